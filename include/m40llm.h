@@ -527,6 +527,132 @@ int m40llm_ext_batched_greedy_step_async(M40llmCudaContext* ctx, const void* d_l
                                          const void* d_table_f16, uint32_t d_model, void* d_x_out_f32);
 const char* m40llm_ext_build_info(void);
 
+/* ---- layered decoders: bf16 weights, bf16 or f32 activations ----------------------------------------------------------------
+ * Building blocks of decoders that are described layer by layer (no counterpart in the reference).  All of them are
+ * asynchronous on the stream stream_kind names.  act_dtype: 0 = bf16 activations (f32 sums), 1 = f32 throughout (products
+ * on the f32 matrix instruction).  Weights are bf16 in packed tiles: a [N][K] matrix is ceil(N/16) x ceil(K/32) tiles of
+ * 512 elements, row tile after row tile, zero past the matrix; the element order inside a tile is the operand order of
+ * the 16x16x32 matrix instruction. */
+#define M40LLM_ACT_BF16 0u
+#define M40LLM_ACT_F32 1u
+/* Source element (nb, n, kb, k) = src[nb*sn_block + n*sn + kb*sk_block + k*sk] goes to packed row
+ * n_offset + nb*n_block_pad + n and packed column k_offset + kb*k_block_pad + k of a matrix with k_tiles tiles per row
+ * tile; row tile t of that counting is stored as row tile tile_first + t*tile_stride.  dst must have been cleared. */
+typedef struct M40llmPackPlan {
+    uint32_t n_blocks, n, n_block_pad, n_offset;
+    uint32_t k_blocks, k, k_block_pad, k_offset;
+    uint64_t sn_block, sn, sk_block, sk;
+    uint32_t k_tiles, tile_first, tile_stride;
+} M40llmPackPlan;
+int m40llm_ext_pack_tiles_async(M40llmCudaContext* ctx, const void* d_src_bf16, void* d_dst, const M40llmPackPlan* plan,
+                                uint32_t stream_kind);
+/* n bf16 values, uniform with mean 0 and the given standard deviation, from a counter-based generator */
+int m40llm_ext_fill_random_bf16_async(M40llmCudaContext* ctx, void* d_dst, uint64_t n, uint64_t seed, float std_dev,
+                                      uint32_t stream_kind);
+/* clears n 32-bit words with a kernel */
+int m40llm_ext_clear_u32_async(M40llmCudaContext* ctx, void* d_dst, size_t n, uint32_t stream_kind);
+
+/* what a packed product does with its sums */
+#define M40LLM_PACKED_STORE 0u      /* out_f32[row][col] = v */
+#define M40LLM_PACKED_ADD 1u        /* out_f32[row][col] += v */
+#define M40LLM_PACKED_STORE_ACT 2u  /* out_act[row][col] = v */
+#define M40LLM_PACKED_GATED 3u      /* out_act[row][col] = v * sigmoid(gate[row][batch]) */
+#define M40LLM_PACKED_ROTATE 4u     /* heads of [plain | rotated] columns: pairs (2i, 2i+1) of the rotated part are rotated */
+#define M40LLM_PACKED_PROJECT 5u    /* the first plain_tiles tiles: as STORE; then pairs of tiles (gate, up):
+                                       out_act[row][16*pair + c] = gelu_tanh(gate) * up */
+typedef struct M40llmPackedGemm {
+    uint32_t act_dtype, epilogue;
+    const void* a;                /* [rows][lda] activations, the columns past the matrix (to k_tiles*32) zero */
+    uint64_t lda, a_batch;        /* elements; lda a multiple of 8 */
+    const void* w;
+    uint32_t n_tiles, k_tiles;
+    uint64_t w_batch;             /* elements */
+    uint32_t rows, batches;
+    void* out_f32;
+    uint64_t ld_out, out_batch;
+    void* out_act;
+    uint64_t ld_act, act_batch;
+    uint32_t cols, plain_tiles;
+    const void* gate;
+    uint64_t ld_gate;
+    uint32_t head_width, rot_start, heads, split_row, rot_half;
+    const void* angles;
+    void* rot_out;
+    uint64_t ld_rot;
+} M40llmPackedGemm;
+int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm* g, uint32_t stream_kind);
+
+/* x[row] = table[token] (+ pair_table[(prev*mul_prev + token*mul_cur) mod buckets], row `buckets` where prev is
+ * 0xffffffff = the token opens its sequence; pair_table NULL = none).  bf16 tables, f32 rows. */
+int m40llm_ext_embed_pairs_async(M40llmCudaContext* ctx, const void* d_table_bf16, const void* d_pair_table_bf16,
+                                 const uint32_t* d_tokens, const uint32_t* d_prev, uint32_t rows, uint32_t vocab, uint32_t width,
+                                 uint32_t buckets, uint32_t mul_prev, uint32_t mul_cur, void* d_x_f32, uint32_t stream_kind);
+/* out[r] = layer norm of x[row_index ? row_index[r] : r] (mean taken off, eps inside the root, weight, no bias);
+ * out has ld_out columns, those past width zero */
+int m40llm_ext_layer_norm_rows_async(M40llmCudaContext* ctx, const void* d_x_f32, const void* d_w_f32,
+                                     const uint32_t* d_row_index, uint32_t rows, uint32_t width, float eps, void* d_out,
+                                     uint32_t ld_out, uint32_t act_dtype, uint32_t stream_kind);
+/* angles[row][i] = (cos, sin)(position * freq[i]) * magnitude for i < pairs, (1, 0) for pairs <= i < ld_pairs; the angle is
+ * formed in double precision */
+int m40llm_ext_rotation_angles_async(M40llmCudaContext* ctx, const uint32_t* d_positions, uint32_t rows, const double* d_freq,
+                                     uint32_t pairs, uint32_t ld_pairs, float magnitude, void* d_angles, uint32_t stream_kind);
+
+/* ---- latent attention over a paged cache ------------------------------------------------------------------------------------
+ * A page holds 64 tokens; a token's entry is its normed latent (kv_rank, padded to a multiple of 32) followed by the rotated
+ * key part all heads share (rot_dim, padded to a multiple of 32): entry_width elements of the activation type, in packed
+ * tile order (4 x entry_width/32 tiles a page).  Page p of a layer starts at base + p*64*entry_width.  Sequence slot s
+ * finds its pages in page_table[s*max_pages + position/64]. */
+#define M40LLM_PAGE_TOKENS 64u
+/* From the projected row [q latent | kv latent | rotated key part | ...] (f32, parts padded to multiples of 16 / 32):
+ * cq[row] = RMSNorm(q latent) (ld_cq columns, zero past q_rank), and where cache is not NULL RMSNorm(kv latent) and the
+ * rotated key part go to the row's place in the cache. */
+typedef struct M40llmLatentSplit {
+    uint32_t act_dtype, rows;
+    const void* proj;                 /* f32 [rows][ld_proj] */
+    uint64_t ld_proj;
+    uint32_t q_rank, kv_offset, kv_rank, rot_offset, rot_dim;
+    const void *q_norm, *kv_norm;     /* f32 weights */
+    float eps;
+    void* cq;
+    uint32_t ld_cq;
+    void* cache;                      /* NULL = the layer reads another layer's entries */
+    uint32_t latent_pad, entry_width, rot_half;
+    const void* angles;
+    const uint32_t *row_slot, *row_pos, *page_table;
+    uint32_t max_pages;
+} M40llmLatentSplit;
+int m40llm_ext_latent_split_append_async(M40llmCudaContext* ctx, const M40llmLatentSplit* s, uint32_t stream_kind);
+/* Attention of query rows i = row*heads + head given in latent space (queries [rows*heads][entry_width]: W_uk^T q, then the
+ * rotated part): score = q . entry * scale over the positions <= row_pos[row] of the row's slot, softmax whose denominator
+ * also holds exp(sink[head]), result = weighted sum of the latents, out [rows*heads][latent_pad].
+ * tiles[t] = {first query row, query rows}: all of one slot, at most 16*m_tiles.  splits > 1 divides the pages of a tile over
+ * that many workgroups; partial sums go to `partial` (m40llm_ext_latent_attention_partial_floats) and are joined by a
+ * second launch. */
+typedef struct M40llmLatentAttention {
+    uint32_t act_dtype, heads, kv_rank, latent_pad, entry_width;
+    float scale;
+    const void* queries;
+    const void* cache;
+    const void* sink;                 /* f32 [heads] */
+    const uint32_t *row_slot, *row_pos, *page_table;
+    uint32_t max_pages;
+    const uint32_t* tiles;            /* device, 2 words a tile */
+    uint32_t n_tiles, m_tiles, splits;
+    uint32_t first_query, n_queries;  /* the range the tiles cover (partials and the joining launch) */
+    void* partial;
+    uint64_t partial_floats;
+    void* out;
+} M40llmLatentAttention;
+int m40llm_ext_latent_attention_async(M40llmCudaContext* ctx, const M40llmLatentAttention* a, uint32_t stream_kind);
+uint64_t m40llm_ext_latent_attention_partial_floats(uint32_t n_queries, uint32_t latent_pad, uint32_t splits);
+/* the largest m_tiles the kernels serve for an entry width (0 = the width is not served) */
+uint32_t m40llm_ext_latent_attention_max_m_tiles(uint32_t act_dtype, uint32_t kv_rank, uint32_t entry_width);
+/* Greedy step of a device-driven decode loop: token r = picks[r] (gap[r] beside it) is recorded at ids[r*capacity + step] /
+ * gaps[...], becomes the input token (prev = the token before), positions advance by one.  state[0] = step counter. */
+int m40llm_ext_advance_rows_async(M40llmCudaContext* ctx, const uint32_t* d_picks, const float* d_gap, uint32_t rows,
+                                  uint32_t* d_tokens, uint32_t* d_prev, uint32_t* d_positions, uint32_t* d_state,
+                                  uint32_t* d_ids, float* d_gaps, uint32_t capacity, uint32_t stream_kind);
+
 /* ---- present but unavailable (return -1, as cuda/stub.c does) ---------------------- */
 int m40llm_kvcache_build_q8_old_from_dense(M40llmCudaContext*, M40llmKVCache*, uint32_t, uint32_t, uint32_t);
 int m40llm_kvcache_build_compressed_from_dense(M40llmCudaContext*, M40llmKVCache*, const M40llmKVCache*, uint32_t);

@@ -168,6 +168,38 @@ int m40host_model_decode_batch_greedy(M40HostModel* model, const uint32_t* seque
 int m40host_model_forward_prefill(M40HostModel* model, const uint32_t* sequence_ids, const uint32_t* lens,
                                   const uint32_t* tokens, uint32_t batch, float* hidden_last_host, float* logits_last_host);
 
+/* ---- model folders (config.json + model.safetensors): decoders described layer by layer -------------------------- */
+typedef struct M40HostModelOptions {
+    uint32_t act_dtype;        /* M40LLM_ACT_BF16 or M40LLM_ACT_F32 */
+    uint32_t max_tokens;       /* what the cache pool holds, rounded up to whole pages of 64; 0 = 4096 */
+    uint32_t max_sequences;    /* 0 = 4 */
+    uint32_t max_rows;         /* rows of one pass (longer steps run in several); 0 = 4096 */
+} M40HostModelOptions;
+typedef struct M40HostStepEntry {
+    uint32_t sequence_id, n_tokens, n_want;
+    const uint32_t* tokens;    /* the sequence's next tokens */
+    const uint32_t* want;      /* places among them whose logits are asked for */
+} M40HostStepEntry;
+/* The design comes from the folder's config.json ("architecture"); options NULL = defaults. */
+M40HostModel* m40host_model_open(M40llmCudaContext* ctx, const char* path, const M40HostModelOptions* options);
+/* the same with random weights of the shapes config_json gives (throughput runs) */
+M40HostModel* m40host_model_open_random(M40llmCudaContext* ctx, const char* config_json, uint64_t seed, float std_dev,
+                                        const M40HostModelOptions* options);
+const char* m40host_model_family(M40HostModel* model);
+uint32_t m40host_model_vocab(M40HostModel* model);
+uint32_t m40host_model_max_seq_len(M40HostModel* model);
+/* One step: every entry's tokens behind what its sequence holds, all entries one batch.  logits_out: [wanted places in entry
+ * order][vocab], may be NULL when nothing is wanted. */
+int m40host_model_step(M40HostModel* model, const M40HostStepEntry* entries, uint32_t n, float* logits_out);
+/* diagnosis: a step of one entry that also reads the residual stream after every layer, [layers][n_tokens][width] */
+int m40host_model_step_layers(M40HostModel* model, const M40HostStepEntry* entry, float* layers_out);
+/* gives back the pages and the state of a sequence */
+int m40host_model_release(M40HostModel* model, uint32_t sequence_id);
+/* throughput runs: the sequence counts as holding `tokens` tokens (entries: whatever its pages contain) */
+int m40host_model_assume_length(M40HostModel* model, uint32_t sequence_id, uint32_t tokens);
+uint32_t m40host_model_length(M40HostModel* model, uint32_t sequence_id);
+uint32_t m40host_model_free_pages(M40HostModel* model);
+
 /* ---- continuous-batching decode scheduler (src/server.rs:203-770 without HTTP, tokenizer and channels) ---------- */
 typedef struct M40HostScheduler M40HostScheduler;
 typedef struct M40HostTickReport {

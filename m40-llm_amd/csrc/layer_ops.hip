@@ -1,0 +1,229 @@
+// Row-wise steps of layered decoders: token + token-pair embedding, layer norm, rotation angles, and the step between a latent
+// attention's projections and its attention (norms of the two latents, rotation, cache append).
+#include "packed_gemm.hpp"
+
+namespace {
+
+constexpr int kThreads = 256;
+
+__global__ __launch_bounds__(kThreads) void embed_pairs_kernel(const uint16_t* __restrict__ table, const uint16_t* __restrict__ pairs,
+                                                               const uint32_t* __restrict__ tokens, const uint32_t* __restrict__ prev,
+                                                               uint32_t vocab, uint32_t width, uint32_t buckets, uint32_t mul_prev,
+                                                               uint32_t mul_cur, float* __restrict__ x) {
+    const uint32_t row = blockIdx.x;
+    uint32_t tok = tokens[row];
+    tok = tok < vocab ? tok : vocab - 1u;
+    const uint16_t* a = table + (size_t)tok * width;
+    const uint16_t* b = nullptr;
+    if (pairs) {
+        const uint32_t p = prev[row];
+        const uint32_t r = p == 0xffffffffu ? buckets : (uint32_t)(((uint64_t)p * mul_prev + (uint64_t)tok * mul_cur) % buckets);
+        b = pairs + (size_t)r * width;
+    }
+    for (uint32_t i = threadIdx.x; i < width; i += kThreads) {
+        float v = m40_bf16_bits(a[i]);
+        if (b) v += m40_bf16_bits(b[i]);
+        x[(size_t)row * width + i] = v;
+    }
+}
+
+// sum over the workgroup, the same bits in every thread
+__device__ __forceinline__ float block_sum(float v, float* scratch) {
+    v = m40_sum64(v);
+    __syncthreads();
+    if ((threadIdx.x & 63u) == 0u) scratch[threadIdx.x >> 6] = v;
+    __syncthreads();
+    float s = scratch[0];
+#pragma unroll
+    for (int i = 1; i < kThreads / 64; ++i) s += scratch[i];
+    return s;
+}
+
+template <class T>
+__global__ __launch_bounds__(kThreads) void layer_norm_rows_kernel(const float* __restrict__ x, const float* __restrict__ w,
+                                                                   const uint32_t* __restrict__ row_index, uint32_t width, float eps,
+                                                                   T* __restrict__ out, uint32_t ld_out) {
+    __shared__ float scratch[kThreads / 64];
+    constexpr int kKeep = 16;            // elements a thread keeps in registers (width up to 4096)
+    const float* src = x + (size_t)(row_index ? row_index[blockIdx.x] : blockIdx.x) * width;
+    T* dst = out + (size_t)blockIdx.x * ld_out;
+    float keep[kKeep];
+    const bool kept = width <= (uint32_t)(kKeep * kThreads);
+    float s = 0.0f;
+    if (kept) {
+#pragma unroll
+        for (int j = 0; j < kKeep; ++j) {
+            const uint32_t i = threadIdx.x + j * kThreads;
+            keep[j] = i < width ? src[i] : 0.0f;
+            s += keep[j];
+        }
+    } else {
+        for (uint32_t i = threadIdx.x; i < width; i += kThreads) s += src[i];
+    }
+    const float mean = block_sum(s, scratch) / (float)width;
+    float q = 0.0f;
+    if (kept) {
+#pragma unroll
+        for (int j = 0; j < kKeep; ++j) {
+            const float d = threadIdx.x + j * kThreads < width ? keep[j] - mean : 0.0f;
+            q = fmaf(d, d, q);
+        }
+    } else {
+        for (uint32_t i = threadIdx.x; i < width; i += kThreads) {
+            const float d = src[i] - mean;
+            q = fmaf(d, d, q);
+        }
+    }
+    const float inv = 1.0f / sqrtf(block_sum(q, scratch) / (float)width + eps);
+    if (kept) {
+#pragma unroll
+        for (int j = 0; j < kKeep; ++j) {
+            const uint32_t i = threadIdx.x + j * kThreads;
+            if (i < width) dst[i] = M40Act<T>::from((keep[j] - mean) * inv * w[i]);
+        }
+    } else {
+        for (uint32_t i = threadIdx.x; i < width; i += kThreads) dst[i] = M40Act<T>::from((src[i] - mean) * inv * w[i]);
+    }
+    for (uint32_t i = width + threadIdx.x; i < ld_out; i += kThreads) dst[i] = M40Act<T>::from(0.0f);
+}
+
+__global__ __launch_bounds__(kThreads) void rotation_angles_kernel(const uint32_t* __restrict__ positions, const double* __restrict__ freq,
+                                                                   uint32_t rows, uint32_t pairs, uint32_t ld_pairs, float magnitude,
+                                                                   float2* __restrict__ angles) {
+    const size_t i = (size_t)blockIdx.x * kThreads + threadIdx.x;
+    if (i >= (size_t)rows * ld_pairs) return;
+    const uint32_t row = (uint32_t)(i / ld_pairs), p = (uint32_t)(i % ld_pairs);
+    if (p >= pairs) {
+        angles[i] = make_float2(1.0f, 0.0f);
+        return;
+    }
+    double s, c;
+    sincos((double)positions[row] * freq[p], &s, &c);
+    angles[i] = make_float2((float)(c * (double)magnitude), (float)(s * (double)magnitude));
+}
+
+template <class T>
+__global__ __launch_bounds__(kThreads) void latent_split_append_kernel(M40llmLatentSplit a) {
+    __shared__ float scratch[kThreads / 64];
+    const uint32_t row = blockIdx.x, tid = threadIdx.x;
+    const float* src = static_cast<const float*>(a.proj) + (size_t)row * a.ld_proj;
+    float s = 0.0f;
+    for (uint32_t i = tid; i < a.q_rank; i += kThreads) s = fmaf(src[i], src[i], s);
+    const float q_inv = 1.0f / sqrtf(block_sum(s, scratch) / (float)a.q_rank + a.eps);
+    T* cq = static_cast<T*>(a.cq) + (size_t)row * a.ld_cq;
+    const float* qw = static_cast<const float*>(a.q_norm);
+    for (uint32_t i = tid; i < a.ld_cq; i += kThreads) cq[i] = M40Act<T>::from(i < a.q_rank ? src[i] * q_inv * qw[i] : 0.0f);
+    if (!a.cache) return;
+    const float* kv = src + a.kv_offset;
+    s = 0.0f;
+    for (uint32_t i = tid; i < a.kv_rank; i += kThreads) s = fmaf(kv[i], kv[i], s);
+    const float kv_inv = 1.0f / sqrtf(block_sum(s, scratch) / (float)a.kv_rank + a.eps);
+    const float* kw = static_cast<const float*>(a.kv_norm);
+    const uint32_t pos = a.row_pos[row], page = a.page_table[(size_t)a.row_slot[row] * a.max_pages + pos / M40LLM_PAGE_TOKENS];
+    const uint32_t t = pos % M40LLM_PAGE_TOKENS, k_tiles = a.entry_width / 32u;
+    T* entry = static_cast<T*>(a.cache) + (size_t)page * M40LLM_PAGE_TOKENS * a.entry_width + (size_t)(t / 16u) * k_tiles * kM40Tile;
+    auto place = [&](uint32_t k) { return (size_t)(k / 32u) * kM40Tile + m40_tile_offset(t % 16u, k % 32u); };
+    for (uint32_t i = tid; i < a.latent_pad; i += kThreads)
+        entry[place(i)] = M40Act<T>::from(i < a.kv_rank ? kv[i] * kv_inv * kw[i] : 0.0f);
+    const float* rot = src + a.rot_offset;
+    const float2* ang = static_cast<const float2*>(a.angles) + (size_t)row * a.rot_half;
+    for (uint32_t i = tid; i < a.entry_width - a.latent_pad; i += kThreads) {
+        float y = 0.0f;
+        if (i < a.rot_dim) {
+            const float2 cs = ang[i >> 1];
+            const float u = rot[i & ~1u], v = (i | 1u) < a.rot_dim ? rot[i | 1u] : 0.0f;
+            y = (i & 1u) ? fmaf(v, cs.x, u * cs.y) : fmaf(u, cs.x, -(v * cs.y));
+        }
+        entry[place(a.latent_pad + i)] = M40Act<T>::from(y);
+    }
+}
+
+__global__ __launch_bounds__(kThreads) void advance_rows_kernel(const uint32_t* __restrict__ picks, const float* __restrict__ gap,
+                                                                uint32_t rows, uint32_t* __restrict__ tokens, uint32_t* __restrict__ prev,
+                                                                uint32_t* __restrict__ positions, uint32_t* __restrict__ state,
+                                                                uint32_t* __restrict__ ids, float* __restrict__ gaps, uint32_t capacity) {
+    const uint32_t step = state[0];
+    __syncthreads();
+    for (uint32_t r = threadIdx.x; r < rows; r += kThreads) {
+        const uint32_t next = picks[r];
+        if (step < capacity) {
+            ids[(size_t)r * capacity + step] = next;
+            gaps[(size_t)r * capacity + step] = gap[r];
+        }
+        prev[r] = tokens[r];
+        tokens[r] = next;
+        positions[r] += 1u;
+    }
+    if (threadIdx.x == 0u) state[0] = step + 1u;
+}
+
+int launched() { return hipGetLastError() == hipSuccess ? 0 : -2; }
+
+}  // namespace
+
+extern "C" {
+
+int m40llm_ext_embed_pairs_async(M40llmCudaContext* ctx, const void* d_table, const void* d_pairs, const uint32_t* d_tokens,
+                                 const uint32_t* d_prev, uint32_t rows, uint32_t vocab, uint32_t width, uint32_t buckets,
+                                 uint32_t mul_prev, uint32_t mul_cur, void* d_x, uint32_t stream_kind) {
+    if (!ctx || !d_table || !d_tokens || !d_x || (d_pairs && !d_prev)) return -1;
+    hipStream_t stream = m40_select_stream(ctx, stream_kind);
+    if (!stream || m40_ensure_device(ctx) != 0) return -2;
+    if (rows == 0 || vocab == 0 || width == 0 || (d_pairs && buckets == 0)) return -3;
+    embed_pairs_kernel<<<rows, kThreads, 0, stream>>>(static_cast<const uint16_t*>(d_table), static_cast<const uint16_t*>(d_pairs), d_tokens,
+                                                      d_prev, vocab, width, buckets, mul_prev, mul_cur, static_cast<float*>(d_x));
+    return launched();
+}
+
+int m40llm_ext_layer_norm_rows_async(M40llmCudaContext* ctx, const void* d_x, const void* d_w, const uint32_t* d_row_index, uint32_t rows,
+                                     uint32_t width, float eps, void* d_out, uint32_t ld_out, uint32_t act_dtype, uint32_t stream_kind) {
+    if (!ctx || !d_x || !d_w || !d_out) return -1;
+    hipStream_t stream = m40_select_stream(ctx, stream_kind);
+    if (!stream || m40_ensure_device(ctx) != 0) return -2;
+    if (rows == 0 || width == 0 || ld_out < width || act_dtype > 1u) return -3;
+    const float *x = static_cast<const float*>(d_x), *w = static_cast<const float*>(d_w);
+    if (act_dtype == M40LLM_ACT_F32)
+        layer_norm_rows_kernel<float><<<rows, kThreads, 0, stream>>>(x, w, d_row_index, width, eps, static_cast<float*>(d_out), ld_out);
+    else
+        layer_norm_rows_kernel<m40_bf16><<<rows, kThreads, 0, stream>>>(x, w, d_row_index, width, eps, static_cast<m40_bf16*>(d_out), ld_out);
+    return launched();
+}
+
+int m40llm_ext_rotation_angles_async(M40llmCudaContext* ctx, const uint32_t* d_positions, uint32_t rows, const double* d_freq, uint32_t pairs,
+                                     uint32_t ld_pairs, float magnitude, void* d_angles, uint32_t stream_kind) {
+    if (!ctx || !d_positions || !d_freq || !d_angles) return -1;
+    hipStream_t stream = m40_select_stream(ctx, stream_kind);
+    if (!stream || m40_ensure_device(ctx) != 0) return -2;
+    if (rows == 0 || ld_pairs == 0 || pairs > ld_pairs) return -3;
+    const size_t n = (size_t)rows * ld_pairs;
+    rotation_angles_kernel<<<(unsigned)((n + kThreads - 1) / kThreads), kThreads, 0, stream>>>(d_positions, d_freq, rows, pairs, ld_pairs,
+                                                                                              magnitude, static_cast<float2*>(d_angles));
+    return launched();
+}
+
+int m40llm_ext_latent_split_append_async(M40llmCudaContext* ctx, const M40llmLatentSplit* s, uint32_t stream_kind) {
+    if (!ctx || !s || !s->proj || !s->q_norm || !s->cq) return -1;
+    hipStream_t stream = m40_select_stream(ctx, stream_kind);
+    if (!stream || m40_ensure_device(ctx) != 0) return -2;
+    if (s->rows == 0 || s->q_rank == 0 || s->ld_cq < s->q_rank || s->act_dtype > 1u) return -3;
+    if (s->cache && (!s->kv_norm || !s->angles || !s->row_slot || !s->row_pos || !s->page_table || s->kv_rank == 0 ||
+                     s->latent_pad < s->kv_rank || s->latent_pad % 32u != 0 || s->entry_width % 32u != 0 ||
+                     s->entry_width < s->latent_pad + s->rot_dim || s->rot_half * 2u < s->rot_dim))
+        return -3;
+    if (s->act_dtype == M40LLM_ACT_F32) latent_split_append_kernel<float><<<s->rows, kThreads, 0, stream>>>(*s);
+    else latent_split_append_kernel<m40_bf16><<<s->rows, kThreads, 0, stream>>>(*s);
+    return launched();
+}
+
+int m40llm_ext_advance_rows_async(M40llmCudaContext* ctx, const uint32_t* d_picks, const float* d_gap, uint32_t rows, uint32_t* d_tokens,
+                                  uint32_t* d_prev, uint32_t* d_positions, uint32_t* d_state, uint32_t* d_ids, float* d_gaps,
+                                  uint32_t capacity, uint32_t stream_kind) {
+    if (!ctx || !d_picks || !d_gap || !d_tokens || !d_prev || !d_positions || !d_state || !d_ids || !d_gaps) return -1;
+    hipStream_t stream = m40_select_stream(ctx, stream_kind);
+    if (!stream || m40_ensure_device(ctx) != 0) return -2;
+    if (rows == 0) return -3;
+    advance_rows_kernel<<<1, kThreads, 0, stream>>>(d_picks, d_gap, rows, d_tokens, d_prev, d_positions, d_state, d_ids, d_gaps, capacity);
+    return launched();
+}
+
+}  // extern "C"

@@ -1,0 +1,368 @@
+// Products of row-major activations with tile-packed bf16 weights (packed_gemm.hpp has the layout and the last steps).
+//
+// rows_packed_kernel   a workgroup owns one or two column tiles for up to 64 rows and its waves share out K: weights go
+//                      straight from memory into the matrix instruction's operand registers, one contiguous kilobyte a
+//                      load, each tile read once per 64 rows; the waves' sums meet in LDS.  Decode steps and short
+//                      portions, and every product in f32.
+// tile_packed_kernel   bf16, more rows: 128 x (128 or 256) tiles of C, both operands staged through LDS by direct
+//                      global-to-LDS loads, three stages of 64 k deep with one barrier a stage.  The stage buffers hold
+//                      operands in instruction order, so LDS reads are contiguous kilobytes as well.
+#include "packed_gemm.hpp"
+
+namespace {
+
+struct PackedArgs {
+    const void* a;
+    const m40_bf16* w;
+    long lda, a_batch, w_batch;
+    int n_tiles, k_tiles, rows;
+};
+
+template <class T, int MT, int NT, int WAVES>
+__global__ __launch_bounds__(WAVES * 64) void rows_packed_kernel(PackedArgs g, M40Epilogue<T> e) {
+    extern __shared__ __align__(16) float red[];       // [WAVES][MT][NT][64][4]
+    typedef typename M40Act<T>::vec8 vec8;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int tile0 = (int)blockIdx.x * NT, row0 = (int)blockIdx.y * 16 * MT, batch = blockIdx.z;
+    const T* a[MT];
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+        const int row = row0 + m * 16 + (lane & 15);
+        a[m] = static_cast<const T*>(g.a) + batch * g.a_batch + (long)(row < g.rows ? row : g.rows - 1) * g.lda + (lane >> 4) * 8;
+    }
+    const m40_bf16* w[NT];
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+        const int t = tile0 + n < g.n_tiles ? tile0 + n : g.n_tiles - 1;
+        w[n] = g.w + batch * g.w_batch + (long)t * g.k_tiles * kM40Tile + lane * 8;
+    }
+    m40_float4 acc[MT][NT];
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+#pragma unroll
+        for (int n = 0; n < NT; ++n) acc[m][n] = m40_float4{0.f, 0.f, 0.f, 0.f};
+    constexpr int U = sizeof(T) == 2 ? (MT * NT <= 2 ? 8 : 4) : 1;
+    int k = wave;
+    for (; k + (U - 1) * WAVES < g.k_tiles; k += U * WAVES) {
+        uint4 wf[U][NT];
+        vec8 af[U][MT];
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+#pragma unroll
+            for (int n = 0; n < NT; ++n) wf[u][n] = m40_load_stream(reinterpret_cast<const uint4*>(w[n] + (long)(k + u * WAVES) * kM40Tile));
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+#pragma unroll
+            for (int m = 0; m < MT; ++m) af[u][m] = M40Act<T>::load8(a[m] + (k + u * WAVES) * 32);
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+#pragma unroll
+            for (int m = 0; m < MT; ++m)
+#pragma unroll
+                for (int n = 0; n < NT; ++n) acc[m][n] = M40Act<T>::mma(af[u][m], __builtin_bit_cast(m40_bf16x8, wf[u][n]), acc[m][n]);
+    }
+    for (; k < g.k_tiles; k += WAVES) {
+        uint4 wf[NT];
+#pragma unroll
+        for (int n = 0; n < NT; ++n) wf[n] = *reinterpret_cast<const uint4*>(w[n] + (long)k * kM40Tile);
+#pragma unroll
+        for (int m = 0; m < MT; ++m) {
+            const vec8 af = M40Act<T>::load8(a[m] + k * 32);
+#pragma unroll
+            for (int n = 0; n < NT; ++n) acc[m][n] = M40Act<T>::mma(af, __builtin_bit_cast(m40_bf16x8, wf[n]), acc[m][n]);
+        }
+    }
+    m40_float4* r4 = reinterpret_cast<m40_float4*>(red);
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+#pragma unroll
+        for (int n = 0; n < NT; ++n) r4[((wave * MT + m) * NT + n) * 64 + lane] = acc[m][n];
+    __syncthreads();
+    for (int m = wave; m < MT; m += WAVES) {
+        if (row0 + m * 16 >= g.rows) continue;
+        m40_float4 s[NT];
+#pragma unroll
+        for (int n = 0; n < NT; ++n) {
+            s[n] = r4[(m * NT + n) * 64 + lane];
+#pragma unroll
+            for (int i = 1; i < WAVES; ++i) s[n] += r4[((i * MT + m) * NT + n) * 64 + lane];
+        }
+        if (NT == 2 && e.kind == M40LLM_PACKED_PROJECT && tile0 >= e.plain_tiles) {
+            m40_epilogue_pair(e, row0 + m * 16, (tile0 - e.plain_tiles) / 2, lane, s[0], s[NT - 1]);
+        } else {
+#pragma unroll
+            for (int n = 0; n < NT; ++n)
+                if (tile0 + n < g.n_tiles) m40_epilogue_tile(e, batch, row0 + m * 16, tile0 + n, lane, s[n]);
+        }
+    }
+}
+
+template <class T, int MT, int NT, int WAVES>
+int launch_rows(hipStream_t stream, const PackedArgs& g, const M40Epilogue<T>& e, int batches) {
+    const dim3 grid((unsigned)((g.n_tiles + NT - 1) / NT), (unsigned)((g.rows + 16 * MT - 1) / (16 * MT)), (unsigned)batches);
+    constexpr size_t lds = (size_t)WAVES * MT * NT * 1024;
+    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(rows_packed_kernel<T, MT, NT, WAVES>),
+                                                       hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (attr != hipSuccess) return -2;
+    rows_packed_kernel<T, MT, NT, WAVES><<<grid, WAVES * 64, lds, stream>>>(g, e);
+    return hipGetLastError() == hipSuccess ? 0 : -2;
+}
+
+template <class T, int MT>
+int launch_rows_m(hipStream_t stream, const PackedArgs& g, const M40Epilogue<T>& e, int batches) {
+    if (e.kind == M40LLM_PACKED_PROJECT) return launch_rows<T, MT, 2, 8>(stream, g, e, batches);
+    if (g.k_tiles >= 64) return launch_rows<T, MT, 1, 16>(stream, g, e, batches);
+    if (g.k_tiles >= 16) return launch_rows<T, MT, 1, 8>(stream, g, e, batches);
+    return launch_rows<T, MT, 1, 4>(stream, g, e, batches);
+}
+template <class T>
+int launch_rows_any(hipStream_t stream, const PackedArgs& g, const M40Epilogue<T>& e, int batches) {
+    if (g.rows <= 16) return launch_rows_m<T, 1>(stream, g, e, batches);
+    if (g.rows <= 32) return launch_rows_m<T, 2>(stream, g, e, batches);
+    return launch_rows_m<T, 4>(stream, g, e, batches);
+}
+
+// ---- many rows, bf16 ---------------------------------------------------------------------------------------------------
+// Workgroup of four waves (2 x 2), wave tile 64 x (16 NTW): C tile 128 x 32 NTW.  A stage is two k tiles of every operand
+// tile: (8 + 2 NTW) * 2 KB, filled by global_load_lds (a wave's instruction moves one 16 x 32 operand tile: for A the lanes
+// gather the rows' 16-byte pieces into instruction order, for W the tile is already contiguous).
+__device__ __forceinline__ constexpr int vm_wait(int n) { return 0x0f70 | (n & 15) | ((n >> 4) << 14); }
+constexpr int kStages = 3;
+
+template <int NTW>
+__global__ __launch_bounds__(256, 1) void tile_packed_kernel(PackedArgs g, M40Epilogue<m40_bf16> e) {
+    typedef __attribute__((address_space(3))) void* lds_dst_t;
+    typedef const __attribute__((address_space(1))) void* global_src_t;
+    extern __shared__ __align__(16) uint8_t stage_lds[];
+    constexpr int kATiles = 8, kBTiles = 2 * NTW;                    // 16-row operand tiles of the workgroup
+    constexpr int kStageBytes = (kATiles + kBTiles) * 2 * 1024;
+    constexpr int kLoads = (kATiles + kBTiles) * 2 / 4;              // per wave and stage
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int tiles_n = (g.n_tiles + kBTiles - 1) / kBTiles;
+    // workgroups are dealt to the eight dies in turn: each die gets a contiguous band of row tiles
+    const int per_die = (int)gridDim.x / 8;
+    const int logical = (int)blockIdx.x < per_die * 8 ? ((int)blockIdx.x % 8) * per_die + (int)blockIdx.x / 8 : (int)blockIdx.x;
+    const int m0 = logical / tiles_n * 128, t0 = logical % tiles_n * kBTiles, batch = blockIdx.z;
+    const m40_bf16* A = static_cast<const m40_bf16*>(g.a) + batch * g.a_batch;
+    const m40_bf16* W = g.w + batch * g.w_batch;
+    // this wave's pieces of a stage: operand tiles wave, wave + 4, ... of the A tiles, then of the W tiles; both k tiles of each
+    const m40_bf16* src[kLoads / 2];
+    uint32_t dst[kLoads / 2];
+#pragma unroll
+    for (int i = 0; i < kLoads / 2; ++i) {
+        const int t = wave + 4 * i;
+        if (i < kATiles / 4) {
+            const int row = m0 + t * 16 + (lane & 15);
+            src[i] = A + (long)(row < g.rows ? row : g.rows - 1) * g.lda + (lane >> 4) * 8;
+        } else {
+            const int n = t0 + t - kATiles;
+            src[i] = W + (long)(n < g.n_tiles ? n : g.n_tiles - 1) * g.k_tiles * kM40Tile + lane * 8;
+        }
+        dst[i] = t * 2048;
+    }
+    const int stages = (g.k_tiles + 1) / 2;
+    auto issue = [&](int buf, int s) {
+        uint8_t* base = stage_lds + buf * kStageBytes;
+        const int k0 = 2 * s, k1 = k0 + 1 < g.k_tiles ? k0 + 1 : k0;     // an odd last k tile is loaded twice, used once
+#pragma unroll
+        for (int i = 0; i < kLoads / 2; ++i) {
+            const int step = i < kATiles / 4 ? 32 : kM40Tile;
+            __builtin_amdgcn_global_load_lds((global_src_t)(src[i] + (long)k0 * step), (lds_dst_t)(base + dst[i]), 16, 0, 0);
+            __builtin_amdgcn_global_load_lds((global_src_t)(src[i] + (long)k1 * step), (lds_dst_t)(base + dst[i] + 1024), 16, 0, 0);
+        }
+    };
+    const int wm = wave >> 1, wn = wave & 1;
+    m40_float4 acc[4][NTW];
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < NTW; ++j) acc[i][j] = m40_float4{0.f, 0.f, 0.f, 0.f};
+    auto compute = [&](const uint8_t* base, int kk) {
+        const uint8_t* a = base + wm * 4 * 2048 + kk * 1024 + lane * 16;
+        const uint8_t* b = base + (kATiles + wn * NTW) * 2048 + kk * 1024 + lane * 16;
+        m40_bf16x8 af[4], bf[NTW];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) af[i] = *reinterpret_cast<const m40_bf16x8*>(a + i * 2048);
+#pragma unroll
+        for (int j = 0; j < NTW; ++j) bf[j] = *reinterpret_cast<const m40_bf16x8*>(b + j * 2048);
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+            for (int j = 0; j < NTW; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(af[i], bf[j], acc[i][j], 0, 0, 0);
+    };
+    issue(0, 0);
+    issue(1, 1 < stages ? 1 : stages - 1);
+    int buf = 0;
+    for (int s = 0; s < stages; ++s) {
+        // stage s is in LDS once at most the newest stage's loads are outstanding; behind the barrier every wave's are, and
+        // every wave is done with stage s - 1, whose buffer takes stage s + 2
+        __builtin_amdgcn_sched_barrier(0);
+        __builtin_amdgcn_s_waitcnt(vm_wait(kLoads));
+        __builtin_amdgcn_s_barrier();
+        __builtin_amdgcn_sched_barrier(0);
+        issue(buf == 0 ? 2 : buf - 1, s + 2 < stages ? s + 2 : stages - 1);
+        const uint8_t* base = stage_lds + buf * kStageBytes;
+        compute(base, 0);
+        if (2 * s + 1 < g.k_tiles) compute(base, 1);
+        buf = buf == kStages - 1 ? 0 : buf + 1;
+    }
+    __builtin_amdgcn_s_waitcnt(vm_wait(0));        // no write into LDS may be outstanding when the workgroup ends
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int row0 = m0 + (wm * 4 + i) * 16;
+        if (row0 >= g.rows) continue;
+#pragma unroll
+        for (int j = 0; j < NTW; j += 2) {
+            const int tile = t0 + wn * NTW + j;
+            if (e.kind == M40LLM_PACKED_PROJECT && tile >= e.plain_tiles) {
+                if (tile + 1 < g.n_tiles) m40_epilogue_pair(e, row0, (tile - e.plain_tiles) / 2, lane, acc[i][j], acc[i][j + 1]);
+            } else {
+                if (tile < g.n_tiles) m40_epilogue_tile(e, batch, row0, tile, lane, acc[i][j]);
+                if (tile + 1 < g.n_tiles) m40_epilogue_tile(e, batch, row0, tile + 1, lane, acc[i][j + 1]);
+            }
+        }
+    }
+}
+
+template <int NTW>
+int launch_tile(hipStream_t stream, const PackedArgs& g, const M40Epilogue<m40_bf16>& e, int batches) {
+    constexpr int lds = (8 + 2 * NTW) * 2 * 1024 * kStages;
+    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(tile_packed_kernel<NTW>),
+                                                       hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    if (attr != hipSuccess) return -2;
+    const long long tiles = (long long)((g.rows + 127) / 128) * ((g.n_tiles + 2 * NTW - 1) / (2 * NTW));
+    tile_packed_kernel<NTW><<<dim3((unsigned)tiles, 1, (unsigned)batches), 256, lds, stream>>>(g, e);
+    return hipGetLastError() == hipSuccess ? 0 : -2;
+}
+
+template <class T>
+M40Epilogue<T> make_epilogue(const M40llmPackedGemm& p) {
+    M40Epilogue<T> e{};
+    e.kind = (int)p.epilogue;
+    e.rows = (int)p.rows;
+    e.out_f32 = static_cast<float*>(p.out_f32);
+    e.out_act = static_cast<T*>(p.out_act);
+    e.ld_out = (long)p.ld_out; e.ld_act = (long)p.ld_act;
+    e.out_batch = (long)p.out_batch; e.act_batch = (long)p.act_batch;
+    e.cols = (int)p.cols;
+    e.plain_tiles = (int)p.plain_tiles;
+    e.gate = static_cast<const float*>(p.gate);
+    e.ld_gate = (long)p.ld_gate;
+    e.head_width = (int)p.head_width; e.rot_start = (int)p.rot_start; e.heads = (int)p.heads;
+    e.split_row = (int)p.split_row; e.rot_half = (int)p.rot_half;
+    e.angles = static_cast<const float2*>(p.angles);
+    e.rot_out = static_cast<T*>(p.rot_out);
+    e.ld_rot = (long)p.ld_rot;
+    return e;
+}
+
+// one thread per source element
+__global__ __launch_bounds__(256) void pack_tiles_kernel(const uint16_t* __restrict__ src, uint16_t* __restrict__ dst,
+                                                         M40llmPackPlan p, size_t total) {
+    for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (size_t)gridDim.x * 256) {
+        size_t r = i;
+        const uint32_t k = (uint32_t)(r % p.k); r /= p.k;
+        const uint32_t kb = (uint32_t)(r % p.k_blocks); r /= p.k_blocks;
+        const uint32_t n = (uint32_t)(r % p.n), nb = (uint32_t)(r / p.n);
+        const uint32_t row = p.n_offset + nb * p.n_block_pad + n, col = p.k_offset + kb * p.k_block_pad + k;
+        const size_t tile = (size_t)(p.tile_first + (row >> 4) * p.tile_stride) * p.k_tiles + (col >> 5);
+        dst[tile * kM40Tile + m40_tile_offset(row & 15u, col & 31u)] = src[nb * p.sn_block + n * p.sn + kb * p.sk_block + k * p.sk];
+    }
+}
+
+__global__ __launch_bounds__(256) void clear_u32_kernel(uint32_t* dst, size_t n) {
+    for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (size_t)gridDim.x * 256) dst[i] = 0u;
+}
+
+__global__ __launch_bounds__(256) void fill_random_bf16_kernel(uint16_t* dst, size_t n, uint64_t seed, float half_range) {
+    for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (size_t)gridDim.x * 256) {
+        uint64_t z = seed + (i + 1) * 0x9e3779b97f4a7c15ull;        // splitmix64
+        z = (z ^ (z >> 30)) * 0xbf58476d1ce4e5b9ull;
+        z = (z ^ (z >> 27)) * 0x94d049bb133111ebull;
+        z ^= z >> 31;
+        const float u = (float)(uint32_t)(z >> 40) * (2.0f / 16777216.0f) - 1.0f;
+        dst[i] = __builtin_bit_cast(uint16_t, static_cast<m40_bf16>(u * half_range));
+    }
+}
+
+}  // namespace
+
+extern "C" {
+
+int m40llm_ext_fill_random_bf16_async(M40llmCudaContext* ctx, void* d_dst, uint64_t n, uint64_t seed, float std_dev, uint32_t stream_kind) {
+    if (!ctx || !d_dst) return -1;
+    hipStream_t stream = m40_select_stream(ctx, stream_kind);
+    if (!stream || m40_ensure_device(ctx) != 0) return -2;
+    if (n == 0) return 0;
+    const uint64_t blocks = (n + 255) / 256;
+    fill_random_bf16_kernel<<<(unsigned)(blocks < 65536 ? blocks : 65536), 256, 0, stream>>>(static_cast<uint16_t*>(d_dst), (size_t)n, seed,
+                                                                                             std_dev * 1.7320508075688772f);
+    return hipGetLastError() == hipSuccess ? 0 : -2;
+}
+
+int m40llm_ext_pack_tiles_async(M40llmCudaContext* ctx, const void* d_src, void* d_dst, const M40llmPackPlan* plan, uint32_t stream_kind) {
+    if (!ctx || !d_src || !d_dst || !plan) return -1;
+    hipStream_t stream = m40_select_stream(ctx, stream_kind);
+    if (!stream || m40_ensure_device(ctx) != 0) return -2;
+    const M40llmPackPlan& p = *plan;
+    const size_t total = (size_t)p.n_blocks * p.n * p.k_blocks * p.k;
+    if (total == 0 || p.tile_stride == 0) return -3;
+    if (p.k_offset + (uint64_t)(p.k_blocks - 1) * p.k_block_pad + p.k > (uint64_t)p.k_tiles * 32u) return -3;
+    const size_t blocks = (total + 255) / 256;
+    pack_tiles_kernel<<<(unsigned)(blocks < 65536 ? blocks : 65536), 256, 0, stream>>>(static_cast<const uint16_t*>(d_src),
+                                                                                       static_cast<uint16_t*>(d_dst), p, total);
+    return hipGetLastError() == hipSuccess ? 0 : -2;
+}
+
+int m40llm_ext_clear_u32_async(M40llmCudaContext* ctx, void* d_dst, size_t n, uint32_t stream_kind) {
+    if (!ctx || !d_dst) return -1;
+    hipStream_t stream = m40_select_stream(ctx, stream_kind);
+    if (!stream || m40_ensure_device(ctx) != 0) return -2;
+    if (n == 0) return 0;
+    const size_t blocks = (n + 255) / 256;
+    clear_u32_kernel<<<(unsigned)(blocks < 4096 ? blocks : 4096), 256, 0, stream>>>(static_cast<uint32_t*>(d_dst), n);
+    return hipGetLastError() == hipSuccess ? 0 : -2;
+}
+
+int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm* p, uint32_t stream_kind) {
+    if (!ctx || !p || !p->a || !p->w) return -1;
+    hipStream_t stream = m40_select_stream(ctx, stream_kind);
+    if (!stream || m40_ensure_device(ctx) != 0) return -2;
+    if (p->act_dtype > 1u || p->epilogue > M40LLM_PACKED_PROJECT || p->rows == 0 || p->batches == 0 || p->batches > 65535u ||
+        p->n_tiles == 0 || p->k_tiles == 0 || p->lda % 8 != 0 || p->lda < (uint64_t)p->k_tiles * 32u || !m40_aligned16(p->a) ||
+        !m40_aligned16(p->w) || p->rows > 0x3fffffffu || (p->batches > 1u && (p->a_batch % 8 != 0 || p->w_batch % 8 != 0)))
+        return -3;
+    switch (p->epilogue) {
+        case M40LLM_PACKED_STORE: case M40LLM_PACKED_ADD: if (!p->out_f32 || p->cols > p->n_tiles * 16u) return -4; break;
+        case M40LLM_PACKED_STORE_ACT: if (!p->out_act || p->cols > p->n_tiles * 16u) return -4; break;
+        case M40LLM_PACKED_GATED: if (!p->out_act || !p->gate || p->cols > p->n_tiles * 16u) return -4; break;
+        case M40LLM_PACKED_ROTATE:
+            if (!p->out_act || !p->angles || p->head_width == 0 || p->head_width % 32 != 0 || p->rot_start % 32 != 0 ||
+                p->rot_start >= p->head_width || p->rot_half * 2u != p->head_width - p->rot_start ||
+                p->heads * p->head_width != p->n_tiles * 16u || (p->split_row > 0 && !p->rot_out))
+                return -4;
+            break;
+        case M40LLM_PACKED_PROJECT:
+            if ((p->plain_tiles > 0 && !p->out_f32) || (p->n_tiles > p->plain_tiles && !p->out_act) || p->plain_tiles % 2 != 0 ||
+                p->n_tiles % 2 != 0 || p->plain_tiles > p->n_tiles)
+                return -4;
+            break;
+    }
+    PackedArgs g{};
+    g.a = p->a;
+    g.w = static_cast<const m40_bf16*>(p->w);
+    g.lda = (long)p->lda; g.a_batch = (long)p->a_batch; g.w_batch = (long)p->w_batch;
+    g.n_tiles = (int)p->n_tiles; g.k_tiles = (int)p->k_tiles; g.rows = (int)p->rows;
+    (void)hipGetLastError();
+    if (p->act_dtype == M40LLM_ACT_F32) {
+        if ((g.rows + 63) / 64 > 65535) return -3;
+        return launch_rows_any<float>(stream, g, make_epilogue<float>(*p), (int)p->batches);
+    }
+    const M40Epilogue<m40_bf16> e = make_epilogue<m40_bf16>(*p);
+    if (g.rows <= 64) return launch_rows_any<m40_bf16>(stream, g, e, (int)p->batches);
+    const long long wide = (long long)((g.rows + 127) / 128) * ((g.n_tiles + 15) / 16) * p->batches;
+    if (wide * 16 >= 9ll * ctx->num_cus) return launch_tile<8>(stream, g, e, (int)p->batches);
+    return launch_tile<4>(stream, g, e, (int)p->batches);
+}
+
+}  // extern "C"

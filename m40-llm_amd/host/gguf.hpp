@@ -94,20 +94,20 @@ inline std::string shape_text(const std::vector<uint64_t>& s) {
 
 class MappedFile {
 public:
-    explicit MappedFile(const std::string& path) {
+    explicit MappedFile(const std::string& path, const char* kind = "GGUF file") {
         fd_ = ::open(path.c_str(), O_RDONLY | O_CLOEXEC);
-        if (fd_ < 0) throw Error("failed to open GGUF file \"" + path + "\": " + std::strerror(errno));
+        if (fd_ < 0) throw Error(std::string("failed to open ") + kind + " \"" + path + "\": " + std::strerror(errno));
         struct stat st {};
         if (::fstat(fd_, &st) != 0 || st.st_size < 0) {
             ::close(fd_);
-            throw Error("failed to stat GGUF file \"" + path + "\"");
+            throw Error(std::string("failed to stat ") + kind + " \"" + path + "\"");
         }
         len_ = static_cast<uint64_t>(st.st_size);
         if (len_ > 0) {
             void* p = ::mmap(nullptr, len_, PROT_READ, MAP_PRIVATE, fd_, 0);
             if (p == MAP_FAILED) {
                 ::close(fd_);
-                throw Error("failed to map GGUF file \"" + path + "\"");
+                throw Error(std::string("failed to map ") + kind + " \"" + path + "\"");
             }
             base_ = static_cast<const uint8_t*>(p);
         }

@@ -11,6 +11,7 @@
 #include "gguf_loader.hpp"
 #include "kv_compression.hpp"
 #include "kv_selection.hpp"
+#include "layered_decoder.hpp"
 #include "model.hpp"
 #include "sampling.hpp"
 #include "scheduler.hpp"
@@ -69,13 +70,33 @@ StoppingCriteria make_stopping(int64_t max_tokens, int64_t eos_id, const uint32_
     return StoppingCriteria::make(mt, eos);
 }
 
+LayeredOptions to_options(const M40HostModelOptions* o) {
+    LayeredOptions r;
+    if (!o) return r;
+    r.act_dtype = o->act_dtype;
+    if (o->max_tokens) r.max_tokens = o->max_tokens;
+    if (o->max_sequences) r.max_sequences = o->max_sequences;
+    if (o->max_rows) r.max_rows = o->max_rows;
+    return r;
+}
+
 struct PlanHolder {
     DecodeBatchPlan plan;
 };
 }  // namespace
 
 struct M40HostModel {
-    std::unique_ptr<DecodeModel> m;
+    std::unique_ptr<ServedModel> m;
+    DecodeModel& dense() {
+        auto* d = dynamic_cast<DecodeModel*>(m.get());
+        if (!d) throw std::invalid_argument("this call needs a dense decoder");
+        return *d;
+    }
+    LayeredDecoder& layered() {
+        auto* d = dynamic_cast<LayeredDecoder*>(m.get());
+        if (!d) throw std::invalid_argument("this call needs a layered decoder");
+        return *d;
+    }
 };
 struct M40HostScheduler {
     std::unique_ptr<DecodeScheduler> s;
@@ -325,9 +346,11 @@ M40HostModel* m40host_model_create(M40llmCudaContext* ctx, const M40HostModelCon
         nullptr);
 }
 void m40host_model_destroy(M40HostModel* m) { delete m; }
-M40llmKVCache* m40host_model_kv(M40HostModel* m) { return m->m->kv(); }
+M40llmKVCache* m40host_model_kv(M40HostModel* m) {
+    return guarded([&]() -> M40llmKVCache* { return m->dense().kv(); }, nullptr);
+}
 uint32_t m40host_model_kv_slot(M40HostModel* m, uint32_t seq, uint32_t layer) {
-    return guarded([&]() -> uint32_t { return m->m->kv_slot(seq, layer); }, 0xffffffffu);
+    return guarded([&]() -> uint32_t { return m->dense().kv_slot(seq, layer); }, 0xffffffffu);
 }
 int m40host_model_set_mode(M40HostModel* m, uint32_t mode) {
     if (mode > 2) return -1;
@@ -338,7 +361,7 @@ int m40host_model_forward_token(M40HostModel* m, uint32_t seq, uint32_t pos, uin
                                 float* logits_host) {
     return guarded(
         [&]() -> int {
-            DecodeModel& d = *m->m;
+            DecodeModel& d = m->dense();
             const float* h = d.forward_token(seq, pos, token);
             if (hidden_host) {
                 M40H_TRY(m40llm_stream_synchronize(d.ctx(), M40LLM_STREAM_DECODE));
@@ -355,7 +378,7 @@ int m40host_model_decode_greedy(M40HostModel* m, uint32_t seq, const uint32_t* p
 }
 int m40host_model_decode_timed(M40HostModel* m, uint32_t seq, const uint32_t* prompt, uint32_t n_prompt, uint32_t warmup,
                                uint32_t steps, uint32_t* ids_out, double* elapsed_ms) {
-    return guarded([&]() -> int { m->m->decode_timed(seq, prompt, n_prompt, warmup, steps, ids_out, elapsed_ms); return 0; }, -100);
+    return guarded([&]() -> int { m->dense().decode_timed(seq, prompt, n_prompt, warmup, steps, ids_out, elapsed_ms); return 0; }, -100);
 }
 int m40host_model_decode_batch_timed(M40HostModel* m, const uint32_t* seq_ids, const uint32_t* kv_lens,
                                      const uint32_t* first_tokens, uint32_t rows, uint32_t warmup, uint32_t steps,
@@ -377,7 +400,7 @@ int m40host_model_forward_batched(M40HostModel* m, const uint32_t* seq_ids, cons
                                   uint32_t rows, float* hidden_host, float* logits_host) {
     return guarded(
         [&]() -> int {
-            DecodeModel& d = *m->m;
+            DecodeModel& d = m->dense();
             const float* h = d.forward_batched(seq_ids, kv_lens, tokens, rows);
             if (hidden_host) {
                 M40H_TRY(m40llm_stream_synchronize(d.ctx(), M40LLM_STREAM_DECODE));
@@ -400,7 +423,7 @@ int m40host_model_forward_prefill(M40HostModel* m, const uint32_t* seq_ids, cons
     return guarded(
         [&]() -> int {
             if (!m || !seq_ids || !lens || !tokens) throw std::invalid_argument("null argument");
-            DecodeModel& d = *m->m;
+            DecodeModel& d = m->dense();
             const float* h = d.forward_prefill(seq_ids, lens, tokens, batch);
             const size_t D = d.config().d_model, V = d.config().vocab;
             size_t row = 0;
@@ -511,68 +534,80 @@ M40HostModel* m40host_model_from_gguf(M40HostGgufWeights* w, uint32_t max_seq_le
         nullptr);
 }
 
+// ---- model folders: layered decoders -------------------------------------------------------------------------
+M40HostModel* m40host_model_open(M40llmCudaContext* ctx, const char* path, const M40HostModelOptions* options) {
+    return guarded(
+        [&]() -> M40HostModel* {
+            if (!ctx || !path) throw std::invalid_argument("null argument");
+            auto h = std::make_unique<M40HostModel>();
+            h->m = open_model_folder(ctx, path, to_options(options));
+            return h.release();
+        },
+        nullptr);
+}
+M40HostModel* m40host_model_open_random(M40llmCudaContext* ctx, const char* config_json, uint64_t seed, float std_dev,
+                                        const M40HostModelOptions* options) {
+    return guarded(
+        [&]() -> M40HostModel* {
+            if (!ctx || !config_json) throw std::invalid_argument("null argument");
+            RandomTensors tensors(seed, std_dev);
+            auto h = std::make_unique<M40HostModel>();
+            h->m = std::make_unique<LayeredDecoder>(ctx, read_decoder_spec(config_json), tensors, to_options(options));
+            return h.release();
+        },
+        nullptr);
+}
+const char* m40host_model_family(M40HostModel* m) { return m ? m->m->family() : ""; }
+uint32_t m40host_model_vocab(M40HostModel* m) { return m ? m->m->vocab() : 0; }
+uint32_t m40host_model_max_seq_len(M40HostModel* m) { return m ? m->m->max_seq_len() : 0; }
+int m40host_model_step(M40HostModel* m, const M40HostStepEntry* entries, uint32_t n, float* logits_out) {
+    return guarded(
+        [&]() -> int {
+            if (!m || (!entries && n)) throw std::invalid_argument("null argument");
+            std::vector<StepEntry> e;
+            for (uint32_t i = 0; i < n; ++i) e.push_back({entries[i].sequence_id, entries[i].tokens, entries[i].n_tokens, entries[i].want, entries[i].n_want});
+            m->layered().step(e, logits_out);
+            return 0;
+        },
+        -100);
+}
+int m40host_model_step_layers(M40HostModel* m, const M40HostStepEntry* entry, float* layers_out) {
+    return guarded(
+        [&]() -> int {
+            if (!m || !entry || !layers_out) throw std::invalid_argument("null argument");
+            LayeredDecoder& d = m->layered();
+            const size_t row = d.spec().width, layer = (size_t)entry->n_tokens * row;
+            std::vector<uint32_t> done(d.spec().layers.size(), 0);
+            d.step({{entry->sequence_id, entry->tokens, entry->n_tokens, nullptr, 0}}, nullptr, [&](uint32_t l, uint32_t rows, const float* x) {
+                M40H_TRY(m40llm_memcpy_d2h(d.ctx(), layers_out + l * layer + done[l] * row, x, (size_t)rows * row * 4));
+                done[l] += rows;
+            });
+            return 0;
+        },
+        -100);
+}
+int m40host_model_release(M40HostModel* m, uint32_t seq) {
+    return guarded([&]() -> int { m->layered().release(seq); return 0; }, -100);
+}
+int m40host_model_assume_length(M40HostModel* m, uint32_t seq, uint32_t tokens) {
+    return guarded([&]() -> int { m->layered().assume_length(seq, tokens); return 0; }, -100);
+}
+uint32_t m40host_model_length(M40HostModel* m, uint32_t seq) {
+    return guarded([&]() -> uint32_t { return m->layered().sequences().length(seq); }, 0xffffffffu);
+}
+uint32_t m40host_model_free_pages(M40HostModel* m) {
+    return guarded([&]() -> uint32_t { return m->layered().sequences().free_pages(); }, 0xffffffffu);
+}
+
 // ---- continuous-batching decode scheduler -----------------------------------------------------------------
 M40HostScheduler* m40host_scheduler_create_for_model(M40HostModel* model, uint32_t sequence_slots) {
     return guarded(
         [&]() -> M40HostScheduler* {
             if (!model) throw std::invalid_argument("null model");
-            DecodeModel* d = model->m.get();
-            const ModelConfig& c = d->config();
-            if (sequence_slots == 0 || sequence_slots > c.max_sequences) sequence_slots = c.max_sequences;
-            SchedulerEngine e;
-            e.vocab = c.vocab;
-            e.max_seq_len = c.max_seq_len;
-            e.prefill = [d](const std::vector<SchedulerPrefillItem>& items, float* logits_out) {
-                const ModelConfig& cfg = d->config();
-                if (d->packed_prefill_available()) {
-                    for (size_t i0 = 0; i0 < items.size();) {   // at most 64 prompts and 65535 rows per packed call
-                        std::vector<uint32_t> seqs, lens, toks;
-                        size_t i = i0;
-                        while (i < items.size() && seqs.size() < 64 && toks.size() + items[i].len <= 65535u) {
-                            seqs.push_back(items[i].sequence_id);
-                            lens.push_back(items[i].len);
-                            toks.insert(toks.end(), items[i].tokens, items[i].tokens + items[i].len);
-                            ++i;
-                        }
-                        if (i == i0) throw std::invalid_argument("prompt longer than one packed prefill call takes");
-                        const float* h = d->forward_prefill(seqs.data(), lens.data(), toks.data(), (uint32_t)seqs.size());
-                        size_t row = 0;
-                        for (size_t j = 0; j < seqs.size(); ++j) {
-                            row += lens[j];
-                            d->logits_from_hidden(h + (row - 1) * cfg.d_model, logits_out + (i0 + j) * (size_t)cfg.vocab);
-                        }
-                        i0 = i;
-                    }
-                } else {   // token by token (DecodeSchedulerRequest::step, server.rs:300-329)
-                    for (size_t i = 0; i < items.size(); ++i) {
-                        const float* h = nullptr;
-                        for (uint32_t p = 0; p < items[i].len; ++p) h = d->forward_token(items[i].sequence_id, p, items[i].tokens[p]);
-                        d->logits_from_hidden(h, logits_out + i * (size_t)cfg.vocab);
-                    }
-                }
-            };
-            e.decode = [d](const std::vector<SchedulerDecodeItem>& items, float* logits_out) {
-                std::vector<uint32_t> seqs, lens, toks;
-                for (const auto& it : items) {
-                    seqs.push_back(it.sequence_id);
-                    lens.push_back(it.kv_len);
-                    toks.push_back(it.token);
-                }
-                d->batched_step_logits(seqs.data(), lens.data(), toks.data(), (uint32_t)items.size(), logits_out);
-            };
-            e.decode_pick = [d](const std::vector<SchedulerDecodeItem>& items, const uint8_t* greedy, float* logits_out,
-                                uint32_t* picks_out, uint8_t* picked_out) {
-                std::vector<uint32_t> seqs, lens, toks;
-                for (const auto& it : items) {
-                    seqs.push_back(it.sequence_id);
-                    lens.push_back(it.kv_len);
-                    toks.push_back(it.token);
-                }
-                d->batched_step_logits(seqs.data(), lens.data(), toks.data(), (uint32_t)items.size(), logits_out, greedy, picks_out,
-                                       picked_out);
-            };
+            ServedModel* d = model->m.get();
+            if (sequence_slots == 0 || sequence_slots > d->max_sequences()) sequence_slots = d->max_sequences();
             auto h = std::make_unique<M40HostScheduler>();
-            h->s = std::make_unique<DecodeScheduler>(std::move(e), sequence_slots);
+            h->s = std::make_unique<DecodeScheduler>(d->scheduler_engine(), sequence_slots);
             return h.release();
         },
         nullptr);

@@ -32,6 +32,7 @@
 #include "kv_compression.hpp"
 #include "kv_selection.hpp"
 #include "sampling.hpp"
+#include "served_model.hpp"
 
 namespace m40host {
 
@@ -124,7 +125,7 @@ struct PrefillWorkspace {   // activations of a packed prefill: no per-row logit
     }
 };
 
-class DecodeModel {
+class DecodeModel : public ServedModel {
 public:
     DecodeModel(M40llmCudaContext* ctx, const ModelConfig& cfg, const LayerWeights* layers, const void* out_norm,
                 const void* lm_head, const void* tok_emb, const KvCompressionConfig& kvcfg)
@@ -148,7 +149,7 @@ public:
         if (!kv_) throw std::runtime_error("KV cache allocation failed");
         ws_.ensure(ctx, cfg, 1);
     }
-    ~DecodeModel() {
+    ~DecodeModel() override {
         drop_graph();
         drop_batch_graph();
         if (kv_) m40llm_kvcache_destroy(kv_);
@@ -156,11 +157,15 @@ public:
     DecodeModel(const DecodeModel&) = delete;
     DecodeModel& operator=(const DecodeModel&) = delete;
 
+    const char* family() const override { return "dense"; }
+    uint32_t vocab() const override { return cfg_.vocab; }
+    uint32_t max_seq_len() const override { return cfg_.max_seq_len; }
+    uint32_t max_sequences() const override { return cfg_.max_sequences; }
     const ModelConfig& config() const { return cfg_; }
     M40llmKVCache* kv() const { return kv_; }
     M40llmCudaContext* ctx() const { return ctx_; }
     uint32_t mode() const { return mode_; }
-    void set_mode(uint32_t m) { mode_ = m; }
+    void set_mode(uint32_t m) override { mode_ = m; }
     uint32_t kv_slot(uint32_t seq, uint32_t layer) const {
         if (seq >= cfg_.max_sequences) throw std::out_of_range("sequence id out of range");   // kv.rs:92-107
         return seq * cfg_.n_layers + layer;
@@ -280,7 +285,7 @@ public:
     // state = {position of the last processed token, step, token, capacity, ids[cap], gaps[cap]}
     static constexpr float kGreedyTieGuard = 1e-6f;
     // the guard in force; tests raise it to drive the host-sampled fallback on purpose
-    void set_tie_guard(float g) { tie_guard_ = g; }
+    void set_tie_guard(float g) override { tie_guard_ = g; }
     float tie_guard() const { return tie_guard_; }
     void ensure_state(uint32_t capacity) {
         if (capacity <= state_cap_) return;
@@ -510,7 +515,7 @@ public:
     // Greedy decode of one sequence: prompt tokens from start_pos, then n_gen sampled tokens
     // (Sampler with top_k = 1).  ids_out holds n_prompt + n_gen ids.
     void decode_greedy(uint32_t seq, const uint32_t* prompt, uint32_t n_prompt, uint32_t n_gen, uint32_t start_pos,
-                       uint32_t* ids_out, float* gaps_out) {
+                       uint32_t* ids_out, float* gaps_out) override {
         if (mode_ >= 1 && fused_available() && n_gen > 0) {
             // The device loop also runs the layers for the last sampled token (its KV entry is written); ids are the same.
             if (decode_greedy_device(seq, prompt, n_prompt, 0, n_gen, start_pos, ids_out, gaps_out, nullptr)) return;
@@ -826,7 +831,7 @@ public:
     // `steps` greedy steps for a batch of sequences whose caches already hold kv_lens[r] tokens;
     // first_tokens[r] is the input of step 0.  ids_out: [rows][steps], gaps_out (optional) likewise.
     void decode_batch_greedy(const uint32_t* seq_ids, const uint32_t* kv_lens, const uint32_t* first_tokens,
-                             uint32_t rows, uint32_t steps, uint32_t* ids_out, float* gaps_out) {
+                             uint32_t rows, uint32_t steps, uint32_t* ids_out, float* gaps_out) override {
         if (mode_ >= 1 && batched_fused_available(rows)) {
             if (decode_batch_device(seq_ids, kv_lens, first_tokens, rows, 0, steps, ids_out, gaps_out, nullptr)) return;
             // near-tie somewhere: redo on the host-sampled path (same cache rows are rewritten)
@@ -884,7 +889,7 @@ public:
     }
 
     void decode_batch_timed(const uint32_t* seq_ids, const uint32_t* kv_lens, const uint32_t* first_tokens, uint32_t rows,
-                            uint32_t warmup, uint32_t steps, uint32_t* ids_out, double* elapsed_ms) {
+                            uint32_t warmup, uint32_t steps, uint32_t* ids_out, double* elapsed_ms) override {
         last_timed_host_fallback_ = false;
         if (mode_ >= 1 && batched_fused_available(rows)) {
             if (decode_batch_device(seq_ids, kv_lens, first_tokens, rows, warmup, steps, ids_out, nullptr, elapsed_ms)) return;
@@ -915,7 +920,7 @@ public:
 
     // true when the last decode_timed / decode_batch_timed call measured the host-sampled path because a device-side
     // greedy pick was a near tie
-    bool last_timed_host_fallback() const { return last_timed_host_fallback_; }
+    bool last_timed_host_fallback() const override { return last_timed_host_fallback_; }
 
     void sync_all() {
         M40H_TRY(m40llm_stream_synchronize(ctx_, M40LLM_STREAM_PREFILL));
@@ -931,6 +936,63 @@ public:
         return a - b;
     }
     static float top2_gap(const std::vector<float>& l) { return top2_gap(l.data(), l.size()); }
+
+    // what the continuous-batching scheduler calls
+    SchedulerEngine scheduler_engine() override {
+        SchedulerEngine e;
+        e.vocab = cfg_.vocab;
+        e.max_seq_len = cfg_.max_seq_len;
+        e.prefill = [this](const std::vector<SchedulerPrefillItem>& items, float* logits_out) {
+            const ModelConfig& cfg = cfg_;
+            if (packed_prefill_available()) {
+                for (size_t i0 = 0; i0 < items.size();) {   // at most 64 prompts and 65535 rows per packed call
+                    std::vector<uint32_t> seqs, lens, toks;
+                    size_t i = i0;
+                    while (i < items.size() && seqs.size() < 64 && toks.size() + items[i].len <= 65535u) {
+                        seqs.push_back(items[i].sequence_id);
+                        lens.push_back(items[i].len);
+                        toks.insert(toks.end(), items[i].tokens, items[i].tokens + items[i].len);
+                        ++i;
+                    }
+                    if (i == i0) throw std::invalid_argument("prompt longer than one packed prefill call takes");
+                    const float* h = forward_prefill(seqs.data(), lens.data(), toks.data(), (uint32_t)seqs.size());
+                    size_t row = 0;
+                    for (size_t j = 0; j < seqs.size(); ++j) {
+                        row += lens[j];
+                        logits_from_hidden(h + (row - 1) * cfg.d_model, logits_out + (i0 + j) * (size_t)cfg.vocab);
+                    }
+                    i0 = i;
+                }
+            } else {   // token by token (DecodeSchedulerRequest::step, server.rs:300-329)
+                for (size_t i = 0; i < items.size(); ++i) {
+                    const float* h = nullptr;
+                    for (uint32_t p = 0; p < items[i].len; ++p) h = forward_token(items[i].sequence_id, p, items[i].tokens[p]);
+                    logits_from_hidden(h, logits_out + i * (size_t)cfg.vocab);
+                }
+            }
+        };
+        e.decode = [this](const std::vector<SchedulerDecodeItem>& items, float* logits_out) {
+            std::vector<uint32_t> seqs, lens, toks;
+            for (const auto& it : items) {
+                seqs.push_back(it.sequence_id);
+                lens.push_back(it.kv_len);
+                toks.push_back(it.token);
+            }
+            batched_step_logits(seqs.data(), lens.data(), toks.data(), (uint32_t)items.size(), logits_out);
+        };
+        e.decode_pick = [this](const std::vector<SchedulerDecodeItem>& items, const uint8_t* greedy, float* logits_out,
+                            uint32_t* picks_out, uint8_t* picked_out) {
+            std::vector<uint32_t> seqs, lens, toks;
+            for (const auto& it : items) {
+                seqs.push_back(it.sequence_id);
+                lens.push_back(it.kv_len);
+                toks.push_back(it.token);
+            }
+            batched_step_logits(seqs.data(), lens.data(), toks.data(), (uint32_t)items.size(), logits_out, greedy, picks_out,
+                                   picked_out);
+        };
+        return e;
+    }
 
     ForwardWorkspace& workspace() { return ws_; }
     const std::vector<LayerWeights>& layers() const { return layers_; }

@@ -14,9 +14,11 @@
 //   a request that finishes in a tick is reported then (send_complete), its lease dropped (slot to the back of the
 //   free list, src/decode_batch.rs:75-85).
 // The engine that runs the model is behind two callbacks (and an optional third that lets the engine pick the token of
-// greedy requests itself), so the scheduling logic can be exercised without a GPU.
+// greedy requests itself), so the scheduling logic can be exercised without a GPU.  An engine that takes mixed steps sets
+// `step`: a tick is then one call with every decode token and portions of the pending prompts.
 #pragma once
 
+#include <algorithm>
 #include <cstdint>
 #include <deque>
 #include <functional>
@@ -44,6 +46,14 @@ struct SchedulerDecodeItem {
     uint32_t token;
 };
 
+struct SchedulerStepItem {   // a sequence's next tokens in a mixed step
+    uint32_t sequence_id;
+    uint32_t start;          // tokens the sequence holds already
+    const uint32_t* tokens;
+    uint32_t len;
+    bool want;               // the last token's logits are asked for
+};
+
 struct SchedulerEngine {
     uint32_t vocab = 0;
     uint32_t max_seq_len = 0;
@@ -56,6 +66,14 @@ struct SchedulerEngine {
     std::function<void(const std::vector<SchedulerDecodeItem>&, const uint8_t* greedy, float* logits_out, uint32_t* picks_out,
                        uint8_t* picked_out)>
         decode_pick;
+    // Optional: one call for decode tokens and portions of prompts together; logits_out has a row per wanting item.  Prompts are
+    // then fed in portions, at most step_tokens tokens a tick in all.
+    std::function<void(const std::vector<SchedulerStepItem>&, float* logits_out)> step;
+    uint32_t step_tokens = 0;
+    // Optional: room for a sequence that may grow to `tokens` tokens is set aside before its first portion (false = not now, the
+    // request waits), and given back with everything else the sequence holds when it leaves.
+    std::function<bool(uint32_t sequence_id, uint64_t tokens)> reserve;
+    std::function<void(uint32_t sequence_id)> release;
 };
 
 enum class SchedulerRequestState : uint32_t { Unknown = 0, PendingPrefill = 1, Decoding = 2, Complete = 3, Cancelled = 4, Failed = 5 };
@@ -90,6 +108,7 @@ public:
         // max_tokens defaults to the context length (server.rs:248-251)
         r->stopping = StoppingCriteria::with_stop_ids(max_tokens ? max_tokens : std::optional<size_t>(engine_.max_seq_len ? engine_.max_seq_len : 32),
                                                       std::move(stop_ids));
+        r->max_tokens = max_tokens;
         const uint64_t id = r->id;
         states_[id] = SchedulerRequestState::PendingPrefill;
         active_.push_back(std::move(r));
@@ -154,11 +173,15 @@ public:
             if (r->stopping.should_stop(r->generated)) {
                 finish(*r, SchedulerRequestState::Complete);
                 ++rep.completed;
-            } else if (r->processed == 0 && r->generated.empty()) {
+            } else if (r->processed < r->prompt_len && r->generated.empty()) {
                 prefill.push_back(std::move(r));
             } else {
                 decode.push_back(std::move(r));
             }
+        }
+        if (engine_.step) {
+            run_step(prefill, decode, rep);
+            return rep;
         }
         if (!prefill.empty()) run_prefill(prefill, rep);
         if (!decode.empty()) run_decode(decode, rep);
@@ -174,13 +197,15 @@ private:
         StoppingCriteria stopping;
         std::vector<uint32_t> ids, generated;
         size_t prompt_len = 0, processed = 0;   // processed: tokens whose KV entries exist
-        bool cancelled = false;
+        bool cancelled = false, admitted = false;
+        std::optional<size_t> max_tokens;
     };
 
     void finish(Request& r, SchedulerRequestState st, const std::string& err = std::string()) {
         states_[r.id] = st;
         results_[r.id] = r.generated;
         if (!err.empty()) errors_[r.id] = err;
+        if (engine_.release && r.admitted) engine_.release(r.lease.sequence_id());
         // the lease is dropped with the request: the slot goes to the back of the free list
     }
 
@@ -204,6 +229,62 @@ private:
             ++rep.failed;
         }
         rs.clear();
+    }
+
+    // One mixed step: every decoding request's next token, then the pending prompts in order of arrival, each with as much of it
+    // as the tick still takes.
+    void run_step(std::vector<std::unique_ptr<Request>>& prefill, std::vector<std::unique_ptr<Request>>& decode, SchedulerTickReport& rep) {
+        std::vector<std::unique_ptr<Request>> taking, waiting;
+        std::vector<SchedulerStepItem> items;
+        uint64_t room = engine_.step_tokens ? engine_.step_tokens : 0xffffffffu;
+        for (auto& r : decode) {
+            if (engine_.max_seq_len && r->processed + 1 > engine_.max_seq_len) {
+                finish(*r, SchedulerRequestState::Failed, "context window exhausted");
+                ++rep.failed;
+                continue;
+            }
+            items.push_back({r->lease.sequence_id(), (uint32_t)r->processed, &r->ids[r->processed], 1, true});
+            room = room > 1 ? room - 1 : 0;
+            ++rep.decode_rows;
+            taking.push_back(std::move(r));
+        }
+        bool closed = false;         // a request that waits for room keeps those behind it waiting
+        for (auto& r : prefill) {
+            if (!closed && !r->admitted) {
+                uint64_t most = engine_.max_seq_len ? engine_.max_seq_len : 0xffffffffu;
+                if (r->max_tokens) most = std::min<uint64_t>(most, (uint64_t)r->prompt_len + *r->max_tokens);
+                r->admitted = !engine_.reserve || engine_.reserve(r->lease.sequence_id(), most);
+                closed = !r->admitted;
+            }
+            if (closed || room == 0) {
+                waiting.push_back(std::move(r));
+                continue;
+            }
+            const uint32_t n = (uint32_t)std::min<uint64_t>(room, r->prompt_len - r->processed);
+            items.push_back({r->lease.sequence_id(), (uint32_t)r->processed, &r->ids[r->processed], n, r->processed + n == r->prompt_len});
+            room -= n;
+            ++rep.prefill_rows;
+            rep.prefill_tokens += n;
+            taking.push_back(std::move(r));
+        }
+        if (!items.empty()) {
+            logits_.resize(items.size() * (size_t)engine_.vocab);
+            bool failed = false;
+            try {
+                engine_.step(items, logits_.data());
+            } catch (const std::exception& e) {
+                fail_all(taking, std::string("step failed: ") + e.what(), rep);
+                failed = true;
+            }
+            size_t row = 0;
+            for (size_t i = 0; !failed && i < taking.size(); ++i) {
+                auto& r = taking[i];
+                r->processed += items[i].len;
+                if (items[i].want) sample_and_route(std::move(r), logits_.data() + (row++) * (size_t)engine_.vocab, rep);
+                else active_.push_back(std::move(r));
+            }
+        }
+        for (auto& r : waiting) active_.push_back(std::move(r));
     }
 
     void run_prefill(std::vector<std::unique_ptr<Request>>& rs, SchedulerTickReport& rep) {
