@@ -1,0 +1,122 @@
+"""Prefill and decode throughput of a layered decoder (the Pimosun design, random weights) beside the dense decoder of the same
+width, depth, feed-forward and vocabulary.  `bench.py --design pimosun` prints what measure() returns.
+
+A case is one shape on one kind of step: a prompt of n tokens run in one step (host clock around the blocking call, the last
+token's logits included), or `batch` sequences of `context` tokens that decode greedily from a replayed graph (timed between
+full synchronisations).  Cache contents do not change how long a step takes, so contexts are assumed, not computed."""
+from __future__ import annotations
+
+import importlib
+import time
+
+import numpy as np
+
+pkg = importlib.import_module(__package__)
+syn = importlib.import_module(__package__ + ".synthetic")
+layered = importlib.import_module(__package__ + ".layered")
+
+SHAPES = {
+    # name: layered decoder, and the dense decoder's heads at the same width
+    "2k": dict(width=2048, heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=768, ff=5632, vocab=32000, layers=8, kv_heads=2),
+    "4k": dict(width=4096, heads=32, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=1536, ff=11008, vocab=32000, layers=4, kv_heads=8),
+}
+PREFILL = (512, 4096)
+DECODE = ((1, 1024), (8, 4096), (32, 4096))
+
+
+def pimosun_config(s: dict) -> dict:
+    rot = dict(base=10000.0, dims=s["rot_dim"], scaling=dict(factor=8.0, original=4096, fast=32.0, slow=1.0))
+    mixer = dict(heads=s["heads"], dim=s["dim"], rot_dim=s["rot_dim"], vdim=s["vdim"], kv_rank=s["kv_rank"], q_rank=s["q_rank"],
+                 scale=float((s["dim"] + s["rot_dim"]) ** -0.5), rot=rot)
+    half = s["layers"] // 2
+    layers = [dict(type="latent_attention", mixer=dict(mixer, **({"kv_from": half - 1} if i >= half else {})), mlp=dict(kind="dense", ff=s["ff"]))
+              for i in range(s["layers"])]
+    return dict(architecture="Pimosun", vocab=s["vocab"], width=s["width"], norm=dict(eps=1e-5),
+                embedding=dict(bigram=dict(buckets=20011, mul_prev=31, mul_cur=7)), layers=layers)
+
+
+def layer_flops_per_token(s: dict, own: bool) -> float:
+    """Matrix-product flops of one layer and token outside attention's own products (keys and values from the latent included)."""
+    w, h = s["width"], s["heads"]
+    n = w * (s["q_rank"] + h) + s["q_rank"] * h * (s["dim"] + s["rot_dim"]) + h * (s["dim"] + s["vdim"]) * s["kv_rank"] + h * s["vdim"] * w + 3 * w * s["ff"]
+    return 2.0 * (n + (w * (s["kv_rank"] + s["rot_dim"]) if own else 0))
+
+
+def layered_cases(ctx, s, prefill=PREFILL, decode=DECODE, reps=3, steps=32, warmup=4):
+    out = {}
+    cfg = pimosun_config(s)
+    rng = np.random.default_rng(0)
+    slots = max([b for b, _ in decode] + [1])
+    tokens = max([b * (c + steps + warmup + 64) for b, c in decode] + [n + 64 for n in prefill])
+    m = layered.LayeredModel.random(ctx, cfg, seed=1, std=0.02, max_tokens=tokens, max_sequences=slots, max_rows=max(list(prefill) + [64]))
+    m.set_tie_guard(-1.0)
+    for n in prefill:
+        prompt = rng.integers(0, s["vocab"], size=n).astype(np.uint32)
+        best = None
+        for r in range(reps + 1):
+            t0 = time.perf_counter()
+            m.step([(0, prompt, [n - 1])])
+            ms = (time.perf_counter() - t0) * 1e3
+            m.release(0)
+            if r and (best is None or ms < best):
+                best = ms
+        out[f"prefill {n}"] = dict(ms=best, tok_s=n / (best * 1e-3))
+    for b, c in decode:
+        for i in range(b):
+            m.assume_length(i, c)
+        first = rng.integers(0, s["vocab"], size=b)
+        _, ms = m.decode_batch_timed(np.arange(b), np.full(b, c), first, warmup, steps)
+        for i in range(b):
+            m.release(i)
+        out[f"decode {b} x {c}"] = dict(ms=ms / steps, tok_s=b * steps / (ms * 1e-3))
+    m.close()
+    return out
+
+
+def dense_cases(ctx, s, prefill=PREFILL, decode=DECODE, reps=3, steps=32, warmup=4):
+    out = {}
+    cfg = dict(syn.TINYLLAMA_1B, n_layers=s["layers"], d_model=s["width"], q_heads=s["heads"], kv_heads=s["kv_heads"],
+               head_dim=s["width"] // s["heads"], ffn=s["ff"], vocab=s["vocab"])
+    W = syn.make_weights(cfg, seed=0, unique_layers=1, tie_embeddings=True)
+    rng = np.random.default_rng(0)
+    slots = max([b for b, _ in decode] + [1])
+    length = max([c + steps + warmup + 8 for _, c in decode] + [n + 8 for n in prefill])
+    dm = syn.DeviceModel(ctx, cfg, W, max_seq_len=length, max_sequences=slots)
+    dm.set_mode(2)
+    dm.H.m40host_model_set_tie_guard(dm.h, -1.0)
+    for n in prefill:
+        prompt = rng.integers(0, s["vocab"], size=n).tolist()
+        best = None
+        for r in range(reps + 1):
+            t0 = time.perf_counter()
+            dm.forward_prefill([0], [prompt])
+            ms = (time.perf_counter() - t0) * 1e3
+            if r and (best is None or ms < best):
+                best = ms
+        out[f"prefill {n}"] = dict(ms=best, tok_s=n / (best * 1e-3))
+    for b, c in decode:
+        k = rng.standard_normal((c, cfg["kv_heads"], cfg["head_dim"]), dtype=np.float32).astype(np.float16).view(np.uint16)
+        dk = ctx.to_device(k)
+        for i in range(b):
+            for l in range(cfg["n_layers"]):
+                pkg.check(ctx.lib.m40llm_ext_kvcache_bulk_fill_f16(ctx.h, dm.kv_handle(), dm.H.m40host_model_kv_slot(dm.h, i, l), dk.ptr, dk.ptr, c),
+                          "m40llm_ext_kvcache_bulk_fill_f16")
+        try:
+            _, ms = dm.decode_batch_timed(np.arange(b), np.full(b, c), rng.integers(0, s["vocab"], size=b), warmup, steps)
+            out[f"decode {b} x {c}"] = dict(ms=ms / steps, tok_s=b * steps / (ms * 1e-3))
+        except RuntimeError as e:
+            out[f"decode {b} x {c}"] = dict(error=str(e))
+        dk.free()
+    dm.close()
+    return out
+
+
+def measure(ctx, shapes=None, steps=32, warmup=4, dense=True) -> dict:
+    out = {}
+    for name in shapes or SHAPES:
+        s = SHAPES[name]
+        out[name] = {"shape": {k: v for k, v in s.items() if k != "kv_heads"}, "pimosun": layered_cases(ctx, s, steps=steps, warmup=warmup)}
+        if dense:
+            out[name]["dense_kv_heads"] = s["kv_heads"]
+            out[name]["dense"] = dense_cases(ctx, s, steps=steps, warmup=warmup)
+    return out
