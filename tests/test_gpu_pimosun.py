@@ -1,0 +1,271 @@
+"""The Pimosun design through the framework's model folders, step function, paged cache and scheduler, against the plain
+restatement in oracle/latent_decoder.py: whole prompts, portions, single tokens, mixed batches, pages and slots used again."""
+import importlib
+
+import numpy as np
+import pytest
+
+pytestmark = pytest.mark.gpu
+
+from pimosun_common import CONFIGS, assert_logits, ld, layered, logits_error, m40, random_tensors, write_folder  # noqa: E402
+
+sch = importlib.import_module("m40-llm_amd.scheduler")
+DTYPES = ["float32", "bfloat16"]
+
+
+@pytest.fixture(scope="module")
+def ctx():
+    yield m40.Context(0)
+
+
+@pytest.fixture(scope="module")
+def folders(tmp_path_factory):
+    made = {}
+
+    def get(name, seed=3):
+        if name not in made:
+            cfg = CONFIGS[name]()
+            made[name] = write_folder(tmp_path_factory.mktemp("pimosun_" + name), cfg, random_tensors(cfg, seed))
+        return made[name]
+    return get
+
+
+@pytest.fixture(scope="module")
+def expected(folders):
+    """(tokens, logits [tokens][vocab], residuals [layers][tokens][width]) of a sequence of n tokens, computed whole."""
+    kept, models = {}, {}
+
+    def get(name, n, seed=0):
+        if (name, n, seed) not in kept:
+            m = models.setdefault(name, ld.Model.load(folders(name)))
+            t = np.random.default_rng(1000 * seed + n).integers(0, m.cfg["vocab"], size=n)
+            s = m.sequence()
+            kept[name, n, seed] = (t, s.feed(t.tolist()), np.stack(s.layer_outputs))
+        return kept[name, n, seed]
+    return get
+
+
+def open_model(ctx, folder, dtype, max_tokens=1024, slots=4, **kw):
+    return layered.LayeredModel.open(ctx, folder, dtype, max_tokens, slots, **kw)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name,n", [("odd", 150), ("even", 200), ("wide", 140), ("one", 70)])
+def test_residual_after_every_layer_and_logits_of_a_whole_prompt(ctx, folders, expected, name, n, dtype):
+    t, want, res = expected(name, n)
+    m = open_model(ctx, folders(name), dtype)
+    x = m.step_layers(0, t, *[res.shape[i] for i in (0, 2)])
+    for i in range(len(res)):
+        e = np.sqrt(((x[i] - res[i]) ** 2).mean(axis=-1)) / np.sqrt((res[i] ** 2).mean())
+        assert e.max() < {"float32": 1e-5, "bfloat16": 0.03}[dtype], (i, int(e.argmax()), float(e.max()))
+    m.release(0)
+    assert_logits(m.step([(1, t, range(n))]), want, dtype)
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name,n,first", [("odd", 135, 60), ("even", 200, 1), ("one", 70, 62)])
+def test_token_by_token_equals_the_whole_prompt(ctx, folders, expected, name, n, first, dtype):
+    t, want, _ = expected(name, n)
+    m = open_model(ctx, folders(name), dtype)
+    got = [m.step([(2, t[:first], range(first))])]
+    for i in range(first, n):
+        got.append(m.step([(2, t[i:i + 1], [0])]))
+    assert_logits(np.concatenate(got), want, dtype)
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name,n", [("odd", 330), ("wide", 330)])
+@pytest.mark.parametrize("cut", [[2], [3, 2, 61, 64, 66], [63, 1], [128, 5], [65], [200, 2]])
+def test_portions_of_any_size(ctx, folders, expected, name, n, cut, dtype):
+    t, want, _ = expected(name, n)
+    m = open_model(ctx, folders(name), dtype)
+    at, k, got = 0, 0, []
+    while at < n:
+        c = min(cut[k % len(cut)], n - at)
+        got.append(m.step([(0, t[at:at + c], range(c))]))
+        at, k = at + c, k + 1
+    assert_logits(np.concatenate(got), want, dtype, cut)
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("max_rows", [0, 7, 100])
+def test_mixed_batches_with_pages_and_slots_used_again(ctx, folders, expected, dtype, max_rows):
+    """Twelve sequences through four slots and a pool that holds four of them: portions of some beside single tokens of others,
+    sequences left out for a step, every position compared; then the pool is whole again."""
+    rng = np.random.default_rng(17)
+    lens = [5, 64, 65, 150, 127, 2, 129, 70, 1, 192, 128, 33]
+    m = open_model(ctx, folders("odd"), dtype, max_tokens=4 * 192, max_rows=max_rows)
+    free0 = m.free_pages()
+    waiting, live, free, errs = list(range(len(lens))), {}, [0, 1, 2, 3], {}
+    seqs = {i: expected("odd", n, seed=1 + i) for i, n in enumerate(lens)}
+    steps = 0
+    while waiting or live:
+        while waiting and free:
+            live[waiting.pop(0)] = [free.pop(rng.integers(len(free))), 0]
+        entries, rows = [], []
+        for i in rng.permutation(list(live)):
+            if len(live) > 1 and rng.random() < 0.2:
+                continue
+            slot, at = live[i]
+            t = seqs[i][0]
+            c = 1 if at > 0 and rng.random() < 0.5 else int(rng.integers(1, 90))
+            c = min(c, len(t) - at)
+            entries.append((slot, t[at:at + c], range(c)))
+            rows += [(i, at + k) for k in range(c)]
+            live[i][1] = at + c
+        if not entries:
+            continue
+        got = m.step(entries)
+        assert_logits(got, np.stack([seqs[i][1][p] for i, p in rows]), dtype, (steps, entries[0][0]))
+        for i in [i for i, (slot, at) in live.items() if at == lens[i]]:
+            slot, _ = live.pop(i)
+            m.release(slot)
+            free.append(slot)
+        steps += 1
+    assert m.free_pages() == free0
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_batch_of_unequal_requests_equals_each_alone(ctx, folders, expected, dtype):
+    m = open_model(ctx, folders("even"), dtype, max_tokens=1024)
+    lens = [200, 3, 129, 64]
+    seqs = [expected("even", n, seed=40) for n in lens]
+    alone = []
+    for t, _, _ in seqs:
+        alone.append(m.step([(0, t, range(len(t)))]))
+        m.release(0)
+    together = m.step([(i, t, range(len(t))) for i, (t, _, _) in enumerate(seqs)])
+    at = 0
+    for (t, want, _), a in zip(seqs, alone):
+        b = together[at:at + len(t)]
+        assert_logits(b, want, dtype)
+        assert logits_error(a, b.astype(np.float64)).max() < {"float32": 5e-6, "bfloat16": 0.02}[dtype]
+        at += len(t)
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_wanted_places_any_order_and_none(ctx, folders, expected, dtype):
+    t, want, _ = expected("odd", 135)
+    m = open_model(ctx, folders("odd"), dtype)
+    assert m.step([(0, t[:40], [])]).shape == (0, want.shape[1])
+    got = m.step([(0, t[40:], [94, 0, 3, 3])])
+    assert_logits(got, want[[134, 40, 43, 43]], dtype)
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_first_tokens_of_a_sequence_and_the_pair_table(ctx, folders, dtype):
+    """A first token takes the table's last row whatever ran in the slot before; the token before counts across a cut."""
+    model = ld.Model.load(folders("odd"))
+    m = open_model(ctx, folders("odd"), dtype)
+    for first in ([7], [0, 0], [100, 3, 100]):
+        want = model.sequence().feed(first)
+        assert_logits(m.step([(1, first[:1], [0])]), want[:1], dtype)
+        for i in range(1, len(first)):
+            assert_logits(m.step([(1, first[i:i + 1], [0])]), want[i:i + 1], dtype)
+        m.release(1)
+    m.close()
+
+
+def test_bad_steps_are_refused_and_change_nothing(ctx, folders, expected):
+    t, want, _ = expected("odd", 135)
+    m = open_model(ctx, folders("odd"), "float32", max_tokens=192, slots=2)
+    m.step([(0, t[:64], [])])
+    for bad in ([(0, [5000], [])], [(2, [1], [])], [(0, [1], [1])], [(0, [1], []), (0, [2], [])], [(0, [], [])],
+                [(1, list(range(100)) + [0] * 40, [])]):
+        with pytest.raises(RuntimeError):
+            m.step(bad)
+    m.release(1)
+    assert m.length(0) == 64
+    assert_logits(m.step([(0, t[64:], range(71))]), want[64:], "float32")
+    m.close()
+
+
+@pytest.mark.parametrize("dtype,mode", [("float32", 0), ("float32", 2), ("bfloat16", 2)])
+def test_long_greedy_decoding_equals_the_oracle(ctx, folders, dtype, mode):
+    """The device-driven loop (plain launches and replayed from a graph) over several page borders.  In 32-bit the ids are the
+    oracle's; in bf16 every pick is the oracle's best up to rounding."""
+    model = ld.Model.load(folders("odd"))
+    m = open_model(ctx, folders("odd"), dtype)
+    m.set_mode(mode)
+    prompt = np.random.default_rng(5).integers(0, 101, size=50).tolist()
+    ids, gaps = m.decode_greedy(0, prompt, 160)
+    s = model.sequence()
+    want = s.feed(ids[:-1].tolist())[len(prompt) - 1:]
+    pick = ids[len(prompt):]
+    if dtype == "float32":
+        assert np.array_equal(want.argmax(axis=1), pick)
+    behind = want.max(axis=1) - want[np.arange(len(pick)), pick]
+    assert behind.max() <= 4 * {"float32": 1e-4, "bfloat16": 0.03}[dtype] * np.std(want)
+    assert m.length(0) == len(prompt) + 159
+    # the loop's state carries on: the next token continues behind it
+    got = m.step([(0, ids[-1:], [0])])
+    assert_logits(got, s.feed(ids[-1:].tolist()), dtype, factor=2)
+    m.close()
+
+
+def test_greedy_batch_loop_on_any_slots_equals_single_sequences(ctx, folders):
+    m = open_model(ctx, folders("odd"), "float32")
+    rng = np.random.default_rng(6)
+    prompts = [rng.integers(0, 101, size=n).tolist() for n in (3, 63, 90)]
+    alone = []
+    for p in prompts:
+        ids, _ = m.decode_greedy(1, p, 40)
+        alone.append(ids[len(p):])
+        m.release(1)
+    slots = [3, 0, 2]
+    last = m.step([(s, p, [len(p) - 1]) for s, p in zip(slots, prompts)]).argmax(axis=1)
+    ids, _ = m.decode_batch_timed(slots, [len(p) for p in prompts], last, 5, 34)
+    for a, f, b in zip(alone, last, ids):
+        assert a.tolist() == [int(f)] + b.tolist()
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("max_rows,max_tokens", [(0, 1024), (24, 320)])
+def test_scheduler_serves_requests_as_each_alone(ctx, folders, dtype, max_rows, max_tokens):
+    """Arrivals over time, prompts cut by the tick's row limit, requests that wait for pages: every request generates what the
+    model generates for it alone, and (32-bit) what the oracle picks."""
+    m = open_model(ctx, folders("odd"), dtype, max_tokens=max_tokens, slots=3, max_rows=max_rows)
+    model = ld.Model.load(folders("odd"))
+    rng = np.random.default_rng(9)
+    specs = [(rng.integers(0, 101, size=n).tolist(), g) for n, g in ((9, 20), (130, 12), (64, 3), (1, 30), (77, 9), (40, 40))]
+    s = sch.Scheduler.for_model(m)
+    free0, rids, pending, ticks, mixed = m.free_pages(), {}, list(enumerate(specs)), 0, 0
+    while pending or s.active():
+        while pending and s.available_slots() and (ticks == 0 or ticks % 3 == 0):
+            i, (p, g) = pending.pop(0)
+            rids[i] = s.submit(p, max_tokens=g)
+        rep = s.tick()
+        mixed += bool(rep.prefill_rows and rep.decode_rows)
+        ticks += 1
+        assert ticks < 400
+    assert mixed > 0 and m.free_pages() == free0
+    for i, (p, g) in enumerate(specs):
+        assert s.state(rids[i]) == "complete", s.error(rids[i])
+        got = s.generated(rids[i])
+        assert len(got) == g
+        want = model.sequence().feed((p + got)[:-1])[len(p) - 1:]
+        if dtype == "float32":
+            assert want.argmax(axis=1).tolist() == got, i
+        behind = want.max(axis=1) - want[np.arange(g), got]
+        assert behind.max() <= 4 * {"float32": 1e-4, "bfloat16": 0.03}[dtype] * np.std(want), i
+    # sampled requests with one seed repeat themselves; a cancelled request gives its pages back
+    two = []
+    for _ in range(2):
+        r = s.submit(specs[0][0], max_tokens=12, temperature=0.9, top_k=20, top_p=0.95, seed=7)
+        s.run_until_idle()
+        two.append(s.generated(r))
+    assert two[0] == two[1] and len(set(two[0])) > 1
+    r = s.submit(specs[1][0], max_tokens=30)
+    s.tick(); s.tick()
+    assert s.cancel(r)
+    s.tick()
+    assert s.state(r) == "cancelled" and m.free_pages() == free0
+    s.close()
+    m.close()
