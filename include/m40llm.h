@@ -532,7 +532,8 @@ const char* m40llm_ext_build_info(void);
  * asynchronous on the stream stream_kind names.  act_dtype: 0 = bf16 activations (f32 sums), 1 = f32 throughout (products
  * on the f32 matrix instruction).  Weights are bf16 in packed tiles: a [N][K] matrix is ceil(N/16) x ceil(K/32) tiles of
  * 512 elements, row tile after row tile, zero past the matrix; the element order inside a tile is the operand order of
- * the 16x16x32 matrix instruction. */
+ * the 16x16x32 matrix instruction.  "Packed" activations ([rows][ld], ld a multiple of 32) lie in the same tiles, their
+ * memory a multiple of 16 rows. */
 #define M40LLM_ACT_BF16 0u
 #define M40LLM_ACT_F32 1u
 /* Source element (nb, n, kb, k) = src[nb*sn_block + n*sn + kb*sk_block + k*sk] goes to packed row
@@ -556,14 +557,21 @@ int m40llm_ext_clear_u32_async(M40llmCudaContext* ctx, void* d_dst, size_t n, ui
 #define M40LLM_PACKED_STORE 0u      /* out_f32[row][col] = v */
 #define M40LLM_PACKED_ADD 1u        /* out_f32[row][col] += v */
 #define M40LLM_PACKED_STORE_ACT 2u  /* out_act[row][col] = v */
-#define M40LLM_PACKED_GATED 3u      /* out_act[row][col] = v * sigmoid(gate[row][batch]) */
-#define M40LLM_PACKED_ROTATE 4u     /* heads of [plain | rotated] columns: pairs (2i, 2i+1) of the rotated part are rotated */
+#define M40LLM_PACKED_GATED 3u      /* out_act[row][batch*act_batch + col] = v * sigmoid(gate[row][batch]), packed */
+#define M40LLM_PACKED_ROTATE 4u     /* heads of [plain | rotated] columns: pairs (2i, 2i+1) of the rotated part are rotated;
+                                       out_act packed, rot_out (rows below split_row) plain */
 #define M40LLM_PACKED_PROJECT 5u    /* the first plain_tiles tiles: as STORE; then pairs of tiles (gate, up):
-                                       out_act[row][16*pair + c] = gelu_tanh(gate) * up */
+                                       out_act[row][act_col + 16*pair + c] = gelu_tanh(gate) * up, packed */
+/* bf16, rows read from cache pages (a = the layer's cache, pages = page numbers, rows = 64 * their number):
+ * KEYS: out_act = the result as a packed operand, 16-row tile after 16-row tile of n_tiles/2 k tiles;
+ * VALUES: out_act = the result transposed, per page and column tile two operand tiles [16 columns][32 rows], row
+ * 16t + 4g + r of 32 at place 8g + 4t + r (the order of m40llm_ext_head_attention_async) */
+#define M40LLM_PACKED_KEYS 6u
+#define M40LLM_PACKED_VALUES 7u
 typedef struct M40llmPackedGemm {
     uint32_t act_dtype, epilogue;
-    const void* a;                /* [rows][lda] activations, the columns past the matrix (to k_tiles*32) zero */
-    uint64_t lda, a_batch;        /* elements; lda a multiple of 8 */
+    const void* a;                /* packed [rows][lda] activations */
+    uint64_t lda, a_batch;        /* columns, multiples of 32 */
     const void* w;
     uint32_t n_tiles, k_tiles;
     uint64_t w_batch;             /* elements */
@@ -572,13 +580,16 @@ typedef struct M40llmPackedGemm {
     uint64_t ld_out, out_batch;
     void* out_act;
     uint64_t ld_act, act_batch;
-    uint32_t cols, plain_tiles;
+    uint32_t cols, plain_tiles, act_col;
     const void* gate;
     uint64_t ld_gate;
     uint32_t head_width, rot_start, heads, split_row, rot_half;
     const void* angles;
     void* rot_out;
     uint64_t ld_rot;
+    uint32_t k_parts;             /* STORE: K in that many parts, part p's sums at out_f32 + p*out_batch (0, 1 = whole) */
+    const uint32_t* pages;        /* KEYS, VALUES: device */
+    uint32_t page_k_tiles;        /* k tiles of a cache entry */
 } M40llmPackedGemm;
 int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm* g, uint32_t stream_kind);
 
@@ -587,11 +598,12 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
 int m40llm_ext_embed_pairs_async(M40llmCudaContext* ctx, const void* d_table_bf16, const void* d_pair_table_bf16,
                                  const uint32_t* d_tokens, const uint32_t* d_prev, uint32_t rows, uint32_t vocab, uint32_t width,
                                  uint32_t buckets, uint32_t mul_prev, uint32_t mul_cur, void* d_x_f32, uint32_t stream_kind);
-/* out[r] = layer norm of x[row_index ? row_index[r] : r] (mean taken off, eps inside the root, weight, no bias);
- * out has ld_out columns, those past width zero */
-int m40llm_ext_layer_norm_rows_async(M40llmCudaContext* ctx, const void* d_x_f32, const void* d_w_f32,
-                                     const uint32_t* d_row_index, uint32_t rows, uint32_t width, float eps, void* d_out,
-                                     uint32_t ld_out, uint32_t act_dtype, uint32_t stream_kind);
+/* out[r] = layer norm of x[row_index ? row_index[r] : r] (mean taken off, eps inside the root, weight, no bias), packed;
+ * out has ld_out columns, those past width zero.  n_planes > 0: x first takes the sum of as many planes of f32 rows, plane_stride
+ * elements apart and laid out like x; without row_index x keeps it. */
+int m40llm_ext_layer_norm_rows_async(M40llmCudaContext* ctx, void* d_x_f32, const void* d_planes_f32, uint32_t n_planes,
+                                     uint64_t plane_stride, const void* d_w_f32, const uint32_t* d_row_index, uint32_t rows,
+                                     uint32_t width, float eps, void* d_out, uint32_t ld_out, uint32_t act_dtype, uint32_t stream_kind);
 /* angles[row][i] = (cos, sin)(position * freq[i]) * magnitude for i < pairs, (1, 0) for pairs <= i < ld_pairs; the angle is
  * formed in double precision */
 int m40llm_ext_rotation_angles_async(M40llmCudaContext* ctx, const uint32_t* d_positions, uint32_t rows, const double* d_freq,
@@ -604,7 +616,7 @@ int m40llm_ext_rotation_angles_async(M40llmCudaContext* ctx, const uint32_t* d_p
  * finds its pages in page_table[s*max_pages + position/64]. */
 #define M40LLM_PAGE_TOKENS 64u
 /* From the projected row [q latent | kv latent | rotated key part | ...] (f32, parts padded to multiples of 16 / 32):
- * cq[row] = RMSNorm(q latent) (ld_cq columns, zero past q_rank), and where cache is not NULL RMSNorm(kv latent) and the
+ * cq[row] = RMSNorm(q latent) (packed, ld_cq columns, zero past q_rank), and where cache is not NULL RMSNorm(kv latent) and the
  * rotated key part go to the row's place in the cache. */
 typedef struct M40llmLatentSplit {
     uint32_t act_dtype, rows;
@@ -624,7 +636,7 @@ typedef struct M40llmLatentSplit {
 int m40llm_ext_latent_split_append_async(M40llmCudaContext* ctx, const M40llmLatentSplit* s, uint32_t stream_kind);
 /* Attention of query rows i = row*heads + head given in latent space (queries [rows*heads][entry_width]: W_uk^T q, then the
  * rotated part): score = q . entry * scale over the positions <= row_pos[row] of the row's slot, softmax whose denominator
- * also holds exp(sink[head]), result = weighted sum of the latents, out [rows*heads][latent_pad].
+ * also holds exp(sink[head]), result = weighted sum of the latents, out packed [rows][heads*latent_pad].
  * tiles[t] = {first query row, query rows}: all of one slot, at most 16*m_tiles.  splits > 1 divides the pages of a tile over
  * that many workgroups; partial sums go to `partial` (m40llm_ext_latent_attention_partial_floats) and are joined by a
  * second launch. */
@@ -647,6 +659,27 @@ int m40llm_ext_latent_attention_async(M40llmCudaContext* ctx, const M40llmLatent
 uint64_t m40llm_ext_latent_attention_partial_floats(uint32_t n_queries, uint32_t latent_pad, uint32_t splits);
 /* the largest m_tiles the kernels serve for an entry width (0 = the width is not served) */
 uint32_t m40llm_ext_latent_attention_max_m_tiles(uint32_t act_dtype, uint32_t kv_rank, uint32_t entry_width);
+/* The same attention for long portions, over keys and values brought out of the latents head by head.  pages: the page lists of the
+ * portions one behind the other; keys / values: what M40LLM_PACKED_KEYS / _VALUES write for that list (heads of 32*plain_tiles key
+ * columns, heads of 16*v_tiles value columns); the rotated key part (the last rot_tiles of a cache entry's entry_tiles) is
+ * read from the cache.  queries: packed [rows][ld_queries], per head [plain | rotated].  jobs[t] = {first row, rows (at most 128),
+ * first page of the portion's sequence in `pages`, 0}.  out[row][head*vdim + d], packed = result * sigmoid(gate[row][head]). */
+typedef struct M40llmHeadAttention {
+    uint32_t heads, plain_tiles, rot_tiles, entry_tiles, vdim, v_tiles;
+    float scale;
+    const void* queries;
+    uint32_t ld_queries;
+    const void *keys, *values, *cache, *sink;
+    const void* gate;
+    uint64_t ld_gate;
+    const uint32_t *row_pos, *pages, *jobs;
+    uint32_t n_jobs;
+    void* out;
+    uint32_t ld_out;
+} M40llmHeadAttention;
+int m40llm_ext_head_attention_async(M40llmCudaContext* ctx, const M40llmHeadAttention* a, uint32_t stream_kind);
+/* whether a head of as many 32-wide key tiles (plain and rotated) and 16-wide value tiles is served */
+int m40llm_ext_head_attention_serves(uint32_t k_tiles, uint32_t v_tiles);
 /* Greedy step of a device-driven decode loop: token r = picks[r] (gap[r] beside it) is recorded at ids[r*capacity + step] /
  * gaps[...], becomes the input token (prev = the token before), positions advance by one.  state[0] = step counter. */
 int m40llm_ext_advance_rows_async(M40llmCudaContext* ctx, const uint32_t* d_picks, const float* d_gap, uint32_t rows,

@@ -39,52 +39,109 @@ __device__ __forceinline__ float block_sum(float v, float* scratch) {
     return s;
 }
 
-template <class T>
-__global__ __launch_bounds__(kThreads) void layer_norm_rows_kernel(const float* __restrict__ x, const float* __restrict__ w,
+// A thread takes groups of eight neighbouring elements: 16-byte pieces of a packed tile.
+template <class T, bool VEC>
+__global__ __launch_bounds__(kThreads) void layer_norm_rows_kernel(float* __restrict__ x, const float* __restrict__ planes, uint32_t n_planes,
+                                                                   size_t plane_stride, const float* __restrict__ w,
                                                                    const uint32_t* __restrict__ row_index, uint32_t width, float eps,
                                                                    T* __restrict__ out, uint32_t ld_out) {
     __shared__ float scratch[kThreads / 64];
-    constexpr int kKeep = 16;            // elements a thread keeps in registers (width up to 4096)
-    const float* src = x + (size_t)(row_index ? row_index[blockIdx.x] : blockIdx.x) * width;
-    T* dst = out + (size_t)blockIdx.x * ld_out;
-    float keep[kKeep];
-    const bool kept = width <= (uint32_t)(kKeep * kThreads);
+    constexpr uint32_t kGroups = 2;      // groups a thread keeps in registers (width up to 4096); beyond, they are read again
+    const uint32_t out_row = m40_tile_row(blockIdx.x, gridDim.x);
+    const size_t at = (size_t)(row_index ? row_index[out_row] : out_row) * width;
+    const uint32_t groups = ld_out / 8u;
+    auto load = [&](uint32_t g, float (&v)[8]) __attribute__((always_inline)) {
+        auto add = [&](const float* src, bool first) __attribute__((always_inline)) {
+            if (VEC) {
+                const float4 a = reinterpret_cast<const float4*>(src + g * 8u)[0], b = reinterpret_cast<const float4*>(src + g * 8u)[1];
+                const float t[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
+#pragma unroll
+                for (int i = 0; i < 8; ++i) v[i] = first ? t[i] : v[i] + t[i];
+            } else {
+#pragma unroll
+                for (uint32_t i = 0; i < 8; ++i) {
+                    const float t = g * 8u + i < width ? src[g * 8u + i] : 0.0f;
+                    v[i] = first ? t : v[i] + t;
+                }
+            }
+        };
+        if (g * 8u >= width) {
+#pragma unroll
+            for (int i = 0; i < 8; ++i) v[i] = 0.0f;
+            return;
+        }
+        add(x + at, true);
+        for (uint32_t p = 0; p < n_planes; ++p) add(planes + p * plane_stride + at, false);
+    };
+    auto keep_sum = [&](uint32_t g, const float (&v)[8]) __attribute__((always_inline)) {      // x takes the planes' sums
+        if (n_planes == 0 || row_index || g * 8u >= width) return;
+        if (VEC) {
+            reinterpret_cast<float4*>(x + at + g * 8u)[0] = make_float4(v[0], v[1], v[2], v[3]);
+            reinterpret_cast<float4*>(x + at + g * 8u)[1] = make_float4(v[4], v[5], v[6], v[7]);
+        } else {
+#pragma unroll
+            for (uint32_t i = 0; i < 8; ++i)
+                if (g * 8u + i < width) x[at + g * 8u + i] = v[i];
+        }
+    };
+    float keep[kGroups][8];
     float s = 0.0f;
-    if (kept) {
+    auto sum8 = [&](const float (&v)[8]) __attribute__((always_inline)) {
 #pragma unroll
-        for (int j = 0; j < kKeep; ++j) {
-            const uint32_t i = threadIdx.x + j * kThreads;
-            keep[j] = i < width ? src[i] : 0.0f;
-            s += keep[j];
-        }
-    } else {
-        for (uint32_t i = threadIdx.x; i < width; i += kThreads) s += src[i];
-    }
-    const float mean = block_sum(s, scratch) / (float)width;
-    float q = 0.0f;
-    if (kept) {
+        for (int i = 0; i < 8; ++i) s += v[i];
+    };
+    float mean = 0.0f, q = 0.0f;
+    auto sq8 = [&](uint32_t g, const float (&v)[8]) __attribute__((always_inline)) {
 #pragma unroll
-        for (int j = 0; j < kKeep; ++j) {
-            const float d = threadIdx.x + j * kThreads < width ? keep[j] - mean : 0.0f;
+        for (uint32_t i = 0; i < 8; ++i) {
+            const float d = g * 8u + i < width ? v[i] - mean : 0.0f;
             q = fmaf(d, d, q);
         }
-    } else {
-        for (uint32_t i = threadIdx.x; i < width; i += kThreads) {
-            const float d = src[i] - mean;
-            q = fmaf(d, d, q);
-        }
-    }
-    const float inv = 1.0f / sqrtf(block_sum(q, scratch) / (float)width + eps);
-    if (kept) {
+    };
+    float inv = 0.0f;
+    auto store = [&](uint32_t g, const float (&v)[8]) __attribute__((always_inline)) {
+        T* o = out + m40_packed_at(out_row, g * 8u, ld_out >> 5);
+        m40_float4 lo, hi;
 #pragma unroll
-        for (int j = 0; j < kKeep; ++j) {
-            const uint32_t i = threadIdx.x + j * kThreads;
-            if (i < width) dst[i] = M40Act<T>::from((keep[j] - mean) * inv * w[i]);
+        for (uint32_t i = 0; i < 4; ++i) {
+            lo[i] = g * 8u + i < width ? (v[i] - mean) * inv * w[g * 8u + i] : 0.0f;
+            hi[i] = g * 8u + 4u + i < width ? (v[4 + i] - mean) * inv * w[g * 8u + 4u + i] : 0.0f;
         }
-    } else {
-        for (uint32_t i = threadIdx.x; i < width; i += kThreads) dst[i] = M40Act<T>::from((src[i] - mean) * inv * w[i]);
+        m40_store4<T>(o, lo);
+        m40_store4<T>(o + 4, hi);
+    };
+#pragma unroll
+    for (uint32_t j = 0; j < kGroups; ++j) {
+        const uint32_t g = threadIdx.x + j * kThreads;
+        load(g < groups ? g : groups, keep[j]);          // past the end: zeros
+        if (g < groups) keep_sum(g, keep[j]);
+        sum8(keep[j]);
     }
-    for (uint32_t i = width + threadIdx.x; i < ld_out; i += kThreads) dst[i] = M40Act<T>::from(0.0f);
+    for (uint32_t g = threadIdx.x + kGroups * kThreads; g < groups; g += kThreads) {
+        float v[8];
+        load(g, v);
+        sum8(v);
+    }
+    mean = block_sum(s, scratch) / (float)width;
+#pragma unroll
+    for (uint32_t j = 0; j < kGroups; ++j) sq8(threadIdx.x + j * kThreads, keep[j]);
+    for (uint32_t g = threadIdx.x + kGroups * kThreads; g < groups; g += kThreads) {
+        float v[8];
+        load(g, v);
+        sq8(g, v);
+    }
+    inv = 1.0f / sqrtf(block_sum(q, scratch) / (float)width + eps);
+#pragma unroll
+    for (uint32_t j = 0; j < kGroups; ++j) {
+        const uint32_t g = threadIdx.x + j * kThreads;
+        if (g < groups) store(g, keep[j]);
+    }
+    for (uint32_t g = threadIdx.x + kGroups * kThreads; g < groups; g += kThreads) {
+        float v[8];
+        load(g, v);
+        store(g, v);
+        keep_sum(g, v);
+    }
 }
 
 __global__ __launch_bounds__(kThreads) void rotation_angles_kernel(const uint32_t* __restrict__ positions, const double* __restrict__ freq,
@@ -105,14 +162,14 @@ __global__ __launch_bounds__(kThreads) void rotation_angles_kernel(const uint32_
 template <class T>
 __global__ __launch_bounds__(kThreads) void latent_split_append_kernel(M40llmLatentSplit a) {
     __shared__ float scratch[kThreads / 64];
-    const uint32_t row = blockIdx.x, tid = threadIdx.x;
+    const uint32_t row = m40_tile_row(blockIdx.x, a.rows), tid = threadIdx.x;
     const float* src = static_cast<const float*>(a.proj) + (size_t)row * a.ld_proj;
     float s = 0.0f;
     for (uint32_t i = tid; i < a.q_rank; i += kThreads) s = fmaf(src[i], src[i], s);
     const float q_inv = 1.0f / sqrtf(block_sum(s, scratch) / (float)a.q_rank + a.eps);
-    T* cq = static_cast<T*>(a.cq) + (size_t)row * a.ld_cq;
+    T* cq = static_cast<T*>(a.cq);
     const float* qw = static_cast<const float*>(a.q_norm);
-    for (uint32_t i = tid; i < a.ld_cq; i += kThreads) cq[i] = M40Act<T>::from(i < a.q_rank ? src[i] * q_inv * qw[i] : 0.0f);
+    for (uint32_t i = tid; i < a.ld_cq; i += kThreads) cq[m40_packed_at(row, i, a.ld_cq >> 5)] = M40Act<T>::from(i < a.q_rank ? src[i] * q_inv * qw[i] : 0.0f);
     if (!a.cache) return;
     const float* kv = src + a.kv_offset;
     s = 0.0f;
@@ -175,17 +232,24 @@ int m40llm_ext_embed_pairs_async(M40llmCudaContext* ctx, const void* d_table, co
     return launched();
 }
 
-int m40llm_ext_layer_norm_rows_async(M40llmCudaContext* ctx, const void* d_x, const void* d_w, const uint32_t* d_row_index, uint32_t rows,
-                                     uint32_t width, float eps, void* d_out, uint32_t ld_out, uint32_t act_dtype, uint32_t stream_kind) {
-    if (!ctx || !d_x || !d_w || !d_out) return -1;
+int m40llm_ext_layer_norm_rows_async(M40llmCudaContext* ctx, void* d_x, const void* d_planes, uint32_t n_planes, uint64_t plane_stride,
+                                     const void* d_w, const uint32_t* d_row_index, uint32_t rows, uint32_t width, float eps, void* d_out,
+                                     uint32_t ld_out, uint32_t act_dtype, uint32_t stream_kind) {
+    if (!ctx || !d_x || !d_w || !d_out || (n_planes && !d_planes)) return -1;
     hipStream_t stream = m40_select_stream(ctx, stream_kind);
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
-    if (rows == 0 || width == 0 || ld_out < width || act_dtype > 1u) return -3;
-    const float *x = static_cast<const float*>(d_x), *w = static_cast<const float*>(d_w);
-    if (act_dtype == M40LLM_ACT_F32)
-        layer_norm_rows_kernel<float><<<rows, kThreads, 0, stream>>>(x, w, d_row_index, width, eps, static_cast<float*>(d_out), ld_out);
-    else
-        layer_norm_rows_kernel<m40_bf16><<<rows, kThreads, 0, stream>>>(x, w, d_row_index, width, eps, static_cast<m40_bf16*>(d_out), ld_out);
+    if (rows == 0 || width == 0 || ld_out < width || ld_out % 32u != 0 || act_dtype > 1u || !m40_aligned16(d_out)) return -3;
+    float* x = static_cast<float*>(d_x);
+    const float *w = static_cast<const float*>(d_w), *p = static_cast<const float*>(d_planes);
+    const bool vec = width % 8u == 0 && plane_stride % 4u == 0 && m40_aligned16(d_x) && (!n_planes || m40_aligned16(d_planes));
+    auto go = [&](auto kernel, auto* out) { kernel<<<rows, kThreads, 0, stream>>>(x, p, n_planes, (size_t)plane_stride, w, d_row_index, width, eps, out, ld_out); };
+    if (act_dtype == M40LLM_ACT_F32) {
+        if (vec) go(layer_norm_rows_kernel<float, true>, static_cast<float*>(d_out));
+        else go(layer_norm_rows_kernel<float, false>, static_cast<float*>(d_out));
+    } else {
+        if (vec) go(layer_norm_rows_kernel<m40_bf16, true>, static_cast<m40_bf16*>(d_out));
+        else go(layer_norm_rows_kernel<m40_bf16, false>, static_cast<m40_bf16*>(d_out));
+    }
     return launched();
 }
 
@@ -205,7 +269,7 @@ int m40llm_ext_latent_split_append_async(M40llmCudaContext* ctx, const M40llmLat
     if (!ctx || !s || !s->proj || !s->q_norm || !s->cq) return -1;
     hipStream_t stream = m40_select_stream(ctx, stream_kind);
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
-    if (s->rows == 0 || s->q_rank == 0 || s->ld_cq < s->q_rank || s->act_dtype > 1u) return -3;
+    if (s->rows == 0 || s->q_rank == 0 || s->ld_cq < s->q_rank || s->ld_cq % 32u != 0 || s->act_dtype > 1u) return -3;
     if (s->cache && (!s->kv_norm || !s->angles || !s->row_slot || !s->row_pos || !s->page_table || s->kv_rank == 0 ||
                      s->latent_pad < s->kv_rank || s->latent_pad % 32u != 0 || s->entry_width % 32u != 0 ||
                      s->entry_width < s->latent_pad + s->rot_dim || s->rot_half * 2u < s->rot_dim))

@@ -1,13 +1,15 @@
-// Products of row-major activations with tile-packed bf16 weights (packed_gemm.hpp has the layout and the last steps).
+// Products of tile-packed activations with tile-packed bf16 weights (packed_gemm.hpp has the layout and the last steps).
 //
 // rows_packed_kernel   a workgroup owns one or two column tiles for up to 64 rows and its waves share out K: weights go
 //                      straight from memory into the matrix instruction's operand registers, one contiguous kilobyte a
 //                      load, each tile read once per 64 rows; the waves' sums meet in LDS.  Decode steps and short
 //                      portions, and every product in f32.
 // tile_packed_kernel   bf16, more rows: 128 x (128 or 256) tiles of C, both operands staged through LDS by direct
-//                      global-to-LDS loads, three stages of 64 k deep with one barrier a stage.  The stage buffers hold
+//                      global-to-LDS loads, five or six steps of 32 k deep with one barrier a step.  The buffers hold
 //                      operands in instruction order, so LDS reads are contiguous kilobytes as well.
 #include "packed_gemm.hpp"
+
+#include <type_traits>
 
 namespace {
 
@@ -16,6 +18,12 @@ struct PackedArgs {
     const m40_bf16* w;
     long lda, a_batch, w_batch;
     int n_tiles, k_tiles, rows;
+    int k_stride;                  // k tiles from one row tile of the weights to the next
+    int k_total;                   // k tiles of all batches together where the batches are parts of K (else 0)
+    // operand rows that lie in cache pages: row tile t is group t % 4 of page pages[t / 4]
+    const uint32_t* pages;
+    int page_k_tiles;
+    __device__ int k_count(int batch) const { return k_total && k_total - batch * k_tiles < k_tiles ? k_total - batch * k_tiles : k_tiles; }
 };
 
 template <class T, int MT, int NT, int WAVES>
@@ -27,15 +35,16 @@ __global__ __launch_bounds__(WAVES * 64) void rows_packed_kernel(PackedArgs g, M
     const T* a[MT];
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
-        const int row = row0 + m * 16 + (lane & 15);
-        a[m] = static_cast<const T*>(g.a) + batch * g.a_batch + (long)(row < g.rows ? row : g.rows - 1) * g.lda + (lane >> 4) * 8;
+        const int rt = row0 / 16 + m, last = (g.rows - 1) / 16;
+        a[m] = static_cast<const T*>(g.a) + batch * g.a_batch + (long)(rt < last ? rt : last) * 16 * g.lda + lane * 8;
     }
     const m40_bf16* w[NT];
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
         const int t = tile0 + n < g.n_tiles ? tile0 + n : g.n_tiles - 1;
-        w[n] = g.w + batch * g.w_batch + (long)t * g.k_tiles * kM40Tile + lane * 8;
+        w[n] = g.w + batch * g.w_batch + (long)t * g.k_stride * kM40Tile + lane * 8;
     }
+    const int k_tiles = g.k_count(batch);
     m40_float4 acc[MT][NT];
 #pragma unroll
     for (int m = 0; m < MT; ++m)
@@ -43,7 +52,7 @@ __global__ __launch_bounds__(WAVES * 64) void rows_packed_kernel(PackedArgs g, M
         for (int n = 0; n < NT; ++n) acc[m][n] = m40_float4{0.f, 0.f, 0.f, 0.f};
     constexpr int U = sizeof(T) == 2 ? (MT * NT <= 2 ? 8 : 4) : 1;
     int k = wave;
-    for (; k + (U - 1) * WAVES < g.k_tiles; k += U * WAVES) {
+    for (; k + (U - 1) * WAVES < k_tiles; k += U * WAVES) {
         uint4 wf[U][NT];
         vec8 af[U][MT];
 #pragma unroll
@@ -53,23 +62,23 @@ __global__ __launch_bounds__(WAVES * 64) void rows_packed_kernel(PackedArgs g, M
 #pragma unroll
         for (int u = 0; u < U; ++u)
 #pragma unroll
-            for (int m = 0; m < MT; ++m) af[u][m] = M40Act<T>::load8(a[m] + (k + u * WAVES) * 32);
+            for (int m = 0; m < MT; ++m) af[u][m] = M40Act<T>::load8(a[m] + (long)(k + u * WAVES) * kM40Tile);
 #pragma unroll
         for (int u = 0; u < U; ++u)
 #pragma unroll
             for (int m = 0; m < MT; ++m)
 #pragma unroll
-                for (int n = 0; n < NT; ++n) acc[m][n] = M40Act<T>::mma(af[u][m], __builtin_bit_cast(m40_bf16x8, wf[u][n]), acc[m][n]);
+                for (int n = 0; n < NT; ++n) acc[m][n] = M40Act<T>::mma(__builtin_bit_cast(m40_bf16x8, wf[u][n]), af[u][m], acc[m][n]);
     }
-    for (; k < g.k_tiles; k += WAVES) {
+    for (; k < k_tiles; k += WAVES) {
         uint4 wf[NT];
 #pragma unroll
         for (int n = 0; n < NT; ++n) wf[n] = *reinterpret_cast<const uint4*>(w[n] + (long)k * kM40Tile);
 #pragma unroll
         for (int m = 0; m < MT; ++m) {
-            const vec8 af = M40Act<T>::load8(a[m] + k * 32);
+            const vec8 af = M40Act<T>::load8(a[m] + (long)k * kM40Tile);
 #pragma unroll
-            for (int n = 0; n < NT; ++n) acc[m][n] = M40Act<T>::mma(af, __builtin_bit_cast(m40_bf16x8, wf[n]), acc[m][n]);
+            for (int n = 0; n < NT; ++n) acc[m][n] = M40Act<T>::mma(__builtin_bit_cast(m40_bf16x8, wf[n]), af, acc[m][n]);
         }
     }
     m40_float4* r4 = reinterpret_cast<m40_float4*>(red);
@@ -123,53 +132,59 @@ int launch_rows_any(hipStream_t stream, const PackedArgs& g, const M40Epilogue<T
 }
 
 // ---- many rows, bf16 ---------------------------------------------------------------------------------------------------
-// Workgroup of four waves (2 x 2), wave tile 64 x (16 NTW): C tile 128 x 32 NTW.  A stage is two k tiles of every operand
-// tile: (8 + 2 NTW) * 2 KB, filled by global_load_lds (a wave's instruction moves one 16 x 32 operand tile: for A the lanes
-// gather the rows' 16-byte pieces into instruction order, for W the tile is already contiguous).
-__device__ __forceinline__ constexpr int vm_wait(int n) { return 0x0f70 | (n & 15) | ((n >> 4) << 14); }
-constexpr int kStages = 3;
+// Workgroup of four waves (2 x 2), wave tile 64 x (16 NTW): C tile 128 x 32 NTW.  A step is one k tile of every operand
+// tile: (8 + 2 NTW) KB, filled by global_load_lds (a wave's instruction moves one 16 x 32 operand tile, a contiguous kilobyte).
+//
+// Memory instructions are issued under matrix instructions: the fragments of the next step and the loads of a step kBufs - 1
+// ahead go out one at a time between the current step's products (sched_group_barrier), so that no wave waits for an address
+// or LDS unit with the matrix pipe idle.  Step t refills the buffer of step t - 1, whose fragments every wave had in registers
+// before the barrier behind that step, and ends with step t + 2 landed.
+enum { kPlainRows = 0, kPageKeys = 1, kPageValues = 2 };
+constexpr int tile_bufs(int ntw) { return ntw == 8 ? 6 : 5; }       // one or two workgroups a CU
 
-template <int NTW>
+template <int NTW, int FORM>
 __global__ __launch_bounds__(256, 1) void tile_packed_kernel(PackedArgs g, M40Epilogue<m40_bf16> e) {
     typedef __attribute__((address_space(3))) void* lds_dst_t;
     typedef const __attribute__((address_space(1))) void* global_src_t;
     extern __shared__ __align__(16) uint8_t stage_lds[];
     constexpr int kATiles = 8, kBTiles = 2 * NTW;                    // 16-row operand tiles of the workgroup
-    constexpr int kStageBytes = (kATiles + kBTiles) * 2 * 1024;
-    constexpr int kLoads = (kATiles + kBTiles) * 2 / 4;              // per wave and stage
+    constexpr int kBufs = tile_bufs(NTW), kStepBytes = (kATiles + kBTiles) * 1024;
+    constexpr int kLoads = (kATiles + kBTiles) / 4;                  // per wave and step
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-    const int tiles_n = (g.n_tiles + kBTiles - 1) / kBTiles;
-    // workgroups are dealt to the eight dies in turn: each die gets a contiguous band of row tiles
+    const int tiles_n = (g.n_tiles + kBTiles - 1) / kBTiles, tiles_m = (g.rows + 127) / 128;
+    // workgroups are dealt to the eight dies in turn: each die gets a contiguous band of tiles, walked in blocks of four row
+    // tiles so that what runs on a die at one time shares both operands
     const int per_die = (int)gridDim.x / 8;
     const int logical = (int)blockIdx.x < per_die * 8 ? ((int)blockIdx.x % 8) * per_die + (int)blockIdx.x / 8 : (int)blockIdx.x;
-    const int m0 = logical / tiles_n * 128, t0 = logical % tiles_n * kBTiles, batch = blockIdx.z;
+    const int group = logical / (4 * tiles_n), in_group = logical - group * 4 * tiles_n, gm = tiles_m - group * 4 < 4 ? tiles_m - group * 4 : 4;
+    const int m0 = (group * 4 + in_group % gm) * 128, t0 = in_group / gm * kBTiles, batch = blockIdx.z;
     const m40_bf16* A = static_cast<const m40_bf16*>(g.a) + batch * g.a_batch;
     const m40_bf16* W = g.w + batch * g.w_batch;
-    // this wave's pieces of a stage: operand tiles wave, wave + 4, ... of the A tiles, then of the W tiles; both k tiles of each
-    const m40_bf16* src[kLoads / 2];
-    uint32_t dst[kLoads / 2];
+    const int k_tiles = g.k_count(batch);
+    // this wave's pieces of a step: operand tiles wave, wave + 4, ... of the A tiles, then of the W tiles
+    const m40_bf16* src[kLoads];
 #pragma unroll
-    for (int i = 0; i < kLoads / 2; ++i) {
+    for (int i = 0; i < kLoads; ++i) {
         const int t = wave + 4 * i;
         if (i < kATiles / 4) {
-            const int row = m0 + t * 16 + (lane & 15);
-            src[i] = A + (long)(row < g.rows ? row : g.rows - 1) * g.lda + (lane >> 4) * 8;
+            if (FORM != kPlainRows) {
+                const int rt = m0 / 16 + t, tiles = g.rows / 16, c = rt < tiles ? rt : tiles - 1;
+                src[i] = A + ((long)g.pages[c >> 2] * 4 + (c & 3)) * g.page_k_tiles * kM40Tile + lane * 8;
+            } else {
+                const int rt = m0 / 16 + t, last = (g.rows - 1) / 16;
+                src[i] = A + (long)(rt < last ? rt : last) * 16 * g.lda + lane * 8;
+            }
         } else {
             const int n = t0 + t - kATiles;
-            src[i] = W + (long)(n < g.n_tiles ? n : g.n_tiles - 1) * g.k_tiles * kM40Tile + lane * 8;
+            src[i] = W + (long)(n < g.n_tiles ? n : g.n_tiles - 1) * g.k_stride * kM40Tile + lane * 8;
         }
-        dst[i] = t * 2048;
     }
-    const int stages = (g.k_tiles + 1) / 2;
-    auto issue = [&](int buf, int s) {
-        uint8_t* base = stage_lds + buf * kStageBytes;
-        const int k0 = 2 * s, k1 = k0 + 1 < g.k_tiles ? k0 + 1 : k0;     // an odd last k tile is loaded twice, used once
+    auto issue = [&](int buf, int t) __attribute__((always_inline)) {
+        uint8_t* base = stage_lds + buf * kStepBytes + wave * 1024;
+        const int k = t < k_tiles ? t : k_tiles - 1;                 // past the end: loaded again, not used
 #pragma unroll
-        for (int i = 0; i < kLoads / 2; ++i) {
-            const int step = i < kATiles / 4 ? 32 : kM40Tile;
-            __builtin_amdgcn_global_load_lds((global_src_t)(src[i] + (long)k0 * step), (lds_dst_t)(base + dst[i]), 16, 0, 0);
-            __builtin_amdgcn_global_load_lds((global_src_t)(src[i] + (long)k1 * step), (lds_dst_t)(base + dst[i] + 1024), 16, 0, 0);
-        }
+        for (int i = 0; i < kLoads; ++i)
+            __builtin_amdgcn_global_load_lds((global_src_t)(src[i] + (long)k * kM40Tile), (lds_dst_t)(base + i * 4096), 16, 0, 0);
     };
     const int wm = wave >> 1, wn = wave & 1;
     m40_float4 acc[4][NTW];
@@ -177,62 +192,111 @@ __global__ __launch_bounds__(256, 1) void tile_packed_kernel(PackedArgs g, M40Ep
     for (int i = 0; i < 4; ++i)
 #pragma unroll
         for (int j = 0; j < NTW; ++j) acc[i][j] = m40_float4{0.f, 0.f, 0.f, 0.f};
-    auto compute = [&](const uint8_t* base, int kk) {
-        const uint8_t* a = base + wm * 4 * 2048 + kk * 1024 + lane * 16;
-        const uint8_t* b = base + (kATiles + wn * NTW) * 2048 + kk * 1024 + lane * 16;
-        m40_bf16x8 af[4], bf[NTW];
+    struct Frags { m40_bf16x8 a[4], b[NTW]; } f[2];
+    auto read_frags = [&](Frags& f, int buf) __attribute__((always_inline)) {
+        const uint8_t* a = stage_lds + buf * kStepBytes + wm * 4096 + lane * 16;
+        const uint8_t* b = stage_lds + buf * kStepBytes + (kATiles + wn * NTW) * 1024 + lane * 16;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) af[i] = *reinterpret_cast<const m40_bf16x8*>(a + i * 2048);
+        for (int i = 0; i < 4; ++i) f.a[i] = *reinterpret_cast<const m40_bf16x8*>(a + i * 1024);
 #pragma unroll
-        for (int j = 0; j < NTW; ++j) bf[j] = *reinterpret_cast<const m40_bf16x8*>(b + j * 2048);
+        for (int j = 0; j < NTW; ++j) f.b[j] = *reinterpret_cast<const m40_bf16x8*>(b + j * 1024);
+    };
+    auto compute = [&](const Frags& f) __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < 4; ++i)
 #pragma unroll
-            for (int j = 0; j < NTW; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(af[i], bf[j], acc[i][j], 0, 0, 0);
+            for (int j = 0; j < NTW; ++j)
+                acc[i][j] = FORM == kPageValues ? __builtin_amdgcn_mfma_f32_16x16x32_bf16(f.a[i], f.b[j], acc[i][j], 0, 0, 0)
+                                                : __builtin_amdgcn_mfma_f32_16x16x32_bf16(f.b[j], f.a[i], acc[i][j], 0, 0, 0);
     };
-    issue(0, 0);
-    issue(1, 1 < stages ? 1 : stages - 1);
+#pragma unroll
+    for (int i = 0; i < kBufs - 1; ++i) issue(i, i);
+    m40_wait_and_meet<(kBufs - 3) * kLoads>();                       // steps 0 and 1 have landed
+    read_frags(f[0], 0);
     int buf = 0;
-    for (int s = 0; s < stages; ++s) {
-        // stage s is in LDS once at most the newest stage's loads are outstanding; behind the barrier every wave's are, and
-        // every wave is done with stage s - 1, whose buffer takes stage s + 2
-        __builtin_amdgcn_sched_barrier(0);
-        __builtin_amdgcn_s_waitcnt(vm_wait(kLoads));
-        __builtin_amdgcn_s_barrier();
-        __builtin_amdgcn_sched_barrier(0);
-        issue(buf == 0 ? 2 : buf - 1, s + 2 < stages ? s + 2 : stages - 1);
-        const uint8_t* base = stage_lds + buf * kStageBytes;
-        compute(base, 0);
-        if (2 * s + 1 < g.k_tiles) compute(base, 1);
-        buf = buf == kStages - 1 ? 0 : buf + 1;
+    auto step = [&](auto parity, int t) __attribute__((always_inline)) {
+        constexpr int ph = decltype(parity)::value;
+        const int next = buf == kBufs - 1 ? 0 : buf + 1;
+        read_frags(f[ph ^ 1], next);
+        issue(buf == 0 ? kBufs - 1 : buf - 1, t + kBufs - 1);
+        compute(f[ph]);
+        constexpr int kPer = 4 * NTW / (4 + NTW);                    // products per fragment read
+#pragma unroll
+        for (int i = 0; i < 4 + NTW; ++i) {
+            __builtin_amdgcn_sched_group_barrier(0x008, kPer, 0);
+            __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+            if (i % 2 == 0) __builtin_amdgcn_sched_group_barrier(0x020, 1, 0);
+        }
+        m40_wait_and_meet<(kBufs - 3) * kLoads>();
+        buf = next;
+    };
+    int t = 0;
+    for (; t + 2 <= k_tiles; t += 2) {
+        step(std::integral_constant<int, 0>(), t);
+        step(std::integral_constant<int, 1>(), t + 1);
     }
-    __builtin_amdgcn_s_waitcnt(vm_wait(0));        // no write into LDS may be outstanding when the workgroup ends
+    if (t < k_tiles) compute(f[0]);
+    m40_wait_and_meet<0>();                                          // every load has landed: the buffers are free
+    // The sums go through LDS (each wave its own) so that the last step is a loop of a few instructions and not 4 NTW copies of it:
+    // run once per workgroup, those would be fetched cold.
+    m40_float4* mine = reinterpret_cast<m40_float4*>(stage_lds) + wave * 4 * NTW * 64 + lane;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        const int row0 = m0 + (wm * 4 + i) * 16;
-        if (row0 >= g.rows) continue;
+    for (int i = 0; i < 4; ++i)
 #pragma unroll
-        for (int j = 0; j < NTW; j += 2) {
-            const int tile = t0 + wn * NTW + j;
-            if (e.kind == M40LLM_PACKED_PROJECT && tile >= e.plain_tiles) {
-                if (tile + 1 < g.n_tiles) m40_epilogue_pair(e, row0, (tile - e.plain_tiles) / 2, lane, acc[i][j], acc[i][j + 1]);
-            } else {
-                if (tile < g.n_tiles) m40_epilogue_tile(e, batch, row0, tile, lane, acc[i][j]);
-                if (tile + 1 < g.n_tiles) m40_epilogue_tile(e, batch, row0, tile + 1, lane, acc[i][j + 1]);
+        for (int j = 0; j < NTW; ++j) mine[(i * NTW + j) * 64] = acc[i][j];
+    if (FORM == kPlainRows && e.kind == M40LLM_PACKED_ADD && e.vec_out && e.cols % 16 == 0) {
+        // the old values of four tiles are requested together, under clamped addresses: loads behind a branch would be awaited one by one
+#pragma unroll 1
+        for (int i = 0; i < NTW; ++i) {
+            const int row = m0 + (wm * 4 + i * 4 / NTW) * 16 + (lane & 15), j0 = i * 4 % NTW;
+            float* o = e.out_f32 + batch * e.out_batch + (long)(row < e.rows ? row : e.rows - 1) * e.ld_out + 4 * (lane >> 4);
+            m40_float4 old[4];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int col = (t0 + wn * NTW + j0 + j) * 16;
+                old[j] = *reinterpret_cast<const m40_float4*>(o + (col < e.cols ? col : 0));
             }
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int col = (t0 + wn * NTW + j0 + j) * 16;
+                if (row < e.rows && col < e.cols) *reinterpret_cast<m40_float4*>(o + col) = old[j] + mine[(i * 4 + j) * 64];
+            }
+        }
+        return;
+    }
+#pragma unroll 1
+    for (int p = 0; p < 2 * NTW; ++p) {
+        const int i = p / (NTW / 2), j = p % (NTW / 2) * 2, row0 = m0 + (wm * 4 + i) * 16, tile = t0 + wn * NTW + j;
+        if (row0 >= g.rows || tile >= g.n_tiles) continue;
+        const m40_float4 v0 = mine[(2 * p) * 64], v1 = mine[(2 * p + 1) * 64];
+        const bool second = tile + 1 < g.n_tiles;
+        if (FORM == kPageValues) {
+            m40_epilogue_values(e, row0, tile, lane, v0);
+            if (second) m40_epilogue_values(e, row0, tile + 1, lane, v1);
+        } else if (e.kind == M40LLM_PACKED_PROJECT && tile >= e.plain_tiles) {
+            if (second) m40_epilogue_pair(e, row0, (tile - e.plain_tiles) / 2, lane, v0, v1);
+        } else {
+#pragma unroll 1
+            for (int k = 0; k < (second ? 2 : 1); ++k) m40_epilogue_tile(e, batch, row0, tile + k, lane, k ? v1 : v0);
         }
     }
 }
 
-template <int NTW>
+template <int NTW, int FORM>
 int launch_tile(hipStream_t stream, const PackedArgs& g, const M40Epilogue<m40_bf16>& e, int batches) {
-    constexpr int lds = (8 + 2 * NTW) * 2 * 1024 * kStages;
-    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(tile_packed_kernel<NTW>),
+    constexpr int lds = (8 + 2 * NTW) * 1024 * tile_bufs(NTW);
+    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(tile_packed_kernel<NTW, FORM>),
                                                        hipFuncAttributeMaxDynamicSharedMemorySize, lds);
     if (attr != hipSuccess) return -2;
     const long long tiles = (long long)((g.rows + 127) / 128) * ((g.n_tiles + 2 * NTW - 1) / (2 * NTW));
-    tile_packed_kernel<NTW><<<dim3((unsigned)tiles, 1, (unsigned)batches), 256, lds, stream>>>(g, e);
+    tile_packed_kernel<NTW, FORM><<<dim3((unsigned)tiles, 1, (unsigned)batches), 256, lds, stream>>>(g, e);
     return hipGetLastError() == hipSuccess ? 0 : -2;
+}
+template <int FORM>
+int launch_tile_any(hipStream_t stream, const PackedArgs& g, const M40Epilogue<m40_bf16>& e, int batches, int num_cus) {
+    const long long wide = (long long)((g.rows + 127) / 128) * ((g.n_tiles + 15) / 16) * batches;
+    if (wide * 16 >= 9ll * num_cus) return launch_tile<8, FORM>(stream, g, e, batches);
+    return launch_tile<4, FORM>(stream, g, e, batches);
 }
 
 template <class T>
@@ -245,7 +309,11 @@ M40Epilogue<T> make_epilogue(const M40llmPackedGemm& p) {
     e.ld_out = (long)p.ld_out; e.ld_act = (long)p.ld_act;
     e.out_batch = (long)p.out_batch; e.act_batch = (long)p.act_batch;
     e.cols = (int)p.cols;
+    auto aligned = [](const void* q, size_t n) { return reinterpret_cast<uintptr_t>(q) % n == 0; };
+    e.vec_out = p.ld_out % 4 == 0 && p.out_batch % 4 == 0 && aligned(p.out_f32, 16);
+    e.vec_act = p.ld_act % 4 == 0 && p.act_batch % 4 == 0 && aligned(p.out_act, 4 * sizeof(T));
     e.plain_tiles = (int)p.plain_tiles;
+    e.n_tiles = (int)p.n_tiles; e.act_col = (int)p.act_col;
     e.gate = static_cast<const float*>(p.gate);
     e.ld_gate = (long)p.ld_gate;
     e.head_width = (int)p.head_width; e.rot_start = (int)p.rot_start; e.heads = (int)p.heads;
@@ -328,10 +396,19 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
     if (!ctx || !p || !p->a || !p->w) return -1;
     hipStream_t stream = m40_select_stream(ctx, stream_kind);
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
-    if (p->act_dtype > 1u || p->epilogue > M40LLM_PACKED_PROJECT || p->rows == 0 || p->batches == 0 || p->batches > 65535u ||
-        p->n_tiles == 0 || p->k_tiles == 0 || p->lda % 8 != 0 || p->lda < (uint64_t)p->k_tiles * 32u || !m40_aligned16(p->a) ||
-        !m40_aligned16(p->w) || p->rows > 0x3fffffffu || (p->batches > 1u && (p->a_batch % 8 != 0 || p->w_batch % 8 != 0)))
+    const bool paged = p->epilogue == M40LLM_PACKED_KEYS || p->epilogue == M40LLM_PACKED_VALUES;
+    const uint32_t k_parts = p->k_parts > 1u ? p->k_parts : 1u, part_tiles = (p->k_tiles + k_parts - 1) / k_parts;
+    if (p->act_dtype > 1u || p->epilogue > M40LLM_PACKED_VALUES || p->rows == 0 || p->batches == 0 || p->batches > 65535u ||
+        p->n_tiles == 0 || p->k_tiles == 0 || !m40_aligned16(p->a) || !m40_aligned16(p->w) || p->rows > 0x3fffffffu ||
+        (p->batches > 1u && (p->a_batch % 32 != 0 || p->w_batch % 8 != 0)))
         return -3;
+    if (!paged && (p->lda % 32 != 0 || p->lda < (uint64_t)p->k_tiles * 32u)) return -3;
+    if (k_parts > 1u && (p->epilogue != M40LLM_PACKED_STORE || p->batches != 1u || (k_parts - 1) * part_tiles >= p->k_tiles)) return -3;
+    // packed results: whole tiles of columns
+    if ((p->epilogue == M40LLM_PACKED_GATED || p->epilogue == M40LLM_PACKED_ROTATE || (p->epilogue == M40LLM_PACKED_PROJECT && p->out_act)) &&
+        (p->ld_act % 32 != 0 || p->act_col % 4 != 0))
+        return -3;
+    const bool wide_stores = p->ld_act % 4 == 0 && reinterpret_cast<uintptr_t>(p->out_act) % (p->act_dtype == M40LLM_ACT_F32 ? 16 : 8) == 0;
     switch (p->epilogue) {
         case M40LLM_PACKED_STORE: case M40LLM_PACKED_ADD: if (!p->out_f32 || p->cols > p->n_tiles * 16u) return -4; break;
         case M40LLM_PACKED_STORE_ACT: if (!p->out_act || p->cols > p->n_tiles * 16u) return -4; break;
@@ -339,30 +416,45 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
         case M40LLM_PACKED_ROTATE:
             if (!p->out_act || !p->angles || p->head_width == 0 || p->head_width % 32 != 0 || p->rot_start % 32 != 0 ||
                 p->rot_start >= p->head_width || p->rot_half * 2u != p->head_width - p->rot_start ||
-                p->heads * p->head_width != p->n_tiles * 16u || (p->split_row > 0 && !p->rot_out))
+                p->heads * p->head_width != p->n_tiles * 16u || !wide_stores || !m40_aligned16(p->angles) ||
+                (p->split_row > 0 && (!p->rot_out || p->ld_rot % 4 != 0 ||
+                                      reinterpret_cast<uintptr_t>(p->rot_out) % (p->act_dtype == M40LLM_ACT_F32 ? 16 : 8) != 0)))
                 return -4;
             break;
         case M40LLM_PACKED_PROJECT:
-            if ((p->plain_tiles > 0 && !p->out_f32) || (p->n_tiles > p->plain_tiles && !p->out_act) || p->plain_tiles % 2 != 0 ||
-                p->n_tiles % 2 != 0 || p->plain_tiles > p->n_tiles)
+            if ((p->plain_tiles > 0 && !p->out_f32) || (p->n_tiles > p->plain_tiles && (!p->out_act || !wide_stores)) ||
+                p->plain_tiles % 2 != 0 || p->n_tiles % 2 != 0 || p->plain_tiles > p->n_tiles)
+                return -4;
+            break;
+        case M40LLM_PACKED_KEYS: case M40LLM_PACKED_VALUES:
+            if (!p->out_act || !m40_aligned16(p->out_act) || !p->pages || p->page_k_tiles < p->k_tiles || p->batches != 1u ||
+                p->act_dtype != M40LLM_ACT_BF16 || p->rows % M40LLM_PAGE_TOKENS != 0 ||
+                (p->epilogue == M40LLM_PACKED_KEYS && p->n_tiles % 2 != 0))
                 return -4;
             break;
     }
     PackedArgs g{};
     g.a = p->a;
     g.w = static_cast<const m40_bf16*>(p->w);
-    g.lda = (long)p->lda; g.a_batch = (long)p->a_batch; g.w_batch = (long)p->w_batch;
-    g.n_tiles = (int)p->n_tiles; g.k_tiles = (int)p->k_tiles; g.rows = (int)p->rows;
+    g.lda = (long)p->lda; g.a_batch = (long)p->a_batch * 16; g.w_batch = (long)p->w_batch;
+    g.n_tiles = (int)p->n_tiles; g.k_tiles = (int)p->k_tiles; g.rows = (int)p->rows; g.k_stride = (int)p->k_tiles;
+    g.pages = p->pages; g.page_k_tiles = (int)p->page_k_tiles;
+    int batches = (int)p->batches;
+    if (k_parts > 1u) {
+        g.k_total = (int)p->k_tiles; g.k_tiles = (int)part_tiles;
+        g.a_batch = (long)part_tiles * kM40Tile; g.w_batch = (long)part_tiles * kM40Tile;
+        batches = (int)k_parts;
+    }
     (void)hipGetLastError();
     if (p->act_dtype == M40LLM_ACT_F32) {
         if ((g.rows + 63) / 64 > 65535) return -3;
-        return launch_rows_any<float>(stream, g, make_epilogue<float>(*p), (int)p->batches);
+        return launch_rows_any<float>(stream, g, make_epilogue<float>(*p), batches);
     }
     const M40Epilogue<m40_bf16> e = make_epilogue<m40_bf16>(*p);
-    if (g.rows <= 64) return launch_rows_any<m40_bf16>(stream, g, e, (int)p->batches);
-    const long long wide = (long long)((g.rows + 127) / 128) * ((g.n_tiles + 15) / 16) * p->batches;
-    if (wide * 16 >= 9ll * ctx->num_cus) return launch_tile<8>(stream, g, e, (int)p->batches);
-    return launch_tile<4>(stream, g, e, (int)p->batches);
+    if (p->epilogue == M40LLM_PACKED_KEYS) return launch_tile_any<kPageKeys>(stream, g, e, batches, ctx->num_cus);
+    if (p->epilogue == M40LLM_PACKED_VALUES) return launch_tile_any<kPageValues>(stream, g, e, batches, ctx->num_cus);
+    if (g.rows <= 64) return launch_rows_any<m40_bf16>(stream, g, e, batches);
+    return launch_tile_any<kPlainRows>(stream, g, e, batches, ctx->num_cus);
 }
 
 }  // extern "C"

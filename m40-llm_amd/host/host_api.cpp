@@ -77,6 +77,7 @@ LayeredOptions to_options(const M40HostModelOptions* o) {
     if (o->max_tokens) r.max_tokens = o->max_tokens;
     if (o->max_sequences) r.max_sequences = o->max_sequences;
     if (o->max_rows) r.max_rows = o->max_rows;
+    r.portion_form = o->portion_form;
     return r;
 }
 

@@ -7,10 +7,16 @@
 //   packed product, PROJECT         [q latent | kv latent | rotated key | gate logits] -> f32, gelu(gate) * up -> bf16
 //   latent split                    norms of the two latents, key rotation, cache append
 //   packed product, ROTATE          queries from their latent, rotated part turned in the last step
+// then for the rows of decoded tokens and short portions
 //   packed product per head         queries into latent space (W_uk^T)
 //   latent attention (+ join)       over the pages, sink in the denominator
 //   packed product per head, GATED  values from latent sums (W_uv), times the head's gate
-//   packed product, ADD             x += [W_o | W_down] [attention ; feed-forward]
+// and for the rows of long portions, where bringing a sequence's keys and values out of the latents costs less than it saves
+//   page products, KEYS and VALUES  the heads' keys and values of the portions' sequences
+//   head attention                  causal, sink, times the head's gate
+// and for all rows
+//   packed product, ADD             x += [W_o | W_down] [attention ; feed-forward]; small launches store the sums of parts of K
+//                                   instead, and the next norm adds them
 #pragma once
 
 #include <algorithm>
@@ -36,6 +42,7 @@ struct LayeredOptions {
     uint32_t max_tokens = 4096;        // what the cache pool holds, in tokens
     uint32_t max_sequences = 4;
     uint32_t max_rows = 4096;          // rows of one pass; longer steps run in several
+    uint32_t portion_form = 0;         // attention of portions: 0 the cheaper, 1 in latent space, 2 head by head where it is served
 };
 
 struct StepEntry {
@@ -50,6 +57,7 @@ class LayeredDecoder : public ServedModel {
 public:
     static constexpr uint32_t kStream = M40LLM_STREAM_DECODE;
     static constexpr uint32_t kPage = M40LLM_PAGE_TOKENS;
+    static constexpr uint32_t kCus = 256, kMaxParts = 8;
 
     LayeredDecoder(M40llmCudaContext* ctx, DecoderSpec spec, TensorSource& tensors, const LayeredOptions& opt)
         : ctx_(ctx), spec_(std::move(spec)), opt_(opt), es_(opt.act_dtype == M40LLM_ACT_F32 ? 4u : 2u),
@@ -105,12 +113,23 @@ public:
         std::vector<uint32_t> done(entries.size(), 0);
         size_t first = 0;
         while (first < entries.size()) {
+            struct Piece { size_t entry; uint32_t n; bool per_head; };
+            std::vector<Piece> pieces;
+            uint32_t taken = 0;
+            for (size_t i = first; i < entries.size() && taken < opt_.max_rows; ++i) {
+                const uint32_t n = std::min(entries[i].n - done[i], opt_.max_rows - taken);
+                pieces.push_back({i, n, per_head(n, seqs_.length(entries[i].sequence))});
+                taken += n;
+            }
+            // rows whose attention runs in latent space come first
+            std::stable_partition(pieces.begin(), pieces.end(), [](const Piece& p) { return !p.per_head; });
             PassPlan plan;
-            for (size_t i = first; i < entries.size() && plan.rows() < opt_.max_rows; ++i) {
+            for (const Piece& piece : pieces) {
+                const size_t i = piece.entry;
                 const StepEntry& e = entries[i];
-                const uint32_t n = std::min(e.n - done[i], opt_.max_rows - plan.rows());
-                const uint32_t len = seqs_.length(e.sequence);
-                plan.portions.push_back({plan.rows(), n});
+                const uint32_t n = piece.n, len = seqs_.length(e.sequence);
+                if (!piece.per_head) plan.latent_rows += n;
+                plan.portions.push_back({plan.rows(), n, e.sequence, len + n, piece.per_head});
                 for (uint32_t k = 0; k < e.n_want; ++k)
                     if (e.want[k] >= done[i] && e.want[k] < done[i] + n) {
                         plan.want.push_back(plan.rows() + e.want[k] - done[i]);
@@ -201,7 +220,7 @@ private:
         int rotation;                         // index into rotations_
         int tile_set;                         // index into tile_sets_
         float scale;
-        DeviceBuf norm1, w_proj, q_norm, kv_norm, w_uq, w_ukt, w_uv, sink, w_out, cache;
+        DeviceBuf norm1, w_proj, q_norm, kv_norm, w_uq, w_ukt, w_uk, w_uv, sink, w_out, cache;
     };
     struct Rotation {
         RotationSpec spec;
@@ -211,17 +230,22 @@ private:
     struct TileSet {
         uint32_t heads, max_m_tiles, latent_pad;
     };
-    struct Portion { uint32_t row, n; };
+    struct Portion { uint32_t row, n, slot, length; bool per_head; };      // length: tokens its sequence holds at its end
     struct PassPlan {
         std::vector<uint32_t> tokens, prev, slot, pos, want;
         std::vector<size_t> want_out;
         std::vector<Portion> portions;
+        uint32_t latent_rows = 0;
         uint32_t rows() const { return (uint32_t)tokens.size(); }
     };
     // device addresses of a pass
     struct Rows {
         uint32_t rows = 0;
+        bool in_place = false;                // every layer leaves its result in x
         uint32_t *tokens = nullptr, *prev = nullptr, *slot = nullptr, *pos = nullptr, *page_table = nullptr;
+        uint32_t latent_rows = 0;             // rows before it: attention in latent space; from it on: head by head
+        const uint32_t *jobs = nullptr, *page_list = nullptr;
+        uint32_t n_jobs = 0, n_pages = 0;
         struct Tiles { const uint32_t* table = nullptr; uint32_t n = 0, m_tiles = 1, splits = 1; };
         std::vector<Tiles> tiles;             // one per tile set
     };
@@ -270,6 +294,10 @@ private:
     }
 
     void load(TensorSource& t) {
+        per_head_served_ = opt_.act_dtype == M40LLM_ACT_BF16 && opt_.portion_form != 1u;
+        for (const LayerSpec& s : spec_.layers)
+            per_head_served_ = per_head_served_ && m40llm_ext_head_attention_serves((round_up(s.mixer.dim, 32) + round_up(s.mixer.rot_dim, 32)) / 32,
+                                                                                    round_up(s.mixer.vdim, 16) / 16);
         const uint32_t D = spec_.width, d_tiles = round_up(D, 32) / 32;
         embed_ = DeviceBuf(ctx_, (size_t)spec_.vocab * D * 2);
         t.read_bf16(ctx_, "embed", {spec_.vocab, D}, embed_.ptr());
@@ -335,6 +363,10 @@ private:
                 q.sn_block = (uint64_t)a.dim * a.kv_rank; q.sn = 1; q.sk = a.kv_rank;
                 q.k_tiles = l.dim_pad / 32; q.tile_stride = 1;
                 M40H_TRY(m40llm_ext_pack_tiles_async(ctx_, src, l.w_ukt.ptr(), &q, kStream));
+                if (per_head_served_) {
+                    l.w_uk = packed(ctx_, a.heads * l.dim_pad / 16, l.latent_pad / 32);
+                    pack_heads(src, a.heads, a.dim, 0, a.dim, a.kv_rank, l.w_uk.ptr(), l.latent_pad / 32, l.dim_pad, 0);
+                }
             }
             {
                 const uint32_t kt = l.latent_pad / 32;
@@ -373,7 +405,7 @@ private:
     }
 
     void allocate() {
-        const size_t R = opt_.max_rows, D = spec_.width;
+        const size_t R = round_up(std::max(opt_.max_rows, opt_.max_sequences), 16), D = spec_.width;
         size_t proj = 0, cat = 0, cq = 0, q = 0, qa = 0, ol = 0;
         for (const Layer& l : layers_) {
             proj = std::max<size_t>(proj, (size_t)l.plain_tiles * 16);
@@ -385,6 +417,13 @@ private:
         }
         d_pad_ = round_up((uint32_t)D, 32);
         x_ = cleared(ctx_, R * D * 4);
+        size_t planes = 0;         // most floats the parts of a step's sums take
+        for (uint32_t rows = 1; rows <= R; ++rows)
+            for (const Layer& l : layers_) {
+                const uint32_t parts = k_parts(round_up((uint32_t)D, 16) / 16, l.cat / 32, rows);
+                if (parts > 1) planes = std::max<size_t>(planes, (size_t)parts * rows * D);
+            }
+        planes_ = DeviceBuf(ctx_, std::max<size_t>(planes, 4) * 4);
         h_ = cleared(ctx_, R * d_pad_ * es_);
         proj_ = cleared(ctx_, R * proj * 4);
         cat_ = cleared(ctx_, R * cat * es_);
@@ -394,34 +433,60 @@ private:
         ol_ = cleared(ctx_, R * ol * es_);
         for (Rotation& r : rotations_) r.angles = cleared(ctx_, R * r.half * 8);
         logits_rows_ = (uint32_t)std::min<size_t>(std::max<size_t>(R, opt_.max_sequences), 256);
-        hn_ = cleared(ctx_, (size_t)logits_rows_ * d_pad_ * es_);
+        hn_ = cleared(ctx_, (size_t)round_up(logits_rows_, 16) * d_pad_ * es_);
         logits_ = DeviceBuf(ctx_, (size_t)logits_rows_ * spec_.vocab * 4);
         pick_ = DeviceBuf(ctx_, (size_t)logits_rows_ * 4);
         gap_ = DeviceBuf(ctx_, (size_t)logits_rows_ * 4);
         M40H_TRY(m40llm_stream_synchronize(ctx_, kStream));
     }
 
+    // Whether a portion of n tokens behind `len` takes the attention head by head: two products over every pair of a query and a key it
+    // sees, against bringing all keys and values out of the latents first.  The latent form's kernel reaches half the rate.
+    bool per_head(uint32_t n, uint32_t len) const {
+        if (!per_head_served_ || n == 1) return false;
+        if (opt_.portion_form == 2u) return true;
+        if (n < 32) return false;
+        double latent = 0.0, head = 0.0;
+        const double keys = (double)len + n, seen = (double)n * (len + n / 2.0);
+        for (const Layer& l : layers_) {
+            latent += 2.0 * seen * l.a.heads * (l.entry_width + l.latent_pad) + (double)n * l.a.heads * l.latent_pad * (l.dim_pad + l.a.vdim);
+            head += seen * l.a.heads * (l.q_width + l.a.vdim) + keys * l.a.heads * l.latent_pad * (l.dim_pad + l.a.vdim);
+        }
+        return head < latent;
+    }
+
     // query tiles of a set for the portions of a pass
     static void make_tiles(const TileSet& set, const std::vector<Portion>& portions, std::vector<uint32_t>& table, uint32_t& m_tiles) {
         uint32_t longest = 0;
-        for (const Portion& p : portions) longest = std::max(longest, p.n * set.heads);
+        for (const Portion& p : portions)
+            if (!p.per_head) longest = std::max(longest, p.n * set.heads);
         m_tiles = longest <= 16 ? 1 : longest <= 32 ? 2 : 4;
         m_tiles = std::min(m_tiles, set.max_m_tiles);
         const uint32_t size = 16 * m_tiles;
         for (const Portion& p : portions)
-            for (uint32_t i = 0; i < p.n * set.heads; i += size) {
+            for (uint32_t i = 0; !p.per_head && i < p.n * set.heads; i += size) {
                 table.push_back(p.row * set.heads + i);
                 table.push_back(std::min(size, p.n * set.heads - i));
             }
     }
     static uint32_t choose_splits(uint32_t n_tiles, uint32_t longest) {
         const uint32_t pages = (longest + kPage - 1) / kPage;
-        return std::max(1u, std::min(pages, 512u / std::max(n_tiles, 1u)));
+        return std::max(1u, std::min(pages, 256u / std::max(n_tiles, 1u)));
     }
-    void ensure_partial(const Rows& r) {
+    void ensure_scratch(const Rows& r) {
         uint64_t need = 0;
         for (size_t i = 0; i < tile_sets_.size(); ++i)
-            need = std::max(need, m40llm_ext_latent_attention_partial_floats(r.rows * tile_sets_[i].heads, tile_sets_[i].latent_pad, r.tiles[i].splits));
+            need = std::max(need, m40llm_ext_latent_attention_partial_floats(r.latent_rows * tile_sets_[i].heads, tile_sets_[i].latent_pad, r.tiles[i].splits));
+        uint64_t keys = 0, values = 0;
+        for (const Layer& l : layers_) {
+            keys = std::max(keys, (uint64_t)r.n_pages * kPage * l.a.heads * l.dim_pad * 2);
+            values = std::max(values, (uint64_t)r.n_pages * kPage * l.a.heads * l.vdim_tiles * 16 * 2);
+        }
+        if (keys > keys_.bytes() || values > values_.bytes()) {
+            M40H_TRY(m40llm_stream_synchronize(ctx_, kStream));
+            keys_ = DeviceBuf(ctx_, keys);
+            values_ = DeviceBuf(ctx_, values);
+        }
         if (need * 4 > partial_.bytes()) {
             M40H_TRY(m40llm_stream_synchronize(ctx_, kStream));
             drop_graph();
@@ -438,22 +503,43 @@ private:
     Rows upload(const PassPlan& plan, DeviceBuf& buf, uint32_t longest, const uint32_t** want) {
         Rows r;
         r.rows = plan.rows();
+        r.latent_rows = plan.latent_rows;
+        // portions whose attention runs head by head: their page lists, and blocks of 128 queries, those that see most keys first
+        std::vector<uint32_t> list;
+        struct Job { uint32_t row, n, first, keys; };
+        std::vector<Job> jobs;
+        for (const Portion& p : plan.portions) {
+            if (!p.per_head) continue;
+            const uint32_t first = (uint32_t)list.size(), len0 = p.length - p.n;
+            list.insert(list.end(), seqs_.pages(p.slot).begin(), seqs_.pages(p.slot).begin() + seqs_.pages_for(p.length));
+            for (uint32_t i = 0; i < p.n; i += 128) {
+                const uint32_t n = std::min(128u, p.n - i);
+                jobs.push_back({p.row + i, n, first, len0 + i + n});
+            }
+        }
+        std::stable_sort(jobs.begin(), jobs.end(), [](const Job& a, const Job& b) { return a.keys > b.keys; });
+        std::vector<uint32_t> job_words;
+        for (const Job& j : jobs) job_words.insert(job_words.end(), {j.row, j.n, j.first, 0u});
+        r.n_jobs = (uint32_t)jobs.size();
+        r.n_pages = (uint32_t)list.size();
         std::vector<uint32_t> all;
         auto put = [&](const std::vector<uint32_t>& v) { const size_t at = all.size(); all.insert(all.end(), v.begin(), v.end()); return at; };
-        const size_t tok = put(plan.tokens), prev = put(plan.prev), slot = put(plan.slot), pos = put(plan.pos), w = put(plan.want), table = put(page_table());
+        const size_t tok = put(plan.tokens), prev = put(plan.prev), slot = put(plan.slot), pos = put(plan.pos), w = put(plan.want), table = put(page_table()),
+                     jobs_at = put(job_words), list_at = put(list);
         std::vector<size_t> tiles_at;
         for (const TileSet& s : tile_sets_) {
             std::vector<uint32_t> t;
             Rows::Tiles d;
             make_tiles(s, plan.portions, t, d.m_tiles);
             d.n = (uint32_t)t.size() / 2;
-            d.splits = choose_splits(opt_.act_dtype == M40LLM_ACT_F32 ? r.rows * s.heads : d.n, longest);
+            d.splits = choose_splits(opt_.act_dtype == M40LLM_ACT_F32 ? r.latent_rows * s.heads : d.n, longest);
             r.tiles.push_back(d);
             tiles_at.push_back(put(t));
         }
         if (buf.bytes() < all.size() * 4) buf = DeviceBuf(ctx_, all.size() * 4 + all.size());
         M40H_TRY(m40llm_memcpy_h2d(ctx_, buf.ptr(), all.data(), all.size() * 4));
         r.tokens = buf.u32(tok); r.prev = buf.u32(prev); r.slot = buf.u32(slot); r.pos = buf.u32(pos); r.page_table = buf.u32(table);
+        r.jobs = buf.u32(jobs_at); r.page_list = buf.u32(list_at);
         for (size_t i = 0; i < tiles_at.size(); ++i) r.tiles[i].table = buf.u32(tiles_at[i]);
         if (want) *want = buf.u32(w);
         return r;
@@ -470,6 +556,7 @@ private:
     char* act(const DeviceBuf& b, size_t elements) const { return static_cast<char*>(b.ptr()) + elements * es_; }
 
     void enqueue_embedding(const Rows& r) {
+        pending_ = 0;
         const BigramSpec b = spec_.bigram.value_or(BigramSpec{});
         M40H_TRY(m40llm_ext_embed_pairs_async(ctx_, embed_.ptr(), spec_.bigram ? bigram_.ptr() : nullptr, r.tokens, r.prev, r.rows, spec_.vocab,
                                               spec_.width, b.buckets, b.mul_prev, b.mul_cur, x_.ptr(), kStream));
@@ -481,14 +568,15 @@ private:
         const LatentAttentionSpec& a = l.a;
         const Rotation& rot = rotations_[(size_t)l.rotation];
         DeviceBuf& cache = a.kv_from >= 0 ? layers_[(size_t)a.kv_from].cache : l.cache;
-        M40H_TRY(m40llm_ext_layer_norm_rows_async(ctx_, x_.ptr(), l.norm1.ptr(), nullptr, r.rows, spec_.width, spec_.eps, h_.ptr(), d_pad_,
-                                                  opt_.act_dtype, kStream));
+        M40H_TRY(m40llm_ext_layer_norm_rows_async(ctx_, x_.ptr(), planes_.ptr(), pending_, (uint64_t)r.rows * spec_.width, l.norm1.ptr(), nullptr,
+                                                  r.rows, spec_.width, spec_.eps, h_.ptr(), d_pad_, opt_.act_dtype, kStream));
+        pending_ = 0;
         const uint32_t ld_proj = l.plain_tiles * 16;
         {
             M40llmPackedGemm g = product(h_.ptr(), d_pad_, l.w_proj, l.proj_tiles, d_pad_ / 32, r.rows, M40LLM_PACKED_PROJECT);
             g.plain_tiles = l.plain_tiles;
             g.out_f32 = proj_.ptr(); g.ld_out = ld_proj;
-            g.out_act = act(cat_, l.o_pad); g.ld_act = l.cat;
+            g.out_act = cat_.ptr(); g.ld_act = l.cat; g.act_col = l.o_pad;
             launch(g);
         }
         {
@@ -507,13 +595,34 @@ private:
         {
             M40llmPackedGemm g = product(cq_.ptr(), l.cq_pad, l.w_uq, a.heads * l.q_width / 16, l.cq_pad / 32, r.rows, M40LLM_PACKED_ROTATE);
             g.out_act = q_.ptr(); g.ld_act = (uint64_t)a.heads * l.q_width;
-            g.head_width = l.q_width; g.rot_start = l.dim_pad; g.heads = a.heads; g.split_row = r.rows; g.rot_half = rot.half;
+            g.head_width = l.q_width; g.rot_start = l.dim_pad; g.heads = a.heads; g.split_row = r.latent_rows; g.rot_half = rot.half;
             g.angles = rot.angles.ptr();
             g.rot_out = act(qa_, l.latent_pad); g.ld_rot = l.entry_width;
             launch(g);
         }
+        if (r.latent_rows) enqueue_latent_attention(l, r, cache);
+        if (r.n_jobs) enqueue_head_attention(l, r, cache);
         {
-            M40llmPackedGemm g = product(q_.ptr(), a.heads * l.q_width, l.w_ukt, l.latent_pad / 16, l.dim_pad / 32, r.rows, M40LLM_PACKED_STORE_ACT);
+            M40llmPackedGemm g = product(cat_.ptr(), l.cat, l.w_out, round_up(spec_.width, 16) / 16, l.cat / 32, r.rows, M40LLM_PACKED_ADD);
+            g.ld_out = spec_.width; g.cols = spec_.width;
+            const uint32_t parts = r.in_place ? 1u : k_parts(g.n_tiles, g.k_tiles, r.rows);
+            if (parts > 1u) {       // sums of parts of K: the next norm adds them to x
+                g.epilogue = M40LLM_PACKED_STORE;
+                g.k_parts = parts;
+                g.out_f32 = planes_.ptr(); g.out_batch = (uint64_t)r.rows * spec_.width;
+                pending_ = parts;
+            } else {
+                g.out_f32 = x_.ptr();
+            }
+            launch(g);
+        }
+    }
+    // decoded tokens and short portions: rows before r.latent_rows
+    void enqueue_latent_attention(Layer& l, const Rows& r, DeviceBuf& cache) {
+        const LatentAttentionSpec& a = l.a;
+        const uint32_t ld_proj = l.plain_tiles * 16;
+        {
+            M40llmPackedGemm g = product(q_.ptr(), a.heads * l.q_width, l.w_ukt, l.latent_pad / 16, l.dim_pad / 32, r.latent_rows, M40LLM_PACKED_STORE_ACT);
             g.batches = a.heads; g.a_batch = l.q_width; g.w_batch = (uint64_t)(l.latent_pad / 16) * (l.dim_pad / 32) * 512;
             g.out_act = qa_.ptr(); g.ld_act = (uint64_t)a.heads * l.entry_width; g.act_batch = l.entry_width; g.cols = l.latent_pad;
             launch(g);
@@ -526,28 +635,53 @@ private:
             g.queries = qa_.ptr(); g.cache = cache.ptr(); g.sink = l.sink.ptr();
             g.row_slot = r.slot; g.row_pos = r.pos; g.page_table = r.page_table; g.max_pages = max_pages_;
             g.tiles = t.table; g.n_tiles = t.n; g.m_tiles = t.m_tiles; g.splits = t.splits;
-            g.first_query = 0; g.n_queries = r.rows * a.heads;
+            g.first_query = 0; g.n_queries = r.latent_rows * a.heads;
             g.partial = partial_.ptr(); g.partial_floats = partial_.bytes() / 4;
             g.out = ol_.ptr();
             M40H_TRY(m40llm_ext_latent_attention_async(ctx_, &g, kStream));
         }
         {
-            M40llmPackedGemm g = product(ol_.ptr(), a.heads * l.latent_pad, l.w_uv, l.vdim_tiles, l.latent_pad / 32, r.rows, M40LLM_PACKED_GATED);
+            M40llmPackedGemm g = product(ol_.ptr(), a.heads * l.latent_pad, l.w_uv, l.vdim_tiles, l.latent_pad / 32, r.latent_rows, M40LLM_PACKED_GATED);
             g.batches = a.heads; g.a_batch = l.latent_pad; g.w_batch = (uint64_t)l.vdim_tiles * (l.latent_pad / 32) * 512;
             g.out_act = cat_.ptr(); g.ld_act = l.cat; g.act_batch = a.vdim; g.cols = a.vdim;
             g.gate = proj_.f32(l.gate_offset); g.ld_gate = ld_proj;
             launch(g);
         }
-        {
-            M40llmPackedGemm g = product(cat_.ptr(), l.cat, l.w_out, round_up(spec_.width, 16) / 16, l.cat / 32, r.rows, M40LLM_PACKED_ADD);
-            g.out_f32 = x_.ptr(); g.ld_out = spec_.width; g.cols = spec_.width;
+    }
+    // long portions: rows from r.latent_rows on
+    void enqueue_head_attention(Layer& l, const Rows& r, DeviceBuf& cache) {
+        const LatentAttentionSpec& a = l.a;
+        for (uint32_t kind : {M40LLM_PACKED_KEYS, M40LLM_PACKED_VALUES}) {
+            const bool keys = kind == M40LLM_PACKED_KEYS;
+            M40llmPackedGemm g = product(cache.ptr(), 0, keys ? l.w_uk : l.w_uv, keys ? a.heads * l.dim_pad / 16 : a.heads * l.vdim_tiles,
+                                         l.latent_pad / 32, r.n_pages * kPage, kind);
+            g.pages = r.page_list; g.page_k_tiles = l.entry_width / 32;
+            g.out_act = keys ? keys_.ptr() : values_.ptr();
             launch(g);
         }
+        M40llmHeadAttention h{};
+        h.heads = a.heads; h.plain_tiles = l.dim_pad / 32; h.rot_tiles = l.rot_pad / 32; h.entry_tiles = l.entry_width / 32;
+        h.vdim = a.vdim; h.v_tiles = l.vdim_tiles; h.scale = l.scale;
+        h.queries = q_.ptr(); h.ld_queries = a.heads * l.q_width;
+        h.keys = keys_.ptr(); h.values = values_.ptr(); h.cache = cache.ptr(); h.sink = l.sink.ptr();
+        h.gate = proj_.f32(l.gate_offset); h.ld_gate = l.plain_tiles * 16;
+        h.row_pos = r.pos; h.pages = r.page_list; h.jobs = r.jobs; h.n_jobs = r.n_jobs;
+        h.out = cat_.ptr(); h.ld_out = l.cat;
+        M40H_TRY(m40llm_ext_head_attention_async(ctx_, &h, kStream));
     }
-    // final norm and head of n rows of x (row_index NULL = the first n)
-    void enqueue_logits(const uint32_t* row_index, uint32_t n) {
-        M40H_TRY(m40llm_ext_layer_norm_rows_async(ctx_, x_.ptr(), final_norm_.ptr(), row_index, n, spec_.width, spec_.eps, hn_.ptr(), d_pad_,
-                                                  opt_.act_dtype, kStream));
+    // Into how many parts the sum over the attention and feed-forward columns is cut where a launch would leave CUs idle.
+    uint32_t k_parts(uint32_t n_tiles, uint32_t k_tiles, uint32_t rows) const {
+        uint32_t groups;
+        if (rows <= 64 || opt_.act_dtype == M40LLM_ACT_F32) groups = n_tiles * ((rows + 63) / 64);
+        else groups = (rows + 127) / 128 * ((n_tiles + 7) / 8);
+        uint32_t parts = 1;
+        while (parts < kMaxParts && groups * parts * 2 <= kCus && k_tiles / (parts * 2) >= 32) parts *= 2;
+        return (parts - 1) * ((k_tiles + parts - 1) / parts) < k_tiles ? parts : 1u;
+    }
+    // final norm and head of n of a pass's rows (row_index NULL = all of them)
+    void enqueue_logits(const uint32_t* row_index, uint32_t n, uint32_t rows) {
+        M40H_TRY(m40llm_ext_layer_norm_rows_async(ctx_, x_.ptr(), planes_.ptr(), pending_, (uint64_t)rows * spec_.width, final_norm_.ptr(), row_index, n,
+                                                  spec_.width, spec_.eps, hn_.ptr(), d_pad_, opt_.act_dtype, kStream));
         M40llmPackedGemm g = product(hn_.ptr(), d_pad_, head_, round_up(spec_.vocab, 16) / 16, d_pad_ / 32, n, M40LLM_PACKED_STORE);
         g.out_f32 = logits_.ptr(); g.ld_out = spec_.vocab; g.cols = spec_.vocab;
         launch(g);
@@ -555,11 +689,13 @@ private:
 
     void run_pass(const PassPlan& plan, float* logits_out, const std::function<void(uint32_t, uint32_t, const float*)>& on_layer) {
         uint32_t longest = 0;
-        for (uint32_t p : plan.pos) longest = std::max(longest, p + 1);
+        for (const Portion& p : plan.portions)
+            if (!p.per_head) longest = std::max(longest, p.length);
         M40H_TRY(m40llm_stream_synchronize(ctx_, kStream));           // the tables of the pass before may still be read
         const uint32_t* want = nullptr;
-        const Rows r = upload(plan, tables_, longest, &want);
-        ensure_partial(r);
+        Rows r = upload(plan, tables_, longest, &want);
+        r.in_place = (bool)on_layer;
+        ensure_scratch(r);
         enqueue_embedding(r);
         for (size_t i = 0; i < layers_.size(); ++i) {
             enqueue_layer(layers_[i], r);
@@ -570,7 +706,7 @@ private:
         }
         for (size_t i = 0; i < plan.want.size(); i += logits_rows_) {
             const uint32_t n = (uint32_t)std::min<size_t>(logits_rows_, plan.want.size() - i);
-            enqueue_logits(want + i, n);
+            enqueue_logits(want + i, n, r.rows);
             M40H_TRY(m40llm_stream_synchronize(ctx_, kStream));
             for (uint32_t k = 0; k < n;) {      // runs of rows that lie together in the output
                 uint32_t m = 1;
@@ -617,20 +753,21 @@ private:
             plan.prev.push_back(prev0[i]);
             plan.slot.push_back(s);
             plan.pos.push_back(kv_lens[i]);
-            plan.portions.push_back({i, 1});
+            plan.portions.push_back({i, 1, s, kv_lens[i] + 1, false});
+            ++plan.latent_rows;
             longest = std::max(longest, kv_lens[i] + total);
         }
         M40H_TRY(m40llm_stream_synchronize(ctx_, kStream));
         drop_graph();
         Rows r = upload(plan, loop_tables_, longest, nullptr);
-        ensure_partial(r);
+        ensure_scratch(r);
         loop_state_ = cleared(ctx_, 16);
         loop_ids_ = DeviceBuf(ctx_, (size_t)rows * total * 4);
         loop_gaps_ = DeviceBuf(ctx_, (size_t)rows * total * 4);
         auto enqueue = [&]() {
             enqueue_embedding(r);
             for (Layer& l : layers_) enqueue_layer(l, r);
-            enqueue_logits(nullptr, rows);
+            enqueue_logits(nullptr, rows, rows);
             M40H_TRY(m40llm_ext_argmax_f32_async(ctx_, logits_.ptr(), rows, spec_.vocab, pick_.u32(), gap_.f32()));
             M40H_TRY(m40llm_ext_advance_rows_async(ctx_, pick_.u32(), gap_.f32(), rows, r.tokens, r.prev, r.pos, loop_state_.u32(), loop_ids_.u32(),
                                                    loop_gaps_.f32(), total, kStream));
@@ -706,13 +843,16 @@ private:
     uint32_t es_;
     SequencePages seqs_;
     uint32_t max_pages_ = 0, d_pad_ = 0, logits_rows_ = 0, mode_ = 2;
+    uint32_t pending_ = 0;             // planes whose sums x has not taken yet
+    bool per_head_served_ = false;
     float tie_guard_ = DecodeModel::kGreedyTieGuard;
     bool timed_fallback_ = false;
     std::vector<Layer> layers_;
     std::vector<Rotation> rotations_;
     std::vector<TileSet> tile_sets_;
     DeviceBuf embed_, bigram_, final_norm_, head_, staging_;
-    DeviceBuf x_, h_, proj_, cat_, cq_, q_, qa_, ol_, hn_, logits_, pick_, gap_, partial_, tables_;
+    DeviceBuf keys_, values_;           // of the long portions' sequences, one layer at a time
+    DeviceBuf x_, planes_, h_, proj_, cat_, cq_, q_, qa_, ol_, hn_, logits_, pick_, gap_, partial_, tables_;
     DeviceBuf loop_tables_, loop_state_, loop_ids_, loop_gaps_;
     M40llmCudaGraphExec* graph_ = nullptr;
 };

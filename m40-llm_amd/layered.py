@@ -13,7 +13,7 @@ ACT = {"bfloat16": 0, "float32": 1}
 
 
 class ModelOptions(C.Structure):
-    _fields_ = [(n, C.c_uint32) for n in ("act_dtype", "max_tokens", "max_sequences", "max_rows")]
+    _fields_ = [(n, C.c_uint32) for n in ("act_dtype", "max_tokens", "max_sequences", "max_rows", "portion_form")]
 
 
 class StepEntryC(C.Structure):
@@ -30,13 +30,13 @@ class LayeredModel:
         self.vocab = self.H.m40host_model_vocab(handle)
 
     @classmethod
-    def open(cls, ctx, folder, dtype="bfloat16", max_tokens=4096, max_sequences=4, max_rows=0):
-        o = ModelOptions(ACT[dtype], max_tokens, max_sequences, max_rows)
+    def open(cls, ctx, folder, dtype="bfloat16", max_tokens=4096, max_sequences=4, max_rows=0, portion_form=0):
+        o = ModelOptions(ACT[dtype], max_tokens, max_sequences, max_rows, portion_form)
         return cls(ctx, host().m40host_model_open(ctx.h, str(folder).encode(), C.byref(o)))
 
     @classmethod
-    def random(cls, ctx, config: dict, seed=0, std=0.02, dtype="bfloat16", max_tokens=4096, max_sequences=4, max_rows=0):
-        o = ModelOptions(ACT[dtype], max_tokens, max_sequences, max_rows)
+    def random(cls, ctx, config: dict, seed=0, std=0.02, dtype="bfloat16", max_tokens=4096, max_sequences=4, max_rows=0, portion_form=0):
+        o = ModelOptions(ACT[dtype], max_tokens, max_sequences, max_rows, portion_form)
         return cls(ctx, host().m40host_model_open_random(ctx.h, json.dumps(config).encode(), seed, std, C.byref(o)))
 
     def close(self):

@@ -49,11 +49,15 @@ def open_model(ctx, folder, dtype, max_tokens=1024, slots=4, **kw):
     return layered.LayeredModel.open(ctx, folder, dtype, max_tokens, slots, **kw)
 
 
-@pytest.mark.parametrize("dtype", DTYPES)
+# (dtype, form of the portions' attention: 0 the cheaper, 1 in latent space, 2 head by head)
+FORMS = [("float32", 0), ("bfloat16", 1), ("bfloat16", 2)]
+
+
+@pytest.mark.parametrize("dtype,form", FORMS)
 @pytest.mark.parametrize("name,n", [("odd", 150), ("even", 200), ("wide", 140), ("one", 70)])
-def test_residual_after_every_layer_and_logits_of_a_whole_prompt(ctx, folders, expected, name, n, dtype):
+def test_residual_after_every_layer_and_logits_of_a_whole_prompt(ctx, folders, expected, name, n, dtype, form):
     t, want, res = expected(name, n)
-    m = open_model(ctx, folders(name), dtype)
+    m = open_model(ctx, folders(name), dtype, portion_form=form)
     x = m.step_layers(0, t, *[res.shape[i] for i in (0, 2)])
     for i in range(len(res)):
         e = np.sqrt(((x[i] - res[i]) ** 2).mean(axis=-1)) / np.sqrt((res[i] ** 2).mean())
@@ -75,12 +79,12 @@ def test_token_by_token_equals_the_whole_prompt(ctx, folders, expected, name, n,
     m.close()
 
 
-@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("dtype,form", FORMS + [("bfloat16", 0)])
 @pytest.mark.parametrize("name,n", [("odd", 330), ("wide", 330)])
 @pytest.mark.parametrize("cut", [[2], [3, 2, 61, 64, 66], [63, 1], [128, 5], [65], [200, 2]])
-def test_portions_of_any_size(ctx, folders, expected, name, n, cut, dtype):
+def test_portions_of_any_size(ctx, folders, expected, name, n, cut, dtype, form):
     t, want, _ = expected(name, n)
-    m = open_model(ctx, folders(name), dtype)
+    m = open_model(ctx, folders(name), dtype, portion_form=form)
     at, k, got = 0, 0, []
     while at < n:
         c = min(cut[k % len(cut)], n - at)
@@ -90,14 +94,14 @@ def test_portions_of_any_size(ctx, folders, expected, name, n, cut, dtype):
     m.close()
 
 
-@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("dtype,form", FORMS + [("bfloat16", 0)])
 @pytest.mark.parametrize("max_rows", [0, 7, 100])
-def test_mixed_batches_with_pages_and_slots_used_again(ctx, folders, expected, dtype, max_rows):
+def test_mixed_batches_with_pages_and_slots_used_again(ctx, folders, expected, dtype, form, max_rows):
     """Twelve sequences through four slots and a pool that holds four of them: portions of some beside single tokens of others,
     sequences left out for a step, every position compared; then the pool is whole again."""
     rng = np.random.default_rng(17)
     lens = [5, 64, 65, 150, 127, 2, 129, 70, 1, 192, 128, 33]
-    m = open_model(ctx, folders("odd"), dtype, max_tokens=4 * 192, max_rows=max_rows)
+    m = open_model(ctx, folders("odd"), dtype, max_tokens=4 * 192, max_rows=max_rows, portion_form=form)
     free0 = m.free_pages()
     waiting, live, free, errs = list(range(len(lens))), {}, [0, 1, 2, 3], {}
     seqs = {i: expected("odd", n, seed=1 + i) for i, n in enumerate(lens)}
@@ -129,9 +133,9 @@ def test_mixed_batches_with_pages_and_slots_used_again(ctx, folders, expected, d
     m.close()
 
 
-@pytest.mark.parametrize("dtype", DTYPES)
-def test_batch_of_unequal_requests_equals_each_alone(ctx, folders, expected, dtype):
-    m = open_model(ctx, folders("even"), dtype, max_tokens=1024)
+@pytest.mark.parametrize("dtype,form", FORMS)
+def test_batch_of_unequal_requests_equals_each_alone(ctx, folders, expected, dtype, form):
+    m = open_model(ctx, folders("even"), dtype, max_tokens=1024, portion_form=form)
     lens = [200, 3, 129, 64]
     seqs = [expected("even", n, seed=40) for n in lens]
     alone = []
