@@ -662,7 +662,7 @@ uint32_t m40llm_ext_latent_attention_max_m_tiles(uint32_t act_dtype, uint32_t kv
 /* The same attention for long portions, over keys and values brought out of the latents head by head.  pages: the page lists of the
  * portions one behind the other; keys / values: what M40LLM_PACKED_KEYS / _VALUES write for that list (heads of 32*plain_tiles key
  * columns, heads of 16*v_tiles value columns); the rotated key part (the last rot_tiles of a cache entry's entry_tiles) is
- * read from the cache.  queries: packed [rows][ld_queries], per head [plain | rotated].  jobs[t] = {first row, rows (at most 128),
+ * read from the cache.  queries: packed [rows][ld_queries], per head [plain | rotated].  jobs[t] = {first row, rows (at most job_rows),
  * first page of the portion's sequence in `pages`, 0}.  out[row][head*vdim + d], packed = result * sigmoid(gate[row][head]). */
 typedef struct M40llmHeadAttention {
     uint32_t heads, plain_tiles, rot_tiles, entry_tiles, vdim, v_tiles;
@@ -673,18 +673,24 @@ typedef struct M40llmHeadAttention {
     const void* gate;
     uint64_t ld_gate;
     const uint32_t *row_pos, *pages, *jobs;
-    uint32_t n_jobs;
+    uint32_t n_jobs, job_rows;        /* job_rows: 64 or 128 */
     void* out;
     uint32_t ld_out;
 } M40llmHeadAttention;
 int m40llm_ext_head_attention_async(M40llmCudaContext* ctx, const M40llmHeadAttention* a, uint32_t stream_kind);
 /* whether a head of as many 32-wide key tiles (plain and rotated) and 16-wide value tiles is served */
 int m40llm_ext_head_attention_serves(uint32_t k_tiles, uint32_t v_tiles);
-/* Greedy step of a device-driven decode loop: token r = picks[r] (gap[r] beside it) is recorded at ids[r*capacity + step] /
- * gaps[...], becomes the input token (prev = the token before), positions advance by one.  state[0] = step counter. */
-int m40llm_ext_advance_rows_async(M40llmCudaContext* ctx, const uint32_t* d_picks, const float* d_gap, uint32_t rows,
-                                  uint32_t* d_tokens, uint32_t* d_prev, uint32_t* d_positions, uint32_t* d_state,
-                                  uint32_t* d_ids, float* d_gaps, uint32_t capacity, uint32_t stream_kind);
+/* Largest and second largest logit of every row, in M40LLM_TOP2_PARTS parts a row: parts[row][part] = {largest, second largest,
+ * first index of the largest, 0} (f32, f32, u32, u32) */
+#define M40LLM_TOP2_PARTS 32u
+int m40llm_ext_top2_parts_async(M40llmCudaContext* ctx, const void* d_logits_f32, uint32_t rows, uint32_t vocab, void* d_parts,
+                                uint32_t stream_kind);
+/* Greedy step of a device-driven decode loop: row r's token is the first index of its largest logit (from parts); it and the gap to
+ * the second largest are recorded at ids[r*capacity + step] / gaps[...], it becomes the input token (prev = the token before), the
+ * position advances by one.  state[0] = step counter. */
+int m40llm_ext_advance_rows_async(M40llmCudaContext* ctx, const void* d_parts, uint32_t rows, uint32_t* d_tokens, uint32_t* d_prev,
+                                  uint32_t* d_positions, uint32_t* d_state, uint32_t* d_ids, float* d_gaps, uint32_t capacity,
+                                  uint32_t stream_kind);
 
 /* ---- present but unavailable (return -1, as cuda/stub.c does) ---------------------- */
 int m40llm_kvcache_build_q8_old_from_dense(M40llmCudaContext*, M40llmKVCache*, uint32_t, uint32_t, uint32_t);

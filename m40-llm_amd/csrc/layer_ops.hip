@@ -20,10 +20,20 @@ __global__ __launch_bounds__(kThreads) void embed_pairs_kernel(const uint16_t* _
         const uint32_t r = p == 0xffffffffu ? buckets : (uint32_t)(((uint64_t)p * mul_prev + (uint64_t)tok * mul_cur) % buckets);
         b = pairs + (size_t)r * width;
     }
+    float* out = x + (size_t)row * width;
+    if (width % 8u == 0) {
+        for (uint32_t i = threadIdx.x; i < width / 8u; i += kThreads) {
+            const m40_bf16x8 va = reinterpret_cast<const m40_bf16x8*>(a)[i];
+            m40_f32x8 v = __builtin_convertvector(va, m40_f32x8);
+            if (b) v += __builtin_convertvector(reinterpret_cast<const m40_bf16x8*>(b)[i], m40_f32x8);
+            reinterpret_cast<m40_f32x8*>(out)[i] = v;
+        }
+        return;
+    }
     for (uint32_t i = threadIdx.x; i < width; i += kThreads) {
         float v = m40_bf16_bits(a[i]);
         if (b) v += m40_bf16_bits(b[i]);
-        x[(size_t)row * width + i] = v;
+        out[i] = v;
     }
 }
 
@@ -195,17 +205,51 @@ __global__ __launch_bounds__(kThreads) void latent_split_append_kernel(M40llmLat
     }
 }
 
-__global__ __launch_bounds__(kThreads) void advance_rows_kernel(const uint32_t* __restrict__ picks, const float* __restrict__ gap,
-                                                                uint32_t rows, uint32_t* __restrict__ tokens, uint32_t* __restrict__ prev,
+struct Top2 {
+    float best, second;
+    uint32_t at, unused;
+};
+__device__ __forceinline__ void top2_join(Top2& a, const Top2& b) {       // the lower index of equal logits
+    const bool take = b.best > a.best || (b.best == a.best && b.at < a.at);
+    a.second = take ? fmaxf(a.best, b.second) : fmaxf(a.second, b.best);
+    a.best = take ? b.best : a.best;
+    a.at = take ? b.at : a.at;
+}
+__device__ __forceinline__ Top2 top2_wave(Top2 t) {
+#pragma unroll
+    for (int d = 1; d < 64; d *= 2) top2_join(t, Top2{__shfl_xor(t.best, d), __shfl_xor(t.second, d), (uint32_t)__shfl_xor((int)t.at, d), 0u});
+    return t;
+}
+__global__ __launch_bounds__(kThreads) void top2_parts_kernel(const float* __restrict__ logits, uint32_t vocab, Top2* __restrict__ parts) {
+    __shared__ Top2 wave_top[kThreads / 64];
+    const uint32_t per = (vocab + M40LLM_TOP2_PARTS - 1u) / M40LLM_TOP2_PARTS, begin = blockIdx.x * per;
+    const uint32_t end = begin + per < vocab ? begin + per : vocab;
+    const float* row = logits + (size_t)blockIdx.y * vocab;
+    Top2 t{-INFINITY, -INFINITY, 0xffffffffu, 0u};
+    for (uint32_t i = begin + threadIdx.x; i < end; i += kThreads) top2_join(t, Top2{row[i], -INFINITY, i, 0u});
+    t = top2_wave(t);
+    if ((threadIdx.x & 63u) == 0u) wave_top[threadIdx.x >> 6] = t;
+    __syncthreads();
+    if (threadIdx.x != 0u) return;
+    for (int w = 1; w < kThreads / 64; ++w) top2_join(t, wave_top[w]);
+    parts[blockIdx.y * M40LLM_TOP2_PARTS + blockIdx.x] = t;
+}
+
+// a wave a row
+__global__ __launch_bounds__(kThreads) void advance_rows_kernel(const Top2* __restrict__ parts, uint32_t rows,
+                                                                uint32_t* __restrict__ tokens, uint32_t* __restrict__ prev,
                                                                 uint32_t* __restrict__ positions, uint32_t* __restrict__ state,
                                                                 uint32_t* __restrict__ ids, float* __restrict__ gaps, uint32_t capacity) {
-    const uint32_t step = state[0];
+    const uint32_t step = state[0], lane = threadIdx.x & 63u;
     __syncthreads();
-    for (uint32_t r = threadIdx.x; r < rows; r += kThreads) {
-        const uint32_t next = picks[r];
+    for (uint32_t r = threadIdx.x >> 6; r < rows; r += kThreads / 64) {
+        Top2 t = lane < M40LLM_TOP2_PARTS ? parts[r * M40LLM_TOP2_PARTS + lane] : Top2{-INFINITY, -INFINITY, 0xffffffffu, 0u};
+        t = top2_wave(t);
+        if (lane != 0u) continue;
+        const uint32_t next = t.at == 0xffffffffu ? 0u : t.at;          // no comparable logit
         if (step < capacity) {
             ids[(size_t)r * capacity + step] = next;
-            gaps[(size_t)r * capacity + step] = gap[r];
+            gaps[(size_t)r * capacity + step] = t.best - t.second;
         }
         prev[r] = tokens[r];
         tokens[r] = next;
@@ -279,14 +323,24 @@ int m40llm_ext_latent_split_append_async(M40llmCudaContext* ctx, const M40llmLat
     return launched();
 }
 
-int m40llm_ext_advance_rows_async(M40llmCudaContext* ctx, const uint32_t* d_picks, const float* d_gap, uint32_t rows, uint32_t* d_tokens,
-                                  uint32_t* d_prev, uint32_t* d_positions, uint32_t* d_state, uint32_t* d_ids, float* d_gaps,
-                                  uint32_t capacity, uint32_t stream_kind) {
-    if (!ctx || !d_picks || !d_gap || !d_tokens || !d_prev || !d_positions || !d_state || !d_ids || !d_gaps) return -1;
+int m40llm_ext_top2_parts_async(M40llmCudaContext* ctx, const void* d_logits, uint32_t rows, uint32_t vocab, void* d_parts, uint32_t stream_kind) {
+    if (!ctx || !d_logits || !d_parts) return -1;
     hipStream_t stream = m40_select_stream(ctx, stream_kind);
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
-    if (rows == 0) return -3;
-    advance_rows_kernel<<<1, kThreads, 0, stream>>>(d_picks, d_gap, rows, d_tokens, d_prev, d_positions, d_state, d_ids, d_gaps, capacity);
+    if (rows == 0 || rows > 65535u || vocab == 0 || !m40_aligned16(d_parts)) return -3;
+    top2_parts_kernel<<<dim3(M40LLM_TOP2_PARTS, rows), kThreads, 0, stream>>>(static_cast<const float*>(d_logits), vocab, static_cast<Top2*>(d_parts));
+    return launched();
+}
+
+int m40llm_ext_advance_rows_async(M40llmCudaContext* ctx, const void* d_parts, uint32_t rows, uint32_t* d_tokens, uint32_t* d_prev,
+                                  uint32_t* d_positions, uint32_t* d_state, uint32_t* d_ids, float* d_gaps, uint32_t capacity,
+                                  uint32_t stream_kind) {
+    if (!ctx || !d_parts || !d_tokens || !d_prev || !d_positions || !d_state || !d_ids || !d_gaps) return -1;
+    hipStream_t stream = m40_select_stream(ctx, stream_kind);
+    if (!stream || m40_ensure_device(ctx) != 0) return -2;
+    if (rows == 0 || !m40_aligned16(d_parts)) return -3;
+    advance_rows_kernel<<<1, kThreads, 0, stream>>>(static_cast<const Top2*>(d_parts), rows, d_tokens, d_prev, d_positions, d_state, d_ids, d_gaps,
+                                                    capacity);
     return launched();
 }
 

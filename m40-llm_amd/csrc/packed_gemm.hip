@@ -295,7 +295,8 @@ int launch_tile(hipStream_t stream, const PackedArgs& g, const M40Epilogue<m40_b
 template <int FORM>
 int launch_tile_any(hipStream_t stream, const PackedArgs& g, const M40Epilogue<m40_bf16>& e, int batches, int num_cus) {
     const long long wide = (long long)((g.rows + 127) / 128) * ((g.n_tiles + 15) / 16) * batches;
-    if (wide * 16 >= 9ll * num_cus) return launch_tile<8, FORM>(stream, g, e, batches);
+    // a short sum is mostly a workgroup's start and end: two narrower workgroups a CU cover each other's
+    if (wide * 16 >= 9ll * num_cus && g.k_tiles > 32) return launch_tile<8, FORM>(stream, g, e, batches);
     return launch_tile<4, FORM>(stream, g, e, batches);
 }
 

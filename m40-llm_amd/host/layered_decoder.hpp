@@ -245,7 +245,7 @@ private:
         uint32_t *tokens = nullptr, *prev = nullptr, *slot = nullptr, *pos = nullptr, *page_table = nullptr;
         uint32_t latent_rows = 0;             // rows before it: attention in latent space; from it on: head by head
         const uint32_t *jobs = nullptr, *page_list = nullptr;
-        uint32_t n_jobs = 0, n_pages = 0;
+        uint32_t n_jobs = 0, job_rows = 128, n_pages = 0;
         struct Tiles { const uint32_t* table = nullptr; uint32_t n = 0, m_tiles = 1, splits = 1; };
         std::vector<Tiles> tiles;             // one per tile set
     };
@@ -435,8 +435,7 @@ private:
         logits_rows_ = (uint32_t)std::min<size_t>(std::max<size_t>(R, opt_.max_sequences), 256);
         hn_ = cleared(ctx_, (size_t)round_up(logits_rows_, 16) * d_pad_ * es_);
         logits_ = DeviceBuf(ctx_, (size_t)logits_rows_ * spec_.vocab * 4);
-        pick_ = DeviceBuf(ctx_, (size_t)logits_rows_ * 4);
-        gap_ = DeviceBuf(ctx_, (size_t)logits_rows_ * 4);
+        pick_parts_ = DeviceBuf(ctx_, (size_t)logits_rows_ * M40LLM_TOP2_PARTS * 16);
         M40H_TRY(m40llm_stream_synchronize(ctx_, kStream));
     }
 
@@ -504,7 +503,11 @@ private:
         Rows r;
         r.rows = plan.rows();
         r.latent_rows = plan.latent_rows;
-        // portions whose attention runs head by head: their page lists, and blocks of 128 queries, those that see most keys first
+        // portions whose attention runs head by head: their page lists, and blocks of queries, those that see most keys first
+        uint32_t fewest_heads = 0xffffffffu, blocks = 0;
+        for (const Layer& l : layers_) fewest_heads = std::min(fewest_heads, l.a.heads);
+        for (const Portion& p : plan.portions) blocks += p.per_head ? (p.n + 127) / 128 : 0;
+        r.job_rows = (uint64_t)blocks * fewest_heads >= kCus ? 128u : 64u;
         std::vector<uint32_t> list;
         struct Job { uint32_t row, n, first, keys; };
         std::vector<Job> jobs;
@@ -512,8 +515,8 @@ private:
             if (!p.per_head) continue;
             const uint32_t first = (uint32_t)list.size(), len0 = p.length - p.n;
             list.insert(list.end(), seqs_.pages(p.slot).begin(), seqs_.pages(p.slot).begin() + seqs_.pages_for(p.length));
-            for (uint32_t i = 0; i < p.n; i += 128) {
-                const uint32_t n = std::min(128u, p.n - i);
+            for (uint32_t i = 0; i < p.n; i += r.job_rows) {
+                const uint32_t n = std::min(r.job_rows, p.n - i);
                 jobs.push_back({p.row + i, n, first, len0 + i + n});
             }
         }
@@ -665,7 +668,7 @@ private:
         h.queries = q_.ptr(); h.ld_queries = a.heads * l.q_width;
         h.keys = keys_.ptr(); h.values = values_.ptr(); h.cache = cache.ptr(); h.sink = l.sink.ptr();
         h.gate = proj_.f32(l.gate_offset); h.ld_gate = l.plain_tiles * 16;
-        h.row_pos = r.pos; h.pages = r.page_list; h.jobs = r.jobs; h.n_jobs = r.n_jobs;
+        h.row_pos = r.pos; h.pages = r.page_list; h.jobs = r.jobs; h.n_jobs = r.n_jobs; h.job_rows = r.job_rows;
         h.out = cat_.ptr(); h.ld_out = l.cat;
         M40H_TRY(m40llm_ext_head_attention_async(ctx_, &h, kStream));
     }
@@ -768,8 +771,8 @@ private:
             enqueue_embedding(r);
             for (Layer& l : layers_) enqueue_layer(l, r);
             enqueue_logits(nullptr, rows, rows);
-            M40H_TRY(m40llm_ext_argmax_f32_async(ctx_, logits_.ptr(), rows, spec_.vocab, pick_.u32(), gap_.f32()));
-            M40H_TRY(m40llm_ext_advance_rows_async(ctx_, pick_.u32(), gap_.f32(), rows, r.tokens, r.prev, r.pos, loop_state_.u32(), loop_ids_.u32(),
+            M40H_TRY(m40llm_ext_top2_parts_async(ctx_, logits_.ptr(), rows, spec_.vocab, pick_parts_.ptr(), kStream));
+            M40H_TRY(m40llm_ext_advance_rows_async(ctx_, pick_parts_.ptr(), rows, r.tokens, r.prev, r.pos, loop_state_.u32(), loop_ids_.u32(),
                                                    loop_gaps_.f32(), total, kStream));
         };
         auto run = [&](uint32_t n) {
@@ -852,7 +855,7 @@ private:
     std::vector<TileSet> tile_sets_;
     DeviceBuf embed_, bigram_, final_norm_, head_, staging_;
     DeviceBuf keys_, values_;           // of the long portions' sequences, one layer at a time
-    DeviceBuf x_, planes_, h_, proj_, cat_, cq_, q_, qa_, ol_, hn_, logits_, pick_, gap_, partial_, tables_;
+    DeviceBuf x_, planes_, h_, proj_, cat_, cq_, q_, qa_, ol_, hn_, logits_, pick_parts_, partial_, tables_;
     DeviceBuf loop_tables_, loop_state_, loop_ids_, loop_gaps_;
     M40llmCudaGraphExec* graph_ = nullptr;
 };
