@@ -53,6 +53,14 @@ struct StepEntry {
     uint32_t n_want;
 };
 
+// Greedy picks of a step's wanted places, in the order of its logits rows: a row flagged greedy whose two best logits are no near
+// tie is decided on the device (picks, picked = 1), and its logits are not brought back.
+struct StepPicks {
+    const uint8_t* greedy;
+    uint32_t* picks;
+    uint8_t* picked;
+};
+
 class LayeredDecoder : public ServedModel {
 public:
     static constexpr uint32_t kStream = M40LLM_STREAM_DECODE;
@@ -94,7 +102,7 @@ public:
     // Runs the entries' tokens behind what their sequences hold.  logits_out: [all wanted places, in entry order][vocab].
     // on_layer (optional): called after every layer with the rows of the pass and the residual on the device (diagnosis).
     void step(const std::vector<StepEntry>& entries, float* logits_out,
-              const std::function<void(uint32_t layer, uint32_t rows, const float* x)>& on_layer = nullptr) {
+              const std::function<void(uint32_t layer, uint32_t rows, const float* x)>& on_layer = nullptr, const StepPicks* picks = nullptr) {
         std::vector<uint8_t> seen(opt_.max_sequences, 0);
         for (const auto& e : entries) {
             if (e.sequence >= opt_.max_sequences) throw std::out_of_range("sequence slot out of range");
@@ -146,7 +154,7 @@ public:
                 done[i] += n;
             }
             while (first < entries.size() && done[first] == entries[first].n) ++first;
-            run_pass(plan, logits_out, on_layer);
+            run_pass(plan, logits_out, on_layer, picks);
         }
         M40H_TRY(m40llm_stream_synchronize(ctx_, kStream));
     }
@@ -165,7 +173,10 @@ public:
             for (const auto& it : items) s.push_back({it.sequence_id, it.kv_len, &it.token, 1, true});
             run_items(s, logits_out);
         };
-        e.step = [this](const std::vector<SchedulerStepItem>& items, float* logits_out) { run_items(items, logits_out); };
+        e.step = [this](const std::vector<SchedulerStepItem>& items, const uint8_t* greedy, float* logits_out, uint32_t* picks, uint8_t* picked) {
+            const StepPicks p{greedy, picks, picked};
+            run_items(items, logits_out, mode_ >= 1 ? &p : nullptr);
+        };
         e.reserve = [this](uint32_t seq, uint64_t tokens) { return seqs_.reserve(seq, tokens); };
         e.release = [this](uint32_t seq) { seqs_.release(seq); };
         e.step_tokens = opt_.max_rows;
@@ -690,7 +701,7 @@ private:
         launch(g);
     }
 
-    void run_pass(const PassPlan& plan, float* logits_out, const std::function<void(uint32_t, uint32_t, const float*)>& on_layer) {
+    void run_pass(const PassPlan& plan, float* logits_out, const std::function<void(uint32_t, uint32_t, const float*)>& on_layer, const StepPicks* picks) {
         uint32_t longest = 0;
         for (const Portion& p : plan.portions)
             if (!p.per_head) longest = std::max(longest, p.length);
@@ -710,10 +721,35 @@ private:
         for (size_t i = 0; i < plan.want.size(); i += logits_rows_) {
             const uint32_t n = (uint32_t)std::min<size_t>(logits_rows_, plan.want.size() - i);
             enqueue_logits(want + i, n, r.rows);
+            std::vector<uint8_t> decided(n, 0);
+            if (picks) {
+                M40H_TRY(m40llm_ext_top2_parts_async(ctx_, logits_.ptr(), n, spec_.vocab, pick_parts_.ptr(), kStream));
+                M40H_TRY(m40llm_stream_synchronize(ctx_, kStream));
+                struct Part { float best, second; uint32_t at, unused; };
+                std::vector<Part> parts((size_t)n * M40LLM_TOP2_PARTS);
+                M40H_TRY(m40llm_memcpy_d2h(ctx_, parts.data(), pick_parts_.ptr(), parts.size() * sizeof(Part)));
+                for (uint32_t k = 0; k < n; ++k) {
+                    Part top = parts[(size_t)k * M40LLM_TOP2_PARTS];
+                    for (uint32_t j = 1; j < M40LLM_TOP2_PARTS; ++j) {      // parts in order of their indices
+                        const Part& p = parts[(size_t)k * M40LLM_TOP2_PARTS + j];
+                        const bool take = p.best > top.best;
+                        top.second = take ? std::max(top.best, p.second) : std::max(top.second, p.best);
+                        if (take) { top.best = p.best; top.at = p.at; }
+                    }
+                    const size_t out = plan.want_out[i + k];
+                    decided[k] = picks->greedy[out] && top.best - top.second >= tie_guard_ && top.at < spec_.vocab;
+                    picks->picked[out] = decided[k];
+                    picks->picks[out] = top.at;
+                }
+            }
             M40H_TRY(m40llm_stream_synchronize(ctx_, kStream));
             for (uint32_t k = 0; k < n;) {      // runs of rows that lie together in the output
+                if (decided[k]) {
+                    ++k;
+                    continue;
+                }
                 uint32_t m = 1;
-                while (k + m < n && plan.want_out[i + k + m] == plan.want_out[i + k] + m) ++m;
+                while (k + m < n && !decided[k + m] && plan.want_out[i + k + m] == plan.want_out[i + k] + m) ++m;
                 M40H_TRY(m40llm_memcpy_d2h(ctx_, logits_out + plan.want_out[i + k] * spec_.vocab, logits_.f32((size_t)k * spec_.vocab),
                                            (size_t)m * spec_.vocab * 4));
                 k += m;
@@ -721,7 +757,7 @@ private:
         }
     }
 
-    void run_items(const std::vector<SchedulerStepItem>& items, float* logits_out) {
+    void run_items(const std::vector<SchedulerStepItem>& items, float* logits_out, const StepPicks* picks = nullptr) {
         std::vector<StepEntry> entries;
         std::vector<uint32_t> last(items.size());
         for (size_t i = 0; i < items.size(); ++i) {
@@ -731,7 +767,7 @@ private:
             last[i] = it.len - 1;
             entries.push_back({it.sequence_id, it.tokens, it.len, &last[i], it.want ? 1u : 0u});
         }
-        step(entries, logits_out);
+        step(entries, logits_out, nullptr, picks);
     }
 
     // Device-driven greedy steps: token, token before, position and step counter stay on the device.  Falls back to the host

@@ -66,9 +66,10 @@ struct SchedulerEngine {
     std::function<void(const std::vector<SchedulerDecodeItem>&, const uint8_t* greedy, float* logits_out, uint32_t* picks_out,
                        uint8_t* picked_out)>
         decode_pick;
-    // Optional: one call for decode tokens and portions of prompts together; logits_out has a row per wanting item.  Prompts are
-    // then fed in portions, at most step_tokens tokens a tick in all.
-    std::function<void(const std::vector<SchedulerStepItem>&, float* logits_out)> step;
+    // Optional: one call for decode tokens and portions of prompts together; logits_out has a row per wanting item, and greedy, picks_out
+    // and picked_out (as for decode_pick) an element.  Prompts are then fed in portions, at most step_tokens tokens a tick in all.
+    std::function<void(const std::vector<SchedulerStepItem>&, const uint8_t* greedy, float* logits_out, uint32_t* picks_out, uint8_t* picked_out)>
+        step;
     uint32_t step_tokens = 0;
     // Optional: room for a sequence that may grow to `tokens` tokens is set aside before its first portion (false = not now, the
     // request waits), and given back with everything else the sequence holds when it leaves.
@@ -269,9 +270,16 @@ private:
         }
         if (!items.empty()) {
             logits_.resize(items.size() * (size_t)engine_.vocab);
+            std::vector<uint8_t> greedy, picked(items.size(), 0);
+            std::vector<uint32_t> picks(items.size(), 0);
+            for (size_t i = 0; i < items.size(); ++i) {
+                if (!items[i].want) continue;
+                const SamplerConfig& c = taking[i]->sampler.config();
+                greedy.push_back(c.top_k && *c.top_k == 1 && !c.top_p);
+            }
             bool failed = false;
             try {
-                engine_.step(items, logits_.data());
+                engine_.step(items, greedy.data(), logits_.data(), picks.data(), picked.data());
             } catch (const std::exception& e) {
                 fail_all(taking, std::string("step failed: ") + e.what(), rep);
                 failed = true;
@@ -280,8 +288,12 @@ private:
             for (size_t i = 0; !failed && i < taking.size(); ++i) {
                 auto& r = taking[i];
                 r->processed += items[i].len;
-                if (items[i].want) sample_and_route(std::move(r), logits_.data() + (row++) * (size_t)engine_.vocab, rep);
-                else active_.push_back(std::move(r));
+                if (!items[i].want) {
+                    active_.push_back(std::move(r));
+                    continue;
+                }
+                sample_and_route(std::move(r), logits_.data() + row * (size_t)engine_.vocab, rep, picked[row] ? &picks[row] : nullptr);
+                ++row;
             }
         }
         for (auto& r : waiting) active_.push_back(std::move(r));

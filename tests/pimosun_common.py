@@ -120,3 +120,55 @@ def logits_error(got, want):
 def assert_logits(got, want, dtype, what="", factor=1.0):
     e = logits_error(got, want)
     assert np.isfinite(e).all() and e.max() <= factor * LIMIT[dtype], (what, dtype, int(e.argmax()), float(e.max()))
+
+
+# ---- kernels one by one: structs of the C header, packed tiles --------------------------------------------------------------
+def c_struct(name):
+    """The ctypes form of a struct in include/m40llm.h."""
+    import ctypes as C
+    import re
+    text = re.sub(r"/\*.*?\*/", "", open(m40.HEADER).read(), flags=re.S)
+    body = re.search(r"typedef struct %s \{(.*?)\} %s;" % (name, name), text, flags=re.S).group(1)
+    fields = []
+    for decl in body.split(";"):
+        decl = decl.strip()
+        if not decl:
+            continue
+        ty, names = re.match(r"(?:const\s+)?(\w+)\s*(.*)", decl, flags=re.S).groups()
+        for n in names.split(","):
+            base = {"uint32_t": C.c_uint32, "uint64_t": C.c_uint64, "float": C.c_float}
+            fields.append((n.strip(" *\n"), C.c_void_p if "*" in n else base[ty]))
+    return type(name, (C.Structure,), {"_fields_": fields})
+
+
+def up32(n):
+    return (n + 31) // 32 * 32
+
+
+def as_act(a, dtype):
+    """Bits of activations: bf16 (rounded) or f32."""
+    return ld.f32_to_bf16(a) if dtype == "bfloat16" else np.ascontiguousarray(a, dtype=np.float32)
+
+
+def from_act(a, dtype):
+    return ld.bf16_to_f32(a) if dtype == "bfloat16" else a
+
+
+def pack_tiles(a):
+    """[N][K] (any dtype) -> 16 x 32 tiles in operand order, zero past the matrix."""
+    n, k = a.shape
+    N, K = (n + 15) // 16 * 16, up32(k)
+    full = np.zeros((N, K), dtype=a.dtype)
+    full[:n, :k] = a
+    return np.ascontiguousarray(full.reshape(N // 16, 16, K // 32, 4, 8).transpose(0, 2, 3, 1, 4)).reshape(-1)
+
+
+def unpack_tiles(flat, n, ld_cols):
+    N = (n + 15) // 16 * 16
+    return flat[:N * ld_cols].reshape(N // 16, ld_cols // 32, 4, 16, 8).transpose(0, 3, 1, 2, 4).reshape(N, ld_cols)[:n]
+
+
+def close_to(got, want, dtype, scale=None, factor=1.0):
+    scale = (np.abs(want).max() or 1.0) if scale is None else scale
+    err = np.abs(np.asarray(got, dtype=np.float64) - want).max() / scale
+    assert err <= factor * {"float32": 3e-6, "bfloat16": 6e-3}[dtype], float(err)

@@ -273,3 +273,46 @@ def test_scheduler_serves_requests_as_each_alone(ctx, folders, dtype, max_rows, 
     assert s.state(r) == "cancelled" and m.free_pages() == free0
     s.close()
     m.close()
+
+
+def test_command_line_generates_what_the_oracle_picks(ctx, folders, capsys):
+    gen = importlib.import_module("m40-llm_amd.generate")
+    model = ld.Model.load(folders("odd"))
+    prompts = [[3, 1, 4, 1, 5], [9] * 70, [2]]
+    gen.main(["--model", folders("odd"), "--dtype", "float32", "--max-tokens", "9", "--slots", "2"] + sum((["--prompt", ",".join(map(str, p))] for p in prompts), []))
+    import json
+    lines = [json.loads(x) for x in capsys.readouterr().out.splitlines()]
+    assert [x["prompt"] for x in lines] == prompts
+    for x in lines:
+        want = model.sequence().feed((x["prompt"] + x["generated"])[:-1])[len(x["prompt"]) - 1:]
+        assert want.argmax(axis=1).tolist() == x["generated"]
+
+
+def test_trace_replay(ctx, folders, expected, tmp_path):
+    """bin/trace_run over a small trace in 32-bit: requests cut into steps, ended and admitted on slots that were used before."""
+    import json
+    import os
+    import subprocess
+    t, want, _ = expected("odd", 135)
+    V = want.shape[1]
+    steps, rows = [], []
+
+    def step(entries, end=()):
+        steps.append(json.dumps({"step": len(steps), "entries": [{"id": i, "tokens": t[a:b].tolist(), "want": w} for i, a, b, w in entries], "end": list(end)}))
+        rows.append([a + x for _, a, _, w in entries for x in w])
+    step([("a", 0, 70, [69, 3])])
+    step([("b", 0, 2, []), ("a", 70, 71, [])])
+    step([("b", 2, 100, [0, 97]), ("a", 71, 72, [0]), ("c", 0, 1, [0]), ("d", 0, 5, [4])], ["a", "c"])
+    step([("e", 0, 64, [63]), ("b", 100, 135, [34])], ["b"])
+    step([("e", 64, 66, [0, 1])], ["e"])
+    exe = os.path.join(m40.ROOT, "bin", "trace_run")
+    p = subprocess.run([exe, "--model", folders("odd"), "--dtype", "float32", "--out", str(tmp_path), "--max-tokens", str(4 * 192)], input="\n".join(steps) + "\n",
+                       capture_output=True, text=True, timeout=100)
+    assert p.returncode == 0, p.stderr[-2000:]
+    assert p.stdout.split("\n")[:-1] == ["done %d" % i for i in range(5)]
+    for i, r in enumerate(rows):
+        f = tmp_path / f"{i}.f32"
+        if not r:
+            assert not f.exists()
+            continue
+        assert_logits(np.fromfile(f, dtype="<f4").reshape(len(r), V), want[r], "float32")
