@@ -220,12 +220,17 @@ __global__ __launch_bounds__(256, 1) void tile_packed_kernel(PackedArgs g, M40Ep
         read_frags(f[ph ^ 1], next);
         issue(buf == 0 ? kBufs - 1 : buf - 1, t + kBufs - 1);
         compute(f[ph]);
-        constexpr int kPer = 4 * NTW / (4 + NTW);                    // products per fragment read
+        // products between two fragment reads, and between two loads
+        constexpr int kPerRead = NTW == 8 ? 2 : 1, kPerLoad = (4 * NTW - kPerRead * (4 + NTW)) / kLoads;
 #pragma unroll
         for (int i = 0; i < 4 + NTW; ++i) {
-            __builtin_amdgcn_sched_group_barrier(0x008, kPer, 0);
+            __builtin_amdgcn_sched_group_barrier(0x008, kPerRead, 0);
             __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
-            if (i % 2 == 0) __builtin_amdgcn_sched_group_barrier(0x020, 1, 0);
+        }
+#pragma unroll
+        for (int i = 0; i < kLoads; ++i) {
+            __builtin_amdgcn_sched_group_barrier(0x008, kPerLoad, 0);
+            __builtin_amdgcn_sched_group_barrier(0x020, 1, 0);
         }
         m40_wait_and_meet<(kBufs - 3) * kLoads>();
         buf = next;
