@@ -25,7 +25,7 @@ HIP_SOURCES = ["context.hip", "elementwise.hip", "gemm.hip", "kvcache.hip", "att
 CPP_SOURCES = ["unavailable.cpp"]
 # per-file additions: matrix-instruction results straight into vector registers (the default form writes them to
 # accumulation registers and copies every element out again)
-HIP_FILE_FLAGS = {name: ["-mllvm", "-amdgpu-mfma-vgpr-form"] for name in ("prefill_attention.hip", "head_attention.hip", "packed_gemm.hip")}
+HIP_FILE_FLAGS = {name: ["-mllvm", "-amdgpu-mfma-vgpr-form"] for name in ("prefill_attention.hip", "head_attention.hip", "packed_gemm.hip", "latent_attention.hip")}
 
 
 def _run(cmd):

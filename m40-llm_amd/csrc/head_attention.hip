@@ -210,8 +210,9 @@ int launch(hipStream_t stream, const M40llmHeadAttention& a) {
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
 template <int DKT, int DVT>
-int launch_any(hipStream_t stream, const M40llmHeadAttention& a) {
-    if (lds_bytes(a.plain_tiles + a.rot_tiles, a.v_tiles, 2) <= kLdsMax)
+int launch_any(hipStream_t stream, const M40llmHeadAttention& a, int num_cus) {
+    // with enough workgroups the short ones fill in behind the long ones, and two independent groups a CU run better than one of eight waves
+    if (lds_bytes(a.plain_tiles + a.rot_tiles, a.v_tiles, 2) <= kLdsMax && (uint64_t)a.heads * a.n_jobs <= 3ull * (uint32_t)num_cus)
         return a.job_rows == 64u ? launch<DKT, DVT, 1, 2>(stream, a) : launch<DKT, DVT, 2, 2>(stream, a);
     return a.job_rows == 64u ? launch<DKT, DVT, 1, 1>(stream, a) : launch<DKT, DVT, 2, 1>(stream, a);
 }
@@ -232,11 +233,11 @@ int m40llm_ext_head_attention_async(M40llmCudaContext* ctx, const M40llmHeadAtte
         !m40llm_ext_head_attention_serves(kt, p->v_tiles))
         return -3;
     (void)hipGetLastError();
-    if (kt <= 3u && p->v_tiles <= 4u) return launch_any<3, 4>(stream, *p);
-    if (kt <= 3u) return launch_any<3, 8>(stream, *p);
-    if (kt <= 6u && p->v_tiles <= 4u) return launch_any<6, 4>(stream, *p);
-    if (kt <= 6u) return launch_any<6, 8>(stream, *p);
-    return launch_any<8, 8>(stream, *p);
+    if (kt <= 3u && p->v_tiles <= 4u) return launch_any<3, 4>(stream, *p, ctx->num_cus);
+    if (kt <= 3u) return launch_any<3, 8>(stream, *p, ctx->num_cus);
+    if (kt <= 6u && p->v_tiles <= 4u) return launch_any<6, 4>(stream, *p, ctx->num_cus);
+    if (kt <= 6u) return launch_any<6, 8>(stream, *p, ctx->num_cus);
+    return launch_any<8, 8>(stream, *p, ctx->num_cus);
 }
 
 }  // extern "C"

@@ -207,7 +207,9 @@ __global__ __launch_bounds__(256, 1) void latent_attention_kernel(LatentArgs a) 
 }
 
 // The same walk for up to two row tiles with the query operands in registers and two page buffers: a page is on its way while the
-// page before is worked on.  Wave w sums latent column tiles w, w + 4, ...
+// page before is worked on.  Wave w sums latent column tiles w, w + 4, ...  Tiles past the entry's are read again and multiplied by
+// zero, columns past the latent's summed and not stored: a branch around either would put an LDS round trip between products.
+// Scores and maxima carry a factor log2(e).
 template <int MT, int VTW, int KT>
 __global__ __launch_bounds__(256, 1) void latent_decode_kernel(LatentArgs a) {
     typedef __attribute__((address_space(3))) void* lds_dst_t;
@@ -243,7 +245,10 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(LatentArgs a) {
         r = r < count ? r : count - 1u;
         const m40_bf16* src = static_cast<const m40_bf16*>(a.queries) + (size_t)(q0 + r) * width + (lane >> 4) * 8;
 #pragma unroll
-        for (int k = 0; k < KT; ++k) qf[m][k] = *reinterpret_cast<const m40_bf16x8*>(src + (k < kt ? k : kt - 1) * 32);
+        for (int k = 0; k < KT; ++k) {
+            qf[m][k] = *reinterpret_cast<const m40_bf16x8*>(src + (k < kt ? k : kt - 1) * 32);
+            if (k >= kt) qf[m][k] = m40_bf16x8{};
+        }
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const uint32_t row = (uint32_t)(m * 16 + 4 * (lane >> 4) + i);
@@ -260,6 +265,7 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(LatentArgs a) {
         for (int r = 0; r < 4; ++r) { mx[m][r] = -INFINITY; ls[m][r] = 0.0f; }
     }
     const int v_tiles = (int)a.latent_pad / 16;
+    const float scale = a.scale * 1.4426950408889634f;
     int buf = 0;
     for (uint32_t p = page0; p < page1; ++p, buf ^= 1) {
         m40_wait_and_meet<0>();              // page p has landed, and nobody reads the other buffer any more
@@ -272,18 +278,17 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(LatentArgs a) {
 #pragma unroll
         for (int m = 0; m < MT; ++m) s[m] = m40_float4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int k = 0; k < KT; ++k)
-            if (k < kt) {
-                const m40_bf16x8 kf = *reinterpret_cast<const m40_bf16x8*>(page_lds + (wave * kt + k) * 1024 + lane * 16);
+        for (int k = 0; k < KT; ++k) {
+            const m40_bf16x8 kf = *reinterpret_cast<const m40_bf16x8*>(page_lds + (wave * kt + (k < kt ? k : kt - 1)) * 1024 + lane * 16);
 #pragma unroll
-                for (int m = 0; m < MT; ++m) s[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[m][k], kf, s[m], 0, 0, 0);
-            }
+            for (int m = 0; m < MT; ++m) s[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[m][k], kf, s[m], 0, 0, 0);
+        }
         const uint32_t key = p * kPage + wave * 16 + (lane & 15);
 #pragma unroll
         for (int m = 0; m < MT; ++m)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-                s[m][r] = key <= pos[m][r] ? s[m][r] * a.scale : -INFINITY;
+                s[m][r] = key <= pos[m][r] ? s[m][r] * scale : -INFINITY;
                 const float t = m40_max16(s[m][r]);
                 if ((lane & 15) == 0) max_lds[wave * 16 * MT + m * 16 + 4 * (lane >> 4) + r] = t;
             }
@@ -298,9 +303,9 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(LatentArgs a) {
 #pragma unroll
                 for (int w = 0; w < 4; ++w) top = fmaxf(top, max_lds[w * 16 * MT + i]);
                 const float safe = top == -INFINITY ? 0.0f : top;       // a row that has seen nothing yet
-                alpha[m][r] = expf(mx[m][r] - safe);
+                alpha[m][r] = __builtin_amdgcn_exp2f(mx[m][r] - safe);
                 mx[m][r] = top;
-                const float e = expf(s[m][r] - safe);
+                const float e = __builtin_amdgcn_exp2f(s[m][r] - safe);
                 ls[m][r] = ls[m][r] * alpha[m][r] + e;
                 const int k = (wave & 1) * 16 + (lane & 15);
                 reinterpret_cast<m40_bf16*>(p_lds)[(m * 2 + (wave >> 1)) * kM40Tile + ((k >> 3) * 16 + (i & 15)) * 8 + (k & 7)] = static_cast<m40_bf16>(e);
@@ -321,14 +326,12 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(LatentArgs a) {
             const uint8_t* group = page_lds + (2 * c + (g >> 1)) * kt * 1024;
 #pragma unroll
             for (int j = 0; j < VTW; ++j) {
-                const int n = j * 4 + wave;
-                if (n < v_tiles) {
-                    const int d = n * 16 + (li & 3) * 4;
-                    const uint8_t* at = group + (d >> 5) * 1024 + (((d & 31) >> 3) * 16 + tok) * 16 + (d & 7) * 2;
-                    const m40_bf16x8 vf = read_transposed(at, at + 4 * 16);
+                const int n = j * 4 + wave < v_tiles ? j * 4 + wave : v_tiles - 1;
+                const int d = n * 16 + (li & 3) * 4;
+                const uint8_t* at = group + (d >> 5) * 1024 + (((d & 31) >> 3) * 16 + tok) * 16 + (d & 7) * 2;
+                const m40_bf16x8 vf = read_transposed(at, at + 4 * 16);
 #pragma unroll
-                    for (int m = 0; m < MT; ++m) o[m][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[m], vf, o[m][j], 0, 0, 0);
-                }
+                for (int m = 0; m < MT; ++m) o[m][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[m], vf, o[m][j], 0, 0, 0);
             }
         }
     }
@@ -351,6 +354,7 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(LatentArgs a) {
 #pragma unroll
             for (int w = 0; w < 4; ++w) l += max_lds[w * 16 * MT + i];
             const uint32_t q = q0 + i;
+            mx[m][r] *= 0.6931471805599453f;
             const float f = a.splits == 1u ? sink_factor(mx[m][r], l, a.sink[q % a.heads]) : 1.0f;
             const uint32_t row = q / a.heads, col = q % a.heads * a.latent_pad + (lane & 15);
             const size_t at = (size_t)blockIdx.y * a.n_queries + (q - a.first_query);
@@ -500,6 +504,8 @@ int launch_bf16_m(hipStream_t stream, const LatentArgs& a, uint32_t n_tiles) {
     const uint32_t per_wave = (a.latent_pad / 16u + 3u) / 4u;
     if constexpr (MT <= 2) {
         if (a.k_tiles <= 6u && per_wave <= 3u) return launch_decode<MT, 3, 6>(stream, a, n_tiles);
+        if (a.k_tiles <= 10u && per_wave <= 4u) return launch_decode<MT, 4, 10>(stream, a, n_tiles);
+        if (a.k_tiles <= 18u && per_wave <= 8u) return launch_decode<MT, 8, 18>(stream, a, n_tiles);
         if (a.k_tiles <= 19u && per_wave <= 10u) return launch_decode<MT, 10, 19>(stream, a, n_tiles);
     }
     if (per_wave <= 1u) return launch_bf16<MT, 1>(stream, a, n_tiles);
