@@ -561,13 +561,16 @@ int m40llm_ext_clear_u32_async(M40llmCudaContext* ctx, void* d_dst, size_t n, ui
 #define M40LLM_PACKED_ROTATE 4u     /* heads of [plain | rotated] columns: pairs (2i, 2i+1) of the rotated part are rotated;
                                        out_act packed, rot_out (rows below split_row) plain */
 #define M40LLM_PACKED_PROJECT 5u    /* the first plain_tiles tiles: as STORE; then pairs of tiles (gate, up):
-                                       out_act[row][act_col + 16*pair + c] = gelu_tanh(gate) * up, packed */
+                                       out_act[row][act_col + 16*pair + c] = activation(gate) * up, packed */
 /* bf16, rows read from cache pages (a = the layer's cache, pages = page numbers, rows = 64 * their number):
  * KEYS: out_act = the result as a packed operand, 16-row tile after 16-row tile of n_tiles/2 k tiles;
  * VALUES: out_act = the result transposed, per page and column tile two operand tiles [16 columns][32 rows], row
  * 16t + 4g + r of 32 at place 8g + 4t + r (the order of m40llm_ext_head_attention_async) */
 #define M40LLM_PACKED_KEYS 6u
 #define M40LLM_PACKED_VALUES 7u
+#define M40LLM_PACKED_SILU 8u       /* the first plain_tiles tiles: as STORE; then out_act[row][act_col + col] = silu(v), packed */
+#define M40LLM_GELU_TANH 0u
+#define M40LLM_SILU 1u
 typedef struct M40llmPackedGemm {
     uint32_t act_dtype, epilogue;
     const void* a;                /* packed [rows][lda] activations */
@@ -590,6 +593,12 @@ typedef struct M40llmPackedGemm {
     uint32_t k_parts;             /* STORE: K in that many parts, part p's sums at out_f32 + p*out_batch (0, 1 = whole) */
     const uint32_t* pages;        /* KEYS, VALUES: device */
     uint32_t page_k_tiles;        /* k tiles of a cache entry */
+    uint32_t activation;          /* PROJECT: M40LLM_GELU_TANH or M40LLM_SILU */
+    /* Products per expert (jobs not NULL; PROJECT without plain tiles, STORE_ACT): job j of the jobs[0] jobs behind word 4 is {expert,
+     * first slot, slots}, slots at most job_rows (16, 32, 64 or 128); weights of expert e start at w + e*w_batch.  With `gather`, the
+     * rows of a are plain rows gather[slot] of lda columns; without, packed rows `slot`.  Results are rows `slot`. */
+    const uint32_t *jobs, *gather;
+    uint32_t max_jobs, job_rows;
 } M40llmPackedGemm;
 int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm* g, uint32_t stream_kind);
 
@@ -608,6 +617,153 @@ int m40llm_ext_layer_norm_rows_async(M40llmCudaContext* ctx, void* d_x_f32, cons
  * formed in double precision */
 int m40llm_ext_rotation_angles_async(M40llmCudaContext* ctx, const uint32_t* d_positions, uint32_t rows, const double* d_freq,
                                      uint32_t pairs, uint32_t ld_pairs, float magnitude, void* d_angles, uint32_t stream_kind);
+
+/* The same with a scale on the token's row and a learned row per position; pair and position tables may be NULL.  h (may be NULL)
+ * takes the row as a packed operand of ld_h columns, zero past width. */
+typedef struct M40llmEmbedTokens {
+    uint32_t act_dtype, rows, vocab, width;
+    const void *table, *pair_table, *pos_table;      /* bf16 */
+    const uint32_t *tokens, *prev, *positions;
+    uint32_t buckets, mul_prev, mul_cur, n_positions;
+    float scale;
+    void* x;
+    void* h;
+    uint32_t ld_h;
+} M40llmEmbedTokens;
+int m40llm_ext_embed_tokens_async(M40llmCudaContext* ctx, const M40llmEmbedTokens* e, uint32_t stream_kind);
+#define M40LLM_NORM_LAYER 0u
+#define M40LLM_NORM_RMS 1u
+/* m40llm_ext_layer_norm_rows_async, or with norm_kind M40LLM_NORM_RMS x / sqrt(mean(x^2) + eps) * w */
+int m40llm_ext_norm_rows_async(M40llmCudaContext* ctx, uint32_t norm_kind, void* d_x_f32, const void* d_planes_f32, uint32_t n_planes,
+                               uint64_t plane_stride, const void* d_w_f32, const uint32_t* d_row_index, uint32_t rows, uint32_t width,
+                               float eps, void* d_out, uint32_t ld_out, uint32_t act_dtype, uint32_t stream_kind);
+/* The end of a sublayer with a norm on its output: x[row] += mult * y / sqrt(mean(y^2) + eps) * w.  y is the sum of n_planes planes of f32
+ * rows, plane_stride elements apart, or, where place is not NULL, sum_j weight[row*top + j] * r_j with r_j = row place[row*top + j] of
+ * expert_out, or x[row] itself where place is M40LLM_PLACE_INPUT.  The new row also goes to h (packed, ld_h columns, zero past width)
+ * and, where h_rows is not NULL, to plain rows of ld_h columns. */
+#define M40LLM_PLACE_INPUT 0xffffffffu
+typedef struct M40llmNormAdd {
+    uint32_t act_dtype, rows, width;
+    float eps, mult;
+    void* x;
+    const void* planes;
+    uint32_t n_planes, top;
+    uint64_t plane_stride;
+    const void* expert_out;          /* act type */
+    uint64_t ld_expert;
+    const uint32_t* place;
+    const void* weight;              /* f32 */
+    const void* w;
+    void *h, *h_rows;
+    uint32_t ld_h;
+} M40llmNormAdd;
+int m40llm_ext_norm_add_rows_async(M40llmCudaContext* ctx, const M40llmNormAdd* n, uint32_t stream_kind);
+/* out[row][c] = y / sqrt(mean(y^2) + eps) * w[c] * sigmoid(gate[row][c]), packed, ld_out columns, zero past cols (f32 rows y, gate) */
+int m40llm_ext_norm_gate_rows_async(M40llmCudaContext* ctx, const void* d_y, uint64_t ld_y, const void* d_w, const void* d_gate,
+                                    uint64_t ld_gate, uint32_t rows, uint32_t cols, float eps, void* d_out, uint32_t ld_out,
+                                    uint32_t act_dtype, uint32_t stream_kind);
+
+/* ---- routed feed-forwards ------------------------------------------------------------------------------------------------------
+ * Of `experts` + `identity` experts each row takes the `top` with the largest softmax(logits) + correction (the lower index of equals);
+ * its weights are the softmax values.  ids / weight: [rows][top].  Then rows are sorted by expert: every expert's rows, in order, take
+ * slots from a multiple of 16 on; rows_of[slot] = row (slots that pad a group of 16 repeat a row), place[row*top + j] = slot, or
+ * M40LLM_PLACE_INPUT for identity experts; jobs (m40llm_ext_packed_gemm_async) of at most job_rows slots.  rows_of holds
+ * m40llm_ext_expert_slots, jobs 4 + 4 * m40llm_ext_expert_max_jobs words. */
+typedef struct M40llmRoute {
+    uint32_t rows, experts, identity, top, job_rows;
+    const void* logits;              /* f32 [rows][ld_logits] */
+    uint64_t ld_logits;
+    const void* correction;          /* f32 [experts + identity] */
+    uint32_t* ids;
+    void* weight;                    /* f32 */
+    uint32_t *rows_of, *place, *jobs;
+} M40llmRoute;
+int m40llm_ext_route_rows_async(M40llmCudaContext* ctx, const M40llmRoute* r, uint32_t stream_kind);
+uint32_t m40llm_ext_expert_slots(uint32_t rows, uint32_t experts, uint32_t top);
+uint32_t m40llm_ext_expert_max_jobs(uint32_t rows, uint32_t experts, uint32_t top, uint32_t job_rows);
+#define M40LLM_MAX_EXPERTS 1024u
+
+/* ---- differential attention over a paged cache of keys and values ----------------------------------------------------------
+ * Every head has two maps: softmaxes of their own queries and keys over the same values, a1 and a2; o = a1 - lambda*a2, then
+ * o / sqrt(mean(o^2) + eps) * out_scale * sigmoid(gate[row][head]).  Query head h uses kv head h / (heads / kv_heads).
+ * A page holds 64 tokens; per kv head first the keys, map after map, as packed rows (4 x k_tiles tiles of 16 tokens x 32 dimensions),
+ * then the values transposed: per 16 dimensions two tiles [16 dimensions][32 tokens], token 16t + 4g + r at place 8g + 4t + r.
+ * k_tiles = dim/32, v_tiles = vdim/16, rounded up; page p starts at element p * m40llm_ext_pair_page_elements. */
+uint64_t m40llm_ext_pair_page_elements(uint32_t kv_heads, uint32_t dim, uint32_t vdim);
+/* From projected rows (f32: heads of [map 1 | map 2] query columns, the same for keys, value columns): causal convolution of `taps` taps
+ * on every column (0 = none), RMS norm over each map's dim of queries and keys; queries out as plain rows [heads][2][32*k_tiles], keys and
+ * values to the row's place in the cache (cache NULL = the layer reads another layer's: no key and value columns).
+ * row_back[row]: rows of the same portion before it, bit 31 set where the portion is one row.  conv_state [slot][taps - 1][ld_state]
+ * holds the columns of the rows before a portion, oldest first (rows before position 0 count as zero); portions of one row update it,
+ * the others by m40llm_ext_conv_state_async afterwards. */
+typedef struct M40llmPairSplit {
+    uint32_t act_dtype, rows, heads, kv_heads, dim, vdim, taps;
+    float eps;
+    const void* proj;
+    uint64_t ld_proj;
+    uint32_t k_offset, v_offset;            /* columns; queries start at 0 */
+    const void *q_conv, *k_conv, *v_conv;   /* f32 [columns][taps] */
+    const void *q_norm, *k_norm;            /* f32 [dim] */
+    void* conv_state;
+    uint64_t ld_state;
+    void* queries;
+    void* cache;
+    const uint32_t *row_slot, *row_pos, *row_back, *page_table;
+    uint32_t max_pages;
+} M40llmPairSplit;
+int m40llm_ext_pair_split_append_async(M40llmCudaContext* ctx, const M40llmPairSplit* s, uint32_t stream_kind);
+/* portions[p] = {first row, rows, slot, first position}: those of two rows and more leave the last taps - 1 of their columns in conv_state */
+int m40llm_ext_conv_state_async(M40llmCudaContext* ctx, const void* d_proj, uint64_t ld_proj, uint32_t cols, uint32_t taps, void* d_conv_state,
+                                uint64_t ld_state, const uint32_t* d_portions, uint32_t n_portions, uint32_t stream_kind);
+/* Query i of a kv head = row * (heads / kv_heads) + head within the group.  tiles[t] = {first query, queries}, all of one slot.
+ * form 0: at most 16 queries a tile, pages divided over waves and over `splits` workgroups (partial:
+ * m40llm_ext_pair_attention_partial_floats; rows first_row .. first_row + n_rows are joined by a second launch); form 1: at most tile_queries
+ * (64 or 128) queries a tile, operands through LDS; f32 takes rows one by one (tiles are not used).  out packed [rows][ld_out]. */
+typedef struct M40llmPairAttention {
+    uint32_t act_dtype, form, heads, kv_heads, dim, vdim;
+    float scale, lambda, out_scale, eps;
+    const void* queries;
+    const void* cache;
+    const void* gate;                 /* f32 */
+    uint64_t ld_gate;
+    const uint32_t *row_slot, *row_pos, *page_table;
+    uint32_t max_pages;
+    const uint32_t* tiles;
+    uint32_t n_tiles, tile_queries, splits, first_row, n_rows;
+    void* partial;
+    uint64_t partial_floats;
+    void* out;
+    uint32_t ld_out;
+} M40llmPairAttention;
+int m40llm_ext_pair_attention_async(M40llmCudaContext* ctx, const M40llmPairAttention* a, uint32_t stream_kind);
+uint64_t m40llm_ext_pair_attention_partial_floats(uint32_t rows, uint32_t heads, uint32_t vdim, uint32_t splits);
+/* most queries of a tile: 128 or 64 where form 1 is served, 16 where only form 0 is, 0 = sizes that are not served */
+uint32_t m40llm_ext_pair_attention_tile_queries(uint32_t act_dtype, uint32_t dim, uint32_t vdim);
+
+/* ---- lightning attention -----------------------------------------------------------------------------------------------------------
+ * Per head S <- decay*S + k v^T, o = S^T q, token by token; S in f32, state[slot][head][dim][32*ceil(vdim/32)], zero before position 0.
+ * qkv: packed rows of the activation type, columns: heads x 32*ceil(dim/32) queries, the same of keys, heads x 32*ceil(vdim/32) values.
+ * o: f32 [rows][heads*vdim].  portions[p] = {first row, rows, slot, first position}.
+ * serial: token after token (any type); chunked (bf16): over the 64-row groups of the pass that a portion touches.  chunk_base[p] = chunks
+ * of the portions before it; chunks[c] = {portion, first row of the group}; scratch: m40llm_ext_lightning_scratch_bytes. */
+typedef struct M40llmLightning {
+    uint32_t act_dtype, chunked, heads, dim, vdim;
+    const void* qkv;
+    uint64_t ld_qkv;
+    const void* log2_decay;           /* f32 [heads] */
+    const void* decay;                /* f32 [heads] */
+    void* state;
+    void* o;
+    uint64_t ld_o;
+    const uint32_t *portions, *chunk_base, *chunks, *row_pos;
+    uint32_t n_portions, n_chunks;
+    void* scratch;
+    uint64_t scratch_bytes;
+} M40llmLightning;
+int m40llm_ext_lightning_async(M40llmCudaContext* ctx, const M40llmLightning* l, uint32_t stream_kind);
+uint64_t m40llm_ext_lightning_scratch_bytes(uint32_t n_chunks, uint32_t heads, uint32_t dim, uint32_t vdim);
+/* whether heads of these sizes are served */
+int m40llm_ext_lightning_serves(uint32_t dim, uint32_t vdim);
 
 /* ---- latent attention over a paged cache ------------------------------------------------------------------------------------
  * A page holds 64 tokens; a token's entry is its normed latent (kv_rank, padded to a multiple of 32) followed by the rotated

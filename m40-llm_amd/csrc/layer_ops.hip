@@ -1,40 +1,54 @@
-// Row-wise steps of layered decoders: token + token-pair embedding, layer norm, rotation angles, and the step between a latent
+// Row-wise steps of layered decoders: embedding (token, token pair, position), norms, rotation angles, and the step between a latent
 // attention's projections and its attention (norms of the two latents, rotation, cache append).
 #include "packed_gemm.hpp"
+
+#include <type_traits>
 
 namespace {
 
 constexpr int kThreads = 256;
 
-__global__ __launch_bounds__(kThreads) void embed_pairs_kernel(const uint16_t* __restrict__ table, const uint16_t* __restrict__ pairs,
-                                                               const uint32_t* __restrict__ tokens, const uint32_t* __restrict__ prev,
-                                                               uint32_t vocab, uint32_t width, uint32_t buckets, uint32_t mul_prev,
-                                                               uint32_t mul_cur, float* __restrict__ x) {
-    const uint32_t row = blockIdx.x;
-    uint32_t tok = tokens[row];
-    tok = tok < vocab ? tok : vocab - 1u;
-    const uint16_t* a = table + (size_t)tok * width;
-    const uint16_t* b = nullptr;
-    if (pairs) {
-        const uint32_t p = prev[row];
-        const uint32_t r = p == 0xffffffffu ? buckets : (uint32_t)(((uint64_t)p * mul_prev + (uint64_t)tok * mul_cur) % buckets);
-        b = pairs + (size_t)r * width;
+template <class T>
+__global__ __launch_bounds__(kThreads) void embed_tokens_kernel(M40llmEmbedTokens e) {
+    const uint32_t row = m40_tile_row(blockIdx.x, e.rows), width = e.width;
+    uint32_t tok = e.tokens[row];
+    tok = tok < e.vocab ? tok : e.vocab - 1u;
+    const uint16_t* a = static_cast<const uint16_t*>(e.table) + (size_t)tok * width;
+    const uint16_t *b = nullptr, *c = nullptr;
+    if (e.pair_table) {
+        const uint32_t p = e.prev[row];
+        const uint32_t r = p == 0xffffffffu ? e.buckets : (uint32_t)(((uint64_t)p * e.mul_prev + (uint64_t)tok * e.mul_cur) % e.buckets);
+        b = static_cast<const uint16_t*>(e.pair_table) + (size_t)r * width;
     }
-    float* out = x + (size_t)row * width;
+    if (e.pos_table) {
+        const uint32_t p = e.positions[row];
+        c = static_cast<const uint16_t*>(e.pos_table) + (size_t)(p < e.n_positions ? p : e.n_positions - 1u) * width;
+    }
+    float* out = static_cast<float*>(e.x) + (size_t)row * width;
+    T* h = static_cast<T*>(e.h);
     if (width % 8u == 0) {
         for (uint32_t i = threadIdx.x; i < width / 8u; i += kThreads) {
-            const m40_bf16x8 va = reinterpret_cast<const m40_bf16x8*>(a)[i];
-            m40_f32x8 v = __builtin_convertvector(va, m40_f32x8);
+            m40_f32x8 v = __builtin_convertvector(reinterpret_cast<const m40_bf16x8*>(a)[i], m40_f32x8) * e.scale;
             if (b) v += __builtin_convertvector(reinterpret_cast<const m40_bf16x8*>(b)[i], m40_f32x8);
+            if (c) v += __builtin_convertvector(reinterpret_cast<const m40_bf16x8*>(c)[i], m40_f32x8);
             reinterpret_cast<m40_f32x8*>(out)[i] = v;
+            if (h) {
+                T* o = h + m40_packed_at(row, i * 8u, e.ld_h >> 5);
+                m40_store4<T>(o, m40_float4{v[0], v[1], v[2], v[3]});
+                m40_store4<T>(o + 4, m40_float4{v[4], v[5], v[6], v[7]});
+            }
         }
-        return;
+    } else {
+        for (uint32_t i = threadIdx.x; i < width; i += kThreads) {
+            float v = m40_bf16_bits(a[i]) * e.scale;
+            if (b) v += m40_bf16_bits(b[i]);
+            if (c) v += m40_bf16_bits(c[i]);
+            out[i] = v;
+            if (h) h[m40_packed_at(row, i, e.ld_h >> 5)] = M40Act<T>::from(v);
+        }
     }
-    for (uint32_t i = threadIdx.x; i < width; i += kThreads) {
-        float v = m40_bf16_bits(a[i]);
-        if (b) v += m40_bf16_bits(b[i]);
-        out[i] = v;
-    }
+    if (h)
+        for (uint32_t i = width + threadIdx.x; i < e.ld_h; i += kThreads) h[m40_packed_at(row, i, e.ld_h >> 5)] = M40Act<T>::from(0.0f);
 }
 
 // sum over the workgroup, the same bits in every thread
@@ -49,8 +63,8 @@ __device__ __forceinline__ float block_sum(float v, float* scratch) {
     return s;
 }
 
-// A thread takes groups of eight neighbouring elements: 16-byte pieces of a packed tile.
-template <class T, bool VEC>
+// A thread takes groups of eight neighbouring elements: 16-byte pieces of a packed tile.  RMS: the mean stays where it is.
+template <class T, bool VEC, bool RMS>
 __global__ __launch_bounds__(kThreads) void layer_norm_rows_kernel(float* __restrict__ x, const float* __restrict__ planes, uint32_t n_planes,
                                                                    size_t plane_stride, const float* __restrict__ w,
                                                                    const uint32_t* __restrict__ row_index, uint32_t width, float eps,
@@ -132,7 +146,7 @@ __global__ __launch_bounds__(kThreads) void layer_norm_rows_kernel(float* __rest
         load(g, v);
         sum8(v);
     }
-    mean = block_sum(s, scratch) / (float)width;
+    if (!RMS) mean = block_sum(s, scratch) / (float)width;
 #pragma unroll
     for (uint32_t j = 0; j < kGroups; ++j) sq8(threadIdx.x + j * kThreads, keep[j]);
     for (uint32_t g = threadIdx.x + kGroups * kThreads; g < groups; g += kThreads) {
@@ -264,37 +278,61 @@ int launched() { return hipGetLastError() == hipSuccess ? 0 : -2; }
 
 extern "C" {
 
+int m40llm_ext_embed_tokens_async(M40llmCudaContext* ctx, const M40llmEmbedTokens* e, uint32_t stream_kind) {
+    if (!ctx || !e || !e->table || !e->tokens || !e->x || (e->pair_table && !e->prev) || (e->pos_table && !e->positions)) return -1;
+    hipStream_t stream = m40_select_stream(ctx, stream_kind);
+    if (!stream || m40_ensure_device(ctx) != 0) return -2;
+    if (e->rows == 0 || e->vocab == 0 || e->width == 0 || e->act_dtype > 1u || (e->pair_table && e->buckets == 0) || (e->pos_table && e->n_positions == 0) ||
+        (e->h && (e->ld_h < e->width || e->ld_h % 32u != 0 || !m40_aligned16(e->h))))
+        return -3;
+    if (e->act_dtype == M40LLM_ACT_F32) embed_tokens_kernel<float><<<e->rows, kThreads, 0, stream>>>(*e);
+    else embed_tokens_kernel<m40_bf16><<<e->rows, kThreads, 0, stream>>>(*e);
+    return launched();
+}
+
 int m40llm_ext_embed_pairs_async(M40llmCudaContext* ctx, const void* d_table, const void* d_pairs, const uint32_t* d_tokens,
                                  const uint32_t* d_prev, uint32_t rows, uint32_t vocab, uint32_t width, uint32_t buckets,
                                  uint32_t mul_prev, uint32_t mul_cur, void* d_x, uint32_t stream_kind) {
-    if (!ctx || !d_table || !d_tokens || !d_x || (d_pairs && !d_prev)) return -1;
+    M40llmEmbedTokens e{};
+    e.rows = rows; e.vocab = vocab; e.width = width;
+    e.table = d_table; e.pair_table = d_pairs; e.tokens = d_tokens; e.prev = d_prev;
+    e.buckets = buckets; e.mul_prev = mul_prev; e.mul_cur = mul_cur;
+    e.scale = 1.0f;
+    e.x = d_x;
+    return m40llm_ext_embed_tokens_async(ctx, &e, stream_kind);
+}
+
+int m40llm_ext_norm_rows_async(M40llmCudaContext* ctx, uint32_t norm_kind, void* d_x, const void* d_planes, uint32_t n_planes, uint64_t plane_stride,
+                               const void* d_w, const uint32_t* d_row_index, uint32_t rows, uint32_t width, float eps, void* d_out,
+                               uint32_t ld_out, uint32_t act_dtype, uint32_t stream_kind) {
+    if (!ctx || !d_x || !d_w || !d_out || (n_planes && !d_planes)) return -1;
     hipStream_t stream = m40_select_stream(ctx, stream_kind);
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
-    if (rows == 0 || vocab == 0 || width == 0 || (d_pairs && buckets == 0)) return -3;
-    embed_pairs_kernel<<<rows, kThreads, 0, stream>>>(static_cast<const uint16_t*>(d_table), static_cast<const uint16_t*>(d_pairs), d_tokens,
-                                                      d_prev, vocab, width, buckets, mul_prev, mul_cur, static_cast<float*>(d_x));
+    if (norm_kind > M40LLM_NORM_RMS || rows == 0 || width == 0 || ld_out < width || ld_out % 32u != 0 || act_dtype > 1u || !m40_aligned16(d_out)) return -3;
+    float* x = static_cast<float*>(d_x);
+    const float *w = static_cast<const float*>(d_w), *p = static_cast<const float*>(d_planes);
+    const bool vec = width % 8u == 0 && plane_stride % 4u == 0 && m40_aligned16(d_x) && (!n_planes || m40_aligned16(d_planes));
+    auto go = [&](auto kernel, auto* out) { kernel<<<rows, kThreads, 0, stream>>>(x, p, n_planes, (size_t)plane_stride, w, d_row_index, width, eps, out, ld_out); };
+    auto pick = [&](auto* out, auto rms) {
+        typedef std::remove_reference_t<decltype(*out)> T;
+        constexpr bool kRms = decltype(rms)::value;
+        if (vec) go(layer_norm_rows_kernel<T, true, kRms>, out);
+        else go(layer_norm_rows_kernel<T, false, kRms>, out);
+    };
+    auto kind = [&](auto* out) {
+        if (norm_kind == M40LLM_NORM_RMS) pick(out, std::true_type());
+        else pick(out, std::false_type());
+    };
+    if (act_dtype == M40LLM_ACT_F32) kind(static_cast<float*>(d_out));
+    else kind(static_cast<m40_bf16*>(d_out));
     return launched();
 }
 
 int m40llm_ext_layer_norm_rows_async(M40llmCudaContext* ctx, void* d_x, const void* d_planes, uint32_t n_planes, uint64_t plane_stride,
                                      const void* d_w, const uint32_t* d_row_index, uint32_t rows, uint32_t width, float eps, void* d_out,
                                      uint32_t ld_out, uint32_t act_dtype, uint32_t stream_kind) {
-    if (!ctx || !d_x || !d_w || !d_out || (n_planes && !d_planes)) return -1;
-    hipStream_t stream = m40_select_stream(ctx, stream_kind);
-    if (!stream || m40_ensure_device(ctx) != 0) return -2;
-    if (rows == 0 || width == 0 || ld_out < width || ld_out % 32u != 0 || act_dtype > 1u || !m40_aligned16(d_out)) return -3;
-    float* x = static_cast<float*>(d_x);
-    const float *w = static_cast<const float*>(d_w), *p = static_cast<const float*>(d_planes);
-    const bool vec = width % 8u == 0 && plane_stride % 4u == 0 && m40_aligned16(d_x) && (!n_planes || m40_aligned16(d_planes));
-    auto go = [&](auto kernel, auto* out) { kernel<<<rows, kThreads, 0, stream>>>(x, p, n_planes, (size_t)plane_stride, w, d_row_index, width, eps, out, ld_out); };
-    if (act_dtype == M40LLM_ACT_F32) {
-        if (vec) go(layer_norm_rows_kernel<float, true>, static_cast<float*>(d_out));
-        else go(layer_norm_rows_kernel<float, false>, static_cast<float*>(d_out));
-    } else {
-        if (vec) go(layer_norm_rows_kernel<m40_bf16, true>, static_cast<m40_bf16*>(d_out));
-        else go(layer_norm_rows_kernel<m40_bf16, false>, static_cast<m40_bf16*>(d_out));
-    }
-    return launched();
+    return m40llm_ext_norm_rows_async(ctx, M40LLM_NORM_LAYER, d_x, d_planes, n_planes, plane_stride, d_w, d_row_index, rows, width, eps, d_out, ld_out,
+                                      act_dtype, stream_kind);
 }
 
 int m40llm_ext_rotation_angles_async(M40llmCudaContext* ctx, const uint32_t* d_positions, uint32_t rows, const double* d_freq, uint32_t pairs,

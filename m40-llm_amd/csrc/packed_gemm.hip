@@ -7,6 +7,9 @@
 // tile_packed_kernel   bf16, more rows: 128 x (128 or 256) tiles of C, both operands staged through LDS by direct
 //                      global-to-LDS loads, five or six steps of 32 k deep with one barrier a step.  The buffers hold
 //                      operands in instruction order, so LDS reads are contiguous kilobytes as well.
+//
+// Products per expert: both kernels take a list of jobs (expert, rows of the list sorted by expert) made on the device; the rows are
+// gathered from plain rows (gate and up) or lie packed in list order (down).
 #include "packed_gemm.hpp"
 
 #include <type_traits>
@@ -23,20 +26,33 @@ struct PackedArgs {
     // operand rows that lie in cache pages: row tile t is group t % 4 of page pages[t / 4]
     const uint32_t* pages;
     int page_k_tiles;
+    const uint32_t *jobs, *gather; // products per expert
     __device__ int k_count(int batch) const { return k_total && k_total - batch * k_tiles < k_tiles ? k_total - batch * k_tiles : k_tiles; }
 };
 
-template <class T, int MT, int NT, int WAVES>
+enum { kAllRows = 0, kJobSlots = 1, kJobGather = 2 };
+
+template <class T, int MT, int NT, int WAVES, int JOBS>
 __global__ __launch_bounds__(WAVES * 64) void rows_packed_kernel(PackedArgs g, M40Epilogue<T> e) {
     extern __shared__ __align__(16) float red[];       // [WAVES][MT][NT][64][4]
     typedef typename M40Act<T>::vec8 vec8;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    const int tile0 = (int)blockIdx.x * NT, row0 = (int)blockIdx.y * 16 * MT, batch = blockIdx.z;
+    const int tile0 = (int)blockIdx.x * NT;
+    int row0 = (int)blockIdx.y * 16 * MT, batch = blockIdx.z;
+    if (JOBS != kAllRows) {
+        if (blockIdx.y >= g.jobs[0]) return;
+        const uint32_t* job = g.jobs + 4 + 4 * blockIdx.y;
+        batch = (int)job[0];
+        row0 = (int)job[1];
+        g.rows = e.rows = row0 + (int)job[2];
+    }
+    constexpr long kStep = JOBS == kJobGather ? 32 : kM40Tile;       // elements from k tile to k tile
     const T* a[MT];
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
-        const int rt = row0 / 16 + m, last = (g.rows - 1) / 16;
-        a[m] = static_cast<const T*>(g.a) + batch * g.a_batch + (long)(rt < last ? rt : last) * 16 * g.lda + lane * 8;
+        const int rt = row0 / 16 + m, last = (g.rows - 1) / 16, c = rt < last ? rt : last;
+        if (JOBS == kJobGather) a[m] = static_cast<const T*>(g.a) + (long)g.gather[c * 16 + (lane & 15)] * g.lda + (lane >> 4) * 8;
+        else a[m] = static_cast<const T*>(g.a) + (JOBS == kAllRows ? batch * g.a_batch : 0) + (long)c * 16 * g.lda + lane * 8;
     }
     const m40_bf16* w[NT];
 #pragma unroll
@@ -62,7 +78,7 @@ __global__ __launch_bounds__(WAVES * 64) void rows_packed_kernel(PackedArgs g, M
 #pragma unroll
         for (int u = 0; u < U; ++u)
 #pragma unroll
-            for (int m = 0; m < MT; ++m) af[u][m] = M40Act<T>::load8(a[m] + (long)(k + u * WAVES) * kM40Tile);
+            for (int m = 0; m < MT; ++m) af[u][m] = M40Act<T>::load8(a[m] + (long)(k + u * WAVES) * kStep);
 #pragma unroll
         for (int u = 0; u < U; ++u)
 #pragma unroll
@@ -76,7 +92,7 @@ __global__ __launch_bounds__(WAVES * 64) void rows_packed_kernel(PackedArgs g, M
         for (int n = 0; n < NT; ++n) wf[n] = *reinterpret_cast<const uint4*>(w[n] + (long)k * kM40Tile);
 #pragma unroll
         for (int m = 0; m < MT; ++m) {
-            const vec8 af = M40Act<T>::load8(a[m] + (long)k * kM40Tile);
+            const vec8 af = M40Act<T>::load8(a[m] + (long)k * kStep);
 #pragma unroll
             for (int n = 0; n < NT; ++n) acc[m][n] = M40Act<T>::mma(__builtin_bit_cast(m40_bf16x8, wf[n]), af, acc[m][n]);
         }
@@ -101,34 +117,39 @@ __global__ __launch_bounds__(WAVES * 64) void rows_packed_kernel(PackedArgs g, M
         } else {
 #pragma unroll
             for (int n = 0; n < NT; ++n)
-                if (tile0 + n < g.n_tiles) m40_epilogue_tile(e, batch, row0 + m * 16, tile0 + n, lane, s[n]);
+                if (tile0 + n < g.n_tiles) m40_epilogue_tile(e, JOBS == kAllRows ? batch : 0, row0 + m * 16, tile0 + n, lane, s[n]);
         }
     }
 }
 
-template <class T, int MT, int NT, int WAVES>
+template <class T, int MT, int NT, int WAVES, int JOBS>
 int launch_rows(hipStream_t stream, const PackedArgs& g, const M40Epilogue<T>& e, int batches) {
-    const dim3 grid((unsigned)((g.n_tiles + NT - 1) / NT), (unsigned)((g.rows + 16 * MT - 1) / (16 * MT)), (unsigned)batches);
+    // g.rows: with jobs, the most jobs there can be
+    const dim3 grid((unsigned)((g.n_tiles + NT - 1) / NT), (unsigned)(JOBS == kAllRows ? (g.rows + 16 * MT - 1) / (16 * MT) : g.rows), (unsigned)batches);
     constexpr size_t lds = (size_t)WAVES * MT * NT * 1024;
-    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(rows_packed_kernel<T, MT, NT, WAVES>),
+    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(rows_packed_kernel<T, MT, NT, WAVES, JOBS>),
                                                        hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (attr != hipSuccess) return -2;
-    rows_packed_kernel<T, MT, NT, WAVES><<<grid, WAVES * 64, lds, stream>>>(g, e);
+    rows_packed_kernel<T, MT, NT, WAVES, JOBS><<<grid, WAVES * 64, lds, stream>>>(g, e);
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
 
-template <class T, int MT>
+template <class T, int MT, int JOBS>
 int launch_rows_m(hipStream_t stream, const PackedArgs& g, const M40Epilogue<T>& e, int batches) {
-    if (e.kind == M40LLM_PACKED_PROJECT) return launch_rows<T, MT, 2, 8>(stream, g, e, batches);
-    if (g.k_tiles >= 64) return launch_rows<T, MT, 1, 16>(stream, g, e, batches);
-    if (g.k_tiles >= 16) return launch_rows<T, MT, 1, 8>(stream, g, e, batches);
-    return launch_rows<T, MT, 1, 4>(stream, g, e, batches);
+    if constexpr (JOBS != kJobSlots)
+        if (e.kind == M40LLM_PACKED_PROJECT) return launch_rows<T, MT, 2, 8, JOBS>(stream, g, e, batches);
+    if constexpr (JOBS != kJobGather) {
+        if (g.k_tiles >= 64) return launch_rows<T, MT, 1, 16, JOBS>(stream, g, e, batches);
+        if (g.k_tiles >= 16) return launch_rows<T, MT, 1, 8, JOBS>(stream, g, e, batches);
+        return launch_rows<T, MT, 1, 4, JOBS>(stream, g, e, batches);
+    }
+    return -3;
 }
-template <class T>
-int launch_rows_any(hipStream_t stream, const PackedArgs& g, const M40Epilogue<T>& e, int batches) {
-    if (g.rows <= 16) return launch_rows_m<T, 1>(stream, g, e, batches);
-    if (g.rows <= 32) return launch_rows_m<T, 2>(stream, g, e, batches);
-    return launch_rows_m<T, 4>(stream, g, e, batches);
+template <class T, int JOBS>
+int launch_rows_any(hipStream_t stream, const PackedArgs& g, const M40Epilogue<T>& e, int batches, int rows) {
+    if (rows <= 16) return launch_rows_m<T, 1, JOBS>(stream, g, e, batches);
+    if (rows <= 32) return launch_rows_m<T, 2, JOBS>(stream, g, e, batches);
+    return launch_rows_m<T, 4, JOBS>(stream, g, e, batches);
 }
 
 // ---- many rows, bf16 ---------------------------------------------------------------------------------------------------
@@ -139,7 +160,7 @@ int launch_rows_any(hipStream_t stream, const PackedArgs& g, const M40Epilogue<T
 // ahead go out one at a time between the current step's products (sched_group_barrier), so that no wave waits for an address
 // or LDS unit with the matrix pipe idle.  Step t refills the buffer of step t - 1, whose fragments every wave had in registers
 // before the barrier behind that step, and ends with step t + 2 landed.
-enum { kPlainRows = 0, kPageKeys = 1, kPageValues = 2 };
+enum { kPlainRows = 0, kPageKeys = 1, kPageValues = 2, kSlots = 3, kGather = 4 };
 constexpr int tile_bufs(int ntw) { return ntw == 8 ? 6 : 5; }       // one or two workgroups a CU
 
 template <int NTW, int FORM>
@@ -151,14 +172,24 @@ __global__ __launch_bounds__(256, 1) void tile_packed_kernel(PackedArgs g, M40Ep
     constexpr int kBufs = tile_bufs(NTW), kStepBytes = (kATiles + kBTiles) * 1024;
     constexpr int kLoads = (kATiles + kBTiles) / 4;                  // per wave and step
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-    const int tiles_n = (g.n_tiles + kBTiles - 1) / kBTiles, tiles_m = (g.rows + 127) / 128;
+    constexpr bool kJobs = FORM == kSlots || FORM == kGather;
+    const int tiles_n = (g.n_tiles + kBTiles - 1) / kBTiles, tiles_m = kJobs ? (int)g.jobs[0] : (g.rows + 127) / 128;
+    const int workgroups = kJobs ? tiles_m * tiles_n : (int)gridDim.x;       // the grid is as large as the list of jobs can be
+    if (kJobs && (int)blockIdx.x >= workgroups) return;
     // workgroups are dealt to the eight dies in turn: each die gets a contiguous band of tiles, walked in blocks of four row
     // tiles so that what runs on a die at one time shares both operands
-    const int per_die = (int)gridDim.x / 8;
+    const int per_die = workgroups / 8;
     const int logical = (int)blockIdx.x < per_die * 8 ? ((int)blockIdx.x % 8) * per_die + (int)blockIdx.x / 8 : (int)blockIdx.x;
     const int group = logical / (4 * tiles_n), in_group = logical - group * 4 * tiles_n, gm = tiles_m - group * 4 < 4 ? tiles_m - group * 4 : 4;
-    const int m0 = (group * 4 + in_group % gm) * 128, t0 = in_group / gm * kBTiles, batch = blockIdx.z;
-    const m40_bf16* A = static_cast<const m40_bf16*>(g.a) + batch * g.a_batch;
+    const int t0 = in_group / gm * kBTiles;
+    int m0 = (group * 4 + in_group % gm) * 128, batch = blockIdx.z;
+    if (kJobs) {
+        const uint32_t* job = g.jobs + 4 + 4 * (group * 4 + in_group % gm);
+        batch = __builtin_amdgcn_readfirstlane((int)job[0]);
+        m0 = __builtin_amdgcn_readfirstlane((int)job[1]);
+        g.rows = e.rows = m0 + __builtin_amdgcn_readfirstlane((int)job[2]);
+    }
+    const m40_bf16* A = static_cast<const m40_bf16*>(g.a) + (kJobs ? 0 : batch * g.a_batch);
     const m40_bf16* W = g.w + batch * g.w_batch;
     const int k_tiles = g.k_count(batch);
     // this wave's pieces of a step: operand tiles wave, wave + 4, ... of the A tiles, then of the W tiles
@@ -167,12 +198,13 @@ __global__ __launch_bounds__(256, 1) void tile_packed_kernel(PackedArgs g, M40Ep
     for (int i = 0; i < kLoads; ++i) {
         const int t = wave + 4 * i;
         if (i < kATiles / 4) {
-            if (FORM != kPlainRows) {
+            if (FORM == kPageKeys || FORM == kPageValues) {
                 const int rt = m0 / 16 + t, tiles = g.rows / 16, c = rt < tiles ? rt : tiles - 1;
                 src[i] = A + ((long)g.pages[c >> 2] * 4 + (c & 3)) * g.page_k_tiles * kM40Tile + lane * 8;
             } else {
-                const int rt = m0 / 16 + t, last = (g.rows - 1) / 16;
-                src[i] = A + (long)(rt < last ? rt : last) * 16 * g.lda + lane * 8;
+                const int rt = m0 / 16 + t, last = (g.rows - 1) / 16, c = rt < last ? rt : last;
+                if (FORM == kGather) src[i] = A + (long)g.gather[c * 16 + (lane & 15)] * g.lda + (lane >> 4) * 8;
+                else src[i] = A + (long)c * 16 * g.lda + lane * 8;
             }
         } else {
             const int n = t0 + t - kATiles;
@@ -184,7 +216,7 @@ __global__ __launch_bounds__(256, 1) void tile_packed_kernel(PackedArgs g, M40Ep
         const int k = t < k_tiles ? t : k_tiles - 1;                 // past the end: loaded again, not used
 #pragma unroll
         for (int i = 0; i < kLoads; ++i)
-            __builtin_amdgcn_global_load_lds((global_src_t)(src[i] + (long)k * kM40Tile), (lds_dst_t)(base + i * 4096), 16, 0, 0);
+            __builtin_amdgcn_global_load_lds((global_src_t)(src[i] + (long)k * (FORM == kGather && i < kATiles / 4 ? 32 : kM40Tile)), (lds_dst_t)(base + i * 4096), 16, 0, 0);
     };
     const int wm = wave >> 1, wn = wave & 1;
     m40_float4 acc[4][NTW];
@@ -282,7 +314,7 @@ __global__ __launch_bounds__(256, 1) void tile_packed_kernel(PackedArgs g, M40Ep
             if (second) m40_epilogue_pair(e, row0, (tile - e.plain_tiles) / 2, lane, v0, v1);
         } else {
 #pragma unroll 1
-            for (int k = 0; k < (second ? 2 : 1); ++k) m40_epilogue_tile(e, batch, row0, tile + k, lane, k ? v1 : v0);
+            for (int k = 0; k < (second ? 2 : 1); ++k) m40_epilogue_tile(e, kJobs ? 0 : batch, row0, tile + k, lane, k ? v1 : v0);
         }
     }
 }
@@ -293,13 +325,14 @@ int launch_tile(hipStream_t stream, const PackedArgs& g, const M40Epilogue<m40_b
     static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(tile_packed_kernel<NTW, FORM>),
                                                        hipFuncAttributeMaxDynamicSharedMemorySize, lds);
     if (attr != hipSuccess) return -2;
-    const long long tiles = (long long)((g.rows + 127) / 128) * ((g.n_tiles + 2 * NTW - 1) / (2 * NTW));
+    constexpr bool kJobs = FORM == kSlots || FORM == kGather;        // g.rows: the most jobs there can be
+    const long long tiles = (long long)(kJobs ? g.rows : (g.rows + 127) / 128) * ((g.n_tiles + 2 * NTW - 1) / (2 * NTW));
     tile_packed_kernel<NTW, FORM><<<dim3((unsigned)tiles, 1, (unsigned)batches), 256, lds, stream>>>(g, e);
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
 template <int FORM>
 int launch_tile_any(hipStream_t stream, const PackedArgs& g, const M40Epilogue<m40_bf16>& e, int batches, int num_cus) {
-    const long long wide = (long long)((g.rows + 127) / 128) * ((g.n_tiles + 15) / 16) * batches;
+    const long long wide = (long long)(FORM == kSlots || FORM == kGather ? g.rows : (g.rows + 127) / 128) * ((g.n_tiles + 15) / 16) * batches;
     // a short sum is mostly a workgroup's start and end: two narrower workgroups a CU cover each other's
     if (wide * 16 >= 9ll * num_cus && g.k_tiles > 32) return launch_tile<8, FORM>(stream, g, e, batches);
     return launch_tile<4, FORM>(stream, g, e, batches);
@@ -319,6 +352,7 @@ M40Epilogue<T> make_epilogue(const M40llmPackedGemm& p) {
     e.vec_out = p.ld_out % 4 == 0 && p.out_batch % 4 == 0 && aligned(p.out_f32, 16);
     e.vec_act = p.ld_act % 4 == 0 && p.act_batch % 4 == 0 && aligned(p.out_act, 4 * sizeof(T));
     e.plain_tiles = (int)p.plain_tiles;
+    e.activation = (int)p.activation;
     e.n_tiles = (int)p.n_tiles; e.act_col = (int)p.act_col;
     e.gate = static_cast<const float*>(p.gate);
     e.ld_gate = (long)p.ld_gate;
@@ -404,14 +438,18 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
     const bool paged = p->epilogue == M40LLM_PACKED_KEYS || p->epilogue == M40LLM_PACKED_VALUES;
     const uint32_t k_parts = p->k_parts > 1u ? p->k_parts : 1u, part_tiles = (p->k_tiles + k_parts - 1) / k_parts;
-    if (p->act_dtype > 1u || p->epilogue > M40LLM_PACKED_VALUES || p->rows == 0 || p->batches == 0 || p->batches > 65535u ||
+    if (p->act_dtype > 1u || p->epilogue > M40LLM_PACKED_SILU || p->activation > M40LLM_SILU || p->rows == 0 || p->batches == 0 || p->batches > 65535u ||
         p->n_tiles == 0 || p->k_tiles == 0 || !m40_aligned16(p->a) || !m40_aligned16(p->w) || p->rows > 0x3fffffffu ||
         (p->batches > 1u && (p->a_batch % 32 != 0 || p->w_batch % 8 != 0)))
+        return -3;
+    if (p->jobs && (p->batches != 1u || k_parts > 1u || p->max_jobs == 0 || p->max_jobs > 65535u || (p->job_rows != 16u && p->job_rows != 32u && p->job_rows != 64u && p->job_rows != 128u) ||
+                    (p->job_rows == 128u && p->act_dtype == M40LLM_ACT_F32) || p->w_batch % 8 != 0 ||
+                    (p->gather ? p->epilogue != M40LLM_PACKED_PROJECT || p->plain_tiles != 0 : p->epilogue != M40LLM_PACKED_STORE_ACT)))
         return -3;
     if (!paged && (p->lda % 32 != 0 || p->lda < (uint64_t)p->k_tiles * 32u)) return -3;
     if (k_parts > 1u && (p->epilogue != M40LLM_PACKED_STORE || p->batches != 1u || (k_parts - 1) * part_tiles >= p->k_tiles)) return -3;
     // packed results: whole tiles of columns
-    if ((p->epilogue == M40LLM_PACKED_GATED || p->epilogue == M40LLM_PACKED_ROTATE || (p->epilogue == M40LLM_PACKED_PROJECT && p->out_act)) &&
+    if ((p->epilogue == M40LLM_PACKED_GATED || p->epilogue == M40LLM_PACKED_ROTATE || p->epilogue == M40LLM_PACKED_SILU || (p->epilogue == M40LLM_PACKED_PROJECT && p->out_act)) &&
         (p->ld_act % 32 != 0 || p->act_col % 4 != 0))
         return -3;
     const bool wide_stores = p->ld_act % 4 == 0 && reinterpret_cast<uintptr_t>(p->out_act) % (p->act_dtype == M40LLM_ACT_F32 ? 16 : 8) == 0;
@@ -431,6 +469,9 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
             if ((p->plain_tiles > 0 && !p->out_f32) || (p->n_tiles > p->plain_tiles && (!p->out_act || !wide_stores)) ||
                 p->plain_tiles % 2 != 0 || p->n_tiles % 2 != 0 || p->plain_tiles > p->n_tiles)
                 return -4;
+            break;
+        case M40LLM_PACKED_SILU:
+            if ((p->plain_tiles > 0 && !p->out_f32) || !p->out_act || !wide_stores || p->plain_tiles > p->n_tiles || p->batches != 1u) return -4;
             break;
         case M40LLM_PACKED_KEYS: case M40LLM_PACKED_VALUES:
             if (!p->out_act || !m40_aligned16(p->out_act) || !p->pages || p->page_k_tiles < p->k_tiles || p->batches != 1u ||
@@ -452,14 +493,26 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
         batches = (int)k_parts;
     }
     (void)hipGetLastError();
+    if (p->jobs) {
+        g.jobs = p->jobs; g.gather = p->gather;
+        g.rows = (int)p->max_jobs;
+        const int rows = (int)p->job_rows;
+        if (p->act_dtype == M40LLM_ACT_F32) {
+            const M40Epilogue<float> e = make_epilogue<float>(*p);
+            return p->gather ? launch_rows_any<float, kJobGather>(stream, g, e, 1, rows) : launch_rows_any<float, kJobSlots>(stream, g, e, 1, rows);
+        }
+        const M40Epilogue<m40_bf16> e = make_epilogue<m40_bf16>(*p);
+        if (rows == 128) return p->gather ? launch_tile_any<kGather>(stream, g, e, 1, ctx->num_cus) : launch_tile_any<kSlots>(stream, g, e, 1, ctx->num_cus);
+        return p->gather ? launch_rows_any<m40_bf16, kJobGather>(stream, g, e, 1, rows) : launch_rows_any<m40_bf16, kJobSlots>(stream, g, e, 1, rows);
+    }
     if (p->act_dtype == M40LLM_ACT_F32) {
         if ((g.rows + 63) / 64 > 65535) return -3;
-        return launch_rows_any<float>(stream, g, make_epilogue<float>(*p), batches);
+        return launch_rows_any<float, kAllRows>(stream, g, make_epilogue<float>(*p), batches, g.rows);
     }
     const M40Epilogue<m40_bf16> e = make_epilogue<m40_bf16>(*p);
     if (p->epilogue == M40LLM_PACKED_KEYS) return launch_tile_any<kPageKeys>(stream, g, e, batches, ctx->num_cus);
     if (p->epilogue == M40LLM_PACKED_VALUES) return launch_tile_any<kPageValues>(stream, g, e, batches, ctx->num_cus);
-    if (g.rows <= 64) return launch_rows_any<m40_bf16>(stream, g, e, batches);
+    if (g.rows <= 64) return launch_rows_any<m40_bf16, kAllRows>(stream, g, e, batches, g.rows);
     return launch_tile_any<kPlainRows>(stream, g, e, batches, ctx->num_cus);
 }
 

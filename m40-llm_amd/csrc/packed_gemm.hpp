@@ -71,6 +71,7 @@ __device__ __forceinline__ uint32_t m40_tile_row(uint32_t b, uint32_t rows) {
     return (b | 127u) < rows ? (b & ~127u) + (b & 7u) * 16u + ((b & 127u) >> 3) : b;
 }
 __device__ __forceinline__ float m40_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float m40_silu(float z) { return z / (1.0f + expf(-z)); }
 // 0.5 z (1 + tanh(u)) = z / (1 + exp(-2 u)), u = sqrt(2 / pi) (z + 0.044715 z^3)
 __device__ __forceinline__ float m40_gelu_tanh(float z) {
     const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
@@ -90,7 +91,8 @@ struct M40Epilogue {
     long out_batch, act_batch;     // elements (packed: columns) from batch (head, part of K) to batch
     int cols;                      // columns stored (STORE, ADD, STORE_ACT, GATED)
     bool vec_out, vec_act;         // four neighbouring columns may be stored at once
-    int plain_tiles, act_col;      // PROJECT: tiles before the gate / up pairs; the first gated column of out_act
+    int plain_tiles, act_col;      // PROJECT, SILU: tiles before the activated ones; the first activated column of out_act
+    int activation;                // PROJECT
     int n_tiles;                   // KEYS, VALUES
     const float* gate;             // GATED: logits, [rows][ld_gate], one column per batch
     long ld_gate;
@@ -134,6 +136,15 @@ __device__ __forceinline__ void m40_epilogue_tile(const M40Epilogue<T>& e, int b
     const int col = tile * 16 + 4 * (lane >> 4), row = row0 + (lane & 15);
     if (row >= e.rows) return;
     switch (e.kind) {
+        case M40LLM_PACKED_SILU:
+            if (tile >= e.plain_tiles) {
+#pragma unroll
+                for (int r = 0; r < 4; ++r) v[r] = m40_silu(v[r]);
+                m40_store_packed<T>(e.out_act, row, e.act_col + col - e.plain_tiles * 16, e.ld_act, v, 4, true);
+                return;
+            }
+            m40_store_cols<float>(e.out_f32 + (long)row * e.ld_out + col, v, 4, e.vec_out);
+            return;
         case M40LLM_PACKED_STORE:
         case M40LLM_PACKED_PROJECT:
             m40_store_cols<float>(e.out_f32 + batch * e.out_batch + (long)row * e.ld_out + col, v, e.kind == M40LLM_PACKED_PROJECT ? 4 : e.cols - col,
@@ -193,7 +204,7 @@ __device__ __forceinline__ void m40_epilogue_pair(const M40Epilogue<T>& e, int r
     if (row >= e.rows) return;
     m40_float4 y;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) y[r] = m40_gelu_tanh(g[r]) * u[r];
+    for (int r = 0; r < 4; ++r) y[r] = (e.activation == M40LLM_SILU ? m40_silu(g[r]) : m40_gelu_tanh(g[r])) * u[r];
     m40_store_packed<T>(e.out_act, row, e.act_col + col, e.ld_act, y, 4, true);
 }
 #endif  // __HIPCC__

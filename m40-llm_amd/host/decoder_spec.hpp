@@ -12,6 +12,7 @@
 #include <optional>
 #include <sstream>
 #include <string>
+#include <variant>
 #include <vector>
 
 #include "json.hpp"
@@ -54,24 +55,62 @@ struct LatentAttentionSpec {
     RotationSpec rotation;
 };
 
-struct GatedMlpSpec {          // down(gelu_tanh(gate h) * (up h))
-    uint32_t ff = 0;
+// Every head two softmax maps over the same values, the second's result taken off the first's; queries, keys and values pass a causal
+// convolution of `taps` taps (0 = none) and per-map norms; a sigmoid gate per head.  kv_from >= 0: reads that layer's cache.
+struct DifferentialAttentionSpec {
+    uint32_t heads = 0, kv_heads = 0, dim = 0, vdim = 0, taps = 0;
+    float scale = 0.0f;
+    double diff = 0.0;             // added to the second map's weight; the result is scaled by one less it
+    int kv_from = -1;
 };
+
+// Linear attention whose state decays by one factor a head; norm over all heads and a sigmoid gate per column before the output product.
+struct LightningSpec {
+    uint32_t heads = 0, dim = 0, vdim = 0;
+    std::vector<double> decay;
+};
+
+typedef std::variant<LatentAttentionSpec, DifferentialAttentionSpec, LightningSpec> MixerSpec;
+
+enum class Activation { GeluTanh, Silu };
+enum class NormKind { Layer, Rms };
+
+struct GatedMlpSpec {          // down(activation(gate h) * (up h))
+    uint32_t ff = 0;
+    Activation activation = Activation::GeluTanh;
+};
+
+// Of `experts` gated feed-forwards and `identity` experts that return their input, each token takes `top` by softmax score + correction
+// and adds up their outputs times their scores.
+struct ExpertMlpSpec {
+    uint32_t experts = 0, identity = 0, top = 0, ff = 0;
+    Activation activation = Activation::Silu;
+};
+
+typedef std::variant<std::monostate, GatedMlpSpec, ExpertMlpSpec> MlpSpec;
 
 struct BigramSpec {            // a second embedding looked up by (token before, token)
     uint32_t buckets = 0, mul_prev = 0, mul_cur = 0;
 };
 
-// A layer with one layer norm whose output both sublayers read: x += mixer(norm(x)) + mlp(norm(x)).
 struct LayerSpec {
-    LatentAttentionSpec mixer;
-    std::optional<GatedMlpSpec> mlp;
+    MixerSpec mixer;
+    MlpSpec mlp;
+};
+
+enum class BlockKind {
+    Parallel,       // one norm whose output both sublayers read: x += mixer(norm(x)) + mlp(norm(x))
+    OutputNorm,     // x += m * norm1(mixer(x)), then x += m * norm2(mlp(x))
 };
 
 struct DecoderSpec {
     std::string architecture;
     uint32_t vocab = 0, width = 0;
     float eps = 0.0f;
+    NormKind norm = NormKind::Layer;
+    BlockKind block = BlockKind::Parallel;
+    float embedding_scale = 1.0f, residual_mult = 1.0f;
+    uint32_t positions = 0;        // rows of a learned position table (0 = none): the most tokens of a sequence
     std::optional<BigramSpec> bigram;
     std::vector<LayerSpec> layers;
 };
@@ -105,7 +144,7 @@ inline DecoderSpec read_pimosun(const json::Value& c) {
         if (l.str("type") != "latent_attention") throw json::Error(where + "unknown mixer '" + l.str("type") + "'");
         const json::Value& m = l.at("mixer");
         LayerSpec s;
-        LatentAttentionSpec& a = s.mixer;
+        LatentAttentionSpec a;
         a.heads = m.u32("heads"); a.dim = m.u32("dim"); a.rot_dim = m.u32("rot_dim"); a.vdim = m.u32("vdim");
         a.kv_rank = m.u32("kv_rank"); a.q_rank = m.u32("q_rank");
         a.scale = (float)m.num("scale");
@@ -115,15 +154,16 @@ inline DecoderSpec read_pimosun(const json::Value& c) {
         if (a.rotation.dims > a.rot_dim || a.rotation.dims % 2 != 0) throw json::Error(where + "rot.dims must be even and at most rot_dim");
         if (a.kv_from >= 0) {
             if ((size_t)a.kv_from >= i) throw json::Error(where + "kv_from must name an earlier layer");
-            const LatentAttentionSpec& o = d.layers[(size_t)a.kv_from].mixer;
+            const LatentAttentionSpec& o = std::get<LatentAttentionSpec>(d.layers[(size_t)a.kv_from].mixer);
             if (o.kv_from >= 0 || o.kv_rank != a.kv_rank || o.rot_dim != a.rot_dim || !(o.rotation == a.rotation))
                 throw json::Error(where + "kv_from must name a layer with entries of its own and the same kv_rank, rot_dim and rotation");
         }
         if (const json::Value* f = l.find("mlp"); f && !f->is_null()) {
             if (f->str("kind") != "dense") throw json::Error(where + "unknown feed-forward '" + f->str("kind") + "'");
-            s.mlp = GatedMlpSpec{f->u32("ff")};
-            if (s.mlp->ff == 0) throw json::Error(where + "a size is zero");
+            s.mlp = GatedMlpSpec{f->u32("ff"), Activation::GeluTanh};
+            if (f->u32("ff") == 0) throw json::Error(where + "a size is zero");
         }
+        s.mixer = a;
         d.layers.push_back(s);
     }
     if (d.vocab == 0 || d.width == 0 || d.layers.empty()) throw json::Error("vocab, width and layers must not be empty");
@@ -131,9 +171,88 @@ inline DecoderSpec read_pimosun(const json::Value& c) {
     return d;
 }
 
+inline uint32_t optional_u32(const json::Value& v, const std::string& key, uint32_t otherwise) {
+    const json::Value* f = v.find(key);
+    return f && !f->is_null() ? f->as_u32(key) : otherwise;
+}
+inline double optional_num(const json::Value& v, const std::string& key, double otherwise) {
+    const json::Value* f = v.find(key);
+    return f && !f->is_null() ? v.num(key) : otherwise;
+}
+
+inline DecoderSpec read_gulidra(const json::Value& c) {
+    DecoderSpec d;
+    d.architecture = "Gulidra";
+    d.vocab = c.u32("vocab");
+    d.width = c.u32("width");
+    d.eps = (float)c.at("norm").num("eps");
+    d.norm = NormKind::Rms;
+    d.block = BlockKind::OutputNorm;
+    d.positions = c.u32("max_positions");
+    d.residual_mult = (float)optional_num(c, "residual_mult", 1.0);
+    if (const json::Value* e = c.find("embedding"); e && !e->is_null()) d.embedding_scale = (float)optional_num(*e, "scale", 1.0);
+    const auto& layers = c.array("layers");
+    for (size_t i = 0; i < layers.size(); ++i) {
+        const json::Value& l = layers[i];
+        const std::string where = "layer " + std::to_string(i) + ": ";
+        auto check = [&](bool ok, const char* what) { if (!ok) throw json::Error(where + what); };
+        const json::Value& m = l.at("mixer");
+        LayerSpec s;
+        if (l.str("type") == "attention") {
+            DifferentialAttentionSpec a;
+            a.heads = m.u32("heads"); a.kv_heads = m.u32("kv_heads"); a.dim = m.u32("dim"); a.vdim = m.u32("vdim");
+            a.taps = optional_u32(m, "conv", 0);
+            a.scale = (float)m.num("scale");
+            a.diff = m.num("diff");
+            check(a.heads && a.kv_heads && a.dim && a.vdim, "a size is zero");
+            check(a.heads % a.kv_heads == 0, "heads must be a multiple of kv_heads");
+            if (const json::Value* j = m.find("kv_from"); j && !j->is_null()) {
+                const uint32_t from = j->as_u32("kv_from");
+                check(from < i, "kv_from must name an earlier layer");
+                const auto* o = std::get_if<DifferentialAttentionSpec>(&d.layers[from].mixer);
+                check(o && o->kv_from < 0 && o->kv_heads == a.kv_heads && o->dim == a.dim && o->vdim == a.vdim,
+                      "kv_from must name an attention layer with keys of its own and the same kv_heads, dim and vdim");
+                a.kv_from = (int)from;
+            }
+            s.mixer = a;
+        } else if (l.str("type") == "lightning") {
+            LightningSpec a;
+            a.heads = m.u32("heads"); a.dim = m.u32("dim"); a.vdim = m.u32("vdim");
+            for (const json::Value& v : m.array("decay")) {
+                check(v.kind == json::Value::Kind::Number && v.number > 0.0, "decay must be positive numbers");
+                a.decay.push_back(v.number);
+            }
+            check(a.heads && a.dim && a.vdim, "a size is zero");
+            check(a.decay.size() == a.heads, "decay must have one number a head");
+            s.mixer = a;
+        } else {
+            throw json::Error(where + "unknown mixer '" + l.str("type") + "'");
+        }
+        if (const json::Value* f = l.find("mlp"); f && !f->is_null()) {
+            if (f->str("kind") == "dense") {
+                s.mlp = GatedMlpSpec{f->u32("ff"), Activation::Silu};
+                check(f->u32("ff") != 0, "a size is zero");
+            } else if (f->str("kind") == "moe") {
+                const json::Value& r = f->at("router");
+                ExpertMlpSpec e;
+                e.experts = r.u32("experts"); e.identity = optional_u32(r, "identity", 0); e.top = r.u32("top");
+                e.ff = f->at("expert").u32("ff");
+                check(e.experts && e.top && e.ff, "a size is zero");
+                check(e.top <= e.experts + e.identity, "router.top is larger than the number of experts");
+                s.mlp = e;
+            } else {
+                throw json::Error(where + "unknown feed-forward '" + f->str("kind") + "'");
+            }
+        }
+        d.layers.push_back(s);
+    }
+    if (d.vocab == 0 || d.width == 0 || d.positions == 0 || d.layers.empty()) throw json::Error("vocab, width, max_positions and layers must not be empty");
+    return d;
+}
+
 // designs by the name config.json gives in "architecture"
 inline const std::map<std::string, std::function<DecoderSpec(const json::Value&)>>& decoder_registry() {
-    static const std::map<std::string, std::function<DecoderSpec(const json::Value&)>> r = {{"Pimosun", read_pimosun}};
+    static const std::map<std::string, std::function<DecoderSpec(const json::Value&)>> r = {{"Pimosun", read_pimosun}, {"Gulidra", read_gulidra}};
     return r;
 }
 inline DecoderSpec read_decoder_spec(const std::string& config_text) {

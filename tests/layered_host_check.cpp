@@ -27,15 +27,30 @@ static void spec(std::istream& in) {
     const DecoderSpec d = read_decoder_spec(read_text_file(path));
     std::cout.precision(17);
     std::cout << "{\"architecture\": " << quoted(d.architecture) << ", \"vocab\": " << d.vocab << ", \"width\": " << d.width << ", \"eps\": " << d.eps
-              << ", \"bigram\": " << (d.bigram ? (int64_t)d.bigram->buckets : -1) << ", \"layers\": [";
+              << ", \"bigram\": " << (d.bigram ? (int64_t)d.bigram->buckets : -1) << ", \"embedding_scale\": " << d.embedding_scale << ", \"residual_mult\": " << d.residual_mult << ", \"positions\": " << d.positions << ", \"layers\": [";
     for (size_t i = 0; i < d.layers.size(); ++i) {
-        const LatentAttentionSpec& a = d.layers[i].mixer;
-        std::cout << (i ? ", " : "") << "{\"sizes\": [" << a.heads << ", " << a.dim << ", " << a.rot_dim << ", " << a.vdim << ", " << a.kv_rank << ", " << a.q_rank
-                  << "], \"scale\": " << a.scale << ", \"kv_from\": " << a.kv_from << ", \"ff\": " << (d.layers[i].mlp ? d.layers[i].mlp->ff : 0)
-                  << ", \"magnitude\": " << a.rotation.magnitude() << ", \"freq\": [";
-        const std::vector<double> f = a.rotation.frequencies();
-        for (size_t k = 0; k < f.size(); ++k) std::cout << (k ? ", " : "") << f[k];
-        std::cout << "]}";
+        std::cout << (i ? ", " : "");
+        const LayerSpec& l = d.layers[i];
+        if (const auto* a = std::get_if<LatentAttentionSpec>(&l.mixer)) {
+            std::cout << "{\"sizes\": [" << a->heads << ", " << a->dim << ", " << a->rot_dim << ", " << a->vdim << ", " << a->kv_rank << ", " << a->q_rank
+                      << "], \"scale\": " << a->scale << ", \"kv_from\": " << a->kv_from << ", \"magnitude\": " << a->rotation.magnitude() << ", \"freq\": [";
+            const std::vector<double> f = a->rotation.frequencies();
+            for (size_t k = 0; k < f.size(); ++k) std::cout << (k ? ", " : "") << f[k];
+            std::cout << "]";
+        } else if (const auto* a = std::get_if<DifferentialAttentionSpec>(&l.mixer)) {
+            std::cout << "{\"sizes\": [" << a->heads << ", " << a->kv_heads << ", " << a->dim << ", " << a->vdim << ", " << a->taps << "], \"scale\": " << a->scale
+                      << ", \"diff\": " << a->diff << ", \"kv_from\": " << a->kv_from;
+        } else {
+            const LightningSpec& n = std::get<LightningSpec>(l.mixer);
+            std::cout << "{\"sizes\": [" << n.heads << ", " << n.dim << ", " << n.vdim << "], \"decay\": [";
+            for (size_t k = 0; k < n.decay.size(); ++k) std::cout << (k ? ", " : "") << n.decay[k];
+            std::cout << "]";
+        }
+        const auto* g = std::get_if<GatedMlpSpec>(&l.mlp);
+        std::cout << ", \"ff\": " << (g ? g->ff : 0) << ", \"silu\": " << (g && g->activation == Activation::Silu ? "true" : "false");
+        if (const auto* e = std::get_if<ExpertMlpSpec>(&l.mlp))
+            std::cout << ", \"experts\": [" << e->experts << ", " << e->identity << ", " << e->top << ", " << e->ff << "]";
+        std::cout << "}";
     }
     std::cout << "]}\n";
 }
