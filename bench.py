@@ -361,10 +361,10 @@ def main():
     ap.add_argument("--traffic-probe", action="store_true",
                     help="also run one 256 MiB device-to-device copy through the library (calibrates rocprofv3 --pmc "
                          "FETCH_SIZE / WRITE_SIZE readings against a transfer of known size)")
-    ap.add_argument("--design", choices=["pimosun"], help="instead of the default workload: prefill and decode throughput of this "
-                    "design beside the dense decoder of equal size (m40-llm_amd/layered_bench.py)")
+    ap.add_argument("--design", choices=["pimosun", "gulidra"], help="instead of the default workload: prefill and decode throughput of "
+                    "this design beside the closest other model of equal size (m40-llm_amd/layered_bench.py)")
     ap.add_argument("--shapes", default="", help="with --design: the shapes to run, with commas between them")
-    ap.add_argument("--no-dense", action="store_true", help="with --design: leave the dense decoder out")
+    ap.add_argument("--no-dense", action="store_true", help="with --design pimosun: leave the dense decoder out")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py measures one GPU: this path has no multi-GPU form (each box has one MI355X); run with --gpus 1",
@@ -380,9 +380,10 @@ def main():
     if args.design:
         lb = importlib.import_module("m40-llm_amd.layered_bench")
         shapes = [x for x in args.shapes.split(",") if x] or None
-        print(json.dumps({"metric": "prefill and decode throughput, Pimosun beside the dense decoder of equal size", "unit": "tok/s",
+        print(json.dumps({"metric": "prefill and decode throughput, %s of equal size" % lb.BESIDE[args.design], "unit": "tok/s",
                           "n_gpus": 1, "dtype": "bf16", "data": "synthetic",
-                          "shapes": lb.measure(pkg.Context(0), shapes, steps=min(args.steps, 32), warmup=4, dense=not args.no_dense)}))
+                          "shapes": lb.measure(pkg.Context(0), shapes, steps=min(args.steps, 32), warmup=4, dense=not args.no_dense,
+                                               design=args.design)}))
         return
 
     cfg = dict(syn.TINYLLAMA_1B)

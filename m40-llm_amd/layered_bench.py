@@ -1,5 +1,6 @@
-"""Prefill and decode throughput of a layered decoder (the Pimosun design, random weights) beside the dense decoder of the same
-width, depth, feed-forward and vocabulary.  `bench.py --design pimosun` prints what measure() returns.
+"""Prefill and decode throughput of layered decoders with random weights beside the framework's closest other model of the same width,
+depth and vocabulary.  `bench.py --design NAME` prints what measure() returns: the Pimosun design beside the dense decoder, the Gulidra
+design beside Pimosun, whose feed-forward is as wide as the experts a token takes together.
 
 A case is one shape on one kind of step: a prompt of n tokens run in one step (host clock around the blocking call, the last
 token's logits included), or `batch` sequences of `context` tokens that decode greedily from a replayed graph (timed between
@@ -15,6 +16,7 @@ pkg = importlib.import_module(__package__)
 syn = importlib.import_module(__package__ + ".synthetic")
 layered = importlib.import_module(__package__ + ".layered")
 
+BESIDE = dict(pimosun="Pimosun beside the dense decoder", gulidra="Gulidra beside Pimosun")
 SHAPES = {
     # name: layered decoder, and the dense decoder's heads at the same width
     "2k": dict(width=2048, heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=768, ff=5632, vocab=32000, layers=8, kv_heads=2),
@@ -35,6 +37,32 @@ def pimosun_config(s: dict) -> dict:
                 embedding=dict(bigram=dict(buckets=20011, mul_prev=31, mul_cur=7)), layers=layers)
 
 
+# Gulidra at Pimosun's sizes: half of the layers routed, one in four a lightning layer, the second half of the attention layers reading the first
+# half's keys; a token's experts together are as wide as the dense feed-forward
+GULIDRA = {
+    "2k": dict(kv_heads=4, dim=64, conv=4, experts=32, identity=2, top=4, expert_ff=1408, light=(16, 128, 128)),
+    "4k": dict(kv_heads=8, dim=64, conv=4, experts=32, identity=2, top=4, expert_ff=2752, light=(32, 128, 128)),
+}
+
+
+def gulidra_config(name: str) -> dict:
+    s, g = SHAPES[name], GULIDRA[name]
+    mixer = dict(heads=s["heads"], kv_heads=g["kv_heads"], dim=g["dim"], vdim=s["vdim"], conv=g["conv"], diff=0.3, scale=float(g["dim"] ** -0.5))
+    heads, dim, vdim = g["light"]
+    light = dict(heads=heads, dim=dim, vdim=vdim, decay=[float(1 - 2.0 ** -(2 + 8 * i / heads)) for i in range(heads)])
+    moe = dict(kind="moe", expert=dict(ff=g["expert_ff"]), router=dict(experts=g["experts"], identity=g["identity"], top=g["top"]))
+    dense = dict(kind="dense", ff=s["ff"])
+    layers = []
+    for i in range(s["layers"]):
+        mlp = moe if i % 2 else dense
+        if i % 4 == 3:
+            layers.append(dict(type="lightning", mixer=light, mlp=mlp))
+        else:
+            layers.append(dict(type="attention", mixer=dict(mixer, **({"kv_from": i - 2} if i % 4 == 2 else {})), mlp=mlp))
+    return dict(architecture="Gulidra", vocab=s["vocab"], width=s["width"], norm=dict(eps=1e-5), embedding=dict(scale=1.0), residual_mult=0.7,
+                max_positions=8192, layers=layers)
+
+
 def layer_flops_per_token(s: dict, own: bool) -> float:
     """Matrix-product flops of one layer and token outside attention's own products (keys and values from the latent included)."""
     w, h = s["width"], s["heads"]
@@ -42,9 +70,9 @@ def layer_flops_per_token(s: dict, own: bool) -> float:
     return 2.0 * (n + (w * (s["kv_rank"] + s["rot_dim"]) if own else 0))
 
 
-def layered_cases(ctx, s, prefill=PREFILL, decode=DECODE, reps=3, steps=32, warmup=4):
+def layered_cases(ctx, s, prefill=PREFILL, decode=DECODE, reps=3, steps=32, warmup=4, cfg=None):
     out = {}
-    cfg = pimosun_config(s)
+    cfg = cfg or pimosun_config(s)
     rng = np.random.default_rng(0)
     slots = max([b for b, _ in decode] + [1])
     tokens = max([b * (c + steps + warmup + 64) for b, c in decode] + [n + 64 for n in prefill])
@@ -111,8 +139,14 @@ def dense_cases(ctx, s, prefill=PREFILL, decode=DECODE, reps=3, steps=32, warmup
     return out
 
 
-def measure(ctx, shapes=None, steps=32, warmup=4, dense=True) -> dict:
+def measure(ctx, shapes=None, steps=32, warmup=4, dense=True, design="pimosun") -> dict:
     out = {}
+    if design == "gulidra":
+        for name in shapes or SHAPES:
+            s = SHAPES[name]
+            out[name] = {"shape": dict(s, **GULIDRA[name]), "gulidra": layered_cases(ctx, s, steps=steps, warmup=warmup, cfg=gulidra_config(name)),
+                         "pimosun": layered_cases(ctx, s, steps=steps, warmup=warmup)}
+        return out
     for name in shapes or SHAPES:
         s = SHAPES[name]
         out[name] = {"shape": {k: v for k, v in s.items() if k != "kv_heads"}, "pimosun": layered_cases(ctx, s, steps=steps, warmup=warmup)}
