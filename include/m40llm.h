@@ -694,15 +694,15 @@ uint64_t m40llm_ext_pair_page_elements(uint32_t kv_heads, uint32_t dim, uint32_t
  * on every column (0 = none), RMS norm over each map's dim of queries and keys; queries out as plain rows [heads][2][32*k_tiles], keys and
  * values to the row's place in the cache (cache NULL = the layer reads another layer's: no key and value columns).
  * row_back[row]: rows of the same portion before it, bit 31 set where the portion is one row.  conv_state [slot][taps - 1][ld_state]
- * holds the columns of the rows before a portion, oldest first (rows before position 0 count as zero); portions of one row update it,
- * the others by m40llm_ext_conv_state_async afterwards. */
+ * holds the columns of the rows before a portion, that of position p at entry p % (taps - 1) (rows before position 0 count as zero);
+ * portions of one row update it, the others by m40llm_ext_conv_state_async afterwards. */
 typedef struct M40llmPairSplit {
     uint32_t act_dtype, rows, heads, kv_heads, dim, vdim, taps;
     float eps;
     const void* proj;
     uint64_t ld_proj;
     uint32_t k_offset, v_offset;            /* columns; queries start at 0 */
-    const void *q_conv, *k_conv, *v_conv;   /* f32 [columns][taps] */
+    const void *q_conv, *k_conv, *v_conv;   /* f32 [taps][columns], the newest row's last */
     const void *q_norm, *k_norm;            /* f32 [dim] */
     void* conv_state;
     uint64_t ld_state;
@@ -712,9 +712,10 @@ typedef struct M40llmPairSplit {
     uint32_t max_pages;
 } M40llmPairSplit;
 int m40llm_ext_pair_split_append_async(M40llmCudaContext* ctx, const M40llmPairSplit* s, uint32_t stream_kind);
-/* portions[p] = {first row, rows, slot, first position}: those of two rows and more leave the last taps - 1 of their columns in conv_state */
+/* portions[p] = {first row, rows, slot, 0}: those of two rows and more leave the last taps - 1 of their columns in conv_state */
 int m40llm_ext_conv_state_async(M40llmCudaContext* ctx, const void* d_proj, uint64_t ld_proj, uint32_t cols, uint32_t taps, void* d_conv_state,
-                                uint64_t ld_state, const uint32_t* d_portions, uint32_t n_portions, uint32_t stream_kind);
+                                uint64_t ld_state, const uint32_t* d_portions, const uint32_t* d_row_pos, uint32_t n_portions,
+                                uint32_t stream_kind);
 /* Query i of a kv head = row * (heads / kv_heads) + head within the group.  tiles[t] = {first query, queries}, all of one slot.
  * form 0: at most 16 queries a tile, pages divided over waves and over `splits` workgroups (partial:
  * m40llm_ext_pair_attention_partial_floats; rows first_row .. first_row + n_rows are joined by a second launch); form 1: at most tile_queries
@@ -743,7 +744,7 @@ uint32_t m40llm_ext_pair_attention_tile_queries(uint32_t act_dtype, uint32_t dim
 /* ---- lightning attention -----------------------------------------------------------------------------------------------------------
  * Per head S <- decay*S + k v^T, o = S^T q, token by token; S in f32, state[slot][head][dim][32*ceil(vdim/32)], zero before position 0.
  * qkv: packed rows of the activation type, columns: heads x 32*ceil(dim/32) queries, the same of keys, heads x 32*ceil(vdim/32) values.
- * o: f32 [rows][heads*vdim].  portions[p] = {first row, rows, slot, first position}.
+ * o: f32 [rows][heads*vdim].  portions[p] = {first row, rows, slot, 0}.
  * serial: token after token (any type); chunked (bf16): over the 64-row groups of the pass that a portion touches.  chunk_base[p] = chunks
  * of the portions before it; chunks[c] = {portion, first row of the group}; scratch: m40llm_ext_lightning_scratch_bytes. */
 typedef struct M40llmLightning {

@@ -5,104 +5,135 @@
 namespace {
 
 constexpr uint32_t kThreads = 256, kWaves = kThreads / 64;
-constexpr uint32_t kMost = M40LLM_MAX_EXPERTS, kPerLane = kMost / 64;
+constexpr uint32_t kListThreads = 1024, kListWaves = kListThreads / 64;
+constexpr uint32_t kMost = M40LLM_MAX_EXPERTS;
 constexpr uint32_t kSmallPairs = 4096;     // (row, choice) pairs one workgroup keeps in LDS
 
-// A wave routes one row: lane l holds experts l, l + 64, ...
+// A wave routes one row: lane l holds experts l, l + 64, ..., N of them.
+template <uint32_t N>
 __device__ __forceinline__ void route_row(const M40llmRoute& a, uint32_t row, uint32_t lane, uint32_t* ids, float* weight) {
     const uint32_t n = a.experts + a.identity;
     const float* z = static_cast<const float*>(a.logits) + (size_t)row * a.ld_logits;
     const float* correction = static_cast<const float*>(a.correction);
-    float s[kPerLane], choice[kPerLane];
+    float s[N], choice[N];
     float top = -INFINITY;
 #pragma unroll
-    for (uint32_t i = 0; i < kPerLane; ++i) {
+    for (uint32_t i = 0; i < N; ++i) {
         const uint32_t e = lane + 64u * i;
         s[i] = e < n ? z[e] : -INFINITY;
+        choice[i] = e < n ? correction[e] : 0.0f;
         top = fmaxf(top, s[i]);
     }
     top = m40_max64(top);
     float sum = 0.0f;
 #pragma unroll
-    for (uint32_t i = 0; i < kPerLane; ++i) {
+    for (uint32_t i = 0; i < N; ++i) {
         s[i] = lane + 64u * i < n ? expf(s[i] - top) : 0.0f;
         sum += s[i];
     }
     sum = m40_sum64(sum);
+    uint32_t left = 0;                       // bit i: this lane's expert i can be chosen
 #pragma unroll
-    for (uint32_t i = 0; i < kPerLane; ++i) {
+    for (uint32_t i = 0; i < N; ++i) {
         const uint32_t e = lane + 64u * i;
         s[i] /= sum;
-        choice[i] = e < n ? s[i] + correction[e] : -INFINITY;
+        choice[i] += s[i];
+        if (e < n) left |= 1u << i;
     }
-    uint32_t taken = 0;                      // bit i: this lane's expert i is chosen
+    uint32_t mine_id = 0;
+    float mine_weight = 0.0f;                // choice `lane`
     for (uint32_t j = 0; j < a.top; ++j) {
         float best = -INFINITY;
-        uint32_t at = 0xffffffffu;
 #pragma unroll
-        for (uint32_t i = 0; i < kPerLane; ++i) {
-            const uint32_t e = lane + 64u * i;
-            if (e < n && !(taken >> i & 1u) && (at == 0xffffffffu || choice[i] > best)) {
-                best = choice[i];
-                at = e;
-            }
-        }
-#pragma unroll
-        for (int d = 1; d < 64; d *= 2) {
-            const float other = __shfl_xor(best, d);
-            const uint32_t where = (uint32_t)__shfl_xor((int)at, d);
-            const bool take = where != 0xffffffffu && (at == 0xffffffffu || other > best || (other == best && where < at));
-            best = take ? other : best;
-            at = take ? where : at;
-        }
+        for (uint32_t i = 0; i < N; ++i) best = left >> i & 1u ? fmaxf(best, choice[i]) : best;
+        best = m40_max64(best);
+        uint32_t at = 0;
         float w = 0.0f;
+        bool found = false;                  // the lowest index of equals: i before lane
 #pragma unroll
-        for (uint32_t i = 0; i < kPerLane; ++i)
-            if (lane + 64u * i == at) {
-                taken |= 1u << i;
-                w = s[i];
+        for (uint32_t i = 0; i < N; ++i) {
+            const unsigned long long hit = __ballot((left >> i & 1u) && choice[i] == best);
+            if (!found && hit) {
+                const uint32_t l = (uint32_t)__ffsll(hit) - 1u;
+                at = l + 64u * i;
+                w = __shfl(s[i], (int)l);
+                if (lane == l) left &= ~(1u << i);
+                found = true;
             }
-        if (at % 64u == lane) {
-            ids[j] = at;
-            weight[j] = w;
+        }
+        if (!found) {                        // nothing comparable is left (not a number): the lowest index that can be chosen
+#pragma unroll
+            for (uint32_t i = 0; i < N; ++i) {
+                const unsigned long long hit = __ballot(left >> i & 1u);
+                if (!found && hit) {
+                    const uint32_t l = (uint32_t)__ffsll(hit) - 1u;
+                    at = l + 64u * i;
+                    w = __shfl(s[i], (int)l);
+                    if (lane == l) left &= ~(1u << i);
+                    found = true;
+                }
+            }
+        }
+        if (lane == (j & 63u)) { mine_id = at; mine_weight = w; }
+        if ((j & 63u) == 63u || j + 1u == a.top) {
+            const uint32_t first = j & ~63u;
+            if (first + lane <= j) {
+                ids[first + lane] = mine_id;
+                weight[first + lane] = mine_weight;
+            }
         }
     }
 }
 
+template <uint32_t N>
 __global__ __launch_bounds__(kThreads) void route_rows_kernel(M40llmRoute a) {
     const uint32_t row = blockIdx.x * kWaves + (threadIdx.x >> 6);
     if (row >= a.rows) return;
-    route_row(a, row, threadIdx.x & 63u, a.ids + (size_t)row * a.top, static_cast<float*>(a.weight) + (size_t)row * a.top);
+    route_row<N>(a, row, threadIdx.x & 63u, a.ids + (size_t)row * a.top, static_cast<float*>(a.weight) + (size_t)row * a.top);
 }
 
-// A workgroup an expert.  SMALL: it first routes all rows itself (one launch for a step of few rows).
-template <bool SMALL>
-__global__ __launch_bounds__(kThreads) void expert_lists_kernel(M40llmRoute a) {
+// A workgroup an expert.  N > 0: it first routes all rows itself (one launch for a step of few rows).
+template <uint32_t N>
+__global__ __launch_bounds__(kListThreads) void expert_lists_kernel(M40llmRoute a) {
+    constexpr bool SMALL = N > 0;
     __shared__ uint32_t count[kMost];
-    __shared__ uint32_t own_ids[SMALL ? kSmallPairs : 1];
+    __shared__ __align__(16) uint32_t own_ids[SMALL ? kSmallPairs : 4];
     __shared__ float own_weight[SMALL ? kSmallPairs : 1];
-    __shared__ uint32_t wave_n[kWaves], wave_slots[kWaves], wave_jobs[kWaves], wave_all[kWaves];
+    __shared__ uint32_t wave_n[2][kListWaves], wave_slots[kListWaves], wave_jobs[kListWaves], wave_all[kListWaves];
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, mine = blockIdx.x, pairs = a.rows * a.top, E = a.experts;
-    for (uint32_t e = tid; e < E; e += kThreads) count[e] = 0u;
-    if (SMALL)
-        for (uint32_t row = wave; row < a.rows; row += kWaves) route_row(a, row, lane, own_ids + row * a.top, own_weight + row * a.top);
+    for (uint32_t e = tid; e < E; e += kListThreads) count[e] = 0u;
+    if constexpr (SMALL)
+        for (uint32_t row = wave; row < a.rows; row += kListWaves) route_row<N>(a, row, lane, own_ids + row * a.top, own_weight + row * a.top);
     __syncthreads();
     const uint32_t* ids = SMALL ? own_ids : a.ids;
-    for (uint32_t p = tid; p < pairs; p += kThreads) {
-        const uint32_t e = ids[p];
-        if (e < E) atomicAdd(&count[e], 1u);
-        if (mine == 0u) {
-            if (e >= E) a.place[p] = M40LLM_PLACE_INPUT;
-            if (SMALL) {
-                a.ids[p] = e;
-                static_cast<float*>(a.weight)[p] = own_weight[p];
+    auto load4 = [&](uint32_t p, uint32_t (&e)[4]) __attribute__((always_inline)) {
+        if (p + 4u <= pairs) {
+            const uint4 v = *reinterpret_cast<const uint4*>(ids + p);
+            e[0] = v.x; e[1] = v.y; e[2] = v.z; e[3] = v.w;
+        } else {
+#pragma unroll
+            for (uint32_t i = 0; i < 4u; ++i) e[i] = p + i < pairs ? ids[p + i] : 0xffffffffu;
+        }
+    };
+    for (uint32_t p = tid * 4u; p < pairs; p += kListThreads * 4u) {
+        uint32_t e[4];
+        load4(p, e);
+#pragma unroll
+        for (uint32_t i = 0; i < 4u; ++i) {
+            if (e[i] < E) atomicAdd(&count[e[i]], 1u);
+            if (mine == 0u && p + i < pairs) {
+                if (e[i] >= E) a.place[p + i] = M40LLM_PLACE_INPUT;
+                if (SMALL) {
+                    a.ids[p + i] = e[i];
+                    static_cast<float*>(a.weight)[p + i] = own_weight[p + i];
+                }
             }
         }
     }
     __syncthreads();
     // slots and jobs of the experts before this one, and all jobs
     uint32_t slots = 0, jobs = 0, all = 0;
-    for (uint32_t e = tid; e < E; e += kThreads) {
+    for (uint32_t e = tid; e < E; e += kListThreads) {
         const uint32_t c = count[e], j = (c + a.job_rows - 1u) / a.job_rows;
         all += j;
         if (e < mine) {
@@ -120,10 +151,10 @@ __global__ __launch_bounds__(kThreads) void expert_lists_kernel(M40llmRoute a) {
     __syncthreads();
     slots = jobs = all = 0u;
 #pragma unroll
-    for (uint32_t w = 0; w < kWaves; ++w) { slots += wave_slots[w]; jobs += wave_jobs[w]; all += wave_all[w]; }
+    for (uint32_t w = 0; w < kListWaves; ++w) { slots += wave_slots[w]; jobs += wave_jobs[w]; all += wave_all[w]; }
     if (mine == 0u && tid == 0u) a.jobs[0] = all;
     const uint32_t n = count[mine];
-    for (uint32_t j = tid; j * a.job_rows < n; j += kThreads) {
+    for (uint32_t j = tid; j * a.job_rows < n; j += kListThreads) {
         uint32_t* job = a.jobs + 4u + 4u * (jobs + j);
         const uint32_t left = n - j * a.job_rows;
         job[0] = mine;
@@ -132,28 +163,47 @@ __global__ __launch_bounds__(kThreads) void expert_lists_kernel(M40llmRoute a) {
         job[3] = 0u;
     }
     if (n == 0u) return;
-    // its rows in order
-    uint32_t found = 0;
-    for (uint32_t p0 = 0; p0 < pairs; p0 += kThreads) {
-        const uint32_t p = p0 + tid;
-        const bool hit = p < pairs && ids[p] == mine;
-        const unsigned long long mask = __ballot(hit);
-        if (lane == 0u) wave_n[wave] = (uint32_t)__popcll(mask);
-        __syncthreads();
-        uint32_t before = found;
+    // its rows in order: four pairs a thread at a time
+    uint32_t found = 0, phase = 0;
+    for (uint32_t p0 = 0; p0 < pairs; p0 += kListThreads * 4u, phase ^= 1u) {
+        const uint32_t p = p0 + tid * 4u;
+        uint32_t e[4];
+        load4(p, e);
+        uint32_t before = 0, total = 0;      // hits of lower lanes, of the wave
 #pragma unroll
-        for (uint32_t w = 0; w < kWaves; ++w) {
-            if (w < wave) before += wave_n[w];
-            found += wave_n[w];
+        for (uint32_t i = 0; i < 4u; ++i) {
+            const unsigned long long mask = __ballot(e[i] == mine);
+            before += (uint32_t)__popcll(mask & ((1ull << lane) - 1ull));
+            total += (uint32_t)__popcll(mask);
         }
-        if (hit) {
-            const uint32_t slot = slots + before + (uint32_t)__popcll(mask & ((1ull << lane) - 1ull));
-            a.rows_of[slot] = p / a.top;
-            a.place[p] = slot;
-        }
+        if (lane == 0u) wave_n[phase][wave] = total;
         __syncthreads();
+        before += found;
+#pragma unroll
+        for (uint32_t w = 0; w < kListWaves; ++w) {
+            const uint32_t k = wave_n[phase][w];
+            if (w < wave) before += k;
+            found += k;
+        }
+#pragma unroll
+        for (uint32_t i = 0; i < 4u; ++i)
+            if (e[i] == mine) {
+                const uint32_t slot = slots + before++;
+                a.rows_of[slot] = (p + i) / a.top;
+                a.place[p + i] = slot;
+            }
     }
     if (tid < ((n + 15u) & ~15u) - n) a.rows_of[slots + n + tid] = 0u;
+}
+
+template <uint32_t N>
+void launch_route(hipStream_t stream, const M40llmRoute& r) {
+    if (r.rows <= 64u && r.rows * r.top <= kSmallPairs) {
+        expert_lists_kernel<N><<<r.experts, kListThreads, 0, stream>>>(r);
+    } else {
+        route_rows_kernel<N><<<(r.rows + kWaves - 1u) / kWaves, kThreads, 0, stream>>>(r);
+        expert_lists_kernel<0><<<r.experts, kListThreads, 0, stream>>>(r);
+    }
 }
 
 }  // namespace
@@ -178,15 +228,14 @@ int m40llm_ext_route_rows_async(M40llmCudaContext* ctx, const M40llmRoute* r, ui
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
     if (r->rows == 0 || r->experts == 0 || r->experts + r->identity > kMost || r->top == 0 || r->top > r->experts + r->identity ||
         r->ld_logits < r->experts + r->identity || (r->job_rows != 16u && r->job_rows != 32u && r->job_rows != 64u && r->job_rows != 128u) ||
-        m40llm_ext_expert_slots(r->rows, r->experts, r->top) == 0 || m40llm_ext_expert_max_jobs(r->rows, r->experts, r->top, r->job_rows) == 0)
+        !m40_aligned16(r->ids) || m40llm_ext_expert_slots(r->rows, r->experts, r->top) == 0 || m40llm_ext_expert_max_jobs(r->rows, r->experts, r->top, r->job_rows) == 0)
         return -3;
     (void)hipGetLastError();
-    if (r->rows <= 64u && r->rows * r->top <= kSmallPairs) {
-        expert_lists_kernel<true><<<r->experts, kThreads, 0, stream>>>(*r);
-    } else {
-        route_rows_kernel<<<(r->rows + kWaves - 1u) / kWaves, kThreads, 0, stream>>>(*r);
-        expert_lists_kernel<false><<<r->experts, kThreads, 0, stream>>>(*r);
-    }
+    const uint32_t all = r->experts + r->identity;
+    if (all <= 64u) launch_route<1>(stream, *r);
+    else if (all <= 128u) launch_route<2>(stream, *r);
+    else if (all <= 256u) launch_route<4>(stream, *r);
+    else launch_route<16>(stream, *r);
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
 

@@ -141,10 +141,21 @@ __global__ __launch_bounds__(256) void lightning_states_kernel(LightArgs a) {
     m40_bf16* out = static_cast<m40_bf16*>(a.l.scratch) + ((size_t)a.l.chunk_base[blockIdx.x] * a.l.heads + head) * dt * vt * 4u * kM40Tile +
                     ((size_t)d32 * vt * 2u + v16) * 2u * kM40Tile + lane * 8;
     const size_t out_step = (size_t)a.l.heads * dt * vt * 4u * kM40Tile;
+    float whole[2][8];                                                 // decay to the end of a whole chunk
+#pragma unroll
+    for (int h = 0; h < 2; ++h)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) whole[h][i] = decay_power(log2_decay, kChunk - 1 - (32 * h + 8 * g + i));
+    const float whole_chunk = decay_power(log2_decay, kChunk);
     int buf = 0;
     for (uint32_t c = 0; c < chunks; ++c) {
-        m40_wait_and_meet<3 * (kBufs - 2)>();                          // chunk c has landed; nobody reads the buffer before it any more
+        // Chunk c has landed, and nobody reads the buffer before it any more.  Behind its three loads a wave has issued those of the two chunks
+        // after it and, once the walk is under way, the two stores of each of three chunks.
+        if (wave_live && c >= 3u) m40_wait_and_meet<3 * (kBufs - 2) + 6>();
+        else m40_wait_and_meet<3 * (kBufs - 2)>();
         issue(buf == 0 ? kBufs - 1 : buf - 1, c + kBufs - 1);
+        asm volatile("" ::: "memory");                                 // the stores stay behind these loads: they are counted
+        __builtin_amdgcn_sched_barrier(0);
         float s8[8];
 #pragma unroll
         for (int i = 0; i < 8; ++i) s8[i] = S[i >> 2][i & 3];
@@ -154,7 +165,8 @@ __global__ __launch_bounds__(256) void lightning_states_kernel(LightArgs a) {
             *reinterpret_cast<m40_bf16x8*>(out + c * out_step + kM40Tile) = sp.lo;
         }
         const int base = (int)((first + c) * kChunk), lo = (int)row0 > base ? (int)row0 - base : 0, end = (int)(row0 + n) - base, hi = end < kChunk ? end : kChunk;
-        const float f = decay_power(log2_decay, hi - lo);
+        const bool all = lo == 0 && hi == kChunk;
+        const float f = all ? whole_chunk : decay_power(log2_decay, hi - lo);
         S[0] *= f;
         S[1] *= f;
         const uint8_t* tiles = lds + buf * kTiles * 1024;
@@ -165,10 +177,15 @@ __global__ __launch_bounds__(256) void lightning_states_kernel(LightArgs a) {
             const uint32_t at = column_address(li, tok, (int)(v16 & 1u)), half = ((v16 >> 1) & 1u) * 1024u;
             const m40_bf16x8 vf = read_columns(tile + 1024 + half + at, tile + 1024 + half + at + 4 * 16);
             float w[8];
+            if (all) {
 #pragma unroll
-            for (int i = 0; i < 8; ++i) {
-                const int j = 32 * h + 8 * g + i;
-                w[i] = j >= lo && j < hi ? static_cast<float>(vf[i]) * decay_power(log2_decay, hi - 1 - j) : 0.0f;
+                for (int i = 0; i < 8; ++i) w[i] = static_cast<float>(vf[i]) * whole[h][i];
+            } else {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) {
+                    const int j = 32 * h + 8 * g + i;
+                    w[i] = j >= lo && j < hi ? static_cast<float>(vf[i]) * decay_power(log2_decay, hi - 1 - j) : 0.0f;
+                }
             }
             const Parts vp = two_parts(w);
 #pragma unroll

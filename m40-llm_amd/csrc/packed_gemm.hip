@@ -512,7 +512,8 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
     const M40Epilogue<m40_bf16> e = make_epilogue<m40_bf16>(*p);
     if (p->epilogue == M40LLM_PACKED_KEYS) return launch_tile_any<kPageKeys>(stream, g, e, batches, ctx->num_cus);
     if (p->epilogue == M40LLM_PACKED_VALUES) return launch_tile_any<kPageValues>(stream, g, e, batches, ctx->num_cus);
-    if (g.rows <= 64) return launch_rows_any<m40_bf16, kAllRows>(stream, g, e, batches, g.rows);
+    // few columns leave most CUs without a wide tile
+    if (g.rows <= 64 || (g.n_tiles <= 8 && batches == 1 && g.rows <= 65535 * 16 && p->epilogue != M40LLM_PACKED_PROJECT)) return launch_rows_any<m40_bf16, kAllRows>(stream, g, e, batches, g.rows);
     return launch_tile_any<kPlainRows>(stream, g, e, batches, ctx->num_cus);
 }
 

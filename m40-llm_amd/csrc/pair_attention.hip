@@ -8,7 +8,8 @@
 //
 // pair_rows_kernel   up to 16 queries: every wave takes whole pages straight from memory into operand registers; the waves' sums, and
 //                    those of the workgroups that share a sequence's pages (pair_join_kernel), meet at the end
-// pair_tile_kernel   64 or 128 queries, a wave 16 or 32 of them: pages go through LDS, one ahead
+// pair_tile_kernel   64 or 128 queries, a wave 16 or 32 of them: pages go through LDS, one ahead.  With two groups of four waves the even and
+//                    the odd pages are walked side by side and the groups' sums meet at the end, which halves the longest walk
 // pair_f32_kernel    one workgroup a row and head, plain f32 arithmetic
 //
 // Maxima are reference points that move only when some score lies 8 (as a power of two) above them.
@@ -55,18 +56,20 @@ struct PairState {
     }
     // the scores of a map become weights: operands of the value product
     __device__ __forceinline__ void weigh(int m, m40_float4 (&s)[4][B], float c, bool whole, uint32_t key0, m40_bf16x8 (&pf)[B][2]) {
+        if (!whole) {
+#pragma unroll
+            for (int b = 0; b < B; ++b)
+#pragma unroll
+                for (int t = 0; t < 4; ++t)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) s[t][b][r] = key0 + t * 16 + r <= pos[b] ? s[t][b][r] : -INFINITY;
+        }
 #pragma unroll
         for (int b = 0; b < B; ++b) {
-            float top = -INFINITY;
+            float top = fmaxf(fmaxf(s[0][b][0], s[0][b][1]), fmaxf(s[0][b][2], s[0][b][3]));
 #pragma unroll
-            for (int t = 0; t < 4; ++t)
-#pragma unroll
-                for (int r = 0; r < 4; ++r) {
-                    float x = s[t][b][r] * c;
-                    if (!whole) x = key0 + t * 16 + r <= pos[b] ? x : -INFINITY;
-                    s[t][b][r] = x;
-                    top = fmaxf(top, x);
-                }
+            for (int t = 1; t < 4; ++t) top = fmaxf(top, fmaxf(fmaxf(s[t][b][0], s[t][b][1]), fmaxf(s[t][b][2], s[t][b][3])));
+            top *= c;
             if (__any(top > ref[m][b] + 8.0f)) {
                 top = m40_max_xor16(top);
                 top = m40_max_xor32(top);
@@ -76,14 +79,17 @@ struct PairState {
 #pragma unroll
                 for (int j = 0; j < DVT; ++j) o[m][j][b] *= f;
             }
+            const float less = -ref[m][b];
+            float l = 0.0f;
 #pragma unroll
             for (int t = 0; t < 4; ++t)
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
-                    const float e = __builtin_amdgcn_exp2f(s[t][b][r] - ref[m][b]);
-                    sum[m][b] += e;
+                    const float e = __builtin_amdgcn_exp2f(fmaf(s[t][b][r], c, less));
+                    l += e;
                     pf[b][t >> 1][(t & 1) * 4 + r] = static_cast<m40_bf16>(e);
                 }
+            sum[m][b] += l;
         }
     }
     // joins sums of other keys (reference, sum and weighted values given as functions of their place)
@@ -290,13 +296,14 @@ __global__ __launch_bounds__(256) void pair_join_kernel(PairArgs p) {
     if (tid < a.vdim) static_cast<T*>(a.out)[m40_packed_at(row, head * a.vdim + tid, a.ld_out >> 5)] = M40Act<T>::from(o * f);
 }
 
-template <int DKT, int DVT, int QB, int PER_CU>
-__global__ __launch_bounds__(256, PER_CU) void pair_tile_kernel(PairArgs p) {
+template <int DKT, int DVT, int QB, int GROUPS, int PER_CU>
+__global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArgs p) {
     typedef __attribute__((address_space(3))) void* lds_dst_t;
     typedef const __attribute__((address_space(1))) void* global_src_t;
     extern __shared__ __align__(16) uint8_t lds[];
     const M40llmPairAttention& a = p.a;
-    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, li = lane & 15;
+    const int lane = threadIdx.x & 63, w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, li = lane & 15;
+    const int wave = w & 3, group = w >> 2;
     const int kt = (int)p.page.k_tiles, vt = (int)p.page.v_tiles, page_tiles = 8 * kt + 2 * vt;
     const uint32_t kv = blockIdx.x, q0 = a.tiles[2 * blockIdx.y], count = a.tiles[2 * blockIdx.y + 1];
     const uint32_t last_row = (q0 + count - 1u) / p.group;
@@ -307,10 +314,12 @@ __global__ __launch_bounds__(256, PER_CU) void pair_tile_kernel(PairArgs p) {
     auto issue = [&](int buf, uint32_t number) __attribute__((always_inline)) {
         const m40_bf16* src = cache + number * p.page.elements();
         for (int i = wave; i < page_tiles; i += 4)
-            __builtin_amdgcn_global_load_lds((global_src_t)(src + (size_t)i * kM40Tile), (lds_dst_t)(lds + (buf * page_tiles + i) * 1024), 16, 0, 0);
+            __builtin_amdgcn_global_load_lds((global_src_t)(src + (size_t)i * kM40Tile), (lds_dst_t)(lds + ((group * 2 + buf) * page_tiles + i) * 1024), 16, 0, 0);
     };
-    issue(0, table[0]);
-    uint32_t next = table[last > 0u ? 1u : 0u];
+    const uint32_t steps = (pages + GROUPS - 1u) / GROUPS;
+    auto page_of = [&](uint32_t step) { const uint32_t n = step * GROUPS + group; return n < last ? n : last; };    // past the end: the last again
+    issue(0, table[page_of(0)]);
+    uint32_t next = table[page_of(1)];
     PairState<DKT, DVT, QB> s;
     s.clear();
     uint32_t row[QB], head[QB];
@@ -338,14 +347,15 @@ __global__ __launch_bounds__(256, PER_CU) void pair_tile_kernel(PairArgs p) {
     const uint32_t pos_first = a.row_pos[(q0 + (wave_live ? i_first : count - 1u)) / p.group], pos_last = a.row_pos[(q0 + (i_last < count ? i_last : count - 1u)) / p.group];
     const float c = a.scale * kLog2e;
     int buf = 0;
-    for (uint32_t n = 0; n < pages; ++n, buf ^= 1) {
-        m40_wait_and_meet<0>();                  // the page has landed, and nobody reads the other buffer any more
-        if (n < last) {
+    for (uint32_t step = 0; step < steps; ++step, buf ^= 1) {
+        m40_wait_and_meet<0>();                  // the pages have landed, and nobody reads the other buffers any more
+        if (step + 1u < steps) {
             issue(buf ^ 1, next);
-            next = table[n + 2u < pages ? n + 2u : last];
+            next = table[page_of(step + 2u)];
         }
-        if (!wave_live || n * kPage > pos_last) continue;
-        const uint8_t* keys = lds + buf * page_tiles * 1024 + lane * 16;
+        const uint32_t n = step * GROUPS + group;
+        if (!wave_live || n > last || n * kPage > pos_last) continue;
+        const uint8_t* keys = lds + (group * 2 + buf) * page_tiles * 1024 + lane * 16;
         const uint8_t* values = keys + 8 * kt * 1024;
         const bool whole = n * kPage + kPage - 1u <= pos_first;
         m40_bf16x8 pf[2][QB][2];
@@ -385,7 +395,16 @@ __global__ __launch_bounds__(256, PER_CU) void pair_tile_kernel(PairArgs p) {
             }
         __builtin_amdgcn_s_setprio(0);
     }
-    __builtin_amdgcn_s_waitcnt(m40_vm_lgkm_wait(0));
+    if constexpr (GROUPS == 2) {
+        m40_wait_and_meet<0>();                  // every buffer is free
+        float* mine = reinterpret_cast<float*>(lds) + (size_t)wave * PairState<DKT, DVT, QB>::kFloats * 64 + lane;
+        if (group == 1) s.put([&](int i, float v) { mine[i * 64] = v; });
+        m40_wait_and_meet<63>();
+        if (group == 1) return;
+        s.join([&](int i) { return mine[i * 64]; });
+    } else {
+        __builtin_amdgcn_s_waitcnt(m40_vm_lgkm_wait(0));
+    }
     if (!wave_live) return;
 #pragma unroll
     for (int b = 0; b < QB; ++b) s.finish(p, b, row[b], head[b], live[b], g);
@@ -447,18 +466,25 @@ int launch_rows(hipStream_t stream, const PairArgs& p) {
     pair_rows_kernel<DKT, DVT><<<dim3(p.a.n_tiles, p.a.kv_heads, p.a.splits), 256, lds, stream>>>(p);
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
-template <int DKT, int DVT, int QB, int PER_CU>
+int page_lds(const PairArgs& p, int groups) { return groups * 2 * (int)(8u * p.page.k_tiles + 2u * p.page.v_tiles) * 1024; }
+template <int DKT, int DVT, int QB, int GROUPS, int PER_CU>
 int launch_tile(hipStream_t stream, const PairArgs& p) {
     static const hipError_t attr =
-        hipFuncSetAttribute(reinterpret_cast<const void*>(pair_tile_kernel<DKT, DVT, QB, PER_CU>), hipFuncAttributeMaxDynamicSharedMemorySize, kLdsMax);
+        hipFuncSetAttribute(reinterpret_cast<const void*>(pair_tile_kernel<DKT, DVT, QB, GROUPS, PER_CU>), hipFuncAttributeMaxDynamicSharedMemorySize, kLdsMax);
     if (attr != hipSuccess) return -2;
-    const int lds = 2 * (int)(8u * p.page.k_tiles + 2u * p.page.v_tiles) * 1024;
-    pair_tile_kernel<DKT, DVT, QB, PER_CU><<<dim3(p.a.kv_heads, p.a.n_tiles), 256, lds, stream>>>(p);
+    constexpr int join = GROUPS == 2 ? 4 * 64 * 4 * PairState<DKT, DVT, QB>::kFloats : 0;
+    static_assert(join <= kLdsMax, "the joining of two groups does not fit");
+    const int pages = page_lds(p, GROUPS);
+    pair_tile_kernel<DKT, DVT, QB, GROUPS, PER_CU><<<dim3(p.a.kv_heads, p.a.n_tiles), GROUPS * 256, pages > join ? pages : join, stream>>>(p);
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
+// PER_CU: workgroups of one group a CU that fit
 template <int DKT, int DVT, int PER_CU>
-int launch_tile_any(hipStream_t stream, const PairArgs& p) {
-    return p.a.tile_queries == 64u ? launch_tile<DKT, DVT, 1, PER_CU>(stream, p) : launch_tile<DKT, DVT, 2, PER_CU>(stream, p);
+int launch_tile_any(hipStream_t stream, const PairArgs& p, int num_cus) {
+    // with enough workgroups the short ones fill in behind the long ones
+    if (page_lds(p, 2) <= kLdsMax && (uint64_t)p.a.kv_heads * p.a.n_tiles <= 3ull * (uint32_t)num_cus)
+        return p.a.tile_queries == 64u ? launch_tile<DKT, DVT, 1, 2, PER_CU>(stream, p) : launch_tile<DKT, DVT, 2, 2, PER_CU>(stream, p);
+    return p.a.tile_queries == 64u ? launch_tile<DKT, DVT, 1, 1, PER_CU>(stream, p) : launch_tile<DKT, DVT, 2, 1, PER_CU>(stream, p);
 }
 
 bool tile_served(uint32_t k_tiles, uint32_t v_tiles) { return 2u * (8u * k_tiles + 2u * v_tiles) * 1024u <= (uint32_t)kLdsMax; }
@@ -483,7 +509,7 @@ int m40llm_ext_pair_attention_async(M40llmCudaContext* ctx, const M40llmPairAtte
     hipStream_t stream = m40_select_stream(ctx, stream_kind);
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
     const uint32_t most = m40llm_ext_pair_attention_tile_queries(a->act_dtype, a->dim, a->vdim);
-    if (a->act_dtype > 1u || a->form > 1u || a->heads == 0 || a->kv_heads == 0 || a->heads % a->kv_heads != 0 || most == 0 || a->ld_out % 32u != 0 ||
+    if (a->act_dtype > 1u || a->form > 1u || a->heads == 0 || a->kv_heads == 0 || a->heads % a->kv_heads != 0 || most == 0 || !(a->scale > 0.0f) || a->ld_out % 32u != 0 ||
         a->ld_out < a->heads * a->vdim || a->n_rows == 0 || !m40_aligned16(a->queries) || !m40_aligned16(a->cache))
         return -3;
     PairArgs p{*a, M40PairPage(a->kv_heads, a->dim, a->vdim), a->heads / a->kv_heads, nullptr, nullptr};
@@ -496,10 +522,10 @@ int m40llm_ext_pair_attention_async(M40llmCudaContext* ctx, const M40llmPairAtte
     const uint32_t kt = p.page.k_tiles, vt = p.page.v_tiles;
     if (a->form == 1u) {
         if ((a->tile_queries != 64u && a->tile_queries != 128u) || a->tile_queries > most || a->n_tiles > 65535u || !tile_served(kt, vt)) return -3;
-        if (kt <= 2u && vt <= 4u) return launch_tile_any<2, 4, 2>(stream, p);
-        if (kt <= 2u && vt <= 8u) return launch_tile_any<2, 8, 2>(stream, p);
-        if (kt <= 4u && vt <= 8u) return launch_tile_any<4, 8, 1>(stream, p);
-        return launch_tile<8, 16, 1, 1>(stream, p);
+        if (kt <= 2u && vt <= 4u) return launch_tile_any<2, 4, 2>(stream, p, ctx->num_cus);
+        if (kt <= 2u && vt <= 8u) return launch_tile_any<2, 8, 2>(stream, p, ctx->num_cus);
+        if (kt <= 4u && vt <= 8u) return launch_tile_any<4, 8, 1>(stream, p, ctx->num_cus);
+        return launch_tile<8, 16, 1, 1, 1>(stream, p);
     }
     if (a->splits == 0 || a->splits > (uint32_t)kJoinSplits || a->kv_heads > 65535u) return -3;
     if (a->splits > 1u) {

@@ -149,102 +149,152 @@ __global__ __launch_bounds__(kThreads) void norm_gate_rows_kernel(const float* _
     }
 }
 
-// A workgroup takes 16 rows and one unit: a map of a query head, a map of a key head, or a value head; 16 lanes a row, lane l the
-// unit's columns l, l + 16, ...
-template <class T>
-__global__ __launch_bounds__(kThreads) void pair_split_append_kernel(M40llmPairSplit a, M40PairPage page) {
-    constexpr uint32_t kMost = 16;       // columns of a lane
-    const uint32_t row = blockIdx.x * 16u + (threadIdx.x >> 4), lane = threadIdx.x & 15u;
-    if (row >= a.rows) return;           // no barrier below; the 16 lanes of a row stay together
-    uint32_t unit = blockIdx.y, n = a.dim, col0;
-    const float *conv = nullptr, *norm = nullptr;
-    int kind = 0;
-    if (unit < 2u * a.heads) {
-        col0 = unit * a.dim;
-        if (a.q_conv) conv = static_cast<const float*>(a.q_conv) + (size_t)unit * a.dim * a.taps;
-        norm = static_cast<const float*>(a.q_norm);
-    } else if (unit < 2u * (a.heads + a.kv_heads)) {
-        kind = 1;
-        unit -= 2u * a.heads;
-        col0 = a.k_offset + unit * a.dim;
-        if (a.k_conv) conv = static_cast<const float*>(a.k_conv) + (size_t)unit * a.dim * a.taps;
-        norm = static_cast<const float*>(a.k_norm);
+// A workgroup takes 16 rows and one unit: a map of a query head, a map of a key head, or a value head; 16 lanes a row, lane l the unit's
+// columns in groups of W at W (l + 16 i), N groups at most (W 4: every size and offset a multiple of 4).
+//
+// What precedes a portion's first row lies in a ring by position, entry p % (taps - 1).  The only row of a portion overwrites the oldest
+// entry, which it has read, with its own.
+template <int W> struct Columns { float v[W]; };
+template <int W>
+__device__ __forceinline__ Columns<W> load_columns(const float* p) {
+    Columns<W> c;
+    if (W == 4) {
+        const float4 t = *reinterpret_cast<const float4*>(p);
+        c.v[0] = t.x; c.v[W > 1 ? 1 : 0] = t.y; c.v[W > 2 ? 2 : 0] = t.z; c.v[W > 3 ? 3 : 0] = t.w;
     } else {
-        kind = 2;
-        unit -= 2u * (a.heads + a.kv_heads);
-        n = a.vdim;
-        col0 = a.v_offset + unit * a.vdim;
-        if (a.v_conv) conv = static_cast<const float*>(a.v_conv) + (size_t)unit * a.vdim * a.taps;
-    }
-    const uint32_t pos = a.row_pos[row], slot = a.row_slot[row], info = a.row_back[row], back = info & 0x7fffffffu;
-    const float* u = static_cast<const float*>(a.proj) + (size_t)row * a.ld_proj + col0;
-    const uint32_t keep = a.taps ? a.taps - 1u : 0u;
-    float* state = static_cast<float*>(a.conv_state) + (size_t)slot * keep * a.ld_state + col0;
-    float y[kMost];
-    float ss = 0.0f;
 #pragma unroll
-    for (uint32_t i = 0; i < kMost; ++i) {
-        const uint32_t c = lane + 16u * i;
-        y[i] = 0.0f;
-        if (c >= n) continue;
-        const float now = u[c];
-        float v = now;
-        if (conv) {
-            const float* w = conv + (size_t)c * a.taps;
-            v = 0.0f;
-            for (uint32_t j = 0; j < keep; ++j) {
-                const uint32_t d = keep - j;             // rows back
-                float before = 0.0f;
-                if (d <= back) before = *(u + c - (size_t)d * a.ld_proj);
-                else if (d <= pos) before = state[(size_t)(keep + back - d) * a.ld_state + c];
-                v = fmaf(w[j], before, v);
-            }
-            v = fmaf(w[keep], now, v);
-            if (info >> 31) {                            // the portion's only row: the state moves on by one
-                for (uint32_t j = 0; j + 1u < keep; ++j) state[(size_t)j * a.ld_state + c] = state[(size_t)(j + 1u) * a.ld_state + c];
-                if (keep) state[(size_t)(keep - 1u) * a.ld_state + c] = now;
+        for (int k = 0; k < W; ++k) c.v[k] = p[k];
+    }
+    return c;
+}
+template <class T, int W>
+__device__ __forceinline__ void store_columns(T* p, const float (&v)[W]) {
+    if (W == 4) m40_store4<T>(p, m40_float4{v[0], v[W > 1 ? 1 : 0], v[W > 2 ? 2 : 0], v[W > 3 ? 3 : 0]});
+    else {
+#pragma unroll
+        for (int k = 0; k < W; ++k) p[k] = M40Act<T>::from(v[k]);
+    }
+}
+enum { kQueries = 0, kKeys = 1, kValues = 2 };
+template <class T, int W, int N>
+__device__ __forceinline__ void split_unit(const M40llmPairSplit& a, const M40PairPage& page, int kind, uint32_t unit, uint32_t row, uint32_t lane) {
+    const uint32_t n = kind == kValues ? a.vdim : a.dim, col0 = (kind == kQueries ? 0u : kind == kKeys ? a.k_offset : a.v_offset) + unit * n;
+    const uint32_t all = (kind == kQueries ? 2u * a.heads : kind == kKeys ? 2u * a.kv_heads : a.kv_heads) * n;      // columns of this kind
+    const float* conv = static_cast<const float*>(kind == kQueries ? a.q_conv : kind == kKeys ? a.k_conv : a.v_conv);
+    const uint32_t pos = a.row_pos[row], slot = a.row_slot[row], info = a.row_back[row], back = info & 0x7fffffffu;
+    const uint32_t number = kind == kQueries ? 0u : a.page_table[(size_t)slot * a.max_pages + pos / M40LLM_PAGE_TOKENS];
+    const float* u = static_cast<const float*>(a.proj) + (size_t)row * a.ld_proj + col0;
+    uint32_t c[N];
+    bool live[N];
+    Columns<W> now[N];
+    float y[N][W];
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+        c[i] = W * (lane + 16u * i);
+        live[i] = c[i] < n;
+        if (!live[i]) c[i] = 0u;             // loads of columns past the unit go to its first
+        now[i] = load_columns<W>(u + c[i]);
+    }
+    if (a.taps) {
+        const uint32_t keep = a.taps - 1u;
+        float* state = static_cast<float*>(a.conv_state) + (size_t)slot * keep * a.ld_state + col0;
+        const float* w = conv + unit * n;
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+            const Columns<W> wn = load_columns<W>(w + (size_t)keep * all + c[i]);
+#pragma unroll
+            for (int k = 0; k < W; ++k) y[i][k] = wn.v[k] * now[i].v[k];
+        }
+#pragma unroll 4
+        for (uint32_t d = 1; d <= keep; ++d) {               // rows back; loads under selected addresses, none behind a branch
+            const bool here = d <= back, some = d <= pos;
+            const float* src = here ? u - (size_t)d * a.ld_proj : some ? state + (size_t)((pos - d) % keep) * a.ld_state : u;
+            const float f = some ? 1.0f : 0.0f;
+#pragma unroll
+            for (int i = 0; i < N; ++i) {
+                const Columns<W> before = load_columns<W>(src + c[i]), wd = load_columns<W>(w + (size_t)(keep - d) * all + c[i]);
+#pragma unroll
+                for (int k = 0; k < W; ++k) y[i][k] = fmaf(wd.v[k] * f, before.v[k], y[i][k]);
             }
         }
-        y[i] = v;
-        ss = fmaf(v, v, ss);
+        if (info >> 31 && keep) {
+            float* own = state + (size_t)(pos % keep) * a.ld_state;
+#pragma unroll
+            for (int i = 0; i < N; ++i)
+                if (live[i]) store_columns<float, W>(own + c[i], now[i].v);
+        }
+    } else {
+#pragma unroll
+        for (int i = 0; i < N; ++i)
+#pragma unroll
+            for (int k = 0; k < W; ++k) y[i][k] = now[i].v[k];
     }
-    if (kind < 2) {
+#pragma unroll
+    for (int i = 0; i < N; ++i)
+#pragma unroll
+        for (int k = 0; k < W; ++k) y[i][k] = live[i] ? y[i][k] : 0.0f;
+    if (kind != kValues) {
+        const float* norm = static_cast<const float*>(kind == kQueries ? a.q_norm : a.k_norm);
+        float ss = 0.0f;
+#pragma unroll
+        for (int i = 0; i < N; ++i)
+#pragma unroll
+            for (int k = 0; k < W; ++k) ss = fmaf(y[i][k], y[i][k], ss);
         const float inv = 1.0f / sqrtf(m40_sum16(ss) / (float)n + a.eps);
 #pragma unroll
-        for (uint32_t i = 0; i < kMost; ++i) {
-            const uint32_t c = lane + 16u * i;
-            if (c < n) y[i] = y[i] * inv * norm[c];
+        for (int i = 0; i < N; ++i) {
+            const Columns<W> w = load_columns<W>(norm + c[i]);
+#pragma unroll
+            for (int k = 0; k < W; ++k) y[i][k] *= inv * w.v[k];
         }
     }
-    if (kind == 0) {
-        const uint32_t pad = page.k_tiles * 32u;
-        T* q = static_cast<T*>(a.queries) + ((size_t)row * 2u * a.heads + unit) * pad;
+    T* cache = static_cast<T*>(a.cache) + number * page.elements() + (kind == kKeys ? unit / 2u : unit) * page.head_elements();
+    const uint32_t t = pos % M40LLM_PAGE_TOKENS, pad = kind == kValues ? page.v_tiles * 16u : page.k_tiles * 32u;
+    T* q = static_cast<T*>(a.queries) + ((size_t)row * 2u * a.heads + unit) * pad;
 #pragma unroll
-        for (uint32_t i = 0; i < kMost; ++i)
-            if (lane + 16u * i < pad) q[lane + 16u * i] = M40Act<T>::from(y[i]);
-        return;
-    }
-    const uint32_t number = a.page_table[(size_t)slot * a.max_pages + pos / M40LLM_PAGE_TOKENS], t = pos % M40LLM_PAGE_TOKENS;
-    T* base = static_cast<T*>(a.cache) + number * page.elements() + (kind == 1 ? unit / 2u : unit) * page.head_elements();
+    for (int i = 0; i < N; ++i) {
+        const uint32_t at = W * (lane + 16u * i);            // pads too: zeros
+        if (at >= pad) continue;
+        if (kind == kQueries) store_columns<T, W>(q + at, y[i]);
+        else if (kind == kKeys) store_columns<T, W>(cache + page.key_at(unit % 2u, t, at), y[i]);
+        else {
 #pragma unroll
-    for (uint32_t i = 0; i < kMost; ++i) {
-        const uint32_t c = lane + 16u * i;
-        if (kind == 1) {
-            if (c < page.k_tiles * 32u) base[page.key_at(unit % 2u, t, c)] = M40Act<T>::from(y[i]);
-        } else {
-            if (c < page.v_tiles * 16u) base[page.value_at(t, c)] = M40Act<T>::from(y[i]);
+            for (int k = 0; k < W; ++k) cache[page.value_at(t, at + k)] = M40Act<T>::from(y[i][k]);
         }
     }
 }
+template <class T, int W, int NQ, int NV>
+__global__ __launch_bounds__(kThreads) void pair_split_append_kernel(M40llmPairSplit a, M40PairPage page) {
+    const uint32_t row = blockIdx.x * 16u + (threadIdx.x >> 4), lane = threadIdx.x & 15u, unit = blockIdx.y;
+    if (row >= a.rows) return;           // no barrier below; the 16 lanes of a row stay together
+    if (unit < 2u * a.heads) split_unit<T, W, NQ>(a, page, kQueries, unit, row, lane);
+    else if (unit < 2u * (a.heads + a.kv_heads)) split_unit<T, W, NQ>(a, page, kKeys, unit - 2u * a.heads, row, lane);
+    else split_unit<T, W, NV>(a, page, kValues, unit - 2u * (a.heads + a.kv_heads), row, lane);
+}
 
-// a thread a column: oldest first, so that a value is read before its place is taken
+// A thread a column: the last rows of a portion take their places in the ring.
 __global__ __launch_bounds__(kThreads) void conv_state_kernel(const float* __restrict__ proj, size_t ld_proj, uint32_t cols, uint32_t keep,
-                                                              float* __restrict__ state, size_t ld_state, const uint32_t* __restrict__ portions) {
+                                                              float* __restrict__ state, size_t ld_state, const uint32_t* __restrict__ portions,
+                                                              const uint32_t* __restrict__ row_pos) {
     const uint32_t row = portions[4 * blockIdx.y], n = portions[4 * blockIdx.y + 1], slot = portions[4 * blockIdx.y + 2];
     const uint32_t c = blockIdx.x * kThreads + threadIdx.x;
     if (n < 2u || c >= cols) return;
     float* s = state + (size_t)slot * keep * ld_state + c;
-    for (uint32_t i = 0; i < keep; ++i) s[i * ld_state] = n + i >= keep ? proj[(size_t)(row + n + i - keep) * ld_proj + c] : s[(i + n) * ld_state];
+    const uint32_t first = row_pos[row];
+    for (uint32_t i = n > keep ? n - keep : 0u; i < n; ++i) s[(size_t)((first + i) % keep) * ld_state] = proj[(size_t)(row + i) * ld_proj + c];
+}
+
+template <class T>
+void launch_split(hipStream_t stream, const M40llmPairSplit& s, const M40PairPage& page) {
+    const dim3 grid((s.rows + 15u) / 16u, 2u * s.heads + (s.cache ? 3u * s.kv_heads : 0u));
+    const bool vec = s.dim % 4u == 0 && s.vdim % 4u == 0 && s.ld_proj % 4u == 0 && s.ld_state % 4u == 0 && s.k_offset % 4u == 0 && s.v_offset % 4u == 0 &&
+                     m40_aligned16(s.proj) && m40_aligned16(s.conv_state) && m40_aligned16(s.q_conv) && m40_aligned16(s.k_conv) && m40_aligned16(s.v_conv) &&
+                     m40_aligned16(s.q_norm) && m40_aligned16(s.k_norm);
+    if (!vec) pair_split_append_kernel<T, 1, 16, 16><<<grid, kThreads, 0, stream>>>(s, page);
+    else if (s.dim <= 64u && s.vdim <= 64u) pair_split_append_kernel<T, 4, 1, 1><<<grid, kThreads, 0, stream>>>(s, page);
+    else if (s.dim <= 64u && s.vdim <= 128u) pair_split_append_kernel<T, 4, 1, 2><<<grid, kThreads, 0, stream>>>(s, page);
+    else if (s.dim <= 128u && s.vdim <= 128u) pair_split_append_kernel<T, 4, 2, 2><<<grid, kThreads, 0, stream>>>(s, page);
+    else pair_split_append_kernel<T, 4, 4, 4><<<grid, kThreads, 0, stream>>>(s, page);
 }
 
 int launched() { return hipGetLastError() == hipSuccess ? 0 : -2; }
@@ -307,20 +357,19 @@ int m40llm_ext_pair_split_append_async(M40llmCudaContext* ctx, const M40llmPairS
                      (s->taps && (!s->k_conv || !s->v_conv))))
         return -4;
     const M40PairPage page(s->kv_heads, s->dim, s->vdim);
-    const dim3 grid((s->rows + 15u) / 16u, 2u * s->heads + (s->cache ? 3u * s->kv_heads : 0u));
-    if (s->act_dtype == M40LLM_ACT_F32) pair_split_append_kernel<float><<<grid, kThreads, 0, stream>>>(*s, page);
-    else pair_split_append_kernel<m40_bf16><<<grid, kThreads, 0, stream>>>(*s, page);
+    if (s->act_dtype == M40LLM_ACT_F32) launch_split<float>(stream, *s, page);
+    else launch_split<m40_bf16>(stream, *s, page);
     return launched();
 }
 
 int m40llm_ext_conv_state_async(M40llmCudaContext* ctx, const void* d_proj, uint64_t ld_proj, uint32_t cols, uint32_t taps, void* d_state, uint64_t ld_state,
-                                const uint32_t* d_portions, uint32_t n_portions, uint32_t stream_kind) {
-    if (!ctx || !d_proj || !d_state || !d_portions) return -1;
+                                const uint32_t* d_portions, const uint32_t* d_row_pos, uint32_t n_portions, uint32_t stream_kind) {
+    if (!ctx || !d_proj || !d_state || !d_portions || !d_row_pos) return -1;
     hipStream_t stream = m40_select_stream(ctx, stream_kind);
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
     if (cols == 0 || taps < 2u || ld_proj < cols || ld_state < cols || n_portions == 0 || n_portions > 65535u) return -3;
     conv_state_kernel<<<dim3((cols + kThreads - 1) / kThreads, n_portions), kThreads, 0, stream>>>(static_cast<const float*>(d_proj), (size_t)ld_proj, cols,
-                                                                                                  taps - 1u, static_cast<float*>(d_state), (size_t)ld_state, d_portions);
+                                                                                                  taps - 1u, static_cast<float*>(d_state), (size_t)ld_state, d_portions, d_row_pos);
     return launched();
 }
 

@@ -206,6 +206,7 @@ inline DecoderSpec read_gulidra(const json::Value& c) {
             a.diff = m.num("diff");
             check(a.heads && a.kv_heads && a.dim && a.vdim, "a size is zero");
             check(a.heads % a.kv_heads == 0, "heads must be a multiple of kv_heads");
+            check(a.scale != 0.0f, "scale is zero");
             if (const json::Value* j = m.find("kv_from"); j && !j->is_null()) {
                 const uint32_t from = j->as_u32("kv_from");
                 check(from < i, "kv_from must name an earlier layer");

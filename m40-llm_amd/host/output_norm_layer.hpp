@@ -66,21 +66,24 @@ public:
         k_offset_ = round_up(q, 16);
         v_offset_ = k_offset_ + (source ? 0 : round_up(k, 16));
         gate_offset_ = v_offset_ + (source ? 0 : round_up(v, 16));
-        conv_cols_ = source ? q : v_offset_ + v;
+        conv_cols_ = round_up(source ? q : v_offset_ + v, 4);
         tiles_in_ = round_up(gate_offset_ + a.heads, 16) / 16;
         o_pad_ = round_up(a.heads * a.vdim, 32);
         const uint32_t D = rt.spec.width, d_tiles = rt.d_pad / 32;
         w_in_ = rt.packed(tiles_in_, d_tiles);
         rt.pack(t, p + "q", q, D, w_in_.ptr(), d_tiles, 0);
-        q_norm_ = rt.upload_f32(t.read_f32(p + "q.norm", {a.dim}));
-        if (a.taps) q_conv_ = rt.upload_f32(t.read_f32(p + "q.conv", {q, a.taps}));
+        std::vector<float> q_norm = t.read_f32(p + "q.norm", {a.dim});
+        if (a.scale < 0.0f)                   // the kernels take the scale's sign from the queries
+            for (float& w : q_norm) w = -w;
+        q_norm_ = rt.upload_f32(q_norm);
+        if (a.taps) q_conv_ = conv_weights(t, p + "q.conv", q);
         if (!source) {
             rt.pack(t, p + "k", k, D, w_in_.ptr(), d_tiles, k_offset_ / 16);
             rt.pack(t, p + "v", v, D, w_in_.ptr(), d_tiles, v_offset_ / 16);
             k_norm_ = rt.upload_f32(t.read_f32(p + "k.norm", {a.dim}));
             if (a.taps) {
-                k_conv_ = rt.upload_f32(t.read_f32(p + "k.conv", {k, a.taps}));
-                v_conv_ = rt.upload_f32(t.read_f32(p + "v.conv", {v, a.taps}));
+                k_conv_ = conv_weights(t, p + "k.conv", k);
+                v_conv_ = conv_weights(t, p + "v.conv", v);
             }
             cache_ = rt.cleared((size_t)rt.max_pages * m40llm_ext_pair_page_elements(a.kv_heads, a.dim, a.vdim) * rt.es);
         }
@@ -137,10 +140,10 @@ public:
         }
         if (a_.taps > 1 && r.multi_row_portions)
             M40H_TRY(m40llm_ext_conv_state_async(rt_.ctx, rt_.proj.ptr(), ld, conv_cols_, a_.taps, conv_state_.ptr(), conv_cols_, portions_.multi(),
-                                                 r.multi_row_portions, rt_.kStream));
+                                                 r.pos, r.multi_row_portions, rt_.kStream));
         M40llmPairAttention h{};
         h.act_dtype = rt_.opt.act_dtype; h.heads = a_.heads; h.kv_heads = a_.kv_heads; h.dim = a_.dim; h.vdim = a_.vdim;
-        h.scale = a_.scale; h.lambda = lambda_; h.out_scale = (float)(1.0 - a_.diff); h.eps = rt_.spec.eps;
+        h.scale = std::fabs(a_.scale); h.lambda = lambda_; h.out_scale = (float)(1.0 - a_.diff); h.eps = rt_.spec.eps;
         h.queries = sh_->queries.ptr(); h.cache = cache.ptr();
         h.gate = rt_.proj.f32(gate_offset_); h.ld_gate = ld;
         h.row_slot = r.slot; h.row_pos = r.pos; h.page_table = r.page_table; h.max_pages = rt_.max_pages;
@@ -165,6 +168,14 @@ public:
     }
 
 private:
+    // [columns][taps] to [taps][columns]
+    DeviceBuf conv_weights(TensorSource& t, const std::string& name, uint32_t cols) {
+        const std::vector<float> w = t.read_f32(name, {cols, a_.taps});
+        std::vector<float> o(w.size());
+        for (uint32_t c = 0; c < cols; ++c)
+            for (uint32_t j = 0; j < a_.taps; ++j) o[(size_t)j * cols + c] = w[(size_t)c * a_.taps + j];
+        return rt_.upload_f32(o);
+    }
     LayerRuntime& rt_;
     std::shared_ptr<PairShared> sh_;
     DifferentialAttentionSpec a_;

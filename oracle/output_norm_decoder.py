@@ -121,6 +121,21 @@ def route(h, w_router, correction, top):
     return chosen, np.take_along_axis(s, chosen, axis=1)
 
 
+def choice_margin(h, w_router, correction, top):
+    """How far the choice is from another one, per token: the difference between the last chosen and the first left out, in units of their
+    scores (how much a router logit would have to move); infinite where every expert is chosen."""
+    z = h @ w_router.T
+    e = np.exp(z - z.max(axis=1, keepdims=True))
+    s = e / e.sum(axis=1, keepdims=True)
+    if top >= s.shape[1]:
+        return np.full(len(h), np.inf)
+    c = s + correction
+    order = np.argsort(-c, axis=1, kind="stable")
+    pair = order[:, top - 1:top + 1]
+    c2, s2 = np.take_along_axis(c, pair, axis=1), np.take_along_axis(s, pair, axis=1)
+    return (c2[:, 0] - c2[:, 1]) / s2.max(axis=1)
+
+
 def expert_mlp(h, T, p, r):
     """The last r.identity of the experts return their input."""
     chosen, weight = route(h, T[p + "router"], T[p + "correction"], r["top"])
@@ -156,6 +171,7 @@ class Sequence:
         self.state = [dict() for _ in model.cfg["layers"]]
         self.kv = {}
         self.layer_outputs = []
+        self.margins = []          # smallest choice_margin of every token fed so far
 
     def mixer(self, i, layer, x, pos):
         T, eps, m, p = self.m.T, self.m.eps, layer["mixer"], f"l{i}.mix."
@@ -178,13 +194,17 @@ class Sequence:
         x = embedding(tokens, pos, T["embed"], cfg["embedding"]["scale"], T["pos"])
         mult = cfg["residual_mult"]
         self.layer_outputs = []
+        margin = np.full(len(tokens), np.inf)
         for i, layer in enumerate(cfg["layers"]):
             p = f"l{i}."
             x = x + mult * rms_norm(self.mixer(i, layer, x, pos), T[p + "norm1"], eps)
             if layer.get("mlp"):
                 l = layer["mlp"]
+                if l["kind"] != "dense":
+                    margin = np.minimum(margin, choice_margin(x, T[p + "mlp.router"], T[p + "mlp.correction"], l["router"]["top"]))
                 y = gated_mlp(x, T, p + "mlp.") if l["kind"] == "dense" else expert_mlp(x, T, p + "mlp.", l["router"])
                 x = x + mult * rms_norm(y, T[p + "norm2"], eps)
             self.layer_outputs.append(x)
         self.n += len(tokens)
+        self.margins += margin.tolist()
         return rms_norm(x, T["final.norm"], eps) @ T["head"].T

@@ -19,20 +19,26 @@ DTYPES = ["float32", "bfloat16"]
 FORMS = [("float32", 0), ("bfloat16", 1), ("bfloat16", 2)]
 
 
-def assert_close(e, dtype, what="", factor=1.0):
-    """In bf16 a token whose choice of experts is a close call may take another: a few positions may be further off, none far."""
+CLOSE_CALL = 0.2      # router logits closer than this may decide otherwise in bf16
+
+
+def assert_close(e, dtype, margins=None, what="", factor=1.0):
+    """e: errors of some positions.  In bf16 a token whose choice of experts is a close call may take another expert; its own error is then of
+    the size of one expert's share, and what later tokens see of it is small."""
+    e = np.asarray(e)
     assert np.isfinite(e).all(), (what, dtype)
     limit = factor * LIMIT[dtype]
-    if dtype == "float32":
+    if dtype == "bfloat16" and margins is not None:
+        close = np.asarray(margins) < CLOSE_CALL
+        assert (e.size < 20 or close.mean() < 0.6) and (not close.any() or e[close].max() < 1.5), (what, float(close.mean()))
+        e = e[~close]
+        assert (e > limit).sum() <= 0.02 * e.size and (e.size == 0 or e.max() <= 4 * limit), (what, dtype, int((e > limit).sum()), e.size, float(e.max()))
+    else:
         assert e.max() <= limit, (what, int(e.argmax()), float(e.max()))
-        return
-    over = int((e > limit).sum())
-    assert over <= max(1, 0.02 * e.size) and e.max() <= 0.5, (what, dtype, over, e.size, float(e.max()))
 
 
-def assert_logits(got, want, dtype, what="", factor=1.0, spread=None):
-    d = logits_error(got, want) * (np.std(want) / spread if spread else 1.0)
-    assert_close(d, dtype, what, factor)
+def assert_logits(got, want, dtype, margins=None, what="", factor=1.0):
+    assert_close(logits_error(got, want), dtype, margins, what, factor)
 
 
 @pytest.fixture(scope="module")
@@ -53,7 +59,8 @@ def folders(tmp_path_factory):
 
 @pytest.fixture(scope="module")
 def expected(folders):
-    """(tokens, logits [tokens][vocab], residuals [layers][tokens][width]) of a sequence of n tokens, computed whole."""
+    """(tokens, logits [tokens][vocab], residuals [layers][tokens][width], margins of the experts' choice) of a sequence of n tokens,
+    computed whole."""
     kept, models = {}, {}
 
     def get(name, n, seed=0):
@@ -61,7 +68,7 @@ def expected(folders):
             m = models.setdefault(name, od.Model.load(folders(name)))
             t = np.random.default_rng(1000 * seed + n).integers(0, m.cfg["vocab"], size=n)
             s = m.sequence()
-            kept[name, n, seed] = (t, s.feed(t.tolist()), np.stack(s.layer_outputs))
+            kept[name, n, seed] = (t, s.feed(t.tolist()), np.stack(s.layer_outputs), np.array(s.margins))
         return kept[name, n, seed]
     return get
 
@@ -73,26 +80,26 @@ def open_model(ctx, folder, dtype, max_tokens=1024, slots=4, **kw):
 @pytest.mark.parametrize("dtype,form", FORMS)
 @pytest.mark.parametrize("name,n", [("odd", 150), ("even", 200), ("wide", 140), ("one", 70)])
 def test_residual_after_every_layer_and_logits_of_a_whole_prompt(ctx, folders, expected, name, n, dtype, form):
-    t, want, res = expected(name, n)
+    t, want, res, margins = expected(name, n)
     m = open_model(ctx, folders(name), dtype, portion_form=form)
     x = m.step_layers(0, t, *[res.shape[i] for i in (0, 2)])
     for i in range(len(res)):
         e = np.sqrt(((x[i] - res[i]) ** 2).mean(axis=-1)) / np.sqrt((res[i] ** 2).mean())
-        assert_close(e, dtype, i)
+        assert_close(e, dtype, margins, i)
     m.release(0)
-    assert_logits(m.step([(1, t, range(n))]), want, dtype)
+    assert_logits(m.step([(1, t, range(n))]), want, dtype, margins)
     m.close()
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("name,n,first", [("odd", 135, 60), ("even", 200, 1), ("wide", 90, 66), ("one", 70, 62)])
 def test_token_by_token_equals_the_whole_prompt(ctx, folders, expected, name, n, first, dtype):
-    t, want, _ = expected(name, n)
+    t, want, _, margins = expected(name, n)
     m = open_model(ctx, folders(name), dtype)
     got = [m.step([(2, t[:first], range(first))])]
     for i in range(first, n):
         got.append(m.step([(2, t[i:i + 1], [0])]))
-    assert_logits(np.concatenate(got), want, dtype)
+    assert_logits(np.concatenate(got), want, dtype, margins)
     m.close()
 
 
@@ -100,14 +107,14 @@ def test_token_by_token_equals_the_whole_prompt(ctx, folders, expected, name, n,
 @pytest.mark.parametrize("name,n", [("odd", 330), ("even", 330), ("wide", 200)])
 @pytest.mark.parametrize("cut", [[2], [3, 2, 61, 64, 66], [63, 1], [128, 5], [65], [200, 2]])
 def test_portions_of_any_size(ctx, folders, expected, name, n, cut, dtype, form):
-    t, want, _ = expected(name, n)
+    t, want, _, margins = expected(name, n)
     m = open_model(ctx, folders(name), dtype, portion_form=form)
     at, k, got = 0, 0, []
     while at < n:
         c = min(cut[k % len(cut)], n - at)
         got.append(m.step([(0, t[at:at + c], range(c))]))
         at, k = at + c, k + 1
-    assert_logits(np.concatenate(got), want, dtype, cut)
+    assert_logits(np.concatenate(got), want, dtype, margins, cut)
     m.close()
 
 
@@ -120,7 +127,7 @@ def test_mixed_batches_with_pages_and_slots_used_again(ctx, folders, expected, d
     lens = [5, 64, 65, 150, 127, 2, 129, 70, 1, 192, 128, 33]
     m = open_model(ctx, folders("odd"), dtype, max_tokens=4 * 192, max_rows=max_rows, portion_form=form)
     free0 = m.free_pages()
-    waiting, live, free, errors = list(range(len(lens))), {}, [0, 1, 2, 3], []
+    waiting, live, free, errors, margins = list(range(len(lens))), {}, [0, 1, 2, 3], [], []
     seqs = {i: expected("odd", n, seed=1 + i) for i, n in enumerate(lens)}
     spread = np.std(np.concatenate([s[1] for s in seqs.values()]))
     while waiting or live:
@@ -143,13 +150,14 @@ def test_mixed_batches_with_pages_and_slots_used_again(ctx, folders, expected, d
         want = np.stack([seqs[i][1][p] for i, p in rows])
         e = logits_error(got, want) * np.std(want) / spread
         if dtype == "float32":
-            assert_close(e, dtype, (rows[0], len(entries)))
+            assert_close(e, dtype, None, (rows[0], len(entries)))
         errors.append(e)
+        margins += [seqs[i][3][p] for i, p in rows]
         for i in [i for i, (slot, at) in live.items() if at == lens[i]]:
             slot, _ = live.pop(i)
             m.release(slot)
             free.append(slot)
-    assert_close(np.concatenate(errors), dtype)
+    assert_close(np.concatenate(errors), dtype, margins)
     assert m.free_pages() == free0
     m.close()
 
@@ -160,15 +168,15 @@ def test_batch_of_unequal_requests_equals_each_alone(ctx, folders, expected, dty
     lens = [200, 3, 129, 64]
     seqs = [expected("even", n, seed=40) for n in lens]
     alone = []
-    for t, _, _ in seqs:
+    for t, _, _, _ in seqs:
         alone.append(m.step([(0, t, range(len(t)))]))
         m.release(0)
-    together = m.step([(i, t, range(len(t))) for i, (t, _, _) in enumerate(seqs)])
+    together = m.step([(i, t, range(len(t))) for i, (t, _, _, _) in enumerate(seqs)])
     at = 0
-    for (t, want, _), a in zip(seqs, alone):
+    for (t, want, _, margins), a in zip(seqs, alone):
         b = together[at:at + len(t)]
-        assert_logits(b, want, dtype)
-        assert_close(logits_error(a, b.astype(np.float64)), dtype, factor={"float32": 0.25, "bfloat16": 0.7}[dtype])
+        assert_logits(b, want, dtype, margins)
+        assert_close(logits_error(a, b.astype(np.float64)), dtype, margins, factor={"float32": 0.25, "bfloat16": 0.7}[dtype])
         at += len(t)
     m.close()
 
@@ -181,25 +189,26 @@ def test_first_tokens_of_a_sequence_on_used_slots(ctx, folders, dtype):
     m.step([(1, np.arange(60) % 101, [])])
     m.release(1)
     for first, cut in (([7], 1), ([0, 0, 5, 9, 9, 100], 1), ([100, 3, 100, 4, 8], 2), ([1, 2, 3, 4, 5, 6, 7], 3)):
-        want = mod.sequence().feed(first)
+        s = mod.sequence()
+        want = s.feed(first)
         got = [m.step([(1, first[i:i + cut], range(len(first[i:i + cut])))]) for i in range(0, len(first), cut)]
-        assert_logits(np.concatenate(got), want, dtype, (first, cut))
+        assert_logits(np.concatenate(got), want, dtype, s.margins, (first, cut))
         m.release(1)
     m.close()
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_wanted_places_any_order_and_none(ctx, folders, expected, dtype):
-    t, want, _ = expected("odd", 135)
+    t, want, _, margins = expected("odd", 135)
     m = open_model(ctx, folders("odd"), dtype)
     assert m.step([(0, t[:40], [])]).shape == (0, want.shape[1])
     got = m.step([(0, t[40:], [94, 0, 3, 3])])
-    assert_logits(got, want[[134, 40, 43, 43]], dtype)
+    assert_logits(got, want[[134, 40, 43, 43]], dtype, margins[[134, 40, 43, 43]])
     m.close()
 
 
 def test_bad_steps_are_refused_and_change_nothing(ctx, folders, expected):
-    t, want, _ = expected("odd", 135)
+    t, want, _, margins = expected("odd", 135)
     m = open_model(ctx, folders("odd"), "float32", max_tokens=192, slots=2)
     m.step([(0, t[:64], [])])
     for bad in ([(0, [5000], [])], [(2, [1], [])], [(0, [1], [1])], [(0, [1], []), (0, [2], [])], [(0, [], [])],
@@ -241,7 +250,7 @@ def test_long_greedy_decoding_equals_the_oracle(ctx, folders, dtype, mode, guard
     assert m.length(0) == len(prompt) + 159
     # the loop's state carries on: the next token continues behind it
     got = m.step([(0, ids[-1:], [0])])
-    assert_logits(got, s.feed(ids[-1:].tolist()), dtype, factor=2)
+    assert_logits(got, s.feed(ids[-1:].tolist()), dtype, s.margins[-1:], factor=2)
     m.close()
 
 
@@ -310,7 +319,7 @@ def test_command_line_generates_what_the_oracle_picks(ctx, folders, capsys):
 
 def test_trace_replay(ctx, folders, expected, tmp_path):
     """bin/trace_run over a small trace in 32-bit: requests cut into steps, ended and admitted on slots that were used before."""
-    t, want, _ = expected("odd", 135)
+    t, want, _, margins = expected("odd", 135)
     V = want.shape[1]
     steps, rows = [], []
 
