@@ -334,7 +334,7 @@ template <int FORM>
 int launch_tile_any(hipStream_t stream, const PackedArgs& g, const M40Epilogue<m40_bf16>& e, int batches, int num_cus) {
     const long long wide = (long long)(FORM == kSlots || FORM == kGather ? g.rows : (g.rows + 127) / 128) * ((g.n_tiles + 15) / 16) * batches;
     // a short sum is mostly a workgroup's start and end: two narrower workgroups a CU cover each other's
-    if (wide * 16 >= 9ll * num_cus && g.k_tiles > 32) return launch_tile<8, FORM>(stream, g, e, batches);
+    if (wide * 16 >= 9ll * num_cus && g.k_tiles > (FORM == kSlots ? 64 : 32)) return launch_tile<8, FORM>(stream, g, e, batches);
     return launch_tile<4, FORM>(stream, g, e, batches);
 }
 
