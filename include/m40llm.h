@@ -594,7 +594,7 @@ typedef struct M40llmPackedGemm {
     const uint32_t* pages;        /* KEYS, VALUES: device */
     uint32_t page_k_tiles;        /* k tiles of a cache entry */
     uint32_t activation;          /* PROJECT: M40LLM_GELU_TANH or M40LLM_SILU */
-    /* Products per expert (jobs not NULL; PROJECT without plain tiles, STORE_ACT): job j of the jobs[0] jobs behind word 4 is {expert,
+    /* Products per expert (jobs not NULL; PROJECT without plain tiles, with `gather` up to 64 rows a job and without for 128; STORE_ACT): job j of the jobs[0] jobs behind word 4 is {expert,
      * first slot, slots}, slots at most job_rows (16, 32, 64 or 128); weights of expert e start at w + e*w_batch.  With `gather`, the
      * rows of a are plain rows gather[slot] of lda columns; without, packed rows `slot`.  Results are rows `slot`. */
     const uint32_t *jobs, *gather;
@@ -667,7 +667,7 @@ int m40llm_ext_norm_gate_rows_async(M40llmCudaContext* ctx, const void* d_y, uin
  * Of `experts` + `identity` experts each row takes the `top` with the largest softmax(logits) + correction (the lower index of equals);
  * its weights are the softmax values.  ids / weight: [rows][top].  Then rows are sorted by expert: every expert's rows, in order, take
  * slots from a multiple of 16 on; rows_of[slot] = row (slots that pad a group of 16 repeat a row), place[row*top + j] = slot, or
- * M40LLM_PLACE_INPUT for identity experts; jobs (m40llm_ext_packed_gemm_async) of at most job_rows slots.  rows_of holds
+ * M40LLM_PLACE_INPUT for identity experts; jobs (m40llm_ext_packed_gemm_async) of at most job_rows slots; jobs[1] = slots in use.  rows_of holds
  * m40llm_ext_expert_slots, jobs 4 + 4 * m40llm_ext_expert_max_jobs words. */
 typedef struct M40llmRoute {
     uint32_t rows, experts, identity, top, job_rows;
@@ -679,6 +679,9 @@ typedef struct M40llmRoute {
     uint32_t *rows_of, *place, *jobs;
 } M40llmRoute;
 int m40llm_ext_route_rows_async(M40llmCudaContext* ctx, const M40llmRoute* r, uint32_t stream_kind);
+/* dst, packed rows of ld columns: slot s = plain row rows_of[s] of src (bf16), for the slots in use; max_slots: m40llm_ext_expert_slots */
+int m40llm_ext_gather_rows_async(M40llmCudaContext* ctx, const void* d_src_bf16, uint32_t ld, const uint32_t* d_rows_of, const uint32_t* d_jobs,
+                                 uint32_t max_slots, void* d_dst_bf16, uint32_t stream_kind);
 uint32_t m40llm_ext_expert_slots(uint32_t rows, uint32_t experts, uint32_t top);
 uint32_t m40llm_ext_expert_max_jobs(uint32_t rows, uint32_t experts, uint32_t top, uint32_t job_rows);
 #define M40LLM_MAX_EXPERTS 1024u

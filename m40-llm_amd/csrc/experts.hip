@@ -152,8 +152,9 @@ __global__ __launch_bounds__(kListThreads) void expert_lists_kernel(M40llmRoute 
     slots = jobs = all = 0u;
 #pragma unroll
     for (uint32_t w = 0; w < kListWaves; ++w) { slots += wave_slots[w]; jobs += wave_jobs[w]; all += wave_all[w]; }
-    if (mine == 0u && tid == 0u) a.jobs[0] = all;
     const uint32_t n = count[mine];
+    if (mine == 0u && tid == 0u) a.jobs[0] = all;
+    if (mine == E - 1u && tid == 0u) a.jobs[1] = slots + ((n + 15u) & ~15u);
     for (uint32_t j = tid; j * a.job_rows < n; j += kListThreads) {
         uint32_t* job = a.jobs + 4u + 4u * (jobs + j);
         const uint32_t left = n - j * a.job_rows;
@@ -196,6 +197,17 @@ __global__ __launch_bounds__(kListThreads) void expert_lists_kernel(M40llmRoute 
     if (tid < ((n + 15u) & ~15u) - n) a.rows_of[slots + n + tid] = 0u;
 }
 
+// A wave moves 16 x 32 operand tiles: 16 rows of the list side by side.
+__global__ __launch_bounds__(kThreads) void gather_rows_kernel(const uint16_t* __restrict__ src, uint32_t ld, const uint32_t* __restrict__ rows_of,
+                                                               const uint32_t* __restrict__ jobs, uint16_t* __restrict__ dst) {
+    const uint32_t slot0 = blockIdx.x * 16u, lane = threadIdx.x & 63u;
+    if (slot0 >= jobs[1]) return;
+    const uint16_t* from = src + (size_t)rows_of[slot0 + (lane & 15u)] * ld + (lane >> 4) * 8u;
+    uint16_t* to = dst + (size_t)slot0 * ld + lane * 8u;
+    for (uint32_t k = threadIdx.x >> 6; k < ld / 32u; k += kWaves)
+        *reinterpret_cast<uint4*>(to + (size_t)k * kM40Tile) = *reinterpret_cast<const uint4*>(from + (size_t)k * 32u);
+}
+
 template <uint32_t N>
 void launch_route(hipStream_t stream, const M40llmRoute& r) {
     if (r.rows <= 64u && r.rows * r.top <= kSmallPairs) {
@@ -236,6 +248,17 @@ int m40llm_ext_route_rows_async(M40llmCudaContext* ctx, const M40llmRoute* r, ui
     else if (all <= 128u) launch_route<2>(stream, *r);
     else if (all <= 256u) launch_route<4>(stream, *r);
     else launch_route<16>(stream, *r);
+    return hipGetLastError() == hipSuccess ? 0 : -2;
+}
+
+int m40llm_ext_gather_rows_async(M40llmCudaContext* ctx, const void* d_src_bf16, uint32_t ld, const uint32_t* d_rows_of, const uint32_t* d_jobs,
+                                 uint32_t max_slots, void* d_dst_bf16, uint32_t stream_kind) {
+    if (!ctx || !d_src_bf16 || !d_rows_of || !d_jobs || !d_dst_bf16) return -1;
+    hipStream_t stream = m40_select_stream(ctx, stream_kind);
+    if (!stream || m40_ensure_device(ctx) != 0) return -2;
+    if (ld == 0 || ld % 32u != 0 || max_slots == 0 || max_slots % 16u != 0 || !m40_aligned16(d_src_bf16) || !m40_aligned16(d_dst_bf16)) return -3;
+    gather_rows_kernel<<<max_slots / 16u, kThreads, 0, stream>>>(static_cast<const uint16_t*>(d_src_bf16), ld, d_rows_of, d_jobs,
+                                                                static_cast<uint16_t*>(d_dst_bf16));
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
 

@@ -9,7 +9,7 @@
 //                      operands in instruction order, so LDS reads are contiguous kilobytes as well.
 //
 // Products per expert: both kernels take a list of jobs (expert, rows of the list sorted by expert) made on the device; the rows are
-// gathered from plain rows (gate and up) or lie packed in list order (down).
+// gathered from plain rows (few rows, gate and up) or lie packed in list order.
 #include "packed_gemm.hpp"
 
 #include <type_traits>
@@ -160,7 +160,7 @@ int launch_rows_any(hipStream_t stream, const PackedArgs& g, const M40Epilogue<T
 // ahead go out one at a time between the current step's products (sched_group_barrier), so that no wave waits for an address
 // or LDS unit with the matrix pipe idle.  Step t refills the buffer of step t - 1, whose fragments every wave had in registers
 // before the barrier behind that step, and ends with step t + 2 landed.
-enum { kPlainRows = 0, kPageKeys = 1, kPageValues = 2, kSlots = 3, kGather = 4 };
+enum { kPlainRows = 0, kPageKeys = 1, kPageValues = 2, kSlots = 3 };
 constexpr int tile_bufs(int ntw) { return ntw == 8 ? 6 : 5; }       // one or two workgroups a CU
 
 template <int NTW, int FORM>
@@ -172,7 +172,7 @@ __global__ __launch_bounds__(256, 1) void tile_packed_kernel(PackedArgs g, M40Ep
     constexpr int kBufs = tile_bufs(NTW), kStepBytes = (kATiles + kBTiles) * 1024;
     constexpr int kLoads = (kATiles + kBTiles) / 4;                  // per wave and step
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-    constexpr bool kJobs = FORM == kSlots || FORM == kGather;
+    constexpr bool kJobs = FORM == kSlots;
     const int tiles_n = (g.n_tiles + kBTiles - 1) / kBTiles, tiles_m = kJobs ? (int)g.jobs[0] : (g.rows + 127) / 128;
     const int workgroups = kJobs ? tiles_m * tiles_n : (int)gridDim.x;       // the grid is as large as the list of jobs can be
     if (kJobs && (int)blockIdx.x >= workgroups) return;
@@ -202,9 +202,8 @@ __global__ __launch_bounds__(256, 1) void tile_packed_kernel(PackedArgs g, M40Ep
                 const int rt = m0 / 16 + t, tiles = g.rows / 16, c = rt < tiles ? rt : tiles - 1;
                 src[i] = A + ((long)g.pages[c >> 2] * 4 + (c & 3)) * g.page_k_tiles * kM40Tile + lane * 8;
             } else {
-                const int rt = m0 / 16 + t, last = (g.rows - 1) / 16, c = rt < last ? rt : last;
-                if (FORM == kGather) src[i] = A + (long)g.gather[c * 16 + (lane & 15)] * g.lda + (lane >> 4) * 8;
-                else src[i] = A + (long)c * 16 * g.lda + lane * 8;
+                const int rt = m0 / 16 + t, last = (g.rows - 1) / 16;
+                src[i] = A + (long)(rt < last ? rt : last) * 16 * g.lda + lane * 8;
             }
         } else {
             const int n = t0 + t - kATiles;
@@ -216,7 +215,7 @@ __global__ __launch_bounds__(256, 1) void tile_packed_kernel(PackedArgs g, M40Ep
         const int k = t < k_tiles ? t : k_tiles - 1;                 // past the end: loaded again, not used
 #pragma unroll
         for (int i = 0; i < kLoads; ++i)
-            __builtin_amdgcn_global_load_lds((global_src_t)(src[i] + (long)k * (FORM == kGather && i < kATiles / 4 ? 32 : kM40Tile)), (lds_dst_t)(base + i * 4096), 16, 0, 0);
+            __builtin_amdgcn_global_load_lds((global_src_t)(src[i] + (long)k * kM40Tile), (lds_dst_t)(base + i * 4096), 16, 0, 0);
     };
     const int wm = wave >> 1, wn = wave & 1;
     m40_float4 acc[4][NTW];
@@ -325,16 +324,16 @@ int launch_tile(hipStream_t stream, const PackedArgs& g, const M40Epilogue<m40_b
     static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(tile_packed_kernel<NTW, FORM>),
                                                        hipFuncAttributeMaxDynamicSharedMemorySize, lds);
     if (attr != hipSuccess) return -2;
-    constexpr bool kJobs = FORM == kSlots || FORM == kGather;        // g.rows: the most jobs there can be
+    constexpr bool kJobs = FORM == kSlots;        // g.rows: the most jobs there can be
     const long long tiles = (long long)(kJobs ? g.rows : (g.rows + 127) / 128) * ((g.n_tiles + 2 * NTW - 1) / (2 * NTW));
     tile_packed_kernel<NTW, FORM><<<dim3((unsigned)tiles, 1, (unsigned)batches), 256, lds, stream>>>(g, e);
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
 template <int FORM>
 int launch_tile_any(hipStream_t stream, const PackedArgs& g, const M40Epilogue<m40_bf16>& e, int batches, int num_cus) {
-    const long long wide = (long long)(FORM == kSlots || FORM == kGather ? g.rows : (g.rows + 127) / 128) * ((g.n_tiles + 15) / 16) * batches;
+    const long long wide = (long long)(FORM == kSlots ? g.rows : (g.rows + 127) / 128) * ((g.n_tiles + 15) / 16) * batches;
     // a short sum is mostly a workgroup's start and end: two narrower workgroups a CU cover each other's
-    if (wide * 16 >= 9ll * num_cus && g.k_tiles > (FORM == kSlots ? 64 : 32)) return launch_tile<8, FORM>(stream, g, e, batches);
+    if (wide * 16 >= 9ll * num_cus && g.k_tiles > (FORM == kSlots && e.kind == M40LLM_PACKED_STORE_ACT ? 64 : 32)) return launch_tile<8, FORM>(stream, g, e, batches);
     return launch_tile<4, FORM>(stream, g, e, batches);
 }
 
@@ -444,7 +443,8 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
         return -3;
     if (p->jobs && (p->batches != 1u || k_parts > 1u || p->max_jobs == 0 || p->max_jobs > 65535u || (p->job_rows != 16u && p->job_rows != 32u && p->job_rows != 64u && p->job_rows != 128u) ||
                     (p->job_rows == 128u && p->act_dtype == M40LLM_ACT_F32) || p->w_batch % 8 != 0 ||
-                    (p->gather ? p->epilogue != M40LLM_PACKED_PROJECT || p->plain_tiles != 0 : p->epilogue != M40LLM_PACKED_STORE_ACT)))
+                    !(p->epilogue == M40LLM_PACKED_STORE_ACT ? !p->gather
+                                                                  : p->epilogue == M40LLM_PACKED_PROJECT && p->plain_tiles == 0 && (p->job_rows == 128u) == !p->gather)))
         return -3;
     if (!paged && (p->lda % 32 != 0 || p->lda < (uint64_t)p->k_tiles * 32u)) return -3;
     if (k_parts > 1u && (p->epilogue != M40LLM_PACKED_STORE || p->batches != 1u || (k_parts - 1) * part_tiles >= p->k_tiles)) return -3;
@@ -502,7 +502,7 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
             return p->gather ? launch_rows_any<float, kJobGather>(stream, g, e, 1, rows) : launch_rows_any<float, kJobSlots>(stream, g, e, 1, rows);
         }
         const M40Epilogue<m40_bf16> e = make_epilogue<m40_bf16>(*p);
-        if (rows == 128) return p->gather ? launch_tile_any<kGather>(stream, g, e, 1, ctx->num_cus) : launch_tile_any<kSlots>(stream, g, e, 1, ctx->num_cus);
+        if (rows == 128) return launch_tile_any<kSlots>(stream, g, e, 1, ctx->num_cus);
         return p->gather ? launch_rows_any<m40_bf16, kJobGather>(stream, g, e, 1, rows) : launch_rows_any<m40_bf16, kJobSlots>(stream, g, e, 1, rows);
     }
     if (p->act_dtype == M40LLM_ACT_F32) {

@@ -243,7 +243,7 @@ private:
         auto light = std::make_shared<LightningShared>();
         auto expert = std::make_shared<ExpertShared>();
         rt_.scratch.insert(rt_.scratch.end(), {&pair->queries, &light->qkv, &light->o, &expert->logits, &expert->ids, &expert->weight, &expert->rows_of,
-                                               &expert->place, &expert->jobs, &expert->act, &expert->out});
+                                               &expert->place, &expert->jobs, &expert->rows, &expert->act, &expert->out});
         shared_ = {pair, light, expert};
         std::vector<DifferentialMixer*> made;
         for (const LayerSpec& s : spec_.layers) {

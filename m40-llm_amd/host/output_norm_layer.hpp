@@ -320,9 +320,10 @@ private:
     DeviceBuf w_in_, w_out_;
 };
 
-struct ExpertShared { Scratch logits, ids, weight, rows_of, place, jobs, act, out; };
+struct ExpertShared { Scratch logits, ids, weight, rows_of, place, jobs, rows, act, out; };
 
-// Launches: product (router logits) | choice and sorted list (two launches above 64 rows) | gate and up per expert | down per expert
+// Launches: product (router logits) | choice and sorted list (two launches above 64 rows) | (many rows: rows in list order) | gate and up per
+// expert | down per expert
 class ExpertFeedForward : public FeedForward {
 public:
     ExpertFeedForward(LayerRuntime& rt, std::shared_ptr<ExpertShared> shared, TensorSource& t, uint32_t index, const ExpertMlpSpec& m)
@@ -355,6 +356,7 @@ public:
         sh_->place.want((size_t)R * m.top * 4);
         sh_->rows_of.want((size_t)slots * 4);
         sh_->jobs.want(16 + (size_t)m40llm_ext_expert_max_jobs(R, m.experts, m.top, 16) * 16);
+        if (rt.bf16() && rows_a_job(R) == 128) sh_->rows.want((size_t)slots * rt.d_pad * rt.es);
         sh_->act.want((size_t)slots * pad_ * rt.es);
         sh_->out.want((size_t)slots * out_cols_ * rt.es);
     }
@@ -378,7 +380,14 @@ public:
         {
             M40llmPackedGemm g = rt_.product(rt_.h_rows.ptr(), rt_.d_pad, w_in_, 2 * tiles_, d_tiles, r.rows, M40LLM_PACKED_PROJECT);
             g.activation = activation_code(m_.activation);
-            g.jobs = sh_->jobs.u32(); g.gather = sh_->rows_of.u32(); g.max_jobs = max_jobs; g.job_rows = job_rows;
+            if (job_rows == 128) {
+                M40H_TRY(m40llm_ext_gather_rows_async(rt_.ctx, rt_.h_rows.ptr(), rt_.d_pad, sh_->rows_of.u32(), sh_->jobs.u32(),
+                                                      m40llm_ext_expert_slots(r.rows, m_.experts, m_.top), sh_->rows.ptr(), rt_.kStream));
+                g.a = sh_->rows.ptr();
+            } else {
+                g.gather = sh_->rows_of.u32();
+            }
+            g.jobs = sh_->jobs.u32(); g.max_jobs = max_jobs; g.job_rows = job_rows;
             g.w_batch = (uint64_t)2 * tiles_ * d_tiles * 512;
             g.out_act = sh_->act.ptr(); g.ld_act = pad_;
             rt_.launch(g);
