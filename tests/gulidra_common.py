@@ -62,6 +62,32 @@ def config_one():
 CONFIGS = dict(odd=config_odd, even=config_even, wide=config_wide, one=config_one)
 
 
+def random_config(seed):
+    """Layers of any kind in any order, sizes of any kind; readers of any earlier layer's keys.  The embedding outweighs what layers add, so
+    that rounding where two maps nearly cancel stays small."""
+    rng = np.random.default_rng(seed)
+
+    def one(*of):
+        return of[int(rng.integers(len(of)))]
+    layers, own = [], []
+    for i in range(int(rng.integers(2, 6))):
+        kind = one("own", "own", "reader", "lightning")
+        if kind == "lightning":
+            H = int(rng.integers(1, 7))
+            l = lightning(H, one(8, 16, 24, 32, 48, 64, 100), one(8, 16, 24, 32, 48, 72, 128), 1 - 2.0 ** -rng.uniform(0.5, 11, size=H))
+        elif kind == "reader" and own:
+            j = one(*own)
+            m = layers[j][0]["mixer"]
+            l = attention(m["kv_heads"] * one(1, 2, 3), m["kv_heads"], m["dim"], m["vdim"], one(1, 2, 3, 4), float(rng.uniform(0, 0.9)), kv_from=j)
+        else:
+            G = one(1, 2, 3, 4)
+            l = attention(G * one(1, 2, 4, 17), G, one(8, 16, 24, 32, 48, 64, 96, 128), one(16, 32, 40, 64, 96, 128), one(None, 1, 2, 3, 4, 6), float(rng.uniform(0, 0.9)))
+            own.append(i)
+        E = one(2, 4, 6, 12, 24)
+        layers.append((l, one(None, dense(one(30, 64, 200)), experts(E, one(0, 1, 3), int(rng.integers(1, min(E, 5) + 1)), one(16, 40, 64)))))
+    return model(one(64, 150, 257), one(48, 100, 128, 192), layers, eps=one(1e-6, 1e-5, 1e-3), scale=one(4.0, 8.0, 15.0), mult=one(0.3, 0.7, 1.0), positions=150)
+
+
 def random_tensors(cfg, seed=0):
     rng = np.random.default_rng(seed)
     T, D = {}, cfg["width"]
@@ -120,4 +146,4 @@ def make_folder(path, name, seed=3):
     return write_folder(path, cfg, random_tensors(cfg, seed))
 
 
-__all__ = ["CONFIGS", "od", "random_tensors", "make_folder", "write_folder"]
+__all__ = ["CONFIGS", "od", "random_config", "random_tensors", "make_folder", "write_folder"]
