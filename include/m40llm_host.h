@@ -174,7 +174,7 @@ typedef struct M40HostModelOptions {
     uint32_t max_tokens;       /* what the cache pool holds, rounded up to whole pages of 64; 0 = 4096 */
     uint32_t max_sequences;    /* 0 = 4 */
     uint32_t max_rows;         /* rows of one pass (longer steps run in several); 0 = 4096 */
-    uint32_t portion_form;     /* attention of portions: 0 the cheaper form, 1 in latent space, 2 head by head where it is served */
+    uint32_t portion_form;     /* attention of portions: 0 the cheaper form, 1 that of single tokens, 2 that of long portions where it is served */
 } M40HostModelOptions;
 typedef struct M40HostStepEntry {
     uint32_t sequence_id, n_tokens, n_want;
