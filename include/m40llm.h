@@ -569,6 +569,7 @@ int m40llm_ext_clear_u32_async(M40llmCudaContext* ctx, void* d_dst, size_t n, ui
 #define M40LLM_PACKED_KEYS 6u
 #define M40LLM_PACKED_VALUES 7u
 #define M40LLM_PACKED_SILU 8u       /* the first plain_tiles tiles: as STORE; then out_act[row][act_col + col] = silu(v), packed */
+#define M40LLM_PACKED_SPLIT 9u      /* the same without silu */
 #define M40LLM_GELU_TANH 0u
 #define M40LLM_SILU 1u
 typedef struct M40llmPackedGemm {
@@ -665,15 +666,17 @@ int m40llm_ext_norm_gate_rows_async(M40llmCudaContext* ctx, const void* d_y, uin
 
 /* ---- routed feed-forwards ------------------------------------------------------------------------------------------------------
  * Of `experts` + `identity` experts each row takes the `top` with the largest softmax(logits) + correction (the lower index of equals);
- * its weights are the softmax values.  ids / weight: [rows][top].  Then rows are sorted by expert: every expert's rows, in order, take
+ * its weights are the softmax values times scale.  groups > 1: experts form that many groups of neighbours, and only those of the `keep` groups
+ * with the largest choice can be taken.  ids / weight: [rows][top].  Then rows are sorted by expert: every expert's rows, in order, take
  * slots from a multiple of 16 on; rows_of[slot] = row (slots that pad a group of 16 repeat a row), place[row*top + j] = slot, or
  * M40LLM_PLACE_INPUT for identity experts; jobs (m40llm_ext_packed_gemm_async) of at most job_rows slots; jobs[1] = slots in use.  rows_of holds
  * m40llm_ext_expert_slots, jobs 4 + 4 * m40llm_ext_expert_max_jobs words. */
 typedef struct M40llmRoute {
-    uint32_t rows, experts, identity, top, job_rows;
+    uint32_t rows, experts, identity, top, job_rows, groups, keep;
+    float scale;
     const void* logits;              /* f32 [rows][ld_logits] */
     uint64_t ld_logits;
-    const void* correction;          /* f32 [experts + identity] */
+    const void* correction;          /* f32 [experts + identity], NULL = none */
     uint32_t* ids;
     void* weight;                    /* f32 */
     uint32_t *rows_of, *place, *jobs;
@@ -686,13 +689,14 @@ uint32_t m40llm_ext_expert_slots(uint32_t rows, uint32_t experts, uint32_t top);
 uint32_t m40llm_ext_expert_max_jobs(uint32_t rows, uint32_t experts, uint32_t top, uint32_t job_rows);
 #define M40LLM_MAX_EXPERTS 1024u
 
-/* ---- differential attention over a paged cache of keys and values ----------------------------------------------------------
- * Every head has two maps: softmaxes of their own queries and keys over the same values, a1 and a2; o = a1 - lambda*a2, then
+/* ---- attention over a paged cache of keys and values, one or two maps a head -------------------------------------------------
+ * One map (maps = 1): softmax attention, its result times out_scale and, where gate is not NULL, times sigmoid(gate[row][head*vdim + d]).
+ * Two maps, differential attention: softmaxes of their own queries and keys over the same values, a1 and a2; o = a1 - lambda*a2, then
  * o / sqrt(mean(o^2) + eps) * out_scale * sigmoid(gate[row][head]).  Query head h uses kv head h / (heads / kv_heads).
- * A page holds 64 tokens; per kv head first the keys, map after map, as packed rows (4 x k_tiles tiles of 16 tokens x 32 dimensions),
+ * A page holds 64 tokens; per kv head first the keys, map after map (`maps` of them), as packed rows (4 x k_tiles tiles of 16 tokens x 32 dimensions),
  * then the values transposed: per 16 dimensions two tiles [16 dimensions][32 tokens], token 16t + 4g + r at place 8g + 4t + r.
  * k_tiles = dim/32, v_tiles = vdim/16, rounded up; page p starts at element p * m40llm_ext_pair_page_elements. */
-uint64_t m40llm_ext_pair_page_elements(uint32_t kv_heads, uint32_t dim, uint32_t vdim);
+uint64_t m40llm_ext_pair_page_elements(uint32_t maps, uint32_t kv_heads, uint32_t dim, uint32_t vdim);
 /* From projected rows (f32: heads of [map 1 | map 2] query columns, the same for keys, value columns): causal convolution of `taps` taps
  * on every column (0 = none), RMS norm over each map's dim of queries and keys; queries out as plain rows [heads][2][32*k_tiles], keys and
  * values to the row's place in the cache (cache NULL = the layer reads another layer's: no key and value columns).
@@ -724,7 +728,7 @@ int m40llm_ext_conv_state_async(M40llmCudaContext* ctx, const void* d_proj, uint
  * m40llm_ext_pair_attention_partial_floats; rows first_row .. first_row + n_rows are joined by a second launch); form 1: at most tile_queries
  * (64 or 128) queries a tile, operands through LDS; f32 takes rows one by one (tiles are not used).  out packed [rows][ld_out]. */
 typedef struct M40llmPairAttention {
-    uint32_t act_dtype, form, heads, kv_heads, dim, vdim;
+    uint32_t act_dtype, form, maps, heads, kv_heads, dim, vdim;
     float scale, lambda, out_scale, eps;
     const void* queries;
     const void* cache;
@@ -740,9 +744,9 @@ typedef struct M40llmPairAttention {
     uint32_t ld_out;
 } M40llmPairAttention;
 int m40llm_ext_pair_attention_async(M40llmCudaContext* ctx, const M40llmPairAttention* a, uint32_t stream_kind);
-uint64_t m40llm_ext_pair_attention_partial_floats(uint32_t rows, uint32_t heads, uint32_t vdim, uint32_t splits);
+uint64_t m40llm_ext_pair_attention_partial_floats(uint32_t maps, uint32_t rows, uint32_t heads, uint32_t vdim, uint32_t splits);
 /* most queries of a tile: 128 or 64 where form 1 is served, 16 where only form 0 is, 0 = sizes that are not served */
-uint32_t m40llm_ext_pair_attention_tile_queries(uint32_t act_dtype, uint32_t dim, uint32_t vdim);
+uint32_t m40llm_ext_pair_attention_tile_queries(uint32_t act_dtype, uint32_t maps, uint32_t dim, uint32_t vdim);
 
 /* ---- lightning attention -----------------------------------------------------------------------------------------------------------
  * Per head S <- decay*S + k v^T, o = S^T q, token by token; S in f32, state[slot][head][dim][32*ceil(vdim/32)], zero before position 0.
@@ -768,6 +772,127 @@ int m40llm_ext_lightning_async(M40llmCudaContext* ctx, const M40llmLightning* l,
 uint64_t m40llm_ext_lightning_scratch_bytes(uint32_t n_chunks, uint32_t heads, uint32_t dim, uint32_t vdim);
 /* whether heads of these sizes are served */
 int m40llm_ext_lightning_serves(uint32_t dim, uint32_t vdim);
+
+/* ---- residual streams ------------------------------------------------------------------------------------------------------------------
+ * x_t <- sum_s mix[s][t] x_s + mult*share[t]*y for all streams at once, then u = sum_t take[t] x_t (take NULL = ones).  x_s: f32 rows of `width`,
+ * stream s at streams_x + s*stream_stride; with x0 every stream holds the row of x0 so far.  y: the sum of n_planes planes or the experts' rows,
+ * as in M40llmNormAdd; neither (n_planes 0, place NULL) = the streams stay as they are.  With w, u / sqrt(mean(u^2) + eps) * w goes to h (packed,
+ * ld_h columns, zero past width) and, where it is not NULL, to plain rows h_rows; without, u goes to x_out.
+ * row_index (may be NULL): only these rows, `rows` of them; discard: the streams' new values are not kept. */
+#define M40LLM_MOST_STREAMS 16u
+typedef struct M40llmStreamUpdate {
+    uint32_t act_dtype, rows, width, streams, discard;
+    float eps, mult;
+    const void* x0;
+    void* streams_x;
+    uint64_t stream_stride;
+    const void *mix, *share, *take;  /* f32 [streams][streams], [streams], [streams] */
+    const void* planes;
+    uint32_t n_planes, top;
+    uint64_t plane_stride;
+    const void* expert_out;
+    uint64_t ld_expert;
+    const uint32_t* place;
+    const void* weight;
+    const void* w;
+    void *h, *h_rows, *x_out;
+    uint32_t ld_h;
+    const uint32_t* row_index;
+} M40llmStreamUpdate;
+int m40llm_ext_stream_update_async(M40llmCudaContext* ctx, const M40llmStreamUpdate* u, uint32_t stream_kind);
+
+/* ---- attention of one map a head: from projections to queries and cache ----------------------------------------------------------
+ * From projected rows (f32: query heads from column 0, key heads from k_offset, value heads from v_offset): biases (f32, may be NULL), RMS norm over
+ * all query and over all key columns (q_norm [heads*dim], k_norm [kv_heads*dim], both or neither), rotation of the first 2*rot_half dimensions of
+ * every query and key head in pairs (2i, 2i+1) by angles[row][rot_half] (may be NULL), queries times q_factor.  Values: keep_values takes them (f32
+ * [row][ld_values]); with first_values (laid out the same) v <- (1 - lambda) v + lambda first.  Queries out as plain rows [heads][32*k_tiles], keys and
+ * values to the row's place in a cache of one map. */
+typedef struct M40llmQkvSplit {
+    uint32_t act_dtype, rows, heads, kv_heads, dim, vdim;
+    float eps, q_factor, lambda;
+    const void* proj;
+    uint64_t ld_proj;
+    uint32_t k_offset, v_offset;
+    const void *q_bias, *k_bias, *v_bias, *q_norm, *k_norm;
+    const void* angles;
+    uint32_t rot_half;
+    const void* first_values;
+    void* keep_values;
+    uint64_t ld_values;
+    void* queries;
+    void* cache;
+    const uint32_t *row_slot, *row_pos, *page_table;
+    uint32_t max_pages;
+} M40llmQkvSplit;
+int m40llm_ext_qkv_split_append_async(M40llmCudaContext* ctx, const M40llmQkvSplit* s, uint32_t stream_kind);
+
+/* ---- recurrent layers with a matrix state --------------------------------------------------------------------------------------------
+ * All in f32, token by token, zero before position 0.  out: packed rows of the activation type, ld_out columns, head h at
+ * out_col + h*vdim: o / sqrt(mean(o^2) + eps) * norm * sigmoid(gate) * out_factor.  portions[p] = {first row, rows, slot, 0}; chunk_base, chunks as in
+ * M40llmLightning; chunked (bf16): a few launches over all chunks instead of token after token; scratch: m40llm_ext_memory_scratch_bytes.
+ *
+ * Matrix memory: log gates i = cap*tanh((zi + i_bias)/cap), f = logsigmoid(cap*tanh((zf + f_bias)/cap)); m' = max(f + m, i); S <- exp(f + m - m') S +
+ * exp(i - m') k v^T, n likewise with k alone; o = S^T q / (max(|n . q|, exp(-m')) + 1e-6), q times q_factor.  proj: f32 rows with query, key, value
+ * and gate columns of all heads, gate logits i and f; norm [heads*vdim]. */
+typedef struct M40llmMatrixMemory {
+    uint32_t act_dtype, chunked, heads, dim, vdim;
+    float cap, q_factor, eps, out_factor;
+    const void* proj;
+    uint64_t ld_proj;
+    uint32_t q_col, k_col, v_col, g_col, i_col, f_col;
+    const void *i_bias, *f_bias, *norm;
+    void* state;                     /* f32 [slot][heads][m40llm_ext_matrix_memory_state_floats]: S [dim][4*ceil(vdim/4)], n, m */
+    void* out;
+    uint32_t ld_out, out_col;
+    const uint32_t *portions, *chunk_base, *chunks, *row_pos;
+    uint32_t n_portions, n_chunks;
+    void* scratch;
+    uint64_t scratch_bytes;
+} M40llmMatrixMemory;
+int m40llm_ext_matrix_memory_async(M40llmCudaContext* ctx, const M40llmMatrixMemory* m, uint32_t stream_kind);
+uint64_t m40llm_ext_matrix_memory_state_floats(uint32_t dim, uint32_t vdim);
+
+/* Delta rule with one decay per head and key channel: g = exp(-exp(A_log) softplus(za + dt_bias)), b = sigmoid(zb); S <- g S (row by row);
+ * u = b (v - S^T k); S <- S + k u^T; o = S^T q.  Head h uses query / key head h / (heads / kv_heads).
+ * First the split: from projected rows (f32: query heads, key heads, value heads) causal convolutions (M40llmPairSplit has conv_state, row_back and
+ * what follows for longer portions), silu, queries and keys x / sqrt(sum x^2 + 1e-6), queries times q_factor; out f32 rows of the same columns. */
+typedef struct M40llmDeltaSplit {
+    uint32_t rows, heads, kv_heads, dim, vdim, taps;
+    float q_factor;
+    const void* proj;
+    uint64_t ld_proj;
+    const void *q_conv, *k_conv, *v_conv;
+    void* conv_state;
+    uint64_t ld_state;
+    void* out;
+    uint64_t ld_out;
+    const uint32_t *row_slot, *row_pos, *row_back;
+} M40llmDeltaSplit;
+int m40llm_ext_delta_split_async(M40llmCudaContext* ctx, const M40llmDeltaSplit* s, uint32_t stream_kind);
+typedef struct M40llmChannelDelta {
+    uint32_t act_dtype, chunked, heads, kv_heads, dim, vdim;
+    float q_factor, eps, out_factor;
+    const void* qkv;                 /* f32 rows of the split */
+    uint64_t ld_qkv;
+    const void* low;                 /* f32 rows: decay logits [heads*dim] from a_col on, gate logits [heads*vdim] from g_col on */
+    uint64_t ld_low;
+    uint32_t a_col, g_col;
+    const void* beta;                /* f32 rows of write strength logits [heads] */
+    uint64_t ld_beta;
+    const void *A_log, *dt_bias, *norm;      /* f32 [heads], [heads*dim], [vdim] */
+    void* state;                     /* f32 [slot][heads][m40llm_ext_channel_delta_state_floats]: S [dim][4*ceil(vdim/4)] */
+    void* out;
+    uint32_t ld_out, out_col;
+    const uint32_t *portions, *chunk_base, *chunks, *row_pos;
+    uint32_t n_portions, n_chunks;
+    void* scratch;
+    uint64_t scratch_bytes;
+} M40llmChannelDelta;
+int m40llm_ext_channel_delta_async(M40llmCudaContext* ctx, const M40llmChannelDelta* m, uint32_t stream_kind);
+uint64_t m40llm_ext_channel_delta_state_floats(uint32_t dim, uint32_t vdim);
+uint64_t m40llm_ext_memory_scratch_bytes(uint32_t delta, uint32_t n_chunks, uint32_t heads, uint32_t dim, uint32_t vdim);
+/* whether heads of these sizes are served */
+int m40llm_ext_memory_serves(uint32_t dim, uint32_t vdim);
 
 /* ---- latent attention over a paged cache ------------------------------------------------------------------------------------
  * A page holds 64 tokens; a token's entry is its normed latent (kv_rank, padded to a multiple of 32) followed by the rotated

@@ -9,6 +9,36 @@ constexpr uint32_t kListThreads = 1024, kListWaves = kListThreads / 64;
 constexpr uint32_t kMost = M40LLM_MAX_EXPERTS;
 constexpr uint32_t kSmallPairs = 4096;     // (row, choice) pairs one workgroup keeps in LDS
 
+// Experts in groups of `size` neighbours: what is left of `left` when only the `keep` groups whose best choice is largest (the lower group of
+// equals) can be chosen from.
+template <uint32_t N>
+__device__ __forceinline__ uint32_t within_groups(const M40llmRoute& a, uint32_t lane, uint32_t size, const float (&choice)[N], uint32_t left) {
+    uint32_t kept = 0, open = left;          // bit i: this lane's expert i is in a group that is taken, in one that still can be
+    for (uint32_t k = 0; k < a.keep; ++k) {
+        float best = -INFINITY;
+#pragma unroll
+        for (uint32_t i = 0; i < N; ++i) best = open >> i & 1u ? fmaxf(best, choice[i]) : best;
+        best = m40_max64(best);
+        uint32_t at = 0xffffffffu;           // its lowest expert (of one that is no number: the lowest that is open)
+#pragma unroll
+        for (uint32_t any = 0; any < 2u; ++any)
+#pragma unroll
+            for (uint32_t i = 0; i < N; ++i) {
+                const unsigned long long hit = __ballot((open >> i & 1u) && (any || choice[i] == best));
+                if (at == 0xffffffffu && hit) at = (uint32_t)__ffsll(hit) - 1u + 64u * i;
+            }
+        if (at == 0xffffffffu) break;
+        const uint32_t group = at / size;
+#pragma unroll
+        for (uint32_t i = 0; i < N; ++i)
+            if ((left >> i & 1u) && (lane + 64u * i) / size == group) {
+                kept |= 1u << i;
+                open &= ~(1u << i);
+            }
+    }
+    return kept;
+}
+
 // A wave routes one row: lane l holds experts l, l + 64, ..., N of them.
 template <uint32_t N>
 __device__ __forceinline__ void route_row(const M40llmRoute& a, uint32_t row, uint32_t lane, uint32_t* ids, float* weight) {
@@ -21,7 +51,7 @@ __device__ __forceinline__ void route_row(const M40llmRoute& a, uint32_t row, ui
     for (uint32_t i = 0; i < N; ++i) {
         const uint32_t e = lane + 64u * i;
         s[i] = e < n ? z[e] : -INFINITY;
-        choice[i] = e < n ? correction[e] : 0.0f;
+        choice[i] = correction && e < n ? correction[e] : 0.0f;
         top = fmaxf(top, s[i]);
     }
     top = m40_max64(top);
@@ -40,6 +70,7 @@ __device__ __forceinline__ void route_row(const M40llmRoute& a, uint32_t row, ui
         choice[i] += s[i];
         if (e < n) left |= 1u << i;
     }
+    if (a.groups > 1u) left = within_groups<N>(a, lane, n / a.groups, choice, left);
     uint32_t mine_id = 0;
     float mine_weight = 0.0f;                // choice `lane`
     for (uint32_t j = 0; j < a.top; ++j) {
@@ -79,7 +110,7 @@ __device__ __forceinline__ void route_row(const M40llmRoute& a, uint32_t row, ui
             const uint32_t first = j & ~63u;
             if (first + lane <= j) {
                 ids[first + lane] = mine_id;
-                weight[first + lane] = mine_weight;
+                weight[first + lane] = mine_weight * a.scale;
             }
         }
     }
@@ -235,15 +266,16 @@ uint32_t m40llm_ext_expert_max_jobs(uint32_t rows, uint32_t experts, uint32_t to
 }
 
 int m40llm_ext_route_rows_async(M40llmCudaContext* ctx, const M40llmRoute* r, uint32_t stream_kind) {
-    if (!ctx || !r || !r->logits || !r->correction || !r->ids || !r->weight || !r->rows_of || !r->place || !r->jobs) return -1;
+    if (!ctx || !r || !r->logits || !r->ids || !r->weight || !r->rows_of || !r->place || !r->jobs) return -1;
     hipStream_t stream = m40_select_stream(ctx, stream_kind);
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
     if (r->rows == 0 || r->experts == 0 || r->experts + r->identity > kMost || r->top == 0 || r->top > r->experts + r->identity ||
         r->ld_logits < r->experts + r->identity || (r->job_rows != 16u && r->job_rows != 32u && r->job_rows != 64u && r->job_rows != 128u) ||
         !m40_aligned16(r->ids) || m40llm_ext_expert_slots(r->rows, r->experts, r->top) == 0 || m40llm_ext_expert_max_jobs(r->rows, r->experts, r->top, r->job_rows) == 0)
         return -3;
-    (void)hipGetLastError();
     const uint32_t all = r->experts + r->identity;
+    if (r->groups > 1u && (all % r->groups != 0 || r->keep == 0 || r->keep > r->groups || r->top > r->keep * (all / r->groups))) return -3;
+    (void)hipGetLastError();
     if (all <= 64u) launch_route<1>(stream, *r);
     else if (all <= 128u) launch_route<2>(stream, *r);
     else if (all <= 256u) launch_route<4>(stream, *r);

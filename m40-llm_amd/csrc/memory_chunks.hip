@@ -1,0 +1,661 @@
+// Recurrent layers with a matrix state, many tokens at once, all in f32 matrix instructions.  A portion is cut at the step's rows that are
+// multiples of 64; within a chunk of up to 64 tokens the recurrence is written out:
+//
+//   S_t = decay_t S_0 + sum_{j <= t} (k_j, decayed from j to t) u_j^T
+//   o_t = (q_t, decayed from the chunk's start)^T S_0 + sum_{j <= t} P[t, j] u_j      P[t, j] = q_t . (k_j, decayed from j to t)
+//
+// Matrix memory: u is the values with a column of ones, whose sums are n; decays are exp of sums of log gates less the running maximum, so no
+// exponent is above zero.  Delta rule: u_t = beta_t (v_t - read_t) depends on the u before it; with A[t, j] = beta_t k_t . (k_j, decayed), j < t,
+// (I + A) u = beta (v - (k, decayed from the start)^T S_0), a triangular system whose solution is U_0 - W S_0.
+//
+// memory_scan_kernel      matrix memory: sums of log gates, the running maximum
+// memory_prepare_kernel   matrix memory: P, decayed queries and keys of all chunks
+// delta_prepare_kernel    delta rule: the same, and the solution of the triangular system.  Decays between two tokens are never formed as
+//                         a quotient: tokens of 16-row blocks meet as a product of the row's decay since its block began and the other's to the
+//                         end of its block (both at most one), tokens of one block pairwise.
+// memory_walk_kernel      chunk after chunk: a workgroup holds 16 value columns of a head's state, leaves them as they are before each chunk
+// memory_outputs_kernel   all chunks at once: outputs, the head's norm, the gate
+//
+// Operands: lane l = 16 g + i of a 16x16x4 f32 instruction holds element (i, g) of either operand and elements (4 g + r, i) of the sums.  Four
+// instructions take k = 4 g + r in turn, so four neighbouring floats of a row are the lane's operands, and a tile of sums is, as it lies, the
+// second operand of 16 more: states and u go from sums to memory to operands in "tile order" [tile][lane][4].
+#include "memory_launch.hpp"
+
+namespace {
+
+constexpr int kChunk = 64;
+constexpr float kNever = -1e30f;
+
+struct Chunk {
+    uint32_t row0, n, slot;
+    __device__ Chunk(const M40MemoryArgs& a, uint32_t c) {
+        const uint32_t *portion = a.portions + 4 * a.chunks[2 * c], base = a.chunks[2 * c + 1], end = portion[0] + portion[1];
+        row0 = base > portion[0] ? base : portion[0];
+        n = (base + kChunk < end ? base + kChunk : end) - row0;
+        slot = portion[2];
+    }
+};
+__device__ __forceinline__ float* block_of(const M40MemoryArgs& a, uint32_t chunk, uint32_t head) { return a.scratch + ((size_t)chunk * a.heads + head) * a.block; }
+__device__ __forceinline__ m40_float4 mma4(const m40_float4& x, const m40_float4& y, m40_float4 c) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) c = __builtin_amdgcn_mfma_f32_16x16x4f32(x[r], y[r], c, 0, 0, 0);
+    return c;
+}
+__device__ __forceinline__ m40_float4 at4(const float* p) { return *reinterpret_cast<const m40_float4*>(p); }
+__device__ __forceinline__ void put4(float* p, const m40_float4& v) { *reinterpret_cast<m40_float4*>(p) = v; }
+
+// ---- matrix memory: gates.  Part `at_gate` of a block: sums of log forget gates to t [64], log input gates [64], running maxima [64], the maximum
+// before the chunk.
+__global__ __launch_bounds__(1024) void memory_scan_kernel(M40MemoryArgs a) {
+    __shared__ float total[2][16], best[2][16];
+    const uint32_t lane = threadIdx.x & 63u, wave = threadIdx.x >> 6;
+    const uint32_t *portion = a.portions + 4 * blockIdx.x, head = blockIdx.y, row0 = portion[0], end = row0 + portion[1];
+    const uint32_t first = row0 / kChunk, chunks = (end - 1u) / kChunk - first + 1u, chunk0 = a.chunk_base[blockIdx.x];
+    float* m_state = a.state + ((size_t)portion[2] * a.heads + head) * a.head_floats + (size_t)a.dim * a.v4 + a.dim4();
+    float top = a.row_pos[row0] == 0u ? 0.0f : *m_state;
+    uint32_t ph = 0;
+    for (uint32_t c0 = 0; c0 < chunks; c0 += 16u, ph ^= 1u) {
+        const uint32_t c = c0 + wave;
+        const bool live = c < chunks;
+        const uint32_t base = (first + c) * kChunk, lo = base > row0 ? base : row0, row = lo + lane;
+        const bool in = live && row < end && row < base + kChunk;
+        const float i = in ? m40_log_input_gate(a, row, head) : kNever;
+        float sum = in ? m40_log_forget_gate(a, row, head) : 0.0f;
+#pragma unroll
+        for (int d = 1; d < 64; d *= 2) {
+            const float y = __shfl_up(sum, d);
+            if ((int)lane >= d) sum += y;
+        }
+        float most = i - sum;
+#pragma unroll
+        for (int d = 1; d < 64; d *= 2) {
+            const float y = __shfl_up(most, d);
+            if ((int)lane >= d) most = fmaxf(most, y);
+        }
+        if (lane == 63u) { total[ph][wave] = sum; best[ph][wave] = most; }
+        __syncthreads();
+        float before = top;
+#pragma unroll
+        for (uint32_t w = 0; w < 16u; ++w) {
+            if (w == wave) before = top;
+            if (c0 + w < chunks) top = total[ph][w] + fmaxf(top, best[ph][w]);
+        }
+        if (live) {
+            float* gate = block_of(a, chunk0 + c, head) + a.at_gate;
+            gate[lane] = sum;
+            gate[64 + lane] = i;
+            gate[128 + lane] = sum + fmaxf(before, most);
+            if (lane == 0u) gate[192] = before;
+        }
+    }
+    if (threadIdx.x == 0u) *m_state = top;
+}
+
+// queries decayed from the start [64][dp], keys decayed to the end in tile order (key dimensions x tokens), P [64][64], values in tile order (tokens x
+// columns), what is left of S_0 per key dimension
+__global__ __launch_bounds__(256) void memory_prepare_kernel(M40MemoryArgs a) {
+    __shared__ float sum[kChunk], input[kChunk], top[kChunk];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, li = lane & 15;
+    const Chunk c(a, blockIdx.x);
+    const uint32_t head = blockIdx.y, dim = a.dim, n = c.n;
+    float* out = block_of(a, blockIdx.x, head);
+    const float* gate = out + a.at_gate;
+    if (threadIdx.x < kChunk) {
+        sum[threadIdx.x] = gate[threadIdx.x];
+        input[threadIdx.x] = gate[64 + threadIdx.x];
+        top[threadIdx.x] = gate[128 + threadIdx.x];
+    }
+    __syncthreads();
+    const float m0 = gate[192], f_end = sum[n - 1u], m_end = top[n - 1u];
+    auto row_of = [&](uint32_t t) { return (size_t)(c.row0 + (t < n ? t : n - 1u)) * a.ld; };
+    const bool vec = dim % 4u == 0 && a.ld % 4u == 0 && m40_aligned16(a.q) && m40_aligned16(a.k);
+    const float *qh = a.q + (head / a.share) * dim, *kh = a.k + (head / a.share) * dim;
+    // scores of this wave's 16 rows with the keys of blocks 0 .. wave
+    m40_float4 s[4];
+#pragma unroll
+    for (int b = 0; b < 4; ++b) s[b] = m40_float4{0.f, 0.f, 0.f, 0.f};
+    const uint32_t t = wave * 16 + li;
+    for (uint32_t d = 4u * g; d < a.dp; d += 16u) {
+        if (d - 4u * g >= dim) break;
+        const uint32_t left = d < dim ? dim - d : 0u;
+        const m40_float4 qf = m40_load4(qh + row_of(t) + d, left, vec);
+#pragma unroll
+        for (int b = 0; b < 4; ++b)
+            if (b <= wave) s[b] = mma4(m40_load4(kh + row_of(b * 16 + li) + d, left, vec), qf, s[b]);
+    }
+#pragma unroll
+    for (int b = 0; b < 4; ++b) {
+        if (b > wave) continue;
+        m40_float4 p;
+#pragma unroll
+        for (uint32_t r = 0; r < 4; ++r) {
+            const uint32_t j = b * 16 + 4 * g + r;
+            p[r] = j <= t && t < n ? s[b][r] * a.q_factor * __builtin_amdgcn_exp2f((sum[t] - sum[j] + input[j] - top[t]) * kM40Log2e) : 0.0f;
+        }
+        put4(out + a.at_p + t * kChunk + b * 16 + 4 * g, p);
+    }
+    for (uint32_t x = threadIdx.x; x < kChunk * (a.dp / 4u); x += 256u) {
+        const uint32_t tt = x / (a.dp / 4u), d = x % (a.dp / 4u) * 4u;
+        const float f = tt < n ? a.q_factor * __builtin_amdgcn_exp2f((sum[tt] + m0 - top[tt]) * kM40Log2e) : 0.0f;
+        put4(out + tt * a.dp + d, m40_load4(qh + row_of(tt) + d, d < dim ? dim - d : 0u, vec) * f);
+    }
+    for (uint32_t x = wave; x < a.dp / 16u * 4u; x += 4u) {
+        const uint32_t d = x / 4u * 16u + li;
+        m40_float4 y;
+#pragma unroll
+        for (uint32_t r = 0; r < 4; ++r) {
+            const uint32_t tt = x % 4u * 16u + 4u * g + r;
+            const float v = kh[row_of(tt) + (d < dim ? d : 0u)];
+            y[r] = tt < n && d < dim ? v * __builtin_amdgcn_exp2f((f_end - sum[tt] + input[tt] - m_end) * kM40Log2e) : 0.0f;
+        }
+        put4(out + a.at_k + (x * 64 + lane) * 4, y);
+    }
+    for (uint32_t x = wave; x < a.vt * 4u; x += 4u) {
+        const uint32_t v = x % a.vt * 16u + li;
+        m40_float4 y;
+#pragma unroll
+        for (uint32_t r = 0; r < 4; ++r) {
+            const uint32_t tt = x / a.vt * 16u + 4u * g + r;
+            const float u = a.v[row_of(tt) + head * a.vdim + (v < a.vdim ? v : 0u)];
+            y[r] = tt >= n || v > a.vdim ? 0.0f : v == a.vdim ? 1.0f : u;
+        }
+        put4(out + a.at_u + (x * 64 + lane) * 4, y);
+    }
+    if (threadIdx.x < a.dp) out[a.at_decay + threadIdx.x] = __builtin_amdgcn_exp2f((f_end + m0 - m_end) * kM40Log2e);
+}
+
+// ---- delta rule -------------------------------------------------------------------------------------------------------------------------
+constexpr int kSlab = 32, kLdSlab = 36, kLdA = 68;
+struct DeltaLds {
+    float k[kChunk][kLdSlab], q[kChunk][kLdSlab], l[kChunk][kLdSlab];          // l: log2 of the decay since the 16-row block began
+    float ke[kChunk][kLdSlab], qe[kChunk][kLdSlab], ks[kChunk][kLdSlab];       // k, q decayed since the block began; k decayed to its end
+    float whole[4][kSlab], start[4][kSlab], rest[4][kSlab];                    // of a block: its own decay, all before it, all behind it
+    float a[kChunk][kLdA];                                                     // minus A
+    float inverse[4][16][20];                                                  // of I + A's diagonal blocks
+    float beta[kChunk];
+};
+__global__ __launch_bounds__(256) void delta_prepare_kernel(M40MemoryArgs a) {
+    extern __shared__ __align__(16) uint8_t delta_lds[];
+    DeltaLds& lds = *reinterpret_cast<DeltaLds*>(delta_lds);
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, li = lane & 15;
+    const Chunk c(a, blockIdx.x);
+    const uint32_t head = blockIdx.y, dim = a.dim, n = c.n;
+    float* out = block_of(a, blockIdx.x, head);
+    float* W = out + a.at_w;
+    auto row_of = [&](uint32_t t) { return c.row0 + (t < n ? t : n - 1u); };
+    const bool vec = dim % 4u == 0 && a.ld % 4u == 0 && m40_aligned16(a.q) && m40_aligned16(a.k);
+    const float *qh = a.q + (head / a.share) * dim, *kh = a.k + (head / a.share) * dim;
+    if (tid < kChunk) lds.beta[tid] = tid < (int)n ? m40_sigmoid(a.beta[(size_t)row_of(tid) * a.ld_beta + head]) : 0.0f;
+    const float rate = -kM40Log2e * expf(a.A_log[head]);
+    float own_a[16], own_p[16];                     // rows of this wave's block with row lane / 4 of it, a quarter of the key dimensions
+#pragma unroll
+    for (int t = 0; t < 16; ++t) own_a[t] = own_p[t] = 0.0f;
+    m40_float4 off_a[3], off_p[3];                  // with the rows of the blocks before
+#pragma unroll
+    for (int b = 0; b < 3; ++b) off_a[b] = off_p[b] = m40_float4{0.f, 0.f, 0.f, 0.f};
+    const int t_in = tid >> 2, d_in = (tid & 3) * 8;
+    for (uint32_t slab = 0; slab < a.dp; slab += kSlab) {
+        {
+            const size_t row = row_of(t_in);
+            const bool live = t_in < (int)n;
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {
+                const uint32_t d = slab + d_in + 4 * h, left = live && d < dim ? dim - d : 0u;
+                const m40_float4 kk = m40_load4(kh + row * a.ld + d, left, vec), qq = m40_load4(qh + row * a.ld + d, left, vec) * a.q_factor;
+                m40_float4 l;
+#pragma unroll
+                for (uint32_t r = 0; r < 4; ++r) l[r] = r < left ? rate * m40_channel_step(a, (uint32_t)row, head, d + r) : 0.0f;
+                put4(&lds.k[t_in][d_in + 4 * h], kk);
+                put4(&lds.q[t_in][d_in + 4 * h], qq);
+                put4(&lds.l[t_in][d_in + 4 * h], l);
+            }
+        }
+        __syncthreads();
+        if (tid < 4 * kSlab) {
+            const int b = tid / kSlab, d = tid % kSlab;
+            float s = 0.0f;
+#pragma unroll
+            for (int t = 0; t < 16; ++t) {
+                s += lds.l[b * 16 + t][d];
+                lds.l[b * 16 + t][d] = s;
+            }
+            lds.whole[b][d] = s;
+        }
+        __syncthreads();
+        if (tid < 4 * kSlab) {
+            const int b = tid / kSlab, d = tid % kSlab;
+            float before = 0.0f, behind = 0.0f;
+            for (int x = 0; x < 4; ++x) {
+                if (x < b) before += lds.whole[x][d];
+                if (x > b) behind += lds.whole[x][d];
+            }
+            lds.start[b][d] = __builtin_amdgcn_exp2f(before);
+            lds.rest[b][d] = __builtin_amdgcn_exp2f(behind);
+            if (b == 3) out[a.at_decay + slab + d] = __builtin_amdgcn_exp2f(before + lds.whole[3][d]);
+        }
+        {
+            const int b = t_in >> 4;
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {
+                const int d = d_in + 4 * h;
+                const m40_float4 l = at4(&lds.l[t_in][d]), kk = at4(&lds.k[t_in][d]), qq = at4(&lds.q[t_in][d]), end = at4(&lds.whole[b][d]);
+                m40_float4 since, until;
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    since[r] = __builtin_amdgcn_exp2f(l[r]);
+                    until[r] = __builtin_amdgcn_exp2f(end[r] - l[r]);
+                }
+                put4(&lds.ke[t_in][d], kk * since);
+                put4(&lds.qe[t_in][d], qq * since);
+                put4(&lds.ks[t_in][d], kk * until);
+            }
+        }
+        __syncthreads();
+        {                                           // decayed from the start, to the end
+            const int b = t_in >> 4;
+            const float beta = lds.beta[t_in];
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {
+                const int d = d_in + 4 * h;
+                const m40_float4 f = at4(&lds.start[b][d]);
+                put4(out + t_in * a.dp + slab + d, at4(&lds.qe[t_in][d]) * f);
+                put4(W + t_in * a.dp + slab + d, at4(&lds.ke[t_in][d]) * f * beta);
+            }
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {           // block `wave` of tokens, 16 dimensions
+                const int d = h * 16 + li;
+                m40_float4 y;
+#pragma unroll
+                for (int r = 0; r < 4; ++r) y[r] = lds.ks[wave * 16 + 4 * g + r][d] * lds.rest[wave][d];
+                put4(out + a.at_k + (((slab / 16u + h) * 4u + wave) * 64 + lane) * 4, y);
+            }
+        }
+        {                                           // pairs of the block's own rows
+            const int j = lane >> 2, d = (lane & 3) * 8;
+            float kj[8], lj[8];
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {
+                const m40_float4 x = at4(&lds.k[wave * 16 + j][d + 4 * h]), y = at4(&lds.l[wave * 16 + j][d + 4 * h]);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) { kj[4 * h + r] = x[r]; lj[4 * h + r] = y[r]; }
+            }
+#pragma unroll
+            for (int t = 0; t < 16; ++t) {
+#pragma unroll
+                for (int h = 0; h < 2; ++h) {
+                    const m40_float4 kt = at4(&lds.k[wave * 16 + t][d + 4 * h]), qt = at4(&lds.q[wave * 16 + t][d + 4 * h]), lt = at4(&lds.l[wave * 16 + t][d + 4 * h]);
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) {
+                        const float e = kj[4 * h + r] * __builtin_amdgcn_exp2f(fminf(lt[r] - lj[4 * h + r], 0.0f));
+                        own_a[t] = fmaf(kt[r], e, own_a[t]);
+                        own_p[t] = fmaf(qt[r], e, own_p[t]);
+                    }
+                }
+            }
+        }
+#pragma unroll
+        for (int b = 0; b < 3; ++b) {               // with the rows of block b
+            if (b >= wave) continue;
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {
+                const int d = h * 16 + 4 * g;
+                m40_float4 f = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int x = 1; x < 3; ++x)
+                    if (x > b && x < wave) f += at4(&lds.whole[x][d]);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) f[r] = __builtin_amdgcn_exp2f(f[r]);
+                const m40_float4 j = at4(&lds.ks[b * 16 + li][d]);
+                off_a[b] = mma4(j, at4(&lds.ke[wave * 16 + li][d]) * f, off_a[b]);
+                off_p[b] = mma4(j, at4(&lds.qe[wave * 16 + li][d]) * f, off_p[b]);
+            }
+        }
+        __syncthreads();
+    }
+    {
+        const int j = lane >> 2;
+#pragma unroll
+        for (int t = 0; t < 16; ++t) {
+            float x = own_a[t], y = own_p[t];
+            x += m40_dpp_f<M40_DPP_XOR1>(x);
+            y += m40_dpp_f<M40_DPP_XOR1>(y);
+            x += m40_dpp_f<M40_DPP_XOR2>(x);
+            y += m40_dpp_f<M40_DPP_XOR2>(y);
+            if ((lane & 3) == (t & 3)) {
+                lds.a[wave * 16 + t][wave * 16 + j] = j < t ? -lds.beta[wave * 16 + t] * x : 0.0f;
+                out[a.at_p + (wave * 16 + t) * kChunk + wave * 16 + j] = j <= t ? y : 0.0f;
+            }
+        }
+        const float beta = lds.beta[wave * 16 + li];
+#pragma unroll
+        for (int b = 0; b < 3; ++b) {
+            if (b >= wave) continue;
+            put4(&lds.a[wave * 16 + li][b * 16 + 4 * g], off_a[b] * -beta);
+            put4(out + a.at_p + (wave * 16 + li) * kChunk + b * 16 + 4 * g, off_p[b]);
+        }
+    }
+    __syncthreads();
+    {                                               // column li of the inverse of I + A's block, by substitution
+        float x[16];
+#pragma unroll
+        for (int t = 0; t < 16; ++t) {
+            x[t] = t == li ? 1.0f : 0.0f;
+#pragma unroll
+            for (int j = 0; j < t; ++j) x[t] = fmaf(lds.a[wave * 16 + t][wave * 16 + j], x[j], x[t]);
+        }
+        if (g == 0) {
+#pragma unroll
+            for (int t = 0; t < 16; ++t) lds.inverse[wave][t][li] = x[t];
+        }
+    }
+    __syncthreads();
+    const uint32_t w_tiles = a.dp / 16u;
+    for (uint32_t x = wave; x < w_tiles + a.vt; x += 4u) {
+        m40_float4 X[4];
+#pragma unroll
+        for (int b = 0; b < 4; ++b) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const uint32_t t = b * 16 + 4 * g + r;
+                if (x < w_tiles) {
+                    X[b][r] = W[t * a.dp + x * 16u + li];
+                } else {
+                    const uint32_t v = (x - w_tiles) * 16u + li;
+                    const float y = a.v[(size_t)row_of(t) * a.ld + head * a.vdim + (v < a.vdim ? v : 0u)];
+                    X[b][r] = v < a.vdim && t < n ? y * lds.beta[t] : 0.0f;
+                }
+            }
+        }
+#pragma unroll
+        for (int b = 0; b < 4; ++b) {
+#pragma unroll
+            for (int j = 0; j < b; ++j) X[b] = mma4(at4(&lds.a[b * 16 + li][j * 16 + 4 * g]), X[j], X[b]);
+            X[b] = mma4(at4(&lds.inverse[b][li][4 * g]), X[b], m40_float4{0.f, 0.f, 0.f, 0.f});
+        }
+#pragma unroll
+        for (int b = 0; b < 4; ++b) {
+            if (x < w_tiles) {
+#pragma unroll
+                for (int r = 0; r < 4; ++r) W[(b * 16 + 4 * g + r) * a.dp + x * 16u + li] = X[b][r];
+            } else {
+                put4(out + a.at_u + ((b * a.vt + x - w_tiles) * 64 + lane) * 4, X[b]);
+            }
+        }
+    }
+}
+
+// ---- the walk ---------------------------------------------------------------------------------------------------------------------------
+// Wave w holds key dimensions 16 DT w .. of 16 value columns.  What a chunk needs is requested while the chunk before it is worked on.
+template <int DT, bool DELTA>
+__global__ __launch_bounds__(256) void memory_walk_kernel(M40MemoryArgs a) {
+    __shared__ m40_float4 part[DELTA ? 2 : 1][DELTA ? 4 : 1][4][64];
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, li = lane & 15;
+    const uint32_t p = blockIdx.x / a.heads, head = blockIdx.x % a.heads, V = blockIdx.y, v = V * 16u + li;
+    const uint32_t *portion = a.portions + 4 * p, row0 = portion[0], end = row0 + portion[1];
+    const uint32_t chunks = (end - 1u) / kChunk - row0 / kChunk + 1u;
+    float* state = a.state + ((size_t)portion[2] * a.heads + head) * a.head_floats;
+    float* own = state + (v < a.vdim ? v : (size_t)a.dim * a.v4);                  // column v of S; behind the last, n
+    const size_t step_d = v < a.vdim ? a.v4 : 1u;
+    const bool stored = v < a.vdim || (!DELTA && v == a.vdim), fresh = a.row_pos[row0] == 0u;
+    m40_float4 S[DT];
+#pragma unroll
+    for (int i = 0; i < DT; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const uint32_t d = (wave * DT + i) * 16 + 4 * g + r;
+            S[i][r] = stored && !fresh && d < a.dim ? own[d * step_d] : 0.0f;
+        }
+    float* block = block_of(a, a.chunk_base[p], head);
+    const size_t next = (size_t)a.heads * a.block;
+    m40_float4 wf[DELTA ? 4 : 1][DT], kf[DT][4], u[4], decay[DT];
+    auto load_w = [&](const float* b) __attribute__((always_inline)) {
+        if (!DELTA) return;
+#pragma unroll
+        for (int t = 0; t < 4; ++t)
+#pragma unroll
+            for (int i = 0; i < DT; ++i) wf[DELTA ? t : 0][i] = at4(b + a.at_w + (t * 16 + li) * a.dp + (wave * DT + i) * 16 + 4 * g);
+    };
+    auto load_u = [&](const float* b) __attribute__((always_inline)) {
+#pragma unroll
+        for (int t = 0; t < 4; ++t) u[t] = at4(b + a.at_u + ((t * a.vt + V) * 64 + lane) * 4);
+    };
+    auto load_k = [&](const float* b) __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < DT; ++i) {
+            decay[i] = at4(b + a.at_decay + (wave * DT + i) * 16 + 4 * g);
+#pragma unroll
+            for (int t = 0; t < 4; ++t) kf[i][t] = at4(b + a.at_k + (((wave * DT + i) * 4 + t) * 64 + lane) * 4);
+        }
+    };
+    load_w(block);
+    load_u(block);
+    load_k(block);
+    for (uint32_t c = 0; c < chunks; ++c) {
+        const float* ahead = c + 1u < chunks ? block + next : block;
+#pragma unroll
+        for (int i = 0; i < DT; ++i) put4(block + a.at_s + (((wave * DT + i) * a.vt + V) * 64 + lane) * 4, S[i]);
+        if (DELTA) {
+            m40_float4 read[4];
+#pragma unroll
+            for (int t = 0; t < 4; ++t) {
+                read[t] = m40_float4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int i = 0; i < DT; ++i) read[t] = mma4(wf[DELTA ? t : 0][i], S[i], read[t]);
+                part[DELTA ? c & 1u : 0][DELTA ? wave : 0][t][lane] = read[t];
+            }
+            load_w(ahead);
+            m40_wait_and_meet<63>();
+#pragma unroll
+            for (int t = 0; t < 4; ++t)
+#pragma unroll
+                for (int w = 0; w < 4; ++w) u[t] -= part[DELTA ? c & 1u : 0][DELTA ? w : 0][t][lane];
+#pragma unroll
+            for (int t = 0; t < 4; ++t)
+                if (t == wave) put4(block + a.at_u + ((t * a.vt + V) * 64 + lane) * 4, u[t]);
+        }
+#pragma unroll
+        for (int i = 0; i < DT; ++i) {
+            S[i] *= decay[i];
+#pragma unroll
+            for (int t = 0; t < 4; ++t) S[i] = mma4(kf[i][t], u[t], S[i]);
+        }
+        load_u(ahead);
+        load_k(ahead);
+        block += next;
+    }
+    if (!stored) return;
+#pragma unroll
+    for (int i = 0; i < DT; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const uint32_t d = (wave * DT + i) * 16 + 4 * g + r;
+            if (d < a.dim) own[d * step_d] = S[i][r];
+        }
+}
+
+// ---- outputs: wave w takes the chunk's rows 16 w ..; VT: the most column tiles
+template <int VT, bool DELTA>
+__global__ __launch_bounds__(256) void memory_outputs_kernel(M40MemoryArgs a) {
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, li = lane & 15;
+    const Chunk c(a, blockIdx.x);
+    const uint32_t head = blockIdx.y;
+    if (wave * 16 >= (int)c.n) return;
+    const float* block = block_of(a, blockIdx.x, head);
+    const int vt = (int)a.vt, t = wave * 16 + li;
+    m40_float4 o[VT];
+#pragma unroll
+    for (int j = 0; j < VT; ++j) o[j] = m40_float4{0.f, 0.f, 0.f, 0.f};
+    for (uint32_t d = 0; d < (a.dim + 15u) / 16u; ++d) {
+        const m40_float4 q = at4(block + t * a.dp + d * 16 + 4 * g);
+#pragma unroll
+        for (int j = 0; j < VT; ++j)
+            if (j < vt) o[j] = mma4(at4(block + a.at_s + ((d * vt + j) * 64 + lane) * 4), q, o[j]);
+    }
+    for (int b = 0; b <= wave; ++b) {
+        const m40_float4 p = at4(block + a.at_p + t * kChunk + b * 16 + 4 * g);
+#pragma unroll
+        for (int j = 0; j < VT; ++j)
+            if (j < vt) o[j] = mma4(at4(block + a.at_u + ((b * vt + j) * 64 + lane) * 4), p, o[j]);
+    }
+    const int vdim = (int)a.vdim;
+    float f = 1.0f;
+    if (!DELTA) {                                   // column vdim: n . q
+        float x = 0.0f;
+#pragma unroll
+        for (int j = 0; j < VT; ++j)
+            if (j == vdim / 16) {
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+                    if (r == vdim % 4) {
+                        x = o[j][r];
+                        if (g == vdim % 16 / 4) o[j][r] = 0.0f;
+                    }
+            }
+        x = __shfl(x, vdim % 16 / 4 * 16 + li);
+        f = 1.0f / (fmaxf(fabsf(x), expf(-block[a.at_gate + 128 + t])) + 1e-6f);
+    }
+    float ss = 0.0f;
+#pragma unroll
+    for (int j = 0; j < VT; ++j) {
+        o[j] *= f;
+        ss += o[j][0] * o[j][0] + o[j][1] * o[j][1] + o[j][2] * o[j][2] + o[j][3] * o[j][3];
+    }
+    ss = m40_add_xor32(m40_add_xor16(ss));
+    if (t >= (int)c.n) return;
+    const float inv = a.out_factor / sqrtf(ss / (float)vdim + a.eps);
+    const uint32_t row = c.row0 + t;
+    const float *gate = a.gate + (size_t)row * a.ld_gate + head * a.vdim, *norm = a.norm + head * a.norm_stride;
+    const bool vec = vdim % 4 == 0 && a.ld_gate % 4u == 0 && m40_aligned16(a.gate) && m40_aligned16(a.norm);
+#pragma unroll
+    for (int j = 0; j < VT; ++j) {
+        const int v = j * 16 + 4 * g;
+        if (j >= vt || v >= vdim) continue;
+        const m40_float4 z = m40_load4(gate + v, vdim - v, vec), w = m40_load4(norm + v, vdim - v, vec);
+        m40_float4 y;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) y[r] = o[j][r] * inv * w[r] * m40_sigmoid(z[r]);
+        m40_store_packed<m40_bf16>(static_cast<m40_bf16*>(a.out), (int)row, (int)(a.out_col + head * a.vdim) + v, (long)a.ld_out, y, vdim - v, vdim % 4 == 0 && a.out_col % 4u == 0);
+    }
+}
+
+template <int DT, bool DELTA>
+void walk(hipStream_t stream, const M40MemoryArgs& a, uint32_t n_portions) {
+    memory_walk_kernel<DT, DELTA><<<dim3(n_portions * a.heads, a.vt), 256, 0, stream>>>(a);
+}
+template <bool DELTA>
+int chunked(hipStream_t stream, const M40MemoryArgs& a, uint32_t n_portions, uint32_t n_chunks) {
+    if constexpr (DELTA) {
+        static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(delta_prepare_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)sizeof(DeltaLds));
+        if (attr != hipSuccess) return -2;
+        delta_prepare_kernel<<<dim3(n_chunks, a.heads), 256, sizeof(DeltaLds), stream>>>(a);
+    } else {
+        memory_scan_kernel<<<dim3(n_portions, a.heads), 1024, 0, stream>>>(a);
+        memory_prepare_kernel<<<dim3(n_chunks, a.heads), 256, 0, stream>>>(a);
+    }
+    switch (a.dp / 64u) {
+        case 1: walk<1, DELTA>(stream, a, n_portions); break;
+        case 2: walk<2, DELTA>(stream, a, n_portions); break;
+        case 3: walk<3, DELTA>(stream, a, n_portions); break;
+        default: walk<4, DELTA>(stream, a, n_portions); break;
+    }
+    const dim3 grid(n_chunks, a.heads);
+    if (a.vt <= 4u) memory_outputs_kernel<4, DELTA><<<grid, 256, 0, stream>>>(a);
+    else if (a.vt <= 9u) memory_outputs_kernel<9, DELTA><<<grid, 256, 0, stream>>>(a);
+    else memory_outputs_kernel<17, DELTA><<<grid, 256, 0, stream>>>(a);
+    return hipGetLastError() == hipSuccess ? 0 : -2;
+}
+
+constexpr uint32_t kMost = 256;
+// the parts of a block of scratch
+void lay_out(M40MemoryArgs& a, bool delta) {
+    a.dp = (a.dim + 63u) / 64u * 64u;
+    a.vt = (a.vdim + (delta ? 0u : 1u) + 15u) / 16u;
+    uint32_t at = kChunk * a.dp;
+    auto part = [&](uint32_t n) { const uint32_t x = at; at += n; return x; };
+    a.at_k = part(kChunk * a.dp);
+    a.at_p = part(kChunk * kChunk);
+    a.at_u = part(kChunk * 16u * a.vt);
+    a.at_decay = part(a.dp);
+    a.at_s = part(a.dp * 16u * a.vt);
+    a.at_w = part(delta ? kChunk * a.dp : 0u);
+    a.at_gate = part(delta ? 0u : 256u);
+    a.block = at;
+}
+uint64_t state_floats(bool delta, uint32_t dim, uint32_t vdim) {
+    const uint64_t s = (uint64_t)dim * ((vdim + 3u) & ~3u);
+    return delta ? s : s + ((dim + 3u) & ~3u) + 4u;
+}
+
+// what both rules' structs have in common
+template <class P>
+int run(M40llmCudaContext* ctx, M40MemoryArgs& a, const P& p, bool delta, uint32_t stream_kind) {
+    hipStream_t stream = m40_select_stream(ctx, stream_kind);
+    if (!stream || m40_ensure_device(ctx) != 0) return -2;
+    if (p.act_dtype > 1u || p.heads == 0 || p.heads > 65535u || p.n_portions == 0 || !m40llm_ext_memory_serves(p.dim, p.vdim) || p.ld_out % 32u != 0 ||
+        p.ld_out < p.out_col + (uint64_t)p.heads * p.vdim || !m40_aligned16(p.state) || !m40_aligned16(p.out))
+        return -3;
+    a.heads = p.heads; a.dim = p.dim; a.vdim = p.vdim; a.v4 = (p.vdim + 3u) & ~3u;
+    a.q_factor = p.q_factor; a.eps = p.eps; a.out_factor = p.out_factor;
+    a.state = static_cast<float*>(p.state);
+    a.head_floats = state_floats(delta, p.dim, p.vdim);
+    a.out = p.out; a.ld_out = p.ld_out; a.out_col = p.out_col;
+    a.portions = p.portions; a.chunk_base = p.chunk_base; a.chunks = p.chunks; a.row_pos = p.row_pos;
+    a.scratch = static_cast<float*>(p.scratch);
+    lay_out(a, delta);
+    (void)hipGetLastError();
+    if (!p.chunked) return m40_launch_memory_serial(stream, a, delta, p.act_dtype, p.n_portions);
+    if (p.act_dtype != M40LLM_ACT_BF16 || !p.chunk_base || !p.chunks || p.n_chunks == 0 || !p.scratch || !m40_aligned16(p.scratch) ||
+        p.scratch_bytes < (uint64_t)p.n_chunks * p.heads * a.block * 4u)
+        return -4;
+    return delta ? chunked<true>(stream, a, p.n_portions, p.n_chunks) : chunked<false>(stream, a, p.n_portions, p.n_chunks);
+}
+
+}  // namespace
+
+extern "C" {
+
+int m40llm_ext_memory_serves(uint32_t dim, uint32_t vdim) { return dim >= 1u && dim <= kMost && vdim >= 1u && vdim <= kMost; }
+uint64_t m40llm_ext_matrix_memory_state_floats(uint32_t dim, uint32_t vdim) { return state_floats(false, dim, vdim); }
+uint64_t m40llm_ext_channel_delta_state_floats(uint32_t dim, uint32_t vdim) { return state_floats(true, dim, vdim); }
+uint64_t m40llm_ext_memory_scratch_bytes(uint32_t delta, uint32_t n_chunks, uint32_t heads, uint32_t dim, uint32_t vdim) {
+    M40MemoryArgs a{};
+    a.dim = dim; a.vdim = vdim;
+    lay_out(a, delta != 0u);
+    return (uint64_t)n_chunks * heads * a.block * 4u;
+}
+
+int m40llm_ext_matrix_memory_async(M40llmCudaContext* ctx, const M40llmMatrixMemory* m, uint32_t stream_kind) {
+    if (!ctx || !m || !m->proj || !m->i_bias || !m->f_bias || !m->norm || !m->state || !m->out || !m->portions || !m->row_pos) return -1;
+    const uint64_t q = (uint64_t)m->heads * m->dim, v = (uint64_t)m->heads * m->vdim;
+    if (m->ld_proj < m->q_col + q || m->ld_proj < m->k_col + q || m->ld_proj < m->v_col + v || m->ld_proj < m->g_col + v || m->ld_proj < (uint64_t)m->i_col + m->heads ||
+        m->ld_proj < (uint64_t)m->f_col + m->heads || !(m->cap > 0.0f))
+        return -3;
+    M40MemoryArgs a{};
+    const float* x = static_cast<const float*>(m->proj);
+    a.share = 1u;
+    a.q = x + m->q_col; a.k = x + m->k_col; a.v = x + m->v_col; a.ld = m->ld_proj;
+    a.i = x + m->i_col; a.f = x + m->f_col; a.i_bias = static_cast<const float*>(m->i_bias); a.f_bias = static_cast<const float*>(m->f_bias);
+    a.cap = m->cap;
+    a.norm = static_cast<const float*>(m->norm); a.norm_stride = m->vdim;
+    a.gate = x + m->g_col; a.ld_gate = m->ld_proj;
+    return run(ctx, a, *m, false, stream_kind);
+}
+
+int m40llm_ext_channel_delta_async(M40llmCudaContext* ctx, const M40llmChannelDelta* m, uint32_t stream_kind) {
+    if (!ctx || !m || !m->qkv || !m->low || !m->beta || !m->A_log || !m->dt_bias || !m->norm || !m->state || !m->out || !m->portions || !m->row_pos) return -1;
+    if (m->kv_heads == 0 || m->heads % m->kv_heads != 0 || m->ld_qkv < 2ull * m->kv_heads * m->dim + (uint64_t)m->heads * m->vdim ||
+        m->ld_low < m->a_col + (uint64_t)m->heads * m->dim || m->ld_low < m->g_col + (uint64_t)m->heads * m->vdim || m->ld_beta < m->heads)
+        return -3;
+    M40MemoryArgs a{};
+    const float *x = static_cast<const float*>(m->qkv), *low = static_cast<const float*>(m->low);
+    a.share = m->heads / m->kv_heads;
+    a.q = x; a.k = x + (size_t)m->kv_heads * m->dim; a.v = x + 2u * (size_t)m->kv_heads * m->dim; a.ld = m->ld_qkv;
+    a.a = low + m->a_col; a.ld_a = m->ld_low;
+    a.beta = static_cast<const float*>(m->beta); a.ld_beta = m->ld_beta;
+    a.A_log = static_cast<const float*>(m->A_log); a.dt_bias = static_cast<const float*>(m->dt_bias);
+    a.norm = static_cast<const float*>(m->norm); a.norm_stride = 0;
+    a.gate = low + m->g_col; a.ld_gate = m->ld_low;
+    return run(ctx, a, *m, true, stream_kind);
+}
+
+}  // extern "C"

@@ -437,7 +437,7 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
     const bool paged = p->epilogue == M40LLM_PACKED_KEYS || p->epilogue == M40LLM_PACKED_VALUES;
     const uint32_t k_parts = p->k_parts > 1u ? p->k_parts : 1u, part_tiles = (p->k_tiles + k_parts - 1) / k_parts;
-    if (p->act_dtype > 1u || p->epilogue > M40LLM_PACKED_SILU || p->activation > M40LLM_SILU || p->rows == 0 || p->batches == 0 || p->batches > 65535u ||
+    if (p->act_dtype > 1u || p->epilogue > M40LLM_PACKED_SPLIT || p->activation > M40LLM_SILU || p->rows == 0 || p->batches == 0 || p->batches > 65535u ||
         p->n_tiles == 0 || p->k_tiles == 0 || !m40_aligned16(p->a) || !m40_aligned16(p->w) || p->rows > 0x3fffffffu ||
         (p->batches > 1u && (p->a_batch % 32 != 0 || p->w_batch % 8 != 0)))
         return -3;
@@ -449,7 +449,7 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
     if (!paged && (p->lda % 32 != 0 || p->lda < (uint64_t)p->k_tiles * 32u)) return -3;
     if (k_parts > 1u && (p->epilogue != M40LLM_PACKED_STORE || p->batches != 1u || (k_parts - 1) * part_tiles >= p->k_tiles)) return -3;
     // packed results: whole tiles of columns
-    if ((p->epilogue == M40LLM_PACKED_GATED || p->epilogue == M40LLM_PACKED_ROTATE || p->epilogue == M40LLM_PACKED_SILU || (p->epilogue == M40LLM_PACKED_PROJECT && p->out_act)) &&
+    if ((p->epilogue == M40LLM_PACKED_GATED || p->epilogue == M40LLM_PACKED_ROTATE || p->epilogue == M40LLM_PACKED_SILU || p->epilogue == M40LLM_PACKED_SPLIT || (p->epilogue == M40LLM_PACKED_PROJECT && p->out_act)) &&
         (p->ld_act % 32 != 0 || p->act_col % 4 != 0))
         return -3;
     const bool wide_stores = p->ld_act % 4 == 0 && reinterpret_cast<uintptr_t>(p->out_act) % (p->act_dtype == M40LLM_ACT_F32 ? 16 : 8) == 0;
@@ -470,7 +470,7 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
                 p->plain_tiles % 2 != 0 || p->n_tiles % 2 != 0 || p->plain_tiles > p->n_tiles)
                 return -4;
             break;
-        case M40LLM_PACKED_SILU:
+        case M40LLM_PACKED_SILU: case M40LLM_PACKED_SPLIT:
             if ((p->plain_tiles > 0 && !p->out_f32) || !p->out_act || !wide_stores || p->plain_tiles > p->n_tiles || p->batches != 1u) return -4;
             break;
         case M40LLM_PACKED_KEYS: case M40LLM_PACKED_VALUES:

@@ -91,7 +91,7 @@ struct M40Epilogue {
     long out_batch, act_batch;     // elements (packed: columns) from batch (head, part of K) to batch
     int cols;                      // columns stored (STORE, ADD, STORE_ACT, GATED)
     bool vec_out, vec_act;         // four neighbouring columns may be stored at once
-    int plain_tiles, act_col;      // PROJECT, SILU: tiles before the activated ones; the first activated column of out_act
+    int plain_tiles, act_col;      // PROJECT, SILU, SPLIT: tiles before those that go to out_act; the first column of out_act they take
     int activation;                // PROJECT
     int n_tiles;                   // KEYS, VALUES
     const float* gate;             // GATED: logits, [rows][ld_gate], one column per batch
@@ -137,9 +137,10 @@ __device__ __forceinline__ void m40_epilogue_tile(const M40Epilogue<T>& e, int b
     if (row >= e.rows) return;
     switch (e.kind) {
         case M40LLM_PACKED_SILU:
+        case M40LLM_PACKED_SPLIT:
             if (tile >= e.plain_tiles) {
 #pragma unroll
-                for (int r = 0; r < 4; ++r) v[r] = m40_silu(v[r]);
+                for (int r = 0; r < 4; ++r) v[r] = e.kind == M40LLM_PACKED_SILU ? m40_silu(v[r]) : v[r];
                 m40_store_packed<T>(e.out_act, row, e.act_col + col - e.plain_tiles * 16, e.ld_act, v, 4, true);
                 return;
             }

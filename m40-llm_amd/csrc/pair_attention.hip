@@ -1,6 +1,7 @@
-// Differential attention over a paged cache of keys and values (include/m40llm.h has the page order): every head has two maps, softmaxes
-// of their own queries and keys over the same values; the second map's result is taken off the first's, lambda times, and what is left is
-// normed over the head's value dimensions and gated.
+// Attention over a paged cache of keys and values (include/m40llm.h has the page order), in kernels for one or two maps a head (M).
+// Two maps, differential attention: softmaxes of their own queries and keys over the same values; the second map's result is taken off the
+// first's, lambda times, and what is left is normed over the head's value dimensions and gated.  One map: softmax attention, its result
+// scaled and, where there is a gate, gated column by column.
 //
 // Products are formed transposed, S' = K Q' and O' = V' P': a lane holds the scores of one query (lane % 16) for keys 4 g + r of every
 // 16, and pages hold values with their tokens in exactly that order, so the weights a lane computes are its operand of the second
@@ -25,8 +26,8 @@ struct PairArgs {
     M40llmPairAttention a;
     M40PairPage page;
     uint32_t group;
-    float* partial_o;      // [splits][rows * heads][2][16 v_tiles]
-    float* partial_ml;     // [splits][rows * heads][2][2]: reference, sum
+    float* partial_o;      // [splits][rows * heads][maps][16 v_tiles]
+    float* partial_ml;     // [splits][rows * heads][maps][2]: reference, sum
 };
 
 // what o (map 1's sums times f1 less map 2's times f2) is multiplied by: sum of squares of o over the head's dimensions in ss
@@ -34,18 +35,22 @@ __device__ __forceinline__ float last_factor(const M40llmPairAttention& a, float
     const float z = static_cast<const float*>(a.gate)[(size_t)row * a.ld_gate + head];
     return a.out_scale * m40_sigmoid(z) / sqrtf(ss / (float)a.vdim + a.eps);
 }
+// one map: what column v of a head's result is multiplied by
+__device__ __forceinline__ float column_factor(const M40llmPairAttention& a, uint32_t row, uint32_t head, uint32_t v) {
+    return a.gate ? a.out_scale * m40_sigmoid(static_cast<const float*>(a.gate)[(size_t)row * a.ld_gate + head * a.vdim + v]) : a.out_scale;
+}
 
 // One page (its tiles at `keys` / `values`, a kilobyte a tile, lane offset included) for B blocks of 16 queries.
-template <int DKT, int DVT, int B>
+template <int M, int DKT, int DVT, int B>
 struct PairState {
-    m40_bf16x8 q[2][B][DKT];
-    m40_float4 o[2][DVT][B];
-    float ref[2][B], sum[2][B];
+    m40_bf16x8 q[M][B][DKT];
+    m40_float4 o[M][DVT][B];
+    float ref[M][B], sum[M][B];
     uint32_t pos[B];
 
     __device__ __forceinline__ void clear() {
 #pragma unroll
-        for (int m = 0; m < 2; ++m)
+        for (int m = 0; m < M; ++m)
 #pragma unroll
             for (int b = 0; b < B; ++b) {
                 ref[m][b] = kNothing;
@@ -96,7 +101,7 @@ struct PairState {
     template <class G>
     __device__ __forceinline__ void join(G get) {
 #pragma unroll
-        for (int m = 0; m < 2; ++m)
+        for (int m = 0; m < M; ++m)
 #pragma unroll
             for (int b = 0; b < B; ++b) {
                 const int at = (m * B + b) * (2 + 4 * DVT);
@@ -110,11 +115,11 @@ struct PairState {
                     for (int r = 0; r < 4; ++r) o[m][j][b][r] = o[m][j][b][r] * f0 + get(at + 2 + j * 4 + r) * f1;
             }
     }
-    static constexpr int kFloats = 2 * B * (2 + 4 * DVT);       // of a lane
+    static constexpr int kFloats = M * B * (2 + 4 * DVT);       // of a lane
     template <class P>
     __device__ __forceinline__ void put(P set) const {
 #pragma unroll
-        for (int m = 0; m < 2; ++m)
+        for (int m = 0; m < M; ++m)
 #pragma unroll
             for (int b = 0; b < B; ++b) {
                 const int at = (m * B + b) * (2 + 4 * DVT);
@@ -128,16 +133,34 @@ struct PairState {
     }
     // the result of query block b to its row
     __device__ __forceinline__ void finish(const PairArgs& p, int b, uint32_t row, uint32_t head, bool live, int g) const {
-        float l1 = sum[0][b], l2 = sum[1][b];
-        l1 = m40_add_xor32(m40_add_xor16(l1));
-        l2 = m40_add_xor32(m40_add_xor16(l2));
-        const float f1 = 1.0f / l1, f2 = p.a.lambda / l2;
         const int vt = (int)p.page.v_tiles, vdim = (int)p.a.vdim;
+        const float f1 = 1.0f / m40_add_xor32(m40_add_xor16(sum[0][b]));
+        if constexpr (M == 1) {
+            if (!live) return;
+            const bool vec = p.a.gate && vdim % 4 == 0 && p.a.ld_gate % 4 == 0 && m40_aligned16(p.a.gate);
+            const float* gate = static_cast<const float*>(p.a.gate) + (p.a.gate ? (size_t)row * p.a.ld_gate + head * vdim : 0);
+#pragma unroll
+            for (int j = 0; j < DVT; ++j) {
+                const int v = j * 16 + 4 * g;
+                if (j >= vt || v >= vdim) continue;
+                m40_float4 y = o[0][j][b] * f1;
+                if (vec) {
+                    const m40_float4 z = *reinterpret_cast<const m40_float4*>(gate + v);
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) y[r] *= p.a.out_scale * m40_sigmoid(z[r]);
+                } else {
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) y[r] *= column_factor(p.a, row, head, (uint32_t)(v + r < vdim ? v + r : vdim - 1));
+                }
+                m40_store_packed<m40_bf16>(static_cast<m40_bf16*>(p.a.out), (int)row, (int)head * vdim + v, (long)p.a.ld_out, y, vdim - v, vdim % 4 == 0);
+            }
+        } else {
+        const float f2 = p.a.lambda / m40_add_xor32(m40_add_xor16(sum[M - 1][b]));
         float ss = 0.0f;
         m40_float4 d[DVT];
 #pragma unroll
         for (int j = 0; j < DVT; ++j) {
-            d[j] = o[0][j][b] * f1 - o[1][j][b] * f2;       // dimensions past vdim are zero in every page
+            d[j] = o[0][j][b] * f1 - o[M - 1][j][b] * f2;       // dimensions past vdim are zero in every page
             if (j < vt) ss += d[j][0] * d[j][0] + d[j][1] * d[j][1] + d[j][2] * d[j][2] + d[j][3] * d[j][3];
         }
         ss = m40_add_xor32(m40_add_xor16(ss));
@@ -149,10 +172,11 @@ struct PairState {
             if (j < vt && v < vdim)
                 m40_store_packed<m40_bf16>(static_cast<m40_bf16*>(p.a.out), (int)row, (int)head * vdim + v, (long)p.a.ld_out, d[j] * f, vdim - v, vdim % 4 == 0);
         }
+        }
     }
 };
 
-template <int DKT, int DVT>
+template <int M, int DKT, int DVT>
 __global__ __launch_bounds__(256, 1) void pair_rows_kernel(PairArgs p) {
     extern __shared__ __align__(16) float join_lds[];      // three waves' sums
     const M40llmPairAttention& a = p.a;
@@ -165,13 +189,13 @@ __global__ __launch_bounds__(256, 1) void pair_rows_kernel(PairArgs p) {
     const uint32_t pages = a.row_pos[last_row] / kPage + 1u, per = (pages + a.splits - 1u) / a.splits;
     const uint32_t page0 = blockIdx.z * per, page1 = page0 + per < pages ? page0 + per : pages;
     const uint32_t* table = a.page_table + (size_t)a.row_slot[last_row] * a.max_pages;
-    PairState<DKT, DVT, 1> s;
+    PairState<M, DKT, DVT, 1> s;
     s.clear();
     s.pos[0] = a.row_pos[row];
     const uint32_t first_pos = a.row_pos[q0 / p.group];
-    const m40_bf16* q = static_cast<const m40_bf16*>(a.queries) + ((size_t)row * a.heads + head) * (2u * kt * 32u) + g * 8;
+    const m40_bf16* q = static_cast<const m40_bf16*>(a.queries) + ((size_t)row * a.heads + head) * ((uint32_t)M * kt * 32u) + g * 8;
 #pragma unroll
-    for (int m = 0; m < 2; ++m)
+    for (int m = 0; m < M; ++m)
 #pragma unroll
         for (int k = 0; k < DKT; ++k) {
             s.q[m][0][k] = *reinterpret_cast<const m40_bf16x8*>(q + (m * kt + (k < kt ? k : kt - 1)) * 32);
@@ -183,9 +207,9 @@ __global__ __launch_bounds__(256, 1) void pair_rows_kernel(PairArgs p) {
         const m40_bf16* keys = cache + table[n] * p.page.elements();
         const m40_bf16* values = keys + p.page.key_elements();
         const bool whole = n * kPage + kPage - 1u <= first_pos;
-        m40_bf16x8 pf[2][1][2], vf[DVT][2];
+        m40_bf16x8 pf[M][1][2], vf[DVT][2];
 #pragma unroll
-        for (int m = 0; m < 2; ++m) {
+        for (int m = 0; m < M; ++m) {
             m40_float4 sc[4][1];
 #pragma unroll
             for (int t = 0; t < 4; ++t) {
@@ -207,11 +231,11 @@ __global__ __launch_bounds__(256, 1) void pair_rows_kernel(PairArgs p) {
 #pragma unroll
         for (int j = 0; j < DVT; ++j)
 #pragma unroll
-            for (int m = 0; m < 2; ++m)
+            for (int m = 0; m < M; ++m)
 #pragma unroll
                 for (int h = 0; h < 2; ++h) s.o[m][j][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[j][h], pf[m][0][h], s.o[m][j][0], 0, 0, 0);
     }
-    constexpr int kFloats = PairState<DKT, DVT, 1>::kFloats;
+    constexpr int kFloats = PairState<M, DKT, DVT, 1>::kFloats;
     if (wave > 0) {
         float* mine = join_lds + (size_t)(wave - 1) * kFloats * 64 + lane;
         s.put([&](int i, float v) { mine[i * 64] = v; });
@@ -227,38 +251,38 @@ __global__ __launch_bounds__(256, 1) void pair_rows_kernel(PairArgs p) {
         s.finish(p, 0, row, head, live, g);
         return;
     }
-    float l[2];
+    float l[M];
 #pragma unroll
-    for (int m = 0; m < 2; ++m) l[m] = m40_add_xor32(m40_add_xor16(s.sum[m][0]));
+    for (int m = 0; m < M; ++m) l[m] = m40_add_xor32(m40_add_xor16(s.sum[m][0]));
     if (!live) return;
     const size_t at = (size_t)blockIdx.z * a.n_rows * a.heads + (size_t)(row - a.first_row) * a.heads + head;
 #pragma unroll
-    for (int m = 0; m < 2; ++m) {
+    for (int m = 0; m < M; ++m) {
         if (g == 0) {
-            p.partial_ml[(at * 2 + m) * 2] = s.ref[m][0];
-            p.partial_ml[(at * 2 + m) * 2 + 1] = l[m];
+            p.partial_ml[(at * M + m) * 2] = s.ref[m][0];
+            p.partial_ml[(at * M + m) * 2 + 1] = l[m];
         }
 #pragma unroll
         for (int j = 0; j < DVT; ++j)
-            if (j < vt) *reinterpret_cast<m40_float4*>(p.partial_o + ((at * 2 + m) * vt + j) * 16 + 4 * g) = s.o[m][j][0];
+            if (j < vt) *reinterpret_cast<m40_float4*>(p.partial_o + ((at * M + m) * vt + j) * 16 + 4 * g) = s.o[m][j][0];
     }
 }
 
 // A workgroup a row and head: the splits' weights first, then eight groups of 32 lanes take every eighth split.
 constexpr int kJoinSplits = 256;
-template <class T>
+template <class T, int M>
 __global__ __launch_bounds__(256) void pair_join_kernel(PairArgs p) {
-    __shared__ float weight[2][kJoinSplits];
+    __shared__ float weight[M][kJoinSplits];
     __shared__ m40_float4 sums[8][32];
     __shared__ float part[4];
-    __shared__ float o_lds[2][M40LLM_PAIR_MOST_DIM];
+    __shared__ float o_lds[M][M40LLM_PAIR_MOST_DIM];
     const M40llmPairAttention& a = p.a;
     const uint32_t i = blockIdx.x, row = a.first_row + i / a.heads, head = i % a.heads, tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6;
     const uint32_t width = p.page.v_tiles * 16u, group = tid >> 5;
     const size_t stride = (size_t)a.n_rows * a.heads;
-    for (uint32_t m = 0; m < 2u; ++m) {
-        const float* ml = p.partial_ml + ((size_t)i * 2u + m) * 2u;
-        const float ref = tid < a.splits ? ml[tid * stride * 4u] : kNothing, l = tid < a.splits ? ml[tid * stride * 4u + 1u] : 0.0f;
+    for (uint32_t m = 0; m < (uint32_t)M; ++m) {
+        const float* ml = p.partial_ml + ((size_t)i * M + m) * 2u;
+        const float ref = tid < a.splits ? ml[tid * stride * 2u * M] : kNothing, l = tid < a.splits ? ml[tid * stride * 2u * M + 1u] : 0.0f;
         const float top = m40_max64(ref);
         if (lane == 0) part[wave] = top;
         __syncthreads();
@@ -273,9 +297,9 @@ __global__ __launch_bounds__(256) void pair_join_kernel(PairArgs p) {
             const uint32_t d = d0 + (tid & 31u) * 4u;
             m40_float4 acc = {0.f, 0.f, 0.f, 0.f};
             if (d < width) {
-                const float* o = p.partial_o + ((size_t)i * 2u + m) * width + d;
+                const float* o = p.partial_o + ((size_t)i * M + m) * width + d;
 #pragma unroll 4
-                for (uint32_t s = group; s < a.splits; s += 8u) acc += *reinterpret_cast<const m40_float4*>(o + s * stride * 2u * width) * weight[m][s];
+                for (uint32_t s = group; s < a.splits; s += 8u) acc += *reinterpret_cast<const m40_float4*>(o + s * stride * M * width) * weight[m][s];
             }
             sums[group][tid & 31u] = acc;
             __syncthreads();
@@ -288,7 +312,12 @@ __global__ __launch_bounds__(256) void pair_join_kernel(PairArgs p) {
             __syncthreads();
         }
     }
-    const float o = tid < a.vdim ? o_lds[0][tid] + o_lds[1][tid] : 0.0f;
+    if constexpr (M == 1) {
+        if (tid < a.vdim)
+            static_cast<T*>(a.out)[m40_packed_at(row, head * a.vdim + tid, a.ld_out >> 5)] = M40Act<T>::from(o_lds[0][tid] * column_factor(a, row, head, tid));
+        return;
+    }
+    const float o = tid < a.vdim ? o_lds[0][tid] + o_lds[M - 1][tid] : 0.0f;
     const float ss = m40_sum64(o * o);
     if (lane == 0) part[wave] = ss;
     __syncthreads();
@@ -296,7 +325,7 @@ __global__ __launch_bounds__(256) void pair_join_kernel(PairArgs p) {
     if (tid < a.vdim) static_cast<T*>(a.out)[m40_packed_at(row, head * a.vdim + tid, a.ld_out >> 5)] = M40Act<T>::from(o * f);
 }
 
-template <int DKT, int DVT, int QB, int GROUPS, int PER_CU>
+template <int M, int DKT, int DVT, int QB, int GROUPS, int PER_CU>
 __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArgs p) {
     typedef __attribute__((address_space(3))) void* lds_dst_t;
     typedef const __attribute__((address_space(1))) void* global_src_t;
@@ -304,7 +333,7 @@ __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArg
     const M40llmPairAttention& a = p.a;
     const int lane = threadIdx.x & 63, w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, li = lane & 15;
     const int wave = w & 3, group = w >> 2;
-    const int kt = (int)p.page.k_tiles, vt = (int)p.page.v_tiles, page_tiles = 8 * kt + 2 * vt;
+    const int kt = (int)p.page.k_tiles, vt = (int)p.page.v_tiles, page_tiles = 4 * M * kt + 2 * vt;
     const uint32_t kv = blockIdx.x, q0 = a.tiles[2 * blockIdx.y], count = a.tiles[2 * blockIdx.y + 1];
     const uint32_t last_row = (q0 + count - 1u) / p.group;
     const uint32_t pages = a.row_pos[last_row] / kPage + 1u, last = pages - 1u;
@@ -320,7 +349,7 @@ __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArg
     auto page_of = [&](uint32_t step) { const uint32_t n = step * GROUPS + group; return n < last ? n : last; };    // past the end: the last again
     issue(0, table[page_of(0)]);
     uint32_t next = table[page_of(1)];
-    PairState<DKT, DVT, QB> s;
+    PairState<M, DKT, DVT, QB> s;
     s.clear();
     uint32_t row[QB], head[QB];
     bool live[QB];
@@ -332,9 +361,9 @@ __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArg
         row[b] = query / p.group;
         head[b] = kv * p.group + query % p.group;
         s.pos[b] = a.row_pos[row[b]];
-        const m40_bf16* q = static_cast<const m40_bf16*>(a.queries) + ((size_t)row[b] * a.heads + head[b]) * (2u * kt * 32u) + g * 8;
+        const m40_bf16* q = static_cast<const m40_bf16*>(a.queries) + ((size_t)row[b] * a.heads + head[b]) * ((uint32_t)M * kt * 32u) + g * 8;
 #pragma unroll
-        for (int m = 0; m < 2; ++m)
+        for (int m = 0; m < M; ++m)
 #pragma unroll
             for (int k = 0; k < DKT; ++k) {
                 s.q[m][b][k] = *reinterpret_cast<const m40_bf16x8*>(q + (m * kt + (k < kt ? k : kt - 1)) * 32);
@@ -356,11 +385,11 @@ __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArg
         const uint32_t n = step * GROUPS + group;
         if (!wave_live || n > last || n * kPage > pos_last) continue;
         const uint8_t* keys = lds + (group * 2 + buf) * page_tiles * 1024 + lane * 16;
-        const uint8_t* values = keys + 8 * kt * 1024;
+        const uint8_t* values = keys + 4 * M * kt * 1024;
         const bool whole = n * kPage + kPage - 1u <= pos_first;
-        m40_bf16x8 pf[2][QB][2];
+        m40_bf16x8 pf[M][QB][2];
 #pragma unroll
-        for (int m = 0; m < 2; ++m) {
+        for (int m = 0; m < M; ++m) {
             m40_float4 sc[4][QB];
 #pragma unroll
             for (int t = 0; t < 4; ++t)
@@ -388,7 +417,7 @@ __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArg
                 for (int h = 0; h < 2; ++h) {
                     const m40_bf16x8 vf = *reinterpret_cast<const m40_bf16x8*>(values + (j * 2 + h) * 1024);
 #pragma unroll
-                    for (int m = 0; m < 2; ++m)
+                    for (int m = 0; m < M; ++m)
 #pragma unroll
                         for (int b = 0; b < QB; ++b) s.o[m][j][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[m][b][h], s.o[m][j][b], 0, 0, 0);
                 }
@@ -397,7 +426,7 @@ __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArg
     }
     if constexpr (GROUPS == 2) {
         m40_wait_and_meet<0>();                  // every buffer is free
-        float* mine = reinterpret_cast<float*>(lds) + (size_t)wave * PairState<DKT, DVT, QB>::kFloats * 64 + lane;
+        float* mine = reinterpret_cast<float*>(lds) + (size_t)wave * PairState<M, DKT, DVT, QB>::kFloats * 64 + lane;
         if (group == 1) s.put([&](int i, float v) { mine[i * 64] = v; });
         m40_wait_and_meet<63>();
         if (group == 1) return;
@@ -410,29 +439,32 @@ __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArg
     for (int b = 0; b < QB; ++b) s.finish(p, b, row[b], head[b], live[b], g);
 }
 
+template <int M>
 __global__ __launch_bounds__(256) void pair_f32_kernel(PairArgs p) {
-    __shared__ float q[2][M40LLM_PAIR_MOST_DIM], o[2][M40LLM_PAIR_MOST_DIM], s[2][kPage];
-    __shared__ float stat[2][3];             // maximum, sum, factor on what came before
+    __shared__ float q[M][M40LLM_PAIR_MOST_DIM], o[M][M40LLM_PAIR_MOST_DIM], s[M][kPage];
+    __shared__ float stat[M][3];             // maximum, sum, factor on what came before
     __shared__ float part[4];
     const M40llmPairAttention& a = p.a;
     const uint32_t tid = threadIdx.x, row = a.first_row + blockIdx.x / a.heads, head = blockIdx.x % a.heads, kv = head / p.group;
     const uint32_t width = p.page.k_tiles * 32u;
-    for (uint32_t i = tid; i < 2u * width; i += 256u) q[i / width][i % width] = static_cast<const float*>(a.queries)[((size_t)row * a.heads + head) * 2u * width + i];
-    for (uint32_t i = tid; i < 2u * a.vdim; i += 256u) o[i / a.vdim][i % a.vdim] = 0.0f;
-    if (tid < 2u) { stat[tid][0] = -INFINITY; stat[tid][1] = 0.0f; }
+    for (uint32_t i = tid; i < M * width; i += 256u) q[i / width][i % width] = static_cast<const float*>(a.queries)[((size_t)row * a.heads + head) * M * width + i];
+    for (uint32_t i = tid; i < M * a.vdim; i += 256u) o[i / a.vdim][i % a.vdim] = 0.0f;
+    if (tid < (uint32_t)M) { stat[tid][0] = -INFINITY; stat[tid][1] = 0.0f; }
     const uint32_t pos = a.row_pos[row], pages = pos / kPage + 1u;
     const uint32_t* table = a.page_table + (size_t)a.row_slot[row] * a.max_pages;
     __syncthreads();
     for (uint32_t n = 0; n < pages; ++n) {
         const float* page = static_cast<const float*>(a.cache) + table[n] * p.page.elements() + kv * p.page.head_elements();
-        // two lanes a token and map
-        const uint32_t map = tid >> 7, t = (tid & 127u) >> 1;
+        // two lanes a token and map of two, four a token of one
+        constexpr uint32_t kLanes = 4u / M;
+        const uint32_t map = tid / (kPage * kLanes), t = tid / kLanes % kPage;
         float x = 0.0f;
-        for (uint32_t d = tid & 1u; d < a.dim; d += 2u) x = fmaf(q[map][d], page[p.page.key_at(map, t, d)], x);
+        for (uint32_t d = tid % kLanes; d < a.dim; d += kLanes) x = fmaf(q[map][d], page[p.page.key_at(map, t, d)], x);
         x += m40_dpp_f<M40_DPP_XOR1>(x);
-        if ((tid & 1u) == 0u) s[map][t] = n * kPage + t <= pos ? x * a.scale : -INFINITY;
+        if (kLanes == 4u) x += m40_dpp_f<M40_DPP_XOR2>(x);
+        if (tid % kLanes == 0u) s[map][t] = n * kPage + t <= pos ? x * a.scale : -INFINITY;
         __syncthreads();
-        if (tid < 128u) {                    // a wave a map; a page of the range holds a seen token
+        if (tid < 64u * M) {                 // a wave a map; a page of the range holds a seen token
             const uint32_t m = tid >> 6, l = tid & 63u;
             const float v = s[m][l], before = stat[m][0], top = fmaxf(before, m40_max64(v));
             const float e = expf(v - top), f = expf(before - top), sum = m40_sum64(e);
@@ -440,7 +472,7 @@ __global__ __launch_bounds__(256) void pair_f32_kernel(PairArgs p) {
             if (l == 0u) { stat[m][0] = top; stat[m][1] = stat[m][1] * f + sum; stat[m][2] = f; }
         }
         __syncthreads();
-        for (uint32_t i = tid; i < 2u * a.vdim; i += 256u) {
+        for (uint32_t i = tid; i < M * a.vdim; i += 256u) {
             const uint32_t m = i / a.vdim, d = i % a.vdim;
             float acc = o[m][d] * stat[m][2];
             for (uint32_t k = 0; k < (uint32_t)kPage; ++k) acc = fmaf(s[m][k], page[p.page.value_at(k, d)], acc);
@@ -448,7 +480,12 @@ __global__ __launch_bounds__(256) void pair_f32_kernel(PairArgs p) {
         }
         __syncthreads();
     }
-    const float y = tid < a.vdim ? o[0][tid] / stat[0][1] - a.lambda * (o[1][tid] / stat[1][1]) : 0.0f;
+    if constexpr (M == 1) {
+        if (tid < a.vdim)
+            static_cast<float*>(a.out)[m40_packed_at(row, head * a.vdim + tid, a.ld_out >> 5)] = o[0][tid] / stat[0][1] * column_factor(a, row, head, tid);
+        return;
+    }
+    const float y = tid < a.vdim ? o[0][tid] / stat[0][1] - a.lambda * (o[M - 1][tid] / stat[M - 1][1]) : 0.0f;
     const float ss = m40_sum64(y * y);
     if ((tid & 63u) == 0u) part[tid >> 6] = ss;
     __syncthreads();
@@ -458,91 +495,102 @@ __global__ __launch_bounds__(256) void pair_f32_kernel(PairArgs p) {
 
 constexpr int kLdsMax = 160 * 1024;
 
-template <int DKT, int DVT>
+template <int M, int DKT, int DVT>
 int launch_rows(hipStream_t stream, const PairArgs& p) {
-    constexpr int lds = 3 * 64 * 4 * PairState<DKT, DVT, 1>::kFloats;
-    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(pair_rows_kernel<DKT, DVT>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    constexpr int lds = 3 * 64 * 4 * PairState<M, DKT, DVT, 1>::kFloats;
+    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(pair_rows_kernel<M, DKT, DVT>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
     if (attr != hipSuccess) return -2;
-    pair_rows_kernel<DKT, DVT><<<dim3(p.a.n_tiles, p.a.kv_heads, p.a.splits), 256, lds, stream>>>(p);
+    pair_rows_kernel<M, DKT, DVT><<<dim3(p.a.n_tiles, p.a.kv_heads, p.a.splits), 256, lds, stream>>>(p);
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
-int page_lds(const PairArgs& p, int groups) { return groups * 2 * (int)(8u * p.page.k_tiles + 2u * p.page.v_tiles) * 1024; }
-template <int DKT, int DVT, int QB, int GROUPS, int PER_CU>
+int page_lds(const PairArgs& p, int groups) { return groups * 2 * (int)(4u * p.page.maps * p.page.k_tiles + 2u * p.page.v_tiles) * 1024; }
+template <int M, int DKT, int DVT, int QB, int GROUPS, int PER_CU>
 int launch_tile(hipStream_t stream, const PairArgs& p) {
     static const hipError_t attr =
-        hipFuncSetAttribute(reinterpret_cast<const void*>(pair_tile_kernel<DKT, DVT, QB, GROUPS, PER_CU>), hipFuncAttributeMaxDynamicSharedMemorySize, kLdsMax);
+        hipFuncSetAttribute(reinterpret_cast<const void*>(pair_tile_kernel<M, DKT, DVT, QB, GROUPS, PER_CU>), hipFuncAttributeMaxDynamicSharedMemorySize, kLdsMax);
     if (attr != hipSuccess) return -2;
-    constexpr int join = GROUPS == 2 ? 4 * 64 * 4 * PairState<DKT, DVT, QB>::kFloats : 0;
+    constexpr int join = GROUPS == 2 ? 4 * 64 * 4 * PairState<M, DKT, DVT, QB>::kFloats : 0;
     static_assert(join <= kLdsMax, "the joining of two groups does not fit");
     const int pages = page_lds(p, GROUPS);
-    pair_tile_kernel<DKT, DVT, QB, GROUPS, PER_CU><<<dim3(p.a.kv_heads, p.a.n_tiles), GROUPS * 256, pages > join ? pages : join, stream>>>(p);
+    pair_tile_kernel<M, DKT, DVT, QB, GROUPS, PER_CU><<<dim3(p.a.kv_heads, p.a.n_tiles), GROUPS * 256, pages > join ? pages : join, stream>>>(p);
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
 // PER_CU: workgroups of one group a CU that fit
-template <int DKT, int DVT, int PER_CU>
+template <int M, int DKT, int DVT, int PER_CU>
 int launch_tile_any(hipStream_t stream, const PairArgs& p, int num_cus) {
     // with enough workgroups the short ones fill in behind the long ones
     if (page_lds(p, 2) <= kLdsMax && (uint64_t)p.a.kv_heads * p.a.n_tiles <= 3ull * (uint32_t)num_cus)
-        return p.a.tile_queries == 64u ? launch_tile<DKT, DVT, 1, 2, PER_CU>(stream, p) : launch_tile<DKT, DVT, 2, 2, PER_CU>(stream, p);
-    return p.a.tile_queries == 64u ? launch_tile<DKT, DVT, 1, 1, PER_CU>(stream, p) : launch_tile<DKT, DVT, 2, 1, PER_CU>(stream, p);
+        return p.a.tile_queries == 64u ? launch_tile<M, DKT, DVT, 1, 2, PER_CU>(stream, p) : launch_tile<M, DKT, DVT, 2, 2, PER_CU>(stream, p);
+    return p.a.tile_queries == 64u ? launch_tile<M, DKT, DVT, 1, 1, PER_CU>(stream, p) : launch_tile<M, DKT, DVT, 2, 1, PER_CU>(stream, p);
 }
 
-bool tile_served(uint32_t k_tiles, uint32_t v_tiles) { return 2u * (8u * k_tiles + 2u * v_tiles) * 1024u <= (uint32_t)kLdsMax; }
+bool tile_served(uint32_t maps, uint32_t k_tiles, uint32_t v_tiles) { return 2u * (4u * maps * k_tiles + 2u * v_tiles) * 1024u <= (uint32_t)kLdsMax; }
+
+// PER_CU of heads of 128 dimensions
+template <int M, int PER_CU>
+int launch_form(hipStream_t stream, const PairArgs& p, uint32_t form, int num_cus) {
+    const uint32_t kt = p.page.k_tiles, vt = p.page.v_tiles;
+    if (form == 1u) {
+        if (kt <= 2u && vt <= 4u) return launch_tile_any<M, 2, 4, 2>(stream, p, num_cus);
+        if (kt <= 2u && vt <= 8u) return launch_tile_any<M, 2, 8, 2>(stream, p, num_cus);
+        if (kt <= 4u && vt <= 8u) return launch_tile_any<M, 4, 8, PER_CU>(stream, p, num_cus);
+        return launch_tile<M, 8, 16, 1, 1, 1>(stream, p);
+    }
+    int rc;
+    if (kt <= 2u && vt <= 4u) rc = launch_rows<M, 2, 4>(stream, p);
+    else if (kt <= 2u && vt <= 8u) rc = launch_rows<M, 2, 8>(stream, p);
+    else if (kt <= 4u && vt <= 8u) rc = launch_rows<M, 4, 8>(stream, p);
+    else rc = launch_rows<M, 8, 16>(stream, p);
+    if (rc != 0 || p.a.splits == 1u) return rc;
+    pair_join_kernel<m40_bf16, M><<<p.a.n_rows * p.a.heads, 256, 0, stream>>>(p);
+    return hipGetLastError() == hipSuccess ? 0 : -2;
+}
 
 }  // namespace
 
 extern "C" {
 
-uint64_t m40llm_ext_pair_attention_partial_floats(uint32_t rows, uint32_t heads, uint32_t vdim, uint32_t splits) {
-    return splits <= 1u ? 0u : (uint64_t)splits * rows * heads * 2u * ((vdim + 15u) / 16u * 16u + 2u);
+uint64_t m40llm_ext_pair_attention_partial_floats(uint32_t maps, uint32_t rows, uint32_t heads, uint32_t vdim, uint32_t splits) {
+    return splits <= 1u ? 0u : (uint64_t)splits * rows * heads * maps * ((vdim + 15u) / 16u * 16u + 2u);
 }
 
-uint32_t m40llm_ext_pair_attention_tile_queries(uint32_t act_dtype, uint32_t dim, uint32_t vdim) {
-    if (dim == 0 || vdim == 0 || dim > M40LLM_PAIR_MOST_DIM || vdim > M40LLM_PAIR_MOST_DIM) return 0;
+uint32_t m40llm_ext_pair_attention_tile_queries(uint32_t act_dtype, uint32_t maps, uint32_t dim, uint32_t vdim) {
+    if (maps == 0 || maps > 2u || dim == 0 || vdim == 0 || dim > M40LLM_PAIR_MOST_DIM || vdim > M40LLM_PAIR_MOST_DIM) return 0;
     if (act_dtype == M40LLM_ACT_F32) return 128u;
     const uint32_t kt = (dim + 31u) / 32u, vt = (vdim + 15u) / 16u;
-    return !tile_served(kt, vt) ? 16u : vt <= 8u && kt <= 4u ? 128u : 64u;
+    return !tile_served(maps, kt, vt) ? 16u : vt <= 8u && kt <= 4u ? 128u : 64u;
 }
 
 int m40llm_ext_pair_attention_async(M40llmCudaContext* ctx, const M40llmPairAttention* a, uint32_t stream_kind) {
-    if (!ctx || !a || !a->queries || !a->cache || !a->gate || !a->row_slot || !a->row_pos || !a->page_table || !a->out) return -1;
+    if (!ctx || !a || !a->queries || !a->cache || (!a->gate && a->maps != 1u) || !a->row_slot || !a->row_pos || !a->page_table || !a->out) return -1;
     hipStream_t stream = m40_select_stream(ctx, stream_kind);
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
-    const uint32_t most = m40llm_ext_pair_attention_tile_queries(a->act_dtype, a->dim, a->vdim);
+    const uint32_t most = m40llm_ext_pair_attention_tile_queries(a->act_dtype, a->maps, a->dim, a->vdim);
     if (a->act_dtype > 1u || a->form > 1u || a->heads == 0 || a->kv_heads == 0 || a->heads % a->kv_heads != 0 || most == 0 || !(a->scale > 0.0f) || a->ld_out % 32u != 0 ||
         a->ld_out < a->heads * a->vdim || a->n_rows == 0 || !m40_aligned16(a->queries) || !m40_aligned16(a->cache))
         return -3;
-    PairArgs p{*a, M40PairPage(a->kv_heads, a->dim, a->vdim), a->heads / a->kv_heads, nullptr, nullptr};
+    PairArgs p{*a, M40PairPage(a->maps, a->kv_heads, a->dim, a->vdim), a->heads / a->kv_heads, nullptr, nullptr};
     (void)hipGetLastError();
     if (a->act_dtype == M40LLM_ACT_F32) {
-        pair_f32_kernel<<<a->n_rows * a->heads, 256, 0, stream>>>(p);
+        if (a->maps == 1u) pair_f32_kernel<1><<<a->n_rows * a->heads, 256, 0, stream>>>(p);
+        else pair_f32_kernel<2><<<a->n_rows * a->heads, 256, 0, stream>>>(p);
         return hipGetLastError() == hipSuccess ? 0 : -2;
     }
     if (!a->tiles || a->n_tiles == 0) return -1;
     const uint32_t kt = p.page.k_tiles, vt = p.page.v_tiles;
     if (a->form == 1u) {
-        if ((a->tile_queries != 64u && a->tile_queries != 128u) || a->tile_queries > most || a->n_tiles > 65535u || !tile_served(kt, vt)) return -3;
-        if (kt <= 2u && vt <= 4u) return launch_tile_any<2, 4, 2>(stream, p, ctx->num_cus);
-        if (kt <= 2u && vt <= 8u) return launch_tile_any<2, 8, 2>(stream, p, ctx->num_cus);
-        if (kt <= 4u && vt <= 8u) return launch_tile_any<4, 8, 1>(stream, p, ctx->num_cus);
-        return launch_tile<8, 16, 1, 1, 1>(stream, p);
+        if ((a->tile_queries != 64u && a->tile_queries != 128u) || a->tile_queries > most || a->n_tiles > 65535u || !tile_served(a->maps, kt, vt)) return -3;
+        return a->maps == 1u ? launch_form<1, 2>(stream, p, 1u, ctx->num_cus) : launch_form<2, 1>(stream, p, 1u, ctx->num_cus);
     }
     if (a->splits == 0 || a->splits > (uint32_t)kJoinSplits || a->kv_heads > 65535u) return -3;
     if (a->splits > 1u) {
         if (!a->partial || !m40_aligned16(a->partial) ||
-            a->partial_floats < m40llm_ext_pair_attention_partial_floats(a->n_rows, a->heads, a->vdim, a->splits))
+            a->partial_floats < m40llm_ext_pair_attention_partial_floats(a->maps, a->n_rows, a->heads, a->vdim, a->splits))
             return -4;
         p.partial_o = static_cast<float*>(a->partial);
-        p.partial_ml = p.partial_o + (size_t)a->splits * a->n_rows * a->heads * 2u * vt * 16u;
+        p.partial_ml = p.partial_o + (size_t)a->splits * a->n_rows * a->heads * a->maps * vt * 16u;
     }
-    int rc = -3;
-    if (kt <= 2u && vt <= 4u) rc = launch_rows<2, 4>(stream, p);
-    else if (kt <= 2u && vt <= 8u) rc = launch_rows<2, 8>(stream, p);
-    else if (kt <= 4u && vt <= 8u) rc = launch_rows<4, 8>(stream, p);
-    else rc = launch_rows<8, 16>(stream, p);
-    if (rc != 0 || a->splits == 1u) return rc;
-    pair_join_kernel<m40_bf16><<<a->n_rows * a->heads, 256, 0, stream>>>(p);
-    return hipGetLastError() == hipSuccess ? 0 : -2;
+    return a->maps == 1u ? launch_form<1, 2>(stream, p, 0u, ctx->num_cus) : launch_form<2, 1>(stream, p, 0u, ctx->num_cus);
 }
 
 }  // extern "C"

@@ -1,4 +1,4 @@
-// Pages of a cache of keys and values whose keys come in two maps a head (include/m40llm.h has the order).
+// Pages of a cache of keys and values whose keys come in one or two maps a head (include/m40llm.h has the order).
 #pragma once
 
 #include "packed_gemm.hpp"
@@ -6,9 +6,9 @@
 #define M40LLM_PAIR_MOST_DIM 256u
 
 struct M40PairPage {
-    uint32_t kv_heads, k_tiles, v_tiles;
-    M40_HD M40PairPage(uint32_t heads, uint32_t dim, uint32_t vdim) : kv_heads(heads), k_tiles((dim + 31u) / 32u), v_tiles((vdim + 15u) / 16u) {}
-    M40_HD size_t key_elements() const { return (size_t)8u * k_tiles * 512u; }                       // both maps of a kv head
+    uint32_t maps, kv_heads, k_tiles, v_tiles;
+    M40_HD M40PairPage(uint32_t maps_, uint32_t heads, uint32_t dim, uint32_t vdim) : maps(maps_), kv_heads(heads), k_tiles((dim + 31u) / 32u), v_tiles((vdim + 15u) / 16u) {}
+    M40_HD size_t key_elements() const { return (size_t)4u * maps * k_tiles * 512u; }                // all maps of a kv head
     M40_HD size_t head_elements() const { return key_elements() + (size_t)2u * v_tiles * 512u; }
     M40_HD size_t elements() const { return kv_heads * head_elements(); }
 #ifdef __HIPCC__

@@ -2,6 +2,7 @@
 // attention's projections and its attention (short convolution, query and key norms, cache append).
 #include "packed_gemm.hpp"
 #include "pair_cache.hpp"
+#include "short_conv.hpp"
 
 namespace {
 
@@ -149,101 +150,27 @@ __global__ __launch_bounds__(kThreads) void norm_gate_rows_kernel(const float* _
     }
 }
 
-// A workgroup takes 16 rows and one unit: a map of a query head, a map of a key head, or a value head; 16 lanes a row, lane l the unit's
-// columns in groups of W at W (l + 16 i), N groups at most (W 4: every size and offset a multiple of 4).
-//
-// What precedes a portion's first row lies in a ring by position, entry p % (taps - 1).  The only row of a portion overwrites the oldest
-// entry, which it has read, with its own.
-template <int W> struct Columns { float v[W]; };
-template <int W>
-__device__ __forceinline__ Columns<W> load_columns(const float* p) {
-    Columns<W> c;
-    if (W == 4) {
-        const float4 t = *reinterpret_cast<const float4*>(p);
-        c.v[0] = t.x; c.v[W > 1 ? 1 : 0] = t.y; c.v[W > 2 ? 2 : 0] = t.z; c.v[W > 3 ? 3 : 0] = t.w;
-    } else {
-#pragma unroll
-        for (int k = 0; k < W; ++k) c.v[k] = p[k];
-    }
-    return c;
-}
-template <class T, int W>
-__device__ __forceinline__ void store_columns(T* p, const float (&v)[W]) {
-    if (W == 4) m40_store4<T>(p, m40_float4{v[0], v[W > 1 ? 1 : 0], v[W > 2 ? 2 : 0], v[W > 3 ? 3 : 0]});
-    else {
-#pragma unroll
-        for (int k = 0; k < W; ++k) p[k] = M40Act<T>::from(v[k]);
-    }
-}
+// A workgroup takes 16 rows and one unit: a map of a query head, a map of a key head, or a value head; 16 lanes a row.
 enum { kQueries = 0, kKeys = 1, kValues = 2 };
 template <class T, int W, int N>
 __device__ __forceinline__ void split_unit(const M40llmPairSplit& a, const M40PairPage& page, int kind, uint32_t unit, uint32_t row, uint32_t lane) {
     const uint32_t n = kind == kValues ? a.vdim : a.dim, col0 = (kind == kQueries ? 0u : kind == kKeys ? a.k_offset : a.v_offset) + unit * n;
     const uint32_t all = (kind == kQueries ? 2u * a.heads : kind == kKeys ? 2u * a.kv_heads : a.kv_heads) * n;      // columns of this kind
     const float* conv = static_cast<const float*>(kind == kQueries ? a.q_conv : kind == kKeys ? a.k_conv : a.v_conv);
-    const uint32_t pos = a.row_pos[row], slot = a.row_slot[row], info = a.row_back[row], back = info & 0x7fffffffu;
+    const uint32_t pos = a.row_pos[row], slot = a.row_slot[row], info = a.row_back[row];
     const uint32_t number = kind == kQueries ? 0u : a.page_table[(size_t)slot * a.max_pages + pos / M40LLM_PAGE_TOKENS];
-    const float* u = static_cast<const float*>(a.proj) + (size_t)row * a.ld_proj + col0;
-    uint32_t c[N];
-    bool live[N];
-    Columns<W> now[N];
+    const uint32_t keep = a.taps ? a.taps - 1u : 0u;
+    const M40ConvRow r{static_cast<const float*>(a.proj) + (size_t)row * a.ld_proj + col0, (size_t)a.ld_proj, a.taps ? conv + unit * n : nullptr, all, a.taps,
+                       keep ? static_cast<float*>(a.conv_state) + (size_t)slot * keep * a.ld_state + col0 : nullptr, (size_t)a.ld_state, pos, info};
     float y[N][W];
-#pragma unroll
-    for (int i = 0; i < N; ++i) {
-        c[i] = W * (lane + 16u * i);
-        live[i] = c[i] < n;
-        if (!live[i]) c[i] = 0u;             // loads of columns past the unit go to its first
-        now[i] = load_columns<W>(u + c[i]);
-    }
-    if (a.taps) {
-        const uint32_t keep = a.taps - 1u;
-        float* state = static_cast<float*>(a.conv_state) + (size_t)slot * keep * a.ld_state + col0;
-        const float* w = conv + unit * n;
-#pragma unroll
-        for (int i = 0; i < N; ++i) {
-            const Columns<W> wn = load_columns<W>(w + (size_t)keep * all + c[i]);
-#pragma unroll
-            for (int k = 0; k < W; ++k) y[i][k] = wn.v[k] * now[i].v[k];
-        }
-#pragma unroll 4
-        for (uint32_t d = 1; d <= keep; ++d) {               // rows back; loads under selected addresses, none behind a branch
-            const bool here = d <= back, some = d <= pos;
-            const float* src = here ? u - (size_t)d * a.ld_proj : some ? state + (size_t)((pos - d) % keep) * a.ld_state : u;
-            const float f = some ? 1.0f : 0.0f;
-#pragma unroll
-            for (int i = 0; i < N; ++i) {
-                const Columns<W> before = load_columns<W>(src + c[i]), wd = load_columns<W>(w + (size_t)(keep - d) * all + c[i]);
-#pragma unroll
-                for (int k = 0; k < W; ++k) y[i][k] = fmaf(wd.v[k] * f, before.v[k], y[i][k]);
-            }
-        }
-        if (info >> 31 && keep) {
-            float* own = state + (size_t)(pos % keep) * a.ld_state;
-#pragma unroll
-            for (int i = 0; i < N; ++i)
-                if (live[i]) store_columns<float, W>(own + c[i], now[i].v);
-        }
-    } else {
-#pragma unroll
-        for (int i = 0; i < N; ++i)
-#pragma unroll
-            for (int k = 0; k < W; ++k) y[i][k] = now[i].v[k];
-    }
-#pragma unroll
-    for (int i = 0; i < N; ++i)
-#pragma unroll
-        for (int k = 0; k < W; ++k) y[i][k] = live[i] ? y[i][k] : 0.0f;
+    m40_short_conv<W, N>(r, n, lane, y);
     if (kind != kValues) {
         const float* norm = static_cast<const float*>(kind == kQueries ? a.q_norm : a.k_norm);
-        float ss = 0.0f;
-#pragma unroll
-        for (int i = 0; i < N; ++i)
-#pragma unroll
-            for (int k = 0; k < W; ++k) ss = fmaf(y[i][k], y[i][k], ss);
-        const float inv = 1.0f / sqrtf(m40_sum16(ss) / (float)n + a.eps);
+        const float inv = 1.0f / sqrtf(m40_sum_squares16<W, N>(y) / (float)n + a.eps);
 #pragma unroll
         for (int i = 0; i < N; ++i) {
-            const Columns<W> w = load_columns<W>(norm + c[i]);
+            const uint32_t c = W * (lane + 16u * i);
+            const M40Columns<W> w = m40_load_columns<W>(norm + (c < n ? c : 0u));
 #pragma unroll
             for (int k = 0; k < W; ++k) y[i][k] *= inv * w.v[k];
         }
@@ -255,8 +182,8 @@ __device__ __forceinline__ void split_unit(const M40llmPairSplit& a, const M40Pa
     for (int i = 0; i < N; ++i) {
         const uint32_t at = W * (lane + 16u * i);            // pads too: zeros
         if (at >= pad) continue;
-        if (kind == kQueries) store_columns<T, W>(q + at, y[i]);
-        else if (kind == kKeys) store_columns<T, W>(cache + page.key_at(unit % 2u, t, at), y[i]);
+        if (kind == kQueries) m40_store_columns<T, W>(q + at, y[i]);
+        else if (kind == kKeys) m40_store_columns<T, W>(cache + page.key_at(unit % 2u, t, at), y[i]);
         else {
 #pragma unroll
             for (int k = 0; k < W; ++k) cache[page.value_at(t, at + k)] = M40Act<T>::from(y[i][k]);
@@ -341,7 +268,7 @@ int m40llm_ext_norm_gate_rows_async(M40llmCudaContext* ctx, const void* d_y, uin
     return launched();
 }
 
-uint64_t m40llm_ext_pair_page_elements(uint32_t kv_heads, uint32_t dim, uint32_t vdim) { return M40PairPage(kv_heads, dim, vdim).elements(); }
+uint64_t m40llm_ext_pair_page_elements(uint32_t maps, uint32_t kv_heads, uint32_t dim, uint32_t vdim) { return M40PairPage(maps, kv_heads, dim, vdim).elements(); }
 
 int m40llm_ext_pair_split_append_async(M40llmCudaContext* ctx, const M40llmPairSplit* s, uint32_t stream_kind) {
     if (!ctx || !s || !s->proj || !s->q_norm || !s->queries || !s->row_slot || !s->row_pos || !s->row_back) return -1;
@@ -356,7 +283,7 @@ int m40llm_ext_pair_split_append_async(M40llmCudaContext* ctx, const M40llmPairS
     if (s->cache && (!s->k_norm || !s->page_table || s->k_offset < 2u * s->heads * s->dim || s->v_offset < s->k_offset + 2u * s->kv_heads * s->dim ||
                      (s->taps && (!s->k_conv || !s->v_conv))))
         return -4;
-    const M40PairPage page(s->kv_heads, s->dim, s->vdim);
+    const M40PairPage page(2u, s->kv_heads, s->dim, s->vdim);
     if (s->act_dtype == M40LLM_ACT_F32) launch_split<float>(stream, *s, page);
     else launch_split<m40_bf16>(stream, *s, page);
     return launched();

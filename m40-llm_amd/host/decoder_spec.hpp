@@ -70,7 +70,35 @@ struct LightningSpec {
     std::vector<double> decay;
 };
 
-typedef std::variant<LatentAttentionSpec, DifferentialAttentionSpec, LightningSpec> MixerSpec;
+// Softmax attention.  Optional: biases on the projections, RMS norm over all query and over all key columns, rotation, a sigmoid gate per
+// column; values mixed with those of the first layer that shares its own (share_values).
+struct AttentionSpec {
+    uint32_t heads = 0, kv_heads = 0, dim = 0, vdim = 0;
+    float scale = 0.0f;
+    bool biases = false, projection_norm = false, column_gate = false, share_values = false;
+    std::optional<RotationSpec> rotation;
+};
+
+// A matrix state with exponential gates whose logits are capped; norm per head, weights per column, a sigmoid gate per column.
+struct MatrixMemorySpec {
+    uint32_t heads = 0, dim = 0, vdim = 0;
+    float gate_cap = 0.0f;
+};
+
+// Attention and a matrix memory that read the same input; their outputs times a factor each.
+struct ParallelSpec {
+    AttentionSpec left;
+    MatrixMemorySpec right;
+    float left_scale = 1.0f, right_scale = 1.0f;
+};
+
+// Delta rule with one decay per head and key channel; queries, keys and values behind a short convolution and silu; decays and output gates from
+// low-rank products whose rank the tensors give.
+struct ChannelDeltaSpec {
+    uint32_t heads = 0, kv_heads = 0, dim = 0, vdim = 0, taps = 0;
+};
+
+typedef std::variant<LatentAttentionSpec, DifferentialAttentionSpec, LightningSpec, AttentionSpec, ParallelSpec, ChannelDeltaSpec> MixerSpec;
 
 enum class Activation { GeluTanh, Silu };
 enum class NormKind { Layer, Rms };
@@ -80,10 +108,13 @@ struct GatedMlpSpec {          // down(activation(gate h) * (up h))
     Activation activation = Activation::GeluTanh;
 };
 
-// Of `experts` gated feed-forwards and `identity` experts that return their input, each token takes `top` by softmax score + correction
-// and adds up their outputs times their scores.
+// Of `experts` gated feed-forwards and `identity` experts that return their input, each token takes `top` by softmax score (+ correction)
+// and adds up their outputs times scale times their scores.  groups > 1: experts form groups of neighbours, and only those of the `keep` groups with
+// the best expert can be taken.
 struct ExpertMlpSpec {
-    uint32_t experts = 0, identity = 0, top = 0, ff = 0;
+    uint32_t experts = 0, identity = 0, top = 0, ff = 0, groups = 1, keep = 1;
+    float scale = 1.0f;
+    bool correction = true;
     Activation activation = Activation::Silu;
 };
 
@@ -101,6 +132,7 @@ struct LayerSpec {
 enum class BlockKind {
     Parallel,       // one norm whose output both sublayers read: x += mixer(norm(x)) + mlp(norm(x))
     OutputNorm,     // x += m * norm1(mixer(x)), then x += m * norm2(mlp(x))
+    Streams,        // several streams: u = in . x, y = mixer(norm1(u)), x_t = sum_s mix[s][t] x_s + m * out[t] * y; the same with the mlp
 };
 
 struct DecoderSpec {
@@ -108,6 +140,9 @@ struct DecoderSpec {
     uint32_t vocab = 0, width = 0;
     float eps = 0.0f;
     NormKind norm = NormKind::Layer;
+    bool norm_around_zero = false;     // norm weights are stored less one
+    bool tied_head = false;            // logits from the embedding table
+    uint32_t streams = 1;              // BlockKind::Streams
     BlockKind block = BlockKind::Parallel;
     float embedding_scale = 1.0f, residual_mult = 1.0f;
     uint32_t positions = 0;        // rows of a learned position table (0 = none): the most tokens of a sequence
@@ -251,9 +286,100 @@ inline DecoderSpec read_gulidra(const json::Value& c) {
     return d;
 }
 
+inline AttentionSpec read_attention_sizes(const json::Value& m, const std::string& where) {
+    AttentionSpec a;
+    a.heads = m.u32("heads"); a.kv_heads = m.u32("kv_heads"); a.dim = m.u32("dim"); a.vdim = m.u32("vdim");
+    a.scale = (float)m.num("scale");
+    if (!a.heads || !a.kv_heads || !a.dim || !a.vdim) throw json::Error(where + "a size is zero");
+    if (a.heads % a.kv_heads != 0) throw json::Error(where + "heads must be a multiple of kv_heads");
+    if (a.scale == 0.0f) throw json::Error(where + "scale is zero");
+    return a;
+}
+
+inline bool optional_flag(const json::Value& v, const std::string& key) {
+    const json::Value* f = v.find(key);
+    if (!f || f->is_null()) return false;
+    if (f->kind != json::Value::Kind::Bool) throw json::Error("'" + key + "' is not true or false");
+    return f->boolean;
+}
+
+inline DecoderSpec read_natatar(const json::Value& c) {
+    DecoderSpec d;
+    d.architecture = "Natatar";
+    d.vocab = c.u32("vocab");
+    d.width = c.u32("width");
+    d.eps = (float)c.at("norm").num("eps");
+    d.norm = NormKind::Rms;
+    d.norm_around_zero = true;
+    d.tied_head = true;
+    d.block = BlockKind::Streams;
+    d.streams = c.u32("streams");
+    d.residual_mult = (float)optional_num(c, "residual_mult", 1.0);
+    if (const json::Value* e = c.find("embedding"); e && !e->is_null()) d.embedding_scale = (float)optional_num(*e, "scale", 1.0);
+    const auto& layers = c.array("layers");
+    uint32_t shared_columns = 0;
+    for (size_t i = 0; i < layers.size(); ++i) {
+        const json::Value& l = layers[i];
+        const std::string where = "layer " + std::to_string(i) + ": ";
+        auto check = [&](bool ok, const char* what) { if (!ok) throw json::Error(where + what); };
+        const json::Value& m = l.at("mixer");
+        LayerSpec s;
+        if (l.str("type") == "attention") {
+            AttentionSpec a = read_attention_sizes(m, where);
+            a.biases = a.projection_norm = true;
+            a.share_values = optional_flag(m, "v_mix");
+            if (a.share_values) {
+                check(shared_columns == 0 || shared_columns == a.kv_heads * a.vdim, "layers that mix values must have equally many value columns");
+                shared_columns = a.kv_heads * a.vdim;
+            }
+            s.mixer = a;
+        } else if (l.str("type") == "parallel") {
+            ParallelSpec p;
+            const json::Value &left = m.at("left"), &right = m.at("right");
+            p.left = read_attention_sizes(left, where);
+            p.left.column_gate = true;
+            p.left.rotation = read_rotation(left.at("rot"));
+            check(p.left.rotation->dims <= p.left.dim && p.left.rotation->dims % 2 == 0, "rot.dims must be even and at most dim");
+            p.right.heads = right.u32("heads"); p.right.dim = right.u32("dim"); p.right.vdim = right.u32("vdim");
+            p.right.gate_cap = (float)right.num("gate_cap");
+            check(p.right.heads && p.right.dim && p.right.vdim, "a size is zero");
+            check(p.right.gate_cap > 0.0f, "gate_cap must be positive");
+            p.left_scale = (float)optional_num(m, "left_scale", 1.0);
+            p.right_scale = (float)optional_num(m, "right_scale", 1.0);
+            s.mixer = p;
+        } else if (l.str("type") == "channel_delta") {
+            ChannelDeltaSpec a;
+            a.heads = m.u32("heads"); a.kv_heads = m.u32("kv_heads"); a.dim = m.u32("dim"); a.vdim = m.u32("vdim"); a.taps = m.u32("conv");
+            check(a.heads && a.kv_heads && a.dim && a.vdim && a.taps, "a size is zero");
+            check(a.heads % a.kv_heads == 0, "heads must be a multiple of kv_heads");
+            s.mixer = a;
+        } else {
+            throw json::Error(where + "unknown mixer '" + l.str("type") + "'");
+        }
+        if (const json::Value* f = l.find("mlp"); f && !f->is_null()) {
+            if (f->str("kind") != "moe") throw json::Error(where + "unknown feed-forward '" + f->str("kind") + "'");
+            const json::Value& r = f->at("router");
+            ExpertMlpSpec e;
+            e.correction = false;
+            e.experts = r.u32("experts"); e.top = r.u32("top");
+            e.ff = f->at("expert").u32("ff");
+            e.scale = (float)optional_num(r, "scale", 1.0);
+            if (const json::Value* g = r.find("groups"); g && !g->is_null()) { e.groups = g->u32("count"); e.keep = g->u32("keep"); }
+            check(e.experts && e.top && e.ff && e.groups && e.keep, "a size is zero");
+            check(e.experts % e.groups == 0, "router.experts must be a multiple of groups.count");
+            check(e.keep <= e.groups, "groups.keep is larger than groups.count");
+            check(e.top <= e.keep * (e.experts / e.groups), "router.top is larger than the number of experts to choose from");
+            s.mlp = e;
+        }
+        d.layers.push_back(s);
+    }
+    if (d.vocab == 0 || d.width == 0 || d.streams == 0 || d.layers.empty()) throw json::Error("vocab, width, streams and layers must not be empty");
+    return d;
+}
+
 // designs by the name config.json gives in "architecture"
 inline const std::map<std::string, std::function<DecoderSpec(const json::Value&)>>& decoder_registry() {
-    static const std::map<std::string, std::function<DecoderSpec(const json::Value&)>> r = {{"Pimosun", read_pimosun}, {"Gulidra", read_gulidra}};
+    static const std::map<std::string, std::function<DecoderSpec(const json::Value&)>> r = {{"Pimosun", read_pimosun}, {"Gulidra", read_gulidra}, {"Natatar", read_natatar}};
     return r;
 }
 inline DecoderSpec read_decoder_spec(const std::string& config_text) {

@@ -19,26 +19,6 @@
 
 namespace m40host {
 
-// cosines and sines of a pass's rows
-struct RotationAngles : PassTable {
-    RotationAngles(LayerRuntime* rt, RotationSpec s, uint32_t h) : rt_(rt), spec(s), half(h) {
-        const std::vector<double> f = spec.frequencies();
-        freq_ = DeviceBuf(rt->ctx, std::max<size_t>(f.size(), 1) * 8);
-        if (!f.empty()) M40H_TRY(m40llm_memcpy_h2d(rt->ctx, freq_.ptr(), f.data(), f.size() * 8));
-        angles = rt->cleared((size_t)rt->rows_pad * half * 8);
-    }
-    bool same(LayerRuntime*, const RotationSpec& s, uint32_t h) const { return spec == s && half == h; }
-    std::vector<uint32_t> build(const PassPlan&, const SequencePages&, uint32_t) override { return {}; }
-    void enqueue(const Rows& r) override {
-        M40H_TRY(m40llm_ext_rotation_angles_async(rt_->ctx, r.pos, r.rows, static_cast<const double*>(freq_.ptr()), spec.dims / 2, half,
-                                                  (float)spec.magnitude(), angles.ptr(), LayerRuntime::kStream));
-    }
-    LayerRuntime* rt_;
-    RotationSpec spec;
-    uint32_t half;                        // padded pairs of a row
-    DeviceBuf freq_, angles;
-};
-
 // Tiles of query rows (row, head) for the rows of single tokens and short portions.
 struct LatentTiles : PassTable {
     LatentTiles(uint32_t act, uint32_t h, uint32_t most, uint32_t pad) : act_dtype(act), heads(h), max_m_tiles(most), latent_pad(pad) {}

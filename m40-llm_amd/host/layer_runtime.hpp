@@ -129,6 +129,20 @@ public:
         M40H_TRY(m40llm_memcpy_h2d(ctx, b.ptr(), v.data(), v.size() * 4));
         return b;
     }
+    DeviceBuf upload_norm(TensorSource& t, const std::string& name) {         // of the residual's width
+        std::vector<float> w = t.read_f32(name, {spec.width});
+        if (spec.norm_around_zero)
+            for (float& x : w) x += 1.0f;
+        return upload_f32(w);
+    }
+    // [columns][taps] to [taps][columns]
+    DeviceBuf upload_taps(TensorSource& t, const std::string& name, uint32_t cols, uint32_t taps) {
+        const std::vector<float> w = t.read_f32(name, {cols, taps});
+        std::vector<float> o(w.size());
+        for (uint32_t c = 0; c < cols; ++c)
+            for (uint32_t j = 0; j < taps; ++j) o[(size_t)j * cols + c] = w[(size_t)c * taps + j];
+        return upload_f32(o);
+    }
     void* stage(TensorSource& t, const std::string& name, const std::vector<uint64_t>& shape) {
         const size_t bytes = tensor_elements(shape) * 2;
         M40H_TRY(m40llm_stream_synchronize(ctx, kStream));       // the tensor before may still be being packed
@@ -228,6 +242,26 @@ public:
 private:
     DeviceBuf staging_;
     PortionTable* portions_ = nullptr;
+};
+
+// cosines and sines of a pass's rows
+struct RotationAngles : PassTable {
+    RotationAngles(LayerRuntime* rt, RotationSpec s, uint32_t h) : rt_(rt), spec(s), half(h) {
+        const std::vector<double> f = spec.frequencies();
+        freq_ = DeviceBuf(rt->ctx, std::max<size_t>(f.size(), 1) * 8);
+        if (!f.empty()) M40H_TRY(m40llm_memcpy_h2d(rt->ctx, freq_.ptr(), f.data(), f.size() * 8));
+        angles = rt->cleared((size_t)rt->rows_pad * half * 8);
+    }
+    bool same(LayerRuntime*, const RotationSpec& s, uint32_t h) const { return spec == s && half == h; }
+    std::vector<uint32_t> build(const PassPlan&, const SequencePages&, uint32_t) override { return {}; }
+    void enqueue(const Rows& r) override {
+        M40H_TRY(m40llm_ext_rotation_angles_async(rt_->ctx, r.pos, r.rows, static_cast<const double*>(freq_.ptr()), spec.dims / 2, half,
+                                                  (float)spec.magnitude(), angles.ptr(), LayerRuntime::kStream));
+    }
+    LayerRuntime* rt_;
+    RotationSpec spec;
+    uint32_t half;                        // padded pairs of a row
+    DeviceBuf freq_, angles;
 };
 
 // One layer (or block) of a decoder.

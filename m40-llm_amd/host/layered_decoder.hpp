@@ -1,7 +1,7 @@
 // Decoder that runs a DecoderSpec: bf16 weights in packed tiles, bf16 or f32 activations, an f32 residual stream, a paged cache and, per
 // sequence slot, what recurrent layers carry from token to token.  One step function takes any mixture of sequences and portions (whole
 // prompts, parts of prompts, single tokens); everything that serves or generates goes through it or through the same layer launches
-// replayed from a graph.  The layers themselves: latent_layer.hpp (parallel blocks), output_norm_layer.hpp.
+// replayed from a graph.  The layers themselves: latent_layer.hpp (parallel blocks), output_norm_layer.hpp, stream_layer.hpp.
 #pragma once
 
 #include <algorithm>
@@ -14,6 +14,7 @@
 
 #include "latent_layer.hpp"
 #include "output_norm_layer.hpp"
+#include "stream_layer.hpp"
 #include "served_model.hpp"
 
 namespace m40host {
@@ -214,11 +215,14 @@ private:
         embed_ = table("embed", spec_.vocab);
         if (spec_.bigram) bigram_ = table("bigram", (uint64_t)spec_.bigram->buckets + 1);
         if (spec_.positions) positions_ = table("pos", spec_.positions);
-        if (spec_.block == BlockKind::Parallel) load_parallel(t);
-        else load_output_norm(t);
-        final_norm_ = rt_.upload_f32(t.read_f32("final.norm", {D}));
+        switch (spec_.block) {
+            case BlockKind::Parallel: load_parallel(t); break;
+            case BlockKind::OutputNorm: load_output_norm(t); break;
+            case BlockKind::Streams: load_streams(t); break;
+        }
+        final_norm_ = rt_.upload_norm(t, "final.norm");
         head_ = rt_.packed(round_up(spec_.vocab, 16) / 16, d_tiles);
-        rt_.pack(t, "head", spec_.vocab, D, head_.ptr(), d_tiles, 0);
+        rt_.pack(t, spec_.tied_head ? "embed" : "head", spec_.vocab, D, head_.ptr(), d_tiles, 0);
         rt_.finish_loading();
     }
     void load_parallel(TensorSource& t) {
@@ -259,11 +263,40 @@ private:
             } else {
                 throw std::invalid_argument("layer " + std::to_string(i) + ": this mixer has no form with a norm on its output");
             }
-            std::unique_ptr<FeedForward> ff;
-            if (const auto* m = std::get_if<GatedMlpSpec>(&s.mlp)) ff = std::make_unique<DenseFeedForward>(rt_, t, i, *m);
-            else if (const auto* m = std::get_if<ExpertMlpSpec>(&s.mlp)) ff = std::make_unique<ExpertFeedForward>(rt_, expert, t, i, *m);
-            layers_.push_back(std::make_unique<OutputNormLayer>(rt_, t, i, std::move(mixer), std::move(ff)));
+            layers_.push_back(std::make_unique<OutputNormLayer>(rt_, t, i, std::move(mixer), feed_forward(t, expert, i, s.mlp)));
         }
+    }
+    void load_streams(TensorSource& t) {
+        if (spec_.streams > M40LLM_MOST_STREAMS) throw std::invalid_argument("more residual streams than the kernels serve");
+        auto shared = std::make_shared<StreamShared>();
+        auto expert = std::make_shared<ExpertShared>();
+        rt_.scratch.insert(rt_.scratch.end(), {&shared->queries, &shared->first_values, &shared->recurrent, &shared->low, &shared->low_act, &expert->logits, &expert->ids,
+                                               &expert->weight, &expert->rows_of, &expert->place, &expert->jobs, &expert->rows, &expert->act, &expert->out});
+        shared_ = {shared, expert};
+        streams_ = std::make_unique<ResidualStreams>(rt_);
+        bool values_kept = false;
+        for (const LayerSpec& s : spec_.layers) {
+            const uint32_t i = (uint32_t)layers_.size();
+            std::unique_ptr<Mixer> mixer;
+            if (const auto* a = std::get_if<AttentionSpec>(&s.mixer)) {
+                mixer = std::make_unique<AttentionMixer>(rt_, shared, t, i, *a, a->share_values && values_kept);
+                values_kept = values_kept || a->share_values;
+            } else if (const auto* a = std::get_if<ParallelSpec>(&s.mixer)) {
+                mixer = std::make_unique<ParallelMixer>(rt_, shared, t, i, *a);
+            } else if (const auto* a = std::get_if<ChannelDeltaSpec>(&s.mixer)) {
+                mixer = std::make_unique<ChannelDeltaMixer>(rt_, shared, t, i, *a);
+            } else {
+                throw std::invalid_argument("layer " + std::to_string(i) + ": this mixer has no form over residual streams");
+            }
+            if (const auto* e = std::get_if<ExpertMlpSpec>(&s.mlp); e && e->identity)
+                throw std::invalid_argument("layer " + std::to_string(i) + ": experts that return their input have no form over residual streams");
+            layers_.push_back(std::make_unique<StreamLayer>(rt_, *streams_, t, i, std::move(mixer), feed_forward(t, expert, i, s.mlp)));
+        }
+    }
+    std::unique_ptr<FeedForward> feed_forward(TensorSource& t, const std::shared_ptr<ExpertShared>& expert, uint32_t i, const MlpSpec& mlp) {
+        if (const auto* m = std::get_if<GatedMlpSpec>(&mlp)) return std::make_unique<DenseFeedForward>(rt_, t, i, *m);
+        if (const auto* m = std::get_if<ExpertMlpSpec>(&mlp)) return std::make_unique<ExpertFeedForward>(rt_, expert, t, i, *m);
+        return nullptr;
     }
 
     void allocate() {
@@ -333,10 +366,12 @@ private:
         e.x = rt_.x.ptr();
         if (spec_.block == BlockKind::OutputNorm) { e.h = rt_.h.ptr(); e.ld_h = rt_.d_pad; }
         M40H_TRY(m40llm_ext_embed_tokens_async(ctx_, &e, kStream));
+        if (streams_) streams_->begin();
         for (auto& t : rt_.tables) t->enqueue(r);
     }
     // final norm and head of n of a pass's rows (row_index NULL = all of them)
     void enqueue_logits(const uint32_t* row_index, uint32_t n, uint32_t rows) {
+        if (streams_) streams_->last_sum(row_index, n);
         M40H_TRY(m40llm_ext_norm_rows_async(ctx_, spec_.norm == NormKind::Rms ? M40LLM_NORM_RMS : M40LLM_NORM_LAYER, rt_.x.ptr(), rt_.planes.ptr(), rt_.pending,
                                             (uint64_t)rows * spec_.width, final_norm_.ptr(), row_index, n, spec_.width, spec_.eps, hn_.ptr(), rt_.d_pad,
                                             opt_.act_dtype, kStream));
@@ -546,6 +581,7 @@ private:
     float tie_guard_ = DecodeModel::kGreedyTieGuard;
     bool timed_fallback_ = false;
     std::vector<std::shared_ptr<void>> shared_;       // buffers the layers share
+    std::unique_ptr<ResidualStreams> streams_;        // BlockKind::Streams
     std::vector<std::unique_ptr<DecoderLayer>> layers_;
     size_t state_bytes_ = 0;                          // of a slot, all layers
     DeviceBuf embed_, bigram_, positions_, final_norm_, head_, hn_, logits_, pick_parts_, tables_;

@@ -60,7 +60,7 @@ public:
     DifferentialMixer(LayerRuntime& rt, std::shared_ptr<PairShared> shared, TensorSource& t, uint32_t index, const DifferentialAttentionSpec& a, DifferentialMixer* source)
         : rt_(rt), sh_(std::move(shared)), a_(a), source_(source), portions_(rt.portions()) {
         const std::string p = "l" + std::to_string(index) + ".mix.";
-        most_queries_ = m40llm_ext_pair_attention_tile_queries(rt.opt.act_dtype, a.dim, a.vdim);
+        most_queries_ = m40llm_ext_pair_attention_tile_queries(rt.opt.act_dtype, 2, a.dim, a.vdim);
         if (most_queries_ == 0) throw std::invalid_argument("layer " + std::to_string(index) + ": head sizes beyond what the attention kernels serve");
         const uint32_t q = 2 * a.heads * a.dim, k = 2 * a.kv_heads * a.dim, v = a.kv_heads * a.vdim;
         k_offset_ = round_up(q, 16);
@@ -76,16 +76,16 @@ public:
         if (a.scale < 0.0f)                   // the kernels take the scale's sign from the queries
             for (float& w : q_norm) w = -w;
         q_norm_ = rt.upload_f32(q_norm);
-        if (a.taps) q_conv_ = conv_weights(t, p + "q.conv", q);
+        if (a.taps) q_conv_ = rt.upload_taps(t, p + "q.conv", q, a.taps);
         if (!source) {
             rt.pack(t, p + "k", k, D, w_in_.ptr(), d_tiles, k_offset_ / 16);
             rt.pack(t, p + "v", v, D, w_in_.ptr(), d_tiles, v_offset_ / 16);
             k_norm_ = rt.upload_f32(t.read_f32(p + "k.norm", {a.dim}));
             if (a.taps) {
-                k_conv_ = conv_weights(t, p + "k.conv", k);
-                v_conv_ = conv_weights(t, p + "v.conv", v);
+                k_conv_ = rt.upload_taps(t, p + "k.conv", k, a.taps);
+                v_conv_ = rt.upload_taps(t, p + "v.conv", v, a.taps);
             }
-            cache_ = rt.cleared((size_t)rt.max_pages * m40llm_ext_pair_page_elements(a.kv_heads, a.dim, a.vdim) * rt.es);
+            cache_ = rt.cleared((size_t)rt.max_pages * m40llm_ext_pair_page_elements(2, a.kv_heads, a.dim, a.vdim) * rt.es);
         }
         rt.pack(t, p + "g", a.heads, D, w_in_.ptr(), d_tiles, gate_offset_ / 16);
         w_out_ = rt.packed(round_up(D, 16) / 16, o_pad_ / 32);
@@ -104,7 +104,7 @@ public:
         }
         tiles_ = &rt.table<PairTiles>(a.heads / a.kv_heads, most_queries_);
         tiles_->fewest_kv_heads = std::min(tiles_->fewest_kv_heads, a.kv_heads);
-        tiles_->floats_a_row = std::max(tiles_->floats_a_row, m40llm_ext_pair_attention_partial_floats(1, a.heads, a.vdim, 2) / 2);
+        tiles_->floats_a_row = std::max(tiles_->floats_a_row, m40llm_ext_pair_attention_partial_floats(2, 1, a.heads, a.vdim, 2) / 2);
         rt.proj.want(rt.f32_bytes((size_t)tiles_in_ * 16));
         rt.cat.want(rt.act_bytes(o_pad_));
         sh_->queries.want(rt.act_bytes((size_t)a.heads * 2 * round_up(a.dim, 32)));
@@ -142,7 +142,7 @@ public:
             M40H_TRY(m40llm_ext_conv_state_async(rt_.ctx, rt_.proj.ptr(), ld, conv_cols_, a_.taps, conv_state_.ptr(), conv_cols_, portions_.multi(),
                                                  r.pos, r.multi_row_portions, rt_.kStream));
         M40llmPairAttention h{};
-        h.act_dtype = rt_.opt.act_dtype; h.heads = a_.heads; h.kv_heads = a_.kv_heads; h.dim = a_.dim; h.vdim = a_.vdim;
+        h.act_dtype = rt_.opt.act_dtype; h.maps = 2; h.heads = a_.heads; h.kv_heads = a_.kv_heads; h.dim = a_.dim; h.vdim = a_.vdim;
         h.scale = std::fabs(a_.scale); h.lambda = lambda_; h.out_scale = (float)(1.0 - a_.diff); h.eps = rt_.spec.eps;
         h.queries = sh_->queries.ptr(); h.cache = cache.ptr();
         h.gate = rt_.proj.f32(gate_offset_); h.ld_gate = ld;
@@ -168,14 +168,6 @@ public:
     }
 
 private:
-    // [columns][taps] to [taps][columns]
-    DeviceBuf conv_weights(TensorSource& t, const std::string& name, uint32_t cols) {
-        const std::vector<float> w = t.read_f32(name, {cols, a_.taps});
-        std::vector<float> o(w.size());
-        for (uint32_t c = 0; c < cols; ++c)
-            for (uint32_t j = 0; j < a_.taps; ++j) o[(size_t)j * cols + c] = w[(size_t)c * a_.taps + j];
-        return rt_.upload_f32(o);
-    }
     LayerRuntime& rt_;
     std::shared_ptr<PairShared> sh_;
     DifferentialAttentionSpec a_;
@@ -278,12 +270,27 @@ private:
     DeviceBuf w_in_, norm_, w_out_, decay_, log2_decay_, state_;
 };
 
-// A feed-forward leaves its output in the fields of the norm that adds it to the residual.
+// Where a sublayer leaves its output for the launch that takes it to the residual: in planes, or as the experts' rows.
+struct SublayerOut {
+    const void* planes = nullptr;
+    uint32_t n_planes = 0, top = 0;
+    uint64_t plane_stride = 0;
+    const void* expert_out = nullptr;
+    uint64_t ld_expert = 0;
+    const uint32_t* place = nullptr;
+    const void* weight = nullptr;
+    template <class N>
+    void put(N& n) const {
+        n.planes = planes; n.n_planes = n_planes; n.plane_stride = plane_stride;
+        n.expert_out = expert_out; n.ld_expert = ld_expert; n.place = place; n.weight = weight; n.top = top;
+    }
+};
+
 class FeedForward {
 public:
     virtual ~FeedForward() = default;
-    virtual void enqueue(const Rows& r, M40llmNormAdd& n) = 0;
-    virtual bool reads_plain_rows() const { return false; }      // it wants x as plain rows (h_rows) as well
+    virtual SublayerOut enqueue(const Rows& r) = 0;
+    virtual bool reads_plain_rows() const { return false; }      // it wants its input as plain rows (h_rows) as well
 };
 
 inline uint32_t activation_code(Activation a) { return a == Activation::Silu ? M40LLM_SILU : M40LLM_GELU_TANH; }
@@ -303,7 +310,8 @@ public:
         rt.cat.want(rt.act_bytes(pad_));
         rt.want_planes(pad_ / 32, true);
     }
-    void enqueue(const Rows& r, M40llmNormAdd& n) override {
+    SublayerOut enqueue(const Rows& r) override {
+        SublayerOut n;
         M40llmPackedGemm g = rt_.product(rt_.h.ptr(), rt_.d_pad, w_in_, 2 * tiles_, rt_.d_pad / 32, r.rows, M40LLM_PACKED_PROJECT);
         g.activation = activation_code(m_.activation);
         g.out_act = rt_.cat.ptr(); g.ld_act = pad_;
@@ -311,6 +319,7 @@ public:
         n.planes = rt_.planes.ptr();
         n.n_planes = rt_.into_planes(rt_.product(rt_.cat.ptr(), pad_, w_out_, round_up(rt_.spec.width, 16) / 16, pad_ / 32, r.rows, M40LLM_PACKED_STORE), r.rows);
         n.plane_stride = (uint64_t)r.rows * rt_.spec.width;
+        return n;
     }
 
 private:
@@ -337,7 +346,7 @@ public:
         router_tiles_ = round_up(all, 16) / 16;
         w_router_ = rt.packed(router_tiles_, d_tiles);
         rt.pack(t, p + "router", all, D, w_router_.ptr(), d_tiles, 0);
-        correction_ = rt.upload_f32(t.read_f32(p + "correction", {all}));
+        if (m.correction) correction_ = rt.upload_f32(t.read_f32(p + "correction", {all}));
         const uint32_t down_tiles = round_up(D, 16) / 16;
         w_in_ = rt.packed(m.experts * 2 * tiles_, d_tiles);
         w_out_ = rt.packed(m.experts * down_tiles, pad_ / 32);
@@ -361,7 +370,8 @@ public:
         sh_->out.want((size_t)slots * out_cols_ * rt.es);
     }
     bool reads_plain_rows() const override { return true; }
-    void enqueue(const Rows& r, M40llmNormAdd& n) override {
+    SublayerOut enqueue(const Rows& r) override {
+        SublayerOut n;
         {
             M40llmPackedGemm g = rt_.product(rt_.h.ptr(), rt_.d_pad, w_router_, router_tiles_, rt_.d_pad / 32, r.rows, M40LLM_PACKED_STORE);
             g.out_f32 = sh_->logits.ptr(); g.ld_out = router_tiles_ * 16; g.cols = router_tiles_ * 16;
@@ -370,7 +380,7 @@ public:
         const uint32_t job_rows = rows_a_job(r.rows), max_jobs = m40llm_ext_expert_max_jobs(r.rows, m_.experts, m_.top, job_rows);
         {
             M40llmRoute q{};
-            q.rows = r.rows; q.experts = m_.experts; q.identity = m_.identity; q.top = m_.top; q.job_rows = job_rows;
+            q.rows = r.rows; q.experts = m_.experts; q.identity = m_.identity; q.top = m_.top; q.job_rows = job_rows; q.groups = m_.groups; q.keep = m_.keep; q.scale = m_.scale;
             q.logits = sh_->logits.ptr(); q.ld_logits = router_tiles_ * 16; q.correction = correction_.ptr();
             q.ids = sh_->ids.u32(); q.weight = sh_->weight.ptr();
             q.rows_of = sh_->rows_of.u32(); q.place = sh_->place.u32(); q.jobs = sh_->jobs.u32();
@@ -401,6 +411,7 @@ public:
         }
         n.expert_out = sh_->out.ptr(); n.ld_expert = out_cols_;
         n.place = sh_->place.u32(); n.weight = sh_->weight.ptr(); n.top = m_.top;
+        return n;
     }
 
 private:
@@ -441,7 +452,7 @@ public:
         m.h_rows = ff_ && ff_->reads_plain_rows() ? rt_.h_rows.ptr() : nullptr;
         M40H_TRY(m40llm_ext_norm_add_rows_async(rt_.ctx, &m, rt_.kStream));
         if (!ff_) return;
-        ff_->enqueue(r, n);
+        ff_->enqueue(r).put(n);
         n.w = norm2_.ptr();
         M40H_TRY(m40llm_ext_norm_add_rows_async(rt_.ctx, &n, rt_.kStream));
     }

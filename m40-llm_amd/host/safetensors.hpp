@@ -22,6 +22,8 @@ public:
     virtual void read_bf16(M40llmCudaContext* ctx, const std::string& name, const std::vector<uint64_t>& shape, void* d_dst) = 0;
     // the same to the host, widened
     virtual std::vector<float> read_f32(const std::string& name, const std::vector<uint64_t>& shape) = 0;
+    // rows of a matrix whose size only the tensor itself gives
+    virtual uint64_t rows_of(const std::string& name, uint64_t otherwise) = 0;
 };
 
 inline uint64_t tensor_elements(const std::vector<uint64_t>& shape) {
@@ -76,11 +78,20 @@ public:
         return out;
     }
 
+    uint64_t rows_of(const std::string& name, uint64_t) override {
+        const Entry& e = find(name);
+        if (e.shape.empty() || e.shape[0] == 0 || e.shape[0] > 0xffffffffull) throw json::Error("tensor '" + name + "' has no rows");
+        return e.shape[0];
+    }
+
 private:
-    const Entry& find(const std::string& name, const std::vector<uint64_t>& shape) const {
+    const Entry& find(const std::string& name) const {
         const auto it = entries_.find(name);
         if (it == entries_.end()) throw json::Error("no tensor named '" + name + "'");
-        const Entry& e = it->second;
+        return it->second;
+    }
+    const Entry& find(const std::string& name, const std::vector<uint64_t>& shape) const {
+        const Entry& e = find(name);
         if (e.dtype != "BF16") throw json::Error("tensor '" + name + "' is " + e.dtype + ", not BF16");
         if (e.shape != shape || e.end - e.begin != 2 * tensor_elements(shape)) throw json::Error("tensor '" + name + "' has another shape than config.json gives");
         return e;
@@ -102,6 +113,7 @@ public:
     std::vector<float> read_f32(const std::string&, const std::vector<uint64_t>& shape) override {
         return std::vector<float>(tensor_elements(shape), 1.0f);
     }
+    uint64_t rows_of(const std::string&, uint64_t otherwise) override { return otherwise; }
 
 private:
     uint64_t seed_, count_ = 0;

@@ -146,7 +146,7 @@ def route(ctx, z, correction, experts, top, job_rows):
     keep = []
     ids, weight, rows_of, place, job = (ctx.to_device(np.full(n, 77, t)) for n, t in ((rows * top, np.uint32), (rows * top, np.float32), (slots, np.uint32),
                                                                                       (rows * top, np.uint32), (4 + 4 * jobs, np.uint32)))
-    r = Route(rows=rows, experts=experts, identity=all_ - experts, top=top, job_rows=job_rows, logits=dev(ctx, keep, z, np.float32), ld_logits=all_,
+    r = Route(rows=rows, experts=experts, identity=all_ - experts, top=top, job_rows=job_rows, scale=1.0, logits=dev(ctx, keep, z, np.float32), ld_logits=all_,
               correction=dev(ctx, keep, correction, np.float32), ids=ids.ptr, weight=weight.ptr, rows_of=rows_of.ptr, place=place.ptr, jobs=job.ptr)
     call(ctx, "m40llm_ext_route_rows_async", C.byref(r), 1)
     return (ids.download(np.uint32, (rows, top)), weight.download(np.float32, (rows, top)), rows_of, place, job, slots, jobs, keep)
@@ -235,7 +235,7 @@ class Cache:
 
     def __init__(self, ctx, dtype, G, dim, vdim, slots, max_pages, seed=0):
         ctx.lib.m40llm_ext_pair_page_elements.restype = C.c_uint64
-        self.n = ctx.lib.m40llm_ext_pair_page_elements(G, dim, vdim)
+        self.n = ctx.lib.m40llm_ext_pair_page_elements(2, G, dim, vdim)
         self.max_pages = max_pages
         self.table = np.random.default_rng(seed).permutation(slots * max_pages).astype(np.uint32).reshape(slots, max_pages)
         self.d_table = ctx.to_device(self.table)
@@ -340,11 +340,11 @@ def attend(ctx, dtype, cache, cfg, q, gate, slot, pos, portions, form, splits=1,
     size = 16 if form == 0 else tile_queries
     tiles = [(r * group + i, min(size, n * group - i)) for r, n in portions for i in range(0, n * group, size)]
     ctx.lib.m40llm_ext_pair_attention_partial_floats.restype = C.c_uint64
-    floats = ctx.lib.m40llm_ext_pair_attention_partial_floats(rows, H, vdim, splits)
+    floats = ctx.lib.m40llm_ext_pair_attention_partial_floats(2, rows, H, vdim, splits)
     partial = ctx.alloc(max(floats, 4) * 4)
     ldo = up32(H * vdim)
     out = ctx.to_device(filled((rows + 15) // 16 * 16 * ldo, dtype))
-    a = Attn(act_dtype=ACT[dtype], form=form, heads=H, kv_heads=G, dim=dim, vdim=vdim, scale=scale, out_scale=out_scale, eps=eps,
+    a = Attn(act_dtype=ACT[dtype], maps=2, form=form, heads=H, kv_heads=G, dim=dim, vdim=vdim, scale=scale, out_scale=out_scale, eps=eps,
              queries=dev(ctx, keep, as_act(qq, dtype)), cache=cache.pages.ptr, gate=dev(ctx, keep, gate, np.float32), ld_gate=gate.shape[1],
              row_slot=u32(ctx, keep, slot), row_pos=u32(ctx, keep, pos), page_table=cache.d_table.ptr, max_pages=cache.max_pages, tiles=u32(ctx, keep, tiles),
              n_tiles=len(tiles), tile_queries=tile_queries, splits=splits, first_row=0, n_rows=rows, partial=partial.ptr, partial_floats=floats, out=out.ptr, ld_out=ldo)
@@ -372,7 +372,7 @@ def test_differential_attention_with_one_key_that_stands_out(ctx, dtype, form, s
     """Every query row looks for one key by its first map (far away, at page borders, itself, the first) and for another by its second: what it
     finds is that token's values, less lambda times the other's."""
     if form == 1:
-        most = ctx.lib.m40llm_ext_pair_attention_tile_queries(0, dim, vdim)
+        most = ctx.lib.m40llm_ext_pair_attention_tile_queries(0, 2, dim, vdim)
         if most < tile:
             pytest.skip("these sizes have no such tile")
     rng = np.random.default_rng(dim)
@@ -478,9 +478,9 @@ def test_lightning_recurrence(ctx, dtype, chunked, H, dim, vdim):
 def test_kernels_refuse_what_they_do_not_serve(ctx):
     b = ctx.alloc(1 << 16)
     p = {n: b.ptr for n in ("queries", "cache", "gate", "row_slot", "row_pos", "page_table", "tiles", "out")}
-    ok = dict(heads=2, kv_heads=1, dim=32, vdim=32, scale=1.0, ld_out=64, n_rows=1, n_tiles=1, splits=1, max_pages=1, **p)
+    ok = dict(maps=2, heads=2, kv_heads=1, dim=32, vdim=32, scale=1.0, ld_out=64, n_rows=1, n_tiles=1, splits=1, max_pages=1, **p)
     for bad, rc in ((dict(kv_heads=3), -3), (dict(dim=300), -3), (dict(scale=0.0), -3), (dict(ld_out=32), -3), (dict(form=1, tile_queries=96), -3),
-                    (dict(splits=300), -3), (dict(splits=2), -4), (dict(cache=None), -1)):
+                    (dict(splits=300), -3), (dict(maps=3), -3), (dict(splits=2), -4), (dict(cache=None), -1)):
         call(ctx, "m40llm_ext_pair_attention_async", C.byref(Attn(**dict(ok, **bad))), 1, rc=rc)
     p = {n: b.ptr for n in ("qkv", "decay", "log2_decay", "state", "o", "portions", "row_pos")}
     ok = dict(heads=1, dim=32, vdim=32, ld_qkv=96, ld_o=32, n_portions=1, **p)
