@@ -60,17 +60,14 @@ __global__ __launch_bounds__(1024) void memory_scan_kernel(M40MemoryArgs a) {
         const uint32_t base = (first + c) * kChunk, lo = base > row0 ? base : row0, row = lo + lane;
         const bool in = live && row < end && row < base + kChunk;
         const float i = in ? m40_log_input_gate(a, row, head) : kNever;
-        float sum = in ? m40_log_forget_gate(a, row, head) : 0.0f;
+        float sum = in ? m40_log_forget_gate(a, row, head) : 0.0f, most = i;       // most: the largest log input gate, decayed to this token
 #pragma unroll
         for (int d = 1; d < 64; d *= 2) {
-            const float y = __shfl_up(sum, d);
-            if ((int)lane >= d) sum += y;
-        }
-        float most = i - sum;
-#pragma unroll
-        for (int d = 1; d < 64; d *= 2) {
-            const float y = __shfl_up(most, d);
-            if ((int)lane >= d) most = fmaxf(most, y);
+            const float s = __shfl_up(sum, d), m = __shfl_up(most, d);
+            if ((int)lane >= d) {
+                most = fmaxf(most, m + sum);
+                sum += s;
+            }
         }
         if (lane == 63u) { total[ph][wave] = sum; best[ph][wave] = most; }
         __syncthreads();
@@ -78,13 +75,13 @@ __global__ __launch_bounds__(1024) void memory_scan_kernel(M40MemoryArgs a) {
 #pragma unroll
         for (uint32_t w = 0; w < 16u; ++w) {
             if (w == wave) before = top;
-            if (c0 + w < chunks) top = total[ph][w] + fmaxf(top, best[ph][w]);
+            if (c0 + w < chunks) top = fmaxf(total[ph][w] + top, best[ph][w]);
         }
         if (live) {
             float* gate = block_of(a, chunk0 + c, head) + a.at_gate;
             gate[lane] = sum;
             gate[64 + lane] = i;
-            gate[128 + lane] = sum + fmaxf(before, most);
+            gate[128 + lane] = fmaxf(sum + before, most);
             if (lane == 0u) gate[192] = before;
         }
     }
