@@ -44,6 +44,21 @@ __device__ __forceinline__ m40_float4 mma4(const m40_float4& x, const m40_float4
 __device__ __forceinline__ m40_float4 at4(const float* p) { return *reinterpret_cast<const m40_float4*>(p); }
 __device__ __forceinline__ void put4(float* p, const m40_float4& v) { *reinterpret_cast<m40_float4*>(p) = v; }
 
+// Dimensions d .. d + 3 of a row, zero from dim on: loads under clamped addresses, none behind a branch.  VEC: everything a multiple of 4.
+template <bool VEC>
+__device__ __forceinline__ m40_float4 dims4(const float* row, uint32_t d, uint32_t dim) {
+    m40_float4 v;
+    if (VEC) {
+        v = at4(row + (d < dim ? d : 0u));
+    } else {
+#pragma unroll
+        for (uint32_t r = 0; r < 4; ++r) v[r] = row[d + r < dim ? d + r : 0u];
+    }
+#pragma unroll
+    for (uint32_t r = 0; r < 4; ++r) v[r] = d + r < dim ? v[r] : 0.0f;
+    return v;
+}
+
 // ---- matrix memory: gates.  Part `at_gate` of a block: sums of log forget gates to t [64], log input gates [64], running maxima [64], the maximum
 // before the chunk.
 __global__ __launch_bounds__(1024) void memory_scan_kernel(M40MemoryArgs a) {
@@ -53,14 +68,20 @@ __global__ __launch_bounds__(1024) void memory_scan_kernel(M40MemoryArgs a) {
     const uint32_t first = row0 / kChunk, chunks = (end - 1u) / kChunk - first + 1u, chunk0 = a.chunk_base[blockIdx.x];
     float* m_state = a.state + ((size_t)portion[2] * a.heads + head) * a.head_floats + (size_t)a.dim * a.v4 + a.dim4();
     float top = a.row_pos[row0] == 0u ? 0.0f : *m_state;
-    uint32_t ph = 0;
+    // row of this lane in chunk c, and whether there is one
+    auto row_of = [&](uint32_t c, bool& in) __attribute__((always_inline)) {
+        const uint32_t base = (first + c) * kChunk, row = (base > row0 ? base : row0) + lane;
+        in = c < chunks && row < end && row < base + kChunk;
+        return in ? row : row0;
+    };
+    bool in;
+    uint32_t row = row_of(wave, in), ph = 0;
+    float zi = a.i[(size_t)row * a.ld + head], zf = a.f[(size_t)row * a.ld + head];          // a round ahead
     for (uint32_t c0 = 0; c0 < chunks; c0 += 16u, ph ^= 1u) {
         const uint32_t c = c0 + wave;
         const bool live = c < chunks;
-        const uint32_t base = (first + c) * kChunk, lo = base > row0 ? base : row0, row = lo + lane;
-        const bool in = live && row < end && row < base + kChunk;
-        const float i = in ? m40_log_input_gate(a, row, head) : kNever;
-        float sum = in ? m40_log_forget_gate(a, row, head) : 0.0f, most = i;       // most: the largest log input gate, decayed to this token
+        const float i = in ? m40_log_input_gate(a, zi, head) : kNever;
+        float sum = in ? m40_log_forget_gate(a, zf, head) : 0.0f, most = i;       // most: the largest log input gate, decayed to this token
 #pragma unroll
         for (int d = 1; d < 64; d *= 2) {
             const float s = __shfl_up(sum, d), m = __shfl_up(most, d);
@@ -70,6 +91,9 @@ __global__ __launch_bounds__(1024) void memory_scan_kernel(M40MemoryArgs a) {
             }
         }
         if (lane == 63u) { total[ph][wave] = sum; best[ph][wave] = most; }
+        row = row_of(c + 16u, in);
+        zi = a.i[(size_t)row * a.ld + head];
+        zf = a.f[(size_t)row * a.ld + head];
         __syncthreads();
         float before = top;
 #pragma unroll
@@ -90,9 +114,10 @@ __global__ __launch_bounds__(1024) void memory_scan_kernel(M40MemoryArgs a) {
 
 // queries decayed from the start [64][dp], keys decayed to the end in tile order (key dimensions x tokens), P [64][64], values in tile order (tokens x
 // columns), what is left of S_0 per key dimension
+template <bool VEC>
 __global__ __launch_bounds__(256) void memory_prepare_kernel(M40MemoryArgs a) {
     __shared__ float sum[kChunk], input[kChunk], top[kChunk];
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, li = lane & 15;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, li = lane & 15;
     const Chunk c(a, blockIdx.x);
     const uint32_t head = blockIdx.y, dim = a.dim, n = c.n;
     float* out = block_of(a, blockIdx.x, head);
@@ -105,20 +130,32 @@ __global__ __launch_bounds__(256) void memory_prepare_kernel(M40MemoryArgs a) {
     __syncthreads();
     const float m0 = gate[192], f_end = sum[n - 1u], m_end = top[n - 1u];
     auto row_of = [&](uint32_t t) { return (size_t)(c.row0 + (t < n ? t : n - 1u)) * a.ld; };
-    const bool vec = dim % 4u == 0 && a.ld % 4u == 0 && m40_aligned16(a.q) && m40_aligned16(a.k);
     const float *qh = a.q + (head / a.share) * dim, *kh = a.k + (head / a.share) * dim;
     // scores of this wave's 16 rows with the keys of blocks 0 .. wave
     m40_float4 s[4];
 #pragma unroll
     for (int b = 0; b < 4; ++b) s[b] = m40_float4{0.f, 0.f, 0.f, 0.f};
     const uint32_t t = wave * 16 + li;
-    for (uint32_t d = 4u * g; d < a.dp; d += 16u) {
-        if (d - 4u * g >= dim) break;
-        const uint32_t left = d < dim ? dim - d : 0u;
-        const m40_float4 qf = m40_load4(qh + row_of(t) + d, left, vec);
+    struct Operands { m40_float4 q, k[4]; } even, odd;             // requested a step ahead
+    const float *q_row = qh + row_of(t), *k_row[4] = {kh + row_of(li), kh + row_of(16 + li), kh + row_of(32 + li), kh + row_of(48 + li)};
+    auto load = [&](Operands& f, uint32_t d) __attribute__((always_inline)) {
+        f.q = dims4<VEC>(q_row, d + 4u * g, dim);
+#pragma unroll
+        for (int b = 0; b < 4; ++b) f.k[b] = dims4<VEC>(k_row[b <= wave ? b : 0], d + 4u * g, dim);
+    };
+    auto add = [&](const Operands& f) __attribute__((always_inline)) {
 #pragma unroll
         for (int b = 0; b < 4; ++b)
-            if (b <= wave) s[b] = mma4(m40_load4(kh + row_of(b * 16 + li) + d, left, vec), qf, s[b]);
+            if (b <= wave) s[b] = mma4(f.k[b], f.q, s[b]);
+    };
+    load(even, 0u);
+    for (uint32_t d = 0; d < dim; d += 32u) {
+        load(odd, d + 16u);
+        __builtin_amdgcn_sched_barrier(0);
+        add(even);
+        load(even, d + 32u);
+        __builtin_amdgcn_sched_barrier(0);
+        add(odd);
     }
 #pragma unroll
     for (int b = 0; b < 4; ++b) {
@@ -134,7 +171,7 @@ __global__ __launch_bounds__(256) void memory_prepare_kernel(M40MemoryArgs a) {
     for (uint32_t x = threadIdx.x; x < kChunk * (a.dp / 4u); x += 256u) {
         const uint32_t tt = x / (a.dp / 4u), d = x % (a.dp / 4u) * 4u;
         const float f = tt < n ? a.q_factor * __builtin_amdgcn_exp2f((sum[tt] + m0 - top[tt]) * kM40Log2e) : 0.0f;
-        put4(out + tt * a.dp + d, m40_load4(qh + row_of(tt) + d, d < dim ? dim - d : 0u, vec) * f);
+        put4(out + tt * a.dp + d, dims4<VEC>(qh + row_of(tt), d, dim) * f);
     }
     for (uint32_t x = wave; x < a.dp / 16u * 4u; x += 4u) {
         const uint32_t d = x / 4u * 16u + li;
@@ -161,6 +198,12 @@ __global__ __launch_bounds__(256) void memory_prepare_kernel(M40MemoryArgs a) {
     if (threadIdx.x < a.dp) out[a.at_decay + threadIdx.x] = __builtin_amdgcn_exp2f((f_end + m0 - m_end) * kM40Log2e);
 }
 
+// loads and arithmetic stay on their side
+__device__ __forceinline__ void stay() {
+    asm volatile("" ::: "memory");
+    __builtin_amdgcn_sched_barrier(0);
+}
+
 // ---- delta rule -------------------------------------------------------------------------------------------------------------------------
 constexpr int kSlab = 32, kLdSlab = 36, kLdA = 68;
 struct DeltaLds {
@@ -171,42 +214,58 @@ struct DeltaLds {
     float inverse[4][16][20];                                                  // of I + A's diagonal blocks
     float beta[kChunk];
 };
-__global__ __launch_bounds__(256) void delta_prepare_kernel(M40MemoryArgs a) {
+template <bool VEC>
+__global__ __launch_bounds__(256, 2) void delta_prepare_kernel(M40MemoryArgs a) {
     extern __shared__ __align__(16) uint8_t delta_lds[];
     DeltaLds& lds = *reinterpret_cast<DeltaLds*>(delta_lds);
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, li = lane & 15;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), g = lane >> 4, li = lane & 15;
     const Chunk c(a, blockIdx.x);
     const uint32_t head = blockIdx.y, dim = a.dim, n = c.n;
     float* out = block_of(a, blockIdx.x, head);
     float* W = out + a.at_w;
     auto row_of = [&](uint32_t t) { return c.row0 + (t < n ? t : n - 1u); };
-    const bool vec = dim % 4u == 0 && a.ld % 4u == 0 && m40_aligned16(a.q) && m40_aligned16(a.k);
-    const float *qh = a.q + (head / a.share) * dim, *kh = a.k + (head / a.share) * dim;
     if (tid < kChunk) lds.beta[tid] = tid < (int)n ? m40_sigmoid(a.beta[(size_t)row_of(tid) * a.ld_beta + head]) : 0.0f;
     const float rate = -kM40Log2e * expf(a.A_log[head]);
     float own_a[16], own_p[16];                     // rows of this wave's block with row lane / 4 of it, a quarter of the key dimensions
 #pragma unroll
     for (int t = 0; t < 16; ++t) own_a[t] = own_p[t] = 0.0f;
-    m40_float4 off_a[3], off_p[3];                  // with the rows of the blocks before
+    // rows of a block with those of one before it: six pairs of blocks, waves 0 and 1 for A, waves 2 and 3 for P
+    const int x_of[6] = {1, 2, 2, 3, 3, 3}, y_of[6] = {0, 0, 1, 0, 1, 2};
+    const bool for_p = wave >= 2;
+    const int pair0 = (wave & 1) * 3;
+    m40_float4 off[3];
 #pragma unroll
-    for (int b = 0; b < 3; ++b) off_a[b] = off_p[b] = m40_float4{0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < 3; ++i) off[i] = m40_float4{0.f, 0.f, 0.f, 0.f};
     const int t_in = tid >> 2, d_in = (tid & 3) * 8;
-    for (uint32_t slab = 0; slab < a.dp; slab += kSlab) {
-        {
-            const size_t row = row_of(t_in);
-            const bool live = t_in < (int)n;
+    // a slab's rows, requested a slab ahead
+    struct Rows { m40_float4 k[2], q[2], z[2], bias[2]; } in;
+    const bool live = t_in < (int)n;
+    const size_t row_in = row_of(t_in);
+    const float *k_row = a.k + row_in * a.ld + (head / a.share) * dim, *q_row = a.q + row_in * a.ld + (head / a.share) * dim, *z_row = a.a + row_in * a.ld_a + head * dim,
+                *bias_row = a.dt_bias + head * dim;
+    auto load = [&](uint32_t slab) __attribute__((always_inline)) {
 #pragma unroll
-            for (int h = 0; h < 2; ++h) {
-                const uint32_t d = slab + d_in + 4 * h, left = live && d < dim ? dim - d : 0u;
-                const m40_float4 kk = m40_load4(kh + row * a.ld + d, left, vec), qq = m40_load4(qh + row * a.ld + d, left, vec) * a.q_factor;
-                m40_float4 l;
-#pragma unroll
-                for (uint32_t r = 0; r < 4; ++r) l[r] = r < left ? rate * m40_channel_step(a, (uint32_t)row, head, d + r) : 0.0f;
-                put4(&lds.k[t_in][d_in + 4 * h], kk);
-                put4(&lds.q[t_in][d_in + 4 * h], qq);
-                put4(&lds.l[t_in][d_in + 4 * h], l);
-            }
+        for (int h = 0; h < 2; ++h) {
+            const uint32_t d = slab + d_in + 4 * h;
+            in.k[h] = dims4<VEC>(k_row, d, dim);
+            in.q[h] = dims4<VEC>(q_row, d, dim);
+            in.z[h] = dims4<VEC>(z_row, d, dim);
+            in.bias[h] = dims4<VEC>(bias_row, d, dim);
         }
+    };
+    load(0u);
+    for (uint32_t slab = 0; slab < a.dp; slab += kSlab) {
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+            const uint32_t d = slab + d_in + 4 * h;
+            m40_float4 l;
+#pragma unroll
+            for (uint32_t r = 0; r < 4; ++r) l[r] = live && d + r < dim ? rate * m40_softplus(in.z[h][r] + in.bias[h][r]) : 0.0f;
+            put4(&lds.k[t_in][d_in + 4 * h], in.k[h] * (live ? 1.0f : 0.0f));
+            put4(&lds.q[t_in][d_in + 4 * h], in.q[h] * (live ? a.q_factor : 0.0f));
+            put4(&lds.l[t_in][d_in + 4 * h], l);
+        }
+        load(slab + kSlab);
         __syncthreads();
         if (tid < 4 * kSlab) {
             const int b = tid / kSlab, d = tid % kSlab;
@@ -288,23 +347,22 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(M40MemoryArgs a) {
                         own_p[t] = fmaf(qt[r], e, own_p[t]);
                     }
                 }
+                if (t & 1) stay();                  // operands of two rows at a time in registers
             }
         }
+        const float(*own)[kLdSlab] = for_p ? lds.qe : lds.ke;
 #pragma unroll
-        for (int b = 0; b < 3; ++b) {               // with the rows of block b
-            if (b >= wave) continue;
+        for (int i = 0; i < 3; ++i) {
+            const int x = pair0 ? x_of[3 + i] : x_of[i], y = pair0 ? y_of[3 + i] : y_of[i];
 #pragma unroll
             for (int h = 0; h < 2; ++h) {
                 const int d = h * 16 + 4 * g;
-                m40_float4 f = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                for (int x = 1; x < 3; ++x)
-                    if (x > b && x < wave) f += at4(&lds.whole[x][d]);
+                // decays of the blocks between: at most the second and the third
+                const float f1 = y < 1 && x > 1 ? 1.0f : 0.0f, f2 = y < 2 && x > 2 ? 1.0f : 0.0f;
+                m40_float4 f = at4(&lds.whole[1][d]) * f1 + at4(&lds.whole[2][d]) * f2;
 #pragma unroll
                 for (int r = 0; r < 4; ++r) f[r] = __builtin_amdgcn_exp2f(f[r]);
-                const m40_float4 j = at4(&lds.ks[b * 16 + li][d]);
-                off_a[b] = mma4(j, at4(&lds.ke[wave * 16 + li][d]) * f, off_a[b]);
-                off_p[b] = mma4(j, at4(&lds.qe[wave * 16 + li][d]) * f, off_p[b]);
+                off[i] = mma4(at4(&lds.ks[y * 16 + li][d]), at4(&own[x * 16 + li][d]) * f, off[i]);
             }
         }
         __syncthreads();
@@ -323,12 +381,11 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(M40MemoryArgs a) {
                 out[a.at_p + (wave * 16 + t) * kChunk + wave * 16 + j] = j <= t ? y : 0.0f;
             }
         }
-        const float beta = lds.beta[wave * 16 + li];
 #pragma unroll
-        for (int b = 0; b < 3; ++b) {
-            if (b >= wave) continue;
-            put4(&lds.a[wave * 16 + li][b * 16 + 4 * g], off_a[b] * -beta);
-            put4(out + a.at_p + (wave * 16 + li) * kChunk + b * 16 + 4 * g, off_p[b]);
+        for (int i = 0; i < 3; ++i) {
+            const int x = pair0 ? x_of[3 + i] : x_of[i], y = pair0 ? y_of[3 + i] : y_of[i], t = x * 16 + li;
+            if (for_p) put4(out + a.at_p + t * kChunk + y * 16 + 4 * g, off[i]);
+            else put4(&lds.a[t][y * 16 + 4 * g], off[i] * -lds.beta[t]);
         }
     }
     __syncthreads();
@@ -339,6 +396,7 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(M40MemoryArgs a) {
             x[t] = t == li ? 1.0f : 0.0f;
 #pragma unroll
             for (int j = 0; j < t; ++j) x[t] = fmaf(lds.a[wave * 16 + t][wave * 16 + j], x[j], x[t]);
+            if (t & 1) stay();
         }
         if (g == 0) {
 #pragma unroll
@@ -382,7 +440,7 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(M40MemoryArgs a) {
 }
 
 // ---- the walk ---------------------------------------------------------------------------------------------------------------------------
-// Wave w holds key dimensions 16 DT w .. of 16 value columns.  What a chunk needs is requested while the chunk before it is worked on.
+// Wave w holds key dimensions 16 DT w .. of 16 value columns.
 template <int DT, bool DELTA>
 __global__ __launch_bounds__(256) void memory_walk_kernel(M40MemoryArgs a) {
     __shared__ m40_float4 part[DELTA ? 2 : 1][DELTA ? 4 : 1][4][64];
@@ -404,61 +462,66 @@ __global__ __launch_bounds__(256) void memory_walk_kernel(M40MemoryArgs a) {
         }
     float* block = block_of(a, a.chunk_base[p], head);
     const size_t next = (size_t)a.heads * a.block;
-    m40_float4 wf[DELTA ? 4 : 1][DT], kf[DT][4], u[4], decay[DT];
-    auto load_w = [&](const float* b) __attribute__((always_inline)) {
-        if (!DELTA) return;
+    struct Operands { m40_float4 w[DELTA ? 4 : 1][DT], k[DT][4], u[4], decay[DT]; };
+    auto load = [&](Operands& f, const float* b) __attribute__((always_inline)) {
+        if (DELTA) {
 #pragma unroll
-        for (int t = 0; t < 4; ++t)
+            for (int t = 0; t < 4; ++t)
 #pragma unroll
-            for (int i = 0; i < DT; ++i) wf[DELTA ? t : 0][i] = at4(b + a.at_w + (t * 16 + li) * a.dp + (wave * DT + i) * 16 + 4 * g);
-    };
-    auto load_u = [&](const float* b) __attribute__((always_inline)) {
+                for (int i = 0; i < DT; ++i) f.w[DELTA ? t : 0][i] = at4(b + a.at_w + (t * 16 + li) * a.dp + (wave * DT + i) * 16 + 4 * g);
+        }
 #pragma unroll
-        for (int t = 0; t < 4; ++t) u[t] = at4(b + a.at_u + ((t * a.vt + V) * 64 + lane) * 4);
-    };
-    auto load_k = [&](const float* b) __attribute__((always_inline)) {
+        for (int t = 0; t < 4; ++t) f.u[t] = at4(b + a.at_u + ((t * a.vt + V) * 64 + lane) * 4);
 #pragma unroll
         for (int i = 0; i < DT; ++i) {
-            decay[i] = at4(b + a.at_decay + (wave * DT + i) * 16 + 4 * g);
+            f.decay[i] = at4(b + a.at_decay + (wave * DT + i) * 16 + 4 * g);
 #pragma unroll
-            for (int t = 0; t < 4; ++t) kf[i][t] = at4(b + a.at_k + (((wave * DT + i) * 4 + t) * 64 + lane) * 4);
+            for (int t = 0; t < 4; ++t) f.k[i][t] = at4(b + a.at_k + (((wave * DT + i) * 4 + t) * 64 + lane) * 4);
         }
     };
-    load_w(block);
-    load_u(block);
-    load_k(block);
-    for (uint32_t c = 0; c < chunks; ++c) {
-        const float* ahead = c + 1u < chunks ? block + next : block;
+    auto step = [&](Operands& f, uint32_t c, int phase) __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < DT; ++i) put4(block + a.at_s + (((wave * DT + i) * a.vt + V) * 64 + lane) * 4, S[i]);
         if (DELTA) {
-            m40_float4 read[4];
 #pragma unroll
             for (int t = 0; t < 4; ++t) {
-                read[t] = m40_float4{0.f, 0.f, 0.f, 0.f};
+                m40_float4 read = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                for (int i = 0; i < DT; ++i) read[t] = mma4(wf[DELTA ? t : 0][i], S[i], read[t]);
-                part[DELTA ? c & 1u : 0][DELTA ? wave : 0][t][lane] = read[t];
+                for (int i = 0; i < DT; ++i) read = mma4(f.w[DELTA ? t : 0][i], S[i], read);
+                part[DELTA ? phase : 0][DELTA ? wave : 0][t][lane] = read;
             }
-            load_w(ahead);
             m40_wait_and_meet<63>();
 #pragma unroll
             for (int t = 0; t < 4; ++t)
 #pragma unroll
-                for (int w = 0; w < 4; ++w) u[t] -= part[DELTA ? c & 1u : 0][DELTA ? w : 0][t][lane];
+                for (int w = 0; w < 4; ++w) f.u[t] -= part[DELTA ? phase : 0][DELTA ? w : 0][t][lane];
 #pragma unroll
             for (int t = 0; t < 4; ++t)
-                if (t == wave) put4(block + a.at_u + ((t * a.vt + V) * 64 + lane) * 4, u[t]);
+                if (t == wave) put4(block + a.at_u + ((t * a.vt + V) * 64 + lane) * 4, f.u[t]);
         }
 #pragma unroll
         for (int i = 0; i < DT; ++i) {
-            S[i] *= decay[i];
+            S[i] *= f.decay[i];
 #pragma unroll
-            for (int t = 0; t < 4; ++t) S[i] = mma4(kf[i][t], u[t], S[i]);
+            for (int t = 0; t < 4; ++t) S[i] = mma4(f.k[i][t], f.u[t], S[i]);
         }
-        load_u(ahead);
-        load_k(ahead);
         block += next;
+    };
+    // the operands of the next chunk are requested before the current one is worked on; wide heads have registers for one set only
+    constexpr bool kAhead = DT <= 2;
+    Operands even, odd;
+    load(even, block);
+    for (uint32_t c = 0; c < chunks; c += 2u) {
+        const bool more = c + 1u < chunks;
+        if (kAhead) load(odd, more ? block + next : block);
+        __builtin_amdgcn_sched_barrier(0);
+        step(even, c, 0);
+        if (!more) break;
+        if (!kAhead) load(odd, block);
+        if (kAhead) load(even, c + 2u < chunks ? block + next : block);
+        __builtin_amdgcn_sched_barrier(0);
+        step(odd, c + 1u, 1);
+        if (!kAhead && c + 2u < chunks) load(even, block);
     }
     if (!stored) return;
 #pragma unroll
@@ -482,17 +545,31 @@ __global__ __launch_bounds__(256) void memory_outputs_kernel(M40MemoryArgs a) {
     m40_float4 o[VT];
 #pragma unroll
     for (int j = 0; j < VT; ++j) o[j] = m40_float4{0.f, 0.f, 0.f, 0.f};
-    for (uint32_t d = 0; d < (a.dim + 15u) / 16u; ++d) {
-        const m40_float4 q = at4(block + t * a.dp + d * 16 + 4 * g);
+    // 16 key dimensions of the state a step, then 16 of the chunk's tokens; operands are requested a step ahead
+    const int d_steps = (int)(a.dim + 15u) / 16, steps = d_steps + wave + 1;
+    struct Operands { m40_float4 x, y[VT]; } even, odd;
+    auto load = [&](Operands& f, int n) __attribute__((always_inline)) {
+        n = n < steps ? n : steps - 1;
+        const bool state = n < d_steps;
+        const float* tiles = block + (state ? a.at_s + n * vt * 256 : a.at_u + (n - d_steps) * vt * 256) + lane * 4;
+        f.x = at4(state ? block + t * a.dp + n * 16 + 4 * g : block + a.at_p + t * kChunk + (n - d_steps) * 16 + 4 * g);
+#pragma unroll
+        for (int j = 0; j < VT; ++j) f.y[j] = at4(tiles + (j < vt ? j : vt - 1) * 256);
+    };
+    auto add = [&](const Operands& f) __attribute__((always_inline)) {
 #pragma unroll
         for (int j = 0; j < VT; ++j)
-            if (j < vt) o[j] = mma4(at4(block + a.at_s + ((d * vt + j) * 64 + lane) * 4), q, o[j]);
-    }
-    for (int b = 0; b <= wave; ++b) {
-        const m40_float4 p = at4(block + a.at_p + t * kChunk + b * 16 + 4 * g);
-#pragma unroll
-        for (int j = 0; j < VT; ++j)
-            if (j < vt) o[j] = mma4(at4(block + a.at_u + ((b * vt + j) * 64 + lane) * 4), p, o[j]);
+            if (j < vt) o[j] = mma4(f.y[j], f.x, o[j]);
+    };
+    load(even, 0);
+    for (int n = 0; n < steps; n += 2) {
+        load(odd, n + 1);
+        __builtin_amdgcn_sched_barrier(0);
+        add(even);
+        if (n + 1 >= steps) break;
+        load(even, n + 2);
+        __builtin_amdgcn_sched_barrier(0);
+        add(odd);
     }
     const int vdim = (int)a.vdim;
     float f = 1.0f;
@@ -541,13 +618,18 @@ void walk(hipStream_t stream, const M40MemoryArgs& a, uint32_t n_portions) {
 }
 template <bool DELTA>
 int chunked(hipStream_t stream, const M40MemoryArgs& a, uint32_t n_portions, uint32_t n_chunks) {
+    const bool vec = a.dim % 4u == 0 && a.ld % 4u == 0 && a.ld_a % 4u == 0 && m40_aligned16(a.q) && m40_aligned16(a.k) && m40_aligned16(a.a) && m40_aligned16(a.dt_bias);
+    const dim3 grid(n_chunks, a.heads);
     if constexpr (DELTA) {
-        static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(delta_prepare_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)sizeof(DeltaLds));
-        if (attr != hipSuccess) return -2;
-        delta_prepare_kernel<<<dim3(n_chunks, a.heads), 256, sizeof(DeltaLds), stream>>>(a);
+        static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(delta_prepare_kernel<true>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)sizeof(DeltaLds)),
+                                attr2 = hipFuncSetAttribute(reinterpret_cast<const void*>(delta_prepare_kernel<false>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)sizeof(DeltaLds));
+        if (attr != hipSuccess || attr2 != hipSuccess) return -2;
+        if (vec) delta_prepare_kernel<true><<<grid, 256, sizeof(DeltaLds), stream>>>(a);
+        else delta_prepare_kernel<false><<<grid, 256, sizeof(DeltaLds), stream>>>(a);
     } else {
         memory_scan_kernel<<<dim3(n_portions, a.heads), 1024, 0, stream>>>(a);
-        memory_prepare_kernel<<<dim3(n_chunks, a.heads), 256, 0, stream>>>(a);
+        if (vec) memory_prepare_kernel<true><<<grid, 256, 0, stream>>>(a);
+        else memory_prepare_kernel<false><<<grid, 256, 0, stream>>>(a);
     }
     switch (a.dp / 64u) {
         case 1: walk<1, DELTA>(stream, a, n_portions); break;
@@ -555,8 +637,8 @@ int chunked(hipStream_t stream, const M40MemoryArgs& a, uint32_t n_portions, uin
         case 3: walk<3, DELTA>(stream, a, n_portions); break;
         default: walk<4, DELTA>(stream, a, n_portions); break;
     }
-    const dim3 grid(n_chunks, a.heads);
     if (a.vt <= 4u) memory_outputs_kernel<4, DELTA><<<grid, 256, 0, stream>>>(a);
+    else if (a.vt <= 8u) memory_outputs_kernel<8, DELTA><<<grid, 256, 0, stream>>>(a);
     else if (a.vt <= 9u) memory_outputs_kernel<9, DELTA><<<grid, 256, 0, stream>>>(a);
     else memory_outputs_kernel<17, DELTA><<<grid, 256, 0, stream>>>(a);
     return hipGetLastError() == hipSuccess ? 0 : -2;

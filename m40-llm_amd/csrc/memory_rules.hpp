@@ -32,13 +32,15 @@ struct M40MemoryArgs {
 #ifdef __HIPCC__
 constexpr float kM40Log2e = 1.4426950408889634f;
 __device__ __forceinline__ float m40_soft_cap(float z, float cap) { return cap * tanhf(z / cap); }
-__device__ __forceinline__ float m40_softplus(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
-__device__ __forceinline__ float m40_log_input_gate(const M40MemoryArgs& a, uint32_t row, uint32_t head) {
-    return m40_soft_cap(a.i[(size_t)row * a.ld + head] + a.i_bias[head], a.cap);
+// log(1 + e^z): max(z, 0) + log(1 + y) with y = e^-|z|, the logarithm by its series where 1 + y would round y off
+__device__ __forceinline__ float m40_softplus(float z) {
+    const float y = __builtin_amdgcn_exp2f(-fabsf(z) * kM40Log2e);
+    const float series = y * fmaf(-y, fmaf(-y, fmaf(-y, 0.25f, 1.0f / 3.0f), 0.5f), 1.0f);
+    return fmaxf(z, 0.0f) + (y < 0.03125f ? series : __builtin_amdgcn_logf(1.0f + y) * 0.6931471805599453f);
 }
-__device__ __forceinline__ float m40_log_forget_gate(const M40MemoryArgs& a, uint32_t row, uint32_t head) {
-    return -m40_softplus(-m40_soft_cap(a.f[(size_t)row * a.ld + head] + a.f_bias[head], a.cap));
-}
+// logits of a row's gates
+__device__ __forceinline__ float m40_log_input_gate(const M40MemoryArgs& a, float z, uint32_t head) { return m40_soft_cap(z + a.i_bias[head], a.cap); }
+__device__ __forceinline__ float m40_log_forget_gate(const M40MemoryArgs& a, float z, uint32_t head) { return -m40_softplus(-m40_soft_cap(z + a.f_bias[head], a.cap)); }
 // minus the log of a key channel's decay, less the head's factor exp(A_log)
 __device__ __forceinline__ float m40_channel_step(const M40MemoryArgs& a, uint32_t row, uint32_t head, uint32_t d) {
     return m40_softplus(a.a[(size_t)row * a.ld_a + head * a.dim + d] + a.dt_bias[head * a.dim + d]);

@@ -51,7 +51,7 @@ __global__ __launch_bounds__(kThreads) void memory_serial_kernel(M40MemoryArgs a
         if (DELTA) {
             beta = m40_sigmoid(a.beta[(size_t)row * a.ld_beta + head]);
         } else {
-            const float i = m40_log_input_gate(a, row, head), f = m40_log_forget_gate(a, row, head), next = fmaxf(f + top, i);
+            const float i = m40_log_input_gate(a, a.i[(size_t)row * a.ld + head], head), f = m40_log_forget_gate(a, a.f[(size_t)row * a.ld + head], head), next = fmaxf(f + top, i);
             keep = expf(f + top - next);
             add = expf(i - next);
             top = next;

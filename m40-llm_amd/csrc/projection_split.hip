@@ -1,7 +1,7 @@
 // Steps between a mixer's projections and what it does with them.
 //
 // qkv_split_kernel     attention of one map a head: biases, RMS norm over whole projections, rotation, values mixed with another layer's;
-//                      queries out, keys and values to the cache.  A workgroup a row.
+//                      queries out, keys and values to the cache.  A workgroup a row, or several for few rows (each forms the norms).
 // delta_split_kernel   delta rule: short convolution and silu, queries and keys as unit vectors; f32 rows out.  A workgroup takes 16 rows of
 //                      one head.
 #include "packed_gemm.hpp"
@@ -96,9 +96,9 @@ __global__ __launch_bounds__(kThreads) void qkv_split_kernel(M40llmQkvSplit a, M
             y[0] = at & 1u ? fmaf(v.v[0], cs.x, w * cs.y) : fmaf(v.v[0], cs.x, -(w * cs.y));
         }
     };
-    const uint32_t k_pad = page.k_tiles * 32u, v_pad = page.v_tiles * 16u;
+    const uint32_t k_pad = page.k_tiles * 32u, v_pad = page.v_tiles * 16u, first = (blockIdx.y * kThreads + tid) * W;
     T* q = static_cast<T*>(a.queries) + (size_t)row * a.heads * k_pad;
-    for (uint32_t i = tid * W; i < a.heads * k_pad; i += kThreads * W) {
+    for (uint32_t i = first; i < a.heads * k_pad; i += kThreads * W * gridDim.y) {
         float y[W];
         turned(0u, a.q_bias, a.q_norm, q_inv * a.q_factor, i / k_pad, i % k_pad, y);
         if (!a.q_norm) {
@@ -108,13 +108,13 @@ __global__ __launch_bounds__(kThreads) void qkv_split_kernel(M40llmQkvSplit a, M
         m40_store_columns<T, W>(q + i, y);
     }
     T* cache = static_cast<T*>(a.cache) + number * page.elements();
-    for (uint32_t i = tid * W; i < a.kv_heads * k_pad; i += kThreads * W) {
+    for (uint32_t i = first; i < a.kv_heads * k_pad; i += kThreads * W * gridDim.y) {
         float y[W];
         turned(a.k_offset, a.k_bias, a.k_norm, k_inv, i / k_pad, i % k_pad, y);
         m40_store_columns<T, W>(cache + i / k_pad * page.head_elements() + page.key_at(0u, t, i % k_pad), y);
     }
     const float lambda = a.lambda;
-    for (uint32_t i = tid * W; i < a.kv_heads * v_pad; i += kThreads * W) {
+    for (uint32_t i = first; i < a.kv_heads * v_pad; i += kThreads * W * gridDim.y) {
         const uint32_t unit = i / v_pad, at = i % v_pad, c = unit * a.vdim + at;
         T* to = cache + unit * page.head_elements();
         M40Columns<W> v{};
@@ -194,13 +194,16 @@ int m40llm_ext_qkv_split_append_async(M40llmCudaContext* ctx, const M40llmQkvSpl
     bool vec = s->dim % 4u == 0 && s->vdim % 4u == 0 && s->ld_proj % 4u == 0 && s->k_offset % 4u == 0 && s->v_offset % 4u == 0 && s->ld_values % 4u == 0;
     for (const void* p : {s->proj, s->q_bias, s->k_bias, s->v_bias, s->q_norm, s->k_norm, s->first_values, static_cast<const void*>(s->keep_values)})
         vec = vec && m40_aligned16(p);
+    // parts of a row's queries
+    const uint32_t most = (s->heads * page.k_tiles * 32u + 1023u) / 1024u, parts = s->rows > 64u ? 1u : most < 8u ? most : 8u;
+    const dim3 grid(s->rows, parts);
     (void)hipGetLastError();
     if (s->act_dtype == M40LLM_ACT_F32) {
-        if (vec) qkv_split_kernel<float, 4><<<s->rows, kThreads, 0, stream>>>(*s, page);
-        else qkv_split_kernel<float, 1><<<s->rows, kThreads, 0, stream>>>(*s, page);
+        if (vec) qkv_split_kernel<float, 4><<<grid, kThreads, 0, stream>>>(*s, page);
+        else qkv_split_kernel<float, 1><<<grid, kThreads, 0, stream>>>(*s, page);
     } else {
-        if (vec) qkv_split_kernel<m40_bf16, 4><<<s->rows, kThreads, 0, stream>>>(*s, page);
-        else qkv_split_kernel<m40_bf16, 1><<<s->rows, kThreads, 0, stream>>>(*s, page);
+        if (vec) qkv_split_kernel<m40_bf16, 4><<<grid, kThreads, 0, stream>>>(*s, page);
+        else qkv_split_kernel<m40_bf16, 1><<<grid, kThreads, 0, stream>>>(*s, page);
     }
     return launched();
 }

@@ -49,6 +49,19 @@ __global__ __launch_bounds__(kThreads) void stream_update_kernel(M40llmStreamUpd
     const float* x0 = a.x0 ? static_cast<const float*>(a.x0) + (size_t)row * width : nullptr;
     float* xs = static_cast<float*>(a.streams_x) + (size_t)row * width;
     const bool write = a.place || a.n_planes;
+    // up to four streams: all coefficients in registers before anything is stored
+    constexpr bool kFew = S <= 4;
+    float mx[kFew ? S : 1][kFew ? S : 1], sh[kFew ? S : 1], tk[kFew ? S : 1];
+    if (kFew) {
+#pragma unroll
+        for (int t = 0; t < S; ++t) {
+            tk[kFew ? t : 0] = take ? take[t] : 1.0f;
+            sh[kFew ? t : 0] = write ? a.mult * share[t] : 0.0f;
+#pragma unroll
+            for (int s = 0; s < S; ++s) mx[kFew ? s : 0][kFew ? t : 0] = write ? mix[s * S + t] : 0.0f;
+        }
+    }
+    auto taken = [&](uint32_t t) __attribute__((always_inline)) { return kFew ? tk[kFew ? t : 0] : take ? take[t] : 1.0f; };
     auto old = [&](uint32_t s, uint32_t g, float (&v)[8]) __attribute__((always_inline)) {
         load8<float, VEC>(x0 ? x0 : xs + s * (size_t)a.stream_stride, g * 8u, width, v);
     };
@@ -87,13 +100,13 @@ __global__ __launch_bounds__(kThreads) void stream_update_kernel(M40llmStreamUpd
             if (t >= streams) continue;
             float z[8];
             if (write) {
-                const float f = a.mult * share[t];
+                const float f = kFew ? sh[kFew ? t : 0] : a.mult * share[t];
 #pragma unroll
                 for (int i = 0; i < 8; ++i) z[i] = f * y[i];
 #pragma unroll
                 for (uint32_t s = 0; s < S; ++s)
                     if (s < streams) {
-                        const float m = mix[s * streams + t];
+                        const float m = kFew ? mx[kFew ? s : 0][kFew ? t : 0] : mix[s * streams + t];
 #pragma unroll
                         for (int i = 0; i < 8; ++i) z[i] = fmaf(m, x[s][i], z[i]);
                     }
@@ -102,7 +115,7 @@ __global__ __launch_bounds__(kThreads) void stream_update_kernel(M40llmStreamUpd
 #pragma unroll
                 for (int i = 0; i < 8; ++i) z[i] = x[t][i];
             }
-            const float f = take ? take[t] : 1.0f;
+            const float f = taken(t);
 #pragma unroll
             for (int i = 0; i < 8; ++i) u[i] = fmaf(f, z[i], u[i]);
         }

@@ -1,6 +1,7 @@
 """Prefill and decode throughput of layered decoders with random weights beside the framework's closest other model of the same width,
 depth and vocabulary.  `bench.py --design NAME` prints what measure() returns: the Pimosun design beside the dense decoder, the Gulidra
-design beside Pimosun, whose feed-forward is as wide as the experts a token takes together.
+design beside Pimosun, whose feed-forward is as wide as the experts a token takes together, the Natatar design beside Gulidra with the same
+experts in every layer.
 
 A case is one shape on one kind of step: a prompt of n tokens run in one step (host clock around the blocking call, the last
 token's logits included), or `batch` sequences of `context` tokens that decode greedily from a replayed graph (timed between
@@ -16,7 +17,7 @@ pkg = importlib.import_module(__package__)
 syn = importlib.import_module(__package__ + ".synthetic")
 layered = importlib.import_module(__package__ + ".layered")
 
-BESIDE = dict(pimosun="Pimosun beside the dense decoder", gulidra="Gulidra beside Pimosun")
+BESIDE = dict(pimosun="Pimosun beside the dense decoder", gulidra="Gulidra beside Pimosun", natatar="Natatar beside Gulidra")
 SHAPES = {
     # name: layered decoder, and the dense decoder's heads at the same width
     "2k": dict(width=2048, heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=768, ff=5632, vocab=32000, layers=8, kv_heads=2),
@@ -45,13 +46,16 @@ GULIDRA = {
 }
 
 
-def gulidra_config(name: str) -> dict:
+def gulidra_config(name: str, routed=False) -> dict:
+    """routed: experts in every layer, none of them the identity."""
     s, g = SHAPES[name], GULIDRA[name]
     mixer = dict(heads=s["heads"], kv_heads=g["kv_heads"], dim=g["dim"], vdim=s["vdim"], conv=g["conv"], diff=0.3, scale=float(g["dim"] ** -0.5))
     heads, dim, vdim = g["light"]
     light = dict(heads=heads, dim=dim, vdim=vdim, decay=[float(1 - 2.0 ** -(2 + 8 * i / heads)) for i in range(heads)])
     moe = dict(kind="moe", expert=dict(ff=g["expert_ff"]), router=dict(experts=g["experts"], identity=g["identity"], top=g["top"]))
-    dense = dict(kind="dense", ff=s["ff"])
+    if routed:
+        moe["router"]["identity"] = 0
+    dense = moe if routed else dict(kind="dense", ff=s["ff"])
     layers = []
     for i in range(s["layers"]):
         mlp = moe if i % 2 else dense
@@ -61,6 +65,28 @@ def gulidra_config(name: str) -> dict:
             layers.append(dict(type="attention", mixer=dict(mixer, **({"kv_from": i - 2} if i % 4 == 2 else {})), mlp=mlp))
     return dict(architecture="Gulidra", vocab=s["vocab"], width=s["width"], norm=dict(eps=1e-5), embedding=dict(scale=1.0), residual_mult=0.7,
                 max_positions=8192, layers=layers)
+
+
+# Natatar at the same sizes: of four layers one with attention beside a matrix memory, two of attention, one of the delta rule; four streams
+NATATAR = {
+    "2k": dict(streams=4, kv_heads=4, dim=128, conv=4, experts=32, top=4, expert_ff=1408, groups=(8, 4), memory=(16, 128, 128), delta=(16, 16, 128, 128)),
+    "4k": dict(streams=4, kv_heads=8, dim=128, conv=4, experts=32, top=4, expert_ff=2752, groups=(8, 4), memory=(32, 128, 128), delta=(32, 32, 128, 128)),
+}
+
+
+def natatar_config(name: str) -> dict:
+    s, g = SHAPES[name], NATATAR[name]
+    mixer = dict(heads=s["heads"], kv_heads=g["kv_heads"], dim=g["dim"], vdim=s["vdim"], scale=float(g["dim"] ** -0.5))
+    rot = dict(base=500000.0, dims=g["dim"], scaling=dict(factor=8.0, original=4096, fast=32.0, slow=1.0))
+    h, d, v = g["memory"]
+    parallel = dict(left=dict(mixer, rot=rot), left_scale=0.7, right=dict(heads=h, dim=d, vdim=v, gate_cap=12.0), right_scale=1.1)
+    h, k, d, v = g["delta"]
+    delta = dict(heads=h, kv_heads=k, dim=d, vdim=v, conv=g["conv"])
+    kinds = [dict(type="parallel", mixer=parallel), dict(type="attention", mixer=dict(mixer, v_mix=True)), dict(type="channel_delta", mixer=delta),
+             dict(type="attention", mixer=dict(mixer, v_mix=True))]
+    moe = dict(kind="moe", expert=dict(ff=g["expert_ff"]), router=dict(experts=g["experts"], top=g["top"], scale=2.0, groups=dict(count=g["groups"][0], keep=g["groups"][1])))
+    return dict(architecture="Natatar", vocab=s["vocab"], width=s["width"], streams=g["streams"], norm=dict(eps=1e-5), embedding=dict(scale=1.0), residual_mult=0.3,
+                layers=[dict(kinds[i % 4], mlp=moe) for i in range(s["layers"])])
 
 
 def layer_flops_per_token(s: dict, own: bool) -> float:
@@ -141,6 +167,12 @@ def dense_cases(ctx, s, prefill=PREFILL, decode=DECODE, reps=3, steps=32, warmup
 
 def measure(ctx, shapes=None, steps=32, warmup=4, dense=True, design="pimosun") -> dict:
     out = {}
+    if design == "natatar":
+        for name in shapes or SHAPES:
+            s = SHAPES[name]
+            out[name] = {"shape": dict(s, **NATATAR[name]), "natatar": layered_cases(ctx, s, steps=steps, warmup=warmup, cfg=natatar_config(name)),
+                         "gulidra": layered_cases(ctx, s, steps=steps, warmup=warmup, cfg=gulidra_config(name, routed=True))}
+        return out
     if design == "gulidra":
         for name in shapes or SHAPES:
             s = SHAPES[name]
