@@ -17,8 +17,9 @@
 // memory_outputs_kernel   all chunks at once: outputs, the head's norm, the gate
 //
 // Operands: lane l = 16 g + i of a 16x16x4 f32 instruction holds element (i, g) of either operand and elements (4 g + r, i) of the sums.  Four
-// instructions take k = 4 g + r in turn, so four neighbouring floats of a row are the lane's operands, and a tile of sums is, as it lies, the
-// second operand of 16 more: states and u go from sums to memory to operands in "tile order" [tile][lane][4].
+// instructions take k = 4 g + r in turn, so a lane's operands are four neighbouring floats of row i, and a tile of sums is, as it lies, the
+// second operand of four more.  Everything goes through memory in "tile order" [tile][lane][4], tiles of 16 x 16, so that a wave's load is a
+// contiguous kilobyte and already an operand.
 #include "memory_launch.hpp"
 
 namespace {
@@ -43,6 +44,9 @@ __device__ __forceinline__ m40_float4 mma4(const m40_float4& x, const m40_float4
 }
 __device__ __forceinline__ m40_float4 at4(const float* p) { return *reinterpret_cast<const m40_float4*>(p); }
 __device__ __forceinline__ void put4(float* p, const m40_float4& v) { *reinterpret_cast<m40_float4*>(p) = v; }
+
+// four columns from d on (a multiple of 4) of row t of a matrix in tile order whose rows have `tiles` tiles
+__device__ __forceinline__ size_t tile_at(uint32_t t, uint32_t d, uint32_t tiles) { return (((t >> 4) * tiles + (d >> 4)) * 64u + (d >> 2 & 3u) * 16u + (t & 15u)) * 4u; }
 
 // Dimensions d .. d + 3 of a row, zero from dim on: loads under clamped addresses, none behind a branch.  VEC: everything a multiple of 4.
 template <bool VEC>
@@ -112,7 +116,7 @@ __global__ __launch_bounds__(1024) void memory_scan_kernel(M40MemoryArgs a) {
     if (threadIdx.x == 0u) *m_state = top;
 }
 
-// queries decayed from the start [64][dp], keys decayed to the end in tile order (key dimensions x tokens), P [64][64], values in tile order (tokens x
+// queries decayed from the start (tokens x key dimensions), keys decayed to the end (key dimensions x tokens), P (tokens x tokens), values (tokens x
 // columns), what is left of S_0 per key dimension
 template <bool VEC>
 __global__ __launch_bounds__(256) void memory_prepare_kernel(M40MemoryArgs a) {
@@ -166,12 +170,12 @@ __global__ __launch_bounds__(256) void memory_prepare_kernel(M40MemoryArgs a) {
             const uint32_t j = b * 16 + 4 * g + r;
             p[r] = j <= t && t < n ? s[b][r] * a.q_factor * __builtin_amdgcn_exp2f((sum[t] - sum[j] + input[j] - top[t]) * kM40Log2e) : 0.0f;
         }
-        put4(out + a.at_p + t * kChunk + b * 16 + 4 * g, p);
+        put4(out + a.at_p + ((wave * 4 + b) * 64 + lane) * 4, p);
     }
-    for (uint32_t x = threadIdx.x; x < kChunk * (a.dp / 4u); x += 256u) {
-        const uint32_t tt = x / (a.dp / 4u), d = x % (a.dp / 4u) * 4u;
+    for (uint32_t x = wave; x < a.dp / 4u; x += 4u) {            // 16 x 16 tiles: 4 dp / 16 of them
+        const uint32_t tt = x / (a.dp / 16u) * 16u + li, d = x % (a.dp / 16u) * 16u + 4u * g;
         const float f = tt < n ? a.q_factor * __builtin_amdgcn_exp2f((sum[tt] + m0 - top[tt]) * kM40Log2e) : 0.0f;
-        put4(out + tt * a.dp + d, dims4<VEC>(qh + row_of(tt), d, dim) * f);
+        put4(out + (x * 64 + lane) * 4, dims4<VEC>(qh + row_of(tt), d, dim) * f);
     }
     for (uint32_t x = wave; x < a.dp / 16u * 4u; x += 4u) {
         const uint32_t d = x / 4u * 16u + li;
@@ -314,8 +318,9 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(M40MemoryArgs a) 
             for (int h = 0; h < 2; ++h) {
                 const int d = d_in + 4 * h;
                 const m40_float4 f = at4(&lds.start[b][d]);
-                put4(out + t_in * a.dp + slab + d, at4(&lds.qe[t_in][d]) * f);
-                put4(W + t_in * a.dp + slab + d, at4(&lds.ke[t_in][d]) * f * beta);
+                const size_t at = tile_at(t_in, slab + d, a.dp / 16u);
+                put4(out + at, at4(&lds.qe[t_in][d]) * f);
+                put4(W + at, at4(&lds.ke[t_in][d]) * f * beta);
             }
 #pragma unroll
             for (int h = 0; h < 2; ++h) {           // block `wave` of tokens, 16 dimensions
@@ -378,13 +383,13 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(M40MemoryArgs a) 
             y += m40_dpp_f<M40_DPP_XOR2>(y);
             if ((lane & 3) == (t & 3)) {
                 lds.a[wave * 16 + t][wave * 16 + j] = j < t ? -lds.beta[wave * 16 + t] * x : 0.0f;
-                out[a.at_p + (wave * 16 + t) * kChunk + wave * 16 + j] = j <= t ? y : 0.0f;
+                out[a.at_p + tile_at(wave * 16 + t, wave * 16 + (j & 12), 4u) + (j & 3)] = j <= t ? y : 0.0f;
             }
         }
 #pragma unroll
         for (int i = 0; i < 3; ++i) {
             const int x = pair0 ? x_of[3 + i] : x_of[i], y = pair0 ? y_of[3 + i] : y_of[i], t = x * 16 + li;
-            if (for_p) put4(out + a.at_p + t * kChunk + y * 16 + 4 * g, off[i]);
+            if (for_p) put4(out + a.at_p + ((x * 4 + y) * 64 + lane) * 4, off[i]);
             else put4(&lds.a[t][y * 16 + 4 * g], off[i] * -lds.beta[t]);
         }
     }
@@ -413,7 +418,7 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(M40MemoryArgs a) 
             for (int r = 0; r < 4; ++r) {
                 const uint32_t t = b * 16 + 4 * g + r;
                 if (x < w_tiles) {
-                    X[b][r] = W[t * a.dp + x * 16u + li];
+                    X[b][r] = W[tile_at(t, x * 16u + (li & 12), w_tiles) + (li & 3)];
                 } else {
                     const uint32_t v = (x - w_tiles) * 16u + li;
                     const float y = a.v[(size_t)row_of(t) * a.ld + head * a.vdim + (v < a.vdim ? v : 0u)];
@@ -431,7 +436,7 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(M40MemoryArgs a) 
         for (int b = 0; b < 4; ++b) {
             if (x < w_tiles) {
 #pragma unroll
-                for (int r = 0; r < 4; ++r) W[(b * 16 + 4 * g + r) * a.dp + x * 16u + li] = X[b][r];
+                for (int r = 0; r < 4; ++r) W[tile_at(b * 16 + 4 * g + r, x * 16u + (li & 12), w_tiles) + (li & 3)] = X[b][r];
             } else {
                 put4(out + a.at_u + ((b * a.vt + x - w_tiles) * 64 + lane) * 4, X[b]);
             }
@@ -440,10 +445,10 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(M40MemoryArgs a) 
 }
 
 // ---- the walk ---------------------------------------------------------------------------------------------------------------------------
-// Wave w holds key dimensions 16 DT w .. of 16 value columns.
-template <int DT, bool DELTA>
-__global__ __launch_bounds__(256) void memory_walk_kernel(M40MemoryArgs a) {
-    __shared__ m40_float4 part[DELTA ? 2 : 1][DELTA ? 4 : 1][4][64];
+// Wave w holds key dimensions 16 DT w .. of 16 value columns.  A chunk's operands are requested SETS - 1 chunks ahead.
+template <int WAVES, int DT, int SETS, bool DELTA>
+__global__ __launch_bounds__(WAVES * 64) void memory_walk_kernel(M40MemoryArgs a) {
+    __shared__ m40_float4 part[DELTA ? WAVES : 1][4][64], whole[4][64];            // what the waves read of S; u
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, li = lane & 15;
     const uint32_t p = blockIdx.x / a.heads, head = blockIdx.x % a.heads, V = blockIdx.y, v = V * 16u + li;
     const uint32_t *portion = a.portions + 4 * p, row0 = portion[0], end = row0 + portion[1];
@@ -462,16 +467,20 @@ __global__ __launch_bounds__(256) void memory_walk_kernel(M40MemoryArgs a) {
         }
     float* block = block_of(a, a.chunk_base[p], head);
     const size_t next = (size_t)a.heads * a.block;
-    struct Operands { m40_float4 w[DELTA ? 4 : 1][DT], k[DT][4], u[4], decay[DT]; };
-    auto load = [&](Operands& f, const float* b) __attribute__((always_inline)) {
+    // u: of the delta rule, tile `wave` only (waves 0 to 3)
+    struct Operands { m40_float4 w[DELTA ? 4 : 1][DT], k[DT][4], u[DELTA ? 1 : 4], decay[DT]; } set[SETS];
+    auto load = [&](Operands& f, uint32_t c) __attribute__((always_inline)) {
+        const float* b = block + (c < chunks ? c : chunks - 1u) * next;
         if (DELTA) {
 #pragma unroll
             for (int t = 0; t < 4; ++t)
 #pragma unroll
-                for (int i = 0; i < DT; ++i) f.w[DELTA ? t : 0][i] = at4(b + a.at_w + (t * 16 + li) * a.dp + (wave * DT + i) * 16 + 4 * g);
-        }
+                for (int i = 0; i < DT; ++i) f.w[DELTA ? t : 0][i] = at4(b + a.at_w + ((t * (a.dp / 16u) + wave * DT + i) * 64 + lane) * 4);
+            f.u[0] = at4(b + a.at_u + (((wave & 3) * a.vt + V) * 64 + lane) * 4);
+        } else {
 #pragma unroll
-        for (int t = 0; t < 4; ++t) f.u[t] = at4(b + a.at_u + ((t * a.vt + V) * 64 + lane) * 4);
+            for (int t = 0; t < 4; ++t) f.u[DELTA ? 0 : t] = at4(b + a.at_u + ((t * a.vt + V) * 64 + lane) * 4);
+        }
 #pragma unroll
         for (int i = 0; i < DT; ++i) {
             f.decay[i] = at4(b + a.at_decay + (wave * DT + i) * 16 + 4 * g);
@@ -479,49 +488,51 @@ __global__ __launch_bounds__(256) void memory_walk_kernel(M40MemoryArgs a) {
             for (int t = 0; t < 4; ++t) f.k[i][t] = at4(b + a.at_k + (((wave * DT + i) * 4 + t) * 64 + lane) * 4);
         }
     };
-    auto step = [&](Operands& f, uint32_t c, int phase) __attribute__((always_inline)) {
+    auto step = [&](const Operands& f, uint32_t c) __attribute__((always_inline)) {
+        float* b = block + c * next;
 #pragma unroll
-        for (int i = 0; i < DT; ++i) put4(block + a.at_s + (((wave * DT + i) * a.vt + V) * 64 + lane) * 4, S[i]);
+        for (int i = 0; i < DT; ++i) put4(b + a.at_s + (((wave * DT + i) * a.vt + V) * 64 + lane) * 4, S[i]);
+        m40_float4 u[4];
         if (DELTA) {
 #pragma unroll
             for (int t = 0; t < 4; ++t) {
                 m40_float4 read = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
                 for (int i = 0; i < DT; ++i) read = mma4(f.w[DELTA ? t : 0][i], S[i], read);
-                part[DELTA ? phase : 0][DELTA ? wave : 0][t][lane] = read;
+                part[DELTA ? wave : 0][t][lane] = read;
+            }
+            m40_wait_and_meet<63>();
+            if (wave < 4) {
+                m40_float4 x = f.u[0];
+#pragma unroll
+                for (int w = 0; w < WAVES; ++w) x -= part[DELTA ? w : 0][wave][lane];
+                whole[wave][lane] = x;
+                put4(b + a.at_u + ((wave * a.vt + V) * 64 + lane) * 4, x);
             }
             m40_wait_and_meet<63>();
 #pragma unroll
-            for (int t = 0; t < 4; ++t)
+            for (int t = 0; t < 4; ++t) u[t] = whole[t][lane];
+        } else {
 #pragma unroll
-                for (int w = 0; w < 4; ++w) f.u[t] -= part[DELTA ? phase : 0][DELTA ? w : 0][t][lane];
-#pragma unroll
-            for (int t = 0; t < 4; ++t)
-                if (t == wave) put4(block + a.at_u + ((t * a.vt + V) * 64 + lane) * 4, f.u[t]);
+            for (int t = 0; t < 4; ++t) u[t] = f.u[DELTA ? 0 : t];
         }
 #pragma unroll
         for (int i = 0; i < DT; ++i) {
             S[i] *= f.decay[i];
 #pragma unroll
-            for (int t = 0; t < 4; ++t) S[i] = mma4(f.k[i][t], f.u[t], S[i]);
+            for (int t = 0; t < 4; ++t) S[i] = mma4(f.k[i][t], u[t], S[i]);
         }
-        block += next;
     };
-    // the operands of the next chunk are requested before the current one is worked on; wide heads have registers for one set only
-    constexpr bool kAhead = DT <= 2;
-    Operands even, odd;
-    load(even, block);
-    for (uint32_t c = 0; c < chunks; c += 2u) {
-        const bool more = c + 1u < chunks;
-        if (kAhead) load(odd, more ? block + next : block);
-        __builtin_amdgcn_sched_barrier(0);
-        step(even, c, 0);
-        if (!more) break;
-        if (!kAhead) load(odd, block);
-        if (kAhead) load(even, c + 2u < chunks ? block + next : block);
-        __builtin_amdgcn_sched_barrier(0);
-        step(odd, c + 1u, 1);
-        if (!kAhead && c + 2u < chunks) load(even, block);
+#pragma unroll
+    for (int i = 0; i + 1 < SETS; ++i) load(set[i], i);
+    for (uint32_t c = 0; c < chunks; c += SETS) {
+#pragma unroll
+        for (int i = 0; i < SETS; ++i) {
+            if (c + i >= chunks) break;
+            load(set[(i + SETS - 1) % SETS], c + i + SETS - 1);
+            __builtin_amdgcn_sched_barrier(0);
+            step(set[i], c + i);
+        }
     }
     if (!stored) return;
 #pragma unroll
@@ -552,7 +563,7 @@ __global__ __launch_bounds__(256) void memory_outputs_kernel(M40MemoryArgs a) {
         n = n < steps ? n : steps - 1;
         const bool state = n < d_steps;
         const float* tiles = block + (state ? a.at_s + n * vt * 256 : a.at_u + (n - d_steps) * vt * 256) + lane * 4;
-        f.x = at4(state ? block + t * a.dp + n * 16 + 4 * g : block + a.at_p + t * kChunk + (n - d_steps) * 16 + 4 * g);
+        f.x = at4((state ? block + (wave * (int)(a.dp / 16u) + n) * 256 : block + a.at_p + (wave * 4 + n - d_steps) * 256) + lane * 4);
 #pragma unroll
         for (int j = 0; j < VT; ++j) f.y[j] = at4(tiles + (j < vt ? j : vt - 1) * 256);
     };
@@ -612,9 +623,9 @@ __global__ __launch_bounds__(256) void memory_outputs_kernel(M40MemoryArgs a) {
     }
 }
 
-template <int DT, bool DELTA>
+template <int WAVES, int DT, int SETS, bool DELTA>
 void walk(hipStream_t stream, const M40MemoryArgs& a, uint32_t n_portions) {
-    memory_walk_kernel<DT, DELTA><<<dim3(n_portions * a.heads, a.vt), 256, 0, stream>>>(a);
+    memory_walk_kernel<WAVES, DT, SETS, DELTA><<<dim3(n_portions * a.heads, a.vt), WAVES * 64, 0, stream>>>(a);
 }
 template <bool DELTA>
 int chunked(hipStream_t stream, const M40MemoryArgs& a, uint32_t n_portions, uint32_t n_chunks) {
@@ -632,10 +643,10 @@ int chunked(hipStream_t stream, const M40MemoryArgs& a, uint32_t n_portions, uin
         else memory_prepare_kernel<false><<<grid, 256, 0, stream>>>(a);
     }
     switch (a.dp / 64u) {
-        case 1: walk<1, DELTA>(stream, a, n_portions); break;
-        case 2: walk<2, DELTA>(stream, a, n_portions); break;
-        case 3: walk<3, DELTA>(stream, a, n_portions); break;
-        default: walk<4, DELTA>(stream, a, n_portions); break;
+        case 1: walk<4, 1, 3, DELTA>(stream, a, n_portions); break;
+        case 2: walk<DELTA ? 8 : 4, DELTA ? 1 : 2, 3, DELTA>(stream, a, n_portions); break;
+        case 3: walk<12, 1, 2, DELTA>(stream, a, n_portions); break;
+        default: walk<8, 2, 2, DELTA>(stream, a, n_portions); break;
     }
     if (a.vt <= 4u) memory_outputs_kernel<4, DELTA><<<grid, 256, 0, stream>>>(a);
     else if (a.vt <= 8u) memory_outputs_kernel<8, DELTA><<<grid, 256, 0, stream>>>(a);
