@@ -68,20 +68,32 @@ __global__ __launch_bounds__(kThreads) void stream_update_kernel(M40llmStreamUpd
     auto output = [&](uint32_t g, float (&y)[8]) __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < 8; ++i) y[i] = 0.0f;
-        float v[8];
         if (a.place) {
-            for (uint32_t j = 0; j < a.top; ++j) {
-                const uint32_t at = a.place[(size_t)row * a.top + j];
-                const float f = static_cast<const float*>(a.weight)[(size_t)row * a.top + j];
-                load8<T, VEC>(static_cast<const T*>(a.expert_out) + (size_t)at * a.ld_expert, g * 8u, width, v);
+            for (uint32_t j0 = 0; j0 < a.top; j0 += 4u) {                 // places, then rows of four experts at a time
+                uint32_t at[4];
+                float f[4], v[4][8];
 #pragma unroll
-                for (int i = 0; i < 8; ++i) y[i] = fmaf(f, v[i], y[i]);
+                for (uint32_t j = 0; j < 4; ++j) {
+                    const size_t pick = (size_t)row * a.top + (j0 + j < a.top ? j0 + j : j0);
+                    at[j] = a.place[pick];
+                    f[j] = j0 + j < a.top ? static_cast<const float*>(a.weight)[pick] : 0.0f;
+                }
+#pragma unroll
+                for (uint32_t j = 0; j < 4; ++j) load8<T, VEC>(static_cast<const T*>(a.expert_out) + (size_t)at[j] * a.ld_expert, g * 8u, width, v[j]);
+#pragma unroll
+                for (uint32_t j = 0; j < 4; ++j)
+#pragma unroll
+                    for (int i = 0; i < 8; ++i) y[i] = fmaf(f[j], v[j][i], y[i]);
             }
         } else {
-            for (uint32_t p = 0; p < a.n_planes; ++p) {
-                load8<float, VEC>(static_cast<const float*>(a.planes) + p * (size_t)a.plane_stride + (size_t)row * width, g * 8u, width, v);
+            const float* plane = static_cast<const float*>(a.planes) + (size_t)row * width;
+            for (uint32_t p = 0; p < a.n_planes; p += 2u) {
+                float v[2][8];
+                const bool both = p + 1u < a.n_planes;
+                load8<float, VEC>(plane + p * (size_t)a.plane_stride, g * 8u, width, v[0]);
+                if (both) load8<float, VEC>(plane + (p + 1u) * (size_t)a.plane_stride, g * 8u, width, v[1]);
 #pragma unroll
-                for (int i = 0; i < 8; ++i) y[i] += v[i];
+                for (int i = 0; i < 8; ++i) y[i] += both ? v[0][i] + v[1][i] : v[0][i];
             }
         }
     };
@@ -146,15 +158,23 @@ __global__ __launch_bounds__(kThreads) void stream_update_kernel(M40llmStreamUpd
         for (int i = 0; i < 8; ++i) q = fmaf(u[i], u[i], q);
     }
     const float* w = static_cast<const float*>(a.w);
+    float kept_w[kGroups][8];
+#pragma unroll
+    for (uint32_t j = 0; j < kGroups; ++j)
+#pragma unroll
+        for (uint32_t i = 0; i < 8; ++i) {
+            const uint32_t c = (threadIdx.x + j * kThreads) * 8u + i;
+            kept_w[j][i] = w && c < width ? w[c] : 0.0f;
+        }
     const float inv = w ? 1.0f / sqrtf(block_sum(q, scratch) / (float)width + a.eps) : 1.0f;
-    auto finish = [&](uint32_t g, const float (&u)[8]) __attribute__((always_inline)) {
+    auto finish = [&](uint32_t g, const float (&u)[8], const float (&wg)[8]) __attribute__((always_inline)) {
         if (!w) {
             if (g * 8u < width) store8<VEC>(static_cast<float*>(a.x_out) + (size_t)row * width, g * 8u, width, u);
             return;
         }
         float v[8];
 #pragma unroll
-        for (uint32_t i = 0; i < 8; ++i) v[i] = g * 8u + i < width ? u[i] * inv * w[g * 8u + i] : 0.0f;
+        for (uint32_t i = 0; i < 8; ++i) v[i] = u[i] * inv * wg[i];          // both zero past the width
         const m40_float4 lo = {v[0], v[1], v[2], v[3]}, hi = {v[4], v[5], v[6], v[7]};
         T* o = static_cast<T*>(a.h) + m40_packed_at(row, g * 8u, a.ld_h >> 5);
         m40_store4<T>(o, lo);
@@ -168,13 +188,15 @@ __global__ __launch_bounds__(kThreads) void stream_update_kernel(M40llmStreamUpd
 #pragma unroll
     for (uint32_t j = 0; j < kGroups; ++j) {
         const uint32_t g = threadIdx.x + j * kThreads;
-        if (g < groups) finish(g, keep[j]);
+        if (g < groups) finish(g, keep[j], kept_w[j]);
     }
     for (uint32_t g = threadIdx.x + kGroups * kThreads; g < groups; g += kThreads) {
-        float u[8];
+        float u[8], wg[8];
         if (a.discard) turn(g, u);
         else again(g, u);
-        finish(g, u);
+#pragma unroll
+        for (uint32_t i = 0; i < 8; ++i) wg[i] = w && g * 8u + i < width ? w[g * 8u + i] : 0.0f;
+        finish(g, u, wg);
     }
 }
 
