@@ -21,25 +21,47 @@ static std::string quoted(const std::string& s) {
     return o + "\"";
 }
 
+static void rotation(const RotationSpec& r) {
+    std::cout << ", \"rot_dims\": " << r.dims << ", \"magnitude\": " << r.magnitude() << ", \"freq\": [";
+    const std::vector<double> f = r.frequencies();
+    for (size_t k = 0; k < f.size(); ++k) std::cout << (k ? ", " : "") << f[k];
+    std::cout << "]";
+}
+
+static void attention(const AttentionSpec& a) {
+    std::cout << "\"sizes\": [" << a.heads << ", " << a.kv_heads << ", " << a.dim << ", " << a.vdim << "], \"scale\": " << a.scale << ", \"flags\": [" << a.biases << ", "
+              << a.projection_norm << ", " << a.column_gate << ", " << a.share_values << "]";
+    if (a.rotation) rotation(*a.rotation);
+}
+
 static void spec(std::istream& in) {
     std::string path;
     in >> path;
     const DecoderSpec d = read_decoder_spec(read_text_file(path));
     std::cout.precision(17);
     std::cout << "{\"architecture\": " << quoted(d.architecture) << ", \"vocab\": " << d.vocab << ", \"width\": " << d.width << ", \"eps\": " << d.eps
-              << ", \"bigram\": " << (d.bigram ? (int64_t)d.bigram->buckets : -1) << ", \"embedding_scale\": " << d.embedding_scale << ", \"residual_mult\": " << d.residual_mult << ", \"positions\": " << d.positions << ", \"layers\": [";
+              << ", \"bigram\": " << (d.bigram ? (int64_t)d.bigram->buckets : -1) << ", \"embedding_scale\": " << d.embedding_scale << ", \"residual_mult\": " << d.residual_mult << ", \"positions\": " << d.positions << ", \"streams\": " << d.streams
+              << ", \"tied_head\": " << (d.tied_head ? "true" : "false") << ", \"around_zero\": " << (d.norm_around_zero ? "true" : "false") << ", \"layers\": [";
     for (size_t i = 0; i < d.layers.size(); ++i) {
         std::cout << (i ? ", " : "");
         const LayerSpec& l = d.layers[i];
         if (const auto* a = std::get_if<LatentAttentionSpec>(&l.mixer)) {
             std::cout << "{\"sizes\": [" << a->heads << ", " << a->dim << ", " << a->rot_dim << ", " << a->vdim << ", " << a->kv_rank << ", " << a->q_rank
-                      << "], \"scale\": " << a->scale << ", \"kv_from\": " << a->kv_from << ", \"magnitude\": " << a->rotation.magnitude() << ", \"freq\": [";
-            const std::vector<double> f = a->rotation.frequencies();
-            for (size_t k = 0; k < f.size(); ++k) std::cout << (k ? ", " : "") << f[k];
-            std::cout << "]";
+                      << "], \"scale\": " << a->scale << ", \"kv_from\": " << a->kv_from ;
+            rotation(a->rotation);
         } else if (const auto* a = std::get_if<DifferentialAttentionSpec>(&l.mixer)) {
             std::cout << "{\"sizes\": [" << a->heads << ", " << a->kv_heads << ", " << a->dim << ", " << a->vdim << ", " << a->taps << "], \"scale\": " << a->scale
                       << ", \"diff\": " << a->diff << ", \"kv_from\": " << a->kv_from;
+        } else if (const auto* a = std::get_if<AttentionSpec>(&l.mixer)) {
+            std::cout << "{";
+            attention(*a);
+        } else if (const auto* a = std::get_if<ParallelSpec>(&l.mixer)) {
+            std::cout << "{\"left\": {";
+            attention(a->left);
+            std::cout << "}, \"right\": [" << a->right.heads << ", " << a->right.dim << ", " << a->right.vdim << ", " << a->right.gate_cap << "], \"factors\": ["
+                      << a->left_scale << ", " << a->right_scale << "]";
+        } else if (const auto* a = std::get_if<ChannelDeltaSpec>(&l.mixer)) {
+            std::cout << "{\"sizes\": [" << a->heads << ", " << a->kv_heads << ", " << a->dim << ", " << a->vdim << ", " << a->taps << "]";
         } else {
             const LightningSpec& n = std::get<LightningSpec>(l.mixer);
             std::cout << "{\"sizes\": [" << n.heads << ", " << n.dim << ", " << n.vdim << "], \"decay\": [";
@@ -49,7 +71,8 @@ static void spec(std::istream& in) {
         const auto* g = std::get_if<GatedMlpSpec>(&l.mlp);
         std::cout << ", \"ff\": " << (g ? g->ff : 0) << ", \"silu\": " << (g && g->activation == Activation::Silu ? "true" : "false");
         if (const auto* e = std::get_if<ExpertMlpSpec>(&l.mlp))
-            std::cout << ", \"experts\": [" << e->experts << ", " << e->identity << ", " << e->top << ", " << e->ff << "]";
+            std::cout << ", \"experts\": [" << e->experts << ", " << e->identity << ", " << e->top << ", " << e->ff << "], \"groups\": [" << e->groups << ", " << e->keep << "], \"router_scale\": " << e->scale
+                      << ", \"correction\": " << (e->correction ? "true" : "false");
         std::cout << "}";
     }
     std::cout << "]}\n";
@@ -82,6 +105,12 @@ static void pages(std::istream& in) {
         std::cout << "], \"length\": " << (slot < slots ? p.length(slot) : 0) << ", \"prev\": " << (slot < slots ? p.previous_token(slot) : 0) << "}";
     }
     std::cout << "]\n";
+}
+
+static void rows(std::istream& in) {
+    std::string path, name;
+    in >> path >> name;
+    std::cout << SafetensorsFile(path).rows_of(name, 7) << "\n";
 }
 
 static void tensors(std::istream& in) {
@@ -172,6 +201,7 @@ int main() {
             if (what == "spec") spec(in);
             else if (what == "pages") pages(in);
             else if (what == "tensors") tensors(in);
+            else if (what == "rows") rows(in);
             else if (what == "scheduler") scheduler(in);
         } catch (const std::exception& e) {
             std::cout << "{\"error\": " << quoted(e.what()) << "}\n";

@@ -44,7 +44,8 @@ YARN = dict(factor=6.0, original=64, fast=8.0, slow=0.5)
 
 
 def config_odd():
-    """Sizes that fill no tile, values mixed across other layers and not at all, part of a head rotated, other taps, layers without feed-forward."""
+    """Sizes that fill no tile, values mixed across other layers and not at all, part of a head rotated, other taps, layers without feed-forward; an eps
+    that lets the normalizer of the matrix memory show through the norm behind it."""
     return model(101, 84, 3, [(attention(6, 2, 20, 37, v_mix=False), experts(6, 2, 24, (3, 2), 1.7)),
                               (delta(6, 3, 20, 37, 4), None),
                               (parallel((3, 1, 21, 24), (5, 19, 30), rot_dims=10, scaling=YARN), experts(9, 3, 40, (3, 2))),
@@ -52,7 +53,7 @@ def config_odd():
                               (attention(9, 3, 10, 12, v_mix=True, scale=-0.4), None),
                               (delta(2, 1, 33, 50, 2), experts(8, 3, 17, (2, 1), 2.0)),
                               (parallel((4, 4, 12, 20), (2, 40, 9), cap=3.0, scales=(1.5, -0.4)), None),
-                              (attention(2, 1, 30, 36, v_mix=True), experts(4, 2, 24, (4, 3)))], eps=2e-3, mult=0.4)
+                              (attention(2, 1, 30, 36, v_mix=True), experts(4, 2, 24, (4, 3)))], eps=0.1, mult=0.4)
 
 
 def config_even():
