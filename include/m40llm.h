@@ -570,8 +570,11 @@ int m40llm_ext_clear_u32_async(M40llmCudaContext* ctx, void* d_dst, size_t n, ui
 #define M40LLM_PACKED_VALUES 7u
 #define M40LLM_PACKED_SILU 8u       /* the first plain_tiles tiles: as STORE; then out_act[row][act_col + col] = silu(v), packed */
 #define M40LLM_PACKED_SPLIT 9u      /* the same without silu */
+#define M40LLM_PACKED_TANH 10u      /* the same with tanh */
+#define M40LLM_PACKED_CAP 11u       /* as STORE, v = out_cap * tanh(v * out_scale / out_cap), or v * out_scale where out_cap is 0 */
 #define M40LLM_GELU_TANH 0u
 #define M40LLM_SILU 1u
+#define M40LLM_LIMITED_GATE 2u      /* for PROJECT, with g = min(gate, act_limit), u = up held within +-act_limit: g * sigmoid(act_alpha*g) * (u + 1) */
 typedef struct M40llmPackedGemm {
     uint32_t act_dtype, epilogue;
     const void* a;                /* packed [rows][lda] activations */
@@ -600,6 +603,9 @@ typedef struct M40llmPackedGemm {
      * rows of a are plain rows gather[slot] of lda columns; without, packed rows `slot`.  Results are rows `slot`. */
     const uint32_t *jobs, *gather;
     uint32_t max_jobs, job_rows;
+    const void* row_scale;        /* PROJECT: f32 [rows] (or slots), gate and up are multiplied by it before the activation; NULL = ones */
+    float act_alpha, act_limit, out_scale, out_cap;
+    uint32_t segment_tiles;       /* column tile t reads columns t / segment_tiles * a_batch on of a (0 = all read the same; else a multiple of 16, one batch) */
 } M40llmPackedGemm;
 int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm* g, uint32_t stream_kind);
 
@@ -665,14 +671,17 @@ int m40llm_ext_norm_gate_rows_async(M40llmCudaContext* ctx, const void* d_y, uin
                                     uint32_t act_dtype, uint32_t stream_kind);
 
 /* ---- routed feed-forwards ------------------------------------------------------------------------------------------------------
- * Of `experts` + `identity` experts each row takes the `top` with the largest softmax(logits) + correction (the lower index of equals);
- * its weights are the softmax values times scale.  groups > 1: experts form that many groups of neighbours, and only those of the `keep` groups
+ * Of `experts` + `identity` experts each row takes the `top` with the largest score + correction (the lower index of equals), scores being
+ * softmax(logits) or, with M40LLM_SCORE_SIGMOID, sigmoid(logits) of each; its weights are the scores times scale; slot_weight (f32 by slot, may be
+ * NULL) takes them in the order of the list, for experts whose input is weighted.  groups > 1: experts form that many groups of neighbours, and only those of the `keep` groups
  * with the largest choice can be taken.  ids / weight: [rows][top].  Then rows are sorted by expert: every expert's rows, in order, take
  * slots from a multiple of 16 on; rows_of[slot] = row (slots that pad a group of 16 repeat a row), place[row*top + j] = slot, or
  * M40LLM_PLACE_INPUT for identity experts; jobs (m40llm_ext_packed_gemm_async) of at most job_rows slots; jobs[1] = slots in use.  rows_of holds
  * m40llm_ext_expert_slots, jobs 4 + 4 * m40llm_ext_expert_max_jobs words. */
+#define M40LLM_SCORE_SOFTMAX 0u
+#define M40LLM_SCORE_SIGMOID 1u
 typedef struct M40llmRoute {
-    uint32_t rows, experts, identity, top, job_rows, groups, keep;
+    uint32_t rows, experts, identity, top, job_rows, groups, keep, score;
     float scale;
     const void* logits;              /* f32 [rows][ld_logits] */
     uint64_t ld_logits;
@@ -680,6 +689,7 @@ typedef struct M40llmRoute {
     uint32_t* ids;
     void* weight;                    /* f32 */
     uint32_t *rows_of, *place, *jobs;
+    void* slot_weight;
 } M40llmRoute;
 int m40llm_ext_route_rows_async(M40llmCudaContext* ctx, const M40llmRoute* r, uint32_t stream_kind);
 /* dst, packed rows of ld columns: slot s = plain row rows_of[s] of src (bf16), for the slots in use; max_slots: m40llm_ext_expert_slots */
@@ -691,20 +701,22 @@ uint32_t m40llm_ext_expert_max_jobs(uint32_t rows, uint32_t experts, uint32_t to
 
 /* ---- attention over a paged cache of keys and values, one or two maps a head -------------------------------------------------
  * One map (maps = 1): softmax attention, its result times out_scale and, where gate is not NULL, times sigmoid(gate[row][head*vdim + d]).
+ * Its scores may be capped, s = cap * tanh(q.k * scale / cap) (cap 0 = not), lose slopes[head] * (distance of key and query) (f32, NULL = nothing),
+ * be limited to the `window` newest tokens (0 = all), and share the denominator with a sink, exp(sink[head]) (f32, NULL = none).
  * Two maps, differential attention: softmaxes of their own queries and keys over the same values, a1 and a2; o = a1 - lambda*a2, then
  * o / sqrt(mean(o^2) + eps) * out_scale * sigmoid(gate[row][head]).  Query head h uses kv head h / (heads / kv_heads).
  * A page holds 64 tokens; per kv head first the keys, map after map (`maps` of them), as packed rows (4 x k_tiles tiles of 16 tokens x 32 dimensions),
  * then the values transposed: per 16 dimensions two tiles [16 dimensions][32 tokens], token 16t + 4g + r at place 8g + 4t + r.
  * k_tiles = dim/32, v_tiles = vdim/16, rounded up; page p starts at element p * m40llm_ext_pair_page_elements. */
 uint64_t m40llm_ext_pair_page_elements(uint32_t maps, uint32_t kv_heads, uint32_t dim, uint32_t vdim);
-/* From projected rows (f32: heads of [map 1 | map 2] query columns, the same for keys, value columns): causal convolution of `taps` taps
- * on every column (0 = none), RMS norm over each map's dim of queries and keys; queries out as plain rows [heads][2][32*k_tiles], keys and
+/* From projected rows (f32: heads of [map 1 | map 2] query columns, or of one map; the same for keys, value columns): causal convolution of `taps` taps
+ * on every column (0 = none), RMS norm over each map's dim of queries and keys; queries out as plain rows [heads][maps][32*k_tiles], keys and
  * values to the row's place in the cache (cache NULL = the layer reads another layer's: no key and value columns).
  * row_back[row]: rows of the same portion before it, bit 31 set where the portion is one row.  conv_state [slot][taps - 1][ld_state]
  * holds the columns of the rows before a portion, that of position p at entry p % (taps - 1) (rows before position 0 count as zero);
  * portions of one row update it, the others by m40llm_ext_conv_state_async afterwards. */
 typedef struct M40llmPairSplit {
-    uint32_t act_dtype, rows, heads, kv_heads, dim, vdim, taps;
+    uint32_t act_dtype, rows, maps, heads, kv_heads, dim, vdim, taps;
     float eps;
     const void* proj;
     uint64_t ld_proj;
@@ -742,18 +754,23 @@ typedef struct M40llmPairAttention {
     uint64_t partial_floats;
     void* out;
     uint32_t ld_out;
+    uint32_t window;
+    float cap;
+    const void *slopes, *sink;
 } M40llmPairAttention;
 int m40llm_ext_pair_attention_async(M40llmCudaContext* ctx, const M40llmPairAttention* a, uint32_t stream_kind);
 uint64_t m40llm_ext_pair_attention_partial_floats(uint32_t maps, uint32_t rows, uint32_t heads, uint32_t vdim, uint32_t splits);
 /* most queries of a tile: 128 or 64 where form 1 is served, 16 where only form 0 is, 0 = sizes that are not served */
 uint32_t m40llm_ext_pair_attention_tile_queries(uint32_t act_dtype, uint32_t maps, uint32_t dim, uint32_t vdim);
 
-/* ---- lightning attention -----------------------------------------------------------------------------------------------------------
+/* ---- linear attention with one decay a head: lightning attention, state space layers ---------------------------------------------
  * Per head S <- decay*S + k v^T, o = S^T q, token by token; S in f32, state[slot][head][dim][32*ceil(vdim/32)], zero before position 0.
  * qkv: packed rows of the activation type, columns: heads x 32*ceil(dim/32) queries, the same of keys, heads x 32*ceil(vdim/32) values.
  * o: f32 [rows][heads*vdim].  portions[p] = {first row, rows, slot, 0}.
  * serial: token after token (any type); chunked (bf16): over the 64-row groups of the pass that a portion touches.  chunk_base[p] = chunks
- * of the portions before it; chunks[c] = {portion, first row of the group}; scratch: m40llm_ext_lightning_scratch_bytes. */
+ * of the portions before it; chunks[c] = {portion, first row of the group}; scratch: m40llm_ext_lightning_scratch_bytes.
+ * With step_logits the decay depends on the token (Mamba-2): d = softplus(step_logits[row][head] + step_bias[head]), S <- exp(-exp(A_log[head])*d)*S +
+ * d*k v^T, o = S^T q + skip[head]*v.  Head h uses query / key head h / (heads / kv_heads) (kv_heads 0 = heads): queries and keys of kv_heads heads. */
 typedef struct M40llmLightning {
     uint32_t act_dtype, chunked, heads, dim, vdim;
     const void* qkv;
@@ -767,6 +784,10 @@ typedef struct M40llmLightning {
     uint32_t n_portions, n_chunks;
     void* scratch;
     uint64_t scratch_bytes;
+    uint32_t kv_heads;
+    const void* step_logits;          /* f32 rows */
+    uint64_t ld_step;
+    const void *step_bias, *A_log, *skip;        /* f32 [heads] */
 } M40llmLightning;
 int m40llm_ext_lightning_async(M40llmCudaContext* ctx, const M40llmLightning* l, uint32_t stream_kind);
 uint64_t m40llm_ext_lightning_scratch_bytes(uint32_t n_chunks, uint32_t heads, uint32_t dim, uint32_t vdim);
@@ -780,6 +801,7 @@ int m40llm_ext_lightning_serves(uint32_t dim, uint32_t vdim);
  * ld_h columns, zero past width) and, where it is not NULL, to plain rows h_rows; without, u goes to x_out.
  * row_index (may be NULL): only these rows, `rows` of them; discard: the streams' new values are not kept. */
 #define M40LLM_MOST_STREAMS 16u
+/* (experts' rows without weights, weight NULL, count once each) */
 typedef struct M40llmStreamUpdate {
     uint32_t act_dtype, rows, width, streams, discard;
     float eps, mult;
@@ -800,6 +822,44 @@ typedef struct M40llmStreamUpdate {
     const uint32_t* row_index;
 } M40llmStreamUpdate;
 int m40llm_ext_stream_update_async(M40llmCudaContext* ctx, const M40llmStreamUpdate* u, uint32_t stream_kind);
+
+/* ---- row-wise steps of pre-norm layers ------------------------------------------------------------------------------------------------
+ * Mixes of each token's row with the one before: out column m*ld + c = h + (h' - h)*mu[m][c] for m < mixes, packed rows of mixes*ld columns.  h: plain
+ * rows of the activation type, ld columns; h' is the row before of the same portion, state[slot] (f32 rows of ld) for a portion's first,
+ * zero before position 0.  mu: f32 [mixes][ld].  state takes every portion's last row. */
+typedef struct M40llmTokenMix {
+    uint32_t act_dtype, rows, ld, mixes;
+    const void* h;
+    const void* mu;
+    void* state;
+    void* out;
+    const uint32_t *portions, *row_pos, *row_back;       /* as in M40llmLightning and M40llmPairSplit */
+    uint32_t n_portions;
+} M40llmTokenMix;
+int m40llm_ext_token_mix_async(M40llmCudaContext* ctx, const M40llmTokenMix* m, uint32_t stream_kind);
+/* Normed polynomial, in place on packed rows of ld columns (zero past cols): a N(z) + b N(z^2) + c N(z^3) + e, N(y) = y / sqrt(mean(y^2) + eps) over
+ * a row's cols columns; coefficients {a, b, c, e} in act (f32) */
+int m40llm_ext_poly_norm_rows_async(M40llmCudaContext* ctx, void* d_z, uint32_t ld, const void* d_act, uint32_t rows, uint32_t cols, float eps, uint32_t act_dtype,
+                                    uint32_t stream_kind);
+/* u = y * silu(gate) (f32 rows), then each of `groups` equal parts of cols over its own sqrt(mean(u^2) + eps), times w (f32 [cols]); packed, ld_out
+ * columns, zero past cols */
+int m40llm_ext_gate_group_norm_rows_async(M40llmCudaContext* ctx, const void* d_y, uint64_t ld_y, const void* d_gate, uint64_t ld_gate, const void* d_w, uint32_t rows,
+                                          uint32_t cols, uint32_t groups, float eps, void* d_out, uint32_t ld_out, uint32_t act_dtype, uint32_t stream_kind);
+/* Causal convolution with bias and silu over projected rows (f32) whose columns are `units` blocks: heads x vdim values, then twice kv_heads x dim
+ * (keys, then queries); out: the packed rows m40llm_ext_lightning_async reads (queries, keys, values, each head padded).  conv: f32 [taps][all], the newest
+ * row's last; conv_state, row_back and what follows for longer portions: M40llmPairSplit. */
+typedef struct M40llmSpaceSplit {
+    uint32_t act_dtype, rows, heads, kv_heads, dim, vdim, taps;
+    const void* proj;
+    uint64_t ld_proj;
+    const void *conv, *bias;
+    void* conv_state;
+    uint64_t ld_state;
+    void* out;
+    uint64_t ld_out;
+    const uint32_t *row_slot, *row_pos, *row_back;
+} M40llmSpaceSplit;
+int m40llm_ext_space_split_async(M40llmCudaContext* ctx, const M40llmSpaceSplit* s, uint32_t stream_kind);
 
 /* ---- attention of one map a head: from projections to queries and cache ----------------------------------------------------------
  * From projected rows (f32: query heads from column 0, key heads from k_offset, value heads from v_offset): biases (f32, may be NULL), RMS norm over
@@ -890,7 +950,30 @@ typedef struct M40llmChannelDelta {
 } M40llmChannelDelta;
 int m40llm_ext_channel_delta_async(M40llmCudaContext* ctx, const M40llmChannelDelta* m, uint32_t stream_kind);
 uint64_t m40llm_ext_channel_delta_state_floats(uint32_t dim, uint32_t vdim);
-uint64_t m40llm_ext_memory_scratch_bytes(uint32_t delta, uint32_t n_chunks, uint32_t heads, uint32_t dim, uint32_t vdim);
+/* Time mixing with a bonus (RWKV): w = exp(-exp(zw + w0)) per head and key channel; o = (S + diag(u) k v^T)^T r; then S <- diag(w) S + k v^T.
+ * rkv: f32 rows, receptance, key, value and gate columns of all heads; out: o / sqrt(mean(o^2) + eps) * norm * silu(gate) * out_factor (norm [heads*dim]). */
+typedef struct M40llmTimeMixing {
+    uint32_t act_dtype, chunked, heads, dim;
+    float eps, out_factor;
+    const void* rkv;
+    uint64_t ld_rkv;
+    uint32_t r_col, k_col, v_col, g_col;
+    const void* decay;               /* f32 rows of zw, heads*dim columns */
+    uint64_t ld_decay;
+    const void *w0, *u, *norm;       /* f32 [heads*dim] */
+    void* state;                     /* f32 [slot][heads][m40llm_ext_channel_delta_state_floats(dim, dim)] */
+    void* out;
+    uint32_t ld_out, out_col;
+    const uint32_t *portions, *chunk_base, *chunks, *row_pos;
+    uint32_t n_portions, n_chunks;
+    void* scratch;
+    uint64_t scratch_bytes;
+} M40llmTimeMixing;
+int m40llm_ext_time_mixing_async(M40llmCudaContext* ctx, const M40llmTimeMixing* m, uint32_t stream_kind);
+#define M40LLM_RULE_MEMORY 0u
+#define M40LLM_RULE_DELTA 1u
+#define M40LLM_RULE_MIXING 2u
+uint64_t m40llm_ext_memory_scratch_bytes(uint32_t rule, uint32_t n_chunks, uint32_t heads, uint32_t dim, uint32_t vdim);
 /* whether heads of these sizes are served */
 int m40llm_ext_memory_serves(uint32_t dim, uint32_t vdim);
 

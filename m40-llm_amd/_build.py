@@ -22,7 +22,7 @@ HIP_FLAGS = [
 HIP_SOURCES = ["context.hip", "elementwise.hip", "gemm.hip", "kvcache.hip", "attention.hip", "block_select.hip",
                "decode_fused.hip", "skinny_mfma.hip", "attention_mfma.hip", "rows_gemv.hip", "rows_mfma.hip", "rows_khalf_mfma.hip", "prefill_attention.hip", "gemm_tiled.hip", "q80_i8.hip",
                "packed_gemm.hip", "layer_ops.hip", "latent_attention.hip", "head_attention.hip", "sublayer_ops.hip", "experts.hip", "pair_attention.hip", "lightning.hip",
-               "stream_ops.hip", "projection_split.hip", "memory_serial.hip", "memory_chunks.hip"]
+               "stream_ops.hip", "mix_ops.hip", "projection_split.hip", "memory_serial.hip", "memory_chunks.hip"]
 CPP_SOURCES = ["unavailable.cpp"]
 # per-file additions: matrix-instruction results straight into vector registers (the default form writes them to
 # accumulation registers and copies every element out again)

@@ -45,6 +45,7 @@ __device__ __forceinline__ void route_row(const M40llmRoute& a, uint32_t row, ui
     const uint32_t n = a.experts + a.identity;
     const float* z = static_cast<const float*>(a.logits) + (size_t)row * a.ld_logits;
     const float* correction = static_cast<const float*>(a.correction);
+    const bool sigmoid = a.score == M40LLM_SCORE_SIGMOID;
     float s[N], choice[N];
     float top = -INFINITY;
 #pragma unroll
@@ -58,16 +59,21 @@ __device__ __forceinline__ void route_row(const M40llmRoute& a, uint32_t row, ui
     float sum = 0.0f;
 #pragma unroll
     for (uint32_t i = 0; i < N; ++i) {
-        s[i] = lane + 64u * i < n ? expf(s[i] - top) : 0.0f;
+        const float logit = s[i];
+        s[i] = lane + 64u * i >= n ? 0.0f : sigmoid ? m40_sigmoid(logit) : expf(logit - top);
         sum += s[i];
+        // sigmoids of large logits are equal in f32 where the logits are not: without a correction the logits decide
+        if (sigmoid) choice[i] = correction ? choice[i] + s[i] : logit;
     }
     sum = m40_sum64(sum);
     uint32_t left = 0;                       // bit i: this lane's expert i can be chosen
 #pragma unroll
     for (uint32_t i = 0; i < N; ++i) {
         const uint32_t e = lane + 64u * i;
-        s[i] /= sum;
-        choice[i] += s[i];
+        if (!sigmoid) {
+            s[i] /= sum;
+            choice[i] += s[i];
+        }
         if (e < n) left |= 1u << i;
     }
     if (a.groups > 1u) left = within_groups<N>(a, lane, n / a.groups, choice, left);
@@ -223,9 +229,13 @@ __global__ __launch_bounds__(kListThreads) void expert_lists_kernel(M40llmRoute 
                 const uint32_t slot = slots + before++;
                 a.rows_of[slot] = (p + i) / a.top;
                 a.place[p + i] = slot;
+                if (a.slot_weight) static_cast<float*>(a.slot_weight)[slot] = SMALL ? own_weight[SMALL ? p + i : 0] : static_cast<const float*>(a.weight)[p + i];
             }
     }
-    if (tid < ((n + 15u) & ~15u) - n) a.rows_of[slots + n + tid] = 0u;
+    if (tid < ((n + 15u) & ~15u) - n) {
+        a.rows_of[slots + n + tid] = 0u;
+        if (a.slot_weight) static_cast<float*>(a.slot_weight)[slots + n + tid] = 0.0f;
+    }
 }
 
 // A wave moves 16 x 32 operand tiles: 16 rows of the list side by side.
@@ -269,7 +279,7 @@ int m40llm_ext_route_rows_async(M40llmCudaContext* ctx, const M40llmRoute* r, ui
     if (!ctx || !r || !r->logits || !r->ids || !r->weight || !r->rows_of || !r->place || !r->jobs) return -1;
     hipStream_t stream = m40_select_stream(ctx, stream_kind);
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
-    if (r->rows == 0 || r->experts == 0 || r->experts + r->identity > kMost || r->top == 0 || r->top > r->experts + r->identity ||
+    if (r->rows == 0 || r->experts == 0 || r->score > M40LLM_SCORE_SIGMOID || r->experts + r->identity > kMost || r->top == 0 || r->top > r->experts + r->identity ||
         r->ld_logits < r->experts + r->identity || (r->job_rows != 16u && r->job_rows != 32u && r->job_rows != 64u && r->job_rows != 128u) ||
         !m40_aligned16(r->ids) || m40llm_ext_expert_slots(r->rows, r->experts, r->top) == 0 || m40llm_ext_expert_max_jobs(r->rows, r->experts, r->top, r->job_rows) == 0)
         return -3;

@@ -6,13 +6,15 @@
 //
 // Matrix memory: u is the values with a column of ones, whose sums are n; decays are exp of sums of log gates less the running maximum, so no
 // exponent is above zero.  Delta rule: u_t = beta_t (v_t - read_t) depends on the u before it; with A[t, j] = beta_t k_t . (k_j, decayed), j < t,
-// (I + A) u = beta (v - (k, decayed from the start)^T S_0), a triangular system whose solution is U_0 - W S_0.
+// (I + A) u = beta (v - (k, decayed from the start)^T S_0), a triangular system whose solution is U_0 - W S_0.  Time mixing: u is the values;
+// queries are decayed to the token before, P[t, t] is q_t . (bonus k_t).
 //
 // memory_scan_kernel      matrix memory: sums of log gates, the running maximum
 // memory_prepare_kernel   matrix memory: P, decayed queries and keys of all chunks
 // delta_prepare_kernel    delta rule: the same, and the solution of the triangular system.  Decays between two tokens are never formed as
 //                         a quotient: tokens of 16-row blocks meet as a product of the row's decay since its block began and the other's to the
 //                         end of its block (both at most one), tokens of one block pairwise.
+// mixing_prepare_kernel   time mixing: P, decayed queries and keys, with decays as in the delta rule
 // memory_walk_kernel      chunk after chunk: a workgroup holds 16 value columns of a head's state, leaves them as they are before each chunk
 // memory_outputs_kernel   all chunks at once: outputs, the head's norm, the gate
 //
@@ -444,10 +446,189 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(M40MemoryArgs a) 
     }
 }
 
+// ---- time mixing ------------------------------------------------------------------------------------------------------------------------
+struct MixingLds {
+    float k[kChunk][kLdSlab], q[kChunk][kLdSlab], l[kChunk][kLdSlab];          // l: log2 of the decay since the 16-row block began
+    float qe[kChunk][kLdSlab], ks[kChunk][kLdSlab];                            // q decayed since the block began, up to the token before; k decayed to its end
+    float whole[4][kSlab], start[4][kSlab], rest[4][kSlab];                    // of a block: its own decay, all before it, all behind it
+};
+template <bool VEC>
+__global__ __launch_bounds__(256, 2) void mixing_prepare_kernel(M40MemoryArgs a) {
+    __shared__ __align__(16) MixingLds lds;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), g = lane >> 4, li = lane & 15;
+    const Chunk c(a, blockIdx.x);
+    const uint32_t head = blockIdx.y, dim = a.dim, n = c.n;
+    float* out = block_of(a, blockIdx.x, head);
+    auto row_of = [&](uint32_t t) { return c.row0 + (t < n ? t : n - 1u); };
+    float own[16], bonus = 0.0f;                    // own: rows of this wave's block with row lane / 4 of it, a quarter of the key dimensions
+#pragma unroll
+    for (int t = 0; t < 16; ++t) own[t] = 0.0f;
+    // rows of a block x with those of one before it, y: six pairs, a wave's own and one of the last two
+    m40_float4 off[2];
+    int x_of[2], y_of[2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+        const int pair = wave + 4 * i < 6 ? wave + 4 * i : 5;
+        x_of[i] = pair == 0 ? 1 : pair < 3 ? 2 : 3;
+        y_of[i] = pair - x_of[i] * (x_of[i] - 1) / 2;
+        off[i] = m40_float4{0.f, 0.f, 0.f, 0.f};
+    }
+    const int t_in = tid >> 2, d_in = (tid & 3) * 8;
+    struct Rows { m40_float4 k[2], q[2], z[2], bias[2], u[2]; } in;            // a slab's rows, requested a slab ahead
+    const bool live = t_in < (int)n;
+    const size_t row_in = row_of(t_in);
+    const float *k_row = a.k + row_in * a.ld + head * dim, *q_row = a.q + row_in * a.ld + head * dim, *z_row = a.a + row_in * a.ld_a + head * dim, *bias_row = a.dt_bias + head * dim,
+                *u_row = a.bonus + head * dim;
+    auto load = [&](uint32_t slab) __attribute__((always_inline)) {
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+            const uint32_t d = slab + d_in + 4 * h;
+            in.k[h] = dims4<VEC>(k_row, d, dim);
+            in.q[h] = dims4<VEC>(q_row, d, dim);
+            in.z[h] = dims4<VEC>(z_row, d, dim);
+            in.bias[h] = dims4<VEC>(bias_row, d, dim);
+            in.u[h] = dims4<VEC>(u_row, d, dim);
+        }
+    };
+    load(0u);
+    for (uint32_t slab = 0; slab < a.dp; slab += kSlab) {
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+            const uint32_t d = slab + d_in + 4 * h;
+            const m40_float4 k = in.k[h] * (live ? 1.0f : 0.0f), q = in.q[h] * (live ? a.q_factor : 0.0f);
+            m40_float4 l;
+#pragma unroll
+            for (uint32_t r = 0; r < 4; ++r) {
+                l[r] = live && d + r < dim ? m40_mixing_log2_decay(in.z[h][r] + in.bias[h][r]) : 0.0f;
+                bonus = fmaf(q[r] * in.u[h][r], k[r], bonus);
+            }
+            put4(&lds.k[t_in][d_in + 4 * h], k);
+            put4(&lds.q[t_in][d_in + 4 * h], q);
+            put4(&lds.l[t_in][d_in + 4 * h], l);
+        }
+        load(slab + kSlab);
+        __syncthreads();
+        if (tid < 4 * kSlab) {
+            const int b = tid / kSlab, d = tid % kSlab;
+            float s = 0.0f;
+#pragma unroll
+            for (int t = 0; t < 16; ++t) {
+                s += lds.l[b * 16 + t][d];
+                lds.l[b * 16 + t][d] = s;
+            }
+            lds.whole[b][d] = s;
+        }
+        __syncthreads();
+        if (tid < 4 * kSlab) {
+            const int b = tid / kSlab, d = tid % kSlab;
+            float before = 0.0f, behind = 0.0f;
+            for (int x = 0; x < 4; ++x) {
+                if (x < b) before += lds.whole[x][d];
+                if (x > b) behind += lds.whole[x][d];
+            }
+            lds.start[b][d] = __builtin_amdgcn_exp2f(before);
+            lds.rest[b][d] = __builtin_amdgcn_exp2f(behind);
+            if (b == 3) out[a.at_decay + slab + d] = __builtin_amdgcn_exp2f(before + lds.whole[3][d]);
+        }
+        {
+            const int b = t_in >> 4, before = t_in & 15 ? t_in - 1 : t_in;
+            const float f = t_in & 15 ? 1.0f : 0.0f;
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {
+                const int d = d_in + 4 * h;
+                const m40_float4 l = at4(&lds.l[t_in][d]), past = at4(&lds.l[before][d]), end = at4(&lds.whole[b][d]);
+                m40_float4 since, until;
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    since[r] = __builtin_amdgcn_exp2f(past[r] * f);
+                    until[r] = __builtin_amdgcn_exp2f(end[r] - l[r]);
+                }
+                put4(&lds.qe[t_in][d], at4(&lds.q[t_in][d]) * since);
+                put4(&lds.ks[t_in][d], at4(&lds.k[t_in][d]) * until);
+            }
+        }
+        __syncthreads();
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {               // decayed from the start, to the end
+            const int d = d_in + 4 * h;
+            put4(out + tile_at(t_in, slab + d, a.dp / 16u), at4(&lds.qe[t_in][d]) * at4(&lds.start[t_in >> 4][d]));
+        }
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {               // block `wave` of tokens, 16 dimensions
+            const int d = h * 16 + li;
+            m40_float4 y;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) y[r] = lds.ks[wave * 16 + 4 * g + r][d] * lds.rest[wave][d];
+            put4(out + a.at_k + (((slab / 16u + h) * 4u + wave) * 64 + lane) * 4, y);
+        }
+        {                                           // pairs of the block's own rows
+            const int j = lane >> 2, d = (lane & 3) * 8;
+            float kj[8], lj[8];
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {
+                const m40_float4 x = at4(&lds.k[wave * 16 + j][d + 4 * h]), y = at4(&lds.l[wave * 16 + j][d + 4 * h]);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) { kj[4 * h + r] = x[r]; lj[4 * h + r] = y[r]; }
+            }
+#pragma unroll
+            for (int t = 1; t < 16; ++t) {
+#pragma unroll
+                for (int h = 0; h < 2; ++h) {
+                    const m40_float4 qt = at4(&lds.q[wave * 16 + t][d + 4 * h]), lt = at4(&lds.l[wave * 16 + t - 1][d + 4 * h]);
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) own[t] = fmaf(qt[r], kj[4 * h + r] * __builtin_amdgcn_exp2f(fminf(lt[r] - lj[4 * h + r], 0.0f)), own[t]);
+                }
+                if (t & 1) stay();                  // operands of two rows at a time in registers
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {
+                const int d = h * 16 + 4 * g, x = x_of[i], y = y_of[i];
+                // decays of the blocks between: at most the second and the third
+                const float f1 = y < 1 && x > 1 ? 1.0f : 0.0f, f2 = y < 2 && x > 2 ? 1.0f : 0.0f;
+                m40_float4 f = at4(&lds.whole[1][d]) * f1 + at4(&lds.whole[2][d]) * f2;
+#pragma unroll
+                for (int r = 0; r < 4; ++r) f[r] = __builtin_amdgcn_exp2f(f[r]);
+                off[i] = mma4(at4(&lds.ks[y * 16 + li][d]), at4(&lds.qe[x * 16 + li][d]) * f, off[i]);
+            }
+        __syncthreads();
+    }
+    {
+        const int j = lane >> 2;
+#pragma unroll
+        for (int t = 0; t < 16; ++t) {
+            float y = own[t];
+            y += m40_dpp_f<M40_DPP_XOR1>(y);
+            y += m40_dpp_f<M40_DPP_XOR2>(y);
+            if ((lane & 3) == (t & 3) && j != t) out[a.at_p + tile_at(wave * 16 + t, wave * 16 + (j & 12), 4u) + (j & 3)] = j < t ? y : 0.0f;
+        }
+        bonus += m40_dpp_f<M40_DPP_XOR1>(bonus);
+        bonus += m40_dpp_f<M40_DPP_XOR2>(bonus);
+        if ((lane & 3) == 0) out[a.at_p + tile_at(t_in, t_in & 60, 4u) + (t_in & 3)] = bonus;
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+            if (wave + 4 * i < 6) put4(out + a.at_p + ((x_of[i] * 4 + y_of[i]) * 64 + lane) * 4, off[i]);
+    }
+    for (uint32_t x = wave; x < a.vt * 4u; x += 4u) {
+        const uint32_t v = x % a.vt * 16u + li;
+        m40_float4 y;
+#pragma unroll
+        for (uint32_t r = 0; r < 4; ++r) {
+            const uint32_t t = x / a.vt * 16u + 4u * g + r;
+            const float u = a.v[(size_t)row_of(t) * a.ld + head * a.vdim + (v < a.vdim ? v : 0u)];
+            y[r] = t < n && v < a.vdim ? u : 0.0f;
+        }
+        put4(out + a.at_u + (x * 64 + lane) * 4, y);
+    }
+}
+
 // ---- the walk ---------------------------------------------------------------------------------------------------------------------------
 // Wave w holds key dimensions 16 DT w .. of 16 value columns.  A chunk's operands are requested SETS - 1 chunks ahead.
-template <int WAVES, int DT, int SETS, bool DELTA>
+template <int WAVES, int DT, int SETS, M40MemoryRule RULE>
 __global__ __launch_bounds__(WAVES * 64) void memory_walk_kernel(M40MemoryArgs a) {
+    constexpr bool DELTA = RULE == kM40Delta;
     __shared__ m40_float4 part[DELTA ? WAVES : 1][4][64], whole[4][64];            // what the waves read of S; u
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, li = lane & 15;
     const uint32_t p = blockIdx.x / a.heads, head = blockIdx.x % a.heads, V = blockIdx.y, v = V * 16u + li;
@@ -456,7 +637,7 @@ __global__ __launch_bounds__(WAVES * 64) void memory_walk_kernel(M40MemoryArgs a
     float* state = a.state + ((size_t)portion[2] * a.heads + head) * a.head_floats;
     float* own = state + (v < a.vdim ? v : (size_t)a.dim * a.v4);                  // column v of S; behind the last, n
     const size_t step_d = v < a.vdim ? a.v4 : 1u;
-    const bool stored = v < a.vdim || (!DELTA && v == a.vdim), fresh = a.row_pos[row0] == 0u;
+    const bool stored = v < a.vdim || (RULE == kM40Memory && v == a.vdim), fresh = a.row_pos[row0] == 0u;
     m40_float4 S[DT];
 #pragma unroll
     for (int i = 0; i < DT; ++i)
@@ -545,7 +726,7 @@ __global__ __launch_bounds__(WAVES * 64) void memory_walk_kernel(M40MemoryArgs a
 }
 
 // ---- outputs: wave w takes the chunk's rows 16 w ..; VT: the most column tiles
-template <int VT, bool DELTA>
+template <int VT, M40MemoryRule RULE>
 __global__ __launch_bounds__(256) void memory_outputs_kernel(M40MemoryArgs a) {
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, li = lane & 15;
     const Chunk c(a, blockIdx.x);
@@ -584,7 +765,7 @@ __global__ __launch_bounds__(256) void memory_outputs_kernel(M40MemoryArgs a) {
     }
     const int vdim = (int)a.vdim;
     float f = 1.0f;
-    if (!DELTA) {                                   // column vdim: n . q
+    if (RULE == kM40Memory) {                       // column vdim: n . q
         float x = 0.0f;
 #pragma unroll
         for (int j = 0; j < VT; ++j)
@@ -618,20 +799,24 @@ __global__ __launch_bounds__(256) void memory_outputs_kernel(M40MemoryArgs a) {
         const m40_float4 z = m40_load4(gate + v, vdim - v, vec), w = m40_load4(norm + v, vdim - v, vec);
         m40_float4 y;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) y[r] = o[j][r] * inv * w[r] * m40_sigmoid(z[r]);
+        for (int r = 0; r < 4; ++r) y[r] = o[j][r] * inv * w[r] * (RULE == kM40Mixing ? m40_silu(z[r]) : m40_sigmoid(z[r]));
         m40_store_packed<m40_bf16>(static_cast<m40_bf16*>(a.out), (int)row, (int)(a.out_col + head * a.vdim) + v, (long)a.ld_out, y, vdim - v, vdim % 4 == 0 && a.out_col % 4u == 0);
     }
 }
 
-template <int WAVES, int DT, int SETS, bool DELTA>
+template <int WAVES, int DT, int SETS, M40MemoryRule RULE>
 void walk(hipStream_t stream, const M40MemoryArgs& a, uint32_t n_portions) {
-    memory_walk_kernel<WAVES, DT, SETS, DELTA><<<dim3(n_portions * a.heads, a.vt), WAVES * 64, 0, stream>>>(a);
+    memory_walk_kernel<WAVES, DT, SETS, RULE><<<dim3(n_portions * a.heads, a.vt), WAVES * 64, 0, stream>>>(a);
 }
-template <bool DELTA>
+template <M40MemoryRule RULE>
 int chunked(hipStream_t stream, const M40MemoryArgs& a, uint32_t n_portions, uint32_t n_chunks) {
     const bool vec = a.dim % 4u == 0 && a.ld % 4u == 0 && a.ld_a % 4u == 0 && m40_aligned16(a.q) && m40_aligned16(a.k) && m40_aligned16(a.a) && m40_aligned16(a.dt_bias);
     const dim3 grid(n_chunks, a.heads);
-    if constexpr (DELTA) {
+    constexpr bool DELTA = RULE == kM40Delta;
+    if constexpr (RULE == kM40Mixing) {
+        if (vec && m40_aligned16(a.bonus)) mixing_prepare_kernel<true><<<grid, 256, 0, stream>>>(a);
+        else mixing_prepare_kernel<false><<<grid, 256, 0, stream>>>(a);
+    } else if constexpr (DELTA) {
         static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(delta_prepare_kernel<true>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)sizeof(DeltaLds)),
                                 attr2 = hipFuncSetAttribute(reinterpret_cast<const void*>(delta_prepare_kernel<false>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)sizeof(DeltaLds));
         if (attr != hipSuccess || attr2 != hipSuccess) return -2;
@@ -643,23 +828,23 @@ int chunked(hipStream_t stream, const M40MemoryArgs& a, uint32_t n_portions, uin
         else memory_prepare_kernel<false><<<grid, 256, 0, stream>>>(a);
     }
     switch (a.dp / 64u) {
-        case 1: walk<4, 1, 3, DELTA>(stream, a, n_portions); break;
-        case 2: walk<DELTA ? 8 : 4, DELTA ? 1 : 2, 3, DELTA>(stream, a, n_portions); break;
-        case 3: walk<12, 1, 2, DELTA>(stream, a, n_portions); break;
-        default: walk<8, 2, 2, DELTA>(stream, a, n_portions); break;
+        case 1: walk<4, 1, 3, RULE>(stream, a, n_portions); break;
+        case 2: walk<DELTA ? 8 : 4, DELTA ? 1 : 2, 3, RULE>(stream, a, n_portions); break;
+        case 3: walk<12, 1, 2, RULE>(stream, a, n_portions); break;
+        default: walk<8, 2, 2, RULE>(stream, a, n_portions); break;
     }
-    if (a.vt <= 4u) memory_outputs_kernel<4, DELTA><<<grid, 256, 0, stream>>>(a);
-    else if (a.vt <= 8u) memory_outputs_kernel<8, DELTA><<<grid, 256, 0, stream>>>(a);
-    else if (a.vt <= 9u) memory_outputs_kernel<9, DELTA><<<grid, 256, 0, stream>>>(a);
-    else memory_outputs_kernel<17, DELTA><<<grid, 256, 0, stream>>>(a);
+    if (a.vt <= 4u) memory_outputs_kernel<4, RULE><<<grid, 256, 0, stream>>>(a);
+    else if (a.vt <= 8u) memory_outputs_kernel<8, RULE><<<grid, 256, 0, stream>>>(a);
+    else if (a.vt <= 9u) memory_outputs_kernel<9, RULE><<<grid, 256, 0, stream>>>(a);
+    else memory_outputs_kernel<17, RULE><<<grid, 256, 0, stream>>>(a);
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
 
 constexpr uint32_t kMost = 256;
 // the parts of a block of scratch
-void lay_out(M40MemoryArgs& a, bool delta) {
+void lay_out(M40MemoryArgs& a, M40MemoryRule rule) {
     a.dp = (a.dim + 63u) / 64u * 64u;
-    a.vt = (a.vdim + (delta ? 0u : 1u) + 15u) / 16u;
+    a.vt = (a.vdim + (rule == kM40Memory ? 1u : 0u) + 15u) / 16u;
     uint32_t at = kChunk * a.dp;
     auto part = [&](uint32_t n) { const uint32_t x = at; at += n; return x; };
     a.at_k = part(kChunk * a.dp);
@@ -667,37 +852,41 @@ void lay_out(M40MemoryArgs& a, bool delta) {
     a.at_u = part(kChunk * 16u * a.vt);
     a.at_decay = part(a.dp);
     a.at_s = part(a.dp * 16u * a.vt);
-    a.at_w = part(delta ? kChunk * a.dp : 0u);
-    a.at_gate = part(delta ? 0u : 256u);
+    a.at_w = part(rule == kM40Delta ? kChunk * a.dp : 0u);
+    a.at_gate = part(rule == kM40Memory ? 256u : 0u);
     a.block = at;
 }
-uint64_t state_floats(bool delta, uint32_t dim, uint32_t vdim) {
+uint64_t state_floats(M40MemoryRule rule, uint32_t dim, uint32_t vdim) {
     const uint64_t s = (uint64_t)dim * ((vdim + 3u) & ~3u);
-    return delta ? s : s + ((dim + 3u) & ~3u) + 4u;
+    return rule != kM40Memory ? s : s + ((dim + 3u) & ~3u) + 4u;
 }
 
-// what both rules' structs have in common
+// what the rules' structs have in common
 template <class P>
-int run(M40llmCudaContext* ctx, M40MemoryArgs& a, const P& p, bool delta, uint32_t stream_kind) {
+int run(M40llmCudaContext* ctx, M40MemoryArgs& a, const P& p, uint32_t vdim, M40MemoryRule rule, uint32_t stream_kind) {
     hipStream_t stream = m40_select_stream(ctx, stream_kind);
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
-    if (p.act_dtype > 1u || p.heads == 0 || p.heads > 65535u || p.n_portions == 0 || !m40llm_ext_memory_serves(p.dim, p.vdim) || p.ld_out % 32u != 0 ||
-        p.ld_out < p.out_col + (uint64_t)p.heads * p.vdim || !m40_aligned16(p.state) || !m40_aligned16(p.out))
+    if (p.act_dtype > 1u || p.heads == 0 || p.heads > 65535u || p.n_portions == 0 || !m40llm_ext_memory_serves(p.dim, vdim) || p.ld_out % 32u != 0 ||
+        p.ld_out < p.out_col + (uint64_t)p.heads * vdim || !m40_aligned16(p.state) || !m40_aligned16(p.out))
         return -3;
-    a.heads = p.heads; a.dim = p.dim; a.vdim = p.vdim; a.v4 = (p.vdim + 3u) & ~3u;
-    a.q_factor = p.q_factor; a.eps = p.eps; a.out_factor = p.out_factor;
+    a.heads = p.heads; a.dim = p.dim; a.vdim = vdim; a.v4 = (vdim + 3u) & ~3u;
+    a.eps = p.eps; a.out_factor = p.out_factor;
     a.state = static_cast<float*>(p.state);
-    a.head_floats = state_floats(delta, p.dim, p.vdim);
+    a.head_floats = state_floats(rule, p.dim, vdim);
     a.out = p.out; a.ld_out = p.ld_out; a.out_col = p.out_col;
     a.portions = p.portions; a.chunk_base = p.chunk_base; a.chunks = p.chunks; a.row_pos = p.row_pos;
     a.scratch = static_cast<float*>(p.scratch);
-    lay_out(a, delta);
+    lay_out(a, rule);
     (void)hipGetLastError();
-    if (!p.chunked) return m40_launch_memory_serial(stream, a, delta, p.act_dtype, p.n_portions);
+    if (!p.chunked) return m40_launch_memory_serial(stream, a, rule, p.act_dtype, p.n_portions);
     if (p.act_dtype != M40LLM_ACT_BF16 || !p.chunk_base || !p.chunks || p.n_chunks == 0 || !p.scratch || !m40_aligned16(p.scratch) ||
         p.scratch_bytes < (uint64_t)p.n_chunks * p.heads * a.block * 4u)
         return -4;
-    return delta ? chunked<true>(stream, a, p.n_portions, p.n_chunks) : chunked<false>(stream, a, p.n_portions, p.n_chunks);
+    switch (rule) {
+        case kM40Delta: return chunked<kM40Delta>(stream, a, p.n_portions, p.n_chunks);
+        case kM40Mixing: return chunked<kM40Mixing>(stream, a, p.n_portions, p.n_chunks);
+        default: return chunked<kM40Memory>(stream, a, p.n_portions, p.n_chunks);
+    }
 }
 
 }  // namespace
@@ -705,12 +894,12 @@ int run(M40llmCudaContext* ctx, M40MemoryArgs& a, const P& p, bool delta, uint32
 extern "C" {
 
 int m40llm_ext_memory_serves(uint32_t dim, uint32_t vdim) { return dim >= 1u && dim <= kMost && vdim >= 1u && vdim <= kMost; }
-uint64_t m40llm_ext_matrix_memory_state_floats(uint32_t dim, uint32_t vdim) { return state_floats(false, dim, vdim); }
-uint64_t m40llm_ext_channel_delta_state_floats(uint32_t dim, uint32_t vdim) { return state_floats(true, dim, vdim); }
-uint64_t m40llm_ext_memory_scratch_bytes(uint32_t delta, uint32_t n_chunks, uint32_t heads, uint32_t dim, uint32_t vdim) {
+uint64_t m40llm_ext_matrix_memory_state_floats(uint32_t dim, uint32_t vdim) { return state_floats(kM40Memory, dim, vdim); }
+uint64_t m40llm_ext_channel_delta_state_floats(uint32_t dim, uint32_t vdim) { return state_floats(kM40Delta, dim, vdim); }
+uint64_t m40llm_ext_memory_scratch_bytes(uint32_t rule, uint32_t n_chunks, uint32_t heads, uint32_t dim, uint32_t vdim) {
     M40MemoryArgs a{};
     a.dim = dim; a.vdim = vdim;
-    lay_out(a, delta != 0u);
+    lay_out(a, (M40MemoryRule)rule);
     return (uint64_t)n_chunks * heads * a.block * 4u;
 }
 
@@ -728,7 +917,8 @@ int m40llm_ext_matrix_memory_async(M40llmCudaContext* ctx, const M40llmMatrixMem
     a.cap = m->cap;
     a.norm = static_cast<const float*>(m->norm); a.norm_stride = m->vdim;
     a.gate = x + m->g_col; a.ld_gate = m->ld_proj;
-    return run(ctx, a, *m, false, stream_kind);
+    a.q_factor = m->q_factor;
+    return run(ctx, a, *m, m->vdim, kM40Memory, stream_kind);
 }
 
 int m40llm_ext_channel_delta_async(M40llmCudaContext* ctx, const M40llmChannelDelta* m, uint32_t stream_kind) {
@@ -745,7 +935,24 @@ int m40llm_ext_channel_delta_async(M40llmCudaContext* ctx, const M40llmChannelDe
     a.A_log = static_cast<const float*>(m->A_log); a.dt_bias = static_cast<const float*>(m->dt_bias);
     a.norm = static_cast<const float*>(m->norm); a.norm_stride = 0;
     a.gate = low + m->g_col; a.ld_gate = m->ld_low;
-    return run(ctx, a, *m, true, stream_kind);
+    a.q_factor = m->q_factor;
+    return run(ctx, a, *m, m->vdim, kM40Delta, stream_kind);
+}
+
+int m40llm_ext_time_mixing_async(M40llmCudaContext* ctx, const M40llmTimeMixing* m, uint32_t stream_kind) {
+    if (!ctx || !m || !m->rkv || !m->decay || !m->w0 || !m->u || !m->norm || !m->state || !m->out || !m->portions || !m->row_pos) return -1;
+    const uint64_t cols = (uint64_t)m->heads * m->dim;
+    if (m->ld_rkv < m->r_col + cols || m->ld_rkv < m->k_col + cols || m->ld_rkv < m->v_col + cols || m->ld_rkv < m->g_col + cols || m->ld_decay < cols) return -3;
+    M40MemoryArgs a{};
+    const float* x = static_cast<const float*>(m->rkv);
+    a.share = 1u;
+    a.q = x + m->r_col; a.k = x + m->k_col; a.v = x + m->v_col; a.ld = m->ld_rkv;
+    a.q_factor = 1.0f;
+    a.a = static_cast<const float*>(m->decay); a.ld_a = m->ld_decay;
+    a.dt_bias = static_cast<const float*>(m->w0); a.bonus = static_cast<const float*>(m->u);
+    a.norm = static_cast<const float*>(m->norm); a.norm_stride = m->dim;
+    a.gate = x + m->g_col; a.ld_gate = m->ld_rkv;
+    return run(ctx, a, *m, m->dim, kM40Mixing, stream_kind);
 }
 
 }  // extern "C"

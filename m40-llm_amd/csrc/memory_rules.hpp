@@ -1,8 +1,11 @@
 // What the kernels of recurrent layers with a matrix state share: matrix memory with exponential gates (a running maximum keeps its
-// exponents small; beside S a vector n), and the delta rule with one decay per key channel.  All of it is f32.
+// exponents small; beside S a vector n), the delta rule with one decay per key channel, and time mixing (one decay per key channel, what a token
+// writes is read by later tokens only, itself it sees through a bonus).  All of it is f32.
 #pragma once
 
 #include "packed_gemm.hpp"
+
+enum M40MemoryRule { kM40Memory = M40LLM_RULE_MEMORY, kM40Delta = M40LLM_RULE_DELTA, kM40Mixing = M40LLM_RULE_MIXING };
 
 struct M40MemoryArgs {
     uint32_t heads, share, dim, vdim, v4;          // share: heads that use one query / key head; v4: floats of a state row
@@ -11,6 +14,7 @@ struct M40MemoryArgs {
     const float *i, *f, *i_bias, *f_bias;          // matrix memory: gate logits of a row, ld apart
     float cap;
     const float *a, *beta, *A_log, *dt_bias;       // delta rule: decay logits (heads x dim, ld_a apart), write strength logits (ld_beta)
+    const float* bonus;                            // time mixing: heads x dim; its decay logits are a + dt_bias
     size_t ld_a, ld_beta;
     const float *norm, *gate;                      // the head's norm weights (norm_stride from head to head), gate logits (heads x vdim)
     uint32_t norm_stride;
@@ -41,6 +45,8 @@ __device__ __forceinline__ float m40_softplus(float z) {
 // logits of a row's gates
 __device__ __forceinline__ float m40_log_input_gate(const M40MemoryArgs& a, float z, uint32_t head) { return m40_soft_cap(z + a.i_bias[head], a.cap); }
 __device__ __forceinline__ float m40_log_forget_gate(const M40MemoryArgs& a, float z, uint32_t head) { return -m40_softplus(-m40_soft_cap(z + a.f_bias[head], a.cap)); }
+// time mixing: log2 of a key channel's decay; what is below this is nothing in f32
+__device__ __forceinline__ float m40_mixing_log2_decay(float z) { return fmaxf(-expf(z) * kM40Log2e, -160.0f); }
 // minus the log of a key channel's decay, less the head's factor exp(A_log)
 __device__ __forceinline__ float m40_channel_step(const M40MemoryArgs& a, uint32_t row, uint32_t head, uint32_t d) {
     return m40_softplus(a.a[(size_t)row * a.ld_a + head * a.dim + d] + a.dt_bias[head * a.dim + d]);

@@ -27,6 +27,7 @@ struct PackedArgs {
     const uint32_t* pages;
     int page_k_tiles;
     const uint32_t *jobs, *gather; // products per expert
+    int segment;                   // column tiles that read the same columns of a (0 = all): the next ones read those a_batch further
     __device__ int k_count(int batch) const { return k_total && k_total - batch * k_tiles < k_tiles ? k_total - batch * k_tiles : k_tiles; }
 };
 
@@ -52,7 +53,7 @@ __global__ __launch_bounds__(WAVES * 64) void rows_packed_kernel(PackedArgs g, M
     for (int m = 0; m < MT; ++m) {
         const int rt = row0 / 16 + m, last = (g.rows - 1) / 16, c = rt < last ? rt : last;
         if (JOBS == kJobGather) a[m] = static_cast<const T*>(g.a) + (long)g.gather[c * 16 + (lane & 15)] * g.lda + (lane >> 4) * 8;
-        else a[m] = static_cast<const T*>(g.a) + (JOBS == kAllRows ? batch * g.a_batch : 0) + (long)c * 16 * g.lda + lane * 8;
+        else a[m] = static_cast<const T*>(g.a) + (JOBS == kAllRows ? (g.segment ? tile0 / g.segment : batch) * g.a_batch : 0) + (long)c * 16 * g.lda + lane * 8;
     }
     const m40_bf16* w[NT];
 #pragma unroll
@@ -189,7 +190,7 @@ __global__ __launch_bounds__(256, 1) void tile_packed_kernel(PackedArgs g, M40Ep
         m0 = __builtin_amdgcn_readfirstlane((int)job[1]);
         g.rows = e.rows = m0 + __builtin_amdgcn_readfirstlane((int)job[2]);
     }
-    const m40_bf16* A = static_cast<const m40_bf16*>(g.a) + (kJobs ? 0 : batch * g.a_batch);
+    const m40_bf16* A = static_cast<const m40_bf16*>(g.a) + (kJobs ? 0 : (g.segment ? t0 / g.segment : batch) * g.a_batch);
     const m40_bf16* W = g.w + batch * g.w_batch;
     const int k_tiles = g.k_count(batch);
     // this wave's pieces of a step: operand tiles wave, wave + 4, ... of the A tiles, then of the W tiles
@@ -352,6 +353,9 @@ M40Epilogue<T> make_epilogue(const M40llmPackedGemm& p) {
     e.vec_act = p.ld_act % 4 == 0 && p.act_batch % 4 == 0 && aligned(p.out_act, 4 * sizeof(T));
     e.plain_tiles = (int)p.plain_tiles;
     e.activation = (int)p.activation;
+    e.act_alpha = p.act_alpha; e.act_limit = p.act_limit;
+    e.row_scale = static_cast<const float*>(p.row_scale);
+    e.out_scale = p.out_scale; e.out_cap = p.out_cap;
     e.n_tiles = (int)p.n_tiles; e.act_col = (int)p.act_col;
     e.gate = static_cast<const float*>(p.gate);
     e.ld_gate = (long)p.ld_gate;
@@ -437,7 +441,7 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
     const bool paged = p->epilogue == M40LLM_PACKED_KEYS || p->epilogue == M40LLM_PACKED_VALUES;
     const uint32_t k_parts = p->k_parts > 1u ? p->k_parts : 1u, part_tiles = (p->k_tiles + k_parts - 1) / k_parts;
-    if (p->act_dtype > 1u || p->epilogue > M40LLM_PACKED_SPLIT || p->activation > M40LLM_SILU || p->rows == 0 || p->batches == 0 || p->batches > 65535u ||
+    if (p->act_dtype > 1u || p->epilogue > M40LLM_PACKED_CAP || p->activation > M40LLM_LIMITED_GATE || p->rows == 0 || p->batches == 0 || p->batches > 65535u ||
         p->n_tiles == 0 || p->k_tiles == 0 || !m40_aligned16(p->a) || !m40_aligned16(p->w) || p->rows > 0x3fffffffu ||
         (p->batches > 1u && (p->a_batch % 32 != 0 || p->w_batch % 8 != 0)))
         return -3;
@@ -447,13 +451,19 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
                                                                   : p->epilogue == M40LLM_PACKED_PROJECT && p->plain_tiles == 0 && (p->job_rows == 128u) == !p->gather)))
         return -3;
     if (!paged && (p->lda % 32 != 0 || p->lda < (uint64_t)p->k_tiles * 32u)) return -3;
+    // a workgroup's column tiles lie in one segment
+    if (p->segment_tiles && (paged || p->jobs || p->batches != 1u || k_parts > 1u || p->epilogue == M40LLM_PACKED_PROJECT || p->segment_tiles % 16u != 0 || p->a_batch % 32 != 0 ||
+                             p->lda < (p->n_tiles - 1u) / p->segment_tiles * p->a_batch + (uint64_t)p->k_tiles * 32u))
+        return -3;
     if (k_parts > 1u && (p->epilogue != M40LLM_PACKED_STORE || p->batches != 1u || (k_parts - 1) * part_tiles >= p->k_tiles)) return -3;
     // packed results: whole tiles of columns
-    if ((p->epilogue == M40LLM_PACKED_GATED || p->epilogue == M40LLM_PACKED_ROTATE || p->epilogue == M40LLM_PACKED_SILU || p->epilogue == M40LLM_PACKED_SPLIT || (p->epilogue == M40LLM_PACKED_PROJECT && p->out_act)) &&
+    if ((p->epilogue == M40LLM_PACKED_GATED || p->epilogue == M40LLM_PACKED_ROTATE || p->epilogue == M40LLM_PACKED_SILU || p->epilogue == M40LLM_PACKED_SPLIT || p->epilogue == M40LLM_PACKED_TANH ||
+         (p->epilogue == M40LLM_PACKED_PROJECT && p->out_act)) &&
         (p->ld_act % 32 != 0 || p->act_col % 4 != 0))
         return -3;
     const bool wide_stores = p->ld_act % 4 == 0 && reinterpret_cast<uintptr_t>(p->out_act) % (p->act_dtype == M40LLM_ACT_F32 ? 16 : 8) == 0;
     switch (p->epilogue) {
+        case M40LLM_PACKED_CAP: if (p->batches != 1u || !(p->out_cap >= 0.0f)) return -4; [[fallthrough]];
         case M40LLM_PACKED_STORE: case M40LLM_PACKED_ADD: if (!p->out_f32 || p->cols > p->n_tiles * 16u) return -4; break;
         case M40LLM_PACKED_STORE_ACT: if (!p->out_act || p->cols > p->n_tiles * 16u) return -4; break;
         case M40LLM_PACKED_GATED: if (!p->out_act || !p->gate || p->cols > p->n_tiles * 16u) return -4; break;
@@ -470,7 +480,7 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
                 p->plain_tiles % 2 != 0 || p->n_tiles % 2 != 0 || p->plain_tiles > p->n_tiles)
                 return -4;
             break;
-        case M40LLM_PACKED_SILU: case M40LLM_PACKED_SPLIT:
+        case M40LLM_PACKED_SILU: case M40LLM_PACKED_SPLIT: case M40LLM_PACKED_TANH:
             if ((p->plain_tiles > 0 && !p->out_f32) || !p->out_act || !wide_stores || p->plain_tiles > p->n_tiles || p->batches != 1u) return -4;
             break;
         case M40LLM_PACKED_KEYS: case M40LLM_PACKED_VALUES:
@@ -486,6 +496,7 @@ int m40llm_ext_packed_gemm_async(M40llmCudaContext* ctx, const M40llmPackedGemm*
     g.lda = (long)p->lda; g.a_batch = (long)p->a_batch * 16; g.w_batch = (long)p->w_batch;
     g.n_tiles = (int)p->n_tiles; g.k_tiles = (int)p->k_tiles; g.rows = (int)p->rows; g.k_stride = (int)p->k_tiles;
     g.pages = p->pages; g.page_k_tiles = (int)p->page_k_tiles;
+    g.segment = (int)p->segment_tiles;
     int batches = (int)p->batches;
     if (k_parts > 1u) {
         g.k_total = (int)p->k_tiles; g.k_tiles = (int)part_tiles;

@@ -91,8 +91,11 @@ struct M40Epilogue {
     long out_batch, act_batch;     // elements (packed: columns) from batch (head, part of K) to batch
     int cols;                      // columns stored (STORE, ADD, STORE_ACT, GATED)
     bool vec_out, vec_act;         // four neighbouring columns may be stored at once
-    int plain_tiles, act_col;      // PROJECT, SILU, SPLIT: tiles before those that go to out_act; the first column of out_act they take
+    int plain_tiles, act_col;      // PROJECT, SILU, SPLIT, TANH: tiles before those that go to out_act; the first column of out_act they take
     int activation;                // PROJECT
+    float act_alpha, act_limit;
+    const float* row_scale;        // PROJECT: on both sums of a row (NULL = ones)
+    float out_scale, out_cap;      // CAP
     int n_tiles;                   // KEYS, VALUES
     const float* gate;             // GATED: logits, [rows][ld_gate], one column per batch
     long ld_gate;
@@ -136,11 +139,17 @@ __device__ __forceinline__ void m40_epilogue_tile(const M40Epilogue<T>& e, int b
     const int col = tile * 16 + 4 * (lane >> 4), row = row0 + (lane & 15);
     if (row >= e.rows) return;
     switch (e.kind) {
+        case M40LLM_PACKED_CAP:
+#pragma unroll
+            for (int r = 0; r < 4; ++r) v[r] = e.out_cap > 0.0f ? e.out_cap * tanhf(v[r] * e.out_scale / e.out_cap) : v[r] * e.out_scale;
+            m40_store_cols<float>(e.out_f32 + (long)row * e.ld_out + col, v, e.cols - col, e.vec_out);
+            return;
         case M40LLM_PACKED_SILU:
         case M40LLM_PACKED_SPLIT:
+        case M40LLM_PACKED_TANH:
             if (tile >= e.plain_tiles) {
 #pragma unroll
-                for (int r = 0; r < 4; ++r) v[r] = e.kind == M40LLM_PACKED_SILU ? m40_silu(v[r]) : v[r];
+                for (int r = 0; r < 4; ++r) v[r] = e.kind == M40LLM_PACKED_SILU ? m40_silu(v[r]) : e.kind == M40LLM_PACKED_TANH ? tanhf(v[r]) : v[r];
                 m40_store_packed<T>(e.out_act, row, e.act_col + col - e.plain_tiles * 16, e.ld_act, v, 4, true);
                 return;
             }
@@ -204,8 +213,18 @@ __device__ __forceinline__ void m40_epilogue_pair(const M40Epilogue<T>& e, int r
     const int col = pair * 16 + 4 * (lane >> 4), row = row0 + (lane & 15);
     if (row >= e.rows) return;
     m40_float4 y;
+    if (e.activation == M40LLM_LIMITED_GATE) {
+        const float f = e.row_scale ? e.row_scale[row] : 1.0f;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) y[r] = (e.activation == M40LLM_SILU ? m40_silu(g[r]) : m40_gelu_tanh(g[r])) * u[r];
+        for (int r = 0; r < 4; ++r) {
+            const float z = fminf(g[r] * f, e.act_limit), up = fminf(fmaxf(u[r] * f, -e.act_limit), e.act_limit);
+            y[r] = z * m40_sigmoid(e.act_alpha * z) * (up + 1.0f);
+        }
+    } else {
+        const float f = e.row_scale ? e.row_scale[row] : 1.0f;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) y[r] = (e.activation == M40LLM_SILU ? m40_silu(g[r] * f) : m40_gelu_tanh(g[r] * f)) * (u[r] * f);
+    }
     m40_store_packed<T>(e.out_act, row, e.act_col + col, e.ld_act, y, 4, true);
 }
 #endif  // __HIPCC__

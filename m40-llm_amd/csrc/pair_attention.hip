@@ -1,7 +1,8 @@
 // Attention over a paged cache of keys and values (include/m40llm.h has the page order), in kernels for one or two maps a head (M).
 // Two maps, differential attention: softmaxes of their own queries and keys over the same values; the second map's result is taken off the
 // first's, lambda times, and what is left is normed over the head's value dimensions and gated.  One map: softmax attention, its result
-// scaled and, where there is a gate, gated column by column.
+// scaled and, where there is a gate, gated column by column.  One map in the extended form (X): scores capped by a tanh, less a slope times the
+// distance of key and query, within a window of the newest tokens, beside a sink in the denominator; all of these are optional.
 //
 // Products are formed transposed, S' = K Q' and O' = V' P': a lane holds the scores of one query (lane % 16) for keys 4 g + r of every
 // 16, and pages hold values with their tokens in exactly that order, so the weights a lane computes are its operand of the second
@@ -13,7 +14,7 @@
 //                    the odd pages are walked side by side and the groups' sums meet at the end, which halves the longest walk
 // pair_f32_kernel    one workgroup a row and head, plain f32 arithmetic
 //
-// Maxima are reference points that move only when some score lies 8 (as a power of two) above them.
+// Maxima are reference points that move only when some score lies 8 (as a power of two) above them.  The sink joins once, when everything is summed.
 #include "pair_cache.hpp"
 
 namespace {
@@ -29,6 +30,25 @@ struct PairArgs {
     float* partial_o;      // [splits][rows * heads][maps][16 v_tiles]
     float* partial_ml;     // [splits][rows * heads][maps][2]: reference, sum
 };
+
+// Window of the newest tokens (all: more than there can be), the first page that a query at `pos` sees, and whether every query of a range
+// sees the whole page.
+__device__ __forceinline__ uint32_t window_of(const M40llmPairAttention& a) { return a.window ? a.window : 0x7fffffffu; }
+template <bool X>
+__device__ __forceinline__ uint32_t first_page(const M40llmPairAttention& a, uint32_t pos) {
+    const uint32_t w = window_of(a);
+    return X && pos + 1u > w ? (pos + 1u - w) / kPage : 0u;
+}
+template <bool X>
+__device__ __forceinline__ bool whole_page(const M40llmPairAttention& a, uint32_t page, uint32_t first_pos, uint32_t last_pos) {
+    return page * kPage + kPage - 1u <= first_pos && (!X || page * kPage + window_of(a) > last_pos);
+}
+// one over the sum l of weights relative to 2^ref, the sink's included
+__device__ __forceinline__ float inverse_sum(const M40llmPairAttention& a, uint32_t head, float ref, float l) {
+    if (!a.sink) return 1.0f / l;
+    const float sink = static_cast<const float*>(a.sink)[head] * kLog2e, to = fmaxf(ref, sink), f = __builtin_amdgcn_exp2f(ref - to);
+    return f / (l * f + __builtin_amdgcn_exp2f(sink - to));
+}
 
 // what o (map 1's sums times f1 less map 2's times f2) is multiplied by: sum of squares of o over the head's dimensions in ss
 __device__ __forceinline__ float last_factor(const M40llmPairAttention& a, float ss, uint32_t row, uint32_t head) {
@@ -58,6 +78,31 @@ struct PairState {
 #pragma unroll
                 for (int j = 0; j < DVT; ++j) o[m][j][b] = m40_float4{0.f, 0.f, 0.f, 0.f};
             }
+    }
+    // X: products of queries and keys become powers of two that weigh() takes as they are
+    __device__ __forceinline__ void extend(const M40llmPairAttention& a, const float (&slope)[B], m40_float4 (&s)[4][B], bool whole, uint32_t key0) const {
+        const float window = (float)window_of(a), c = a.cap > 0.0f ? a.scale * 2.0f * kLog2e / a.cap : a.scale * kLog2e, cap = a.cap * kLog2e;
+#pragma unroll
+        for (int b = 0; b < B; ++b) {
+            const float back = (float)((int)key0 - (int)pos[b]);
+            if (a.cap > 0.0f) {              // cap tanh(x) = cap - 2 cap / (1 + exp(2 x))
+#pragma unroll
+                for (int t = 0; t < 4; ++t)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) s[t][b][r] = fmaf(-2.0f * cap, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(s[t][b][r] * c)), cap);
+            } else {
+#pragma unroll
+                for (int t = 0; t < 4; ++t) s[t][b] *= c;
+            }
+#pragma unroll
+            for (int t = 0; t < 4; ++t)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const float d = back + (float)(t * 16 + r);
+                    s[t][b][r] = fmaf(slope[b], d, s[t][b][r]);
+                    if (!whole) s[t][b][r] = d <= 0.0f && d > -window ? s[t][b][r] : -INFINITY;
+                }
+        }
     }
     // the scores of a map become weights: operands of the value product
     __device__ __forceinline__ void weigh(int m, m40_float4 (&s)[4][B], float c, bool whole, uint32_t key0, m40_bf16x8 (&pf)[B][2]) {
@@ -134,7 +179,7 @@ struct PairState {
     // the result of query block b to its row
     __device__ __forceinline__ void finish(const PairArgs& p, int b, uint32_t row, uint32_t head, bool live, int g) const {
         const int vt = (int)p.page.v_tiles, vdim = (int)p.a.vdim;
-        const float f1 = 1.0f / m40_add_xor32(m40_add_xor16(sum[0][b]));
+        const float l = m40_add_xor32(m40_add_xor16(sum[0][b])), f1 = M == 1 ? inverse_sum(p.a, head, ref[0][b], l) : 1.0f / l;
         if constexpr (M == 1) {
             if (!live) return;
             const bool vec = p.a.gate && vdim % 4 == 0 && p.a.ld_gate % 4 == 0 && m40_aligned16(p.a.gate);
@@ -176,7 +221,10 @@ struct PairState {
     }
 };
 
-template <int M, int DKT, int DVT>
+// what a power of two loses per token of distance
+__device__ __forceinline__ float slope_of(const M40llmPairAttention& a, uint32_t head) { return a.slopes ? static_cast<const float*>(a.slopes)[head] * kLog2e : 0.0f; }
+
+template <int M, int DKT, int DVT, bool X>
 __global__ __launch_bounds__(256, 1) void pair_rows_kernel(PairArgs p) {
     extern __shared__ __align__(16) float join_lds[];      // three waves' sums
     const M40llmPairAttention& a = p.a;
@@ -186,13 +234,14 @@ __global__ __launch_bounds__(256, 1) void pair_rows_kernel(PairArgs p) {
     const bool live = (uint32_t)li < count;
     const uint32_t query = q0 + (live ? (uint32_t)li : count - 1u), row = query / p.group, head = kv * p.group + query % p.group;
     const uint32_t last_row = (q0 + count - 1u) / p.group;
-    const uint32_t pages = a.row_pos[last_row] / kPage + 1u, per = (pages + a.splits - 1u) / a.splits;
-    const uint32_t page0 = blockIdx.z * per, page1 = page0 + per < pages ? page0 + per : pages;
+    const uint32_t first_pos = a.row_pos[q0 / p.group], last_pos = a.row_pos[last_row];
+    const uint32_t pages = last_pos / kPage + 1u, skipped = first_page<X>(a, first_pos), per = (pages - skipped + a.splits - 1u) / a.splits;
+    const uint32_t page0 = skipped + blockIdx.z * per, page1 = page0 + per < pages ? page0 + per : pages;
     const uint32_t* table = a.page_table + (size_t)a.row_slot[last_row] * a.max_pages;
     PairState<M, DKT, DVT, 1> s;
     s.clear();
     s.pos[0] = a.row_pos[row];
-    const uint32_t first_pos = a.row_pos[q0 / p.group];
+    const float slope[1] = {X ? slope_of(a, head) : 0.0f};
     const m40_bf16* q = static_cast<const m40_bf16*>(a.queries) + ((size_t)row * a.heads + head) * ((uint32_t)M * kt * 32u) + g * 8;
 #pragma unroll
     for (int m = 0; m < M; ++m)
@@ -206,7 +255,7 @@ __global__ __launch_bounds__(256, 1) void pair_rows_kernel(PairArgs p) {
     for (uint32_t n = page0 + wave; n < page1; n += 4u) {
         const m40_bf16* keys = cache + table[n] * p.page.elements();
         const m40_bf16* values = keys + p.page.key_elements();
-        const bool whole = n * kPage + kPage - 1u <= first_pos;
+        const bool whole = whole_page<X>(a, n, first_pos, last_pos);
         m40_bf16x8 pf[M][1][2], vf[DVT][2];
 #pragma unroll
         for (int m = 0; m < M; ++m) {
@@ -226,7 +275,8 @@ __global__ __launch_bounds__(256, 1) void pair_rows_kernel(PairArgs p) {
 #pragma unroll
                     for (int h = 0; h < 2; ++h) vf[j][h] = *reinterpret_cast<const m40_bf16x8*>(values + ((j < vt ? j : vt - 1) * 2 + h) * kM40Tile);
             }
-            s.weigh(m, sc, c, whole, n * kPage + 4 * g, pf[m]);
+            if constexpr (X) s.extend(a, slope, sc, whole, n * kPage + 4 * g);
+            s.weigh(m, sc, X ? 1.0f : c, X || whole, n * kPage + 4 * g, pf[m]);
         }
 #pragma unroll
         for (int j = 0; j < DVT; ++j)
@@ -286,13 +336,15 @@ __global__ __launch_bounds__(256) void pair_join_kernel(PairArgs p) {
         const float top = m40_max64(ref);
         if (lane == 0) part[wave] = top;
         __syncthreads();
-        const float to = fmaxf(fmaxf(part[0], part[1]), fmaxf(part[2], part[3]));
+        const bool sunk = M == 1 && a.sink;
+        const float sink = sunk ? static_cast<const float*>(a.sink)[head] * kLog2e : kNothing;
+        const float to = fmaxf(fmaxf(fmaxf(part[0], part[1]), fmaxf(part[2], part[3])), sink);
         const float e = __builtin_amdgcn_exp2f(ref - to), den = m40_sum64(l * e);
         __syncthreads();
         if (tid < a.splits) weight[m][tid] = e;
         if (lane == 0) part[wave] = den;
         __syncthreads();
-        const float inv = (m ? -a.lambda : 1.0f) / (part[0] + part[1] + part[2] + part[3]);
+        const float inv = (m ? -a.lambda : 1.0f) / (part[0] + part[1] + part[2] + part[3] + (sunk ? __builtin_amdgcn_exp2f(sink - to) : 0.0f));
         for (uint32_t d0 = 0; d0 < width; d0 += 128u) {
             const uint32_t d = d0 + (tid & 31u) * 4u;
             m40_float4 acc = {0.f, 0.f, 0.f, 0.f};
@@ -325,7 +377,7 @@ __global__ __launch_bounds__(256) void pair_join_kernel(PairArgs p) {
     if (tid < a.vdim) static_cast<T*>(a.out)[m40_packed_at(row, head * a.vdim + tid, a.ld_out >> 5)] = M40Act<T>::from(o * f);
 }
 
-template <int M, int DKT, int DVT, int QB, int GROUPS, int PER_CU>
+template <int M, int DKT, int DVT, int QB, int GROUPS, int PER_CU, bool X>
 __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArgs p) {
     typedef __attribute__((address_space(3))) void* lds_dst_t;
     typedef const __attribute__((address_space(1))) void* global_src_t;
@@ -336,7 +388,7 @@ __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArg
     const int kt = (int)p.page.k_tiles, vt = (int)p.page.v_tiles, page_tiles = 4 * M * kt + 2 * vt;
     const uint32_t kv = blockIdx.x, q0 = a.tiles[2 * blockIdx.y], count = a.tiles[2 * blockIdx.y + 1];
     const uint32_t last_row = (q0 + count - 1u) / p.group;
-    const uint32_t pages = a.row_pos[last_row] / kPage + 1u, last = pages - 1u;
+    const uint32_t last = a.row_pos[last_row] / kPage, skipped = first_page<X>(a, a.row_pos[q0 / p.group]), pages = last + 1u - skipped;
     const uint32_t* table = a.page_table + (size_t)a.row_slot[last_row] * a.max_pages;
     const m40_bf16* cache = static_cast<const m40_bf16*>(a.cache) + kv * p.page.head_elements() + lane * 8;
     // a kv head's part of a page is contiguous: keys, then values
@@ -346,7 +398,7 @@ __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArg
             __builtin_amdgcn_global_load_lds((global_src_t)(src + (size_t)i * kM40Tile), (lds_dst_t)(lds + ((group * 2 + buf) * page_tiles + i) * 1024), 16, 0, 0);
     };
     const uint32_t steps = (pages + GROUPS - 1u) / GROUPS;
-    auto page_of = [&](uint32_t step) { const uint32_t n = step * GROUPS + group; return n < last ? n : last; };    // past the end: the last again
+    auto page_of = [&](uint32_t step) { const uint32_t n = skipped + step * GROUPS + group; return n < last ? n : last; };    // past the end: the last again
     issue(0, table[page_of(0)]);
     uint32_t next = table[page_of(1)];
     PairState<M, DKT, DVT, QB> s;
@@ -375,6 +427,9 @@ __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArg
     const bool wave_live = i_first < count;
     const uint32_t pos_first = a.row_pos[(q0 + (wave_live ? i_first : count - 1u)) / p.group], pos_last = a.row_pos[(q0 + (i_last < count ? i_last : count - 1u)) / p.group];
     const float c = a.scale * kLog2e;
+    float slope[QB];
+#pragma unroll
+    for (int b = 0; b < QB; ++b) slope[b] = X ? slope_of(a, head[b]) : 0.0f;
     int buf = 0;
     for (uint32_t step = 0; step < steps; ++step, buf ^= 1) {
         m40_wait_and_meet<0>();                  // the pages have landed, and nobody reads the other buffers any more
@@ -382,11 +437,11 @@ __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArg
             issue(buf ^ 1, next);
             next = table[page_of(step + 2u)];
         }
-        const uint32_t n = step * GROUPS + group;
-        if (!wave_live || n > last || n * kPage > pos_last) continue;
+        const uint32_t n = skipped + step * GROUPS + group;
+        if (!wave_live || n > last || n * kPage > pos_last || (X && n < first_page<X>(a, pos_first))) continue;
         const uint8_t* keys = lds + (group * 2 + buf) * page_tiles * 1024 + lane * 16;
         const uint8_t* values = keys + 4 * M * kt * 1024;
-        const bool whole = n * kPage + kPage - 1u <= pos_first;
+        const bool whole = whole_page<X>(a, n, pos_first, pos_last);
         m40_bf16x8 pf[M][QB][2];
 #pragma unroll
         for (int m = 0; m < M; ++m) {
@@ -407,7 +462,8 @@ __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArg
                     }
                 }
             __builtin_amdgcn_s_setprio(0);
-            s.weigh(m, sc, c, whole, n * kPage + 4 * g, pf[m]);
+            if constexpr (X) s.extend(a, slope, sc, whole, n * kPage + 4 * g);
+            s.weigh(m, sc, X ? 1.0f : c, X || whole, n * kPage + 4 * g, pf[m]);
         }
         __builtin_amdgcn_s_setprio(1);
 #pragma unroll
@@ -452,8 +508,9 @@ __global__ __launch_bounds__(256) void pair_f32_kernel(PairArgs p) {
     if (tid < (uint32_t)M) { stat[tid][0] = -INFINITY; stat[tid][1] = 0.0f; }
     const uint32_t pos = a.row_pos[row], pages = pos / kPage + 1u;
     const uint32_t* table = a.page_table + (size_t)a.row_slot[row] * a.max_pages;
+    const float slope = M == 1 && a.slopes ? static_cast<const float*>(a.slopes)[head] : 0.0f;
     __syncthreads();
-    for (uint32_t n = 0; n < pages; ++n) {
+    for (uint32_t n = first_page<M == 1>(a, pos); n < pages; ++n) {
         const float* page = static_cast<const float*>(a.cache) + table[n] * p.page.elements() + kv * p.page.head_elements();
         // two lanes a token and map of two, four a token of one
         constexpr uint32_t kLanes = 4u / M;
@@ -462,7 +519,13 @@ __global__ __launch_bounds__(256) void pair_f32_kernel(PairArgs p) {
         for (uint32_t d = tid % kLanes; d < a.dim; d += kLanes) x = fmaf(q[map][d], page[p.page.key_at(map, t, d)], x);
         x += m40_dpp_f<M40_DPP_XOR1>(x);
         if (kLanes == 4u) x += m40_dpp_f<M40_DPP_XOR2>(x);
-        if (tid % kLanes == 0u) s[map][t] = n * kPage + t <= pos ? x * a.scale : -INFINITY;
+        x *= a.scale;
+        if (M == 1) {
+            if (a.cap > 0.0f) x = a.cap * tanhf(x / a.cap);
+            x -= slope * ((float)pos - (float)(n * kPage + t));
+        }
+        const uint32_t key = n * kPage + t;
+        if (tid % kLanes == 0u) s[map][t] = key <= pos && (M != 1 || pos - key < window_of(a)) ? x : -INFINITY;
         __syncthreads();
         if (tid < 64u * M) {                 // a wave a map; a page of the range holds a seen token
             const uint32_t m = tid >> 6, l = tid & 63u;
@@ -481,8 +544,14 @@ __global__ __launch_bounds__(256) void pair_f32_kernel(PairArgs p) {
         __syncthreads();
     }
     if constexpr (M == 1) {
+        float below = stat[0][1], f = 1.0f;
+        if (a.sink) {
+            const float sink = static_cast<const float*>(a.sink)[head], to = fmaxf(stat[0][0], sink);
+            f = expf(stat[0][0] - to);
+            below = below * f + expf(sink - to);
+        }
         if (tid < a.vdim)
-            static_cast<float*>(a.out)[m40_packed_at(row, head * a.vdim + tid, a.ld_out >> 5)] = o[0][tid] / stat[0][1] * column_factor(a, row, head, tid);
+            static_cast<float*>(a.out)[m40_packed_at(row, head * a.vdim + tid, a.ld_out >> 5)] = o[0][tid] * f / below * column_factor(a, row, head, tid);
         return;
     }
     const float y = tid < a.vdim ? o[0][tid] / stat[0][1] - a.lambda * (o[M - 1][tid] / stat[M - 1][1]) : 0.0f;
@@ -495,55 +564,61 @@ __global__ __launch_bounds__(256) void pair_f32_kernel(PairArgs p) {
 
 constexpr int kLdsMax = 160 * 1024;
 
-template <int M, int DKT, int DVT>
+template <int M, int DKT, int DVT, bool X>
 int launch_rows(hipStream_t stream, const PairArgs& p) {
     constexpr int lds = 3 * 64 * 4 * PairState<M, DKT, DVT, 1>::kFloats;
-    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(pair_rows_kernel<M, DKT, DVT>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(pair_rows_kernel<M, DKT, DVT, X>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
     if (attr != hipSuccess) return -2;
-    pair_rows_kernel<M, DKT, DVT><<<dim3(p.a.n_tiles, p.a.kv_heads, p.a.splits), 256, lds, stream>>>(p);
+    pair_rows_kernel<M, DKT, DVT, X><<<dim3(p.a.n_tiles, p.a.kv_heads, p.a.splits), 256, lds, stream>>>(p);
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
 int page_lds(const PairArgs& p, int groups) { return groups * 2 * (int)(4u * p.page.maps * p.page.k_tiles + 2u * p.page.v_tiles) * 1024; }
-template <int M, int DKT, int DVT, int QB, int GROUPS, int PER_CU>
+template <int M, int DKT, int DVT, int QB, int GROUPS, int PER_CU, bool X>
 int launch_tile(hipStream_t stream, const PairArgs& p) {
     static const hipError_t attr =
-        hipFuncSetAttribute(reinterpret_cast<const void*>(pair_tile_kernel<M, DKT, DVT, QB, GROUPS, PER_CU>), hipFuncAttributeMaxDynamicSharedMemorySize, kLdsMax);
+        hipFuncSetAttribute(reinterpret_cast<const void*>(pair_tile_kernel<M, DKT, DVT, QB, GROUPS, PER_CU, X>), hipFuncAttributeMaxDynamicSharedMemorySize, kLdsMax);
     if (attr != hipSuccess) return -2;
     constexpr int join = GROUPS == 2 ? 4 * 64 * 4 * PairState<M, DKT, DVT, QB>::kFloats : 0;
     static_assert(join <= kLdsMax, "the joining of two groups does not fit");
     const int pages = page_lds(p, GROUPS);
-    pair_tile_kernel<M, DKT, DVT, QB, GROUPS, PER_CU><<<dim3(p.a.kv_heads, p.a.n_tiles), GROUPS * 256, pages > join ? pages : join, stream>>>(p);
+    pair_tile_kernel<M, DKT, DVT, QB, GROUPS, PER_CU, X><<<dim3(p.a.kv_heads, p.a.n_tiles), GROUPS * 256, pages > join ? pages : join, stream>>>(p);
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
 // PER_CU: workgroups of one group a CU that fit
-template <int M, int DKT, int DVT, int PER_CU>
+template <int M, int DKT, int DVT, int PER_CU, bool X>
 int launch_tile_any(hipStream_t stream, const PairArgs& p, int num_cus) {
     // with enough workgroups the short ones fill in behind the long ones
     if (page_lds(p, 2) <= kLdsMax && (uint64_t)p.a.kv_heads * p.a.n_tiles <= 3ull * (uint32_t)num_cus)
-        return p.a.tile_queries == 64u ? launch_tile<M, DKT, DVT, 1, 2, PER_CU>(stream, p) : launch_tile<M, DKT, DVT, 2, 2, PER_CU>(stream, p);
-    return p.a.tile_queries == 64u ? launch_tile<M, DKT, DVT, 1, 1, PER_CU>(stream, p) : launch_tile<M, DKT, DVT, 2, 1, PER_CU>(stream, p);
+        return p.a.tile_queries == 64u ? launch_tile<M, DKT, DVT, 1, 2, PER_CU, X>(stream, p) : launch_tile<M, DKT, DVT, 2, 2, PER_CU, X>(stream, p);
+    return p.a.tile_queries == 64u ? launch_tile<M, DKT, DVT, 1, 1, PER_CU, X>(stream, p) : launch_tile<M, DKT, DVT, 2, 1, PER_CU, X>(stream, p);
 }
 
 bool tile_served(uint32_t maps, uint32_t k_tiles, uint32_t v_tiles) { return 2u * (4u * maps * k_tiles + 2u * v_tiles) * 1024u <= (uint32_t)kLdsMax; }
 
 // PER_CU of heads of 128 dimensions
-template <int M, int PER_CU>
+template <int M, int PER_CU, bool X>
 int launch_form(hipStream_t stream, const PairArgs& p, uint32_t form, int num_cus) {
     const uint32_t kt = p.page.k_tiles, vt = p.page.v_tiles;
     if (form == 1u) {
-        if (kt <= 2u && vt <= 4u) return launch_tile_any<M, 2, 4, 2>(stream, p, num_cus);
-        if (kt <= 2u && vt <= 8u) return launch_tile_any<M, 2, 8, 2>(stream, p, num_cus);
-        if (kt <= 4u && vt <= 8u) return launch_tile_any<M, 4, 8, PER_CU>(stream, p, num_cus);
-        return launch_tile<M, 8, 16, 1, 1, 1>(stream, p);
+        if (kt <= 2u && vt <= 4u) return launch_tile_any<M, 2, 4, 2, X>(stream, p, num_cus);
+        if (kt <= 2u && vt <= 8u) return launch_tile_any<M, 2, 8, 2, X>(stream, p, num_cus);
+        if (kt <= 4u && vt <= 8u) return launch_tile_any<M, 4, 8, PER_CU, X>(stream, p, num_cus);
+        return launch_tile<M, 8, 16, 1, 1, 1, X>(stream, p);
     }
     int rc;
-    if (kt <= 2u && vt <= 4u) rc = launch_rows<M, 2, 4>(stream, p);
-    else if (kt <= 2u && vt <= 8u) rc = launch_rows<M, 2, 8>(stream, p);
-    else if (kt <= 4u && vt <= 8u) rc = launch_rows<M, 4, 8>(stream, p);
-    else rc = launch_rows<M, 8, 16>(stream, p);
+    if (kt <= 2u && vt <= 4u) rc = launch_rows<M, 2, 4, X>(stream, p);
+    else if (kt <= 2u && vt <= 8u) rc = launch_rows<M, 2, 8, X>(stream, p);
+    else if (kt <= 4u && vt <= 8u) rc = launch_rows<M, 4, 8, X>(stream, p);
+    else rc = launch_rows<M, 8, 16, X>(stream, p);
     if (rc != 0 || p.a.splits == 1u) return rc;
     pair_join_kernel<m40_bf16, M><<<p.a.n_rows * p.a.heads, 256, 0, stream>>>(p);
     return hipGetLastError() == hipSuccess ? 0 : -2;
+}
+
+int launch(hipStream_t stream, const PairArgs& p, uint32_t form, int num_cus) {
+    if (p.a.maps == 2u) return launch_form<2, 1, false>(stream, p, form, num_cus);
+    if (p.a.window || p.a.cap > 0.0f || p.a.slopes) return launch_form<1, 2, true>(stream, p, form, num_cus);
+    return launch_form<1, 2, false>(stream, p, form, num_cus);
 }
 
 }  // namespace
@@ -567,7 +642,8 @@ int m40llm_ext_pair_attention_async(M40llmCudaContext* ctx, const M40llmPairAtte
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
     const uint32_t most = m40llm_ext_pair_attention_tile_queries(a->act_dtype, a->maps, a->dim, a->vdim);
     if (a->act_dtype > 1u || a->form > 1u || a->heads == 0 || a->kv_heads == 0 || a->heads % a->kv_heads != 0 || most == 0 || !(a->scale > 0.0f) || a->ld_out % 32u != 0 ||
-        a->ld_out < a->heads * a->vdim || a->n_rows == 0 || !m40_aligned16(a->queries) || !m40_aligned16(a->cache))
+        a->ld_out < a->heads * a->vdim || a->n_rows == 0 || !m40_aligned16(a->queries) || !m40_aligned16(a->cache) || a->window > 0x7fffffffu || !(a->cap >= 0.0f) ||
+        (a->maps != 1u && (a->window || a->cap > 0.0f || a->slopes || a->sink)))
         return -3;
     PairArgs p{*a, M40PairPage(a->maps, a->kv_heads, a->dim, a->vdim), a->heads / a->kv_heads, nullptr, nullptr};
     (void)hipGetLastError();
@@ -580,7 +656,7 @@ int m40llm_ext_pair_attention_async(M40llmCudaContext* ctx, const M40llmPairAtte
     const uint32_t kt = p.page.k_tiles, vt = p.page.v_tiles;
     if (a->form == 1u) {
         if ((a->tile_queries != 64u && a->tile_queries != 128u) || a->tile_queries > most || a->n_tiles > 65535u || !tile_served(a->maps, kt, vt)) return -3;
-        return a->maps == 1u ? launch_form<1, 2>(stream, p, 1u, ctx->num_cus) : launch_form<2, 1>(stream, p, 1u, ctx->num_cus);
+        return launch(stream, p, 1u, ctx->num_cus);
     }
     if (a->splits == 0 || a->splits > (uint32_t)kJoinSplits || a->kv_heads > 65535u) return -3;
     if (a->splits > 1u) {
@@ -590,7 +666,7 @@ int m40llm_ext_pair_attention_async(M40llmCudaContext* ctx, const M40llmPairAtte
         p.partial_o = static_cast<float*>(a->partial);
         p.partial_ml = p.partial_o + (size_t)a->splits * a->n_rows * a->heads * a->maps * vt * 16u;
     }
-    return a->maps == 1u ? launch_form<1, 2>(stream, p, 0u, ctx->num_cus) : launch_form<2, 1>(stream, p, 0u, ctx->num_cus);
+    return launch(stream, p, 0u, ctx->num_cus);
 }
 
 }  // extern "C"

@@ -76,7 +76,7 @@ __global__ __launch_bounds__(kThreads) void stream_update_kernel(M40llmStreamUpd
                 for (uint32_t j = 0; j < 4; ++j) {
                     const size_t pick = (size_t)row * a.top + (j0 + j < a.top ? j0 + j : j0);
                     at[j] = a.place[pick];
-                    f[j] = j0 + j < a.top ? static_cast<const float*>(a.weight)[pick] : 0.0f;
+                    f[j] = j0 + j >= a.top ? 0.0f : a.weight ? static_cast<const float*>(a.weight)[pick] : 1.0f;
                 }
 #pragma unroll
                 for (uint32_t j = 0; j < 4; ++j) load8<T, VEC>(static_cast<const T*>(a.expert_out) + (size_t)at[j] * a.ld_expert, g * 8u, width, v[j]);
@@ -227,7 +227,7 @@ extern "C" int m40llm_ext_stream_update_async(M40llmCudaContext* ctx, const M40l
         (u->w && (u->ld_h < u->width || u->ld_h % 32u != 0 || !m40_aligned16(u->h) || (u->h_rows && !m40_aligned16(u->h_rows)))))
         return -3;
     if (u->row_index && u->w) return -4;           // rows of h are those of the step
-    if (write && (!u->streams_x || !u->mix || !u->share || (u->place ? !u->expert_out || !u->weight || u->top == 0 : !u->planes))) return -4;
+    if (write && (!u->streams_x || !u->mix || !u->share || (u->place ? !u->expert_out || u->top == 0 : !u->planes))) return -4;
     const bool vec = u->width % 8u == 0 && u->stream_stride % 4u == 0 && m40_aligned16(u->streams_x) && (!u->x0 || m40_aligned16(u->x0)) && (!u->x_out || m40_aligned16(u->x_out)) &&
                      (u->place ? u->ld_expert % 8u == 0 && m40_aligned16(u->expert_out) : u->plane_stride % 4u == 0 && (!u->n_planes || m40_aligned16(u->planes)));
     (void)hipGetLastError();

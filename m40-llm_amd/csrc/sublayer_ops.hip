@@ -150,12 +150,12 @@ __global__ __launch_bounds__(kThreads) void norm_gate_rows_kernel(const float* _
     }
 }
 
-// A workgroup takes 16 rows and one unit: a map of a query head, a map of a key head, or a value head; 16 lanes a row.
+// A workgroup takes 16 rows and one unit: a map (of one or two) of a query head, a map of a key head, or a value head; 16 lanes a row.
 enum { kQueries = 0, kKeys = 1, kValues = 2 };
 template <class T, int W, int N>
 __device__ __forceinline__ void split_unit(const M40llmPairSplit& a, const M40PairPage& page, int kind, uint32_t unit, uint32_t row, uint32_t lane) {
     const uint32_t n = kind == kValues ? a.vdim : a.dim, col0 = (kind == kQueries ? 0u : kind == kKeys ? a.k_offset : a.v_offset) + unit * n;
-    const uint32_t all = (kind == kQueries ? 2u * a.heads : kind == kKeys ? 2u * a.kv_heads : a.kv_heads) * n;      // columns of this kind
+    const uint32_t all = (kind == kQueries ? a.maps * a.heads : kind == kKeys ? a.maps * a.kv_heads : a.kv_heads) * n;      // columns of this kind
     const float* conv = static_cast<const float*>(kind == kQueries ? a.q_conv : kind == kKeys ? a.k_conv : a.v_conv);
     const uint32_t pos = a.row_pos[row], slot = a.row_slot[row], info = a.row_back[row];
     const uint32_t number = kind == kQueries ? 0u : a.page_table[(size_t)slot * a.max_pages + pos / M40LLM_PAGE_TOKENS];
@@ -175,15 +175,15 @@ __device__ __forceinline__ void split_unit(const M40llmPairSplit& a, const M40Pa
             for (int k = 0; k < W; ++k) y[i][k] *= inv * w.v[k];
         }
     }
-    T* cache = static_cast<T*>(a.cache) + number * page.elements() + (kind == kKeys ? unit / 2u : unit) * page.head_elements();
+    T* cache = static_cast<T*>(a.cache) + number * page.elements() + (kind == kKeys ? unit / a.maps : unit) * page.head_elements();
     const uint32_t t = pos % M40LLM_PAGE_TOKENS, pad = kind == kValues ? page.v_tiles * 16u : page.k_tiles * 32u;
-    T* q = static_cast<T*>(a.queries) + ((size_t)row * 2u * a.heads + unit) * pad;
+    T* q = static_cast<T*>(a.queries) + ((size_t)row * a.maps * a.heads + unit) * pad;
 #pragma unroll
     for (int i = 0; i < N; ++i) {
         const uint32_t at = W * (lane + 16u * i);            // pads too: zeros
         if (at >= pad) continue;
         if (kind == kQueries) m40_store_columns<T, W>(q + at, y[i]);
-        else if (kind == kKeys) m40_store_columns<T, W>(cache + page.key_at(unit % 2u, t, at), y[i]);
+        else if (kind == kKeys) m40_store_columns<T, W>(cache + page.key_at(unit % a.maps, t, at), y[i]);
         else {
 #pragma unroll
             for (int k = 0; k < W; ++k) cache[page.value_at(t, at + k)] = M40Act<T>::from(y[i][k]);
@@ -194,9 +194,10 @@ template <class T, int W, int NQ, int NV>
 __global__ __launch_bounds__(kThreads) void pair_split_append_kernel(M40llmPairSplit a, M40PairPage page) {
     const uint32_t row = blockIdx.x * 16u + (threadIdx.x >> 4), lane = threadIdx.x & 15u, unit = blockIdx.y;
     if (row >= a.rows) return;           // no barrier below; the 16 lanes of a row stay together
-    if (unit < 2u * a.heads) split_unit<T, W, NQ>(a, page, kQueries, unit, row, lane);
-    else if (unit < 2u * (a.heads + a.kv_heads)) split_unit<T, W, NQ>(a, page, kKeys, unit - 2u * a.heads, row, lane);
-    else split_unit<T, W, NV>(a, page, kValues, unit - 2u * (a.heads + a.kv_heads), row, lane);
+    const uint32_t queries = a.maps * a.heads, keys = a.maps * a.kv_heads;
+    if (unit < queries) split_unit<T, W, NQ>(a, page, kQueries, unit, row, lane);
+    else if (unit < queries + keys) split_unit<T, W, NQ>(a, page, kKeys, unit - queries, row, lane);
+    else split_unit<T, W, NV>(a, page, kValues, unit - queries - keys, row, lane);
 }
 
 // A thread a column: the last rows of a portion take their places in the ring.
@@ -213,7 +214,7 @@ __global__ __launch_bounds__(kThreads) void conv_state_kernel(const float* __res
 
 template <class T>
 void launch_split(hipStream_t stream, const M40llmPairSplit& s, const M40PairPage& page) {
-    const dim3 grid((s.rows + 15u) / 16u, 2u * s.heads + (s.cache ? 3u * s.kv_heads : 0u));
+    const dim3 grid((s.rows + 15u) / 16u, s.maps * s.heads + (s.cache ? (s.maps + 1u) * s.kv_heads : 0u));
     const bool vec = s.dim % 4u == 0 && s.vdim % 4u == 0 && s.ld_proj % 4u == 0 && s.ld_state % 4u == 0 && s.k_offset % 4u == 0 && s.v_offset % 4u == 0 &&
                      m40_aligned16(s.proj) && m40_aligned16(s.conv_state) && m40_aligned16(s.q_conv) && m40_aligned16(s.k_conv) && m40_aligned16(s.v_conv) &&
                      m40_aligned16(s.q_norm) && m40_aligned16(s.k_norm);
@@ -274,16 +275,16 @@ int m40llm_ext_pair_split_append_async(M40llmCudaContext* ctx, const M40llmPairS
     if (!ctx || !s || !s->proj || !s->q_norm || !s->queries || !s->row_slot || !s->row_pos || !s->row_back) return -1;
     hipStream_t stream = m40_select_stream(ctx, stream_kind);
     if (!stream || m40_ensure_device(ctx) != 0) return -2;
-    if (s->rows == 0 || s->act_dtype > 1u || s->heads == 0 || s->kv_heads == 0 || s->heads % s->kv_heads != 0 || s->dim == 0 || s->dim > M40LLM_PAIR_MOST_DIM ||
-        s->vdim == 0 || s->vdim > M40LLM_PAIR_MOST_DIM)
+    if (s->rows == 0 || s->act_dtype > 1u || s->maps == 0 || s->maps > 2u || s->heads == 0 || s->kv_heads == 0 || s->heads % s->kv_heads != 0 || s->dim == 0 ||
+        s->dim > M40LLM_PAIR_MOST_DIM || s->vdim == 0 || s->vdim > M40LLM_PAIR_MOST_DIM || s->maps * (s->heads + (uint64_t)s->kv_heads) + s->kv_heads > 65535u)
         return -3;
-    const uint64_t cols = s->cache ? (uint64_t)s->v_offset + (uint64_t)s->kv_heads * s->vdim : 2ull * s->heads * s->dim;
+    const uint64_t cols = s->cache ? (uint64_t)s->v_offset + (uint64_t)s->kv_heads * s->vdim : (uint64_t)s->maps * s->heads * s->dim;
     if (s->ld_proj < cols) return -3;
     if (s->taps && (!s->q_conv || (s->taps > 1u && (!s->conv_state || s->ld_state < cols)))) return -4;
-    if (s->cache && (!s->k_norm || !s->page_table || s->k_offset < 2u * s->heads * s->dim || s->v_offset < s->k_offset + 2u * s->kv_heads * s->dim ||
+    if (s->cache && (!s->k_norm || !s->page_table || s->k_offset < s->maps * s->heads * s->dim || s->v_offset < s->k_offset + s->maps * s->kv_heads * s->dim ||
                      (s->taps && (!s->k_conv || !s->v_conv))))
         return -4;
-    const M40PairPage page(2u, s->kv_heads, s->dim, s->vdim);
+    const M40PairPage page(s->maps, s->kv_heads, s->dim, s->vdim);
     if (s->act_dtype == M40LLM_ACT_F32) launch_split<float>(stream, *s, page);
     else launch_split<m40_bf16>(stream, *s, page);
     return launched();

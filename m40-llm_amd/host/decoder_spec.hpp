@@ -71,11 +71,15 @@ struct LightningSpec {
 };
 
 // Softmax attention.  Optional: biases on the projections, RMS norm over all query and over all key columns, rotation, a sigmoid gate per
-// column; values mixed with those of the first layer that shares its own (share_values).
+// column; values mixed with those of the first layer that shares its own (share_values); RMS norm of every query and key head without a weight;
+// scores held within +-cap by a tanh; less a slope times the distance of key and query, 2^(-8 (h + 1) / heads) for head h; a window of the newest
+// tokens; a sink per head in the denominator.
 struct AttentionSpec {
     uint32_t heads = 0, kv_heads = 0, dim = 0, vdim = 0;
     float scale = 0.0f;
-    bool biases = false, projection_norm = false, column_gate = false, share_values = false;
+    bool biases = false, projection_norm = false, column_gate = false, share_values = false, head_norm = false, distance_slopes = false, sink = false;
+    float cap = 0.0f;              // 0 = none
+    uint32_t window = 0;           // 0 = all
     std::optional<RotationSpec> rotation;
 };
 
@@ -98,9 +102,22 @@ struct ChannelDeltaSpec {
     uint32_t heads = 0, kv_heads = 0, dim = 0, vdim = 0, taps = 0;
 };
 
-typedef std::variant<LatentAttentionSpec, DifferentialAttentionSpec, LightningSpec, AttentionSpec, ParallelSpec, ChannelDeltaSpec> MixerSpec;
+// Time mixing (RWKV): receptance, keys, values, gates and decays each from their own mix of a token with the one before; one decay per head and key
+// channel, from a low-rank product whose rank the tensors give; a bonus for the current token.
+struct TimeMixingSpec {
+    uint32_t heads = 0, dim = 0;
+};
 
-enum class Activation { GeluTanh, Silu };
+// State space layer (Mamba-2): values, keys and queries (heads of a group share the latter two) behind a short convolution; decay and input weight from a
+// step size per token and head; a direct part; a gate, then an RMS norm over each of norm_groups parts.
+struct StateSpaceSpec {
+    uint32_t heads = 0, groups = 0, state = 0, vdim = 0, taps = 0, norm_groups = 0;
+};
+
+typedef std::variant<LatentAttentionSpec, DifferentialAttentionSpec, LightningSpec, AttentionSpec, ParallelSpec, ChannelDeltaSpec, TimeMixingSpec, StateSpaceSpec> MixerSpec;
+
+enum class Activation { GeluTanh, Silu, LimitedGate };
+enum class RouterScore { Softmax, Sigmoid };
 enum class NormKind { Layer, Rms };
 
 struct GatedMlpSpec {          // down(activation(gate h) * (up h))
@@ -108,17 +125,23 @@ struct GatedMlpSpec {          // down(activation(gate h) * (up h))
     Activation activation = Activation::GeluTanh;
 };
 
-// Of `experts` gated feed-forwards and `identity` experts that return their input, each token takes `top` by softmax score (+ correction)
-// and adds up their outputs times scale times their scores.  groups > 1: experts form groups of neighbours, and only those of the `keep` groups with
+struct PolyMlpSpec {           // down(p(up h)), p a polynomial whose powers are each divided by their root mean square
+    uint32_t ff = 0;
+};
+
+// Of `experts` gated feed-forwards and `identity` experts that return their input, each token takes `top` by score (+ correction)
+// and adds up their outputs times scale times their scores, or (weight_input) their outputs for its input times scale times their scores.  groups > 1: experts form groups of neighbours, and only those of the `keep` groups with
 // the best expert can be taken.
 struct ExpertMlpSpec {
     uint32_t experts = 0, identity = 0, top = 0, ff = 0, groups = 1, keep = 1;
     float scale = 1.0f;
-    bool correction = true;
+    bool correction = true, weight_input = false;
+    RouterScore score = RouterScore::Softmax;
     Activation activation = Activation::Silu;
+    float limit = 0.0f, alpha = 1.0f;        // LimitedGate
 };
 
-typedef std::variant<std::monostate, GatedMlpSpec, ExpertMlpSpec> MlpSpec;
+typedef std::variant<std::monostate, GatedMlpSpec, ExpertMlpSpec, PolyMlpSpec> MlpSpec;
 
 struct BigramSpec {            // a second embedding looked up by (token before, token)
     uint32_t buckets = 0, mul_prev = 0, mul_cur = 0;
@@ -127,11 +150,13 @@ struct BigramSpec {            // a second embedding looked up by (token before,
 struct LayerSpec {
     MixerSpec mixer;
     MlpSpec mlp;
+    int tensors_of = -1;               // the layer whose tensors it uses (-1 = its own)
 };
 
 enum class BlockKind {
     Parallel,       // one norm whose output both sublayers read: x += mixer(norm(x)) + mlp(norm(x))
     OutputNorm,     // x += m * norm1(mixer(x)), then x += m * norm2(mlp(x))
+    PreNorm,        // x += mixer(norm1(x)), then x += mlp(norm2(x))
     Streams,        // several streams: u = in . x, y = mixer(norm1(u)), x_t = sum_s mix[s][t] x_s + m * out[t] * y; the same with the mlp
 };
 
@@ -141,6 +166,8 @@ struct DecoderSpec {
     float eps = 0.0f;
     NormKind norm = NormKind::Layer;
     bool norm_around_zero = false;     // norm weights are stored less one
+    bool norm_scalar = false;          // norm weights are one number for all coordinates
+    float logit_scale = 1.0f, logit_cap = 0.0f;      // logits are scaled, then held within +-cap by a tanh (0 = not)
     bool tied_head = false;            // logits from the embedding table
     uint32_t streams = 1;              // BlockKind::Streams
     BlockKind block = BlockKind::Parallel;
@@ -377,9 +404,97 @@ inline DecoderSpec read_natatar(const json::Value& c) {
     return d;
 }
 
+// The layer whose tensors layer i uses, through any number of layers that use another's themselves.
+inline int read_tensors_of(const std::vector<json::Value>& layers, size_t i, const std::string& where) {
+    size_t at = i;
+    for (size_t n = 0;; ++n) {
+        const json::Value* j = layers[at].find("weights_of");
+        if (!j || j->is_null()) return at == i ? -1 : (int)at;
+        at = j->as_u32("weights_of");
+        if (at >= layers.size() || n >= layers.size()) throw json::Error(where + "weights_of must lead to a layer with tensors of its own");
+        for (const char* key : {"type", "mixer", "mlp"}) {
+            const json::Value *a = layers[i].find(key), *b = layers[at].find(key);
+            if ((a && !a->is_null()) != (b && !b->is_null()) || (a && b && *a != *b)) throw json::Error(where + "weights_of must name a layer of the same kind and sizes");
+        }
+    }
+}
+
+inline DecoderSpec read_fomunex(const json::Value& c) {
+    DecoderSpec d;
+    d.architecture = "Fomunex";
+    d.vocab = c.u32("vocab");
+    d.width = c.u32("width");
+    d.eps = (float)c.at("norm").num("eps");
+    d.norm = NormKind::Rms;
+    d.norm_scalar = true;
+    d.block = BlockKind::PreNorm;
+    d.positions = c.u32("max_positions");
+    d.logit_scale = (float)optional_num(c, "logit_scale", 1.0);
+    d.logit_cap = (float)optional_num(c, "logit_softcap", 0.0);
+    if (d.logit_cap < 0.0f) throw json::Error("logit_softcap must not be negative");
+    const auto& layers = c.array("layers");
+    for (size_t i = 0; i < layers.size(); ++i) {
+        const json::Value& l = layers[i];
+        const std::string where = "layer " + std::to_string(i) + ": ";
+        auto check = [&](bool ok, const char* what) { if (!ok) throw json::Error(where + what); };
+        const json::Value& m = l.at("mixer");
+        LayerSpec s;
+        s.tensors_of = read_tensors_of(layers, i, where);
+        if (l.str("type") == "attention") {
+            AttentionSpec a = read_attention_sizes(m, where);
+            a.head_norm = a.distance_slopes = a.sink = true;
+            a.cap = (float)optional_num(m, "softcap", 0.0);
+            check(a.cap >= 0.0f, "softcap must not be negative");
+            if (const json::Value* w = m.find("mask"); w && !w->is_null()) {
+                a.window = w->u32("size");
+                check(a.window > 0 && a.window <= 0x7fffffffu, "mask.size must be positive");
+            }
+            s.mixer = a;
+        } else if (l.str("type") == "wkv") {
+            const TimeMixingSpec a{m.u32("heads"), m.u32("dim")};
+            check(a.heads && a.dim, "a size is zero");
+            s.mixer = a;
+        } else if (l.str("type") == "mamba2") {
+            const StateSpaceSpec a{m.u32("heads"), m.u32("groups"), m.u32("state"), m.u32("vdim"), m.u32("conv"), m.u32("norm_groups")};
+            check(a.heads && a.groups && a.state && a.vdim && a.taps && a.norm_groups, "a size is zero");
+            check(a.heads % a.groups == 0, "heads must be a multiple of groups");
+            check((uint64_t)a.heads * a.vdim % a.norm_groups == 0, "heads * vdim must be a multiple of norm_groups");
+            s.mixer = a;
+        } else {
+            throw json::Error(where + "unknown mixer '" + l.str("type") + "'");
+        }
+        if (const json::Value* f = l.find("mlp"); f && !f->is_null()) {
+            if (f->str("kind") == "dense") {
+                s.mlp = PolyMlpSpec{f->u32("ff")};
+                check(f->u32("ff") != 0, "a size is zero");
+            } else if (f->str("kind") == "moe") {
+                ExpertMlpSpec e;
+                const json::Value &r = f->at("router"), &x = f->at("expert");
+                e.correction = false;
+                e.weight_input = true;
+                e.score = RouterScore::Sigmoid;
+                e.experts = r.u32("experts"); e.top = r.u32("top");
+                e.ff = x.u32("ff");
+                e.activation = Activation::LimitedGate;
+                e.limit = (float)x.num("limit");
+                e.alpha = 1.702f;
+                check(e.experts && e.top && e.ff, "a size is zero");
+                check(e.top <= e.experts, "router.top is larger than the number of experts");
+                check(e.limit >= 0.0f, "expert.limit must not be negative");
+                s.mlp = e;
+            } else {
+                throw json::Error(where + "unknown feed-forward '" + f->str("kind") + "'");
+            }
+        }
+        d.layers.push_back(s);
+    }
+    if (d.vocab == 0 || d.width == 0 || d.positions == 0 || d.layers.empty()) throw json::Error("vocab, width, max_positions and layers must not be empty");
+    return d;
+}
+
 // designs by the name config.json gives in "architecture"
 inline const std::map<std::string, std::function<DecoderSpec(const json::Value&)>>& decoder_registry() {
-    static const std::map<std::string, std::function<DecoderSpec(const json::Value&)>> r = {{"Pimosun", read_pimosun}, {"Gulidra", read_gulidra}, {"Natatar", read_natatar}};
+    static const std::map<std::string, std::function<DecoderSpec(const json::Value&)>> r = {{"Pimosun", read_pimosun}, {"Gulidra", read_gulidra}, {"Natatar", read_natatar}, {"Fomunex", read_fomunex}};
     return r;
 }
 inline DecoderSpec read_decoder_spec(const std::string& config_text) {

@@ -56,6 +56,16 @@ public:
         if (v.kind != Kind::String) throw Error("'" + key + "' is not a string");
         return v.string;
     }
+    // the same value, members in any order
+    bool operator==(const Value& o) const {
+        if (kind != o.kind || boolean != o.boolean || number != o.number || string != o.string || items != o.items || members.size() != o.members.size()) return false;
+        for (const auto& m : members) {
+            const Value* v = o.find(m.first);
+            if (!v || !(m.second == *v)) return false;
+        }
+        return true;
+    }
+    bool operator!=(const Value& o) const { return !(*this == o); }
     const std::vector<Value>& array(const std::string& key) const {
         const Value& v = at(key);
         if (v.kind != Kind::Array) throw Error("'" + key + "' is not a list");

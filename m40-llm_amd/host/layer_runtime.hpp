@@ -130,6 +130,7 @@ public:
         return b;
     }
     DeviceBuf upload_norm(TensorSource& t, const std::string& name) {         // of the residual's width
+        if (spec.norm_scalar) return upload_f32(std::vector<float>(spec.width, t.read_f32(name, {})[0]));
         std::vector<float> w = t.read_f32(name, {spec.width});
         if (spec.norm_around_zero)
             for (float& x : w) x += 1.0f;

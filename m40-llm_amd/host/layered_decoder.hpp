@@ -1,13 +1,14 @@
 // Decoder that runs a DecoderSpec: bf16 weights in packed tiles, bf16 or f32 activations, an f32 residual stream, a paged cache and, per
 // sequence slot, what recurrent layers carry from token to token.  One step function takes any mixture of sequences and portions (whole
 // prompts, parts of prompts, single tokens); everything that serves or generates goes through it or through the same layer launches
-// replayed from a graph.  The layers themselves: latent_layer.hpp (parallel blocks), output_norm_layer.hpp, stream_layer.hpp.
+// replayed from a graph.  The layers themselves: latent_layer.hpp (parallel blocks), output_norm_layer.hpp, stream_layer.hpp, prenorm_layer.hpp.
 #pragma once
 
 #include <algorithm>
 #include <chrono>
 #include <cmath>
 #include <cstring>
+#include <map>
 #include <memory>
 #include <string>
 #include <vector>
@@ -15,6 +16,7 @@
 #include "latent_layer.hpp"
 #include "output_norm_layer.hpp"
 #include "stream_layer.hpp"
+#include "prenorm_layer.hpp"
 #include "served_model.hpp"
 
 namespace m40host {
@@ -219,6 +221,7 @@ private:
             case BlockKind::Parallel: load_parallel(t); break;
             case BlockKind::OutputNorm: load_output_norm(t); break;
             case BlockKind::Streams: load_streams(t); break;
+            case BlockKind::PreNorm: load_pre_norm(t); break;
         }
         final_norm_ = rt_.upload_norm(t, "final.norm");
         head_ = rt_.packed(round_up(spec_.vocab, 16) / 16, d_tiles);
@@ -263,7 +266,7 @@ private:
             } else {
                 throw std::invalid_argument("layer " + std::to_string(i) + ": this mixer has no form with a norm on its output");
             }
-            layers_.push_back(std::make_unique<OutputNormLayer>(rt_, t, i, std::move(mixer), feed_forward(t, expert, i, s.mlp)));
+            layers_.push_back(std::make_unique<OutputNormLayer>(rt_, t, i, std::move(mixer), feed_forward(t, expert, tensor_prefix(i), s.mlp)));
         }
     }
     void load_streams(TensorSource& t) {
@@ -290,12 +293,45 @@ private:
             }
             if (const auto* e = std::get_if<ExpertMlpSpec>(&s.mlp); e && e->identity)
                 throw std::invalid_argument("layer " + std::to_string(i) + ": experts that return their input have no form over residual streams");
-            layers_.push_back(std::make_unique<StreamLayer>(rt_, *streams_, t, i, std::move(mixer), feed_forward(t, expert, i, s.mlp)));
+            layers_.push_back(std::make_unique<StreamLayer>(rt_, *streams_, t, i, std::move(mixer), feed_forward(t, expert, tensor_prefix(i), s.mlp)));
         }
     }
-    std::unique_ptr<FeedForward> feed_forward(TensorSource& t, const std::shared_ptr<ExpertShared>& expert, uint32_t i, const MlpSpec& mlp) {
-        if (const auto* m = std::get_if<GatedMlpSpec>(&mlp)) return std::make_unique<DenseFeedForward>(rt_, t, i, *m);
-        if (const auto* m = std::get_if<ExpertMlpSpec>(&mlp)) return std::make_unique<ExpertFeedForward>(rt_, expert, t, i, *m);
+    // Layers over one stream; those that use another layer's tensors (in whichever order the two come) share them and have a cache or state of
+    // their own.
+    void load_pre_norm(TensorSource& t) {
+        auto shared = std::make_shared<StreamShared>();
+        auto expert = std::make_shared<ExpertShared>();
+        rt_.scratch.insert(rt_.scratch.end(), {&shared->queries, &shared->recurrent, &shared->low, &shared->low_act, &shared->mixes, &shared->heads, &expert->logits, &expert->ids,
+                                               &expert->weight, &expert->rows_of, &expert->place, &expert->jobs, &expert->rows, &expert->act, &expert->out,
+                                               &expert->slot_weight});
+        shared_ = {shared, expert};
+        streams_ = std::make_unique<ResidualStreams>(rt_);
+        std::map<uint32_t, const StreamLayer*> made;        // by the layer whose tensors it has
+        for (const LayerSpec& s : spec_.layers) {
+            const uint32_t i = (uint32_t)layers_.size(), own = s.tensors_of >= 0 ? (uint32_t)s.tensors_of : i;
+            const StreamLayer* twin = made.count(own) ? made[own] : nullptr;
+            const Mixer* other = twin ? twin->mixer() : nullptr;
+            std::unique_ptr<Mixer> mixer;
+            if (const auto* a = std::get_if<AttentionSpec>(&s.mixer)) {
+                mixer = std::make_unique<AttentionMixer>(rt_, shared, t, own, *a, false, dynamic_cast<const AttentionMixer*>(other));
+            } else if (const auto* a = std::get_if<TimeMixingSpec>(&s.mixer)) {
+                mixer = std::make_unique<TimeMixingMixer>(rt_, shared, t, own, *a, dynamic_cast<const TimeMixingMixer*>(other));
+            } else if (const auto* a = std::get_if<StateSpaceSpec>(&s.mixer)) {
+                mixer = std::make_unique<StateSpaceMixer>(rt_, shared, t, own, *a, dynamic_cast<const StateSpaceMixer*>(other));
+            } else {
+                throw std::invalid_argument("layer " + std::to_string(i) + ": this mixer has no pre-norm form");
+            }
+            auto layer = twin ? std::make_unique<StreamLayer>(*twin, std::move(mixer))
+                              : std::make_unique<StreamLayer>(rt_, *streams_, t, own, std::move(mixer), feed_forward(t, expert, tensor_prefix(own), s.mlp));
+            if (!twin) made[own] = layer.get();
+            layers_.push_back(std::move(layer));
+        }
+    }
+    static std::string tensor_prefix(uint32_t layer) { return "l" + std::to_string(layer) + "."; }
+    std::unique_ptr<FeedForward> feed_forward(TensorSource& t, const std::shared_ptr<ExpertShared>& expert, const std::string& layer, const MlpSpec& mlp) {
+        if (const auto* m = std::get_if<GatedMlpSpec>(&mlp)) return std::make_unique<DenseFeedForward>(rt_, t, layer, *m);
+        if (const auto* m = std::get_if<PolyMlpSpec>(&mlp)) return std::make_unique<PolyFeedForward>(rt_, t, layer, *m);
+        if (const auto* m = std::get_if<ExpertMlpSpec>(&mlp)) return std::make_unique<ExpertFeedForward>(rt_, expert, t, layer, *m);
         return nullptr;
     }
 
@@ -376,6 +412,10 @@ private:
                                             (uint64_t)rows * spec_.width, final_norm_.ptr(), row_index, n, spec_.width, spec_.eps, hn_.ptr(), rt_.d_pad,
                                             opt_.act_dtype, kStream));
         M40llmPackedGemm g = rt_.product(hn_.ptr(), rt_.d_pad, head_, round_up(spec_.vocab, 16) / 16, rt_.d_pad / 32, n, M40LLM_PACKED_STORE);
+        if (spec_.logit_scale != 1.0f || spec_.logit_cap > 0.0f) {
+            g.epilogue = M40LLM_PACKED_CAP;
+            g.out_scale = spec_.logit_scale; g.out_cap = spec_.logit_cap;
+        }
         g.out_f32 = logits_.ptr(); g.ld_out = spec_.vocab; g.cols = spec_.vocab;
         rt_.launch(g);
     }
@@ -581,7 +621,7 @@ private:
     float tie_guard_ = DecodeModel::kGreedyTieGuard;
     bool timed_fallback_ = false;
     std::vector<std::shared_ptr<void>> shared_;       // buffers the layers share
-    std::unique_ptr<ResidualStreams> streams_;        // BlockKind::Streams
+    std::unique_ptr<ResidualStreams> streams_;        // BlockKind::Streams, PreNorm
     std::vector<std::unique_ptr<DecoderLayer>> layers_;
     size_t state_bytes_ = 0;                          // of a slot, all layers
     DeviceBuf embed_, bigram_, positions_, final_norm_, head_, hn_, logits_, pick_parts_, tables_;

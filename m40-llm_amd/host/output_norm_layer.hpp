@@ -13,13 +13,15 @@ public:
     virtual uint32_t enqueue(const Rows& r) = 0;         // returns the number of planes
     virtual void prepare(const Rows&) {}
     virtual bool portion_cost(uint32_t, uint32_t, double&, double&) const { return true; }
+    virtual bool reads_plain_rows() const { return false; }      // it wants its input as plain rows (h_rows) as well
 };
 
-// Tiles of queries (row, head of a kv head's group): 16 a tile for single tokens and short portions, 64 or 128 for long ones.
+// Tiles of queries (row, head of a kv head's group): 16 a tile for single tokens and short portions, 64 or 128 for long ones.  window: of the
+// newest tokens, which is all that queries see (0 = everything).
 struct PairTiles : PassTable {
-    PairTiles(uint32_t g, uint32_t most) : group(g), most_queries(most) {}
-    bool same(uint32_t g, uint32_t most) const { return group == g && most_queries == most; }
-    uint32_t group, most_queries, fewest_kv_heads = 0xffffffffu, n_short = 0, n_long = 0, long_queries = 64, splits = 1;
+    PairTiles(uint32_t g, uint32_t most, uint32_t w) : group(g), most_queries(most), window(w ? w : 0x7fffffffu) {}
+    bool same(uint32_t g, uint32_t most, uint32_t w) const { return group == g && most_queries == most && window == (w ? w : 0x7fffffffu); }
+    uint32_t group, most_queries, window, fewest_kv_heads = 0xffffffffu, n_short = 0, n_long = 0, long_queries = 64, splits = 1;
     uint64_t floats_a_row = 0;            // of a split's partial sums, the largest layer's
     const uint32_t* long_tiles() const { return at + 2 * n_short; }
     std::vector<uint32_t> build(const PassPlan& plan, const SequencePages&, uint32_t longest) override {
@@ -38,14 +40,16 @@ struct PairTiles : PassTable {
             const uint32_t n = p.n * group;
             for (uint32_t i = 0; p.is_long && i < n; i += long_queries) {
                 const uint32_t m = std::min(long_queries, n - i);
-                tiles.push_back({p.row * group + i, m, p.length - p.n + (i + m + group - 1) / group});
+                const uint32_t first = p.length - p.n + i / group + 1, last = p.length - p.n + (i + m + group - 1) / group;
+                tiles.push_back({p.row * group + i, m, last - (first > window ? first - window : 0)});
             }
         }
         std::stable_sort(tiles.begin(), tiles.end(), [](const Tile& a, const Tile& b) { return a.keys > b.keys; });     // the longest walks first
         for (const Tile& x : tiles) t.insert(t.end(), {x.first, x.n});
         n_long = (uint32_t)tiles.size();
         // the pages of a tile over as many workgroups as fill the CUs twice, a page a wave at least
-        const uint32_t pages = (longest + LayerRuntime::kPage - 1) / LayerRuntime::kPage, groups = std::max(1u, n_short * fewest_kv_heads);
+        const uint32_t seen = longest > window ? window + LayerRuntime::kPage : longest;
+        const uint32_t pages = (seen + LayerRuntime::kPage - 1) / LayerRuntime::kPage, groups = std::max(1u, n_short * fewest_kv_heads);
         splits = std::max(1u, std::min({(pages + 3) / 4, 2 * LayerRuntime::kCus / groups, 256u}));
         return t;
     }
@@ -102,7 +106,7 @@ public:
             conv_state_ = rt.cleared(slot * rt.opt.max_sequences);
             rt.states.push_back({&conv_state_, slot});
         }
-        tiles_ = &rt.table<PairTiles>(a.heads / a.kv_heads, most_queries_);
+        tiles_ = &rt.table<PairTiles>(a.heads / a.kv_heads, most_queries_, 0u);
         tiles_->fewest_kv_heads = std::min(tiles_->fewest_kv_heads, a.kv_heads);
         tiles_->floats_a_row = std::max(tiles_->floats_a_row, m40llm_ext_pair_attention_partial_floats(2, 1, a.heads, a.vdim, 2) / 2);
         rt.proj.want(rt.f32_bytes((size_t)tiles_in_ * 16));
@@ -127,7 +131,7 @@ public:
         DeviceBuf& cache = source_ ? source_->cache_ : cache_;
         {
             M40llmPairSplit s{};
-            s.act_dtype = rt_.opt.act_dtype; s.rows = r.rows; s.heads = a_.heads; s.kv_heads = a_.kv_heads; s.dim = a_.dim; s.vdim = a_.vdim; s.taps = a_.taps;
+            s.act_dtype = rt_.opt.act_dtype; s.rows = r.rows; s.maps = 2; s.heads = a_.heads; s.kv_heads = a_.kv_heads; s.dim = a_.dim; s.vdim = a_.vdim; s.taps = a_.taps;
             s.eps = rt_.spec.eps;
             s.proj = rt_.proj.ptr(); s.ld_proj = ld; s.k_offset = k_offset_; s.v_offset = v_offset_;
             s.q_conv = q_conv_.ptr(); s.k_conv = k_conv_.ptr(); s.v_conv = v_conv_.ptr();
@@ -293,12 +297,12 @@ public:
     virtual bool reads_plain_rows() const { return false; }      // it wants its input as plain rows (h_rows) as well
 };
 
-inline uint32_t activation_code(Activation a) { return a == Activation::Silu ? M40LLM_SILU : M40LLM_GELU_TANH; }
+inline uint32_t activation_code(Activation a) { return a == Activation::LimitedGate ? M40LLM_LIMITED_GATE : a == Activation::Silu ? M40LLM_SILU : M40LLM_GELU_TANH; }
 
 class DenseFeedForward : public FeedForward {
 public:
-    DenseFeedForward(LayerRuntime& rt, TensorSource& t, uint32_t index, const GatedMlpSpec& m) : rt_(rt), m_(m) {
-        const std::string p = "l" + std::to_string(index) + ".mlp.";
+    DenseFeedForward(LayerRuntime& rt, TensorSource& t, const std::string& layer, const GatedMlpSpec& m) : rt_(rt), m_(m) {
+        const std::string p = layer + "mlp.";
         const uint32_t D = rt.spec.width, d_tiles = rt.d_pad / 32;
         tiles_ = round_up(m.ff, 16) / 16;
         pad_ = round_up(m.ff, 32);
@@ -329,15 +333,48 @@ private:
     DeviceBuf w_in_, w_out_;
 };
 
-struct ExpertShared { Scratch logits, ids, weight, rows_of, place, jobs, rows, act, out; };
+// Launches: product | polynomial | product
+class PolyFeedForward : public FeedForward {
+public:
+    PolyFeedForward(LayerRuntime& rt, TensorSource& t, const std::string& layer, const PolyMlpSpec& m) : rt_(rt), m_(m), pad_(round_up(m.ff, 32)) {
+        const std::string p = layer + "mlp.";
+        const uint32_t D = rt.spec.width, d_tiles = rt.d_pad / 32;
+        w_in_ = rt.packed(pad_ / 16, d_tiles);             // columns past ff are zeros, which the norms' sums need
+        rt.pack(t, p + "up", m.ff, D, w_in_.ptr(), d_tiles, 0);
+        act_ = rt.upload_f32(t.read_f32(p + "act", {4}));
+        w_out_ = rt.packed(round_up(D, 16) / 16, pad_ / 32);
+        rt.pack(t, p + "down", D, m.ff, w_out_.ptr(), pad_ / 32, 0);
+        rt.cat.want(rt.act_bytes(pad_));
+        rt.want_planes(pad_ / 32, true);
+    }
+    SublayerOut enqueue(const Rows& r) override {
+        SublayerOut n;
+        M40llmPackedGemm g = rt_.product(rt_.h.ptr(), rt_.d_pad, w_in_, pad_ / 16, rt_.d_pad / 32, r.rows, M40LLM_PACKED_SPLIT);
+        g.out_act = rt_.cat.ptr(); g.ld_act = pad_;
+        rt_.launch(g);
+        M40H_TRY(m40llm_ext_poly_norm_rows_async(rt_.ctx, rt_.cat.ptr(), pad_, act_.ptr(), r.rows, m_.ff, rt_.spec.eps, rt_.opt.act_dtype, rt_.kStream));
+        n.planes = rt_.planes.ptr();
+        n.n_planes = rt_.into_planes(rt_.product(rt_.cat.ptr(), pad_, w_out_, round_up(rt_.spec.width, 16) / 16, pad_ / 32, r.rows, M40LLM_PACKED_STORE), r.rows);
+        n.plane_stride = (uint64_t)r.rows * rt_.spec.width;
+        return n;
+    }
+
+private:
+    LayerRuntime& rt_;
+    PolyMlpSpec m_;
+    uint32_t pad_;
+    DeviceBuf w_in_, act_, w_out_;
+};
+
+struct ExpertShared { Scratch logits, ids, weight, rows_of, place, jobs, rows, act, out, slot_weight; };
 
 // Launches: product (router logits) | choice and sorted list (two launches above 64 rows) | (many rows: rows in list order) | gate and up per
 // expert | down per expert
 class ExpertFeedForward : public FeedForward {
 public:
-    ExpertFeedForward(LayerRuntime& rt, std::shared_ptr<ExpertShared> shared, TensorSource& t, uint32_t index, const ExpertMlpSpec& m)
+    ExpertFeedForward(LayerRuntime& rt, std::shared_ptr<ExpertShared> shared, TensorSource& t, const std::string& layer, const ExpertMlpSpec& m)
         : rt_(rt), sh_(std::move(shared)), m_(m) {
-        const std::string p = "l" + std::to_string(index) + ".mlp.", where = "layer " + std::to_string(index) + ": ";
+        const std::string p = layer + "mlp.", where = "layer " + layer.substr(1, layer.size() - 2) + ": ";
         const uint32_t D = rt.spec.width, d_tiles = rt.d_pad / 32, all = m.experts + m.identity;
         if (all > M40LLM_MAX_EXPERTS) throw std::invalid_argument(where + "more experts than the routing kernels serve");
         tiles_ = round_up(m.ff, 16) / 16;
@@ -368,6 +405,7 @@ public:
         if (rt.bf16() && rows_a_job(R) == 128) sh_->rows.want((size_t)slots * rt.d_pad * rt.es);
         sh_->act.want((size_t)slots * pad_ * rt.es);
         sh_->out.want((size_t)slots * out_cols_ * rt.es);
+        if (m.weight_input) sh_->slot_weight.want((size_t)slots * 4);
     }
     bool reads_plain_rows() const override { return true; }
     SublayerOut enqueue(const Rows& r) override {
@@ -384,12 +422,16 @@ public:
             q.logits = sh_->logits.ptr(); q.ld_logits = router_tiles_ * 16; q.correction = correction_.ptr();
             q.ids = sh_->ids.u32(); q.weight = sh_->weight.ptr();
             q.rows_of = sh_->rows_of.u32(); q.place = sh_->place.u32(); q.jobs = sh_->jobs.u32();
+            q.score = m_.score == RouterScore::Sigmoid ? M40LLM_SCORE_SIGMOID : M40LLM_SCORE_SOFTMAX;
+            if (m_.weight_input) q.slot_weight = sh_->slot_weight.ptr();
             M40H_TRY(m40llm_ext_route_rows_async(rt_.ctx, &q, rt_.kStream));
         }
         const uint32_t d_tiles = rt_.d_pad / 32, down_tiles = round_up(rt_.spec.width, 16) / 16;
         {
             M40llmPackedGemm g = rt_.product(rt_.h_rows.ptr(), rt_.d_pad, w_in_, 2 * tiles_, d_tiles, r.rows, M40LLM_PACKED_PROJECT);
             g.activation = activation_code(m_.activation);
+            g.act_limit = m_.limit; g.act_alpha = m_.alpha;
+            if (m_.weight_input) g.row_scale = sh_->slot_weight.ptr();      // gate and up are linear in the input
             if (job_rows == 128) {
                 M40H_TRY(m40llm_ext_gather_rows_async(rt_.ctx, rt_.h_rows.ptr(), rt_.d_pad, sh_->rows_of.u32(), sh_->jobs.u32(),
                                                       m40llm_ext_expert_slots(r.rows, m_.experts, m_.top), sh_->rows.ptr(), rt_.kStream));
@@ -410,7 +452,8 @@ public:
             rt_.launch(g);
         }
         n.expert_out = sh_->out.ptr(); n.ld_expert = out_cols_;
-        n.place = sh_->place.u32(); n.weight = sh_->weight.ptr(); n.top = m_.top;
+        n.place = sh_->place.u32(); n.top = m_.top;
+        n.weight = m_.weight_input ? nullptr : sh_->weight.ptr();
         return n;
     }
 

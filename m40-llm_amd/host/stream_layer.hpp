@@ -1,5 +1,6 @@
 // Layers over residual streams: every sublayer reads a weighted sum of the streams behind a norm, and every stream takes a mixture of all old
-// ones and its share of the output.  Its mixers: softmax attention, attention beside a matrix memory, a delta rule.
+// ones and its share of the output; a pre-norm layer is one over a single stream that takes all of it.  Mixers: softmax attention, attention beside a
+// matrix memory, a delta rule, time mixing, a state space layer.
 #pragma once
 
 #include "output_norm_layer.hpp"
@@ -18,6 +19,11 @@ public:
         const uint32_t s = rt_.spec.streams;
         const std::string p = layer + "hc" + q + ".";
         StreamWeights w;
+        if (rt_.spec.block == BlockKind::PreNorm) {
+            w.mix = rt_.upload_f32({1.0f}); w.share = rt_.upload_f32({1.0f}); w.take = rt_.upload_f32({1.0f});
+            w.norm = rt_.upload_norm(t, layer + "norm" + q);
+            return w;
+        }
         w.mix = rt_.upload_f32(t.read_f32(p + "mix", {s, s}));
         w.share = rt_.upload_f32(t.read_f32(p + "out", {s}));
         w.take = rt_.upload_f32(t.read_f32(p + "in", {s}));
@@ -75,7 +81,7 @@ private:
 };
 
 struct StreamShared {         // buffers the layers of a decoder share
-    Scratch queries, first_values, recurrent, low, low_act;
+    Scratch queries, first_values, recurrent, low, low_act, mixes, heads;
     DeviceBuf chunks;
 };
 
@@ -86,29 +92,20 @@ public:
     // row tiles of the input product that are its own
     static uint32_t input_tiles(const AttentionSpec& a) { return gate_offset(a) / 16 + (a.column_gate ? round_up(a.heads * a.vdim, 16) / 16 : 0); }
 
+    // twin: a part with the same tensors
     AttentionPart(LayerRuntime& rt, StreamShared& sh, TensorSource& t, const std::string& where, const std::string& p, const AttentionSpec& a, float out_factor,
-                  bool takes_first_values)
-        : rt_(rt), sh_(sh), a_(a), out_factor_(out_factor), takes_first_(takes_first_values) {
+                  bool takes_first_values, const AttentionPart* twin = nullptr)
+        : rt_(rt), sh_(sh), a_(a), out_factor_(out_factor), takes_first_(takes_first_values), w_(twin ? twin->w_ : load(rt, t, p, a)) {
         most_queries_ = m40llm_ext_pair_attention_tile_queries(rt.opt.act_dtype, 1, a.dim, a.vdim);
         if (most_queries_ == 0) throw std::invalid_argument(where + "head sizes beyond what the attention kernels serve");
-        const uint32_t q = a.heads * a.dim, k = a.kv_heads * a.dim, v = a.kv_heads * a.vdim;
-        if (a.biases) {
-            q_bias_ = rt.upload_f32(t.read_f32(p + "q.b", {q}));
-            k_bias_ = rt.upload_f32(t.read_f32(p + "k.b", {k}));
-            v_bias_ = rt.upload_f32(t.read_f32(p + "v.b", {v}));
-        }
-        if (a.projection_norm) {
-            q_norm_ = rt.upload_f32(t.read_f32(p + "q.norm", {q}));
-            k_norm_ = rt.upload_f32(t.read_f32(p + "k.norm", {k}));
-        }
         if (a.rotation) rot_ = &rt.table<RotationAngles>(&rt, *a.rotation, std::max(a.rotation->dims / 2, 1u));
         if (takes_first_) lambda_ = t.read_f32(p + "vmix", {})[0];
         cache_ = rt.cleared((size_t)rt.max_pages * m40llm_ext_pair_page_elements(1, a.kv_heads, a.dim, a.vdim) * rt.es);
-        tiles_ = &rt.table<PairTiles>(a.heads / a.kv_heads, most_queries_);
+        tiles_ = &rt.table<PairTiles>(a.heads / a.kv_heads, most_queries_, a.window);
         tiles_->fewest_kv_heads = std::min(tiles_->fewest_kv_heads, a.kv_heads);
         tiles_->floats_a_row = std::max(tiles_->floats_a_row, m40llm_ext_pair_attention_partial_floats(1, 1, a.heads, a.vdim, 2) / 2);
         sh_.queries.want(rt.act_bytes((size_t)a.heads * round_up(a.dim, 32)));
-        if (a.share_values) sh_.first_values.want(rt.f32_bytes(v));
+        if (a.share_values) sh_.first_values.want(rt.f32_bytes(a.kv_heads * a.vdim));
     }
     void pack(TensorSource& t, const std::string& p, const DeviceBuf& w, uint32_t d_tiles) {
         const uint32_t D = rt_.spec.width;
@@ -119,19 +116,28 @@ public:
     }
     bool portion_cost(uint32_t n, uint32_t len, double& as_tokens, double& as_long) const {
         if (!rt_.bf16() || most_queries_ < 64) return false;
-        const double work = 2.0 * n * (len + n / 2.0) * a_.heads * (a_.dim + a_.vdim);
+        const double keys = len + n / 2.0, work = 2.0 * n * (a_.window ? std::min(keys, (double)a_.window) : keys) * a_.heads * (a_.dim + a_.vdim);
         as_tokens += 4.0 * work;              // pages come from memory once for 16 queries instead of 64 or 128
         as_long += work;
         return true;
     }
     void enqueue(const Rows& r, uint32_t ld, uint32_t ld_out) {
-        {
+        if (a_.head_norm) {
+            M40llmPairSplit s{};
+            s.act_dtype = rt_.opt.act_dtype; s.rows = r.rows; s.maps = 1; s.heads = a_.heads; s.kv_heads = a_.kv_heads; s.dim = a_.dim; s.vdim = a_.vdim;
+            s.eps = rt_.spec.eps;
+            s.proj = rt_.proj.ptr(); s.ld_proj = ld; s.k_offset = k_offset(a_); s.v_offset = v_offset(a_);
+            s.q_norm = w_->q_norm.ptr(); s.k_norm = w_->k_norm.ptr();
+            s.queries = sh_.queries.ptr(); s.cache = cache_.ptr();
+            s.row_slot = r.slot; s.row_pos = r.pos; s.row_back = r.back; s.page_table = r.page_table; s.max_pages = rt_.max_pages;
+            M40H_TRY(m40llm_ext_pair_split_append_async(rt_.ctx, &s, rt_.kStream));
+        } else {
             M40llmQkvSplit s{};
             s.act_dtype = rt_.opt.act_dtype; s.rows = r.rows; s.heads = a_.heads; s.kv_heads = a_.kv_heads; s.dim = a_.dim; s.vdim = a_.vdim;
             s.eps = rt_.spec.eps; s.q_factor = a_.scale < 0.0f ? -1.0f : 1.0f;        // the kernels take the scale's sign from the queries
             s.proj = rt_.proj.ptr(); s.ld_proj = ld; s.k_offset = k_offset(a_); s.v_offset = v_offset(a_);
-            s.q_bias = q_bias_.ptr(); s.k_bias = k_bias_.ptr(); s.v_bias = v_bias_.ptr();
-            s.q_norm = q_norm_.ptr(); s.k_norm = k_norm_.ptr();
+            s.q_bias = w_->q_bias.ptr(); s.k_bias = w_->k_bias.ptr(); s.v_bias = w_->v_bias.ptr();
+            s.q_norm = w_->q_norm.ptr(); s.k_norm = w_->k_norm.ptr();
             if (rot_) { s.angles = rot_->angles.ptr(); s.rot_half = rot_->half; }
             if (a_.share_values) {
                 s.ld_values = a_.kv_heads * a_.vdim;
@@ -145,6 +151,7 @@ public:
         M40llmPairAttention h{};
         h.act_dtype = rt_.opt.act_dtype; h.maps = 1; h.heads = a_.heads; h.kv_heads = a_.kv_heads; h.dim = a_.dim; h.vdim = a_.vdim;
         h.scale = std::fabs(a_.scale); h.out_scale = out_factor_;
+        h.window = a_.window; h.cap = a_.cap; h.slopes = w_->slopes.ptr(); h.sink = w_->sink.ptr();
         h.queries = sh_.queries.ptr(); h.cache = cache_.ptr();
         if (a_.column_gate) { h.gate = rt_.proj.f32(gate_offset(a_)); h.ld_gate = ld; }
         h.row_slot = r.slot; h.row_pos = r.pos; h.page_table = r.page_table; h.max_pages = rt_.max_pages;
@@ -168,6 +175,31 @@ public:
     }
 
 private:
+    struct Weights { DeviceBuf q_bias, k_bias, v_bias, q_norm, k_norm, slopes, sink; };
+    static std::shared_ptr<const Weights> load(LayerRuntime& rt, TensorSource& t, const std::string& p, const AttentionSpec& a) {
+        const uint32_t q = a.heads * a.dim, k = a.kv_heads * a.dim, v = a.kv_heads * a.vdim;
+        auto w = std::make_shared<Weights>();
+        if (a.biases) {
+            w->q_bias = rt.upload_f32(t.read_f32(p + "q.b", {q}));
+            w->k_bias = rt.upload_f32(t.read_f32(p + "k.b", {k}));
+            w->v_bias = rt.upload_f32(t.read_f32(p + "v.b", {v}));
+        }
+        if (a.projection_norm) {
+            w->q_norm = rt.upload_f32(t.read_f32(p + "q.norm", {q}));
+            w->k_norm = rt.upload_f32(t.read_f32(p + "k.norm", {k}));
+        }
+        if (a.head_norm) {               // no weights; the kernels take the scale's sign from the queries
+            w->q_norm = rt.upload_f32(std::vector<float>(a.dim, a.scale < 0.0f ? -1.0f : 1.0f));
+            w->k_norm = rt.upload_f32(std::vector<float>(a.dim, 1.0f));
+        }
+        if (a.distance_slopes) {
+            std::vector<float> s(a.heads);
+            for (uint32_t h = 0; h < a.heads; ++h) s[h] = (float)std::exp2(-8.0 * (h + 1) / a.heads);
+            w->slopes = rt.upload_f32(s);
+        }
+        if (a.sink) w->sink = rt.upload_f32(t.read_f32(p + "sink", {a.heads}));
+        return w;
+    }
     static uint32_t k_offset(const AttentionSpec& a) { return round_up(a.heads * a.dim, 16); }
     static uint32_t v_offset(const AttentionSpec& a) { return k_offset(a) + round_up(a.kv_heads * a.dim, 16); }
     static uint32_t gate_offset(const AttentionSpec& a) { return v_offset(a) + round_up(a.kv_heads * a.vdim, 16); }
@@ -176,19 +208,20 @@ private:
     AttentionSpec a_;
     float out_factor_, lambda_ = 0.0f;
     bool takes_first_;
+    std::shared_ptr<const Weights> w_;
     RotationAngles* rot_ = nullptr;
     PairTiles* tiles_;
     uint32_t most_queries_;
-    DeviceBuf q_bias_, k_bias_, v_bias_, q_norm_, k_norm_, cache_;
+    DeviceBuf cache_;
 };
 
-// What both recurrences do with a step's portions: single rows token after token, longer ones of bf16 passes chunk by chunk.
+// What recurrences do with a step's portions: single rows token after token, longer ones of bf16 passes chunk by chunk.
 class RecurrentRows {
 public:
     RecurrentRows(LayerRuntime& rt, StreamShared& sh) : rt_(rt), sh_(sh), portions_(rt.portions()) {}
-    void prepare(bool delta, uint32_t heads, uint32_t dim, uint32_t vdim) {
+    void prepare(uint32_t rule, uint32_t heads, uint32_t dim, uint32_t vdim) { prepare(m40llm_ext_memory_scratch_bytes(rule, portions_.n_chunks, heads, dim, vdim)); }
+    void prepare(uint64_t need) {
         if (!rt_.bf16() || portions_.n_chunks == 0) return;
-        const uint64_t need = m40llm_ext_memory_scratch_bytes(delta, portions_.n_chunks, heads, dim, vdim);
         if (need > sh_.chunks.bytes()) {
             M40H_TRY(m40llm_stream_synchronize(rt_.ctx, rt_.kStream));
             sh_.chunks = DeviceBuf(rt_.ctx, need);
@@ -209,6 +242,7 @@ public:
             M40H_TRY(launch(rt_.ctx, &p, rt_.kStream));
         }
     }
+    const PortionTable& portions() const { return portions_; }
     const uint32_t* multi() const { return portions_.multi(); }
 
 private:
@@ -220,14 +254,21 @@ private:
 // Launches: product (projections) | norms and cache append | attention | product
 class AttentionMixer : public Mixer {
 public:
-    AttentionMixer(LayerRuntime& rt, std::shared_ptr<StreamShared> shared, TensorSource& t, uint32_t index, const AttentionSpec& a, bool takes_first_values)
+    // twin: a mixer with the same tensors
+    AttentionMixer(LayerRuntime& rt, std::shared_ptr<StreamShared> shared, TensorSource& t, uint32_t index, const AttentionSpec& a, bool takes_first_values,
+                   const AttentionMixer* twin = nullptr)
         : rt_(rt), sh_(std::move(shared)), tiles_in_(AttentionPart::input_tiles(a)), o_pad_(round_up(a.heads * a.vdim, 32)) {
         const std::string where = "layer " + std::to_string(index) + ": ", p = "l" + std::to_string(index) + ".mix.";
-        attention_ = std::make_unique<AttentionPart>(rt, *sh_, t, where, p, a, 1.0f, takes_first_values);
-        w_in_ = rt.packed(tiles_in_, rt.d_pad / 32);
-        attention_->pack(t, p, w_in_, rt.d_pad / 32);
-        w_out_ = rt.packed(round_up(rt.spec.width, 16) / 16, o_pad_ / 32);
-        rt.pack(t, p + "o", rt.spec.width, a.heads * a.vdim, w_out_.ptr(), o_pad_ / 32, 0);
+        attention_ = std::make_unique<AttentionPart>(rt, *sh_, t, where, p, a, 1.0f, takes_first_values, twin ? twin->attention_.get() : nullptr);
+        if (twin) {
+            w_ = twin->w_;
+        } else {
+            w_ = std::make_shared<Weights>();
+            w_->in = rt.packed(tiles_in_, rt.d_pad / 32);
+            attention_->pack(t, p, w_->in, rt.d_pad / 32);
+            w_->out = rt.packed(round_up(rt.spec.width, 16) / 16, o_pad_ / 32);
+            rt.pack(t, p + "o", rt.spec.width, a.heads * a.vdim, w_->out.ptr(), o_pad_ / 32, 0);
+        }
         rt.proj.want(rt.f32_bytes((size_t)tiles_in_ * 16));
         rt.cat.want(rt.act_bytes(o_pad_));
         rt.want_planes(o_pad_ / 32, true);
@@ -235,19 +276,20 @@ public:
     bool portion_cost(uint32_t n, uint32_t len, double& as_tokens, double& as_long) const override { return attention_->portion_cost(n, len, as_tokens, as_long); }
     uint32_t enqueue(const Rows& r) override {
         const uint32_t ld = tiles_in_ * 16;
-        M40llmPackedGemm g = rt_.product(rt_.h.ptr(), rt_.d_pad, w_in_, tiles_in_, rt_.d_pad / 32, r.rows, M40LLM_PACKED_STORE);
+        M40llmPackedGemm g = rt_.product(rt_.h.ptr(), rt_.d_pad, w_->in, tiles_in_, rt_.d_pad / 32, r.rows, M40LLM_PACKED_STORE);
         g.out_f32 = rt_.proj.ptr(); g.ld_out = ld; g.cols = ld;
         rt_.launch(g);
         attention_->enqueue(r, ld, o_pad_);
-        return rt_.into_planes(rt_.product(rt_.cat.ptr(), o_pad_, w_out_, round_up(rt_.spec.width, 16) / 16, o_pad_ / 32, r.rows, M40LLM_PACKED_STORE), r.rows);
+        return rt_.into_planes(rt_.product(rt_.cat.ptr(), o_pad_, w_->out, round_up(rt_.spec.width, 16) / 16, o_pad_ / 32, r.rows, M40LLM_PACKED_STORE), r.rows);
     }
 
 private:
+    struct Weights { DeviceBuf in, out; };
     LayerRuntime& rt_;
     std::shared_ptr<StreamShared> sh_;
     uint32_t tiles_in_, o_pad_;
     std::unique_ptr<AttentionPart> attention_;
-    DeviceBuf w_in_, w_out_;
+    std::shared_ptr<Weights> w_;
 };
 
 // Launches: product (both sides' projections) | rotation and cache append | attention | matrix memory (norm and gate included) | product over both
@@ -284,7 +326,7 @@ public:
         rt.cat.want(rt.act_bytes(o_pad_));
         rt.want_planes(o_pad_ / 32, true);
     }
-    void prepare(const Rows&) override { rows_.prepare(false, m_.heads, m_.dim, m_.vdim); }
+    void prepare(const Rows&) override { rows_.prepare(M40LLM_RULE_MEMORY, m_.heads, m_.dim, m_.vdim); }
     bool portion_cost(uint32_t n, uint32_t len, double& as_tokens, double& as_long) const override { return attention_->portion_cost(n, len, as_tokens, as_long); }
     uint32_t enqueue(const Rows& r) override {
         const uint32_t ld = tiles_in_ * 16;
@@ -370,7 +412,7 @@ public:
         sh_->low.want(rt.f32_bytes((size_t)tiles_low_ * 16));
         rt.want_planes(o_pad_ / 32, true);
     }
-    void prepare(const Rows&) override { rows_.prepare(true, a_.heads, a_.dim, a_.vdim); }
+    void prepare(const Rows&) override { rows_.prepare(M40LLM_RULE_DELTA, a_.heads, a_.dim, a_.vdim); }
     uint32_t enqueue(const Rows& r) override {
         const uint32_t ld = plain_tiles_ * 16, ld_low = tiles_low_ * 16, ld_conv = round_up(conv_cols_, 4);
         {
@@ -424,32 +466,41 @@ private:
 class StreamLayer : public DecoderLayer {
 public:
     StreamLayer(LayerRuntime& rt, ResidualStreams& streams, TensorSource& t, uint32_t index, std::unique_ptr<Mixer> mixer, std::unique_ptr<FeedForward> ff)
-        : rt_(rt), streams_(streams), mixer_(std::move(mixer)), ff_(std::move(ff)) {
+        : rt_(rt), streams_(streams), mixer_(std::move(mixer)) {
         const std::string p = "l" + std::to_string(index) + ".";
-        mix_ = streams.load(t, p, "1");
-        if (ff_) feed_ = streams.load(t, p, "2");
+        auto w = std::make_shared<Weights>();
+        w->ff = std::move(ff);
+        w->mix = streams.load(t, p, "1");
+        if (w->ff) w->feed = streams.load(t, p, "2");
+        w_ = std::move(w);
     }
+    // with the tensors of another layer, whose mixer this one's shares them with
+    StreamLayer(const StreamLayer& twin, std::unique_ptr<Mixer> mixer) : rt_(twin.rt_), streams_(twin.streams_), mixer_(std::move(mixer)), w_(twin.w_) {}
+    const Mixer* mixer() const { return mixer_.get(); }
     void prepare(const Rows& r) override { mixer_->prepare(r); }
     bool portion_cost(uint32_t n, uint32_t len, double& as_tokens, double& as_long) const override { return mixer_->portion_cost(n, len, as_tokens, as_long); }
     void enqueue(const Rows& r) override {
-        streams_.read(r, mix_, false);
+        streams_.read(r, w_->mix, mixer_->reads_plain_rows());
         SublayerOut y;
         y.n_planes = mixer_->enqueue(r);
         y.planes = rt_.planes.ptr(); y.plane_stride = (uint64_t)r.rows * rt_.spec.width;
-        streams_.write(mix_, y);
-        if (ff_) {
-            streams_.read(r, feed_, ff_->reads_plain_rows());
-            streams_.write(feed_, ff_->enqueue(r));
+        streams_.write(w_->mix, y);
+        if (w_->ff) {
+            streams_.read(r, w_->feed, w_->ff->reads_plain_rows());
+            streams_.write(w_->feed, w_->ff->enqueue(r));
         }
         if (r.in_place) streams_.sum(r);
     }
 
 private:
     LayerRuntime& rt_;
+    struct Weights {
+        StreamWeights mix, feed;
+        std::unique_ptr<FeedForward> ff;
+    };
     ResidualStreams& streams_;
     std::unique_ptr<Mixer> mixer_;
-    std::unique_ptr<FeedForward> ff_;
-    StreamWeights mix_, feed_;
+    std::shared_ptr<const Weights> w_;
 };
 
 }  // namespace m40host

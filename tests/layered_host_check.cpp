@@ -30,7 +30,8 @@ static void rotation(const RotationSpec& r) {
 
 static void attention(const AttentionSpec& a) {
     std::cout << "\"sizes\": [" << a.heads << ", " << a.kv_heads << ", " << a.dim << ", " << a.vdim << "], \"scale\": " << a.scale << ", \"flags\": [" << a.biases << ", "
-              << a.projection_norm << ", " << a.column_gate << ", " << a.share_values << "]";
+              << a.projection_norm << ", " << a.column_gate << ", " << a.share_values << "], \"scores\": [" << a.head_norm << ", " << a.distance_slopes << ", " << a.sink << ", " << a.cap
+              << ", " << a.window << "]";
     if (a.rotation) rotation(*a.rotation);
 }
 
@@ -41,7 +42,8 @@ static void spec(std::istream& in) {
     std::cout.precision(17);
     std::cout << "{\"architecture\": " << quoted(d.architecture) << ", \"vocab\": " << d.vocab << ", \"width\": " << d.width << ", \"eps\": " << d.eps
               << ", \"bigram\": " << (d.bigram ? (int64_t)d.bigram->buckets : -1) << ", \"embedding_scale\": " << d.embedding_scale << ", \"residual_mult\": " << d.residual_mult << ", \"positions\": " << d.positions << ", \"streams\": " << d.streams
-              << ", \"tied_head\": " << (d.tied_head ? "true" : "false") << ", \"around_zero\": " << (d.norm_around_zero ? "true" : "false") << ", \"layers\": [";
+              << ", \"tied_head\": " << (d.tied_head ? "true" : "false") << ", \"around_zero\": " << (d.norm_around_zero ? "true" : "false") << ", \"logits\": [" << d.logit_scale << ", " << d.logit_cap << "], \"norm_scalar\": "
+              << (d.norm_scalar ? "true" : "false") << ", \"layers\": [";
     for (size_t i = 0; i < d.layers.size(); ++i) {
         std::cout << (i ? ", " : "");
         const LayerSpec& l = d.layers[i];
@@ -62,6 +64,10 @@ static void spec(std::istream& in) {
                       << a->left_scale << ", " << a->right_scale << "]";
         } else if (const auto* a = std::get_if<ChannelDeltaSpec>(&l.mixer)) {
             std::cout << "{\"sizes\": [" << a->heads << ", " << a->kv_heads << ", " << a->dim << ", " << a->vdim << ", " << a->taps << "]";
+        } else if (const auto* a = std::get_if<TimeMixingSpec>(&l.mixer)) {
+            std::cout << "{\"sizes\": [" << a->heads << ", " << a->dim << "]";
+        } else if (const auto* a = std::get_if<StateSpaceSpec>(&l.mixer)) {
+            std::cout << "{\"sizes\": [" << a->heads << ", " << a->groups << ", " << a->state << ", " << a->vdim << ", " << a->taps << ", " << a->norm_groups << "]";
         } else {
             const LightningSpec& n = std::get<LightningSpec>(l.mixer);
             std::cout << "{\"sizes\": [" << n.heads << ", " << n.dim << ", " << n.vdim << "], \"decay\": [";
@@ -70,9 +76,12 @@ static void spec(std::istream& in) {
         }
         const auto* g = std::get_if<GatedMlpSpec>(&l.mlp);
         std::cout << ", \"ff\": " << (g ? g->ff : 0) << ", \"silu\": " << (g && g->activation == Activation::Silu ? "true" : "false");
+        std::cout << ", \"tensors_of\": " << l.tensors_of;
+        if (const auto* p = std::get_if<PolyMlpSpec>(&l.mlp)) std::cout << ", \"poly\": " << p->ff;
         if (const auto* e = std::get_if<ExpertMlpSpec>(&l.mlp))
             std::cout << ", \"experts\": [" << e->experts << ", " << e->identity << ", " << e->top << ", " << e->ff << "], \"groups\": [" << e->groups << ", " << e->keep << "], \"router_scale\": " << e->scale
-                      << ", \"correction\": " << (e->correction ? "true" : "false");
+                      << ", \"correction\": " << (e->correction ? "true" : "false") << ", \"sigmoid\": " << (e->score == RouterScore::Sigmoid ? "true" : "false")
+                      << ", \"weight_input\": " << (e->weight_input ? "true" : "false") << ", \"limit\": [" << e->limit << ", " << e->alpha << "], \"activation\": " << (int)e->activation;
         std::cout << "}";
     }
     std::cout << "]}\n";

@@ -161,7 +161,8 @@ def test_projection_with_gated_feed_forward(ctx, dtype, rows, ff, plain):
 def test_products_refuse_what_they_do_not_serve(ctx):
     b = ctx.alloc(1 << 16)
     ok = dict(act_dtype=0, epilogue=STORE, a=b.ptr, lda=64, w=b.ptr, n_tiles=2, k_tiles=2, rows=4, batches=1, out_f32=b.ptr, ld_out=32, cols=32)
-    for bad, rc in ((dict(rows=0), -3), (dict(lda=40), -3), (dict(lda=32), -3), (dict(act_dtype=2), -3), (dict(epilogue=10), -3), (dict(cols=33), -4),
+    for bad, rc in ((dict(rows=0), -3), (dict(lda=40), -3), (dict(lda=32), -3), (dict(act_dtype=2), -3), (dict(epilogue=12), -3), (dict(segment_tiles=8), -3), (dict(segment_tiles=16, n_tiles=17, a_batch=64), -3),
+                    (dict(segment_tiles=16, batches=2), -3), (dict(epilogue=11, out_cap=-1.0), -4), (dict(cols=33), -4),
                     (dict(k_parts=3), -3), (dict(k_parts=2, epilogue=ADD), -3), (dict(out_f32=None), -4), (dict(a=None), -1),
                     (dict(epilogue=KEYS, out_act=b.ptr, rows=64), -4), (dict(epilogue=GATED, out_act=b.ptr, ld_act=30), -3)):
         call(ctx, "m40llm_ext_packed_gemm_async", C.byref(Gemm(**dict(ok, **bad))), 1, rc=rc)

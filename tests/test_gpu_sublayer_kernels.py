@@ -250,7 +250,7 @@ def split(ctx, dtype, cache, cfg, proj, slot, pos, back, weights, state, source=
     v0 = k0 + (2 * G * dim + 15) // 16 * 16
     pad = up32(dim)
     q = ctx.to_device(filled((rows, H, 2, pad), dtype))
-    s = Split(act_dtype=ACT[dtype], rows=rows, heads=H, kv_heads=G, dim=dim, vdim=vdim, taps=taps, eps=eps, proj=dev(ctx, keep, proj, np.float32),
+    s = Split(act_dtype=ACT[dtype], rows=rows, maps=2, heads=H, kv_heads=G, dim=dim, vdim=vdim, taps=taps, eps=eps, proj=dev(ctx, keep, proj, np.float32),
               ld_proj=proj.shape[1], k_offset=k0, v_offset=v0, conv_state=state.ptr, ld_state=proj.shape[1], queries=q.ptr, cache=None if source else cache.pages.ptr,
               row_slot=u32(ctx, keep, slot), row_pos=u32(ctx, keep, pos), row_back=u32(ctx, keep, back), page_table=cache.d_table.ptr, max_pages=cache.max_pages)
     for n in ("q", "k", "v"):
