@@ -361,7 +361,7 @@ def main():
     ap.add_argument("--traffic-probe", action="store_true",
                     help="also run one 256 MiB device-to-device copy through the library (calibrates rocprofv3 --pmc "
                          "FETCH_SIZE / WRITE_SIZE readings against a transfer of known size)")
-    ap.add_argument("--design", choices=["pimosun", "gulidra", "natatar"], help="instead of the default workload: prefill and decode throughput of "
+    ap.add_argument("--design", choices=["pimosun", "gulidra", "natatar", "fomunex"], help="instead of the default workload: prefill and decode throughput of "
                     "this design beside the closest other model of equal size (m40-llm_amd/layered_bench.py)")
     ap.add_argument("--shapes", default="", help="with --design: the shapes to run, with commas between them")
     ap.add_argument("--no-dense", action="store_true", help="with --design pimosun: leave the dense decoder out")

@@ -757,6 +757,8 @@ typedef struct M40llmPairAttention {
     uint32_t window;
     float cap;
     const void *slopes, *sink;
+    uint32_t even;                    /* form 1: the tiles see about equally many keys (a choice of speed only) */
+    float most;                       /* with a cap: |q.k| is never larger (0 = not known) */
 } M40llmPairAttention;
 int m40llm_ext_pair_attention_async(M40llmCudaContext* ctx, const M40llmPairAttention* a, uint32_t stream_kind);
 uint64_t m40llm_ext_pair_attention_partial_floats(uint32_t maps, uint32_t rows, uint32_t heads, uint32_t vdim, uint32_t splits);

@@ -255,7 +255,7 @@ constexpr uint32_t kTileThreads = 1024, kTileWaves = kTileThreads / 64;
 template <uint32_t KEEP>
 __global__ __launch_bounds__(kTileThreads) void poly_norm_tiles_kernel(m40_bf16* __restrict__ z, uint32_t ld, const float* __restrict__ act, uint32_t cols, float eps) {
     __shared__ float part[3][kTileWaves][16];
-    const uint32_t lane = threadIdx.x & 63u, wave = threadIdx.x >> 6, li = lane & 15u, g = lane >> 4, tiles = ld >> 5;
+    const uint32_t lane = threadIdx.x & 63u, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), li = lane & 15u, g = lane >> 4, tiles = ld >> 5;
     m40_bf16* own = z + (size_t)blockIdx.x * tiles * kM40Tile + lane * 8u;
     m40_bf16x8 kept[KEEP];
     PolySums s;
@@ -269,6 +269,7 @@ __global__ __launch_bounds__(kTileThreads) void poly_norm_tiles_kernel(m40_bf16*
         const float live = wave + j * kTileWaves < tiles ? 1.0f : 0.0f;
 #pragma unroll
         for (int i = 0; i < 8; ++i) s.take(static_cast<float>(kept[j][i]) * live);
+        asm volatile("" : "+v"(kept[j]));        // stays in bf16: its values in f32 are formed again for the result
     }
     for (uint32_t t = wave + KEEP * kTileWaves; t < tiles; t += kTileWaves) {
         const m40_bf16x8 v = *reinterpret_cast<const m40_bf16x8*>(own + (size_t)t * kM40Tile);
@@ -298,7 +299,19 @@ __global__ __launch_bounds__(kTileThreads) void poly_norm_tiles_kernel(m40_bf16*
 }
 
 template <class T>
-void launch_split(hipStream_t stream, const M40llmSpaceSplit& s, bool vec) {
+void launch_split(hipStream_t stream, M40llmSpaceSplit s, bool vec) {
+    // heads without padding lie side by side in the rows on both sides: as many together as fill the lanes
+    auto together = [](uint32_t& heads, uint32_t& size) {
+        if (size % 32u != 0) return;
+        for (uint32_t n = 128u / size; n > 1u; --n)
+            if (heads % n == 0) {
+                heads /= n;
+                size *= n;
+                return;
+            }
+    };
+    together(s.heads, s.vdim);
+    together(s.kv_heads, s.dim);
     const dim3 grid((s.rows + 15u) / 16u, 2u * s.kv_heads + s.heads);
     const uint32_t most = s.dim > s.vdim ? s.dim : s.vdim;
     if (!vec) space_split_kernel<T, 1, 16><<<grid, kThreads, 0, stream>>>(s);

@@ -2,7 +2,9 @@
 // Two maps, differential attention: softmaxes of their own queries and keys over the same values; the second map's result is taken off the
 // first's, lambda times, and what is left is normed over the head's value dimensions and gated.  One map: softmax attention, its result
 // scaled and, where there is a gate, gated column by column.  One map in the extended form (X): scores capped by a tanh, less a slope times the
-// distance of key and query, within a window of the newest tokens, beside a sink in the denominator; all of these are optional.
+// distance of key and query, within a window of the newest tokens, beside a sink in the denominator; all of these are optional.  Scores under a
+// small cap need no maximum (kBounded): weights are powers of two of the scores as they are; where the caller also bounds the products of queries and
+// keys well inside the cap (kInner), the tanh is a polynomial.
 //
 // Products are formed transposed, S' = K Q' and O' = V' P': a lane holds the scores of one query (lane % 16) for keys 4 g + r of every
 // 16, and pages hold values with their tokens in exactly that order, so the weights a lane computes are its operand of the second
@@ -34,12 +36,15 @@ struct PairArgs {
 // Window of the newest tokens (all: more than there can be), the first page that a query at `pos` sees, and whether every query of a range
 // sees the whole page.
 __device__ __forceinline__ uint32_t window_of(const M40llmPairAttention& a) { return a.window ? a.window : 0x7fffffffu; }
-template <bool X>
+enum Scores { kPlain = 0, kExtended = 1, kBounded = 2, kInner = 3 };
+constexpr float kInnerRange = 0.5f;        // of the tanh's argument
+constexpr float kBoundedCap = 60.0f;       // of a score as a power of two: sums of 2^60 and products with values stay far inside f32
+template <int X>
 __device__ __forceinline__ uint32_t first_page(const M40llmPairAttention& a, uint32_t pos) {
     const uint32_t w = window_of(a);
     return X && pos + 1u > w ? (pos + 1u - w) / kPage : 0u;
 }
-template <bool X>
+template <int X>
 __device__ __forceinline__ bool whole_page(const M40llmPairAttention& a, uint32_t page, uint32_t first_pos, uint32_t last_pos) {
     return page * kPage + kPage - 1u <= first_pos && (!X || page * kPage + window_of(a) > last_pos);
 }
@@ -68,12 +73,12 @@ struct PairState {
     float ref[M][B], sum[M][B];
     uint32_t pos[B];
 
-    __device__ __forceinline__ void clear() {
+    __device__ __forceinline__ void clear(float reference) {
 #pragma unroll
         for (int m = 0; m < M; ++m)
 #pragma unroll
             for (int b = 0; b < B; ++b) {
-                ref[m][b] = kNothing;
+                ref[m][b] = reference;
                 sum[m][b] = 0.0f;
 #pragma unroll
                 for (int j = 0; j < DVT; ++j) o[m][j][b] = m40_float4{0.f, 0.f, 0.f, 0.f};
@@ -102,6 +107,39 @@ struct PairState {
                     s[t][b][r] = fmaf(slope[b], d, s[t][b][r]);
                     if (!whole) s[t][b][r] = d <= 0.0f && d > -window ? s[t][b][r] : -INFINITY;
                 }
+        }
+    }
+    // kBounded, kInner: extend() and weigh() in one, without a reference
+    template <int X>
+    __device__ __forceinline__ void weigh_bounded(const M40llmPairAttention& a, const float (&slope)[B], m40_float4 (&s)[4][B], bool whole, uint32_t key0, m40_bf16x8 (&pf)[B][2]) {
+        const float window = (float)window_of(a), c = a.scale * 2.0f * kLog2e / a.cap, cap = a.cap * kLog2e;
+        // kInner: cap tanh(x) as x times a polynomial in x^2, fitted to 1.3e-7 on [-1/2, 1/2], in powers of the product s (x = s scale / cap)
+        const float x = a.scale / a.cap, x2 = x * x, p0 = cap * x, k0 = 0.9999976762f * p0, k1 = -0.3332065518f * p0 * x2, k2 = 0.1314514537f * p0 * x2 * x2,
+                    k3 = -0.04337247714f * p0 * x2 * x2 * x2;
+#pragma unroll
+        for (int b = 0; b < B; ++b) {
+            const float back = (float)((int)key0 - (int)pos[b]), base = fmaf(slope[b], back, X == kInner ? 0.0f : cap);
+            float l = 0.0f;
+#pragma unroll
+            for (int t = 0; t < 4; ++t)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const float z = s[t][b][r], bias = fmaf(slope[b], (float)(t * 16 + r), base);
+                    float e;
+                    if (X == kInner) {
+                        const float u = z * z;
+                        e = __builtin_amdgcn_exp2f(fmaf(z, fmaf(u, fmaf(u, fmaf(u, k3, k2), k1), k0), bias));
+                    } else {
+                        e = __builtin_amdgcn_exp2f(fmaf(-2.0f * cap, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(z * c)), bias));
+                    }
+                    if (!whole) {
+                        const float d = back + (float)(t * 16 + r);
+                        e = d <= 0.0f && d > -window ? e : 0.0f;
+                    }
+                    l += e;
+                    pf[b][t >> 1][(t & 1) * 4 + r] = static_cast<m40_bf16>(e);
+                }
+            sum[0][b] += l;
         }
     }
     // the scores of a map become weights: operands of the value product
@@ -224,7 +262,7 @@ struct PairState {
 // what a power of two loses per token of distance
 __device__ __forceinline__ float slope_of(const M40llmPairAttention& a, uint32_t head) { return a.slopes ? static_cast<const float*>(a.slopes)[head] * kLog2e : 0.0f; }
 
-template <int M, int DKT, int DVT, bool X>
+template <int M, int DKT, int DVT, int X>
 __global__ __launch_bounds__(256, 1) void pair_rows_kernel(PairArgs p) {
     extern __shared__ __align__(16) float join_lds[];      // three waves' sums
     const M40llmPairAttention& a = p.a;
@@ -239,7 +277,7 @@ __global__ __launch_bounds__(256, 1) void pair_rows_kernel(PairArgs p) {
     const uint32_t page0 = skipped + blockIdx.z * per, page1 = page0 + per < pages ? page0 + per : pages;
     const uint32_t* table = a.page_table + (size_t)a.row_slot[last_row] * a.max_pages;
     PairState<M, DKT, DVT, 1> s;
-    s.clear();
+    s.clear(X >= kBounded ? 0.0f : kNothing);
     s.pos[0] = a.row_pos[row];
     const float slope[1] = {X ? slope_of(a, head) : 0.0f};
     const m40_bf16* q = static_cast<const m40_bf16*>(a.queries) + ((size_t)row * a.heads + head) * ((uint32_t)M * kt * 32u) + g * 8;
@@ -275,8 +313,12 @@ __global__ __launch_bounds__(256, 1) void pair_rows_kernel(PairArgs p) {
 #pragma unroll
                     for (int h = 0; h < 2; ++h) vf[j][h] = *reinterpret_cast<const m40_bf16x8*>(values + ((j < vt ? j : vt - 1) * 2 + h) * kM40Tile);
             }
-            if constexpr (X) s.extend(a, slope, sc, whole, n * kPage + 4 * g);
-            s.weigh(m, sc, X ? 1.0f : c, X || whole, n * kPage + 4 * g, pf[m]);
+            if constexpr (X >= kBounded) {
+                s.template weigh_bounded<X>(a, slope, sc, whole, n * kPage + 4 * g, pf[m]);
+            } else {
+                if constexpr (X == kExtended) s.extend(a, slope, sc, whole, n * kPage + 4 * g);
+                s.weigh(m, sc, X ? 1.0f : c, X || whole, n * kPage + 4 * g, pf[m]);
+            }
         }
 #pragma unroll
         for (int j = 0; j < DVT; ++j)
@@ -377,7 +419,7 @@ __global__ __launch_bounds__(256) void pair_join_kernel(PairArgs p) {
     if (tid < a.vdim) static_cast<T*>(a.out)[m40_packed_at(row, head * a.vdim + tid, a.ld_out >> 5)] = M40Act<T>::from(o * f);
 }
 
-template <int M, int DKT, int DVT, int QB, int GROUPS, int PER_CU, bool X>
+template <int M, int DKT, int DVT, int QB, int GROUPS, int PER_CU, int X>
 __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArgs p) {
     typedef __attribute__((address_space(3))) void* lds_dst_t;
     typedef const __attribute__((address_space(1))) void* global_src_t;
@@ -402,7 +444,7 @@ __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArg
     issue(0, table[page_of(0)]);
     uint32_t next = table[page_of(1)];
     PairState<M, DKT, DVT, QB> s;
-    s.clear();
+    s.clear(X >= kBounded ? 0.0f : kNothing);
     uint32_t row[QB], head[QB];
     bool live[QB];
 #pragma unroll
@@ -462,8 +504,12 @@ __global__ __launch_bounds__(GROUPS * 256, PER_CU) void pair_tile_kernel(PairArg
                     }
                 }
             __builtin_amdgcn_s_setprio(0);
-            if constexpr (X) s.extend(a, slope, sc, whole, n * kPage + 4 * g);
-            s.weigh(m, sc, X ? 1.0f : c, X || whole, n * kPage + 4 * g, pf[m]);
+            if constexpr (X >= kBounded) {
+                s.template weigh_bounded<X>(a, slope, sc, whole, n * kPage + 4 * g, pf[m]);
+            } else {
+                if constexpr (X == kExtended) s.extend(a, slope, sc, whole, n * kPage + 4 * g);
+                s.weigh(m, sc, X ? 1.0f : c, X || whole, n * kPage + 4 * g, pf[m]);
+            }
         }
         __builtin_amdgcn_s_setprio(1);
 #pragma unroll
@@ -510,7 +556,7 @@ __global__ __launch_bounds__(256) void pair_f32_kernel(PairArgs p) {
     const uint32_t* table = a.page_table + (size_t)a.row_slot[row] * a.max_pages;
     const float slope = M == 1 && a.slopes ? static_cast<const float*>(a.slopes)[head] : 0.0f;
     __syncthreads();
-    for (uint32_t n = first_page<M == 1>(a, pos); n < pages; ++n) {
+    for (uint32_t n = first_page<M == 1 ? kExtended : kPlain>(a, pos); n < pages; ++n) {
         const float* page = static_cast<const float*>(a.cache) + table[n] * p.page.elements() + kv * p.page.head_elements();
         // two lanes a token and map of two, four a token of one
         constexpr uint32_t kLanes = 4u / M;
@@ -564,7 +610,7 @@ __global__ __launch_bounds__(256) void pair_f32_kernel(PairArgs p) {
 
 constexpr int kLdsMax = 160 * 1024;
 
-template <int M, int DKT, int DVT, bool X>
+template <int M, int DKT, int DVT, int X>
 int launch_rows(hipStream_t stream, const PairArgs& p) {
     constexpr int lds = 3 * 64 * 4 * PairState<M, DKT, DVT, 1>::kFloats;
     static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(pair_rows_kernel<M, DKT, DVT, X>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
@@ -573,7 +619,7 @@ int launch_rows(hipStream_t stream, const PairArgs& p) {
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
 int page_lds(const PairArgs& p, int groups) { return groups * 2 * (int)(4u * p.page.maps * p.page.k_tiles + 2u * p.page.v_tiles) * 1024; }
-template <int M, int DKT, int DVT, int QB, int GROUPS, int PER_CU, bool X>
+template <int M, int DKT, int DVT, int QB, int GROUPS, int PER_CU, int X>
 int launch_tile(hipStream_t stream, const PairArgs& p) {
     static const hipError_t attr =
         hipFuncSetAttribute(reinterpret_cast<const void*>(pair_tile_kernel<M, DKT, DVT, QB, GROUPS, PER_CU, X>), hipFuncAttributeMaxDynamicSharedMemorySize, kLdsMax);
@@ -585,10 +631,12 @@ int launch_tile(hipStream_t stream, const PairArgs& p) {
     return hipGetLastError() == hipSuccess ? 0 : -2;
 }
 // PER_CU: workgroups of one group a CU that fit
-template <int M, int DKT, int DVT, int PER_CU, bool X>
+template <int M, int DKT, int DVT, int PER_CU, int X>
 int launch_tile_any(hipStream_t stream, const PairArgs& p, int num_cus) {
-    // with enough workgroups the short ones fill in behind the long ones
-    if (page_lds(p, 2) <= kLdsMax && (uint64_t)p.a.kv_heads * p.a.n_tiles <= 3ull * (uint32_t)num_cus)
+    // With enough workgroups the short ones fill in behind the long ones.  Where all walks are alike there is nothing to halve, and two workgroups
+    // a CU, whose barriers are their own, overlap products and weights better than two groups of one.
+    const uint64_t workgroups = (uint64_t)p.a.kv_heads * p.a.n_tiles;
+    if (page_lds(p, 2) <= kLdsMax && workgroups <= 3ull * (uint32_t)num_cus && !(p.a.even && workgroups >= 2ull * (uint32_t)num_cus))
         return p.a.tile_queries == 64u ? launch_tile<M, DKT, DVT, 1, 2, PER_CU, X>(stream, p) : launch_tile<M, DKT, DVT, 2, 2, PER_CU, X>(stream, p);
     return p.a.tile_queries == 64u ? launch_tile<M, DKT, DVT, 1, 1, PER_CU, X>(stream, p) : launch_tile<M, DKT, DVT, 2, 1, PER_CU, X>(stream, p);
 }
@@ -596,7 +644,7 @@ int launch_tile_any(hipStream_t stream, const PairArgs& p, int num_cus) {
 bool tile_served(uint32_t maps, uint32_t k_tiles, uint32_t v_tiles) { return 2u * (4u * maps * k_tiles + 2u * v_tiles) * 1024u <= (uint32_t)kLdsMax; }
 
 // PER_CU of heads of 128 dimensions
-template <int M, int PER_CU, bool X>
+template <int M, int PER_CU, int X>
 int launch_form(hipStream_t stream, const PairArgs& p, uint32_t form, int num_cus) {
     const uint32_t kt = p.page.k_tiles, vt = p.page.v_tiles;
     if (form == 1u) {
@@ -605,6 +653,8 @@ int launch_form(hipStream_t stream, const PairArgs& p, uint32_t form, int num_cu
         if (kt <= 4u && vt <= 8u) return launch_tile_any<M, 4, 8, PER_CU, X>(stream, p, num_cus);
         return launch_tile<M, 8, 16, 1, 1, 1, X>(stream, p);
     }
+    if constexpr (X >= kBounded) return -3;      // rows: the extended form hides more of the pages' latency
+    else {
     int rc;
     if (kt <= 2u && vt <= 4u) rc = launch_rows<M, 2, 4, X>(stream, p);
     else if (kt <= 2u && vt <= 8u) rc = launch_rows<M, 2, 8, X>(stream, p);
@@ -613,12 +663,17 @@ int launch_form(hipStream_t stream, const PairArgs& p, uint32_t form, int num_cu
     if (rc != 0 || p.a.splits == 1u) return rc;
     pair_join_kernel<m40_bf16, M><<<p.a.n_rows * p.a.heads, 256, 0, stream>>>(p);
     return hipGetLastError() == hipSuccess ? 0 : -2;
+    }
 }
 
 int launch(hipStream_t stream, const PairArgs& p, uint32_t form, int num_cus) {
-    if (p.a.maps == 2u) return launch_form<2, 1, false>(stream, p, form, num_cus);
-    if (p.a.window || p.a.cap > 0.0f || p.a.slopes) return launch_form<1, 2, true>(stream, p, form, num_cus);
-    return launch_form<1, 2, false>(stream, p, form, num_cus);
+    if (p.a.maps == 2u) return launch_form<2, 1, kPlain>(stream, p, form, num_cus);
+    if (form == 1u && p.a.cap > 0.0f && p.a.cap * kLog2e <= kBoundedCap) {
+        if (p.a.most > 0.0f && p.a.most * p.a.scale <= kInnerRange * p.a.cap) return launch_form<1, 2, kInner>(stream, p, form, num_cus);
+        return launch_form<1, 2, kBounded>(stream, p, form, num_cus);
+    }
+    if (p.a.window || p.a.cap > 0.0f || p.a.slopes) return launch_form<1, 2, kExtended>(stream, p, form, num_cus);
+    return launch_form<1, 2, kPlain>(stream, p, form, num_cus);
 }
 
 }  // namespace

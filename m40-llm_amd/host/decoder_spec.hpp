@@ -166,7 +166,7 @@ struct DecoderSpec {
     float eps = 0.0f;
     NormKind norm = NormKind::Layer;
     bool norm_around_zero = false;     // norm weights are stored less one
-    bool norm_scalar = false;          // norm weights are one number for all coordinates
+    bool norm_scalar = false;          // norm weights are scalars
     float logit_scale = 1.0f, logit_cap = 0.0f;      // logits are scaled, then held within +-cap by a tanh (0 = not)
     bool tied_head = false;            // logits from the embedding table
     uint32_t streams = 1;              // BlockKind::Streams

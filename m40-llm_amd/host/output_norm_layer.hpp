@@ -22,6 +22,7 @@ struct PairTiles : PassTable {
     PairTiles(uint32_t g, uint32_t most, uint32_t w) : group(g), most_queries(most), window(w ? w : 0x7fffffffu) {}
     bool same(uint32_t g, uint32_t most, uint32_t w) const { return group == g && most_queries == most && window == (w ? w : 0x7fffffffu); }
     uint32_t group, most_queries, window, fewest_kv_heads = 0xffffffffu, n_short = 0, n_long = 0, long_queries = 64, splits = 1;
+    bool even = false;                    // long tiles see about equally many keys
     uint64_t floats_a_row = 0;            // of a split's partial sums, the largest layer's
     const uint32_t* long_tiles() const { return at + 2 * n_short; }
     std::vector<uint32_t> build(const PassPlan& plan, const SequencePages&, uint32_t longest) override {
@@ -45,7 +46,12 @@ struct PairTiles : PassTable {
             }
         }
         std::stable_sort(tiles.begin(), tiles.end(), [](const Tile& a, const Tile& b) { return a.keys > b.keys; });     // the longest walks first
-        for (const Tile& x : tiles) t.insert(t.end(), {x.first, x.n});
+        uint64_t keys = 0;
+        for (const Tile& x : tiles) {
+            t.insert(t.end(), {x.first, x.n});
+            keys += x.keys;
+        }
+        even = !tiles.empty() && (uint64_t)tiles[0].keys * tiles.size() <= keys + keys / 4;
         n_long = (uint32_t)tiles.size();
         // the pages of a tile over as many workgroups as fill the CUs twice, a page a wave at least
         const uint32_t seen = longest > window ? window + LayerRuntime::kPage : longest;

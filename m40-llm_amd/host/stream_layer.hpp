@@ -152,6 +152,7 @@ public:
         h.act_dtype = rt_.opt.act_dtype; h.maps = 1; h.heads = a_.heads; h.kv_heads = a_.kv_heads; h.dim = a_.dim; h.vdim = a_.vdim;
         h.scale = std::fabs(a_.scale); h.out_scale = out_factor_;
         h.window = a_.window; h.cap = a_.cap; h.slopes = w_->slopes.ptr(); h.sink = w_->sink.ptr();
+        if (a_.head_norm) h.most = 1.02f * (float)a_.dim;        // both of length sqrt(dim) at most, then rounded
         h.queries = sh_.queries.ptr(); h.cache = cache_.ptr();
         if (a_.column_gate) { h.gate = rt_.proj.f32(gate_offset(a_)); h.ld_gate = ld; }
         h.row_slot = r.slot; h.row_pos = r.pos; h.page_table = r.page_table; h.max_pages = rt_.max_pages;
@@ -169,7 +170,7 @@ public:
         }
         if (tiles_->n_long) {
             h.form = 1;
-            h.tiles = tiles_->long_tiles(); h.n_tiles = tiles_->n_long;
+            h.tiles = tiles_->long_tiles(); h.n_tiles = tiles_->n_long; h.even = tiles_->even;
             M40H_TRY(m40llm_ext_pair_attention_async(rt_.ctx, &h, rt_.kStream));
         }
     }

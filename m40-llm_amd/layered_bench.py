@@ -1,7 +1,7 @@
 """Prefill and decode throughput of layered decoders with random weights beside the framework's closest other model of the same width,
 depth and vocabulary.  `bench.py --design NAME` prints what measure() returns: the Pimosun design beside the dense decoder, the Gulidra
 design beside Pimosun, whose feed-forward is as wide as the experts a token takes together, the Natatar design beside Gulidra with the same
-experts in every layer.
+experts in every layer, the Fomunex design beside Gulidra (dense and routed feed-forwards in turn on both sides) and Natatar.
 
 A case is one shape on one kind of step: a prompt of n tokens run in one step (host clock around the blocking call, the last
 token's logits included), or `batch` sequences of `context` tokens that decode greedily from a replayed graph (timed between
@@ -17,7 +17,7 @@ pkg = importlib.import_module(__package__)
 syn = importlib.import_module(__package__ + ".synthetic")
 layered = importlib.import_module(__package__ + ".layered")
 
-BESIDE = dict(pimosun="Pimosun beside the dense decoder", gulidra="Gulidra beside Pimosun", natatar="Natatar beside Gulidra")
+BESIDE = dict(pimosun="Pimosun beside the dense decoder", gulidra="Gulidra beside Pimosun", natatar="Natatar beside Gulidra", fomunex="Fomunex beside Gulidra and Natatar")
 SHAPES = {
     # name: layered decoder, and the dense decoder's heads at the same width
     "2k": dict(width=2048, heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=768, ff=5632, vocab=32000, layers=8, kv_heads=2),
@@ -87,6 +87,28 @@ def natatar_config(name: str) -> dict:
     moe = dict(kind="moe", expert=dict(ff=g["expert_ff"]), router=dict(experts=g["experts"], top=g["top"], scale=2.0, groups=dict(count=g["groups"][0], keep=g["groups"][1])))
     return dict(architecture="Natatar", vocab=s["vocab"], width=s["width"], streams=g["streams"], norm=dict(eps=1e-5), embedding=dict(scale=1.0), residual_mult=0.3,
                 layers=[dict(kinds[i % 4], mlp=moe) for i in range(s["layers"])])
+
+
+# Fomunex at the same sizes: of four layers two of attention (a window of 1024 tokens, one of all positions), one of time mixing, one state space layer;
+# dense and routed feed-forwards in turn, the dense one without a gate, so wider by half for the same weights
+FOMUNEX = {
+    "2k": dict(kv_heads=4, dim=128, windows=(1024, 8192), mixing=(32, 64), space=(64, 8, 128, 64, 4, 8), ff=8448, experts=32, top=4, expert_ff=1408),
+    "4k": dict(kv_heads=8, dim=128, windows=(1024, 8192), mixing=(64, 64), space=(128, 8, 128, 64, 4, 8), ff=16512, experts=32, top=4, expert_ff=2752),
+}
+
+
+def fomunex_config(name: str) -> dict:
+    s, g = SHAPES[name], FOMUNEX[name]
+    attention = [dict(type="attention", mixer=dict(heads=s["heads"], kv_heads=g["kv_heads"], dim=g["dim"], vdim=s["vdim"], mask=dict(size=w), softcap=30.0,
+                                                   scale=float(g["dim"] ** -0.5))) for w in g["windows"]]
+    h, d = g["mixing"]
+    mixing = dict(type="wkv", mixer=dict(heads=h, dim=d))
+    space = dict(type="mamba2", mixer=dict(zip(("heads", "groups", "state", "vdim", "conv", "norm_groups"), g["space"])))
+    moe = dict(kind="moe", expert=dict(ff=g["expert_ff"], limit=7.0), router=dict(experts=g["experts"], top=g["top"]))
+    dense = dict(kind="dense", ff=g["ff"])
+    kinds = [dict(attention[0], mlp=dense), dict(mixing, mlp=moe), dict(attention[1], mlp=dense), dict(space, mlp=moe)]
+    return dict(architecture="Fomunex", vocab=s["vocab"], width=s["width"], norm=dict(eps=1e-5), max_positions=8192, logit_scale=0.5, logit_softcap=30.0,
+                layers=[kinds[i % 4] for i in range(s["layers"])])
 
 
 def layer_flops_per_token(s: dict, own: bool) -> float:
@@ -167,6 +189,13 @@ def dense_cases(ctx, s, prefill=PREFILL, decode=DECODE, reps=3, steps=32, warmup
 
 def measure(ctx, shapes=None, steps=32, warmup=4, dense=True, design="pimosun") -> dict:
     out = {}
+    if design == "fomunex":
+        for name in shapes or SHAPES:
+            s = SHAPES[name]
+            out[name] = {"shape": dict(s, **FOMUNEX[name]), "fomunex": layered_cases(ctx, s, steps=steps, warmup=warmup, cfg=fomunex_config(name)),
+                         "gulidra": layered_cases(ctx, s, steps=steps, warmup=warmup, cfg=gulidra_config(name)),
+                         "natatar": layered_cases(ctx, s, steps=steps, warmup=warmup, cfg=natatar_config(name))}
+        return out
     if design == "natatar":
         for name in shapes or SHAPES:
             s = SHAPES[name]

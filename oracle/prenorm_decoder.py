@@ -23,7 +23,7 @@ def root_norm(x, eps):
 
 
 def scalar_norm(x, g, eps):
-    """RMS norm with one number for all coordinates."""
+    """RMS norm whose weight is a scalar."""
     return root_norm(x, eps) * g
 
 

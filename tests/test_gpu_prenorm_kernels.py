@@ -175,7 +175,7 @@ def test_heads_over_their_root_mean_square(ctx, dtype, H, G, dim, vdim):
         close_to(gv, p[i * n:(i + 1) * n, v0:v0 + G * vdim].reshape(n, G, vdim), dtype)
 
 
-def attend(ctx, dtype, cache, cfg, q, slot, pos, portions, form, splits, tile_queries, scale, cap, window, slopes, sink):
+def attend(ctx, dtype, cache, cfg, q, slot, pos, portions, form, splits, tile_queries, scale, cap, window, slopes, sink, most=0.0, even=0):
     H, G, dim, vdim = cfg
     keep, rows, pad, group = [], len(q), up32(dim), H // G
     qq = np.zeros((rows, H, pad), np.float32)
@@ -189,7 +189,7 @@ def attend(ctx, dtype, cache, cfg, q, slot, pos, portions, form, splits, tile_qu
     a = Attn(act_dtype=ACT[dtype], form=form, maps=1, heads=H, kv_heads=G, dim=dim, vdim=vdim, scale=scale, out_scale=1.0, queries=dev(ctx, keep, as_act(qq, dtype)),
              cache=cache.pages.ptr, row_slot=u32(ctx, keep, slot), row_pos=u32(ctx, keep, pos), page_table=cache.d_table.ptr, max_pages=cache.max_pages, tiles=u32(ctx, keep, tiles),
              n_tiles=len(tiles), tile_queries=tile_queries, splits=splits, n_rows=rows, partial=partial.ptr, partial_floats=floats, out=out.ptr, ld_out=ldo, window=window or 0,
-             cap=cap or 0.0, slopes=None if slopes is None else dev(ctx, keep, slopes, np.float32), sink=None if sink is None else dev(ctx, keep, sink, np.float32))
+             cap=cap or 0.0, most=most, even=even, slopes=None if slopes is None else dev(ctx, keep, slopes, np.float32), sink=None if sink is None else dev(ctx, keep, sink, np.float32))
     call(ctx, "m40llm_ext_pair_attention_async", C.byref(a), 1)
     return from_act(unpack_tiles(out.download(act_type(dtype), ((rows + 15) // 16 * 16 * ldo,)), rows, ldo), dtype)[:, :H * vdim].reshape(rows, H, vdim)
 
@@ -252,6 +252,28 @@ def test_attention_over_many_like_keys(ctx, dtype, form, splits, tile, cap, wind
     args = (0.125, cap, window, 2.0 ** np.arange(-8, -4) if slopes else None, None if sink is None else sink + rng.standard_normal(4))
     got = attend(ctx, dtype, cache, cfg, q, [1] * 70, pos, [(0, 70)], form, splits, tile, *args)
     close_to(got, attend_want(q, k, v, pos, cfg, *args), dtype, factor=3)
+
+
+@pytest.mark.parametrize("tile", [64, 128])
+@pytest.mark.parametrize("even", [0, 1])
+@pytest.mark.parametrize("H,G,dim,vdim", [(4, 2, 64, 64), (3, 1, 20, 37), (8, 2, 128, 128), (2, 1, 160, 144)])
+@pytest.mark.parametrize("cap,window", [(3.0, None), (12.0, 65), (40.0, 200), (60.0, 100)])
+def test_attention_of_bounded_products(ctx, H, G, dim, vdim, cap, window, tile, even):
+    """Normed queries and keys, whose products are bounded: just inside the polynomial's range, where its error is largest, and beyond it."""
+    if ctx.lib.m40llm_ext_pair_attention_tile_queries(0, 1, dim, vdim) < tile:
+        pytest.skip("these sizes have no such tile")
+    rng, n, rows = np.random.default_rng(dim), 330, 150
+    cfg, cache = (H, G, dim, vdim), Cache(ctx, "bfloat16", G, dim, vdim, 1, 6)
+    k, v = rounded(pd.root_norm(rng.standard_normal((n, G, dim)), 1e-6), "bfloat16"), rounded(rng.standard_normal((n, G, vdim)), "bfloat16")
+    cache.fill(ctx, {0: (k, v)})
+    pos = np.arange(n - rows, n)
+    q = np.stack([k[np.maximum(pos - (7 * h) % 90, 0), h // (H // G)] * (-1) ** h for h in range(H)], axis=1)      # products of dim and minus dim
+    m = 2.0 ** (-8.0 * (np.arange(H) + 1) / H)
+    for reach in (0.49, 1.5):
+        scale = reach * cap / (1.02 * dim)
+        args = (scale, cap, window, m, rng.standard_normal(H))
+        got = attend(ctx, "bfloat16", cache, cfg, q, [0] * rows, pos, [(0, rows)], 1, 1, tile, *args, most=1.02 * dim, even=even)
+        close_to(got, attend_want(q, k, v, pos, cfg, *args), "bfloat16", factor=3)
 
 
 def test_attention_refuses_what_only_one_map_has(ctx):
