@@ -213,15 +213,14 @@ __device__ __forceinline__ void m40_epilogue_pair(const M40Epilogue<T>& e, int r
     const int col = pair * 16 + 4 * (lane >> 4), row = row0 + (lane & 15);
     if (row >= e.rows) return;
     m40_float4 y;
+    const float f = e.row_scale ? e.row_scale[row] : 1.0f;
     if (e.activation == M40LLM_LIMITED_GATE) {
-        const float f = e.row_scale ? e.row_scale[row] : 1.0f;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const float z = fminf(g[r] * f, e.act_limit), up = fminf(fmaxf(u[r] * f, -e.act_limit), e.act_limit);
             y[r] = z * m40_sigmoid(e.act_alpha * z) * (up + 1.0f);
         }
     } else {
-        const float f = e.row_scale ? e.row_scale[row] : 1.0f;
 #pragma unroll
         for (int r = 0; r < 4; ++r) y[r] = (e.activation == M40LLM_SILU ? m40_silu(g[r] * f) : m40_gelu_tanh(g[r] * f)) * (u[r] * f);
     }

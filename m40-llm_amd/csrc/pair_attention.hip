@@ -653,19 +653,19 @@ int launch_form(hipStream_t stream, const PairArgs& p, uint32_t form, int num_cu
         if (kt <= 4u && vt <= 8u) return launch_tile_any<M, 4, 8, PER_CU, X>(stream, p, num_cus);
         return launch_tile<M, 8, 16, 1, 1, 1, X>(stream, p);
     }
-    if constexpr (X >= kBounded) return -3;      // rows: the extended form hides more of the pages' latency
-    else {
-    int rc;
-    if (kt <= 2u && vt <= 4u) rc = launch_rows<M, 2, 4, X>(stream, p);
-    else if (kt <= 2u && vt <= 8u) rc = launch_rows<M, 2, 8, X>(stream, p);
-    else if (kt <= 4u && vt <= 8u) rc = launch_rows<M, 4, 8, X>(stream, p);
-    else rc = launch_rows<M, 8, 16, X>(stream, p);
-    if (rc != 0 || p.a.splits == 1u) return rc;
-    pair_join_kernel<m40_bf16, M><<<p.a.n_rows * p.a.heads, 256, 0, stream>>>(p);
-    return hipGetLastError() == hipSuccess ? 0 : -2;
+    if constexpr (X >= kBounded) {               // rows: the extended form hides more of the pages' latency
+        return -3;
+    } else {
+        int rc;
+        if (kt <= 2u && vt <= 4u) rc = launch_rows<M, 2, 4, X>(stream, p);
+        else if (kt <= 2u && vt <= 8u) rc = launch_rows<M, 2, 8, X>(stream, p);
+        else if (kt <= 4u && vt <= 8u) rc = launch_rows<M, 4, 8, X>(stream, p);
+        else rc = launch_rows<M, 8, 16, X>(stream, p);
+        if (rc != 0 || p.a.splits == 1u) return rc;
+        pair_join_kernel<m40_bf16, M><<<p.a.n_rows * p.a.heads, 256, 0, stream>>>(p);
+        return hipGetLastError() == hipSuccess ? 0 : -2;
     }
 }
-
 int launch(hipStream_t stream, const PairArgs& p, uint32_t form, int num_cus) {
     if (p.a.maps == 2u) return launch_form<2, 1, kPlain>(stream, p, form, num_cus);
     if (form == 1u && p.a.cap > 0.0f && p.a.cap * kLog2e <= kBoundedCap) {
